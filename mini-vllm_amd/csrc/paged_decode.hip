@@ -24,6 +24,11 @@
 #include <cstdlib>
 
 
+__global__ void __launch_bounds__(256) zero_fill_kernel(uint32_t *p, int64_t n) {
+  const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  if (i < n) p[i] = 0u;
+}
+
 // ---- host side -------------------------------------------------------------
 namespace {
 
@@ -263,8 +268,12 @@ int paged_decode_impl(const void *q, int64_t q_stride_tok, const void *k_cache,
   const int esz = dtype == MV_F32 ? 4 : 2;
   if (max_blocks == 0 || num_blocks == 0) {
     // reference: zero-column block tables (warm-up) give zeros, page_attention.py:62-65
-    return mv_check_hip(hipMemsetAsync(out, 0, (size_t)batch * n_heads * head_dim * esz,
-                                       (hipStream_t)stream));
+    // (a fill kernel: a memset node inside a captured graph has given wrong results on later replays)
+    const int64_t words = (int64_t)batch * n_heads * head_dim * esz / 4;
+    hipLaunchKernelGGL(zero_fill_kernel, dim3((unsigned)((words + 255) / 256)), dim3(256), 0, (hipStream_t)stream,
+                       (uint32_t *)out, words);
+    MV_LAUNCH_CHECK();
+    return MV_OK;
   }
   if (!k_cache || !v_cache || !block_tables) return MV_E_NULLPTR;
   DecodePlan pl;

@@ -22,6 +22,7 @@ def asm(tmp_path_factory):
         pytest.skip("hipcc not installed")
     out = tmp_path_factory.mktemp("audit") / "prefill_mfma.s"
     subprocess.run([HIPCC, "-O3", "-std=c++17", "-fPIC", "-ffp-contract=off", "--offload-arch=gfx950", "-fno-slp-vectorize",
+                    "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
                     "--cuda-device-only", "-S", "-o", str(out), os.path.join(ROOT, "mini-vllm_amd", "csrc", "prefill_mfma.hip")],
                    check=True, stderr=subprocess.DEVNULL)
     text = out.read_text()
