@@ -25,8 +25,9 @@ def main():
     ap.add_argument("--top-k", type=int, default=-1)
     ap.add_argument("--dummy", action="store_true", help="random-initialise the weights (no checkpoint needed)")
     ap.add_argument("--eager", action="store_true")
+    ap.add_argument("--dtype", choices=["bfloat16", "float16", "float32"], default="bfloat16")
     a = ap.parse_args()
-    cfg = Config(a.model, dtype="bfloat16", tensor_parallel_size=a.tp, enforce_eager=a.eager, max_num_seqs=256,
+    cfg = Config(a.model, dtype=a.dtype, tensor_parallel_size=a.tp, enforce_eager=a.eager, max_num_seqs=256,
                  load_format="dummy" if a.dummy else "auto")
     llm = LLM(cfg)
     sp = SamplingParams(temperature=a.temperature, top_p=a.top_p, top_k=a.top_k, max_tokens=a.max_tokens,
@@ -35,7 +36,8 @@ def main():
         prompts = ["Introduce yourself.", "List all prime numbers within 100.", "What is the capital of France?",
                    "Explain paged attention in two sentences."]
     else:
-        prompts = [[(7 * i + j) % 1000 + 10 for j in range(16 + 8 * i)] for i in range(4)]
+        vocab = cfg.hf_config.vocab_size
+        prompts = [[((7 * i + j) % 1000 + 10) % vocab for j in range(16 + 8 * i)] for i in range(4)]
     t0 = time.perf_counter()
     outs = llm.generate(prompts, sp)
     dt = time.perf_counter() - t0

@@ -45,6 +45,17 @@ enum {
   MV_E_ALIAS = -7      /* an output overlaps an input other workgroups still read */
 };
 
+/* Options of the attention entry points with the suffix _ex (HOST struct, read during the call; NULL = all defaults):
+ *   interleaved / rot_pairs: rotary layout.  0 / 0: dim i pairs with dim i + D/2 and cos, sin are [max_pos, D/2].
+ *       1 / n: dim 2i pairs with dim 2i + 1 for i < n, dims from 2n on pass unchanged, cos, sin are [max_pos, n].
+ *   chunk: > 0: a query at position i sees only the keys of its own chunk of `chunk` positions (counted from the start of
+ *       the sequence), i / chunk * chunk .. i.  0: every key up to i.
+ *   out_stride: elements between the token rows of `out` (0: dense [.., H, D] rows). */
+typedef struct MvAttnOpts {
+  int rot_pairs, interleaved, chunk, reserved;
+  int64_t out_stride;
+} MvAttnOpts;
+
 int mv_version(void);
 const char *mv_strerror(int code);
 
@@ -97,6 +108,15 @@ int mv_rope_qk_store(const void *q, const void *k, const void *v,
                      const int32_t *slot_mapping, int64_t num_slots, int n_tok,
                      int n_heads, int n_kv_heads, int head_dim, int dtype,
                      void *stream);
+int mv_rope_qk_store_ex(const void *q, const void *k, const void *v,
+                        int64_t q_stride_tok, int64_t k_stride_tok,
+                        int64_t v_stride_tok, const int64_t *positions,
+                        const float *cos, const float *sin, int64_t max_pos,
+                        const void *q_norm_w, const void *k_norm_w, float eps,
+                        void *q_out, void *k_out, void *k_cache, void *v_cache,
+                        const int32_t *slot_mapping, int64_t num_slots, int n_tok,
+                        int n_heads, int n_kv_heads, int head_dim, int dtype,
+                        const MvAttnOpts *opts, void *stream);
 
 /* K3 — paged-KV decode attention (one query token per sequence).
  * Replaces PageAttention.__call__ / flash_attn_with_kvcache
@@ -120,6 +140,9 @@ enum {
 size_t mv_paged_decode_workspace_bytes(int batch, int n_heads, int n_kv_heads,
                                        int head_dim, int block_size,
                                        int max_blocks, int flags);
+size_t mv_paged_decode_workspace_bytes_ex(int batch, int n_heads, int n_kv_heads,
+                                          int head_dim, int block_size,
+                                          int max_blocks, int flags, int chunk);
 int mv_paged_decode(const void *q, int64_t q_stride_tok, const void *k_cache,
                     const void *v_cache, const int32_t *block_tables,
                     int64_t table_stride, const int32_t *context_lens,
@@ -127,6 +150,14 @@ int mv_paged_decode(const void *q, int64_t q_stride_tok, const void *k_cache,
                     int head_dim, int block_size, int max_blocks,
                     int64_t num_blocks, float scale, void *workspace,
                     size_t ws_bytes, int dtype, int flags, void *stream);
+int mv_paged_decode_ex(const void *q, int64_t q_stride_tok, const void *k_cache,
+                       const void *v_cache, const int32_t *block_tables,
+                       int64_t table_stride, const int32_t *context_lens,
+                       void *out, int batch, int n_heads, int n_kv_heads,
+                       int head_dim, int block_size, int max_blocks,
+                       int64_t num_blocks, float scale, void *workspace,
+                       size_t ws_bytes, int dtype, int flags,
+                       const MvAttnOpts *opts, void *stream);
 
 /* K7 + K6 (per head) + K1 + K3 in one launch, for decode steps: q / k / v are the RAW rows of the qkv projection
  * (views of its output: row strides in elements); the attention kernel applies the per-head RMSNorm (q_norm_w /
@@ -144,6 +175,14 @@ int mv_rope_paged_decode(const void *q, int64_t q_stride_tok, const void *k, int
                          void *out, int batch, int n_heads, int n_kv_heads, int head_dim, int block_size,
                          int max_blocks, int64_t num_blocks, float scale, void *workspace, size_t ws_bytes,
                          int dtype, int flags, void *stream);
+int mv_rope_paged_decode_ex(const void *q, int64_t q_stride_tok, const void *k, int64_t k_stride_tok,
+                            const void *v, int64_t v_stride_tok, const int64_t *positions, const float *cos,
+                            const float *sin, int64_t max_pos, const void *q_norm_w, const void *k_norm_w,
+                            float eps, const int32_t *slot_mapping, void *k_cache, void *v_cache,
+                            const int32_t *block_tables, int64_t table_stride, const int32_t *context_lens,
+                            void *out, int batch, int n_heads, int n_kv_heads, int head_dim, int block_size,
+                            int max_blocks, int64_t num_blocks, float scale, void *workspace, size_t ws_bytes,
+                            int dtype, int flags, const MvAttnOpts *opts, void *stream);
 
 
 /* K2 — packed varlen causal prefill attention (flash-style, MFMA).
@@ -167,6 +206,16 @@ int mv_prefill_varlen(const void *q, int64_t q_stride_tok, const void *k,
                       int n_seqs, int max_seqlen_q, int max_seqlen_k,
                       int n_heads, int n_kv_heads, int head_dim,
                       int block_size, float scale, int dtype, int flags, void *stream);
+int mv_prefill_varlen_ex(const void *q, int64_t q_stride_tok, const void *k,
+                         const void *v, int64_t k_stride_tok, int64_t v_stride_tok,
+                         const void *k_cache, const void *v_cache,
+                         const int32_t *block_tables, int64_t table_stride,
+                         int64_t num_blocks, void *out,
+                         const int32_t *cu_seqlens_q, const int32_t *cu_seqlens_k,
+                         int n_seqs, int max_seqlen_q, int max_seqlen_k,
+                         int n_heads, int n_kv_heads, int head_dim,
+                         int block_size, float scale, int dtype, int flags,
+                         const MvAttnOpts *opts, void *stream);
 
 /* K8 — fused temperature / top-k / top-p / min-p / multinomial sampler.
  * Replaces Sampler.forward + sampling/functional.py:34-233,410-437 as driven
@@ -244,6 +293,33 @@ size_t mv_persist_struct_bytes(int which);
 int mv_silu_and_mul(const void *x, int64_t x_stride, void *out,
                     int64_t out_stride, int rows, int cols, int dtype,
                     void *stream);
+/* ... with the tanh form of gelu for silu: out = gelu(x1) * x2, fp32 inside, one rounding. */
+int mv_gelu_and_mul(const void *x, int64_t x_stride, void *out, int64_t out_stride,
+                    int rows, int cols, int dtype, void *stream);
+
+/* K13 — one edge of a residual stream kept in fp32.  Per row, with the stream x [rows][cols] (dense fp32, in place):
+ *     b = x, or (embed_mode 1) nothing;   y' = y, or (y_norm_w) y / sqrt(mean(y^2) + eps) * y_norm_w
+ *     x = b + y' + [embed_mode 1 or 2: embed_scale * embed[ids[row]]] + [vec]
+ *     out = (norm_w) x / sqrt(mean(x^2) + eps) * (norm_offset + norm_w), else x, rounded to dtype   (out NULL: nothing)
+ * y: rows of dtype at stride y_stride, or (y_splits > 0) fp32 partial sums [y_splits][rows][cols]; NULL = nothing.
+ * All weights / tables are of dtype.  Means are over cols_true <= cols columns; the others hold zeros. */
+typedef struct MvResidualArgs {
+  float *x;
+  const void *y, *y_norm_w, *embed;
+  const int64_t *ids;
+  const void *vec, *norm_w;
+  void *out;
+  int64_t y_stride, out_stride, vocab;
+  float embed_scale, norm_offset, eps;
+  int y_splits, embed_mode;
+} MvResidualArgs;
+int mv_residual_update(const MvResidualArgs *args, int rows, int cols, int cols_true, int dtype, void *stream);
+
+/* out[t][j] = gelu(s[t][j]) * table[ids[t]][offset + j] for j < dim, 0 for dim <= j < cols (tanh form of gelu; table
+ * [vocab] rows at table_stride; ids outside the table give zeros). */
+int mv_gated_lookup(const void *s, int64_t s_stride, const void *table, int64_t table_stride, int64_t vocab,
+                    int offset, const int64_t *ids, void *out, int64_t out_stride, int rows, int dim, int cols,
+                    int dtype, void *stream);
 
 /* K10 — decode-sized linear layer: out[m, :] = x[m, :] . W^T (+ bias), 1 <= M <= 64 rows, 16-bit
  * dtypes, fp32 accumulation, one rounding at the end.  Replaces the F.linear calls of the decode step

@@ -11,6 +11,8 @@ from typing import ClassVar
 
 from transformers import AutoConfig, PretrainedConfig
 
+from .native_configs import load_native_config
+
 __all__ = ["Config"]
 
 
@@ -87,6 +89,8 @@ class Config:
                 raise ValueError(f"{name} must be positive, got {getattr(self, name)}")
         self._load_hf_config()
         self._clamp_max_model_len()
+        if getattr(self.hf_config, "max_position_embeddings", 0) is None:
+            self.hf_config.max_position_embeddings = self.max_model_len   # no limit of its own: what the engine serves
         if self.max_num_batched_tokens < self.max_model_len and not self.enable_chunked_prefill:
             raise ValueError(
                 f"max_num_batched_tokens ({self.max_num_batched_tokens}) must be >= max_model_len "
@@ -102,6 +106,9 @@ class Config:
             f"properly downloaded and accessible.")
 
     def _load_hf_config(self) -> None:
+        if self.hf_config is not None:
+            return
+        self.hf_config = load_native_config(self.model)   # architectures no library has a config class for
         if self.hf_config is not None:
             return
         try:
@@ -120,6 +127,8 @@ class Config:
         if self.hf_config is None:
             return
         model_max = getattr(self.hf_config, "max_position_embeddings", self.DEFAULT_MAX_MODEL_LEN)
+        if model_max is None:
+            return
         if (self.max_num_batched_tokens < self.max_model_len and model_max < self.max_model_len
                 and not self.enable_chunked_prefill):
             new_len = min(model_max, self.max_num_batched_tokens)

@@ -132,9 +132,71 @@ __device__ __forceinline__ float wave_max(float x) {
   return x;
 }
 
+// tanh form of gelu: 0.5 z (1 + tanh(u)) = z / (1 + exp(-2 u)), u = sqrt(2/pi) (z + 0.044715 z^3)
+__device__ __forceinline__ float gelu_tanh(float z) {
+  const float u2 = 1.5957691216057308f * (z + 0.044715f * z * z * z);
+  return z / (1.0f + expf(-u2));
+}
+
+// ---- rotary embedding ------------------------------------------------------
+// A head row of D elements lies on LPT = D / VEC adjacent lanes, VEC per lane (sub = lane within the row).  Two layouts:
+//   halves (NeoX):  dim i pairs with dim i + D/2, i < D/2; the partner sits LPT/2 lanes away; cos / sin [max_pos, D/2]
+//   interleaved:    dim 2i pairs with dim 2i + 1, i < pairs, in the same lane; dims from 2 * pairs on pass unchanged;
+//                   cos / sin [max_pos, pairs]
+template <int D, int VEC>
+__device__ __forceinline__ void rot_factors(const float *cos, const float *sin, int64_t pos, bool pos_ok, int sub,
+                                            int pairs, bool interleaved, float (&cs)[VEC], float (&sn)[VEC]) {
+  constexpr int HALF = D / VEC / 2;
+  if (interleaved) {
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+      const int i = (sub * VEC + j) >> 1;
+      const bool ok = pos_ok && i < pairs;
+      cs[j] = ok ? cos[pos * pairs + i] : 1.0f;
+      sn[j] = ok ? sin[pos * pairs + i] : 0.0f;
+    }
+  } else {
+    const int i0 = (sub % HALF) * VEC;
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+      cs[j] = pos_ok ? cos[pos * (D / 2) + i0 + j] : 1.0f;
+      sn[j] = pos_ok ? sin[pos * (D / 2) + i0 + j] : 0.0f;
+    }
+  }
+}
+// y = rotation of x; every product and sum rounded on its own
+template <int D, int VEC>
+__device__ __forceinline__ void rot_apply(const float (&x)[VEC], const float (&cs)[VEC], const float (&sn)[VEC], int sub,
+                                          bool interleaved, float (&y)[VEC]) {
+  constexpr int LPT = D / VEC, HALF = LPT / 2;
+  if (interleaved) {
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+      const float a = __fmul_rn(x[j], cs[j]), b = __fmul_rn(x[j ^ 1], sn[j]);
+      y[j] = (j & 1) ? __fadd_rn(a, b) : __fsub_rn(a, b);
+    }
+  } else {
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+      float other;
+      if constexpr (LPT == 16) other = row_ror<8>(x[j]);
+      else other = __shfl_xor(x[j], HALF, 64);
+      const float a = __fmul_rn(x[j], cs[j]), b = __fmul_rn(other, sn[j]);
+      y[j] = sub < HALF ? __fsub_rn(a, b) : __fadd_rn(a, b);
+    }
+  }
+}
+
 // ---- host-side helpers ------------------------------------------------------
 static inline int mv_check_hip(hipError_t e) { return e == hipSuccess ? 0 : (int)e; }
 static inline bool mv_aligned16(const void *p) { return (((uintptr_t)p) & 15u) == 0; }
+
+// rotary / window options of the attention entry points (NULL = none)
+static inline int mv_check_rot(const MvAttnOpts *o, int head_dim) {
+  if (!o) return MV_OK;
+  if (o->interleaved) return (o->rot_pairs < 0 || o->rot_pairs > head_dim / 2) ? MV_E_SHAPE : MV_OK;
+  return (o->rot_pairs != 0 && o->rot_pairs != head_dim / 2) ? MV_E_SHAPE : MV_OK;   // halves: whole rows only
+}
 
 #define MV_LAUNCH_CHECK()                       \
   do {                                          \

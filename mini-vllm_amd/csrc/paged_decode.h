@@ -34,7 +34,17 @@ struct DecodeParams {
   const void *q_norm_w = nullptr, *k_norm_w = nullptr;
   float eps = 0.f;
   const int32_t *slot_mapping = nullptr;
+  int pairs = 0, interleaved = 0;   // rotary layout (common.h: rot_factors)
+  // chunk > 0: a query at position i reads only the keys of its own chunk of positions, [i / chunk * chunk, i]
+  int chunk = 0;
+  int64_t out_stride = 0;   // elements between token rows of out; 0 = n_heads * D
 };
+
+// first key the query of a sequence with `ctx` tokens (its own included) may read
+__device__ __forceinline__ int decode_first_key(const DecodeParams &p, int ctx) {
+  return p.chunk > 0 && ctx > 0 ? (ctx - 1) / p.chunk * p.chunk : 0;
+}
+
 
 // ---- accesses to bytes that ANOTHER workgroup of the same launch wrote or will read (persistent decode kernel) -------
 // COH = false: plain accesses (one kernel per phase: the kernel boundary makes everything visible).  COH = true: the
@@ -95,11 +105,12 @@ __device__ __forceinline__ void st2(uint16_t *p, uint16_t v) {
 }
 
 // one head row (D elements on LPT lanes, VEC per lane): optional RMSNorm over the row (result rounded to dtype) and
-// the NeoX rotation by (cs, sn) — rope_qk_store_kernel's arithmetic and rounding points, statement for statement
+// the rotation by (cs, sn) — rope_qk_store_kernel's arithmetic and rounding points, statement for statement
 template <typename Tag, int D>
 __device__ __forceinline__ u32x4 norm_rope_row(const u32x4 &raw, const typename elem<Tag>::T *nw, float eps, int sub,
-                                               const float (&cs)[elem<Tag>::VEC], const float (&sn)[elem<Tag>::VEC]) {
-  constexpr int VEC = elem<Tag>::VEC, LPT = D / VEC, HALF = LPT / 2;
+                                               const float (&cs)[elem<Tag>::VEC], const float (&sn)[elem<Tag>::VEC],
+                                               bool interleaved = false) {
+  constexpr int VEC = elem<Tag>::VEC, LPT = D / VEC;
   static_assert(VEC == 8, "16-bit dtypes");
   float x[VEC];
   unpack8<Tag>(raw, x);
@@ -116,15 +127,7 @@ __device__ __forceinline__ u32x4 norm_rope_row(const u32x4 &raw, const typename 
     for (int j = 0; j < VEC; ++j) x[j] = elem<Tag>::ld(elem<Tag>::st(__fmul_rn(__fmul_rn(x[j], rs), w[j])));
   }
   float y[VEC];
-#pragma unroll
-  for (int j = 0; j < VEC; ++j) {
-    float other;
-    if constexpr (LPT == 16) other = row_ror<8>(x[j]);
-    else other = __shfl_xor(x[j], HALF, 64);
-    const float a = __fmul_rn(x[j], cs[j]);
-    const float b = __fmul_rn(other, sn[j]);
-    y[j] = sub < HALF ? __fsub_rn(a, b) : __fadd_rn(a, b);
-  }
+  rot_apply<D, VEC>(x, cs, sn, sub, interleaved, y);
   return pack8<Tag>(y);
 }
 

@@ -20,29 +20,16 @@
 // (The same idea for the matrix-core kernel — a wave per kv head — was measured SLOWER, 94 vs 88 us on Qwen2-7B
 //  heads at B = 256: that kernel is bound by the bytes its 8 resident waves per CU keep in flight, and a wave
 //  that walks twice as many tiles serially keeps no more of them in flight.)
-#include "paged_decode_body.h"
-#include <cstdlib>
+#include "paged_decode_launch.h"
 
 
-__global__ void __launch_bounds__(256) zero_fill_kernel(uint32_t *p, int64_t n) {
+__global__ void __launch_bounds__(256) zero_fill_kernel(uint32_t *p, int64_t n, int64_t row_stride) {
   const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
-  if (i < n) p[i] = 0u;
+  if (i < n) p[blockIdx.y * row_stride + i] = 0u;
 }
 
 // ---- host side -------------------------------------------------------------
 namespace {
-
-struct DecodePlan {
-  int g_chunk;  // q heads served per workgroup (template G)
-  int n_chunks;
-  int nload;
-  int tile;
-  int unit;
-  int nsplit;
-  bool uniform;
-  bool mfma;  // tensor-core variant (paged_decode_mfma.hip)
-  bool wide;  // vector kernel, TPL adjacent kv heads per workgroup (whole-row loads)
-};
 
 constexpr int kTargetWorkgroups = 2048;  // ~8 workgroups per CU
 constexpr int kMaxSplits = 64;
@@ -57,9 +44,9 @@ int pick_g(int g_total) {
 }
 
 bool make_plan(int batch, int n_heads, int n_kv_heads, int head_dim, int block_size,
-               int max_blocks, int dtype, int flags, DecodePlan *pl) {
+               int max_blocks, int dtype, int flags, int chunk, DecodePlan *pl) {
   if (n_kv_heads <= 0 || n_heads % n_kv_heads) return false;
-  if (head_dim != 64 && head_dim != 128) return false;
+  if (head_dim != 64 && head_dim != 128 && head_dim != 256) return false;
   const int g_total = n_heads / n_kv_heads;
   int kv_groups = n_kv_heads;  // workgroups along the kv-head axis
   pl->wide = false;
@@ -86,7 +73,8 @@ bool make_plan(int batch, int n_heads, int n_kv_heads, int head_dim, int block_s
     pl->uniform = block_size % pl->tile == 0;
     if (pl->wide) kv_groups = n_kv_heads / tpl;
   }
-  const int64_t max_ctx = (int64_t)max_blocks * block_size;
+  int64_t max_ctx = (int64_t)max_blocks * block_size;
+  if (chunk > 0 && max_ctx > (int64_t)chunk + pl->unit) max_ctx = (int64_t)chunk + pl->unit;   // (a chunk's edge inside a unit)
   const int max_units = (int)((max_ctx + pl->unit - 1) / pl->unit);
   const int64_t wg = (int64_t)batch * kv_groups * pl->n_chunks;
   // the matrix-core kernel keeps 4 workgroups per CU resident (LDS): one wave of 1024 is enough
@@ -107,89 +95,34 @@ bool make_plan(int batch, int n_heads, int n_kv_heads, int head_dim, int block_s
 
 size_t align256(size_t x) { return (x + 255) & ~(size_t)255; }
 
-template <typename Tag, int D, int G, int NLOAD, bool ROPE>
-void launch_gr(const DecodeParams &p, const DecodePlan &pl, int batch, hipStream_t stream) {
-  dim3 block(256);
-  if constexpr (G <= 4) {
-    if (pl.wide) {
-      dim3 grid(p.n_kv_heads / (64 / (D / elem<Tag>::VEC)), pl.nsplit, batch);
-      if (pl.uniform)
-        hipLaunchKernelGGL((paged_decode_kernel<Tag, D, G, NLOAD, true, true, ROPE>), grid, block, 0, stream, p);
-      else
-        hipLaunchKernelGGL((paged_decode_kernel<Tag, D, G, NLOAD, false, true, ROPE>), grid, block, 0, stream, p);
-      return;
-    }
-  }
-  dim3 grid(p.n_kv_heads * pl.n_chunks, pl.nsplit, batch);
-  if (pl.uniform)
-    hipLaunchKernelGGL((paged_decode_kernel<Tag, D, G, NLOAD, true, false, ROPE>), grid, block, 0, stream, p);
-  else
-    hipLaunchKernelGGL((paged_decode_kernel<Tag, D, G, NLOAD, false, false, ROPE>), grid, block, 0, stream, p);
-}
-
-template <typename Tag, int D, int G, int NLOAD>
-void launch_g(const DecodeParams &p, const DecodePlan &pl, int batch, hipStream_t stream) {
-  if constexpr (elem<Tag>::VEC == 8 && G <= 4) {   // (rope fusion: 16-bit dtypes, up to 4 query heads per kv head)
-    if (p.positions != nullptr) return launch_gr<Tag, D, G, NLOAD, true>(p, pl, batch, stream);
-  }
-  launch_gr<Tag, D, G, NLOAD, false>(p, pl, batch, stream);
-}
-
-template <typename Tag, int D>
-int launch_d(const DecodeParams &p, const DecodePlan &pl, int batch, int dtype, int flags, hipStream_t stream) {
-  if (pl.mfma) {
-    const int klds = (flags & MV_DECODE_KLDS_ON) ? 1 : ((flags & MV_DECODE_KLDS_OFF) ? 0 : -1);
-    const int rc = mv_paged_decode_mfma_launch(p, pl.n_chunks, pl.nsplit, batch, dtype, klds, stream);
-    if (rc != MV_OK) return rc;
-    if (pl.nsplit > 1) {
-      hipLaunchKernelGGL((paged_decode_reduce_kernel<Tag, D>), dim3(batch * p.n_heads), dim3(128), 0,
-                         stream, p.ws_acc, p.ws_ml, (typename elem<Tag>::T *)p.out, pl.nsplit);
-      MV_LAUNCH_CHECK();
-    }
-    return MV_OK;
-  }
-  switch (pl.g_chunk) {
-    case 1: launch_g<Tag, D, 1, 8>(p, pl, batch, stream); break;
-    case 2: launch_g<Tag, D, 2, 8>(p, pl, batch, stream); break;
-    case 3: launch_g<Tag, D, 3, 8>(p, pl, batch, stream); break;
-    case 4: launch_g<Tag, D, 4, 8>(p, pl, batch, stream); break;
-    case 5: launch_g<Tag, D, 5, 4>(p, pl, batch, stream); break;
-    case 6: launch_g<Tag, D, 6, 4>(p, pl, batch, stream); break;
-    case 7: launch_g<Tag, D, 7, 4>(p, pl, batch, stream); break;
-    case 8: launch_g<Tag, D, 8, 4>(p, pl, batch, stream); break;
-    default: return MV_E_SHAPE;
-  }
-  MV_LAUNCH_CHECK();
-  if (pl.nsplit > 1) {
-    hipLaunchKernelGGL((paged_decode_reduce_kernel<Tag, D>), dim3(batch * p.n_heads), dim3(128), 0,
-                       stream, p.ws_acc, p.ws_ml, (typename elem<Tag>::T *)p.out, pl.nsplit);
-    MV_LAUNCH_CHECK();
-  }
-  return MV_OK;
-}
-
 }  // namespace
 
 // the launch plan, for decode_persistent.hip (its attention phase runs the same virtual grid): 0 = ok
 int mv_paged_decode_plan(int batch, int n_heads, int n_kv_heads, int head_dim, int block_size, int max_blocks, int dtype,
                          int flags, int *g_chunk, int *n_chunks, int *nsplit, int *wide, int *mfma, int *uniform) {
   DecodePlan pl;
-  if (!make_plan(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, dtype, flags, &pl)) return MV_E_SHAPE;
+  if (!make_plan(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, dtype, flags, 0, &pl)) return MV_E_SHAPE;
   *g_chunk = pl.g_chunk, *n_chunks = pl.n_chunks, *nsplit = pl.nsplit, *wide = pl.wide, *mfma = pl.mfma, *uniform = pl.uniform;
   return MV_OK;
 }
 
-extern "C" size_t mv_paged_decode_workspace_bytes(int batch, int n_heads, int n_kv_heads,
-                                                  int head_dim, int block_size, int max_blocks, int flags) {
+extern "C" size_t mv_paged_decode_workspace_bytes_ex(int batch, int n_heads, int n_kv_heads, int head_dim, int block_size,
+                                                     int max_blocks, int flags, int chunk) {
   // sized for the widest element type so one buffer serves every dtype
   DecodePlan a, b;
-  if (batch <= 0 || !make_plan(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, MV_BF16, flags, &a) ||
-      !make_plan(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, MV_F32, flags, &b))
+  if (batch <= 0 ||
+      !make_plan(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, MV_BF16, flags, chunk, &a) ||
+      !make_plan(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, MV_F32, flags, chunk, &b))
     return 256;
   const int ns = a.nsplit > b.nsplit ? a.nsplit : b.nsplit;
   if (ns <= 1) return 256;
   const size_t slots = (size_t)batch * n_heads * ns;
   return align256(slots * head_dim * sizeof(float)) + align256(slots * 2 * sizeof(float));
+}
+
+extern "C" size_t mv_paged_decode_workspace_bytes(int batch, int n_heads, int n_kv_heads,
+                                                  int head_dim, int block_size, int max_blocks, int flags) {
+  return mv_paged_decode_workspace_bytes_ex(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, flags, 0);
 }
 
 namespace {
@@ -208,8 +141,21 @@ int paged_decode_impl(const void *q, int64_t q_stride_tok, const void *k_cache,
                       int64_t table_stride, const int32_t *context_lens, void *out,
                       int batch, int n_heads, int n_kv_heads, int head_dim,
                       int block_size, int max_blocks, int64_t num_blocks, float scale,
-                      void *workspace, size_t ws_bytes, int dtype, int flags, void *stream, const RopeArgs *rope);
+                      void *workspace, size_t ws_bytes, int dtype, int flags, void *stream, const RopeArgs *rope,
+                      const MvAttnOpts *opts);
 }  // namespace
+
+extern "C" int mv_paged_decode_ex(const void *q, int64_t q_stride_tok, const void *k_cache,
+                               const void *v_cache, const int32_t *block_tables,
+                               int64_t table_stride, const int32_t *context_lens, void *out,
+                               int batch, int n_heads, int n_kv_heads, int head_dim,
+                               int block_size, int max_blocks, int64_t num_blocks, float scale,
+                               void *workspace, size_t ws_bytes, int dtype, int flags, const MvAttnOpts *opts,
+                               void *stream) {
+  return paged_decode_impl(q, q_stride_tok, k_cache, v_cache, block_tables, table_stride, context_lens, out, batch,
+                           n_heads, n_kv_heads, head_dim, block_size, max_blocks, num_blocks, scale, workspace, ws_bytes,
+                           dtype, flags, stream, nullptr, opts);
+}
 
 extern "C" int mv_paged_decode(const void *q, int64_t q_stride_tok, const void *k_cache,
                                const void *v_cache, const int32_t *block_tables,
@@ -217,9 +163,9 @@ extern "C" int mv_paged_decode(const void *q, int64_t q_stride_tok, const void *
                                int batch, int n_heads, int n_kv_heads, int head_dim,
                                int block_size, int max_blocks, int64_t num_blocks, float scale,
                                void *workspace, size_t ws_bytes, int dtype, int flags, void *stream) {
-  return paged_decode_impl(q, q_stride_tok, k_cache, v_cache, block_tables, table_stride, context_lens, out, batch,
-                           n_heads, n_kv_heads, head_dim, block_size, max_blocks, num_blocks, scale, workspace, ws_bytes,
-                           dtype, flags, stream, nullptr);
+  return mv_paged_decode_ex(q, q_stride_tok, k_cache, v_cache, block_tables, table_stride, context_lens, out, batch,
+                            n_heads, n_kv_heads, head_dim, block_size, max_blocks, num_blocks, scale, workspace, ws_bytes,
+                            dtype, flags, nullptr, stream);
 }
 
 // K7 + K6 (per head) + K1 + K3 in ONE launch for decode steps: q / k / v are the RAW rows of the qkv projection; the
@@ -227,6 +173,34 @@ extern "C" int mv_paged_decode(const void *q, int64_t q_stride_tok, const void *
 // token's K (normed, rotated) and V into the cache (see paged_decode_kernel<ROPE>).  Bit-identical to
 // mv_rope_qk_store followed by mv_paged_decode.  MV_E_SHAPE for layouts the fused form does not take (fp32; more than
 // 16 query heads per kv head): the caller then issues the two launches.
+extern "C" int mv_rope_paged_decode_ex(const void *q, int64_t q_stride_tok, const void *k, int64_t k_stride_tok,
+                                    const void *v, int64_t v_stride_tok, const int64_t *positions, const float *cos,
+                                    const float *sin, int64_t max_pos, const void *q_norm_w, const void *k_norm_w,
+                                    float eps, const int32_t *slot_mapping, void *k_cache, void *v_cache,
+                                    const int32_t *block_tables, int64_t table_stride, const int32_t *context_lens,
+                                    void *out, int batch, int n_heads, int n_kv_heads, int head_dim, int block_size,
+                                    int max_blocks, int64_t num_blocks, float scale, void *workspace, size_t ws_bytes,
+                                    int dtype, int flags, const MvAttnOpts *opts, void *stream) {
+  if (batch == 0) return MV_OK;
+  if (!k || !v || !positions || !cos || !sin || !slot_mapping) return MV_E_NULLPTR;
+  if (dtype != MV_BF16 && dtype != MV_F16) return dtype == MV_F32 ? MV_E_SHAPE : MV_E_DTYPE;
+  if (max_blocks == 0 || num_blocks == 0 || n_kv_heads <= 0 || n_heads % n_kv_heads) return MV_E_SHAPE;
+  if (!mv_aligned16(k) || !mv_aligned16(v) || (k_stride_tok & 7) || (v_stride_tok & 7) ||
+      (q_norm_w && !mv_aligned16(q_norm_w)) || (k_norm_w && !mv_aligned16(k_norm_w)))
+    return MV_E_ALIGN;
+  if (int e = mv_check_rot(opts, head_dim)) return e;
+  DecodePlan pl;
+  if (!make_plan(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, dtype, flags, opts ? opts->chunk : 0, &pl))
+    return MV_E_SHAPE;
+  // vector kernel: up to 4 query heads per kv head; matrix-core kernel: one chunk of <= 16 heads
+  if (pl.n_chunks != 1) return MV_E_SHAPE;
+  if (pl.mfma ? head_dim != 128 : pl.g_chunk > 4) return MV_E_SHAPE;
+  const RopeArgs rope{k, v, k_stride_tok, v_stride_tok, positions, cos, sin, max_pos, q_norm_w, k_norm_w, eps, slot_mapping};
+  return paged_decode_impl(q, q_stride_tok, k_cache, v_cache, block_tables, table_stride, context_lens, out, batch,
+                           n_heads, n_kv_heads, head_dim, block_size, max_blocks, num_blocks, scale, workspace, ws_bytes,
+                           dtype, flags, stream, &rope, opts);
+}
+
 extern "C" int mv_rope_paged_decode(const void *q, int64_t q_stride_tok, const void *k, int64_t k_stride_tok,
                                     const void *v, int64_t v_stride_tok, const int64_t *positions, const float *cos,
                                     const float *sin, int64_t max_pos, const void *q_norm_w, const void *k_norm_w,
@@ -235,22 +209,10 @@ extern "C" int mv_rope_paged_decode(const void *q, int64_t q_stride_tok, const v
                                     void *out, int batch, int n_heads, int n_kv_heads, int head_dim, int block_size,
                                     int max_blocks, int64_t num_blocks, float scale, void *workspace, size_t ws_bytes,
                                     int dtype, int flags, void *stream) {
-  if (batch == 0) return MV_OK;
-  if (!k || !v || !positions || !cos || !sin || !slot_mapping) return MV_E_NULLPTR;
-  if (dtype != MV_BF16 && dtype != MV_F16) return dtype == MV_F32 ? MV_E_SHAPE : MV_E_DTYPE;
-  if (max_blocks == 0 || num_blocks == 0 || n_kv_heads <= 0 || n_heads % n_kv_heads) return MV_E_SHAPE;
-  if (!mv_aligned16(k) || !mv_aligned16(v) || (k_stride_tok & 7) || (v_stride_tok & 7) ||
-      (q_norm_w && !mv_aligned16(q_norm_w)) || (k_norm_w && !mv_aligned16(k_norm_w)))
-    return MV_E_ALIGN;
-  DecodePlan pl;
-  if (!make_plan(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, dtype, flags, &pl)) return MV_E_SHAPE;
-  // vector kernel: up to 4 query heads per kv head; matrix-core kernel: one chunk of <= 16 heads
-  if (pl.n_chunks != 1) return MV_E_SHAPE;
-  if (pl.mfma ? head_dim != 128 : pl.g_chunk > 4) return MV_E_SHAPE;
-  const RopeArgs rope{k, v, k_stride_tok, v_stride_tok, positions, cos, sin, max_pos, q_norm_w, k_norm_w, eps, slot_mapping};
-  return paged_decode_impl(q, q_stride_tok, k_cache, v_cache, block_tables, table_stride, context_lens, out, batch,
-                           n_heads, n_kv_heads, head_dim, block_size, max_blocks, num_blocks, scale, workspace, ws_bytes,
-                           dtype, flags, stream, &rope);
+  return mv_rope_paged_decode_ex(q, q_stride_tok, k, k_stride_tok, v, v_stride_tok, positions, cos, sin, max_pos,
+                                 q_norm_w, k_norm_w, eps, slot_mapping, k_cache, v_cache, block_tables, table_stride,
+                                 context_lens, out, batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks,
+                                 num_blocks, scale, workspace, ws_bytes, dtype, flags, nullptr, stream);
 }
 
 namespace {
@@ -259,7 +221,8 @@ int paged_decode_impl(const void *q, int64_t q_stride_tok, const void *k_cache,
                       int64_t table_stride, const int32_t *context_lens, void *out,
                       int batch, int n_heads, int n_kv_heads, int head_dim,
                       int block_size, int max_blocks, int64_t num_blocks, float scale,
-                      void *workspace, size_t ws_bytes, int dtype, int flags, void *stream, const RopeArgs *rope) {
+                      void *workspace, size_t ws_bytes, int dtype, int flags, void *stream, const RopeArgs *rope,
+                      const MvAttnOpts *opts) {
   if (batch == 0) return MV_OK;
   if (!q || !out || !context_lens) return MV_E_NULLPTR;
   if (batch < 0 || n_heads <= 0 || block_size <= 0 || max_blocks < 0 || num_blocks < 0)
@@ -269,18 +232,21 @@ int paged_decode_impl(const void *q, int64_t q_stride_tok, const void *k_cache,
   if (max_blocks == 0 || num_blocks == 0) {
     // reference: zero-column block tables (warm-up) give zeros, page_attention.py:62-65
     // (a fill kernel: a memset node inside a captured graph has given wrong results on later replays)
-    const int64_t words = (int64_t)batch * n_heads * head_dim * esz / 4;
-    hipLaunchKernelGGL(zero_fill_kernel, dim3((unsigned)((words + 255) / 256)), dim3(256), 0, (hipStream_t)stream,
-                       (uint32_t *)out, words);
+    const int64_t words = (int64_t)n_heads * head_dim * esz / 4, os = opts && opts->out_stride ? opts->out_stride * esz / 4 : words;
+    hipLaunchKernelGGL(zero_fill_kernel, dim3((unsigned)((words + 255) / 256), (unsigned)batch), dim3(256), 0,
+                       (hipStream_t)stream, (uint32_t *)out, words, os);
     MV_LAUNCH_CHECK();
     return MV_OK;
   }
   if (!k_cache || !v_cache || !block_tables) return MV_E_NULLPTR;
   DecodePlan pl;
-  if (!make_plan(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, dtype, flags, &pl))
+  const int chunk = opts ? opts->chunk : 0;
+  const int64_t out_stride = opts && opts->out_stride ? opts->out_stride : (int64_t)n_heads * head_dim;
+  if (chunk < 0 || out_stride < (int64_t)n_heads * head_dim) return MV_E_SHAPE;
+  if (!make_plan(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, dtype, flags, chunk, &pl))
     return MV_E_SHAPE;
   if (!mv_aligned16(q) || !mv_aligned16(k_cache) || !mv_aligned16(v_cache) || !mv_aligned16(out) ||
-      (q_stride_tok * esz) % 16)
+      (q_stride_tok * esz) % 16 || (out_stride * esz) % 16)
     return MV_E_ALIGN;
 
   DecodeParams p;
@@ -300,6 +266,8 @@ int paged_decode_impl(const void *q, int64_t q_stride_tok, const void *k_cache,
   p.bs_shift = (block_size & (block_size - 1)) == 0 ? __builtin_ctz((unsigned)block_size) : -1;
   p.max_blocks = max_blocks;
   p.nsplit = pl.nsplit;
+  p.chunk = chunk;
+  p.out_stride = out_stride;
   p.scale_log2 = scale * 1.4426950408889634f;
   p.ws_acc = nullptr;
   p.ws_ml = nullptr;
@@ -316,8 +284,11 @@ int paged_decode_impl(const void *q, int64_t q_stride_tok, const void *k_cache,
     p.k_new = rope->k_new, p.v_new = rope->v_new, p.k_stride = rope->k_stride, p.v_stride = rope->v_stride;
     p.positions = rope->positions, p.cos = rope->cos, p.sin = rope->sin, p.max_pos = rope->max_pos;
     p.q_norm_w = rope->q_norm_w, p.k_norm_w = rope->k_norm_w, p.eps = rope->eps, p.slot_mapping = rope->slot_mapping;
+    p.interleaved = opts && opts->interleaved;
+    p.pairs = p.interleaved ? opts->rot_pairs : head_dim / 2;
   }
   hipStream_t st = (hipStream_t)stream;
+  if (head_dim == 256) return mv_paged_decode_launch_d256(p, pl, batch, dtype, flags, st);
   if (head_dim == 128) {
     MV_DISPATCH_DTYPE(dtype, return (launch_d<Tag, 128>(p, pl, batch, dtype, flags, st)));
   } else {

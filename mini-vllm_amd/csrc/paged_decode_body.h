@@ -47,6 +47,7 @@ __device__ __forceinline__ float token_sum(float x) {
   x += dpp_mov<0x141>(x);  // row_half_mirror      (other quad of the 8)
   if constexpr (LPT >= 16) x += dpp_mov<0x140>(x);  // row_mirror (other half of the row)
   if constexpr (LPT >= 32) x += __shfl_xor(x, 16, 64);
+  if constexpr (LPT >= 64) x += __shfl_xor(x, 32, 64);
   return x;
 }
 
@@ -97,9 +98,10 @@ __device__ __forceinline__ void paged_decode_body(const DecodeParams &p, const i
   const int64_t cap = (int64_t)p.max_blocks * p.block_size;
   if (ctx > cap) ctx = (int)cap;
   if (ctx < 0) ctx = 0;
-  const int units = (ctx + UNIT - 1) / UNIT;
-  const int ups = (units + p.nsplit - 1) / p.nsplit;
-  const int u_begin = split * ups;
+  const int first = decode_first_key(p, ctx);
+  const int units = (ctx + UNIT - 1) / UNIT, u_first = first / UNIT;
+  const int ups = (units - u_first + p.nsplit - 1) / p.nsplit;
+  const int u_begin = u_first + split * ups;
   const int u_end = min(units, u_begin + ups);
 
   // q fragments: this lane's 16-byte piece of each of the G heads
@@ -116,14 +118,10 @@ __device__ __forceinline__ void paged_decode_body(const DecodeParams &p, const i
     const int64_t pos = p.positions[b];
     const bool pos_ok = pos >= 0 && pos < p.max_pos;
     float cs[VEC], sn[VEC];
-    const int i0 = (sub % (LPT / 2)) * VEC;
+    const bool il = p.interleaved != 0;
+    rot_factors<D, VEC>(p.cos, p.sin, pos, pos_ok, sub, p.pairs, il, cs, sn);
 #pragma unroll
-    for (int j = 0; j < VEC; ++j) {
-      cs[j] = pos_ok ? p.cos[pos * (D / 2) + i0 + j] : 1.0f;
-      sn[j] = pos_ok ? p.sin[pos * (D / 2) + i0 + j] : 0.0f;
-    }
-#pragma unroll
-    for (int g = 0; g < G; ++g) qraw[g] = norm_rope_row<Tag, D>(qraw[g], (const T *)p.q_norm_w, p.eps, sub, cs, sn);
+    for (int g = 0; g < G; ++g) qraw[g] = norm_rope_row<Tag, D>(qraw[g], (const T *)p.q_norm_w, p.eps, sub, cs, sn, il);
     // the workgroup that will read the sequence's last token writes its K / V rows first (one wave; WIDE: its four
     // lane groups are the four kv heads, else lane group 0 has the workgroup's kv head)
     int64_t slot = p.slot_mapping ? (int64_t)p.slot_mapping[b] : -1;
@@ -132,7 +130,7 @@ __device__ __forceinline__ void paged_decode_body(const DecodeParams &p, const i
     if (write && slot >= 0 && u_last >= u_begin && u_last < u_end && wave == 0 && (WIDE || grp == 0)) {
       const u32x4 kraw = ld16<COH>((const T *)p.k_new + (int64_t)b * p.k_stride + (int64_t)hkv * D + sub * VEC);
       const u32x4 vraw = ld16<COH>((const T *)p.v_new + (int64_t)b * p.v_stride + (int64_t)hkv * D + sub * VEC);
-      const u32x4 krot = norm_rope_row<Tag, D>(kraw, (const T *)p.k_norm_w, p.eps, sub, cs, sn);
+      const u32x4 krot = norm_rope_row<Tag, D>(kraw, (const T *)p.k_norm_w, p.eps, sub, cs, sn, il);
       *(MV_AS1 u32x4 *)((T *)p.k_cache + (slot * p.n_kv_heads + hkv) * D + sub * VEC) = krot;
       *(MV_AS1 u32x4 *)((T *)p.v_cache + (slot * p.n_kv_heads + hkv) * D + sub * VEC) = vraw;
       asm volatile("s_waitcnt vmcnt(0)" ::: "memory");   // the rows are in L2 before any wave of the workgroup asks
@@ -171,12 +169,12 @@ __device__ __forceinline__ void paged_decode_body(const DecodeParams &p, const i
       const int off = WIDE ? i : i * TPL + grp;  // token of this lane within the tile
       const int tok = tile_base + off;
       int64_t row;
-      bool ok = tok < ctx;
+      bool ok = tok < ctx && tok >= first;
       if constexpr (UNIFORM) {
         ok = ok && uni_row >= 0;
         row = (uni_row >= 0 ? uni_row : 0) + (ok ? off : 0);
       } else {
-        const int tk = ok ? tok : tile_base;  // tile_base < ctx
+        const int tk = tok < ctx ? tok : tile_base;  // tile_base < ctx
         const int bi = p.bs_shift >= 0 ? (tk >> p.bs_shift) : (tk / p.block_size);
         const int blk = bi < p.max_blocks ? table[bi] : -1;
         const bool blk_ok = blk >= 0 && blk < p.num_blocks;
@@ -294,10 +292,11 @@ __device__ __forceinline__ void paged_decode_body(const DecodeParams &p, const i
       A += lds_acc[w][hg][g][d] * f;
     }
     const int h = (hkv0 + hg) * p.g_total + chunk * G + g;
+    const int64_t os = p.out_stride ? p.out_stride : (int64_t)p.n_heads * D;
     if (p.nsplit == 1) {
       const float o = L > 0.f ? A / L : 0.f;
-      if constexpr (sizeof(T) == 2) st2<COH>((uint16_t *)p.out + ((int64_t)b * p.n_heads + h) * D + d, elem<Tag>::st(o));
-      else ((T *)p.out)[((int64_t)b * p.n_heads + h) * D + d] = elem<Tag>::st(o);
+      if constexpr (sizeof(T) == 2) st2<COH>((uint16_t *)p.out + (int64_t)b * os + h * D + d, elem<Tag>::st(o));
+      else ((T *)p.out)[(int64_t)b * os + h * D + d] = elem<Tag>::st(o);
     } else {
       const int64_t slot = ((int64_t)b * p.n_heads + h) * p.nsplit + split;
       stf<COH>(p.ws_acc + slot * D + d, A);
@@ -399,8 +398,11 @@ template <typename Tag, int D>
 __global__ void __launch_bounds__(128) paged_decode_reduce_kernel(const float *__restrict__ ws_acc,
                                                                   const float *__restrict__ ws_ml,
                                                                   typename elem<Tag>::T *__restrict__ out,
-                                                                  int nsplit) {
+                                                                  int nsplit, int n_heads, int64_t out_stride) {
   __shared__ __attribute__((aligned(16))) float lds[ReduceLds<D>::FLOATS];
-  paged_decode_reduce_body<Tag, D>(ws_acc, ws_ml, out, nsplit, blockIdx.x, threadIdx.x, true, lds);
+  // (the body writes row bh of a dense [B * H, D] array: shift the base so that this row lands in its strided place)
+  const int64_t b = blockIdx.x / n_heads;
+  paged_decode_reduce_body<Tag, D>(ws_acc, ws_ml, out + b * (out_stride - (int64_t)n_heads * D), nsplit, blockIdx.x, threadIdx.x,
+                                   true, lds);
 }
 

@@ -85,9 +85,10 @@ __global__ void __launch_bounds__(256, KLDS ? 2 : 4) paged_decode_mfma_kernel(De
   const int64_t cap = (int64_t)p.max_blocks * p.block_size;
   if (ctx > cap) ctx = (int)cap;
   if (ctx < 0) ctx = 0;
-  const int units = (ctx + UNIT - 1) / UNIT;
-  const int ups = (units + p.nsplit - 1) / p.nsplit;
-  const int u_begin = split * ups;
+  const int first = decode_first_key(p, ctx);
+  const int units = (ctx + UNIT - 1) / UNIT, u_first = first / UNIT;
+  const int ups = (units - u_first + p.nsplit - 1) / p.nsplit;
+  const int u_begin = u_first + split * ups;
   const int u_end = min(units, u_begin + ups);
 
   // Q^T fragments (B operand): lane (q = i16, quad) holds Q[q][32s + 8 quad .. +8)
@@ -130,6 +131,19 @@ __global__ void __launch_bounds__(256, KLDS ? 2 : 4) paged_decode_mfma_kernel(De
         qf[s] = pack8<Tag>(x[s]);
       }
     }
+    if (p.interleaved) {
+      // pairs (2i, 2i+1) sit inside a lane's 8-element fragment: dims 32 s + 8 quad + j, i.e. lane "sub" = 4 s + quad of
+      // rot_apply's row layout
+      const bool live = i16 < g_live;
+#pragma unroll
+      for (int s = 0; s < 4; ++s) {
+        float x[8], cs[8], sn[8], y[8];
+        unpack8<Tag>(qf[s], x);
+        rot_factors<D, 8>(p.cos, p.sin, pos, pos_ok, 4 * s + quad, p.pairs, true, cs, sn);
+        rot_apply<D, 8>(x, cs, sn, 4 * s + quad, true, y);
+        qf[s] = live ? pack8<Tag>(y) : u32x4{0u, 0u, 0u, 0u};
+      }
+    } else {
     // q: dims d = 32 s + 8 quad + j (s = 0, 1) pair with d + 64 (fragment s + 2); products rounded separately, like
     // rope_qk_store_kernel: y[d] = x[d] cos - x[d+64] sin, y[d+64] = x[d+64] cos + x[d] sin
 #pragma unroll
@@ -148,6 +162,7 @@ __global__ void __launch_bounds__(256, KLDS ? 2 : 4) paged_decode_mfma_kernel(De
       qf[s] = live ? pack8<Tag>(ylo) : u32x4{0u, 0u, 0u, 0u};
       qf[s + 2] = live ? pack8<Tag>(yhi) : u32x4{0u, 0u, 0u, 0u};
     }
+    }
     // the new token's K / V rows: written by the workgroup (chunk 0) that will read them, before anybody does
     int64_t slot = p.slot_mapping ? (int64_t)p.slot_mapping[b] : -1;
     if (slot >= p.num_blocks * p.block_size) slot = -1;
@@ -155,15 +170,10 @@ __global__ void __launch_bounds__(256, KLDS ? 2 : 4) paged_decode_mfma_kernel(De
     if (slot >= 0 && chunk == 0 && u_last >= u_begin && u_last < u_end && wave == 0 && lane < 16) {
       const int sub = lane;
       float cs[8], sn[8];
-      const int i0 = (sub % 8) * 8;
-#pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        cs[j] = pos_ok ? p.cos[pos * (D / 2) + i0 + j] : 1.0f;
-        sn[j] = pos_ok ? p.sin[pos * (D / 2) + i0 + j] : 0.0f;
-      }
+      rot_factors<D, 8>(p.cos, p.sin, pos, pos_ok, sub, p.pairs, p.interleaved != 0, cs, sn);
       const u32x4 kraw = *reinterpret_cast<const u32x4 *>((const T *)p.k_new + (int64_t)b * p.k_stride + (int64_t)hkv * D + sub * 8);
       const u32x4 vraw = *reinterpret_cast<const u32x4 *>((const T *)p.v_new + (int64_t)b * p.v_stride + (int64_t)hkv * D + sub * 8);
-      const u32x4 krot = norm_rope_row<Tag, D>(kraw, (const T *)p.k_norm_w, p.eps, sub, cs, sn);
+      const u32x4 krot = norm_rope_row<Tag, D>(kraw, (const T *)p.k_norm_w, p.eps, sub, cs, sn, p.interleaved != 0);
       *reinterpret_cast<u32x4 *>((T *)p.k_cache + (slot * p.n_kv_heads + hkv) * D + sub * 8) = krot;
       *reinterpret_cast<u32x4 *>((T *)p.v_cache + (slot * p.n_kv_heads + hkv) * D + sub * 8) = vraw;
       asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
@@ -259,7 +269,7 @@ __global__ void __launch_bounds__(256, KLDS ? 2 : 4) paged_decode_mfma_kernel(De
       for (int r = 0; r < 4; ++r) {
         const int key = tile_base + 16 * kt + 4 * quad + r;
         float s = sacc[kt][r] * p.scale_log2;
-        s = (blk_ok && key < ctx) ? s : -INFINITY;
+        s = (blk_ok && key < ctx && key >= first) ? s : -INFINITY;
         sacc[kt][r] = s;
         mx = fmaxf(mx, s);
       }
@@ -334,7 +344,8 @@ __global__ void __launch_bounds__(256, KLDS ? 2 : 4) paged_decode_mfma_kernel(De
     }
     const int h = h0 + g;
     if (p.nsplit == 1) {
-      ((T *)p.out)[((int64_t)b * p.n_heads + h) * D + d] = elem<Tag>::st(L > 0.f ? A / L : 0.f);
+      const int64_t os = p.out_stride ? p.out_stride : (int64_t)p.n_heads * D;
+      ((T *)p.out)[(int64_t)b * os + h * D + d] = elem<Tag>::st(L > 0.f ? A / L : 0.f);
     } else {
       const int64_t slot = ((int64_t)b * p.n_heads + h) * p.nsplit + split;
       p.ws_acc[slot * D + d] = A;

@@ -11,9 +11,11 @@ struct PrefillParams {
   int n_seqs, max_seqlen_q, max_seqlen_k;
   int n_heads, n_kv_heads, head_dim, block_size, table_width;
   float scale;
+  int chunk;            // > 0: position i reads only the keys of its chunk of positions, [i / chunk * chunk, i]
+  int64_t out_stride;   // elements between token rows of out
 };
 
-// generic vector-ALU path (every dtype, D in {64,128})
+// generic vector-ALU path (every dtype, D in {64,128,256})
 int mv_prefill_simple_launch(const PrefillParams &p, int64_t max_total_q, int dtype, hipStream_t stream);
 // MFMA flash path (bf16/f16, D in {64,128}); returns MV_E_SHAPE when it does not apply
 // variant: bench switches (flags >> 4 of mv_prefill_varlen), 0 = the shipped kernel

@@ -4,14 +4,14 @@
 // 16-bit tensors and to the vector-ALU kernel otherwise.
 #include "prefill.h"
 
-extern "C" int mv_prefill_varlen(const void *q, int64_t q_stride_tok, const void *k, const void *v,
+extern "C" int mv_prefill_varlen_ex(const void *q, int64_t q_stride_tok, const void *k, const void *v,
                                  int64_t k_stride_tok, int64_t v_stride_tok, const void *k_cache,
                                  const void *v_cache, const int32_t *block_tables,
                                  int64_t table_stride, int64_t num_blocks, void *out,
                                  const int32_t *cu_seqlens_q, const int32_t *cu_seqlens_k,
                                  int n_seqs, int max_seqlen_q, int max_seqlen_k, int n_heads,
                                  int n_kv_heads, int head_dim, int block_size, float scale,
-                                 int dtype, int flags, void *stream) {
+                                 int dtype, int flags, const MvAttnOpts *opts, void *stream) {
   if (n_seqs == 0 || max_seqlen_q == 0) return MV_OK;
   if (!q || !out || !cu_seqlens_q || !cu_seqlens_k) return MV_E_NULLPTR;
   const bool paged = block_tables != nullptr;
@@ -20,10 +20,12 @@ extern "C" int mv_prefill_varlen(const void *q, int64_t q_stride_tok, const void
   if (n_seqs < 0 || max_seqlen_q < 0 || max_seqlen_k < 0 || n_heads <= 0 || n_kv_heads <= 0 ||
       n_heads % n_kv_heads || (paged && (block_size <= 0 || num_blocks <= 0)))
     return MV_E_SHAPE;
-  if (head_dim != 64 && head_dim != 128) return MV_E_SHAPE;
+  if (head_dim != 64 && head_dim != 128 && head_dim != 256) return MV_E_SHAPE;
+  const int64_t out_stride = opts && opts->out_stride ? opts->out_stride : (int64_t)n_heads * head_dim;
+  if (out_stride < (int64_t)n_heads * head_dim || (opts && opts->chunk < 0)) return MV_E_SHAPE;
   if (dtype != MV_BF16 && dtype != MV_F16 && dtype != MV_F32) return MV_E_DTYPE;
   const int esz = dtype == MV_F32 ? 4 : 2;
-  if (!mv_aligned16(q) || !mv_aligned16(out) || (q_stride_tok * esz) % 16 ||
+  if (!mv_aligned16(q) || !mv_aligned16(out) || (q_stride_tok * esz) % 16 || (out_stride * esz) % 16 ||
       (!paged && (!mv_aligned16(k) || !mv_aligned16(v) || (k_stride_tok * esz) % 16 ||
                   (v_stride_tok * esz) % 16)) ||
       (paged && (!mv_aligned16(k_cache) || !mv_aligned16(v_cache))))
@@ -38,6 +40,8 @@ extern "C" int mv_prefill_varlen(const void *q, int64_t q_stride_tok, const void
   p.block_size = block_size;
   p.table_width = paged ? (int)((max_seqlen_k + block_size - 1) / block_size) : 0;
   p.scale = scale;
+  p.chunk = opts ? opts->chunk : 0;
+  p.out_stride = out_stride;
   hipStream_t st = (hipStream_t)stream;
   // MV_PREFILL_SIMPLE routes 16-bit tensors through the vector-ALU kernel (debug aid)
   if (dtype != MV_F32 && !(flags & MV_PREFILL_SIMPLE)) {
@@ -45,4 +49,18 @@ extern "C" int mv_prefill_varlen(const void *q, int64_t q_stride_tok, const void
     if (rc != MV_E_SHAPE) return rc;
   }
   return mv_prefill_simple_launch(p, (int64_t)n_seqs * max_seqlen_q, dtype, st);
+}
+
+extern "C" int mv_prefill_varlen(const void *q, int64_t q_stride_tok, const void *k, const void *v,
+                                 int64_t k_stride_tok, int64_t v_stride_tok, const void *k_cache,
+                                 const void *v_cache, const int32_t *block_tables,
+                                 int64_t table_stride, int64_t num_blocks, void *out,
+                                 const int32_t *cu_seqlens_q, const int32_t *cu_seqlens_k,
+                                 int n_seqs, int max_seqlen_q, int max_seqlen_k, int n_heads,
+                                 int n_kv_heads, int head_dim, int block_size, float scale,
+                                 int dtype, int flags, void *stream) {
+  return mv_prefill_varlen_ex(q, q_stride_tok, k, v, k_stride_tok, v_stride_tok, k_cache, v_cache, block_tables,
+                              table_stride, num_blocks, out, cu_seqlens_q, cu_seqlens_k, n_seqs, max_seqlen_q,
+                              max_seqlen_k, n_heads, n_kv_heads, head_dim, block_size, scale, dtype, flags, nullptr,
+                              stream);
 }

@@ -1,4 +1,4 @@
-// K2 (MFMA path) — packed varlen causal flash attention for gfx950, bf16/f16, D = 128
+// K2 (MFMA path) — packed varlen causal flash attention for gfx950, bf16/f16, D = 64 / 128, whole or chunked context
 // (reference call site: flash_attn_varlen_func, minivllm/models/layers/attention.py:422-433;
 //  semantics of the fallback :467-504,554-597 with bottom-right aligned causal mask).
 //
@@ -114,11 +114,19 @@ __device__ __forceinline__ void half_swap(float x, float &lo, float &hi) {
 // 743 -> 850 TFLOP/s on 4 x 4096 tokens, 28/4 heads.
 // NW = waves per workgroup (32 query rows each): 4 (two workgroups per CU) or 8 (one; the K/V tile and its DMA
 // instructions — ~100 issue cycles apiece — are shared by twice the rows)
-template <typename Tag, int NW, bool PIPE>
+// DH = head dim (64 or 128; the names below shadow the file's D = 128 constants).  CHUNK: position i reads only the keys of its
+// chunk of p.chunk positions: a workgroup starts at the tile of its first row's chunk, a wave skips the tiles in front of its
+// own first row's chunk, and the tiles that hold a chunk's edge take the masked path.
+template <typename Tag, int NW, bool PIPE, int DH, bool CHUNK>
 __global__ void __launch_bounds__(NW * 64, 2) prefill_mfma_kernel(PrefillParams p, float rescale_thr) {
   constexpr int NBUF = 2;   // K|V tile buffers in LDS
+  constexpr int D = DH, NS = D / 16, NDT = D / 32, ROW_BYTES = D * 2, TILE_BYTES = BN * ROW_BYTES;
+  constexpr int CH = D / 8, RPI = 64 / CH;   // 16-byte chunks of a row; rows that one 1-KiB DMA instruction fills
+  // chunk swizzles (XOR) of the K and V tiles: see k_off / v_off; at D = 64 two rows share a 256-byte bank line
+  auto k_swz = [](int row) { return DH == 128 ? (row & 15) : ((row >> 1) & 7); };
+  auto v_swz = [](int row) { return DH == 128 ? (((row & 3) << 2) | ((row >> 2) & 3)) : (((row >> 1) & 1) << 2); };
   constexpr int BM = NW * 32;   // query rows per workgroup
-  constexpr int PP = 16 / NW;   // 1-KiB DMA pieces (4 rows) of a K tile per wave, and as many of the V tile
+  constexpr int PP = TILE_BYTES / 1024 / NW;   // 1-KiB DMA pieces of a K tile per wave, and as many of the V tile
   typedef typename elem<Tag>::T T;
   extern __shared__ __attribute__((aligned(16))) char smem[];
   // two K|V tile buffers: tile t+1 is written while tile t is being read -> ONE barrier per tile
@@ -166,13 +174,18 @@ __global__ void __launch_bounds__(NW * 64, 2) prefill_mfma_kernel(PrefillParams 
   // keys needed by this query block: everything up to its last row's diagonal
   const int q_last = min(sq, (qb + 1) * BM) - 1;
   const int kv_len = min(sk, q_last + shift + 1);
-  const int n_tiles = (kv_len + BN - 1) / BN;
+  // CHUNK: tiles count from the one that holds the first visible key of the workgroup's first row
+  const int kv_base = CHUNK ? (shift + qb * BM) / p.chunk * p.chunk / BN * BN : 0;
+  const int n_tiles = (kv_len - kv_base + BN - 1) / BN;
   const int wave_qpos_min = shift + qb * BM + wave * 32;  // smallest key limit among this wave's rows
   // ... and the largest: tiles that start beyond it are masked out for EVERY row of this wave (the workgroup walks the
   // tiles its LAST wave needs): such a wave skips the tile's arithmetic (p = 0 for all its scores: maximum, sum and
   // accumulator would not move) and only takes part in the DMA and the barrier.  Waves 0..NW-2 save (NW-1-w)/2 tiles
   // each: 5 % of the MFMAs at 4096 tokens, 22 % at 1024, more for short prompts.
   const int wave_qpos_max = wave_qpos_min + 31;
+  // CHUNK: first visible key of the wave's first and last row
+  const int wave_lo_min = CHUNK ? wave_qpos_min / p.chunk * p.chunk : 0;
+  const int wave_lo_max = CHUNK ? wave_qpos_max / p.chunk * p.chunk : 0;
 
   const bool paged = p.block_tables != nullptr;
   const T *ksrc = paged ? (const T *)p.k_cache : (const T *)p.k;
@@ -190,9 +203,9 @@ __global__ void __launch_bounds__(NW * 64, 2) prefill_mfma_kernel(PrefillParams 
   int64_t krel[PP], vrel[PP];
 #pragma unroll
   for (int i = 0; i < PP; ++i) {
-    const int row = 4 * (NW * i + wave) + (lane >> 4), pc = lane & 15;
-    krel[i] = (int64_t)row * kstride + (pc ^ (row & 15)) * 8;
-    vrel[i] = (int64_t)row * vstride + (pc ^ (((row & 3) << 2) | ((row >> 2) & 3))) * 8;
+    const int row = RPI * (NW * i + wave) + lane / CH, pc = lane % CH;
+    krel[i] = (int64_t)row * kstride + (pc ^ k_swz(row)) * 8;
+    vrel[i] = (int64_t)row * vstride + (pc ^ v_swz(row)) * 8;
   }
   bool tile_ok_next = true;
   // (PIPE: through the vector memory path — mbcnt is 0 in every lane but opaque to the compiler — so that no scalar
@@ -204,7 +217,7 @@ __global__ void __launch_bounds__(NW * 64, 2) prefill_mfma_kernel(PrefillParams 
   };
   auto dma = [&](int t, int buf) {
     {
-      const int kv0f = t * BN;
+      const int kv0f = kv_base + t * BN;
       if (kv0f + BN <= sk) {   // a full tile: one scalar base + the per-lane constants
         int64_t base_row = k0 + kv0f;
         tile_ok_next = true;
@@ -227,7 +240,7 @@ __global__ void __launch_bounds__(NW * 64, 2) prefill_mfma_kernel(PrefillParams 
         return;
       }
     }
-    const int kv0 = t * BN;
+    const int kv0 = kv_base + t * BN;
     int64_t base_row = k0 + kv0;
     tile_ok_next = true;
     if (paged) {
@@ -242,12 +255,12 @@ __global__ void __launch_bounds__(NW * 64, 2) prefill_mfma_kernel(PrefillParams 
     char *dk = smem + buf * 2 * TILE_BYTES, *dv = dk + TILE_BYTES;
 #pragma unroll
     for (int i = 0; i < PP; ++i) {
-      // wave `wave`, instruction i fill LDS rows 4 (NW i + wave) .. +3 linearly: lane -> (row, stored chunk)
+      // wave `wave`, instruction i fill RPI LDS rows from RPI (NW i + wave) on linearly: lane -> (row, stored chunk)
       const int wv = wave;
-      const int row = 4 * (NW * i + wv) + (lane >> 4), pc = lane & 15;
+      const int row = RPI * (NW * i + wv) + lane / CH, pc = lane % CH;
       const int srow = min(row, last);
-      const int kch = pc ^ (row & 15);
-      const int vch = pc ^ (((row & 3) << 2) | ((row >> 2) & 3));
+      const int kch = pc ^ k_swz(row);
+      const int vch = pc ^ v_swz(row);
       __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void *)(kt + (int64_t)srow * kstride + kch * 8),
                                        (__attribute__((address_space(3))) void *)(dk + (NW * i + wv) * 1024), 16, 0, 0);
       __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void *)(vt + (int64_t)srow * vstride + vch * 8),
@@ -259,15 +272,15 @@ __global__ void __launch_bounds__(NW * 64, 2) prefill_mfma_kernel(PrefillParams 
   // K, A operand of k-step s: row r (+32 kt), chunk (2s+h) ^ (r & 15)
   int koff[NS];
 #pragma unroll
-  for (int s = 0; s < NS; ++s) koff[s] = r * ROW_BYTES + (((2 * s + h) ^ (r & 15)) << 4);
+  for (int s = 0; s < NS; ++s) koff[s] = r * ROW_BYTES + (((2 * s + h) ^ k_swz(r)) << 4);
   // V^T, A operand of d-tile dt: rows 4h+q4 (+8) (+32 kt + 16 s2), chunk (4dt + 2g + pp/2) ^ swizzle(row)
   const int q4 = i16 >> 2, pp = i16 & 3;
   int voff_lo[NDT], voff_hi[NDT];
 #pragma unroll
   for (int dt = 0; dt < NDT; ++dt) {
     const int ch = 4 * dt + 2 * g + (pp >> 1);
-    voff_lo[dt] = v_off(4 * h + q4, ch) + 8 * (pp & 1);
-    voff_hi[dt] = v_off(4 * h + q4 + 8, ch) + 8 * (pp & 1);
+    voff_lo[dt] = (4 * h + q4) * ROW_BYTES + ((ch ^ v_swz(4 * h + q4)) << 4) + 8 * (pp & 1);
+    voff_hi[dt] = (4 * h + q4 + 8) * ROW_BYTES + ((ch ^ v_swz(4 * h + q4 + 8)) << 4) + 8 * (pp & 1);
   }
 
   bool tile_ok = true;
@@ -338,16 +351,18 @@ __global__ void __launch_bounds__(NW * 64, 2) prefill_mfma_kernel(PrefillParams 
     }
   };
   auto softmax_phase = [&](const int t, const bool tile_ok) __attribute__((always_inline)) {
-    const int kv0 = t * BN;
+    const int kv0 = kv_base + t * BN;
     // ---- mask (only tiles that touch the diagonal / the ragged end: wave-uniform branch)
-    if ((kv0 + BN - 1 > wave_qpos_min) || (kv0 + BN > sk) || !tile_ok) {
+    if ((kv0 + BN - 1 > wave_qpos_min) || (kv0 + BN > sk) || !tile_ok || (CHUNK && kv0 < wave_lo_max)) {
       const int klim = tile_ok ? min(qidx + shift, sk - 1) : -1;  // last key this query row may see
+      // CHUNK: ... and the first.  A chunk is >= 32 positions here, so the wave's 32 rows meet at most one chunk edge
+      const int lane_lo = CHUNK ? (qidx + shift >= wave_lo_max ? wave_lo_max : wave_lo_min) : 0;
 #pragma unroll
       for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
           const int key = kv0 + kt * 32 + (i & 3) + 8 * (i >> 2) + 4 * h;
-          sacc[kt][i] = key <= klim ? sacc[kt][i] : -INFINITY;
+          sacc[kt][i] = key <= klim && (!CHUNK || key >= lane_lo) ? sacc[kt][i] : -INFINITY;
         }
     }
     // ---- online softmax in the log2 domain: p = exp2(s*c - m), one FMA + one exp per score
@@ -408,16 +423,17 @@ __global__ void __launch_bounds__(NW * 64, 2) prefill_mfma_kernel(PrefillParams 
       // group g = (kt, s2) = 16 keys.  ONE set of fragment registers, reused on the fly: the two reads of (g + 1, dt) go
       // out right behind the MFMA that consumed (g, dt), so eight reads stay in flight and the oldest pair is what the
       // next MFMA needs (group 0 was requested behind QK^T)
-      const uint32_t vl[NDT] = {va_lo[0] + add, va_lo[1] + add, va_lo[2] + add, va_lo[3] + add};
-      const uint32_t vh[NDT] = {va_hi[0] + add, va_hi[1] + add, va_hi[2] + add, va_hi[3] + add};
+      uint32_t vl[NDT], vh[NDT];
+#pragma unroll
+      for (int dt = 0; dt < NDT; ++dt) vl[dt] = va_lo[dt] + add, vh[dt] = va_hi[dt] + add;
       auto pv = [&](auto G) __attribute__((always_inline)) {
         constexpr int g = decltype(G)::value;
 #pragma unroll
         for (int dt = 0; dt < NDT; ++dt) {
           if constexpr (g + 1 < 4) lgkm_wait1<2 * NDT - 2>(vlo[0][dt], vhi[0][dt]);
-          else if (dt == 0) lgkm_wait1<6>(vlo[0][dt], vhi[0][dt]);
-          else if (dt == 1) lgkm_wait1<4>(vlo[0][dt], vhi[0][dt]);
-          else if (dt == 2) lgkm_wait1<2>(vlo[0][dt], vhi[0][dt]);
+          else if (dt == NDT - 4) lgkm_wait1<6>(vlo[0][dt], vhi[0][dt]);
+          else if (dt == NDT - 3) lgkm_wait1<4>(vlo[0][dt], vhi[0][dt]);
+          else if (dt == NDT - 2) lgkm_wait1<2>(vlo[0][dt], vhi[0][dt]);
           else lgkm_wait1<0>(vlo[0][dt], vhi[0][dt]);
           const u32x4 a = {vlo[0][dt].x, vlo[0][dt].y, vhi[0][dt].x, vhi[0][dt].y};
           oacc[dt] = mfma<Tag>(a, pf[g >> 1][g & 1], oacc[dt]);
@@ -476,7 +492,7 @@ __global__ void __launch_bounds__(NW * 64, 2) prefill_mfma_kernel(PrefillParams 
   auto tile = [&](const int t, auto BUF) __attribute__((always_inline)) {
     constexpr int BO = decltype(BUF)::value * 2 * TILE_BYTES;   // byte offset of this tile's K|V buffer
     tile_top(t);
-    if (t * BN <= wave_qpos_max) {
+    if (kv_base + t * BN <= wave_qpos_max && (!CHUNK || kv_base + t * BN + BN > wave_lo_min)) {
       qk_phase(std::integral_constant<int, BO>{}, 0u);
       softmax_phase(t, tile_ok);
       pv_phase(std::integral_constant<int, BO>{}, 0u);
@@ -507,17 +523,17 @@ __global__ void __launch_bounds__(NW * 64, 2) prefill_mfma_kernel(PrefillParams 
       u32x2 w;
       w[0] = pack2<Tag>(oacc[dt][4 * c + 0] * inv, oacc[dt][4 * c + 1] * inv);
       w[1] = pack2<Tag>(oacc[dt][4 * c + 2] * inv, oacc[dt][4 * c + 3] * inv);
-      *reinterpret_cast<u32x2 *>(stage + r * ROW_BYTES + (((4 * dt + c) ^ (r & 15)) << 4) + 8 * h) = w;
+      *reinterpret_cast<u32x2 *>(stage + r * ROW_BYTES + (((4 * dt + c) ^ (r & (CH - 1))) << 4) + 8 * h) = w;
     }
   {
-    const int rr = lane >> 4, cc = lane & 15;   // four rows per instruction, sixteen 16-byte chunks per row
+    const int rr = lane / CH, cc = lane % CH;   // RPI rows per instruction, CH 16-byte chunks per row
     const int row0 = qb * BM + wave * 32;
 #pragma unroll
-    for (int it = 0; it < 8; ++it) {
-      const int row = 4 * it + rr;
-      const u32x4 v = *reinterpret_cast<const u32x4 *>(stage + row * ROW_BYTES + ((cc ^ (row & 15)) << 4));
+    for (int it = 0; it < 32 / RPI; ++it) {
+      const int row = RPI * it + rr;
+      const u32x4 v = *reinterpret_cast<const u32x4 *>(stage + row * ROW_BYTES + ((cc ^ (row & (CH - 1))) << 4));
       if (row0 + row < sq && !(rescale_thr <= -2.f && lane != 0)) {   // (thr <= -2: bench ablation, timing only)
-        T *op = (T *)p.out + ((int64_t)(q0 + row0 + row) * p.n_heads + head) * D;
+        T *op = (T *)p.out + (int64_t)(q0 + row0 + row) * p.out_stride + head * D;
         *reinterpret_cast<u32x4 *>(op + 8 * cc) = v;
       }
     }
@@ -951,7 +967,7 @@ __global__ void __launch_bounds__(256, 1) prefill_mfma64_kernel(PrefillParams p,
       w[1] = pack2<Tag>(o_read<base + 2>() * inv, o_read<base + 3>() * inv);
       return w;
     };
-    T *op = (T *)p.out + ((int64_t)(q0 + qidx0 + 32 * b) * p.n_heads + head) * D;
+    T *op = (T *)p.out + (int64_t)(q0 + qidx0 + 32 * b) * p.out_stride + head * D;
     auto row = [&](auto DT) __attribute__((always_inline)) {
       constexpr int dt = decltype(DT)::value;
       const u32x2 w0 = quad(DT, std::integral_constant<int, 0>{}), w1 = quad(DT, std::integral_constant<int, 1>{});
@@ -975,7 +991,8 @@ __global__ void __launch_bounds__(256, 1) prefill_mfma64_kernel(PrefillParams p,
 }  // namespace
 
 int mv_prefill_mfma_launch(const PrefillParams &p, int dtype, int variant, hipStream_t stream) {
-  if (p.head_dim != D || (dtype != MV_BF16 && dtype != MV_F16)) return MV_E_SHAPE;
+  if ((p.head_dim != 64 && p.head_dim != 128) || (dtype != MV_BF16 && dtype != MV_F16)) return MV_E_SHAPE;
+  if (p.chunk > 0 && p.chunk < 32) return MV_E_SHAPE;   // (a handful of keys per query: the vector kernel's job)
   if (p.block_tables && (p.block_size % BN) != 0) return MV_E_SHAPE;  // a 64-key tile must sit in one block
   // 8 waves (256 query rows) per workgroup share a K/V tile where the sequences are long enough that the larger
   // blocks still fill the chip evenly; short prompts keep 4 waves x 2 workgroups per CU (measured per shape,
@@ -992,6 +1009,8 @@ int mv_prefill_mfma_launch(const PrefillParams &p, int dtype, int variant, hipSt
   const int ablate64 = (no_dma ? 1 : 0) | (((variant >> 8) & 3) << 1);   // bench ablations of the 64-rows-per-wave kernel
   const float thr_pick = 6.0f + 2.0f * (float)((variant >> 6) & 3);   // bench switch: rescale threshold 6 / 8 / 10 / 12
   variant &= 7;
+  // the comparison variants (3, 4, 5) exist for whole-context attention at head dim 128
+  if ((p.head_dim != D || p.chunk > 0) && variant > 2) return MV_E_RANGE;
   if (variant == 5) {   // bench switch: 64 query rows per wave, one wave per SIMD (profiles/r03_prefill_kernel.md)
     const int qblocks = (p.max_seqlen_q + 255) / 256;
     if (qblocks == 0 || p.n_seqs == 0) return MV_OK;
@@ -1017,16 +1036,24 @@ int mv_prefill_mfma_launch(const PrefillParams &p, int dtype, int variant, hipSt
   const int q_blocks = (p.max_seqlen_q + bm - 1) / bm;
   if (q_blocks == 0 || p.n_seqs == 0) return MV_OK;
   dim3 grid(p.n_heads, p.n_seqs, q_blocks), block(nw * 64);
-  const size_t lds = 4 * TILE_BYTES;   // 2 x (K tile + V tile) = 64 KiB -> two workgroups per CU
-#define MV_PF_LAUNCH(NWAVES, PIPED)                                                                            \
-  do {                                                                                                        \
-    if (dtype == MV_BF16) hipLaunchKernelGGL((prefill_mfma_kernel<bf16_tag, NWAVES, PIPED>), grid, block, lds, stream, p, thr); \
-    else hipLaunchKernelGGL((prefill_mfma_kernel<f16_tag, NWAVES, PIPED>), grid, block, lds, stream, p, thr);   \
+  const size_t lds = (size_t)4 * BN * p.head_dim * 2;   // 2 x (K tile + V tile): 64 KiB at D = 128 -> two workgroups per CU
+#define MV_PF_LAUNCH(NWAVES, PIPED, DH, CHUNK)                                                                           \
+  do {                                                                                                                  \
+    if (dtype == MV_BF16) hipLaunchKernelGGL((prefill_mfma_kernel<bf16_tag, NWAVES, PIPED, DH, CHUNK>), grid, block, lds, stream, p, thr); \
+    else hipLaunchKernelGGL((prefill_mfma_kernel<f16_tag, NWAVES, PIPED, DH, CHUNK>), grid, block, lds, stream, p, thr);   \
   } while (0)
-  if (nw == 8 && pipe) MV_PF_LAUNCH(8, true);
-  else if (nw == 8) MV_PF_LAUNCH(8, false);
-  else if (pipe) MV_PF_LAUNCH(4, true);
-  else MV_PF_LAUNCH(4, false);
+#define MV_PF_DIMS(NWAVES)                                                   \
+  do {                                                                       \
+    if (p.head_dim == 64 && p.chunk > 0) MV_PF_LAUNCH(NWAVES, true, 64, true);   \
+    else if (p.head_dim == 64) MV_PF_LAUNCH(NWAVES, true, 64, false);          \
+    else if (p.chunk > 0) MV_PF_LAUNCH(NWAVES, true, 128, true);               \
+    else MV_PF_LAUNCH(NWAVES, true, 128, false);                               \
+  } while (0)
+  if (!pipe && nw == 8) MV_PF_LAUNCH(8, false, 128, false);
+  else if (!pipe) MV_PF_LAUNCH(4, false, 128, false);
+  else if (nw == 8) MV_PF_DIMS(8);
+  else MV_PF_DIMS(4);
+#undef MV_PF_DIMS
 #undef MV_PF_LAUNCH
   MV_LAUNCH_CHECK();
   return MV_OK;

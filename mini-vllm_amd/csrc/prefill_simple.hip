@@ -51,7 +51,9 @@ __global__ void __launch_bounds__(256) prefill_simple_kernel(PrefillParams p) {
   while (seq + 1 < p.n_seqs && p.cu_q[seq + 1] <= tok) ++seq;
   const int q0 = p.cu_q[seq], sq = p.cu_q[seq + 1] - q0;
   const int k0 = p.cu_k[seq], sk = p.cu_k[seq + 1] - k0;
-  const int nkeys = min(sk, (tok - q0) + (sk - sq) + 1);  // bottom-right aligned causal
+  const int pos = (tok - q0) + (sk - sq);       // bottom-right aligned causal
+  const int nkeys = min(sk, pos + 1);
+  const int first = p.chunk > 0 ? pos / p.chunk * p.chunk : 0;
 
   const T *qp = (const T *)p.q + (int64_t)tok * p.q_stride + (int64_t)h * D + sub * VEC;
   const u32x4 qraw = *reinterpret_cast<const u32x4 *>(qp);
@@ -60,7 +62,7 @@ __global__ void __launch_bounds__(256) prefill_simple_kernel(PrefillParams p) {
   for (int j = 0; j < VEC; ++j) acc[j] = 0.f;
   const float scale_log2 = p.scale * 1.4426950408889634f;
 
-  for (int base = 0; base < nkeys; base += TPL) {
+  for (int base = first; base < nkeys; base += TPL) {
     const int key = base + grp;
     bool ok = key < nkeys;
     const T *kp = nullptr, *vp = nullptr;
@@ -110,7 +112,7 @@ __global__ void __launch_bounds__(256) prefill_simple_kernel(PrefillParams p) {
     o[j] = ll > 0.f ? a / ll : 0.f;
   }
   if (grp == 0) {
-    T *op = (T *)p.out + ((int64_t)tok * p.n_heads + h) * D + sub * VEC;
+    T *op = (T *)p.out + (int64_t)tok * p.out_stride + h * D + sub * VEC;
     u32x4 packed;
     if constexpr (VEC == 8) packed = pack8<Tag>(o);
     else {
@@ -127,7 +129,9 @@ int mv_prefill_simple_launch(const PrefillParams &p, int64_t max_total_q, int dt
   const int64_t items = max_total_q * p.n_heads;
   if (items == 0) return MV_OK;
   const unsigned blocks = (unsigned)((items + 3) / 4);
-  if (p.head_dim == 128) {
+  if (p.head_dim == 256) {
+    MV_DISPATCH_DTYPE(dtype, hipLaunchKernelGGL((prefill_simple_kernel<Tag, 256>), dim3(blocks), dim3(256), 0, stream, p));
+  } else if (p.head_dim == 128) {
     MV_DISPATCH_DTYPE(dtype, hipLaunchKernelGGL((prefill_simple_kernel<Tag, 128>), dim3(blocks), dim3(256), 0, stream, p));
   } else if (p.head_dim == 64) {
     MV_DISPATCH_DTYPE(dtype, hipLaunchKernelGGL((prefill_simple_kernel<Tag, 64>), dim3(blocks), dim3(256), 0, stream, p));

@@ -1,0 +1,245 @@
+// K13 — steps of a 32-bit residual stream (models whose residual sum stays in fp32 whatever the activation dtype):
+//   mv_residual_update: one launch per edge of the stream — [start the row from a scaled embedding] + the output of the
+//     projections in front (plain, or RMS-normed by a weight of its own; or the fp32 partial sums of a K split)
+//     [+ the scaled embedding] [+ a vector] -> the stream, and what the next projection reads: its RMSNorm or its cast;
+//   mv_gated_lookup: gelu(s) * a slice of a per-token table (the per-token layer input).
+// One workgroup per row, the row in registers between the reductions and the store: the stream is read and written once.
+#include "common.h"
+
+namespace {
+
+struct ResidualParams {
+  float *x;                 // [rows][cols]
+  const void *y;            // [rows] dtype rows (stride y_stride) or, y_splits > 0, fp32 [y_splits][rows][cols]
+  const void *y_norm_w;     // RMS norm of y by a plain weight before it is added; NULL = y as it is
+  const void *embed;        // dtype [vocab][cols]
+  const int64_t *ids;
+  const void *vec;          // dtype [cols], added to every row
+  const void *norm_w;       // out = rms(x) * (norm_offset + norm_w); NULL: out = x rounded to dtype
+  void *out;
+  int64_t y_stride, out_stride, vocab;
+  float embed_scale, norm_offset, eps;
+  int y_splits, embed_mode; // embed_mode: 0 none, 1 the row starts from the embedding, 2 the embedding is added
+  int rows, cols, cols_true;
+};
+
+template <typename Tag>
+__device__ __forceinline__ void load_row_vec(const typename elem<Tag>::T *p, float (&f)[elem<Tag>::VEC]) {
+  const u32x4 raw = *reinterpret_cast<const u32x4 *>(p);
+  if constexpr (elem<Tag>::VEC == 8) {
+    unpack8<Tag>(raw, f);
+  } else {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) f[i] = u2f(raw[i]);
+  }
+}
+template <typename Tag>
+__device__ __forceinline__ void store_row_vec(typename elem<Tag>::T *p, const float (&f)[elem<Tag>::VEC]) {
+  u32x4 raw;
+  if constexpr (elem<Tag>::VEC == 8) {
+    raw = pack8<Tag>(f);
+  } else {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) raw[i] = f2u(f[i]);
+  }
+  *reinterpret_cast<u32x4 *>(p) = raw;
+}
+template <int VEC>
+__device__ __forceinline__ void load_f32(const float *p, float (&f)[VEC]) {
+#pragma unroll
+  for (int q = 0; q < VEC / 4; ++q) {
+    const f32x4 v = *reinterpret_cast<const f32x4 *>(p + 4 * q);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) f[4 * q + e] = v[e];
+  }
+}
+
+// sum over the workgroup, every thread gets it; red: one float per wave
+__device__ __forceinline__ float group_sum(float x, float *red) {
+  x = wave_sum(x);
+  const int nw = blockDim.x >> 6;
+  if (nw == 1) return x;
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = x;
+  __syncthreads();
+  float t = 0.f;
+  for (int i = 0; i < nw; ++i) t += red[i];
+  return t;
+}
+
+// MAXV = vectors per thread
+template <typename Tag, int MAXV>
+__global__ void __launch_bounds__(1024) residual_update_kernel(ResidualParams p) {
+  typedef typename elem<Tag>::T T;
+  constexpr int VEC = elem<Tag>::VEC;
+  __shared__ float red[2][16];
+  const int row = blockIdx.x, nvec = p.cols / VEC;
+  float x[MAXV][VEC], y[MAXV][VEC], e[MAXV][VEC], vv[MAXV][VEC], wy[MAXV][VEC], wn[MAXV][VEC];
+  bool embed_ok = false;
+  int64_t id = 0;
+  if (p.embed_mode) {
+    id = p.ids[row];
+    embed_ok = id >= 0 && id < p.vocab;
+  }
+  // every load of the row before the first reduction
+#pragma unroll
+  for (int i = 0; i < MAXV; ++i) {
+    const int c = (threadIdx.x + i * blockDim.x) * VEC;
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) x[i][j] = y[i][j] = e[i][j] = vv[i][j] = wy[i][j] = wn[i][j] = 0.f;
+    if (c < p.cols) {
+      if (p.embed_mode != 1) load_f32<VEC>(p.x + (int64_t)row * p.cols + c, x[i]);
+      if (p.y) {
+        if (p.y_splits > 0) {
+          const float *pp = (const float *)p.y + (int64_t)row * p.cols + c;
+          load_f32<VEC>(pp, y[i]);
+          for (int s = 1; s < p.y_splits; ++s) {
+            float t[VEC];
+            load_f32<VEC>(pp + (int64_t)s * p.rows * p.cols, t);
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) y[i][j] += t[j];
+          }
+        } else {
+          load_row_vec<Tag>((const T *)p.y + (int64_t)row * p.y_stride + c, y[i]);
+        }
+        if (p.y_norm_w) load_row_vec<Tag>((const T *)p.y_norm_w + c, wy[i]);
+      }
+      if (embed_ok) load_row_vec<Tag>((const T *)p.embed + id * p.cols + c, e[i]);
+      if (p.vec) load_row_vec<Tag>((const T *)p.vec + c, vv[i]);
+      if (p.norm_w) load_row_vec<Tag>((const T *)p.norm_w + c, wn[i]);
+    }
+  }
+  if (p.y_norm_w) {
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < MAXV; ++i)
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) ss = fmaf(y[i][j], y[i][j], ss);
+    ss = group_sum(ss, red[0]);
+    const float rs = 1.0f / sqrtf(ss / (float)p.cols_true + p.eps);
+#pragma unroll
+    for (int i = 0; i < MAXV; ++i)
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) y[i][j] = y[i][j] * rs * wy[i][j];
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < MAXV; ++i) {
+    const int c = (threadIdx.x + i * blockDim.x) * VEC;
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+      x[i][j] = x[i][j] + y[i][j] + e[i][j] * p.embed_scale + vv[i][j];
+      ss = fmaf(x[i][j], x[i][j], ss);
+    }
+    if (c < p.cols) {
+      float *xr = p.x + (int64_t)row * p.cols + c;
+#pragma unroll
+      for (int q = 0; q < VEC / 4; ++q)
+        *reinterpret_cast<f32x4 *>(xr + 4 * q) = f32x4{x[i][4 * q], x[i][4 * q + 1], x[i][4 * q + 2], x[i][4 * q + 3]};
+    }
+  }
+  if (!p.out) return;
+  float rs = 1.0f;
+  if (p.norm_w) {
+    ss = group_sum(ss, red[1]);
+    rs = 1.0f / sqrtf(ss / (float)p.cols_true + p.eps);
+  }
+#pragma unroll
+  for (int i = 0; i < MAXV; ++i) {
+    const int c = (threadIdx.x + i * blockDim.x) * VEC;
+    if (c < p.cols) {
+      float o[VEC];
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) o[j] = p.norm_w ? x[i][j] * rs * (p.norm_offset + wn[i][j]) : x[i][j];
+      store_row_vec<Tag>((T *)p.out + (int64_t)row * p.out_stride + c, o);
+    }
+  }
+}
+
+// out[t][j] = gelu(s[t][j]) * table[ids[t]][offset + j] for j < dim, 0 for dim <= j < cols
+template <typename Tag>
+__global__ void __launch_bounds__(256) gated_lookup_kernel(const typename elem<Tag>::T *s, int64_t s_stride,
+                                                           const typename elem<Tag>::T *table, int64_t table_stride,
+                                                           int64_t vocab, int offset, const int64_t *ids,
+                                                           typename elem<Tag>::T *out, int64_t out_stride, int rows,
+                                                           int dim, int cols, bool table_vec) {
+  constexpr int VEC = elem<Tag>::VEC;
+  const int nvec = cols / VEC;
+  const int64_t n = (int64_t)rows * nvec;
+  for (int64_t v = (int64_t)blockIdx.x * 256 + threadIdx.x; v < n; v += (int64_t)gridDim.x * 256) {
+    const int row = (int)(v / nvec), c = (int)(v - (int64_t)row * nvec) * VEC;
+    const int64_t id = ids[row];
+    const bool ok = id >= 0 && id < vocab;
+    float a[VEC], e[VEC], o[VEC];
+    load_row_vec<Tag>(s + (int64_t)row * s_stride + c, a);
+    const typename elem<Tag>::T *tr = table + (ok ? id : 0) * table_stride + offset + c;
+    if (table_vec && c + VEC <= dim) {
+      load_row_vec<Tag>(tr, e);
+    } else {
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) e[j] = c + j < dim ? elem<Tag>::ld(tr[j]) : 0.f;
+    }
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) o[j] = ok && c + j < dim ? gelu_tanh(a[j]) * e[j] : 0.f;
+    store_row_vec<Tag>(out + (int64_t)row * out_stride + c, o);
+  }
+}
+
+}  // namespace
+
+extern "C" int mv_residual_update(const MvResidualArgs *a, int rows, int cols, int cols_true, int dtype, void *stream) {
+  if (rows == 0) return MV_OK;
+  if (!a || !a->x) return MV_E_NULLPTR;
+  if (rows < 0 || cols <= 0 || cols_true <= 0 || cols_true > cols || a->y_splits < 0) return MV_E_SHAPE;
+  if (dtype != MV_BF16 && dtype != MV_F16 && dtype != MV_F32) return MV_E_DTYPE;
+  if (a->embed_mode < 0 || a->embed_mode > 2) return MV_E_RANGE;
+  if (a->embed_mode && (!a->embed || !a->ids || a->vocab <= 0)) return MV_E_NULLPTR;
+  if (a->y_norm_w && !a->y) return MV_E_NULLPTR;
+  const int vec = dtype == MV_F32 ? 4 : 8;
+  if (cols % vec) return MV_E_SHAPE;
+  if (!mv_aligned16(a->x) || (a->y && !mv_aligned16(a->y)) || (a->y_norm_w && !mv_aligned16(a->y_norm_w)) ||
+      (a->embed_mode && !mv_aligned16(a->embed)) || (a->vec && !mv_aligned16(a->vec)) ||
+      (a->norm_w && !mv_aligned16(a->norm_w)) || (a->out && (!mv_aligned16(a->out) || a->out_stride % vec)) ||
+      (a->y && a->y_splits == 0 && a->y_stride % vec))
+    return MV_E_ALIGN;
+  ResidualParams p;
+  p.x = a->x, p.y = a->y, p.y_norm_w = a->y_norm_w, p.embed = a->embed, p.ids = a->ids, p.vec = a->vec;
+  p.norm_w = a->norm_w, p.out = a->out, p.y_stride = a->y_stride, p.out_stride = a->out_stride, p.vocab = a->vocab;
+  p.embed_scale = a->embed_scale, p.norm_offset = a->norm_offset, p.eps = a->eps;
+  p.y_splits = a->y_splits, p.embed_mode = a->embed_mode, p.rows = rows, p.cols = cols, p.cols_true = cols_true;
+  const int nvec = cols / vec;
+  int threads = (nvec + 63) / 64 * 64;
+  if (threads > 1024) threads = 1024;
+  const int per = (nvec + threads - 1) / threads;
+  hipStream_t st = (hipStream_t)stream;
+#define MV_RES(MV) \
+  MV_DISPATCH_DTYPE(dtype, hipLaunchKernelGGL((residual_update_kernel<Tag, MV>), dim3(rows), dim3(threads), 0, st, p))
+  if (per <= 1) MV_RES(1)
+  else if (per <= 2) MV_RES(2)
+  else return MV_E_SHAPE;   // > 16384 (16-bit) / 8192 (fp32) columns
+#undef MV_RES
+  MV_LAUNCH_CHECK();
+  return MV_OK;
+}
+
+extern "C" int mv_gated_lookup(const void *s, int64_t s_stride, const void *table, int64_t table_stride, int64_t vocab,
+                               int offset, const int64_t *ids, void *out, int64_t out_stride, int rows, int dim, int cols,
+                               int dtype, void *stream) {
+  if (rows == 0) return MV_OK;
+  if (!s || !table || !ids || !out) return MV_E_NULLPTR;
+  if (rows < 0 || dim <= 0 || cols < dim || vocab <= 0 || offset < 0 || offset + dim > table_stride) return MV_E_SHAPE;
+  if (dtype != MV_BF16 && dtype != MV_F16 && dtype != MV_F32) return MV_E_DTYPE;
+  const int vec = dtype == MV_F32 ? 4 : 8;
+  if (cols % vec) return MV_E_SHAPE;
+  if (!mv_aligned16(s) || !mv_aligned16(out) || s_stride % vec || out_stride % vec) return MV_E_ALIGN;
+  const bool table_vec = mv_aligned16(table) && table_stride % vec == 0 && offset % vec == 0;
+  int64_t blocks = ((int64_t)rows * (cols / vec) + 255) / 256;
+  if (blocks > 8192) blocks = 8192;
+  MV_DISPATCH_DTYPE(dtype, {
+    typedef typename elem<Tag>::T T;
+    hipLaunchKernelGGL((gated_lookup_kernel<Tag>), dim3((unsigned)blocks), dim3(256), 0, (hipStream_t)stream, (const T *)s,
+                       s_stride, (const T *)table, table_stride, vocab, offset, ids, (T *)out, out_stride, rows, dim, cols,
+                       table_vec);
+  });
+  MV_LAUNCH_CHECK();
+  return MV_OK;
+}

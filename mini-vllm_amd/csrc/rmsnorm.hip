@@ -202,10 +202,11 @@ extern "C" int mv_add_rmsnorm_partial(const float *partial, int splits, void *re
   return MV_OK;
 }
 
-// K9 — SiluAndMul (reference: minivllm/models/layers/activation.py:70-96).
+// K9 — SiluAndMul (reference: minivllm/models/layers/activation.py:70-96) and, GELU, the tanh form of gelu in its place
+// (one rounding: gelu(x1) * x2 in fp32).
 // The reference rounds silu(x1) to the activation dtype before the multiply;
 // the same two rounding points are kept here.
-template <typename Tag>
+template <typename Tag, bool GELU>
 __global__ void __launch_bounds__(256)
 silu_and_mul_kernel(const typename elem<Tag>::T *__restrict__ x, int64_t x_stride,
                     typename elem<Tag>::T *__restrict__ out, int64_t out_stride, int rows, int cols) {
@@ -238,9 +239,13 @@ silu_and_mul_kernel(const typename elem<Tag>::T *__restrict__ x, int64_t x_strid
           float y[VEC];
 #pragma unroll
           for (int j = 0; j < VEC; ++j) {
-            float s = a[u][j] / (1.0f + expf(-a[u][j]));
-            s = elem<Tag>::ld(elem<Tag>::st(s));
-            y[j] = __fmul_rn(s, b[u][j]);
+            if constexpr (GELU) {
+              y[j] = __fmul_rn(gelu_tanh(a[u][j]), b[u][j]);
+            } else {
+              float s = a[u][j] / (1.0f + expf(-a[u][j]));
+              s = elem<Tag>::ld(elem<Tag>::st(s));
+              y[j] = __fmul_rn(s, b[u][j]);
+            }
           }
           store_vec<Tag>(orow + c * VEC, y);
         }
@@ -249,8 +254,9 @@ silu_and_mul_kernel(const typename elem<Tag>::T *__restrict__ x, int64_t x_strid
   }
 }
 
-extern "C" int mv_silu_and_mul(const void *x, int64_t x_stride, void *out, int64_t out_stride,
-                               int rows, int cols, int dtype, void *stream) {
+template <bool GELU>
+static int act_and_mul(const void *x, int64_t x_stride, void *out, int64_t out_stride, int rows, int cols, int dtype,
+                       void *stream) {
   if (rows == 0) return MV_OK;
   if (!x || !out) return MV_E_NULLPTR;
   if (rows < 0 || cols <= 0) return MV_E_SHAPE;
@@ -266,9 +272,19 @@ extern "C" int mv_silu_and_mul(const void *x, int64_t x_stride, void *out, int64
     if (bx < 1) bx = 1;
     int by = rows < 65535 ? rows : 65535;
     while ((int64_t)bx * by > 16384 && by > 1) by = (by + 1) / 2;
-    hipLaunchKernelGGL((silu_and_mul_kernel<Tag>), dim3((unsigned)bx, (unsigned)by), dim3(256), 0,
+    hipLaunchKernelGGL((silu_and_mul_kernel<Tag, GELU>), dim3((unsigned)bx, (unsigned)by), dim3(256), 0,
                        (hipStream_t)stream, (const T *)x, x_stride, (T *)out, out_stride, rows, cols);
   });
   MV_LAUNCH_CHECK();
   return MV_OK;
+}
+
+extern "C" int mv_silu_and_mul(const void *x, int64_t x_stride, void *out, int64_t out_stride,
+                               int rows, int cols, int dtype, void *stream) {
+  return act_and_mul<false>(x, x_stride, out, out_stride, rows, cols, dtype, stream);
+}
+
+extern "C" int mv_gelu_and_mul(const void *x, int64_t x_stride, void *out, int64_t out_stride,
+                               int rows, int cols, int dtype, void *stream) {
+  return act_and_mul<true>(x, x_stride, out, out_stride, rows, cols, dtype, stream);
 }

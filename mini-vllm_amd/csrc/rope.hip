@@ -1,4 +1,4 @@
-// K7 (+ per-head K6, + K1) — q/k head RMSNorm -> NeoX rotary embedding ->
+// K7 (+ per-head K6, + K1) — q/k head RMSNorm -> rotary embedding (NeoX halves or interleaved pairs) ->
 // K/V cache store in ONE launch
 // (reference: minivllm/models/qwen_base.py:173-190 flat path,
 //  layers/layernorm.py:81-93, layers/rotary_embedding.py:77-81,166-193,
@@ -23,6 +23,7 @@ struct RopeParams {
   const int32_t *slot_mapping;
   int64_t num_slots;
   int n_heads, n_kv_heads;
+  int pairs, interleaved;   // rotary layout (common.h: rot_factors)
 };
 
 template <int LPT>
@@ -37,7 +38,6 @@ __global__ void __launch_bounds__(256) rope_qk_store_kernel(RopeParams p) {
   typedef typename elem<Tag>::T T;
   constexpr int VEC = elem<Tag>::VEC;
   constexpr int LPT = D / VEC;
-  constexpr int HALF = LPT / 2;
   const int tok = blockIdx.x;
   const int sub = threadIdx.x % LPT;
   const int rows_per_iter = blockDim.x / LPT;
@@ -50,14 +50,7 @@ __global__ void __launch_bounds__(256) rope_qk_store_kernel(RopeParams p) {
   const int64_t pos = p.positions[tok];
   const bool pos_ok = pos >= 0 && pos < p.max_pos;
   float cs[VEC], sn[VEC];
-  {
-    const int i0 = (sub % HALF) * VEC;
-#pragma unroll
-    for (int j = 0; j < VEC; ++j) {
-      cs[j] = pos_ok ? p.cos[pos * (D / 2) + i0 + j] : 1.0f;
-      sn[j] = pos_ok ? p.sin[pos * (D / 2) + i0 + j] : 0.0f;
-    }
-  }
+  rot_factors<D, VEC>(p.cos, p.sin, pos, pos_ok, sub, p.pairs, p.interleaved != 0, cs, sn);
 
   for (int r = threadIdx.x / LPT; r < total_rows; r += rows_per_iter) {
     if (r >= H + HKV) {  // raw V row -> cache
@@ -99,15 +92,7 @@ __global__ void __launch_bounds__(256) rope_qk_store_kernel(RopeParams p) {
         x[j] = elem<Tag>::ld(elem<Tag>::st(__fmul_rn(__fmul_rn(x[j], rs), w[j])));
     }
     float y[VEC];
-#pragma unroll
-    for (int j = 0; j < VEC; ++j) {
-      float other;
-      if constexpr (LPT == 16) other = row_ror<8>(x[j]);
-      else other = __shfl_xor(x[j], HALF, 64);
-      const float a = __fmul_rn(x[j], cs[j]);
-      const float b = __fmul_rn(other, sn[j]);
-      y[j] = sub < HALF ? __fsub_rn(a, b) : __fadd_rn(a, b);
-    }
+    rot_apply<D, VEC>(x, cs, sn, sub, p.interleaved != 0, y);
     u32x4 packed;
     if constexpr (VEC == 8) packed = pack8<Tag>(y);
     else {
@@ -130,21 +115,22 @@ __global__ void __launch_bounds__(256) rope_qk_store_kernel(RopeParams p) {
   }
 }
 
-extern "C" int mv_rope_qk_store(const void *q, const void *k, const void *v, int64_t q_stride_tok,
+extern "C" int mv_rope_qk_store_ex(const void *q, const void *k, const void *v, int64_t q_stride_tok,
                                 int64_t k_stride_tok, int64_t v_stride_tok,
                                 const int64_t *positions, const float *cos, const float *sin,
                                 int64_t max_pos, const void *q_norm_w, const void *k_norm_w,
                                 float eps, void *q_out, void *k_out, void *k_cache, void *v_cache,
                                 const int32_t *slot_mapping, int64_t num_slots, int n_tok,
                                 int n_heads, int n_kv_heads, int head_dim, int dtype,
-                                void *stream) {
+                                const MvAttnOpts *opts, void *stream) {
   if (n_tok == 0) return MV_OK;
   if (!q || !k || !positions || !cos || !sin || !q_out) return MV_E_NULLPTR;
   if ((q_norm_w == nullptr) != (k_norm_w == nullptr)) return MV_E_NULLPTR;
   const bool has_cache = k_cache != nullptr || v_cache != nullptr || slot_mapping != nullptr;
   if (has_cache && (!k_cache || !v_cache || !slot_mapping || !v)) return MV_E_NULLPTR;
   if (n_tok < 0 || n_heads <= 0 || n_kv_heads <= 0 || max_pos <= 0) return MV_E_SHAPE;
-  if (head_dim != 64 && head_dim != 128) return MV_E_SHAPE;
+  if (head_dim != 64 && head_dim != 128 && head_dim != 256) return MV_E_SHAPE;
+  if (int e = mv_check_rot(opts, head_dim)) return e;
   if (dtype != MV_BF16 && dtype != MV_F16 && dtype != MV_F32) return MV_E_DTYPE;
   const int esz = dtype == MV_F32 ? 4 : 2;
   if (!mv_aligned16(q) || !mv_aligned16(k) || !mv_aligned16(q_out) ||
@@ -164,12 +150,29 @@ extern "C" int mv_rope_qk_store(const void *q, const void *k, const void *v, int
   p.slot_mapping = has_cache ? slot_mapping : nullptr;
   p.num_slots = num_slots;
   p.n_heads = n_heads; p.n_kv_heads = n_kv_heads;
+  p.interleaved = opts && opts->interleaved;
+  p.pairs = p.interleaved ? opts->rot_pairs : head_dim / 2;
   hipStream_t st = (hipStream_t)stream;
-  if (head_dim == 128) {
+  if (head_dim == 256) {
+    MV_DISPATCH_DTYPE(dtype, hipLaunchKernelGGL((rope_qk_store_kernel<Tag, 256>), dim3(n_tok), dim3(256), 0, st, p));
+  } else if (head_dim == 128) {
     MV_DISPATCH_DTYPE(dtype, hipLaunchKernelGGL((rope_qk_store_kernel<Tag, 128>), dim3(n_tok), dim3(256), 0, st, p));
   } else {
     MV_DISPATCH_DTYPE(dtype, hipLaunchKernelGGL((rope_qk_store_kernel<Tag, 64>), dim3(n_tok), dim3(256), 0, st, p));
   }
   MV_LAUNCH_CHECK();
   return MV_OK;
+}
+
+extern "C" int mv_rope_qk_store(const void *q, const void *k, const void *v, int64_t q_stride_tok,
+                                int64_t k_stride_tok, int64_t v_stride_tok,
+                                const int64_t *positions, const float *cos, const float *sin,
+                                int64_t max_pos, const void *q_norm_w, const void *k_norm_w,
+                                float eps, void *q_out, void *k_out, void *k_cache, void *v_cache,
+                                const int32_t *slot_mapping, int64_t num_slots, int n_tok,
+                                int n_heads, int n_kv_heads, int head_dim, int dtype,
+                                void *stream) {
+  return mv_rope_qk_store_ex(q, k, v, q_stride_tok, k_stride_tok, v_stride_tok, positions, cos, sin, max_pos, q_norm_w,
+                             k_norm_w, eps, q_out, k_out, k_cache, v_cache, slot_mapping, num_slots, n_tok, n_heads,
+                             n_kv_heads, head_dim, dtype, nullptr, stream);
 }

@@ -154,6 +154,17 @@ class BlockManager:
             # byte-identical.
             sequence.num_cached_tokens -= self.block_size
 
+    def reserve(self, sequence: Sequence) -> None:
+        """Grow the block table to cover every token of the sequence with blocks of its own (no digest is looked up or
+        published): for a sequence whose tokens arrive in portions.  All or nothing."""
+        need = sequence.num_blocks - len(sequence.block_table)
+        if need > len(self._free_set):
+            raise RuntimeError(f"No free blocks available: {need} needed, {len(self._free_set)} free")
+        for _ in range(need):
+            block_id = self._get_any_free_block()
+            self._take(block_id)
+            sequence.block_table.append(block_id)
+
     def deallocate(self, sequence: Sequence) -> None:
         for block_id in reversed(sequence.block_table):
             block = self.blocks[block_id]

@@ -45,6 +45,12 @@ def graph_batch_sizes(max_batch_size: int) -> list[int]:
     return sizes
 
 
+def kv_planes(model) -> list[tuple[int, int, int, int]]:
+    """(query heads, kv heads, head dim, chunk) of every attention module that owns a K and a V plane, in cache order."""
+    return [(m.num_heads, m.num_kv_heads, m.head_dim, getattr(m, "chunk", 0)) for m in model.modules()
+            if hasattr(m, "k_cache") and hasattr(m, "v_cache")]
+
+
 def kv_block_bytes(num_layers: int, block_size: int, num_kv_heads_local: int, head_dim: int, itemsize: int) -> int:
     return 2 * num_layers * block_size * num_kv_heads_local * head_dim * itemsize
 
@@ -61,6 +67,13 @@ class InferenceExecutor:
         self.num_kv_heads = max(total_kv // tp, 1)
         self.head_dim = getattr(hf, "head_dim", None) or hf.hidden_size // hf.num_attention_heads
         self.num_layers = hf.num_hidden_layers
+        # layers whose K/V planes differ in shape (heads, head dim) are allocated plane by plane
+        planes = kv_planes(model) if isinstance(model, torch.nn.Module) else []
+        self.kv_shapes = [(hkv, d) for _, hkv, d, _ in planes]
+        if not self.kv_shapes or set(self.kv_shapes) == {(self.num_kv_heads, self.head_dim)}:
+            self.kv_shapes = []          # uniform: one [2, L, blocks, block_size, Hkv, D] tensor
+            self.num_layers = len(planes) or self.num_layers
+        self.attn_shapes = sorted({(h, hkv, d, c) for h, hkv, d, c in planes})
         try:
             self.dtype = next(model.parameters()).dtype
         except (StopIteration, AttributeError):
@@ -120,6 +133,11 @@ class InferenceExecutor:
         self._optimize_model()
         self._warmup_model(max_num_batched_tokens, max_num_seqs)
 
+    def _block_bytes(self) -> int:
+        if self.kv_shapes:
+            return sum(kv_block_bytes(1, self.block_size, hkv, d, self.dtype.itemsize) for hkv, d in self.kv_shapes)
+        return kv_block_bytes(self.num_layers, self.block_size, self.num_kv_heads, self.head_dim, self.dtype.itemsize)
+
     def _calculate_num_kv_blocks(self) -> int:
         """blocks = min(avail // block_bytes, max_num_seqs * ceil(max_model_len / bs)) with
         avail = total*util - used - peak + current (inference_executor.py:245-318)."""
@@ -128,8 +146,7 @@ class InferenceExecutor:
         stats = torch.cuda.memory_stats(self.device)
         peak = stats.get("allocated_bytes.all.peak", 0)
         current = stats.get("allocated_bytes.all.current", 0)
-        block_bytes = kv_block_bytes(self.num_layers, self.block_size, self.num_kv_heads, self.head_dim,
-                                     self.dtype.itemsize)
+        block_bytes = self._block_bytes()
         avail = int(total * cfg.device_memory_utilization - (total - free) - peak + current)
         if avail <= 0:
             raise RuntimeError(f"Insufficient memory for KV cache allocation. Device: {self.device.type}, "
@@ -154,6 +171,8 @@ class InferenceExecutor:
             n = self._calculate_num_kv_blocks()
             self.config.num_kvcache_blocks = n  # the scheduler's BlockManager is sized from this
         shape = (2, self.num_layers, n, self.block_size, self.num_kv_heads, self.head_dim)
+        if self.kv_shapes:   # K plane, V plane of each module, one behind the other
+            shape = (n * self._block_bytes() // self.dtype.itemsize,)
         try:
             self.kv_cache = torch.empty(shape, device=self.device, dtype=self.dtype)
         except torch.cuda.OutOfMemoryError as e:
@@ -164,9 +183,15 @@ class InferenceExecutor:
                     self.kv_cache.numel() * self.kv_cache.element_size() / 2**30, n, self.block_size)
 
     def _assign_kv_cache_to_layers(self) -> None:
-        layer = 0
+        layer, at = 0, 0
         for module in self.model.modules():
             if hasattr(module, "k_cache") and hasattr(module, "v_cache"):
+                if self.kv_shapes:
+                    shape = (2, self.config.num_kvcache_blocks, self.block_size, *self.kv_shapes[layer])
+                    size = 2 * shape[1] * shape[2] * shape[3] * shape[4]
+                    module.k_cache, module.v_cache = self.kv_cache[at:at + size].view(shape).unbind(0)
+                    layer, at = layer + 1, at + size
+                    continue
                 module.k_cache, module.v_cache = self.kv_cache[0, layer], self.kv_cache[1, layer]
                 layer += 1
         if layer == 0:
@@ -244,6 +269,36 @@ class InferenceExecutor:
             self._update_metrics(sequences, prefill)
             self.inference_count += 1
             return logits, tokens
+        finally:
+            reset_context()
+
+    @torch.inference_mode()
+    def score_batch(self, sequences: list[Sequence], rows: list[list[int]]) -> torch.Tensor | None:
+        """One step over the uncomputed tokens of ``sequences`` (portions of prompts and single tokens together), without
+        sampling: -> logits [sum of wanted rows, V], in the order of ``sequences`` and of ``rows[i]`` (places among the
+        step's tokens of sequence i), or None when nothing is wanted.  The same inputs, kernels and cache as
+        ``execute_batch``; eager."""
+        self._drop_speculation()
+        news = [s.prefill_stop - s.num_cached_tokens for s in sequences]
+        is_row = [n == 1 and s.num_cached_tokens > 0 for n, s in zip(news, sequences)]
+        order = sorted(range(len(sequences)), key=lambda i: not is_row[i])   # decode rows lead a mixed batch (stable)
+        batch = [sequences[i] for i in order]
+        try:
+            if all(is_row):
+                ids, pos = self._ship_decode(self.builder.decode(batch))
+            else:
+                ids, pos = self._ship_prefill(self.builder.prefill(batch), batch)
+            hidden = self.model(ids, pos)
+            start, at = {}, 0
+            for i in order:
+                start[i], at = at, at + news[i]
+            want = [start[i] + r for i, rr in enumerate(rows) for r in rr]
+            self._check_peer_waits(True)
+            if not want:
+                return None
+            reset_context()       # plain rows from here on: the head must not pick each prompt's last token
+            pick = torch.tensor(want, dtype=torch.int64).to(self.device)
+            return self.model.compute_logits(hidden.index_select(0, pick))
         finally:
             reset_context()
 
@@ -499,9 +554,10 @@ class InferenceExecutor:
         hf = self.config.hf_config
         heads = hf.num_attention_heads // get_tensor_parallel_world_size()
         # ... sized for every batch an EAGER step can carry too (max_num_seqs may exceed the largest graph bucket)
-        hip_ops.workspace(max(hip_ops.paged_decode_workspace_bytes(bs, heads, self.num_kv_heads, self.head_dim,
-                                                                   self.block_size, self.max_blocks_per_seq)
-                              for bs in list(self.graph_bs) + [self.config.max_num_seqs]), dev)
+        shapes = self.attn_shapes or [(heads, self.num_kv_heads, self.head_dim, 0)]
+        hip_ops.workspace(max(hip_ops.paged_decode_workspace_bytes(bs, h, hkv, d, self.block_size, self.max_blocks_per_seq,
+                                                                   chunk=c)
+                              for bs in list(self.graph_bs) + [self.config.max_num_seqs] for h, hkv, d, c in shapes), dev)
         self._general_capture = "no" if not general_ok else "done"
         try:
             if self.tp_size > 1:   # the family without a backend collective inside (peer-to-peer kernels only)

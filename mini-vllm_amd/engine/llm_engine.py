@@ -131,6 +131,9 @@ class LLMEngine:
             prompt = self.tokenizer.encode(prompt)
         if not prompt:
             raise ValueError("token_ids must contain at least one token")
+        vocab = getattr(self.config.hf_config, "vocab_size", None)
+        if vocab and not (0 <= min(prompt) and max(prompt) < vocab):   # the embedding lookup of a bad id would fault the GPU
+            raise ValueError(f"token ids must be in [0, {vocab}), got {min(prompt)} .. {max(prompt)}")
         # one prefill step takes max_num_batched_tokens; longer prompts are prefilled in chunks (scheduler.py)
         limit = self.config.max_model_len
         if not getattr(self.config, "enable_chunked_prefill", False):

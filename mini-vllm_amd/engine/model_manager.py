@@ -118,6 +118,9 @@ class ModelManager:
     def _dummy_init(model, seed: int) -> None:
         gen = torch.Generator(device=next(model.parameters()).device).manual_seed(seed)
         with torch.no_grad():
+            if hasattr(model, "dummy_weights"):     # checkpoint-shaped tensors through the model's own loaders
+                model.load_weights(model.dummy_weights(gen))
+                return
             for name, p in model.named_parameters():
                 if "norm" in name and name.endswith("weight"):
                     p.fill_(1.0)

@@ -101,6 +101,16 @@ class Sequence:
         self.last_token = token_id
         self.num_tokens += 1
 
+    def extend(self, token_ids: list[int]) -> None:
+        """Append tokens whose values are given (not sampled): everything before them counts as computed, so the next
+        step runs exactly these."""
+        if not token_ids:
+            raise ValueError("extend needs at least one token")
+        self.num_cached_tokens, self.prefill_end = self.num_tokens, None
+        self.token_ids.extend(token_ids)
+        self.last_token = self.token_ids[-1]
+        self.num_tokens += len(token_ids)
+
     # -- compact pickling for the TP control plane (sequence.py:239-365): once a sequence
     #    is decoding, workers only need its last token, never the whole prompt again -------
     def __getstate__(self):

@@ -2,12 +2,14 @@
 it is in none of the benchmark configurations (SURVEY §2 #24)."""
 from typing import Any
 
+from .mofarax import MofaraxForCausalLM
 from .opt import OPTForCausalLM
 from .qwen import Qwen2ForCausalLM, Qwen3ForCausalLM
 
 SUPPORTED_MODELS = {"Qwen2ForCausalLM": Qwen2ForCausalLM, "Qwen3ForCausalLM": Qwen3ForCausalLM,
-                    "OPTForCausalLM": OPTForCausalLM}
-TYPE_TO_ARCH = {"qwen2": "Qwen2ForCausalLM", "qwen3": "Qwen3ForCausalLM", "opt": "OPTForCausalLM"}
+                    "OPTForCausalLM": OPTForCausalLM, "Mofarax": MofaraxForCausalLM}
+TYPE_TO_ARCH = {"qwen2": "Qwen2ForCausalLM", "qwen3": "Qwen3ForCausalLM", "opt": "OPTForCausalLM",
+                "mofarax": "Mofarax"}
 
 
 def create_model(hf_config: Any) -> Any:

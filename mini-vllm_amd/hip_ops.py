@@ -35,24 +35,44 @@ _SIGNATURES = {
                                  c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_float, c_void_p,
                                  c_void_p, c_void_p, c_void_p, c_void_p, c_int64, c_int, c_int, c_int,
                                  c_int, c_int, c_void_p]),
+    "mv_rope_qk_store_ex": (c_int, [c_void_p, c_void_p, c_void_p, c_int64, c_int64, c_int64, c_void_p,
+                                 c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_float, c_void_p,
+                                 c_void_p, c_void_p, c_void_p, c_void_p, c_int64, c_int, c_int, c_int,
+                                 c_int, c_int, c_void_p, c_void_p]),
     "mv_paged_decode_workspace_bytes": (c_size_t, [c_int, c_int, c_int, c_int, c_int, c_int, c_int]),
+    "mv_paged_decode_workspace_bytes_ex": (c_size_t, [c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int]),
     "mv_paged_decode": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_void_p,
                                 c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int64, c_float,
                                 c_void_p, c_size_t, c_int, c_int, c_void_p]),
+    "mv_paged_decode_ex": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_void_p,
+                                c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int64, c_float,
+                                c_void_p, c_size_t, c_int, c_int, c_void_p, c_void_p]),
     "mv_rope_paged_decode": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p,
                                      c_void_p, c_int64, c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_void_p,
                                      c_void_p, c_int64, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
                                      c_int64, c_float, c_void_p, c_size_t, c_int, c_int, c_void_p]),
+    "mv_rope_paged_decode_ex": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p,
+                                     c_void_p, c_int64, c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_void_p,
+                                     c_void_p, c_int64, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
+                                     c_int64, c_float, c_void_p, c_size_t, c_int, c_int, c_void_p, c_void_p]),
     "mv_prefill_varlen": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int64, c_void_p,
                                   c_void_p, c_void_p, c_int64, c_int64, c_void_p, c_void_p, c_void_p,
                                   c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int,
                                   c_int, c_void_p]),
+    "mv_prefill_varlen_ex": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int64, c_void_p,
+                                  c_void_p, c_void_p, c_int64, c_int64, c_void_p, c_void_p, c_void_p,
+                                  c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int,
+                                  c_int, c_void_p, c_void_p]),
     "mv_sample_workspace_bytes": (c_size_t, [c_int, c_int]),
     "mv_sample": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p, c_uint64,
                           c_uint64, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_size_t,
                           c_int, c_void_p]),
     "mv_decode_advance": (c_int, [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p]),
     "mv_silu_and_mul": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int, c_int, c_int, c_void_p]),
+    "mv_gelu_and_mul": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int, c_int, c_int, c_void_p]),
+    "mv_residual_update": (c_int, [c_void_p, c_int, c_int, c_int, c_int, c_void_p]),
+    "mv_gated_lookup": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int64, c_int, c_void_p, c_void_p, c_int64, c_int,
+                                c_int, c_int, c_int, c_void_p]),
     "mv_linear_small_m": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_int, c_int,
                                   c_int, c_int, c_int, c_void_p]),
     "mv_gate_up_silu_small_m": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_int, c_int,
@@ -112,6 +132,32 @@ EXPORTED_SYMBOLS = tuple(_SIGNATURES)
 
 class MvHipError(RuntimeError):
     pass
+
+
+class MvAttnOpts(ctypes.Structure):
+    """Options of the ``_ex`` attention entry points (include/mvhip.h)."""
+    _fields_ = [("rot_pairs", c_int), ("interleaved", c_int), ("chunk", c_int), ("reserved", c_int), ("out_stride", c_int64)]
+
+
+class MvResidualArgs(ctypes.Structure):
+    _fields_ = [("x", c_void_p), ("y", c_void_p), ("y_norm_w", c_void_p), ("embed", c_void_p), ("ids", c_void_p),
+                ("vec", c_void_p), ("norm_w", c_void_p), ("out", c_void_p), ("y_stride", c_int64), ("out_stride", c_int64),
+                ("vocab", c_int64), ("embed_scale", c_float), ("norm_offset", c_float), ("eps", c_float),
+                ("y_splits", c_int), ("embed_mode", c_int)]
+
+
+def _attn_opts(interleaved_pairs=None, chunk: int = 0, out=None):
+    """``interleaved_pairs``: None = rotary halves, n = interleaved layout with n rotated pairs; ``chunk``: chunk size of
+    the causal mask (0 = whole context); ``out``: output tensor [rows, H, D] whose rows may be strided."""
+    il = interleaved_pairs is not None
+    o = MvAttnOpts(int(interleaved_pairs) if il else 0, int(il), int(chunk), 0, out.stride(0) if out is not None else 0)
+    return ctypes.byref(o)
+
+
+def _out_rows(out, rows: int, h: int, d: int):
+    if out.shape != (rows, h, d) or out.stride(2) != 1 or out.stride(1) != d:
+        raise MvHipError(f"output must be [{rows}, {h}, {d}] and dense in its last two dims")
+    return out
 
 
 # ---------------------------------------------------------------- tuning switches
@@ -297,9 +343,17 @@ def add_rmsnorm_partial(partial, residual, weight, eps: float):
 
 
 # ---------------------------------------------------------------- K7
+def _rot_tables_ok(cos, sin, d: int, interleaved_pairs) -> None:
+    want = d // 2 if interleaved_pairs is None else int(interleaved_pairs)
+    if cos.shape != sin.shape or cos.dim() != 2 or cos.shape[1] != want or not (cos.is_contiguous() and sin.is_contiguous()) \
+            or cos.dtype != torch.float32 or sin.dtype != torch.float32:
+        raise MvHipError(f"cos / sin must be dense fp32 [max_pos, {want}] tables")
+
+
 def rope_qk_store(q, k, v, positions, cos, sin, q_norm_w=None, k_norm_w=None, eps: float = 1e-6,
-                  k_cache=None, v_cache=None, slot_mapping=None, want_k_out: bool = True):
+                  k_cache=None, v_cache=None, slot_mapping=None, want_k_out: bool = True, interleaved_pairs=None):
     """q [T,H,D], k/v [T,Hkv,D] (views of the qkv GEMM output are fine).
+    ``interleaved_pairs``: n = the interleaved layout on the first 2n dims (cos / sin [max_pos, n]); None = halves.
     Returns (q_rot [T,H,D], k_rot [T,Hkv,D] or None)."""
     _need_cuda(q, k, positions, cos, sin)
     t, h, d = q.shape
@@ -321,32 +375,36 @@ def rope_qk_store(q, k, v, positions, cos, sin, q_norm_w=None, k_norm_w=None, ep
     pos = positions if positions.dtype == torch.int64 else positions.to(torch.int64)
     qn = q_norm_w if q_norm_w is None or q_norm_w.dtype == q.dtype else q_norm_w.to(q.dtype)
     kn = k_norm_w if k_norm_w is None or k_norm_w.dtype == q.dtype else k_norm_w.to(q.dtype)
-    _check(_lib.mv_rope_qk_store(
+    _rot_tables_ok(cos, sin, d, interleaved_pairs)
+    _check(_lib.mv_rope_qk_store_ex(
         q.data_ptr(), k.data_ptr(), _ptr(v), q.stride(0), k.stride(0), v.stride(0) if v is not None else 0,
         pos.data_ptr(), cos.data_ptr(), sin.data_ptr(), cos.shape[0], _ptr(qn), _ptr(kn), float(eps),
         q_out.data_ptr(), _ptr(k_out),
         k_cache.data_ptr() if has_cache else None, v_cache.data_ptr() if has_cache else None,
         _i32(slot_mapping).data_ptr() if has_cache else None, num_slots, t, h, hkv, d, _dt(q),
-        _stream()), "mv_rope_qk_store")
+        _attn_opts(interleaved_pairs), _stream()), "mv_rope_qk_store")
     return q_out, k_out
 
 
 # ---------------------------------------------------------------- K3
 def paged_decode_workspace_bytes(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks,
-                                 flags: int | None = None) -> int:
-    return int(_lib.mv_paged_decode_workspace_bytes(batch, n_heads, n_kv_heads, head_dim, block_size,
-                                                    max_blocks, DECODE_FLAGS if flags is None else flags))
+                                 flags: int | None = None, chunk: int = 0) -> int:
+    return int(_lib.mv_paged_decode_workspace_bytes_ex(batch, n_heads, n_kv_heads, head_dim, block_size,
+                                                       max_blocks, DECODE_FLAGS if flags is None else flags, int(chunk)))
 
 
-def paged_decode(q, k_cache, v_cache, block_tables, context_lens, scale: float, out=None, flags: int | None = None):
+def paged_decode(q, k_cache, v_cache, block_tables, context_lens, scale: float, out=None, flags: int | None = None,
+                 chunk: int = 0):
     """q [B,H,D]; caches [nb,bs,Hkv,D]; block_tables int [B,nblk] (row-strided view ok);
-    context_lens int [B].  Returns [B,H,D] in q's dtype."""
+    context_lens int [B].  ``chunk``: > 0 = only the keys of the last token's chunk of positions.  Returns [B,H,D] in
+    q's dtype (``out``: a row-strided view is fine)."""
     _need_cuda(q, k_cache, v_cache, block_tables, context_lens)
     b, h, d = q.shape
     if q.stride(-1) != 1 or q.stride(1) != d:
         q = q.contiguous()
     if out is None:
         out = torch.empty((b, h, d), dtype=q.dtype, device=q.device)
+    _out_rows(out, b, h, d)
     nb, bs, hkv = k_cache.shape[0], k_cache.shape[1], k_cache.shape[2]
     bt = _i32(block_tables)
     if bt.dim() != 2 or (bt.shape[1] > 0 and bt.stride(1) != 1):
@@ -354,18 +412,20 @@ def paged_decode(q, k_cache, v_cache, block_tables, context_lens, scale: float, 
     cl = _i32(context_lens)
     max_blocks = bt.shape[1]
     flags = DECODE_FLAGS if flags is None else flags
-    ws_bytes = paged_decode_workspace_bytes(b, h, hkv, d, bs, max_blocks, flags)
+    ws_bytes = paged_decode_workspace_bytes(b, h, hkv, d, bs, max_blocks, flags, chunk)
     ws = workspace(ws_bytes, q.device)
-    _check(_lib.mv_paged_decode(q.data_ptr(), q.stride(0), k_cache.data_ptr(), v_cache.data_ptr(),
+    _check(_lib.mv_paged_decode_ex(q.data_ptr(), q.stride(0), k_cache.data_ptr(), v_cache.data_ptr(),
                                 bt.data_ptr(), bt.stride(0) if max_blocks else 0, cl.data_ptr(),
                                 out.data_ptr(), b, h, hkv, d, bs, max_blocks, nb, float(scale),
-                                ws.data_ptr(), ws.numel(), _dt(q), flags, _stream()), "mv_paged_decode")
+                                ws.data_ptr(), ws.numel(), _dt(q), flags, _attn_opts(None, chunk, out),
+                                   _stream()), "mv_paged_decode")
     return out
 
 
 # ---------------------------------------------------------------- K2
 def rope_paged_decode(q, k, v, positions, cos, sin, q_norm_w, k_norm_w, eps: float, slot_mapping,
-                      k_cache, v_cache, block_tables, context_lens, scale: float, flags: int | None = None):
+                      k_cache, v_cache, block_tables, context_lens, scale: float, flags: int | None = None,
+                      interleaved_pairs=None, chunk: int = 0, out=None):
     """Decode step of one layer in ONE launch: q [B,H,D], k/v [B,Hkv,D] RAW rows of the qkv projection (views are
     fine) -> per-head RMSNorm (weights or None) + RoPE on q and k, the new K/V rows stored at ``slot_mapping``, paged
     attention over ``block_tables`` / ``context_lens`` (which count the new token).  Returns [B,H,D], or None when
@@ -383,17 +443,21 @@ def rope_paged_decode(q, k, v, positions, cos, sin, q_norm_w, k_norm_w, eps: flo
     if bt.dim() != 2 or bt.stride(1) != 1 or bt.shape[1] == 0:
         return None
     flags = DECODE_FLAGS if flags is None else flags
-    ws_bytes = paged_decode_workspace_bytes(b, h, hkv, d, bs, bt.shape[1], flags)
+    ws_bytes = paged_decode_workspace_bytes(b, h, hkv, d, bs, bt.shape[1], flags, chunk)
     ws = workspace(ws_bytes, q.device)
-    out = torch.empty((b, h, d), dtype=q.dtype, device=q.device)
+    if out is None:
+        out = torch.empty((b, h, d), dtype=q.dtype, device=q.device)
+    _out_rows(out, b, h, d)
+    _rot_tables_ok(cos, sin, d, interleaved_pairs)
     pos = positions if positions.dtype == torch.int64 else positions.to(torch.int64)
     qn = q_norm_w if q_norm_w is None or q_norm_w.dtype == q.dtype else q_norm_w.to(q.dtype)
     kn = k_norm_w if k_norm_w is None or k_norm_w.dtype == q.dtype else k_norm_w.to(q.dtype)
-    rc = _lib.mv_rope_paged_decode(
+    rc = _lib.mv_rope_paged_decode_ex(
         q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0), pos.data_ptr(),
         cos.data_ptr(), sin.data_ptr(), cos.shape[0], _ptr(qn), _ptr(kn), float(eps), _i32(slot_mapping).data_ptr(),
         k_cache.data_ptr(), v_cache.data_ptr(), bt.data_ptr(), bt.stride(0), cl.data_ptr(), out.data_ptr(), b, h, hkv,
-        d, bs, bt.shape[1], nb, float(scale), ws.data_ptr(), ws.numel(), _dt(q), flags, _stream())
+        d, bs, bt.shape[1], nb, float(scale), ws.data_ptr(), ws.numel(), _dt(q), flags,
+        _attn_opts(interleaved_pairs, chunk, out), _stream())
     if rc == MV_E_SHAPE:
         return None
     _check(rc, "mv_rope_paged_decode")
@@ -401,15 +465,18 @@ def rope_paged_decode(q, k, v, positions, cos, sin, q_norm_w, k_norm_w, eps: flo
 
 
 def prefill_varlen(q, k, v, cu_seqlens_q, cu_seqlens_k, max_seqlen_q, max_seqlen_k, scale: float,
-                   k_cache=None, v_cache=None, block_tables=None, out=None, flags: int | None = None):
+                   k_cache=None, v_cache=None, block_tables=None, out=None, flags: int | None = None,
+                   chunk: int = 0):
     """Packed causal prefill.  Contiguous K/V (k,v [Tk,Hkv,D]) unless ``block_tables`` is
-    given, in which case keys come from the paged caches (prefix-cache hit)."""
+    given, in which case keys come from the paged caches (prefix-cache hit).  ``chunk``: > 0 = a query sees only the
+    keys of its own chunk of positions."""
     _need_cuda(q, cu_seqlens_q, cu_seqlens_k)
     t, h, d = q.shape
     if q.stride(-1) != 1 or q.stride(1) != d:
         q = q.contiguous()
     if out is None:
         out = torch.empty((t, h, d), dtype=q.dtype, device=q.device)
+    _out_rows(out, t, h, d)
     n_seqs = cu_seqlens_q.numel() - 1
     paged = block_tables is not None
     if paged:
@@ -425,10 +492,11 @@ def prefill_varlen(q, k, v, cu_seqlens_q, cu_seqlens_k, max_seqlen_q, max_seqlen
             if x.stride(-1) != 1 or x.stride(1) != d:
                 raise MvHipError(f"{name} must be dense in its last two dims")
         args_kv = (k.data_ptr(), v.data_ptr(), k.stride(0), v.stride(0), None, None, None, 0, 0)
-    _check(_lib.mv_prefill_varlen(q.data_ptr(), q.stride(0), *args_kv, out.data_ptr(),
+    _check(_lib.mv_prefill_varlen_ex(q.data_ptr(), q.stride(0), *args_kv, out.data_ptr(),
                                   _i32(cu_seqlens_q).data_ptr(), _i32(cu_seqlens_k).data_ptr(), n_seqs,
                                   int(max_seqlen_q), int(max_seqlen_k), h, hkv, d, bs, float(scale),
-                                  _dt(q), PREFILL_FLAGS if flags is None else flags, _stream()), "mv_prefill_varlen")
+                                  _dt(q), PREFILL_FLAGS if flags is None else flags,
+                                     _attn_opts(None, chunk, out), _stream()), "mv_prefill_varlen")
     return out
 
 
@@ -469,6 +537,79 @@ def silu_and_mul(x):
     _check(_lib.mv_silu_and_mul(x2.data_ptr(), x2.stride(0), out.data_ptr(), out.stride(0), x2.shape[0],
                                 cols, _dt(x), _stream()), "mv_silu_and_mul")
     return out.view(*x.shape[:-1], cols)
+
+
+def gelu_and_mul(x, out=None):
+    """x [rows, 2 * cols] (row-strided view ok) -> gelu_tanh(x[:, :cols]) * x[:, cols:]; ``out`` may be row-strided."""
+    _need_cuda(x)
+    if x.dim() != 2 or x.stride(1) != 1 or x.shape[1] % 2:
+        raise ValueError(f"gelu_and_mul wants [rows, 2 * cols] rows, got {tuple(x.shape)}")
+    rows, cols = x.shape[0], x.shape[1] // 2
+    if out is None:
+        out = torch.empty((rows, cols), dtype=x.dtype, device=x.device)
+    if out.shape != (rows, cols) or out.stride(1) != 1 or out.dtype != x.dtype:
+        raise MvHipError("gelu_and_mul: output shape / layout mismatch")
+    _check(_lib.mv_gelu_and_mul(x.data_ptr(), x.stride(0), out.data_ptr(), out.stride(0), rows, cols, _dt(x), _stream()),
+           "mv_gelu_and_mul")
+    return out
+
+
+# ---------------------------------------------------------------- K13
+def residual_update(x, y=None, y_norm_w=None, embed=None, ids=None, embed_scale: float = 1.0, start: bool = False,
+                    vec=None, norm_w=None, norm_offset: float = 0.0, eps: float = 0.0, cols_true: int | None = None,
+                    out=None, want_out: bool = True, dtype=None):
+    """One edge of the fp32 residual stream ``x`` [rows, cols] (updated in place; include/mvhip.h: mv_residual_update).
+    ``y``: [rows, cols] of the activation dtype, or fp32 K-split partial sums [splits, rows, cols]; ``y_norm_w``: its RMS
+    norm.  ``embed`` / ``ids``: the scaled embedding is added (``start``: the row starts from it).  ``vec``: added to every
+    row.  Returns rms(x) * (norm_offset + norm_w), or x cast to ``dtype`` when norm_w is None; None if not want_out."""
+    _need_cuda(x, y, y_norm_w, embed, ids, vec, norm_w)
+    rows, cols = x.shape
+    if x.dtype != torch.float32 or not x.is_contiguous():
+        raise MvHipError("the residual stream must be a dense fp32 [rows, cols] tensor")
+    dt = dtype or next(t.dtype for t in (norm_w, vec, embed, y_norm_w, y) if t is not None)
+    splits = 0
+    if y is not None:
+        if y.dim() == 3:
+            splits = y.shape[0]
+            if y.dtype != torch.float32 or tuple(y.shape[1:]) != (rows, cols) or not y.is_contiguous():
+                raise MvHipError("partial sums must be dense fp32 [splits, rows, cols]")
+        elif tuple(y.shape) != (rows, cols) or y.dtype != dt or y.stride(1) != 1:
+            raise MvHipError(f"y must be [{rows}, {cols}] of {dt}")
+    for name, w in (("y_norm_w", y_norm_w), ("vec", vec), ("norm_w", norm_w)):
+        if w is not None and (w.dtype != dt or w.numel() != cols or not w.is_contiguous()):
+            raise MvHipError(f"{name} must be [{cols}] of {dt}")
+    if embed is not None and (embed.dtype != dt or embed.shape[1] != cols or not embed.is_contiguous()
+                              or ids is None or ids.dtype != torch.int64 or ids.numel() != rows or not ids.is_contiguous()):
+        raise MvHipError("embedding table [vocab, cols] of the activation dtype and int64 ids [rows] required")
+    if start and embed is None:
+        raise MvHipError("a row can only start from an embedding")
+    if want_out and out is None:
+        out = torch.empty((rows, cols), dtype=dt, device=x.device)
+    if out is not None and (tuple(out.shape) != (rows, cols) or out.dtype != dt or out.stride(1) != 1):
+        raise MvHipError(f"out must be [{rows}, {cols}] of {dt}")
+    a = MvResidualArgs(x.data_ptr(), _ptr(y), _ptr(y_norm_w), _ptr(embed), _ptr(ids) if embed is not None else None,
+                       _ptr(vec), _ptr(norm_w), _ptr(out), y.stride(0) if y is not None and splits == 0 else 0,
+                       out.stride(0) if out is not None else 0, embed.shape[0] if embed is not None else 0,
+                       float(embed_scale), float(norm_offset), float(eps), splits,
+                       0 if embed is None else (1 if start else 2))
+    _check(_lib.mv_residual_update(ctypes.byref(a), rows, cols, cols if cols_true is None else int(cols_true), _DTYPES[dt],
+                                   _stream()), "mv_residual_update")
+    return out
+
+
+def gated_lookup(s, table, offset: int, dim: int, ids, out=None):
+    """gelu_tanh(s[:, j]) * table[ids, offset + j] for j < dim, zeros for the padding columns behind."""
+    _need_cuda(s, table, ids)
+    rows, cols = s.shape
+    if s.stride(1) != 1 or table.dtype != s.dtype or not table.is_contiguous() or ids.dtype != torch.int64 \
+            or ids.numel() != rows or not ids.is_contiguous():
+        raise MvHipError("gated_lookup: rows of s, a dense table of the same dtype and int64 ids [rows] required")
+    if out is None:
+        out = torch.empty((rows, cols), dtype=s.dtype, device=s.device)
+    _check(_lib.mv_gated_lookup(s.data_ptr(), s.stride(0), table.data_ptr(), table.stride(0), table.shape[0], int(offset),
+                                ids.data_ptr(), out.data_ptr(), out.stride(0), rows, int(dim), cols, _dt(s), _stream()),
+           "mv_gated_lookup")
+    return out
 
 
 # ---------------------------------------------------------------- K10

@@ -21,26 +21,29 @@ __all__ = ["Attention"]
 
 class Attention(nn.Module):
     def __init__(self, num_heads: int, head_dim: int, scale: float, num_kv_heads: int,
-                 use_buffered_page_attention: bool = False) -> None:
+                 use_buffered_page_attention: bool = False, chunk: int = 0) -> None:
         super().__init__()
         self.num_heads = num_heads
         self.head_dim = head_dim
         self.scale = float(scale) if scale != 0.0 else 1.0 / math.sqrt(head_dim)
         self.num_kv_heads = num_kv_heads
+        # > 0: a query sees only the keys of its own chunk of ``chunk`` positions (counted from the sequence's start)
+        self.chunk = int(chunk)
         self.k_cache: torch.Tensor = torch.tensor([])
         self.v_cache: torch.Tensor = torch.tensor([])
         self._cache_initialized = False
 
     def extra_repr(self) -> str:
         return (f"num_heads={self.num_heads}, head_dim={self.head_dim}, num_kv_heads={self.num_kv_heads}, "
-                f"scale={self.scale}, backend=mvhip")
+                f"scale={self.scale}, chunk={self.chunk}, backend=mvhip")
 
     def store_kv_cache(self, key, value, slot_mapping) -> None:
         hip_ops.store_kvcache(key, value, self.k_cache, self.v_cache, slot_mapping)
 
-    def forward(self, q, k, v, kv_stored: bool = False):
+    def forward(self, q, k, v, kv_stored: bool = False, out=None):
         """``kv_stored=True`` when the caller already wrote k/v into the cache (the fused
-        RoPE+store kernel); otherwise this call stores them first, like the reference."""
+        RoPE+store kernel); otherwise this call stores them first, like the reference.  ``out``: where the result goes
+        ([N, H, D], rows may be strided)."""
         ctx = get_context()
         has_cache = self.k_cache.numel() > 0 and self.v_cache.numel() > 0
         if has_cache:
@@ -60,25 +63,26 @@ class Attention(nn.Module):
                 # mixed batch: the first rows are one-token continuations of cached sequences (the paged-decode
                 # kernel reads their K/V once, at HBM speed), the rest is prefill through the paged cache
                 nd = ctx.decode_rows
-                out = torch.empty_like(q)
+                if out is None:
+                    out = torch.empty((q.shape[0], self.num_heads, q.shape[2]), dtype=q.dtype, device=q.device)
                 hip_ops.paged_decode(q[:nd], self.k_cache, self.v_cache, ctx.block_tables[:nd], ctx.context_lens,
-                                     self.scale, out=out[:nd])
+                                     self.scale, out=out[:nd], chunk=self.chunk)
                 if q.shape[0] > nd:
                     hip_ops.prefill_varlen(q[nd:], None, None, ctx.rest_cum_seqlens_q, ctx.rest_cum_seqlens_k,
                                            ctx.rest_max_seqlen_q, ctx.rest_max_seqlen_k, self.scale,
                                            k_cache=self.k_cache, v_cache=self.v_cache,
-                                           block_tables=ctx.block_tables[nd:], out=out[nd:])
+                                           block_tables=ctx.block_tables[nd:], out=out[nd:], chunk=self.chunk)
                 return out
             if ctx.prefix_cached and has_cache and ctx.block_tables is not None:
                 # prefix-cache hit: the queries are the uncached suffix, the keys live in the cache
                 return hip_ops.prefill_varlen(q, None, None, ctx.cum_seqlens_q, ctx.cum_seqlens_k,
                                               ctx.max_seqlen_q, ctx.max_seqlen_k, self.scale,
                                               k_cache=self.k_cache, v_cache=self.v_cache,
-                                              block_tables=ctx.block_tables)
+                                              block_tables=ctx.block_tables, out=out, chunk=self.chunk)
             return hip_ops.prefill_varlen(q, k, v, ctx.cum_seqlens_q, ctx.cum_seqlens_k,
-                                          ctx.max_seqlen_q, ctx.max_seqlen_k, self.scale)
+                                          ctx.max_seqlen_q, ctx.max_seqlen_k, self.scale, out=out, chunk=self.chunk)
         if ctx.context_lens is None or ctx.block_tables is None:
             raise RuntimeError("Context lengths or block tables not set for decode phase. "
                                "This is a bug in the inference pipeline.")
         return hip_ops.paged_decode(q, self.k_cache, self.v_cache, ctx.block_tables, ctx.context_lens,
-                                    self.scale)
+                                    self.scale, out=out, chunk=self.chunk)

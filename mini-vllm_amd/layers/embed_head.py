@@ -16,8 +16,10 @@ __all__ = ["VocabParallelEmbedding", "ParallelLMHead", "get_tensor_parallel_rank
 
 
 class VocabParallelEmbedding(nn.Module):
-    def __init__(self, num_embeddings: int, embedding_dim: int):
+    def __init__(self, num_embeddings: int, embedding_dim: int, storage_dim: int | None = None):
+        """``storage_dim`` > embedding_dim: rows are stored zero-padded (the activations are padded the same way)."""
         super().__init__()
+        self.embedding_dim = embedding_dim
         self.tp_rank, self.tp_size = get_tensor_parallel_rank(), get_tensor_parallel_world_size()
         if num_embeddings % self.tp_size != 0:
             raise ValueError(f"num_embeddings ({num_embeddings}) must be divisible by "
@@ -26,14 +28,17 @@ class VocabParallelEmbedding(nn.Module):
         self.num_embeddings_per_partition = num_embeddings // self.tp_size
         self.vocab_start_idx = self.num_embeddings_per_partition * self.tp_rank
         self.vocab_end_idx = self.vocab_start_idx + self.num_embeddings_per_partition
-        self.weight = nn.Parameter(torch.empty(self.num_embeddings_per_partition, embedding_dim))
+        storage = storage_dim or embedding_dim
+        self.weight = nn.Parameter(torch.empty(self.num_embeddings_per_partition, storage))
+        if storage > embedding_dim:
+            self.weight.data.zero_()
         self.weight.weight_loader = self.weight_loader
 
     def weight_loader(self, param, loaded_weight, *args, **kwargs):
         from ..utils.loader import materialize
 
         shard = param.data.size(0)
-        param.data.copy_(materialize(loaded_weight.narrow(0, self.tp_rank * shard, shard)))
+        param.data[:, :self.embedding_dim].copy_(materialize(loaded_weight.narrow(0, self.tp_rank * shard, shard)))
 
     def extra_repr(self) -> str:
         return (f"num_embeddings={self.num_embeddings}, embedding_dim={self.weight.shape[1]}, "
@@ -48,10 +53,10 @@ class VocabParallelEmbedding(nn.Module):
 
 
 class ParallelLMHead(VocabParallelEmbedding):
-    def __init__(self, num_embeddings: int, embedding_dim: int, bias: bool = False):
+    def __init__(self, num_embeddings: int, embedding_dim: int, bias: bool = False, storage_dim: int | None = None):
         if bias:
             raise ValueError("bias for ParallelLMHead is not supported")
-        super().__init__(num_embeddings, embedding_dim)
+        super().__init__(num_embeddings, embedding_dim, storage_dim)
         self.weight_packed = None
 
     def pack_for_decode(self) -> bool:

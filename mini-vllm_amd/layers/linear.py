@@ -16,6 +16,8 @@ from __future__ import annotations
 import json
 import os
 
+from dataclasses import dataclass
+
 import torch
 import torch.nn.functional as F
 from torch import nn
@@ -26,7 +28,7 @@ from ..parallel_state import (divide, get_tensor_parallel_rank, get_tensor_paral
 from ..utils.loader import materialize
 
 __all__ = ["LinearBase", "ReplicatedLinear", "ColumnParallelLinear", "MergedColumnParallelLinear",
-           "QKVParallelLinear", "RowParallelLinear", "divide", "linear", "small_m", "PartialSum", "mid_plan",
+           "QKVParallelLinear", "RowParallelLinear", "SegmentedLinear", "Segment", "pad_to", "divide", "linear", "small_m", "PartialSum", "mid_plan",
            "tuned_plan", "mid_m"]
 
 # rows up to which the weight-streaming kernel beats the library GEMM (tools/bench_linear.py); 0 disables
@@ -279,3 +281,66 @@ class RowParallelLinear(LinearBase):
         kind = "row" if partial_ok and self.tp_size == 1 else "col"
         y = linear(x, self.weight, self.bias if self.tp_rank == 0 else None, self.weight_packed, kind)
         return tp_all_reduce(y) if self.tp_size > 1 and reduce else y
+
+
+def pad_to(n: int, multiple: int = 64) -> int:
+    return -(-n // multiple) * multiple
+
+
+@dataclass(frozen=True)
+class Segment:
+    """One checkpoint matrix inside a merged weight: ``units`` (heads, features) of ``unit`` rows or columns each, stored
+    at ``stored`` >= unit apiece (zeros behind); a tensor-parallel rank owns a contiguous run of whole units."""
+    name: str
+    units: int
+    unit: int = 1
+    stored: int | None = None
+
+    def local(self, tp: int) -> int:
+        """Stored rows / columns of one rank: a multiple of 64, so that the next segment starts on a whole tile."""
+        return pad_to(divide(self.units, tp) * (self.stored or self.unit))
+
+
+class SegmentedLinear(LinearBase):
+    """Several projections in one weight, with zero padding wherever a size is not what the kernels take.
+
+    ``split="out"``: segments stack along the output features (they read the same input: q | k | gate | up ...);
+    ``split="in"``: along the input features (their products are SUMMED: attention output | mlp down ...), reduced over
+    the tensor-parallel ranks; ``split="none"``: one replicated matrix.  The other dimension is padded to a multiple of
+    64; ``offsets[name]`` is where a segment starts.  Padding rows / columns are zero and stay zero."""
+
+    def __init__(self, other_size: int, segments: list[Segment], split: str = "out") -> None:
+        if split not in ("out", "in", "none"):
+            raise ValueError(f"unknown split {split!r}")
+        tp = 1 if split == "none" else get_tensor_parallel_world_size()
+        self.segments, self.split, self.other_size = {g.name: g for g in segments}, split, other_size
+        self.offsets, n = {}, 0
+        for g in segments:
+            self.offsets[g.name] = n
+            n += g.local(tp)
+        rows, cols = (pad_to(other_size), n) if split == "in" else (n, pad_to(other_size))
+        super().__init__(cols, rows, False, {"out": 0, "in": 1, "none": None}[split])
+        self.shards = tp
+        self.weight.data.zero_()
+
+    def weight_loader(self, param, loaded_weight, loaded_shard_id: str | None = None, *args, **kwargs):
+        if loaded_shard_id is None and len(self.segments) == 1:
+            loaded_shard_id = next(iter(self.segments))
+        g = self.segments[loaded_shard_id]
+        dim = 1 if self.split == "in" else 0
+        want = [self.other_size, self.other_size]
+        want[dim] = g.units * g.unit
+        if tuple(loaded_weight.shape) != tuple(want):
+            raise ValueError(f"segment {g.name!r}: expected {tuple(want)}, got {tuple(loaded_weight.shape)}")
+        units, stored, off = divide(g.units, self.shards), g.stored or g.unit, self.offsets[g.name]
+        rank = self.tp_rank if self.shards > 1 else 0
+        piece = materialize(loaded_weight.narrow(dim, rank * units * g.unit, units * g.unit))
+        dst = param.data.narrow(dim, off, units * stored).unflatten(dim, (units, stored)).narrow(dim + 1, 0, g.unit)
+        dst = dst.narrow(0 if dim == 1 else 2, 0, self.other_size)
+        dst.copy_(piece.unflatten(dim, (units, g.unit)))
+
+    def forward(self, x, partial_ok: bool = False):
+        """``partial_ok`` (split="in", single rank): the caller takes a ``PartialSum``."""
+        kind = "row" if partial_ok and self.split == "in" and self.shards == 1 else "col"
+        y = linear(x, self.weight, None, self.weight_packed, kind)
+        return tp_all_reduce(y) if self.split == "in" and self.shards > 1 else y

@@ -1,7 +1,10 @@
-"""NeoX rotary embedding (mirror of minivllm/models/layers/rotary_embedding.py:83-242).
+"""Rotary embedding: NeoX halves (mirror of minivllm/models/layers/rotary_embedding.py:83-242).
 The fp32 cos/sin tables are built with the reference's exact operation order (their values
 must match torch's fp32 cos/sin of fp32 ``arange * inv_freq``); application runs in the HIP
-kernel, normally fused with qk-norm and the KV-cache store (see glue/qwen.py)."""
+kernel, normally fused with qk-norm and the KV-cache store (see glue/qwen.py).
+
+``interleaved=True`` is the other layout: dims 2i and 2i + 1 form a pair, on the first ``rotary_dim`` dims of a head; its
+tables are the exact angles (fp64 on the host) rounded once to fp32."""
 from __future__ import annotations
 
 from functools import lru_cache
@@ -32,15 +35,32 @@ def build_cos_sin(rotary_dim: int, max_position: int, base: float,
     return freqs.cos(), freqs.sin()
 
 
+def build_cos_sin_interleaved(rotary_dim: int, max_position: int, base: float):
+    """fp32 cos / sin [max_position, rotary_dim / 2] of position * base^(-2i / rotary_dim)."""
+    i = torch.arange(rotary_dim // 2, dtype=torch.float64, device="cpu")
+    freq = float(base) ** (-2.0 * i / max(rotary_dim, 1))
+    angle = torch.arange(max_position, dtype=torch.float64, device="cpu")[:, None] * freq[None, :]
+    return angle.cos().float(), angle.sin().float()
+
+
 class RotaryEmbedding(nn.Module):
     def __init__(self, head_size: int, rotary_dim: int, max_position_embeddings: int, base: float,
-                 rope_scaling: dict[str, Any] | None = None) -> None:
+                 rope_scaling: dict[str, Any] | None = None, interleaved: bool = False) -> None:
         super().__init__()
-        if rotary_dim != head_size:
+        if interleaved:
+            if rotary_dim % 2 or not 0 <= rotary_dim <= head_size:
+                raise ValueError(f"interleaved rotary dims must be even and at most head_size, got {rotary_dim} of {head_size}")
+            if rope_scaling is not None:
+                raise ValueError("rope_scaling is not defined for the interleaved layout")
+        elif rotary_dim != head_size:
             raise ValueError("rotary_dim must equal head_size")
         self.head_size = head_size
         self.max_position_embeddings = max_position_embeddings
-        cos, sin = build_cos_sin(rotary_dim, max_position_embeddings, base, rope_scaling)
+        self.interleaved_pairs = rotary_dim // 2 if interleaved else None
+        if interleaved:
+            cos, sin = build_cos_sin_interleaved(rotary_dim, max_position_embeddings, base)
+        else:
+            cos, sin = build_cos_sin(rotary_dim, max_position_embeddings, base, rope_scaling)
         self.register_buffer("cos_cache", cos, persistent=False)  # [max_pos, D/2] fp32
         self.register_buffer("sin_cache", sin, persistent=False)
         # the fp32 originals, as plain attributes: ``model.to(dtype)`` rounds the BUFFERS in place, and this module
@@ -64,17 +84,17 @@ class RotaryEmbedding(nn.Module):
 
     def forward(self, positions, query, key):
         """query [T,H,D], key [T,Hkv,D] -> rotated copies."""
-        cos, sin = self._tables(query.device, query.dtype)
-        return hip_ops.rope_qk_store(query, key, None, positions, cos, sin)
+        cos, sin = self._tables(query.device, None if self.interleaved_pairs is not None else query.dtype)
+        return hip_ops.rope_qk_store(query, key, None, positions, cos, sin, interleaved_pairs=self.interleaved_pairs)
 
 
 def get_rope(head_size: int, rotary_dim: int, max_position: int, base: float,
-             rope_scaling: dict[str, Any] | None = None) -> RotaryEmbedding:
+             rope_scaling: dict[str, Any] | None = None, interleaved: bool = False) -> RotaryEmbedding:
     if rope_scaling is not None:  # dicts are unhashable: no cache, as in the reference
-        return RotaryEmbedding(head_size, rotary_dim, max_position, base, rope_scaling)
-    return _get_rope_cached(head_size, rotary_dim, max_position, base)
+        return RotaryEmbedding(head_size, rotary_dim, max_position, base, rope_scaling, interleaved)
+    return _get_rope_cached(head_size, rotary_dim, max_position, base, interleaved)
 
 
-@lru_cache(4)
-def _get_rope_cached(head_size: int, rotary_dim: int, max_position: int, base: float) -> RotaryEmbedding:
-    return RotaryEmbedding(head_size, rotary_dim, max_position, base)
+@lru_cache(16)
+def _get_rope_cached(head_size: int, rotary_dim: int, max_position: int, base: float, interleaved: bool) -> RotaryEmbedding:
+    return RotaryEmbedding(head_size, rotary_dim, max_position, base, None, interleaved)

@@ -1,0 +1,164 @@
+"""Configurations of architectures that are described by this framework's own config.json layout (a top-level
+``"architecture"`` key) instead of a transformers config class."""
+from __future__ import annotations
+
+import json
+import math
+from dataclasses import dataclass
+from pathlib import Path
+
+__all__ = ["AttentionSpec", "LayerSpec", "MofaraxConfig", "NATIVE_CONFIGS", "load_native_config"]
+
+
+def _need(d: dict, key: str, where: str):
+    if not isinstance(d, dict) or key not in d:
+        raise ValueError(f"{where}: missing {key!r}")
+    return d[key]
+
+
+def _size(v, what: str) -> int:
+    if isinstance(v, bool) or not isinstance(v, int) or v <= 0:
+        raise ValueError(f"{what} must be a positive integer, got {v!r}")
+    return v
+
+
+def _real(v, what: str) -> float:
+    if isinstance(v, bool) or not isinstance(v, (int, float)) or not math.isfinite(v):
+        raise ValueError(f"{what} must be a finite number, got {v!r}")
+    return float(v)
+
+
+@dataclass(frozen=True)
+class AttentionSpec:
+    """Grouped-head attention with interleaved rotation and an optional chunk mask; the values are the projected keys."""
+    heads: int
+    kv_heads: int
+    dim: int
+    rot_base: float
+    rot_dims: int
+    scale: float
+    chunk: int          # 0: no mask besides causality
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str) -> "AttentionSpec":
+        heads, kv = _size(_need(m, "heads", where), f"{where}.heads"), _size(_need(m, "kv_heads", where), f"{where}.kv_heads")
+        dim = _size(_need(m, "dim", where), f"{where}.dim")
+        if heads % kv:
+            raise ValueError(f"{where}: {heads} query heads do not divide over {kv} key/value heads")
+        if _size(m.get("vdim", dim), f"{where}.vdim") != dim:
+            raise ValueError(f"{where}: the values are the keys, so vdim ({m['vdim']}) must equal dim ({dim})")
+        rot = _need(m, "rot", where)
+        rot_dims = _size(_need(rot, "dims", f"{where}.rot"), f"{where}.rot.dims")
+        if rot_dims % 2 or rot_dims > dim:
+            raise ValueError(f"{where}.rot.dims must be even and at most dim ({dim}), got {rot_dims!r}")
+        base = _real(_need(rot, "base", f"{where}.rot"), f"{where}.rot.base")
+        mask = m.get("mask") or {}
+        chunk = _size(mask["size"], f"{where}.mask.size") if mask.get("size") is not None else 0
+        scale = _real(_need(m, "scale", where), f"{where}.scale")
+        if scale <= 0 or base <= 0:
+            raise ValueError(f"{where}: scale and rot.base must be positive, got {scale} and {base}")
+        return cls(heads, kv, dim, base, rot_dims, scale, chunk)
+
+
+@dataclass(frozen=True)
+class LayerSpec:
+    attention: AttentionSpec
+    ff: int             # 0: no feed-forward
+
+    @classmethod
+    def from_dict(cls, d: dict, where: str) -> "LayerSpec":
+        kind = _need(d, "type", where)
+        if kind != "attention":
+            raise ValueError(f"{where}: unsupported layer type {kind!r}")
+        mlp, ff = d.get("mlp"), 0
+        if mlp is not None:
+            if mlp.get("kind", "dense") != "dense":
+                raise ValueError(f"{where}: unsupported feed-forward {mlp.get('kind')!r}")
+            ff = _size(_need(mlp, "ff", f"{where}.mlp"), f"{where}.mlp.ff")
+        return cls(AttentionSpec.from_dict(_need(d, "mixer", where), f"{where}.mixer"), ff)
+
+
+class MofaraxConfig:
+    """Parallel attention / feed-forward layers over a 32-bit residual stream, a per-layer token table, and a run of
+    layers that is passed several times over the same weights."""
+    model_type = "mofarax"
+
+    def __init__(self, raw: dict) -> None:
+        self.architectures = ["Mofarax"]
+        self.vocab_size = _size(_need(raw, "vocab", "config"), "vocab")
+        self.hidden_size = _size(_need(raw, "width", "config"), "width")
+        self.embedding_scale = _real((raw.get("embedding") or {}).get("scale", 1.0), "embedding.scale")
+        self.norm_eps = _real(_need(_need(raw, "norm", "config"), "eps", "norm"), "norm.eps")
+        side = raw.get("token_side")
+        self.side_dim = _size(_need(side, "dim", "token_side"), "token_side.dim") if side else 0
+        layers = _need(raw, "layers", "config")
+        if not isinstance(layers, list) or not layers:
+            raise ValueError("config: 'layers' must be a non-empty list")
+        self.layers = [LayerSpec.from_dict(d, f"layers[{i}]") for i, d in enumerate(layers)]
+        loop = raw.get("loop")
+        self.loop = None
+        if loop:
+            start, stop = _need(loop, "start", "loop"), _need(loop, "stop", "loop")
+            times = _size(_need(loop, "times", "loop"), "loop.times")
+            if not 0 <= start < stop <= len(layers):
+                raise ValueError(f"loop: [{start}, {stop}) is not a run of the {len(layers)} layers")
+            self.loop = (start, stop, times)
+        # what the engine asks of any configuration
+        a = [s.attention for s in self.layers]
+        self.num_hidden_layers = len(self.layer_runs())
+        self.num_attention_heads = max(s.heads for s in a)
+        self.num_key_value_heads = max(s.kv_heads for s in a)
+        self.head_dim = max(s.dim for s in a)
+        self.intermediate_size = max(s.ff for s in self.layers)
+        self.max_position_embeddings: int | None = None    # none of its own; the engine's Config fills it in
+        self.torch_dtype = raw.get("dtype", "bfloat16")
+        self.eos_token_id = None
+        self.tie_word_embeddings = False
+
+    def layer_runs(self) -> list[tuple[int, int, bool]]:
+        """The layer runs in order: (layer, pass, does a pass of the loop start here?)."""
+        n = len(self.layers)
+        if self.loop is None:
+            return [(i, 0, False) for i in range(n)]
+        start, stop, times = self.loop
+        runs = [(i, 0, False) for i in range(start)]
+        for t in range(times):
+            runs += [(i, t, i == start) for i in range(start, stop)]
+        return runs + [(i, 0, False) for i in range(stop, n)]
+
+    def weight_shapes(self) -> dict[str, tuple[int, ...]]:
+        """Name -> shape of every tensor of a checkpoint."""
+        v, d, s = self.vocab_size, self.hidden_size, self.side_dim
+        out: dict[str, tuple[int, ...]] = {"embed": (v, d), "final.norm": (d,), "head": (v, d)}
+        if self.loop:
+            out["loop.step"] = (self.loop[2], d)
+        if s:
+            out["side.embed"] = (v, s * len(self.layers))
+        for i, layer in enumerate(self.layers):
+            a, p = layer.attention, f"l{i}."
+            out[p + "norm1"] = (d,)
+            out[p + "mix.q"], out[p + "mix.k"] = (a.heads * a.dim, d), (a.kv_heads * a.dim, d)
+            out[p + "mix.o"] = (d, a.heads * a.dim)
+            if layer.ff:
+                out[p + "mlp.gate"] = out[p + "mlp.up"] = (layer.ff, d)
+                out[p + "mlp.down"] = (d, layer.ff)
+            if s:
+                out[p + "side.gate"], out[p + "side.proj"], out[p + "side.norm"] = (s, d), (d, s), (d,)
+        return out
+
+
+NATIVE_CONFIGS = {"Mofarax": MofaraxConfig}
+
+
+def load_native_config(model_dir: str):
+    """The configuration of a directory whose config.json names one of these architectures, else None."""
+    path = Path(model_dir) / "config.json"
+    if not path.is_file():
+        return None
+    raw = json.loads(path.read_text())
+    name = raw.get("architecture") if isinstance(raw, dict) else None
+    if name is None:
+        return None
+    if name not in NATIVE_CONFIGS:
+        raise ValueError(f"unsupported architecture {name!r} in {path}; known: {sorted(NATIVE_CONFIGS)}")
+    return NATIVE_CONFIGS[name](raw)

@@ -115,6 +115,7 @@ def load_model(model: nn.Module, model_path: str | Path) -> None:
         raise ValueError(f"No .safetensors or .bin files found in {base}")
     mapping = getattr(model, "packed_modules_mapping", {})
     total = loaded = 0
+    names: set[str] = set()      # tensors that found their place
     for path in st_files:
         from safetensors import safe_open
 
@@ -127,13 +128,20 @@ def load_model(model: nn.Module, model_path: str | Path) -> None:
         with safe_open(str(path), framework="pt", device=dev_s) as f:
             for name in f.keys():  # noqa: SIM118
                 total += 1
-                loaded += load_weight(model, name, LazyTensor(f.get_slice(name), dev), mapping)
+                if load_weight(model, name, LazyTensor(f.get_slice(name), dev), mapping):
+                    loaded += 1
+                    names.add(name)
     for path in bin_files:
         state = torch.load(str(path), map_location="cpu", weights_only=True)
         for name, tensor in state.items():
             total += 1
-            loaded += load_weight(model, name, tensor, mapping)
+            if load_weight(model, name, tensor, mapping):
+                loaded += 1
+                names.add(name)
         del state
+    check = getattr(model, "check_loaded", None)   # a model may insist on its exact set of tensors
+    if check is not None:
+        check(names)
     if loaded < total:
         logger.warning("Weight loading completed with %d missing parameter(s) out of %d", total - loaded, total)
     logger.info("Loaded %d/%d weights from %s", loaded, total, base)
