@@ -343,11 +343,11 @@ def add_rmsnorm_partial(partial, residual, weight, eps: float):
 
 
 # ---------------------------------------------------------------- K7
-def _rot_tables_ok(cos, sin, d: int, interleaved_pairs) -> None:
+def _rot_tables_ok(cos, sin, d: int, interleaved_pairs) -> bool:
+    """cos / sin are dense fp32 [max_pos, rotated pairs] tables."""
     want = d // 2 if interleaved_pairs is None else int(interleaved_pairs)
-    if cos.shape != sin.shape or cos.dim() != 2 or cos.shape[1] != want or not (cos.is_contiguous() and sin.is_contiguous()) \
-            or cos.dtype != torch.float32 or sin.dtype != torch.float32:
-        raise MvHipError(f"cos / sin must be dense fp32 [max_pos, {want}] tables")
+    return (cos.shape == sin.shape and cos.dim() == 2 and cos.shape[1] == want and cos.is_contiguous() and sin.is_contiguous()
+            and cos.dtype == torch.float32 and sin.dtype == torch.float32)
 
 
 def rope_qk_store(q, k, v, positions, cos, sin, q_norm_w=None, k_norm_w=None, eps: float = 1e-6,
@@ -375,7 +375,8 @@ def rope_qk_store(q, k, v, positions, cos, sin, q_norm_w=None, k_norm_w=None, ep
     pos = positions if positions.dtype == torch.int64 else positions.to(torch.int64)
     qn = q_norm_w if q_norm_w is None or q_norm_w.dtype == q.dtype else q_norm_w.to(q.dtype)
     kn = k_norm_w if k_norm_w is None or k_norm_w.dtype == q.dtype else k_norm_w.to(q.dtype)
-    _rot_tables_ok(cos, sin, d, interleaved_pairs)
+    if not _rot_tables_ok(cos, sin, d, interleaved_pairs):
+        raise MvHipError(f"cos / sin: dense fp32 [max_pos, rotated pairs] tables required, got {tuple(cos.shape)}")
     _check(_lib.mv_rope_qk_store_ex(
         q.data_ptr(), k.data_ptr(), _ptr(v), q.stride(0), k.stride(0), v.stride(0) if v is not None else 0,
         pos.data_ptr(), cos.data_ptr(), sin.data_ptr(), cos.shape[0], _ptr(qn), _ptr(kn), float(eps),
@@ -448,7 +449,8 @@ def rope_paged_decode(q, k, v, positions, cos, sin, q_norm_w, k_norm_w, eps: flo
     if out is None:
         out = torch.empty((b, h, d), dtype=q.dtype, device=q.device)
     _out_rows(out, b, h, d)
-    _rot_tables_ok(cos, sin, d, interleaved_pairs)
+    if not _rot_tables_ok(cos, sin, d, interleaved_pairs):
+        return None
     pos = positions if positions.dtype == torch.int64 else positions.to(torch.int64)
     qn = q_norm_w if q_norm_w is None or q_norm_w.dtype == q.dtype else q_norm_w.to(q.dtype)
     kn = k_norm_w if k_norm_w is None or k_norm_w.dtype == q.dtype else k_norm_w.to(q.dtype)

@@ -59,6 +59,7 @@ def _executor(tmp_path, cfg_dict, dtype=torch.bfloat16, blocks=160, max_num_seqs
             mod.pack_for_decode()
     ex = InferenceExecutor(cfg, model, torch.device(DEV))
     ex._allocate_kv_cache()
+    ex.kv_cache.zero_()      # whole caches are compared below: slots nobody wrote must not hold another test's NaNs
     ex._initialize_sampler()
     ex._optimize_model()
     return cfg, model, ex
