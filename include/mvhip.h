@@ -423,7 +423,7 @@ int mv_add_rmsnorm_partial(const float *partial, int splits, void *residual, int
 size_t mv_ar_region_bytes(size_t max_bytes);
 int mv_ar_max_world(void);
 int mv_ar_alloc(size_t max_bytes, void **base_out);
-int mv_ar_free(void *base);
+int mv_ar_free(void *base);   /* waits for the device; the memory itself is returned when the process ends */
 int mv_ar_ipc_handle_bytes(void);
 int mv_ar_ipc_export(void *base, void *handle_out);
 int mv_ar_ipc_open(const void *handle, void **ptr_out);

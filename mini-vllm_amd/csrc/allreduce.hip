@@ -507,7 +507,9 @@ extern "C" int mv_ar_set_wait_limit_ms(void *base, size_t max_bytes, uint32_t ms
                                 sizeof(ms), hipMemcpyHostToDevice));
 }
 
-extern "C" int mv_ar_free(void *base) { return base ? mv_check_hip(hipFree(base)) : MV_OK; }
+// Gives the region up without freeing it: after a kernel has read uncached memory, later allocations over the freed range
+// have held wrong values, so it stays mapped until the process ends (a few MiB, one region per process as a rule).
+extern "C" int mv_ar_free(void *base) { return base ? mv_check_hip(hipDeviceSynchronize()) : MV_OK; }
 
 extern "C" int mv_ar_ipc_handle_bytes(void) { return (int)sizeof(hipIpcMemHandle_t); }
 
