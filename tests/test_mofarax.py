@@ -10,6 +10,16 @@ from mofarax_configs import CONFIGS, config, layer, sharp_weights, write_checkpo
 from oracle import mofarax as M
 
 
+@pytest.fixture(autouse=True)
+def _single_rank():
+    """The models are built for one rank, whatever earlier tests of this process left behind."""
+    from minivllm_amd import parallel_state
+
+    parallel_state.reset_tensor_parallel()
+    yield
+    parallel_state.reset_tensor_parallel()
+
+
 # ---- the plain implementation ------------------------------------------------------------------------------------------
 def test_rotation_is_relative_and_leaves_the_tail():
     g = torch.Generator().manual_seed(0)
