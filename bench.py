@@ -76,6 +76,28 @@ MODELS = {
                       rms_norm_eps=1e-6, rope_theta=1000000.0, tie_word_embeddings=False, hidden_act="silu",
                       torch_dtype="bfloat16", eos_token_id=151645),
 }
+
+
+def _mofarax(like: str, side_dim: int = 128, layers: int = 20, loop=(8, 12, 3), chunk: int = 2048) -> dict:
+    """A Mofarax configuration whose layer runs (28: 20 layers, four of them passed three times) have the sizes of
+    ``like``'s layers; the keys behind the first line are what this script itself asks of a model."""
+    c = MODELS[like]
+    heads, kv, width, vocab = (c[k] for k in ("num_attention_heads", "num_key_value_heads", "hidden_size", "vocab_size"))
+    dim = c.get("head_dim") or width // heads
+    mixer = {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "mask": {"size": chunk},
+             "rot": {"base": c["rope_theta"], "dims": dim}}
+    layer = {"type": "attention", "mixer": mixer, "mlp": {"kind": "dense", "ff": c["intermediate_size"]}}
+    assert layers + (loop[1] - loop[0]) * (loop[2] - 1) == c["num_hidden_layers"]
+    return dict(architecture="Mofarax", vocab=vocab, width=width, embedding={"scale": width ** 0.5}, norm={"eps": 1e-6},
+                layers=[layer] * layers, loop=dict(zip(("start", "stop", "times"), loop)), token_side={"dim": side_dim},
+                like=like, chunk=chunk, vocab_size=vocab, hidden_size=width, num_attention_heads=heads, num_key_value_heads=kv,
+                head_dim=dim, intermediate_size=c["intermediate_size"])
+
+
+DESIGNS = {"mofarax": {"mofarax-0.6b": "qwen3-0.6b", "mofarax-1.7b": "qwen3-1.7b", "mofarax-7b": "qwen2-7b"}}
+MODELS.update({name: _mofarax(like) for name, like in DESIGNS["mofarax"].items()})
+DESIGN_DECODE = ((256, 1024), (16, 1024), (1, 1024))      # (batch, context) of a design's decode records
+DESIGN_PREFILL = ((16, 1024), (4, 4096))
 HBM_PEAK_GBS = 8000.0  # MI355X_MICROARCH.md: HBM3E 8.0 TB/s spec (6.29 TB/s measured copy ceiling)
 MFMA_PEAK_TFLOPS = 2500.0  # MI355X_MICROARCH.md: ~2.5 PFLOP/s dense bf16 (the 5 PF headline includes 2:1 sparsity)
 L2_INGEST_GBS_PER_CU = (66.0, 73.0)  # MI355X_MICROARCH.md "Indexed rows: gather into LDS": rows shared by every workgroup, served by the XCD's L2
@@ -113,6 +135,9 @@ def parse(argv=None):
                     help="(with --gpus 2, ranks sharing one card) run the N = 8 record flow on stand-ins: a Qwen2-7B-like model "
                          "whose heads do not divide by 2 (-> the rejection record) and a 4-layer model at Qwen2-72B's per-layer "
                          "dimensions on an explicit KV pool; the records are marked as a rehearsal")
+    ap.add_argument("--design", choices=list(DESIGNS),
+                    help="instead of the headline: decode and prefill throughput of this model design at several sizes, each "
+                         "beside the closest other model with layers of the same size (one GPU, random weights)")
     ap.add_argument("--cpu-config1-only", action="store_true",
                     help="run only the CPU leg of BASELINE config 1 (OPT-125M fp32, reference preset) and print it")
     return ap.parse_args(argv)
@@ -413,6 +438,8 @@ def projection_roofline(engine, rows: int):
     from minivllm_amd.layers.linear import linear, mid_m
 
     ex = engine.model_runner.inference_executor
+    if not hasattr(ex.model, "model"):
+        return None               # (a model without separate q/k/v, o, gate/up and down projections)
     layers = list(ex.model.model.layers)
     dev, dt = ex.device, ex.dtype
     g = torch.Generator(device=dev).manual_seed(7)
@@ -479,13 +506,15 @@ def step_roofline(engine, model, batch, ctx_mid, ms_per_step):
     rows excluded, the tied / untied LM head shard included) + the K/V bytes of the batch at its mean context."""
     ex = engine.model_runner.inference_executor
     seen, wbytes = set(), 0
+    # weights of looped layers are read once a pass
+    passes = {id(m): len(layer.attn) for layer in getattr(ex.model, "stack", []) for m in layer.modules()}
     for mod in ex.model.modules():
         w = getattr(mod, "weight", None)
         if w is None or w.dim() != 2 or w.data_ptr() in seen:
             continue
         if hasattr(mod, "input_size") or type(mod).__name__ == "ParallelLMHead":
             seen.add(w.data_ptr())
-            wbytes += w.numel() * w.element_size()
+            wbytes += w.numel() * w.element_size() * passes.get(id(mod), 1)
     L, nb, bs, hkv, d = ex.kv_cache.shape[1:]
     kv = L * batch * ctx_mid * 2 * hkv * d * ex.dtype.itemsize
     gbs = (wbytes + kv) / (ms_per_step * 1e-3) / 1e9
@@ -510,9 +539,11 @@ def release_all(engine):
     torch.cuda.synchronize()
 
 
-def prefill_flops(heads: int, head_dim: int, lens) -> int:
+def prefill_flops(heads: int, head_dim: int, lens, chunk: int = 0) -> int:
     """Causal flash prefill without a cached prefix, one layer (SURVEY §8 d, K2): sum over sequences of
-    4 H D (Sq Sk - Sq (Sq - 1) / 2) with Sq = Sk = len."""
+    4 H D (Sq Sk - Sq (Sq - 1) / 2) with Sq = Sk = len; a chunk mask cuts a sequence into pieces of ``chunk`` tokens."""
+    if chunk:
+        lens = [m for n in lens for m in [chunk] * (n // chunk) + [n % chunk]]
     return sum(4 * heads * head_dim * (n * n - n * (n - 1) // 2) for n in lens)
 
 
@@ -571,7 +602,7 @@ def prefill_records(engine, model, gpus=1, cases=PREFILL_CASES, reps=5):
         m = statistics.median(t_us)
         kept = [t for t in t_us if t <= 3 * m]
         us = sum(kept) / len(kept)
-        flops = prefill_flops(heads, head_dim, [ln] * n)
+        flops = prefill_flops(heads, head_dim, [ln] * n, cfgm.get("chunk", 0))
         tf = flops / us / 1e6
         out.append({"metric": "prefill tokens/s", "model": model, "tp": gpus, "prompts": n, "prompt_len": ln,
                     "batches_timed": reps, "warmup_batches": 1, "ms_per_batch": round(med * 1e3, 3),
@@ -892,8 +923,62 @@ def init_process_group(args):
     return dist
 
 
+def design_records(args, workdir) -> dict:
+    """``--design``: for every size of the design and for its peer, decode at several batches and prefill, on one engine each."""
+    import gc
+
+    out = {}
+    for name, like in DESIGNS[args.design].items():
+        for model in (name, like):
+            a = argparse.Namespace(**vars(args))
+            a.model, a.batch, a.ctx = model, max(b for b, _ in DESIGN_DECODE), max(c for _, c in DESIGN_DECODE)
+            os.environ["MV_GRAPH_BATCH_SIZES"] = ",".join(str(b) for b, _ in DESIGN_DECODE)
+            note(f"building {model}")
+            engine = build_engine(a, os.path.join(workdir, model), model)
+            os.environ.pop("MV_GRAPH_BATCH_SIZES", None)
+            recs = []
+            for i, (batch, ctx) in enumerate(DESIGN_DECODE):
+                a.batch, a.ctx = batch, ctx
+                rec, _ = decode_record(engine, a, model, None, seed=i, probes=True)
+                recs.append(rec)
+                release_all(engine)
+            for n, ln in DESIGN_PREFILL:
+                note(f"{model} prefill {n} x {ln}")
+                recs += prefill_records(engine, model, cases=((n, ln),))
+            engine.exit()
+            del engine
+            gc.collect()
+            torch.cuda.empty_cache()
+            out[model] = recs
+    return out
+
+
+def design_line(args, records: dict) -> dict:
+    """The JSON line of ``--design``: value = decode tokens/s of the last (largest) size, the pairs beside each other."""
+    pairs = []
+    for name, like in DESIGNS[args.design].items():
+        for mine, peer in zip(records[name], records[like]):
+            what = (f"prefill {mine['prompts']} x {mine['prompt_len']}" if "prompts" in mine
+                    else mine["config"]["workload"].split(" ", 1)[1].split(", kvcache")[0])
+            pairs.append({"model": name, "peer": like, "workload": what, "tokens_per_s": [mine["value"], peer["value"]],
+                          "ratio": round(mine["value"] / peer["value"], 4),
+                          "attention_frac_of_peak": [mine["roofline"]["frac"], peer["roofline"]["frac"]],
+                          "step_frac_of_hbm_peak": [(r.get("step_roofline") or {}).get("frac") for r in (mine, peer)]})
+    last = list(DESIGNS[args.design])[-1]
+    head = records[last][0]
+    return {"metric": f"{args.design} decode tokens/s", "value": head["value"], "unit": "tokens/s", "n_gpus": 1, "steps": args.steps,
+            "warmup": args.warmup, "ms_per_step": head["ms_per_step"], "higher_is_better": True, "scaling": "strong",
+            "vs_baseline": None, "dtype": "bf16", "data": "synthetic", "config": head["config"], "pairs": pairs, "records": records}
+
+
 def main():
     args = parse()
+    if args.design:
+        if args.gpus != 1:
+            raise SystemExit("--design runs on one GPU")
+        with tempfile.TemporaryDirectory() as workdir:
+            print(json.dumps(design_line(args, design_records(args, workdir))))
+        return
     if args.cpu_config1_only:
         print(json.dumps(cpu_config1()))
         return
