@@ -320,6 +320,12 @@ int mv_residual_update(const MvResidualArgs *args, int rows, int cols, int cols_
 int mv_gated_lookup(const void *s, int64_t s_stride, const void *table, int64_t table_stride, int64_t vocab,
                     int offset, const int64_t *ids, void *out, int64_t out_stride, int rows, int dim, int cols,
                     int dtype, void *stream);
+/* ... and the projection behind it in one launch, for decode-sized batches: out[t][i] = sum_j r(g[t][j]) * W[i][j] with g
+ * as above, r() its rounding to dtype, W [n, k] packed by mv_pack_weight (k >= dim: zero columns behind), k % 32 == 0,
+ * k <= 512, n % 4 == 0, 16-bit dtypes; MV_E_SHAPE otherwise. */
+int mv_gated_lookup_linear(const void *s, int64_t s_stride, const void *table, int64_t table_stride, int64_t vocab,
+                           int offset, const int64_t *ids, const void *w_packed, void *out, int64_t out_stride, int rows,
+                           int dim, int k, int n, int dtype, void *stream);
 
 /* K10 — decode-sized linear layer: out[m, :] = x[m, :] . W^T (+ bias), 1 <= M <= 64 rows, 16-bit
  * dtypes, fp32 accumulation, one rounding at the end.  Replaces the F.linear calls of the decode step
@@ -338,7 +344,9 @@ int mv_linear_small_m(const void *x, int64_t x_stride, const void *w,
  * out[m, j] = silu(x[m,:] . Wg[j,:]) * (x[m,:] . Wu[j,:]),  w_gate_up = [Wg ; Wu] of shape [2*n_inter, K]
  * (the merged layout of MergedColumnParallelLinear, minivllm/models/layers/linear.py:166-231), with the
  * rounding points of the unfused pair gate_up_proj -> act_fn (minivllm/models/qwen_base.py:232-234):
- * both GEMM outputs, silu and the product are each rounded to dtype.  Same limits as mv_linear_small_m. */
+ * both GEMM outputs, silu and the product are each rounded to dtype.  Same limits as mv_linear_small_m.
+ * MV_GATE_GELU in `shape` (the mid-M form: in `cfg`): gelu (tanh form) instead of silu, in fp32 up to one rounding. */
+enum { MV_GATE_GELU = 1 << 16 };
 int mv_gate_up_silu_small_m(const void *x, int64_t x_stride, const void *w_gate_up,
                             void *out, int64_t out_stride, int m, int n_inter,
                             int k, int dtype, int shape, void *stream);

@@ -138,6 +138,17 @@ __device__ __forceinline__ float gelu_tanh(float z) {
   return z / (1.0f + expf(-u2));
 }
 
+// act(gate) * up on the fp32 accumulators of a gated projection.  gelu: fp32 throughout.  silu: the rounding points of the
+// unfused pair (GEMM -> dtype, silu -> dtype, product in fp32; the caller rounds it)
+template <typename Tag>
+__device__ __forceinline__ float gated_act(float gate, float up, bool gelu) {
+  if (gelu) return __fmul_rn(gelu_tanh(gate), up);
+  const float gt = elem<Tag>::ld(elem<Tag>::st(gate)), ut = elem<Tag>::ld(elem<Tag>::st(up));
+  float sl = gt / (1.0f + expf(-gt));                        // rmsnorm.hip: silu_and_mul_kernel
+  sl = elem<Tag>::ld(elem<Tag>::st(sl));
+  return __fmul_rn(sl, ut);
+}
+
 // ---- rotary embedding ------------------------------------------------------
 // A head row of D elements lies on LPT = D / VEC adjacent lanes, VEC per lane (sub = lane within the row).  Two layouts:
 //   halves (NeoX):  dim i pairs with dim i + D/2, i < D/2; the partner sits LPT/2 lanes away; cos / sin [max_pos, D/2]

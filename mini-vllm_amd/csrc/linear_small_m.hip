@@ -43,6 +43,7 @@ struct LinearParams {
   void *nres_out = nullptr;
   int64_t nres_stride = 0, nres_out_stride = 0;
   float eps = 0.f;
+  int gelu = 0;          // GATED: gelu (tanh form) instead of silu
   int norm_threads = 0;  // block size of the rmsnorm_kernel launch this prologue re-enacts
 };
 
@@ -341,13 +342,7 @@ linear_small_m_kernel(LinearParams p) {
     if constexpr (GATED) {
       const f32x4 up = tile_sum(t + RPW * MT);
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const float gt = elem<Tag>::ld(elem<Tag>::st(o[i]));  // the GEMM output as the unfused path stores it
-        const float ut = elem<Tag>::ld(elem<Tag>::st(up[i]));
-        float sl = gt / (1.0f + expf(-gt));                     // rmsnorm.hip: silu_and_mul_kernel
-        sl = elem<Tag>::ld(elem<Tag>::st(sl));
-        o[i] = __fmul_rn(sl, ut);
-      }
+      for (int i = 0; i < 4; ++i) o[i] = gated_act<Tag>(o[i], up[i], p.gelu != 0);
     }
     if (m < p.M && n < p.N) {
       if (!GATED && p.bias) {
@@ -535,6 +530,7 @@ extern "C" int mv_gate_up_silu_small_m(const void *x, int64_t x_stride, const vo
   if (m == 0 || n_inter == 0) return MV_OK;
   if (int e = check(x, x_stride, w_gate_up, nullptr, out, out_stride, m, n_inter, k, dtype)) return e;
   LinearParams p{x, w_gate_up, nullptr, out, x_stride, out_stride, m, n_inter, k};
+  p.gelu = (shape & MV_GATE_GELU) ? 1 : 0;
   return run<true>(p, dtype, shape, (hipStream_t)stream);
 }
 
@@ -556,6 +552,7 @@ extern "C" int mv_gate_up_silu_small_m_packed(const void *x, int64_t x_stride, c
   if (n_inter & 15) return MV_E_SHAPE;  // the up rows must start on a tile boundary of the packed copy
   if (int e = check(x, x_stride, w_gate_up_packed, nullptr, out, out_stride, m, n_inter, k, dtype)) return e;
   LinearParams p{x, w_gate_up_packed, nullptr, out, x_stride, out_stride, m, n_inter, k};
+  p.gelu = (shape & MV_GATE_GELU) ? 1 : 0;
   return run<true, true>(p, dtype, shape, (hipStream_t)stream);
 }
 

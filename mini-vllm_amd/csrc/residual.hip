@@ -2,7 +2,8 @@
 //   mv_residual_update: one launch per edge of the stream — [start the row from a scaled embedding] + the output of the
 //     projections in front (plain, or RMS-normed by a weight of its own; or the fp32 partial sums of a K split)
 //     [+ the scaled embedding] [+ a vector] -> the stream, and what the next projection reads: its RMSNorm or its cast;
-//   mv_gated_lookup: gelu(s) * a slice of a per-token table (the per-token layer input).
+//   mv_gated_lookup: gelu(s) * a slice of a per-token table (the per-token layer input);
+//   mv_gated_lookup_linear: the same with the projection behind it, one launch for decode-sized batches.
 // One workgroup per row, the row in registers between the reductions and the store: the stream is read and written once.
 #include "common.h"
 
@@ -184,6 +185,71 @@ __global__ void __launch_bounds__(256) gated_lookup_kernel(const typename elem<T
   }
 }
 
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef _Float16 f16x8 __attribute__((ext_vector_type(8)));
+
+template <typename Tag>
+__device__ __forceinline__ f32x4 side_mfma(u32x4 a, u32x4 b, f32x4 c) {
+  if constexpr (__is_same(Tag, bf16_tag))
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b), c, 0, 0, 0);
+  else
+    return __builtin_amdgcn_mfma_f32_16x16x32_f16(__builtin_bit_cast(f16x8, a), __builtin_bit_cast(f16x8, b), c, 0, 0, 0);
+}
+
+// out[t][n] = sum_j g[t][j] W[n][j], g = gated_lookup_kernel's row rounded to the dtype.  One workgroup: 16 tokens x 64
+// outputs, one 16-wide tile of W per wave.  W comes fragment-ordered (mv_pack_weight: the A operand, 1 KiB per wave-wide
+// load) and its first kAhead k-steps are in flight while the workgroup computes its 16 rows of g into LDS, which holds them
+// in the B operand's order: [k-step][lane][8], lane l = token l & 15, k group l >> 4.
+constexpr int kSideAhead = 4, kSideMaxK = 512;
+template <typename Tag>
+__global__ void __launch_bounds__(256) gated_lookup_linear_kernel(const uint16_t *s, int64_t s_stride, const uint16_t *table,
+                                                                  int64_t table_stride, int64_t vocab, int offset,
+                                                                  const int64_t *ids, const uint16_t *wp, uint16_t *out,
+                                                                  int64_t out_stride, int rows, int dim, int K, int N,
+                                                                  bool table_vec) {
+  __shared__ u32x4 g[kSideMaxK / 32 * 64];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, steps = K / 32;
+  const int m0 = blockIdx.y * 16, tile = blockIdx.x * 4 + wave, tiles = (N + 15) / 16;
+  const u32x4 *w = (const u32x4 *)wp + (int64_t)(tile < tiles ? tile : tiles - 1) * steps * 64 + lane;
+  u32x4 wf[kSideAhead];
+#pragma unroll
+  for (int i = 0; i < kSideAhead; ++i) wf[i] = w[(i < steps ? i : steps - 1) * 64];
+  for (int v = threadIdx.x; v < steps * 64; v += 256) {
+    const int l = v & 63, m = m0 + (l & 15), c = (v >> 6) * 32 + (l >> 4) * 8;
+    float a[8], e[8], o[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) o[j] = 0.f;
+    const int64_t id = m < rows ? ids[m] : -1;
+    if (id >= 0 && id < vocab && c < dim) {
+      load_row_vec<Tag>(s + (int64_t)m * s_stride + c, a);
+      const uint16_t *tr = table + id * table_stride + offset + c;
+      if (table_vec && c + 8 <= dim) {
+        load_row_vec<Tag>(tr, e);
+      } else {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) e[j] = c + j < dim ? elem<Tag>::ld(tr[j]) : 0.f;
+      }
+#pragma unroll
+      for (int j = 0; j < 8; ++j) o[j] = c + j < dim ? gelu_tanh(a[j]) * e[j] : 0.f;
+    }
+    g[v] = pack8<Tag>(o);
+  }
+  __syncthreads();
+  f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int i = 0; i < kSideAhead; ++i)
+    if (i < steps) acc = side_mfma<Tag>(wf[i], g[i * 64 + lane], acc);
+  for (int i = kSideAhead; i < steps; ++i) acc = side_mfma<Tag>(w[i * 64], g[i * 64 + lane], acc);
+  // C layout: lane holds W rows n = (lane >> 4) * 4 + {0..3} (consecutive outputs) of token lane & 15
+  const int m = m0 + (lane & 15), n = tile * 16 + (lane >> 4) * 4;
+  if (m < rows && n < N) {
+    u32x2 pk;
+    pk[0] = (uint32_t)elem<Tag>::st(acc[0]) | ((uint32_t)elem<Tag>::st(acc[1]) << 16);
+    pk[1] = (uint32_t)elem<Tag>::st(acc[2]) | ((uint32_t)elem<Tag>::st(acc[3]) << 16);
+    *(u32x2 *)(out + (int64_t)m * out_stride + n) = pk;
+  }
+}
+
 }  // namespace
 
 extern "C" int mv_residual_update(const MvResidualArgs *a, int rows, int cols, int cols_true, int dtype, void *stream) {
@@ -240,6 +306,29 @@ extern "C" int mv_gated_lookup(const void *s, int64_t s_stride, const void *tabl
                        s_stride, (const T *)table, table_stride, vocab, offset, ids, (T *)out, out_stride, rows, dim, cols,
                        table_vec);
   });
+  MV_LAUNCH_CHECK();
+  return MV_OK;
+}
+
+extern "C" int mv_gated_lookup_linear(const void *s, int64_t s_stride, const void *table, int64_t table_stride, int64_t vocab,
+                                      int offset, const int64_t *ids, const void *w_packed, void *out, int64_t out_stride,
+                                      int rows, int dim, int k, int n, int dtype, void *stream) {
+  if (rows == 0 || n == 0) return MV_OK;
+  if (!s || !table || !ids || !w_packed || !out) return MV_E_NULLPTR;
+  if (dtype != MV_BF16 && dtype != MV_F16) return dtype == MV_F32 ? MV_E_SHAPE : MV_E_DTYPE;
+  if (rows < 0 || dim <= 0 || k < dim || vocab <= 0 || offset < 0 || offset + dim > table_stride || n < 0 || (n & 3))
+    return MV_E_SHAPE;
+  if ((k & 31) || k > kSideMaxK || rows > 16 * 65535) return MV_E_SHAPE;
+  if (!mv_aligned16(s) || !mv_aligned16(w_packed) || (((uintptr_t)out) & 7u) || (s_stride & 7) || (out_stride & 3)) return MV_E_ALIGN;
+  const bool table_vec = mv_aligned16(table) && table_stride % 8 == 0 && offset % 8 == 0;
+  const dim3 grid((unsigned)((n + 63) / 64), (unsigned)((rows + 15) / 16));
+#define MV_SIDE(TAG)                                                                                                          \
+  hipLaunchKernelGGL((gated_lookup_linear_kernel<TAG>), grid, dim3(256), 0, (hipStream_t)stream, (const uint16_t *)s, s_stride, \
+                     (const uint16_t *)table, table_stride, vocab, offset, ids, (const uint16_t *)w_packed, (uint16_t *)out,   \
+                     out_stride, rows, dim, k, n, table_vec)
+  if (dtype == MV_BF16) MV_SIDE(bf16_tag);
+  else MV_SIDE(f16_tag);
+#undef MV_SIDE
   MV_LAUNCH_CHECK();
   return MV_OK;
 }

@@ -1,12 +1,12 @@
 """Mofarax decoder glue.
 
 Attention and feed-forward of a layer read ONE norm and are summed, and the residual stream is fp32, so a layer is
-    [q | k | gate | up] GEMM                                           one merged weight
+    [q | k] GEMM
     -> rotation + K/V store + attention (decode: ONE launch)           into the left columns of `mixed`
-    -> gelu(gate) * up                                                 into its right columns
+    [gate | up] GEMM with gelu(gate) * up                              into its right columns (decode: ONE launch)
     -> [o | down] GEMM over `mixed`                                    both sublayers summed in the accumulators
     -> residual += that; cast                                          (mv_residual_update)
-    -> side gate GEMM -> gelu * token table -> side projection GEMM
+    -> side gate GEMM -> gelu * token table -> side projection GEMM    (decode: the last two in ONE launch)
     -> residual += rms(.) * w [+ embedding + pass vector]; next layer's norm    (mv_residual_update)
 Layers of the loop run several times over the same weights; each pass has attention modules (K/V planes) of its own.
 Values are the projected keys before rotation: the K plane of the cache holds rotated keys, the V plane the raw ones.
@@ -20,7 +20,7 @@ from torch import nn
 
 from .. import hip_ops
 from ..layers import Attention, ParallelLMHead, Segment, SegmentedLinear, get_rope
-from ..layers.linear import divide, pad_to
+from ..layers.linear import MID_M_MAX, divide, gated_linear, pad_to
 from ..parallel_state import get_tensor_parallel_world_size
 from ..utils.context import get_context
 from ..utils.loader import load_weight, materialize
@@ -64,6 +64,9 @@ class SideInput(nn.Module):
         self.norm = _padded(pad_to(width))
 
     def forward(self, x, ids, table):
+        packed, n = self.proj.weight_packed, self.proj.weight.shape[0]
+        if packed is not None and x.shape[0] <= MID_M_MAX and self.proj.weight.shape[1] <= hip_ops.GATED_LOOKUP_LINEAR_MAX_K:
+            return hip_ops.gated_lookup_linear(self.gate(x), table, self.offset, self.dim, ids, packed, n)
         return self.proj(hip_ops.gated_lookup(self.gate(x), table, self.offset, self.dim, ids))
 
 
@@ -75,12 +78,11 @@ class MofaraxLayer(nn.Module):
         self.heads, self.kv_heads, self.ff = divide(a.heads, tp), divide(a.kv_heads, tp), spec.ff
         self.head_dim = d = kernel_head_dim(a.dim)
         self.norm1 = _padded(pad_to(width))
-        cols = [Segment("q", a.heads, a.dim, d), Segment("k", a.kv_heads, a.dim, d)]
         rows = [Segment("o", a.heads, a.dim, d)]
+        self.qk = SegmentedLinear(width, [Segment("q", a.heads, a.dim, d), Segment("k", a.kv_heads, a.dim, d)], split="out")
         if spec.ff:
-            cols += [Segment("gate", spec.ff), Segment("up", spec.ff)]
+            self.gate_up = SegmentedLinear(width, [Segment("gate", spec.ff), Segment("up", spec.ff)], split="out")
             rows += [Segment("down", spec.ff)]
-        self.proj_in = SegmentedLinear(width, cols, split="out")
         self.proj_out = SegmentedLinear(width, rows, split="in")
         self.rotary = get_rope(d, a.rot_dims, config.max_position_embeddings or 4096, a.rot_base, interleaved=True)
         # one per pass of the loop: the weights are shared, the K/V planes are not
@@ -110,21 +112,20 @@ class MofaraxLayer(nn.Module):
     def forward(self, h, positions, run: int):
         """attention(h) + mlp(h) of pass ``run``: [T, width] (or its K-split partial sums)."""
         t, d = h.shape[0], self.head_dim
-        z = self.proj_in(h)
-        at = self.proj_in.offsets
+        z, k_at = self.qk(h), self.qk.offsets["k"]
         q = z[:, :self.heads * d].view(t, self.heads, d)
-        k = z[:, at["k"]:at["k"] + self.kv_heads * d].view(t, self.kv_heads, d)
+        k = z[:, k_at:k_at + self.kv_heads * d].view(t, self.kv_heads, d)
         mixed = torch.empty((t, self.proj_out.weight.shape[1]), dtype=h.dtype, device=h.device)
         self._attend(self.attn[run], q, k, positions, mixed[:, :self.heads * d].view(t, self.heads, d))
         if self.ff:
-            hip_ops.gelu_and_mul(z[:, at["gate"]:], out=mixed[:, self.proj_out.offsets["down"]:])
+            gated_linear(h, self.gate_up, "gelu_tanh", out=mixed[:, self.proj_out.offsets["down"]:])
         return self.proj_out(mixed, partial_ok=True)
 
 
 class MofaraxForCausalLM(nn.Module):
     # checkpoint name fragment -> (parameter, segment); a trailing fragment wins over nothing, so the order is free
-    packed_modules_mapping = {".mix.q": (".proj_in.weight", "q"), ".mix.k": (".proj_in.weight", "k"),
-                              ".mlp.gate": (".proj_in.weight", "gate"), ".mlp.up": (".proj_in.weight", "up"),
+    packed_modules_mapping = {".mix.q": (".qk.weight", "q"), ".mix.k": (".qk.weight", "k"),
+                              ".mlp.gate": (".gate_up.weight", "gate"), ".mlp.up": (".gate_up.weight", "up"),
                               ".mix.o": (".proj_out.weight", "o"), ".mlp.down": (".proj_out.weight", "down"),
                               ".side.gate": (".side.gate.weight", "gate"), ".side.proj": (".side.proj.weight", "proj"),
                               "side.embed": ("side_embed", None), "final.norm": ("final_norm", None),

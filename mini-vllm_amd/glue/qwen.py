@@ -19,7 +19,7 @@ from torch import nn
 from .. import hip_ops
 from ..layers import (Attention, MergedColumnParallelLinear, ParallelLMHead, QKVParallelLinear, RMSNorm,
                       RowParallelLinear, SiluAndMul, VocabParallelEmbedding, get_rope)
-from ..layers.linear import mid_m, mid_plan, small_m
+from ..layers.linear import gated_linear, small_m
 from ..parallel_state import get_tensor_parallel_world_size, tp_all_reduce_add_rmsnorm
 from ..utils.context import get_context
 
@@ -200,23 +200,14 @@ class QwenMLP(nn.Module):
         self.hidden_act, self.intermediate_size, self.hidden_size = hidden_act, intermediate_size, hidden_size
 
     def forward(self, x, reduce: bool = True):
-        w, gu = self.gate_up_proj.weight, self.gate_up_proj
+        gu = self.gate_up_proj
         flat = x.dim() == 2
         if isinstance(x, PendingNorm):   # the post-attention norm rides in the gate_up launch
             act = x.project(gu, gated=True)
             if act is not None:
                 return self.down_proj(act, reduce=reduce, partial_ok=flat)
             x = x.materialize()
-        if small_m(x, w):  # decode-sized batch: SiluAndMul in the epilogue of the weight-streaming gate_up kernel
-            return self.down_proj(hip_ops.gate_up_silu_small_m(x, w, packed=gu.weight_packed), reduce=reduce,
-                                  partial_ok=flat)
-        n_inter = w.shape[0] // 2
-        if mid_m(x, gu.weight_packed) and n_inter % 16 == 0 and hip_ops.linear_mid_m_ok(x, n_inter):
-            cfg, _ = mid_plan("gated", x.numel() // x.shape[-1], n_inter, w.shape[1])
-            if cfg:
-                act = hip_ops.gate_up_silu_mid_m(x, gu.weight_packed, n_inter, cfg)
-                return self.down_proj(act, reduce=reduce, partial_ok=flat)
-        return self.down_proj(self.act_fn(self.gate_up_proj(x)), reduce=reduce, partial_ok=flat)
+        return self.down_proj(gated_linear(x, gu), reduce=reduce, partial_ok=flat)
 
 
 class QwenDecoderLayer(nn.Module):

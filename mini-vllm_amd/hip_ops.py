@@ -73,6 +73,8 @@ _SIGNATURES = {
     "mv_residual_update": (c_int, [c_void_p, c_int, c_int, c_int, c_int, c_void_p]),
     "mv_gated_lookup": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int64, c_int, c_void_p, c_void_p, c_int64, c_int,
                                 c_int, c_int, c_int, c_void_p]),
+    "mv_gated_lookup_linear": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int64, c_int, c_void_p, c_void_p, c_void_p,
+                                       c_int64, c_int, c_int, c_int, c_int, c_int, c_void_p]),
     "mv_linear_small_m": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_int, c_int,
                                   c_int, c_int, c_int, c_void_p]),
     "mv_gate_up_silu_small_m": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_int, c_int,
@@ -529,16 +531,27 @@ def sample(logits, temperatures, top_ks, top_ps, min_ps, seed: int = 0, offset: 
 
 
 # ---------------------------------------------------------------- K9
-def silu_and_mul(x):
+GATE_ACTS = {"silu": 0, "gelu_tanh": 1 << 16}    # include/mvhip.h: MV_GATE_GELU
+
+
+def _gated_out(out, rows: int, n: int, x):
+    if out is None:
+        return torch.empty((rows, n), dtype=x.dtype, device=x.device)
+    if tuple(out.shape) != (rows, n) or out.dtype != x.dtype or out.stride(1) != 1:
+        raise MvHipError(f"act(gate) * up: out must be [{rows}, {n}] rows of {x.dtype}")
+    return out
+
+
+def silu_and_mul(x, out=None):
     _need_cuda(x)
     if x.size(-1) % 2 != 0:
         raise ValueError(f"Input last dimension must be even for SiluAndMul, got {x.size(-1)}")
     x2, cols2 = _rows2d(x)
     cols = cols2 // 2
-    out = torch.empty((x2.shape[0], cols), dtype=x.dtype, device=x.device)
+    given, out = out, _gated_out(out, x2.shape[0], cols, x)
     _check(_lib.mv_silu_and_mul(x2.data_ptr(), x2.stride(0), out.data_ptr(), out.stride(0), x2.shape[0],
                                 cols, _dt(x), _stream()), "mv_silu_and_mul")
-    return out.view(*x.shape[:-1], cols)
+    return out if given is not None else out.view(*x.shape[:-1], cols)
 
 
 def gelu_and_mul(x, out=None):
@@ -547,10 +560,7 @@ def gelu_and_mul(x, out=None):
     if x.dim() != 2 or x.stride(1) != 1 or x.shape[1] % 2:
         raise ValueError(f"gelu_and_mul wants [rows, 2 * cols] rows, got {tuple(x.shape)}")
     rows, cols = x.shape[0], x.shape[1] // 2
-    if out is None:
-        out = torch.empty((rows, cols), dtype=x.dtype, device=x.device)
-    if out.shape != (rows, cols) or out.stride(1) != 1 or out.dtype != x.dtype:
-        raise MvHipError("gelu_and_mul: output shape / layout mismatch")
+    out = _gated_out(out, rows, cols, x)
     _check(_lib.mv_gelu_and_mul(x.data_ptr(), x.stride(0), out.data_ptr(), out.stride(0), rows, cols, _dt(x), _stream()),
            "mv_gelu_and_mul")
     return out
@@ -614,6 +624,25 @@ def gated_lookup(s, table, offset: int, dim: int, ids, out=None):
     return out
 
 
+GATED_LOOKUP_LINEAR_MAX_K = 512
+
+
+def gated_lookup_linear(s, table, offset: int, dim: int, ids, w_packed, n: int):
+    """gated_lookup(s, ...) @ W^T in one launch, W [n, K] packed by ``pack_weight`` (K = columns of ``s`` <= 512)."""
+    _need_cuda(s, table, ids, w_packed)
+    rows, k = s.shape
+    if s.stride(1) != 1 or table.dtype != s.dtype or not table.is_contiguous() or ids.dtype != torch.int64 \
+            or ids.numel() != rows or not ids.is_contiguous():
+        raise MvHipError("gated_lookup_linear: rows of s, a dense table of the same dtype and int64 ids [rows] required")
+    if not _packed_ok(w_packed, n, k, s.dtype):
+        raise MvHipError(f"packed weight does not match [{n}, {k}]")
+    out = torch.empty((rows, n), dtype=s.dtype, device=s.device)
+    _check(_lib.mv_gated_lookup_linear(s.data_ptr(), s.stride(0), table.data_ptr(), table.stride(0), table.shape[0], int(offset),
+                                       ids.data_ptr(), w_packed.data_ptr(), out.data_ptr(), out.stride(0), rows, int(dim), k,
+                                       int(n), _dt(s), _stream()), "mv_gated_lookup_linear")
+    return out
+
+
 # ---------------------------------------------------------------- K10
 LINEAR_SMALL_M_MAX = 64
 
@@ -660,14 +689,16 @@ def linear_small_m(x, weight, bias=None, shape: int = 0, packed=None):
     return out.view(*x.shape[:-1], n)
 
 
-def gate_up_silu_small_m(x, weight, shape: int = 0, packed=None):
-    """x [..., K] (<= 64 rows), weight [2I, K] = [gate rows ; up rows] -> silu(x Wg^T) * (x Wu^T), [..., I]."""
+def gate_up_silu_small_m(x, weight, shape: int = 0, packed=None, act: str = "silu", out=None):
+    """x [..., K] (<= 64 rows), weight [2I, K] = [gate rows ; up rows] -> act(x Wg^T) * (x Wu^T), [..., I].  ``out`` ([rows, I],
+    rows may be strided): where it goes."""
     _need_cuda(x, weight)
     x2, k = _rows2d(x)
     if weight.shape[0] % 2 or weight.shape[1] != k or not weight.is_contiguous():
         raise ValueError(f"weight {tuple(weight.shape)} is not a merged [2I, {k}] gate_up matrix")
     n = weight.shape[0] // 2
-    out = torch.empty((x2.shape[0], n), dtype=x.dtype, device=x.device)
+    given, out = out, _gated_out(out, x2.shape[0], n, x)
+    shape = int(shape) | GATE_ACTS[act]
     if n % 16 == 0 and _packed_ok(packed, 2 * n, k, x.dtype):
         _check(_lib.mv_gate_up_silu_small_m_packed(x2.data_ptr(), x2.stride(0), packed.data_ptr(), out.data_ptr(),
                                                    out.stride(0), x2.shape[0], n, k, _dt(x), int(shape), _stream()),
@@ -676,7 +707,7 @@ def gate_up_silu_small_m(x, weight, shape: int = 0, packed=None):
         _check(_lib.mv_gate_up_silu_small_m(x2.data_ptr(), x2.stride(0), weight.data_ptr(), out.data_ptr(),
                                             out.stride(0), x2.shape[0], n, k, _dt(x), int(shape), _stream()),
                "mv_gate_up_silu_small_m")
-    return out.view(*x.shape[:-1], n)
+    return out if given is not None else out.view(*x.shape[:-1], n)
 
 
 # rows x vectors-per-norm-thread up to which the layer norm rides in the prologue of the small-M projection behind it.  The
@@ -767,17 +798,17 @@ def linear_mid_m(x, w_packed, n: int, bias=None, cfg: int = 0, out=None):
     return out.view(*x.shape[:-1], n)
 
 
-def gate_up_silu_mid_m(x, w_packed, n_inter: int, cfg: int = 0):
-    """x [..., K], w_packed = pack_weight([gate rows ; up rows] of shape [2I, K]) -> silu(x Wg^T) * (x Wu^T)."""
+def gate_up_silu_mid_m(x, w_packed, n_inter: int, cfg: int = 0, act: str = "silu", out=None):
+    """x [..., K], w_packed = pack_weight([gate rows ; up rows] of shape [2I, K]) -> act(x Wg^T) * (x Wu^T)."""
     _need_cuda(x, w_packed)
     x2, k = _rows2d(x)
     if w_packed.numel() != 2 * n_inter * k or n_inter % 16:
         raise ValueError(f"packed weight of {w_packed.numel()} elements is not a merged [2*{n_inter}, {k}] matrix")
-    out = torch.empty((x2.shape[0], n_inter), dtype=x.dtype, device=x.device)
+    given, out = out, _gated_out(out, x2.shape[0], n_inter, x)
     _check(_lib.mv_gate_up_silu_mid_m(x2.data_ptr(), x2.stride(0), w_packed.data_ptr(), out.data_ptr(),
-                                      out.stride(0), x2.shape[0], n_inter, k, _dt(x), int(cfg), _stream()),
+                                      out.stride(0), x2.shape[0], n_inter, k, _dt(x), int(cfg) | GATE_ACTS[act], _stream()),
            "mv_gate_up_silu_mid_m")
-    return out.view(*x.shape[:-1], n_inter)
+    return out if given is not None else out.view(*x.shape[:-1], n_inter)
 
 
 def linear_mid_m_partial(x, w_packed, n: int, splits: int, cfg: int = 0):

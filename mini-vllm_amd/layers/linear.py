@@ -28,7 +28,7 @@ from ..parallel_state import (divide, get_tensor_parallel_rank, get_tensor_paral
 from ..utils.loader import materialize
 
 __all__ = ["LinearBase", "ReplicatedLinear", "ColumnParallelLinear", "MergedColumnParallelLinear",
-           "QKVParallelLinear", "RowParallelLinear", "SegmentedLinear", "Segment", "pad_to", "divide", "linear", "small_m", "PartialSum", "mid_plan",
+           "QKVParallelLinear", "RowParallelLinear", "SegmentedLinear", "Segment", "gated_linear", "pad_to", "divide", "linear", "small_m", "PartialSum", "mid_plan",
            "tuned_plan", "mid_m"]
 
 # rows up to which the weight-streaming kernel beats the library GEMM (tools/bench_linear.py); 0 disables
@@ -155,6 +155,20 @@ def linear(x, weight, bias=None, packed=None, kind: str = "col"):
             if cfg:
                 return hip_ops.linear_mid_m(x, packed, n, bias, cfg)
     return F.linear(x, weight, bias)
+
+
+def gated_linear(x, lin, act: str = "silu", out=None):
+    """act(x W_gate^T) * (x W_up^T) for ``lin`` with the merged weight [gate rows ; up rows]: in the projection's epilogue for
+    decode-sized inputs, else the library GEMM and the activation kernel.  ``out``: where it goes (2-D, rows may be strided)."""
+    w = lin.weight
+    if small_m(x, w):
+        return hip_ops.gate_up_silu_small_m(x, w, packed=lin.weight_packed, act=act, out=out)
+    n_inter = w.shape[0] // 2
+    if mid_m(x, lin.weight_packed) and n_inter % 16 == 0 and hip_ops.linear_mid_m_ok(x, n_inter):
+        cfg, _ = mid_plan("gated", x.numel() // x.shape[-1], n_inter, w.shape[1])
+        if cfg:
+            return hip_ops.gate_up_silu_mid_m(x, lin.weight_packed, n_inter, cfg, act=act, out=out)
+    return (hip_ops.silu_and_mul if act == "silu" else hip_ops.gelu_and_mul)(lin(x), out=out)
 
 
 class LinearBase(nn.Module):

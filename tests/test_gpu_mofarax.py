@@ -115,6 +115,37 @@ def test_gelu_and_mul_and_gated_lookup(H, dtype):
         assert got[:, dim:].abs().sum() == 0
 
 
+@pytest.mark.parametrize("m, inter, k", [(1, 80, 256), (5, 192, 320), (16, 64, 512), (33, 208, 192), (200, 144, 256)])
+def test_gelu_in_the_epilogue_of_the_gated_projection(H, m, inter, k):
+    """Row counts of the small-M and the mid-M kernel, row-major and packed weights, into strided rows."""
+    from minivllm_amd.layers.linear import MID_CFGS
+
+    dtype = torch.bfloat16
+    x, w = _rand(m, k, dtype=dtype, seed=1), (_rand(2 * inter, k, seed=2) * 3 * k ** -0.5).to(dtype)
+    gate, up = x.double() @ w.double().T[:, :inter], x.double() @ w.double().T[:, inter:]
+    want, wp = M.gelu_tanh(gate) * up, H.pack_weight(w.to(DEV))
+    wide = torch.zeros(m, inter + 96, dtype=dtype, device=DEV)
+    out = wide[:, 64:64 + inter]
+    if k >= 256 and m <= 64:
+        for packed in (None, wp):
+            _close(H.gate_up_silu_small_m(x.to(DEV), w.to(DEV), packed=packed, act="gelu_tanh", out=out), want, dtype)
+    for cfg in [0] + [c for c, (_, _, gated) in MID_CFGS.items() if gated]:
+        wide.zero_()
+        _close(H.gate_up_silu_mid_m(x.to(DEV), wp, inter, cfg, act="gelu_tanh", out=out), want, dtype, f"tile {cfg}")
+        assert wide[:, :64].abs().sum() == 0 and wide[:, 64 + inter:].abs().sum() == 0
+
+
+@pytest.mark.parametrize("dtype", [torch.bfloat16, torch.float16])
+@pytest.mark.parametrize("rows, dim, k, off, total, n", [(1, 20, 64, 20, 60, 64), (9, 128, 128, 128, 384, 1100), (16, 40, 64, 40, 80, 192),
+                                                         (17, 200, 256, 0, 200, 52), (300, 96, 128, 96, 288, 448), (33, 500, 512, 8, 512, 320)])
+def test_lookup_and_side_projection_in_one_launch(H, dtype, rows, dim, k, off, total, n):
+    s, table, w = _rand(rows, k, dtype=dtype, seed=2), _rand(17, total, dtype=dtype, seed=3), _rand(n, k, dtype=dtype, seed=4)
+    ids = torch.arange(rows) * 3 % 17
+    got = H.gated_lookup_linear(s.to(DEV), table.to(DEV), off, dim, ids.to(DEV), H.pack_weight(w.to(DEV)), n)
+    g = (M.gelu_tanh(s.double()[:, :dim]) * table.double()[ids][:, off:off + dim]).to(dtype).double()
+    _close(got, g @ w.double()[:, :dim].T, dtype)
+
+
 def _paged(kv, lens, nk, D, bs, dtype, seed):
     """Scatter per-sequence rows into shuffled blocks; the other slots hold huge values (a wrong slot shows)."""
     nb = sum(-(-n // bs) for n in lens) + 2

@@ -124,11 +124,13 @@ def test_weights_land_in_the_merged_matrices_with_zero_padding(tmp_path):
     w = M.random_model(cfg, 3)
     m = _built(tmp_path, cfg, w)
     f = {k: v.float() for k, v in w.items()}
-    lin, at = m.l0.proj_in, m.l0.proj_in.offsets                      # q: 6 heads of 48 stored at 64; width 200 at 256
-    assert lin.weight.shape == (6 * 64 + 2 * 64 + 128 + 128, 256) and at == {"q": 0, "k": 384, "gate": 512, "up": 640}
+    lin, ffn = m.l0.qk, m.l0.gate_up                                   # q: 6 heads of 48 stored at 64; width 200 at 256
+    assert lin.weight.shape == (6 * 64 + 2 * 64, 256) and lin.offsets == {"q": 0, "k": 384}
+    assert ffn.weight.shape == (128 + 128, 256) and ffn.offsets == {"gate": 0, "up": 128}
     q = lin.weight[:384].view(6, 64, 256)
     assert torch.equal(q[:, :48, :200], f["l0.mix.q"].view(6, 48, 200)) and q[:, 48:].abs().sum() == 0
-    assert torch.equal(lin.weight[512:632, :200], f["l0.mlp.gate"]) and lin.weight[632:640].abs().sum() == 0
+    assert torch.equal(ffn.weight[:120, :200], f["l0.mlp.gate"]) and ffn.weight[120:128].abs().sum() == 0
+    assert torch.equal(ffn.weight[128:248, :200], f["l0.mlp.up"])
     assert lin.weight[:, 200:].abs().sum() == 0
     o = m.l0.proj_out.weight[:200, :384].view(200, 6, 64)
     assert torch.equal(o[:, :, :48], f["l0.mix.o"].view(200, 6, 48)) and o[:, :, 48:].abs().sum() == 0
@@ -168,10 +170,10 @@ def test_tensor_parallel_shards_sum_to_the_whole(tmp_path):
             ps.reset_tensor_parallel()
         lay = m.l0
         assert (lay.heads, lay.kv_heads) == (2, 1) and m.head.weight.shape[0] == 20
-        z = h_pad @ lay.proj_in.weight.T
+        z, y = h_pad @ lay.qk.weight.T, h_pad @ lay.gate_up.weight.T
         qs.append(z[:, :128].view(7, 2, 64)[:, :, :32])
-        at = lay.proj_in.offsets
-        act = M.gelu_tanh(z[:, at["gate"]:at["up"]]) * z[:, at["up"]:]
+        up = lay.gate_up.offsets["up"]
+        act = M.gelu_tanh(y[:, :up]) * y[:, up:]
         mixed = torch.cat([z[:, :128], act], 1)                        # (the queries stand in for the attention output)
         total += (mixed @ lay.proj_out.weight.T)[:, :96]
     q = h @ f["l0.mix.q"].T
