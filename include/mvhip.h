@@ -320,9 +320,9 @@ int mv_residual_update(const MvResidualArgs *args, int rows, int cols, int cols_
 int mv_gated_lookup(const void *s, int64_t s_stride, const void *table, int64_t table_stride, int64_t vocab,
                     int offset, const int64_t *ids, void *out, int64_t out_stride, int rows, int dim, int cols,
                     int dtype, void *stream);
-/* ... and the projection behind it in one launch, for decode-sized batches: out[t][i] = sum_j r(g[t][j]) * W[i][j] with g
+/* ... and the projection behind it in one launch: out[t][i] = sum_j r(g[t][j]) * W[i][j] with g
  * as above, r() its rounding to dtype, W [n, k] packed by mv_pack_weight (k >= dim: zero columns behind), k % 32 == 0,
- * k <= 512, n % 4 == 0, 16-bit dtypes; MV_E_SHAPE otherwise. */
+ * k <= 512, n % 4 == 0, 16-bit dtypes; MV_E_SHAPE otherwise.  out and its rows 16-byte aligned. */
 int mv_gated_lookup_linear(const void *s, int64_t s_stride, const void *table, int64_t table_stride, int64_t vocab,
                            int offset, const int64_t *ids, const void *w_packed, void *out, int64_t out_stride, int rows,
                            int dim, int k, int n, int dtype, void *stream);
@@ -353,7 +353,10 @@ int mv_gate_up_silu_small_m(const void *x, int64_t x_stride, const void *w_gate_
 
 /* K10 on the fragment-ordered weight copy of mv_pack_weight (below): the same two operations, the same summation
  * order and rounding points (results bit-identical to the row-major entry points); only the weight address stream
- * differs — 1 KiB contiguous per wave-wide load instead of 16 pieces of 64 B.  The gated form needs n_inter % 16 == 0. */
+ * differs — 1 KiB contiguous per wave-wide load instead of 16 pieces of 64 B.  The gated form needs n_inter % 16 == 0.
+ * MV_LINEAR_ROW_GROUPS in `shape` (plain form): any m, the rows in groups of 16 with workgroups of their own (each re-reads
+ * the weight: for narrow matrices, whose few tiles would leave most of the chip idle otherwise). */
+enum { MV_LINEAR_ROW_GROUPS = 1 << 17 };
 int mv_linear_small_m_packed(const void *x, int64_t x_stride, const void *w_packed,
                              const void *bias, void *out, int64_t out_stride, int m,
                              int n, int k, int dtype, int shape, void *stream);

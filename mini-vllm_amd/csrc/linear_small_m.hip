@@ -153,6 +153,12 @@ __global__ void __launch_bounds__((GATED ? 2 : 1) * RPW * MT >= 12 ? 512 : 1024)
 linear_small_m_kernel(LinearParams p) {
   static_assert(!NORM || (PACKED && MT == 1 && !XLDS), "the norm prologue exists for the packed, <= 16-row form");  // (>= 12 tiles per wave: the 64 KB of partial-tile LDS allow <= 5 waves)
   typedef uint16_t T;
+  if constexpr (PACKED && !GATED && !NORM) {   // row groups (narrow projections of wider batches): 16 * MT rows per blockIdx.y
+    const int mb = blockIdx.y * (16 * MT);
+    p.x = (const T *)p.x + (int64_t)mb * p.x_stride;
+    p.out = (T *)p.out + (int64_t)mb * p.out_stride;
+    p.M = min(p.M - mb, 16 * MT);
+  }
   extern __shared__ float red[];  // [waves][RPW*MT][64][4]; XLDS: first the per-wave x blocks
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nwaves = blockDim.x >> 6;
   const int r16 = lane & 15, g = lane >> 4;
@@ -399,7 +405,8 @@ static void norm_block(int cols, int *threads, int *per_thread) {
 
 template <bool GATED, bool PACKED = false, bool NORM = false>
 int run(LinearParams p, int dtype, int shape, hipStream_t st) {
-  const int m = p.M, n = p.N, mt = (m + 15) / 16, steps = p.K / 32;
+  const bool groups = PACKED && !GATED && !NORM && (shape & MV_LINEAR_ROW_GROUPS) && p.M > 16;
+  const int m = groups ? 16 : p.M, n = p.N, mt = (m + 15) / 16, steps = p.K / 32;
   int rpw = GATED ? (m > 2 && n >= 16384 ? 2 : 1) : (m <= 2 ? 1 : (n >= 65536 ? 4 : (n >= 8192 ? 2 : 1)));
   // (on the packed copy 4 row tiles per wave never measured fastest, nor 2 + 2 tiles for the gated form:
   //  Qwen2-7B gate_up at 16 rows 44 us with 1 + 1 tiles over 7 waves, 64 us with 2 + 2)
@@ -465,7 +472,7 @@ int run(LinearParams p, int dtype, int shape, hipStream_t st) {
   while (xlds && waves > 1 && waves * xblock > 65536) waves /= 2;
   size_t lds = (size_t)waves * na * mt * 64 * sizeof(f32x4);
   if (xlds && waves * xblock > lds) lds = waves * xblock;
-  dim3 grid(tiles), block(waves * 64);
+  dim3 grid(tiles, groups ? (p.M + 15) / 16 : 1), block(waves * 64);
   // one or two weight tiles per wave and more than one block per K slice (K >= 3584, or 6144 over 8 waves): the
   // weight block also comes in by whole-row DMA (+13..25 % on the down / Qwen2-7B qkv projections at M <= 8,
   // -5 % on single-block slices and on the LM head, tools/dbg/wlds_bench.sh); MV_LINEAR_WLDS=1/-1 forces
@@ -504,10 +511,10 @@ int run(LinearParams p, int dtype, int shape, hipStream_t st) {
 }
 
 int check(const void *x, int64_t x_stride, const void *w, const void *bias, void *out, int64_t out_stride, int m,
-          int n, int k, int dtype) {
+          int n, int k, int dtype, int m_max = 64) {
   if (!x || !w || !out) return MV_E_NULLPTR;
   if (dtype != MV_BF16 && dtype != MV_F16) return dtype == MV_F32 ? MV_E_SHAPE : MV_E_DTYPE;
-  if (m < 0 || m > 64 || n < 0 || k < 256 || (k & 31) || (n & 3)) return MV_E_SHAPE;
+  if (m < 0 || m > m_max || n < 0 || k < 256 || (k & 31) || (n & 3)) return MV_E_SHAPE;
   if (!mv_aligned16(x) || !mv_aligned16(w) || (((uintptr_t)out) & 7u) || (x_stride & 7) || (out_stride & 3) ||
       (bias && (((uintptr_t)bias) & 7u)))
     return MV_E_ALIGN;
@@ -540,7 +547,8 @@ extern "C" int mv_linear_small_m_packed(const void *x, int64_t x_stride, const v
                                         void *out, int64_t out_stride, int m, int n, int k, int dtype, int shape,
                                         void *stream) {
   if (m == 0 || n == 0) return MV_OK;
-  if (int e = check(x, x_stride, w_packed, bias, out, out_stride, m, n, k, dtype)) return e;
+  if (int e = check(x, x_stride, w_packed, bias, out, out_stride, m, n, k, dtype, (shape & MV_LINEAR_ROW_GROUPS) ? 16 * 65535 : 64))
+    return e;
   LinearParams p{x, w_packed, bias, out, x_stride, out_stride, m, n, k};
   return run<false, true>(p, dtype, shape, (hipStream_t)stream);
 }

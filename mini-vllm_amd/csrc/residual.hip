@@ -3,7 +3,7 @@
 //     projections in front (plain, or RMS-normed by a weight of its own; or the fp32 partial sums of a K split)
 //     [+ the scaled embedding] [+ a vector] -> the stream, and what the next projection reads: its RMSNorm or its cast;
 //   mv_gated_lookup: gelu(s) * a slice of a per-token table (the per-token layer input);
-//   mv_gated_lookup_linear: the same with the projection behind it, one launch for decode-sized batches.
+//   mv_gated_lookup_linear: the same with the projection behind it, in one launch (decode-sized batches).
 // One workgroup per row, the row in registers between the reductions and the store: the stream is read and written once.
 #include "common.h"
 
@@ -196,10 +196,12 @@ __device__ __forceinline__ f32x4 side_mfma(u32x4 a, u32x4 b, f32x4 c) {
     return __builtin_amdgcn_mfma_f32_16x16x32_f16(__builtin_bit_cast(f16x8, a), __builtin_bit_cast(f16x8, b), c, 0, 0, 0);
 }
 
-// out[t][n] = sum_j g[t][j] W[n][j], g = gated_lookup_kernel's row rounded to the dtype.  One workgroup: 16 tokens x 64
-// outputs, one 16-wide tile of W per wave.  W comes fragment-ordered (mv_pack_weight: the A operand, 1 KiB per wave-wide
-// load) and its first kAhead k-steps are in flight while the workgroup computes its 16 rows of g into LDS, which holds them
-// in the B operand's order: [k-step][lane][8], lane l = token l & 15, k group l >> 4.
+// out[t][n] = sum_j g[t][j] W[n][j], g = gated_lookup_kernel's row rounded to the dtype.  One workgroup: 16 tokens, whose rows
+// of g it computes once, into LDS, in the MFMA B operand's order ([k-step][lane][8], lane l = token l & 15, k group l >> 4);
+// then each wave walks blocks of 32 outputs.  W comes fragment-ordered (mv_pack_weight: [tile of 16][k-step][lane][8], lane =
+// row + 16 * k group).  The two A fragments of a block take its rows as 8 (r >> 2) + (r & 3) and that + 4, so that a lane ends
+// up with 8 consecutive outputs of its token: one 16-byte store.  The first kSideAhead k-steps of a wave's first block are in
+// flight while the rows of g are computed.
 constexpr int kSideAhead = 4, kSideMaxK = 512;
 template <typename Tag>
 __global__ void __launch_bounds__(256) gated_lookup_linear_kernel(const uint16_t *s, int64_t s_stride, const uint16_t *table,
@@ -207,21 +209,36 @@ __global__ void __launch_bounds__(256) gated_lookup_linear_kernel(const uint16_t
                                                                   const int64_t *ids, const uint16_t *wp, uint16_t *out,
                                                                   int64_t out_stride, int rows, int dim, int K, int N,
                                                                   bool table_vec) {
-  __shared__ u32x4 g[kSideMaxK / 32 * 64];
+  extern __shared__ u32x4 g[];   // [K / 32][64]
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, steps = K / 32;
-  const int m0 = blockIdx.y * 16, tile = blockIdx.x * 4 + wave, tiles = (N + 15) / 16;
-  const u32x4 *w = (const u32x4 *)wp + (int64_t)(tile < tiles ? tile : tiles - 1) * steps * 64 + lane;
-  u32x4 wf[kSideAhead];
+  const int64_t m0 = (int64_t)blockIdx.y * 16;
+  const int r16 = lane & 15, kg = lane >> 4, n_pad = (N + 15) / 16 * 16, blocks = (N + 31) / 32, stride = gridDim.x * 4;
+  const u32x4 *w = (const u32x4 *)wp;
+  auto w_row = [&](int blk, int half) {   // this lane's row of W in half `half` of a block (clamped into the packed copy)
+    int n = blk * 32 + (r16 >> 2) * 8 + (r16 & 3) + half * 4;
+    n = n < n_pad ? n : n_pad - 1;
+    return w + (int64_t)(n >> 4) * steps * 64 + kg * 16 + (n & 15);
+  };
+  u32x4 wf[kSideAhead][2];
+  auto preload = [&](int blk) {
+    const u32x4 *a = w_row(blk, 0), *b = w_row(blk, 1);
 #pragma unroll
-  for (int i = 0; i < kSideAhead; ++i) wf[i] = w[(i < steps ? i : steps - 1) * 64];
+    for (int i = 0; i < kSideAhead; ++i) {
+      const int k = i < steps ? i : steps - 1;
+      wf[i][0] = a[k * 64], wf[i][1] = b[k * 64];
+    }
+  };
+  int blk = blockIdx.x * 4 + wave;
+  preload(blk < blocks ? blk : blocks - 1);
   for (int v = threadIdx.x; v < steps * 64; v += 256) {
-    const int l = v & 63, m = m0 + (l & 15), c = (v >> 6) * 32 + (l >> 4) * 8;
+    const int l = v & 63, c = (v >> 6) * 32 + (l >> 4) * 8;
+    const int64_t m = m0 + (l & 15);
     float a[8], e[8], o[8];
 #pragma unroll
     for (int j = 0; j < 8; ++j) o[j] = 0.f;
     const int64_t id = m < rows ? ids[m] : -1;
     if (id >= 0 && id < vocab && c < dim) {
-      load_row_vec<Tag>(s + (int64_t)m * s_stride + c, a);
+      load_row_vec<Tag>(s + m * s_stride + c, a);
       const uint16_t *tr = table + id * table_stride + offset + c;
       if (table_vec && c + 8 <= dim) {
         load_row_vec<Tag>(tr, e);
@@ -235,18 +252,34 @@ __global__ void __launch_bounds__(256) gated_lookup_linear_kernel(const uint16_t
     g[v] = pack8<Tag>(o);
   }
   __syncthreads();
-  f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+  for (; blk < blocks; blk += stride) {
+    f32x4 acc[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
 #pragma unroll
-  for (int i = 0; i < kSideAhead; ++i)
-    if (i < steps) acc = side_mfma<Tag>(wf[i], g[i * 64 + lane], acc);
-  for (int i = kSideAhead; i < steps; ++i) acc = side_mfma<Tag>(w[i * 64], g[i * 64 + lane], acc);
-  // C layout: lane holds W rows n = (lane >> 4) * 4 + {0..3} (consecutive outputs) of token lane & 15
-  const int m = m0 + (lane & 15), n = tile * 16 + (lane >> 4) * 4;
-  if (m < rows && n < N) {
-    u32x2 pk;
-    pk[0] = (uint32_t)elem<Tag>::st(acc[0]) | ((uint32_t)elem<Tag>::st(acc[1]) << 16);
-    pk[1] = (uint32_t)elem<Tag>::st(acc[2]) | ((uint32_t)elem<Tag>::st(acc[3]) << 16);
-    *(u32x2 *)(out + (int64_t)m * out_stride + n) = pk;
+    for (int i = 0; i < kSideAhead; ++i)
+      if (i < steps) {
+        const u32x4 x = g[i * 64 + lane];
+        acc[0] = side_mfma<Tag>(wf[i][0], x, acc[0]);
+        acc[1] = side_mfma<Tag>(wf[i][1], x, acc[1]);
+      }
+    if (steps > kSideAhead) {
+      const u32x4 *a = w_row(blk, 0), *b = w_row(blk, 1);
+#pragma unroll 4
+      for (int i = kSideAhead; i < steps; ++i) {
+        const u32x4 x = g[i * 64 + lane];
+        acc[0] = side_mfma<Tag>(a[i * 64], x, acc[0]);
+        acc[1] = side_mfma<Tag>(b[i * 64], x, acc[1]);
+      }
+    }
+    if (blk + stride < blocks) preload(blk + stride);
+    const int64_t m = m0 + r16;
+    const int n = blk * 32 + kg * 8;
+    if (m < rows && n < N) {
+      const float o[8] = {acc[0][0], acc[0][1], acc[0][2], acc[0][3], acc[1][0], acc[1][1], acc[1][2], acc[1][3]};
+      const u32x4 pk = pack8<Tag>(o);
+      uint16_t *dst = out + m * out_stride + n;
+      if (n + 8 <= N) *(u32x4 *)dst = pk;
+      else *(u32x2 *)dst = u32x2{pk[0], pk[1]};   // N % 4 == 0: four outputs are left
+    }
   }
 }
 
@@ -318,14 +351,17 @@ extern "C" int mv_gated_lookup_linear(const void *s, int64_t s_stride, const voi
   if (dtype != MV_BF16 && dtype != MV_F16) return dtype == MV_F32 ? MV_E_SHAPE : MV_E_DTYPE;
   if (rows < 0 || dim <= 0 || k < dim || vocab <= 0 || offset < 0 || offset + dim > table_stride || n < 0 || (n & 3))
     return MV_E_SHAPE;
-  if ((k & 31) || k > kSideMaxK || rows > 16 * 65535) return MV_E_SHAPE;
-  if (!mv_aligned16(s) || !mv_aligned16(w_packed) || (((uintptr_t)out) & 7u) || (s_stride & 7) || (out_stride & 3)) return MV_E_ALIGN;
+  if ((k & 31) || k > kSideMaxK) return MV_E_SHAPE;
+  if (!mv_aligned16(s) || !mv_aligned16(w_packed) || !mv_aligned16(out) || (s_stride & 7) || (out_stride & 7)) return MV_E_ALIGN;
   const bool table_vec = mv_aligned16(table) && table_stride % 8 == 0 && offset % 8 == 0;
-  const dim3 grid((unsigned)((n + 63) / 64), (unsigned)((rows + 15) / 16));
+  const int row_blocks = (rows + 15) / 16, split_max = (n + 127) / 128;
+  if (row_blocks > 65535) return MV_E_SHAPE;
+  const int split = (2048 + row_blocks - 1) / row_blocks;
+  const dim3 grid((unsigned)(split < split_max ? split : split_max), (unsigned)row_blocks);
 #define MV_SIDE(TAG)                                                                                                          \
-  hipLaunchKernelGGL((gated_lookup_linear_kernel<TAG>), grid, dim3(256), 0, (hipStream_t)stream, (const uint16_t *)s, s_stride, \
-                     (const uint16_t *)table, table_stride, vocab, offset, ids, (const uint16_t *)w_packed, (uint16_t *)out,   \
-                     out_stride, rows, dim, k, n, table_vec)
+  hipLaunchKernelGGL((gated_lookup_linear_kernel<TAG>), grid, dim3(256), (size_t)k * 32, (hipStream_t)stream,                   \
+                     (const uint16_t *)s, s_stride, (const uint16_t *)table, table_stride, vocab, offset, ids,                  \
+                     (const uint16_t *)w_packed, (uint16_t *)out, out_stride, rows, dim, k, n, table_vec)
   if (dtype == MV_BF16) MV_SIDE(bf16_tag);
   else MV_SIDE(f16_tag);
 #undef MV_SIDE

@@ -6,7 +6,7 @@ Attention and feed-forward of a layer read ONE norm and are summed, and the resi
     [gate | up] GEMM with gelu(gate) * up                              into its right columns (decode: ONE launch)
     -> [o | down] GEMM over `mixed`                                    both sublayers summed in the accumulators
     -> residual += that; cast                                          (mv_residual_update)
-    -> side gate GEMM -> gelu * token table -> side projection GEMM    (decode: the last two in ONE launch)
+    -> side gate GEMM -> gelu * token table -> side projection         (decode: the last two in ONE launch)
     -> residual += rms(.) * w [+ embedding + pass vector]; next layer's norm    (mv_residual_update)
 Layers of the loop run several times over the same weights; each pass has attention modules (K/V planes) of its own.
 Values are the projected keys before rotation: the K plane of the cache holds rotated keys, the V plane the raw ones.
@@ -65,6 +65,7 @@ class SideInput(nn.Module):
 
     def forward(self, x, ids, table):
         packed, n = self.proj.weight_packed, self.proj.weight.shape[0]
+        # (prefill: the library product and a launch of its own for the lookup were as fast or faster)
         if packed is not None and x.shape[0] <= MID_M_MAX and self.proj.weight.shape[1] <= hip_ops.GATED_LOOKUP_LINEAR_MAX_K:
             return hip_ops.gated_lookup_linear(self.gate(x), table, self.offset, self.dim, ids, packed, n)
         return self.proj(hip_ops.gated_lookup(self.gate(x), table, self.offset, self.dim, ids))

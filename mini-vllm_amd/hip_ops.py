@@ -636,7 +636,7 @@ def gated_lookup_linear(s, table, offset: int, dim: int, ids, w_packed, n: int):
         raise MvHipError("gated_lookup_linear: rows of s, a dense table of the same dtype and int64 ids [rows] required")
     if not _packed_ok(w_packed, n, k, s.dtype):
         raise MvHipError(f"packed weight does not match [{n}, {k}]")
-    out = torch.empty((rows, n), dtype=s.dtype, device=s.device)
+    out = torch.empty((rows, -(-n // 8) * 8), dtype=s.dtype, device=s.device)[:, :n]
     _check(_lib.mv_gated_lookup_linear(s.data_ptr(), s.stride(0), table.data_ptr(), table.stride(0), table.shape[0], int(offset),
                                        ids.data_ptr(), w_packed.data_ptr(), out.data_ptr(), out.stride(0), rows, int(dim), k,
                                        int(n), _dt(s), _stream()), "mv_gated_lookup_linear")
@@ -665,6 +665,19 @@ def small_m_shape(rpw: int = 0, waves: int = 0, xlds: int = 0, wlds: int = 0) ->
 def _packed_ok(packed, n_rows: int, k: int, dtype) -> bool:
     return (packed is not None and packed.dtype == dtype and packed.is_contiguous()
             and packed.numel() == -(-n_rows // 16) * 16 * k)
+
+
+def linear_narrow(x, packed, n: int, bias=None):
+    """x [..., K] (any number of rows), packed = pack_weight(W [n, K]), n small -> [..., n]: rows in groups of 16."""
+    _need_cuda(x, packed)
+    x2, k = _rows2d(x)
+    if not _packed_ok(packed, n, k, x.dtype) or (bias is not None and (bias.dtype != x.dtype or bias.shape[0] != n)):
+        raise ValueError(f"packed weight / bias do not match [{n}, {k}] of {x.dtype}")
+    out = torch.empty((x2.shape[0], n), dtype=x.dtype, device=x.device)
+    _check(_lib.mv_linear_small_m_packed(x2.data_ptr(), x2.stride(0), packed.data_ptr(), _ptr(bias), out.data_ptr(),
+                                         out.stride(0), x2.shape[0], n, k, _dt(x), 1 << 17, _stream()),   # MV_LINEAR_ROW_GROUPS
+           "mv_linear_small_m_packed")
+    return out.view(*x.shape[:-1], n)
 
 
 def linear_small_m(x, weight, bias=None, shape: int = 0, packed=None):

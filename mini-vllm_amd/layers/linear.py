@@ -53,6 +53,9 @@ def small_m(x, weight) -> bool:
 
 # ---- decode batches of SMALL_M_MAX+1 .. MID_M_MAX rows: csrc/linear_mid_m.hip --------------------------------
 MID_M_MAX = int(os.environ.get("MV_LINEAR_MID_M_MAX", "512"))   # 0 disables (everything above small-M on the library)
+# output features up to which a projection of such a batch is split over groups of 16 rows and over K inside a workgroup
+# (mv_linear_small_m_packed with row groups) instead of over output tiles, of which it has too few for 256 CUs; 0 disables
+NARROW_N_MAX = int(os.environ.get("MV_LINEAR_NARROW_N_MAX", "256"))
 # workgroup tiles of mv_linear_mid_m (ids of the table in csrc/linear_mid_m.hip): id -> (BM, BN, takes the gated form)
 MID_CFGS = {1: (128, 96, True), 2: (256, 48, False), 3: (128, 32, True), 4: (64, 32, False), 5: (256, 64, True),
             6: (128, 128, True), 7: (256, 160, True), 8: (256, 128, True), 9: (128, 48, False), 10: (64, 64, True),
@@ -147,6 +150,8 @@ def linear(x, weight, bias=None, packed=None, kind: str = "col"):
         return hip_ops.linear_small_m(x, weight, bias, packed=packed)
     if mid_m(x, packed):
         n, k = weight.shape
+        if n <= NARROW_N_MAX and k >= 256 and hip_ops.linear_mid_m_ok(x, n):
+            return hip_ops.linear_narrow(x, packed, n, bias)
         if hip_ops.linear_mid_m_ok(x, n):
             rows = x.numel() // k
             cfg, splits = mid_plan(kind if bias is None else "col", rows, n, k)

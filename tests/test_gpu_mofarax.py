@@ -136,8 +136,22 @@ def test_gelu_in_the_epilogue_of_the_gated_projection(H, m, inter, k):
 
 
 @pytest.mark.parametrize("dtype", [torch.bfloat16, torch.float16])
+@pytest.mark.parametrize("m, n, k", [(17, 64, 256), (64, 52, 2048), (255, 128, 2048), (256, 192, 640), (500, 256, 3584)])
+def test_narrow_projection_in_row_groups(H, dtype, m, n, k):
+    x, w = _rand(m, k, dtype=dtype, seed=1), (_rand(n, k, seed=2) * k ** -0.5).to(dtype)
+    wide = x.new_zeros(m, k + 64)
+    wide[:, :k] = x
+    b = _rand(n, dtype=dtype, seed=3)
+    for bias in (None, b):
+        got = H.linear_narrow(wide.to(DEV)[:, :k], H.pack_weight(w.to(DEV)), n, None if bias is None else bias.to(DEV))
+        want = x.double() @ w.double().T + (0 if bias is None else bias.double())
+        _close(got, want, dtype)
+
+
+@pytest.mark.parametrize("dtype", [torch.bfloat16, torch.float16])
 @pytest.mark.parametrize("rows, dim, k, off, total, n", [(1, 20, 64, 20, 60, 64), (9, 128, 128, 128, 384, 1100), (16, 40, 64, 40, 80, 192),
-                                                         (17, 200, 256, 0, 200, 52), (300, 96, 128, 96, 288, 448), (33, 500, 512, 8, 512, 320)])
+                                                         (17, 200, 256, 0, 200, 52), (300, 96, 128, 96, 288, 448), (33, 500, 512, 8, 512, 320),
+                                                         (2500, 72, 128, 72, 144, 1100), (4099, 190, 192, 0, 190, 64), (2049, 500, 512, 0, 500, 320)])
 def test_lookup_and_side_projection_in_one_launch(H, dtype, rows, dim, k, off, total, n):
     s, table, w = _rand(rows, k, dtype=dtype, seed=2), _rand(17, total, dtype=dtype, seed=3), _rand(n, k, dtype=dtype, seed=4)
     ids = torch.arange(rows) * 3 % 17
