@@ -923,6 +923,36 @@ def init_process_group(args):
     return dist
 
 
+def attention_graph_roofline(engine, model) -> dict:
+    """The decode attention launches of one step (every layer run, on the running batch's tables, lengths and K/V planes, query
+    rows random) captured into a graph and replayed.  A design's small batches are launch-bound when run eagerly: event pairs
+    around its launches would time the host."""
+    from minivllm_amd import hip_ops
+    from minivllm_amd.utils.context import get_context, reset_context
+
+    ex = engine.model_runner.inference_executor
+    seqs = list(engine.scheduler.running)
+    ex._drop_speculation()
+    torch.cuda.synchronize()
+    ex._ship_decode(ex.builder.decode(seqs))
+    ctx = get_context()
+    tables, lens = ctx.block_tables, ctx.context_lens
+    reset_context()
+    mods = [m for m in ex.model.modules() if hasattr(m, "k_cache") and hasattr(m, "v_cache")]
+    m0 = mods[0]
+    q = torch.randn((len(seqs), m0.num_heads, m0.head_dim), device=ex.device).to(ex.dtype)
+
+    def run():
+        for m in mods:
+            hip_ops.paged_decode(q, m.k_cache, m.v_cache, tables, lens, m.scale, chunk=m.chunk)
+    us = _graph_time_us(run, len(mods))
+    seen = [n - (n - 1) // m0.chunk * m0.chunk if m0.chunk else n for n in lens.tolist()]
+    algo = (sum(seen) * 2 * m0.num_kv_heads * m0.head_dim + 2 * q.numel()) * ex.dtype.itemsize
+    return {"bound": "hbm", "achieved": round(algo / us / 1e3, 1), "peak": HBM_PEAK_GBS, "unit": "GB/s",
+            "frac": round(algo / us / 1e3 / HBM_PEAK_GBS, 4), "bytes_per_launch": algo, "us_per_launch": round(us, 2),
+            "timing": f"{len(mods)} launches (split-KV combine included) captured into a hipGraph, median of 5 replays / launches"}
+
+
 def design_records(args, workdir) -> dict:
     """``--design``: for every size of the design and for its peer, decode at several batches and prefill, on one engine each."""
     import gc
@@ -939,7 +969,9 @@ def design_records(args, workdir) -> dict:
             recs = []
             for i, (batch, ctx) in enumerate(DESIGN_DECODE):
                 a.batch, a.ctx = batch, ctx
-                rec, _ = decode_record(engine, a, model, None, seed=i, probes=True)
+                rec, _ = decode_record(engine, a, model, None, seed=i, probes=False)
+                rec["roofline"] = attention_graph_roofline(engine, model)
+                rec["step_roofline"] = step_roofline(engine, model, batch, ctx + a.warmup + a.steps // 2, rec["ms_per_step"])
                 recs.append(rec)
                 release_all(engine)
             for n, ln in DESIGN_PREFILL:

@@ -159,12 +159,19 @@ __device__ __forceinline__ void rot_factors(const float *cos, const float *sin, 
                                             int pairs, bool interleaved, float (&cs)[VEC], float (&sn)[VEC]) {
   constexpr int HALF = D / VEC / 2;
   if (interleaved) {
+    // (clamped addresses and a select behind the loads: no branch around each of them)
+    const int64_t base = pos_ok ? pos * pairs : 0;
 #pragma unroll
-    for (int j = 0; j < VEC; ++j) {
+    for (int j = 0; j < VEC; j += 2) {
       const int i = (sub * VEC + j) >> 1;
+      float c = 1.0f, s = 0.0f;
+      if (pairs > 0) {   // (uniform)
+        const int ic = i < pairs ? i : pairs - 1;
+        c = cos[base + ic], s = sin[base + ic];
+      }
       const bool ok = pos_ok && i < pairs;
-      cs[j] = ok ? cos[pos * pairs + i] : 1.0f;
-      sn[j] = ok ? sin[pos * pairs + i] : 0.0f;
+      cs[j] = cs[j + 1] = ok ? c : 1.0f;
+      sn[j] = sn[j + 1] = ok ? s : 0.0f;
     }
   } else {
     const int i0 = (sub % HALF) * VEC;

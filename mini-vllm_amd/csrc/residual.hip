@@ -263,7 +263,6 @@ __global__ void __launch_bounds__(256) gated_lookup_linear_kernel(const uint16_t
       }
     if (steps > kSideAhead) {
       const u32x4 *a = w_row(blk, 0), *b = w_row(blk, 1);
-#pragma unroll 4
       for (int i = kSideAhead; i < steps; ++i) {
         const u32x4 x = g[i * 64 + lane];
         acc[0] = side_mfma<Tag>(a[i * 64], x, acc[0]);

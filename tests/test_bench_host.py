@@ -131,3 +131,22 @@ def test_run_records_executes_the_n8_plan_in_order(monkeypatch, tmp_path):
     # the headline engine is gone before the rejected construction, the last engine at the end
     order = [e[:2] for e in events if e[0] in ("build", "exit")]
     assert order == [("build", "qwen3-1.7b"), ("exit", "qwen3-1.7b"), ("build", "qwen2-7b"), ("build", "qwen2-72b"), ("exit", "qwen2-72b")]
+
+
+def test_design_configurations_have_the_layer_sizes_of_their_peers():
+    """`bench.py --design`: every layer run of a design's configuration is the size of the peer's layers, their number too,
+    and the framework reads the configuration."""
+    from minivllm_amd.native_configs import NATIVE_CONFIGS
+
+    for design, pairs in bench.DESIGNS.items():
+        for name, like in pairs.items():
+            c, p = NATIVE_CONFIGS[bench.MODELS[name]["architecture"]](bench.MODELS[name]), bench.MODELS[like]
+            assert c.num_hidden_layers == p["num_hidden_layers"] and c.vocab_size == p["vocab_size"]
+            for run, _, _ in c.layer_runs():
+                a = c.layers[run].attention
+                assert (a.heads, a.kv_heads) == (p["num_attention_heads"], p["num_key_value_heads"])
+                assert a.dim == (p.get("head_dim") or p["hidden_size"] // p["num_attention_heads"]) and c.layers[run].ff == p["intermediate_size"]
+    args = bench.parse(["--design", "mofarax"])
+    assert args.design == "mofarax" and bench.parse([]).design is None and bench.parse([]).model == "qwen3-1.7b"
+    # a chunk mask cuts the work of a prompt into the chunks' triangles
+    assert bench.prefill_flops(2, 64, [100], 30) == bench.prefill_flops(2, 64, [30, 30, 30, 10])

@@ -30,6 +30,9 @@ SHAPES = {
                    ("row", 2048, 6144, False)],
     "qwen2-7b": [("col", 4608, 3584, True), ("row", 3584, 3584, False), ("gated", 18944, 3584, False),
                  ("row", 3584, 18944, False)],
+    # q | k and attention output | down of Mofarax layers with the sizes of the three models above (bench.py --design)
+    "mofarax": [("col", 3072, 1024, False), ("row", 1024, 5120, False), ("col", 3072, 2048, False), ("row", 2048, 8192, False),
+                ("col", 4096, 3584, False), ("row", 3584, 22528, False)],
     "lm-heads": [("col", 151936, 1024, False), ("col", 151936, 2048, False), ("col", 152064, 3584, False),
                  ("col", 19008, 8192, False)],
     # the per-rank shards of Qwen3-1.7B under TP = 2 / 4 / 8 (bench.py --gpus N)
