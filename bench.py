@@ -5,7 +5,7 @@
     (N>1: one rank per GPU.  Started WITHOUT torch.distributed.run, the script starts it itself as a child
     process — before anything has touched the GPU — relays the child's output and exits with its code.)
 
-Workload (BASELINE.json configs[2], SURVEY §8d config 3): Qwen3-1.7B, bf16, kvcache_block_size=64,
+Workload (BASELINE.json configs[2]): Qwen3-1.7B, bf16, kvcache_block_size=64,
 hipGraph decode, max_num_seqs=256 — B=256 sequences at context 1024, synthetic token ids,
 random-initialised weights at the true architecture dimensions (no checkpoints offline; throughput is
 value-independent).  One "step" = one engine decode step over the whole batch: scheduler ->
@@ -54,7 +54,7 @@ sys.path.insert(0, ROOT)
 import torch  # noqa: E402
 
 MODELS = {
-    # public HF config.json values (SURVEY §8 table)
+    # public HF config.json values
     "qwen3-1.7b": dict(model_type="qwen3", architectures=["Qwen3ForCausalLM"], hidden_size=2048,
                        num_hidden_layers=28, num_attention_heads=16, num_key_value_heads=8, head_dim=128,
                        intermediate_size=6144, vocab_size=151936, max_position_embeddings=40960,
@@ -101,7 +101,7 @@ DESIGN_PREFILL = ((16, 1024), (4, 4096))
 HBM_PEAK_GBS = 8000.0  # MI355X_MICROARCH.md: HBM3E 8.0 TB/s spec (6.29 TB/s measured copy ceiling)
 MFMA_PEAK_TFLOPS = 2500.0  # MI355X_MICROARCH.md: ~2.5 PFLOP/s dense bf16 (the 5 PF headline includes 2:1 sparsity)
 L2_INGEST_GBS_PER_CU = (66.0, 73.0)  # MI355X_MICROARCH.md "Indexed rows: gather into LDS": rows shared by every workgroup, served by the XCD's L2
-PREFILL_CASES = ((16, 1024), (4, 4096), (64, 256))        # SURVEY §8(d) config 4 prompt shapes
+PREFILL_CASES = ((16, 1024), (4, 4096), (64, 256))        # config 4 prompt shapes
 SAMPLED = dict(temperature=0.6, top_p=0.95, top_k=40)      # reference examples/cpu_inference_opt.py:153-158
 _T0 = time.perf_counter()
 
@@ -502,7 +502,7 @@ def projection_roofline(engine, rows: int):
 
 
 def step_roofline(engine, model, batch, ctx_mid, ms_per_step):
-    """The whole decode step against HBM (SURVEY §8 d): per GPU, every matrix weight of this rank touched once (embedding
+    """The whole decode step against HBM: per GPU, every matrix weight of this rank touched once (embedding
     rows excluded, the tied / untied LM head shard included) + the K/V bytes of the batch at its mean context."""
     ex = engine.model_runner.inference_executor
     seen, wbytes = set(), 0
@@ -540,7 +540,7 @@ def release_all(engine):
 
 
 def prefill_flops(heads: int, head_dim: int, lens, chunk: int = 0) -> int:
-    """Causal flash prefill without a cached prefix, one layer (SURVEY §8 d, K2): sum over sequences of
+    """Causal flash prefill without a cached prefix, one layer (K2): sum over sequences of
     4 H D (Sq Sk - Sq (Sq - 1) / 2) with Sq = Sk = len; a chunk mask cuts a sequence into pieces of ``chunk`` tokens."""
     if chunk:
         lens = [m for n in lens for m in [chunk] * (n // chunk) + [n % chunk]]
@@ -559,7 +559,7 @@ def _mfma_busy_quote():
 
 
 def prefill_records(engine, model, gpus=1, cases=PREFILL_CASES, reps=5):
-    """Prefill tokens/s of the whole model step (SURVEY §8 d(ii), config-4 prompt shapes): n prompts x len fresh
+    """Prefill tokens/s of the whole model step (config-4 prompt shapes): n prompts x len fresh
     random tokens through ``execute_batch(prefill=True)`` -- input build, H2D, every layer, LM head on the last
     tokens, sampler, D2H of the n tokens.  One warm-up per shape, then the median of ``reps`` timed batches; then ONE more
     batch whose mv_prefill_varlen launches (one per layer) are bracketed by HIP event pairs -> ``roofline``."""

@@ -126,7 +126,7 @@ int mv_rope_qk_store_ex(const void *q, const void *k, const void *v,
  * context_lens int32 [B]; out [B,H,D] contiguous.  Rows with
  * context_len <= 0 or max_blocks == 0 produce zeros
  * (page_attention.py:62-65).  Block ids outside [0,num_blocks) inside the
- * context contribute nothing (reference: zero K/V rows; see DESIGN.md Q9).
+ * context contribute nothing (reference: zero K/V rows).
  * workspace: mv_paged_decode_workspace_bytes() bytes, 16-byte aligned. */
 /* `flags` (same value for the size query and the call), 0 = kernel variant chosen from the shape: */
 enum {
@@ -222,7 +222,7 @@ int mv_prefill_varlen_ex(const void *q, int64_t q_stride_tok, const void *k,
  * by InferenceExecutor._sample_tokens (inference_executor.py:776-806).
  * logits [B,V] row stride ld; temperatures/top_ps/min_ps fp32 [B];
  * top_ks int64 [B] (<=0 or >=V disables); out_tokens int64 [B].
- * temperature == 0 -> argmax (lowest index on ties; SURVEY §9 Q4).
+ * temperature == 0 -> argmax (lowest index on ties).
  * RNG: Philox4x32-10 keyed by (seed, offset + *offset_dev, row); offset_dev
  * (device u64, may be NULL) lets a captured graph draw fresh numbers.
  * keep_mask (uint8 [B,V], may be NULL) receives the post-filter support set

@@ -1,4 +1,4 @@
-// C1 (SURVEY §8 b: mv_allreduce_*) — small-message all-reduce over xGMI peer-to-peer loads, for the
+// C1 (mv_allreduce_*) — small-message all-reduce over xGMI peer-to-peer loads, for the
 // [tokens, hidden] sums after o_proj / down_proj of a tensor-parallel decode step
 // (minivllm/models/layers/linear.py:316-318 calls dist.all_reduce; RCCL's ring needs 2(W-1) latency-bound
 // steps for a 1-2 MB message).  Two-shot, one launch, no host involvement, hipGraph-capturable:
@@ -184,7 +184,7 @@ __global__ void __launch_bounds__(kArThreads) allreduce_two_shot_kernel(ArParams
   }
 }
 
-// f1 (SURVEY §8) — all-reduce + residual add + RMSNorm in ONE launch, for a [M, K] activation with
+// f1 — all-reduce + residual add + RMSNorm in ONE launch, for a [M, K] activation with
 // M % world == 0: the same two-shot protocol with ROWS as the unit.  Row r belongs to slice r / (M/W) (the
 // rank that reduces it) and to block r % NB on every rank (so the per-block barriers cover every hand-off);
 // inside a block, wave (r / NB) % 8 owns it: a whole row per wave, the row norm is a wave reduction, no LDS.
@@ -350,7 +350,7 @@ __global__ void __launch_bounds__(kArThreads) allreduce_rows_kernel(ArRowParams 
   }
 }
 
-// f2 (SURVEY §8): greedy decoding under tensor parallelism without gathering the logits.  Every rank packs,
+// f2: greedy decoding under tensor parallelism without gathering the logits.  Every rank packs,
 // per row, the maximum of its vocab shard and the global index of that maximum into four 16-bit floats that
 // are EXACT in bf16/f16 (the logit itself; three 8-bit pieces of the index) at slot [rank] of a zeroed
 // [world][rows][4] buffer; the all-reduce above (sum with zeros = gather, exact) then hands every rank all

@@ -11,8 +11,7 @@
 //   top-p : smallest key v with mass(keys > v) <= p * mass(top-k set)
 //   min-p : weight threshold  exp((x-max)/T) >= min_p
 // then a single multinomial draw (Philox4x32-10) over the surviving weights.
-// Math is fp32 throughout (the reference computes in the logits dtype; see
-// DESIGN.md "sampler parity").
+// Math is fp32 throughout (the reference computes in the logits dtype).
 #include "common.h"
 
 namespace {
@@ -245,7 +244,7 @@ __global__ void __launch_bounds__(kThreads) sample_kernel(SampleParams p) {
     if (ok && (x > best || (x == best && i < best_i))) { best = x; best_i = i; }
   });
   const float xmax = block_max(best, sh);
-  if (temp == 0.0f) {  // greedy (SURVEY §9 Q4: argmax, not multinomial over softmax(l/1e-8))
+  if (temp == 0.0f) {  // greedy (argmax, not multinomial over softmax(l/1e-8))
     int cand = (best == xmax) ? best_i : 0x7fffffff;
 #pragma unroll
     for (int off = 32; off >= 1; off >>= 1) cand = min(cand, __shfl_xor(cand, off, 64));
@@ -611,7 +610,7 @@ __global__ void __launch_bounds__(kThreads) sample_kernel(SampleParams p) {
 }
 
 
-// f2 (SURVEY §8) for SAMPLED rows under tensor parallelism: instead of all-gathering [B, V/tp] logits, every
+// f2 for SAMPLED rows under tensor parallelism: instead of all-gathering [B, V/tp] logits, every
 // rank reduces its vocab shard of a row to its kTopC largest logits (+ their global indices).  For a row whose
 // top_k is in 1..kTopC (or that is greedy) the union of the per-rank candidates contains a complete top-k set, the
 // filters after it (top-p, min-p) and the draw only ever look at that set, so running the ordinary sampler on the
@@ -719,7 +718,7 @@ __global__ void topc_unpack_kernel(const uint16_t *buf, int world, int rows, int
 // candidate position -> token id.  Sampled rows: the global index of the drawn candidate.  Greedy rows
 // (temperature 0): the LOWEST global index among the candidates equal to the row maximum — candidates are laid out in
 // shard-visiting order, not in index order, so "first maximum by candidate position" could name a higher token id than
-// TP = 1 (argmax: lowest index on ties, DESIGN.md Q4) and the all-greedy path (mv_greedy_merge) do, and the same greedy
+// TP = 1 (argmax: lowest index on ties) and the all-greedy path (mv_greedy_merge) do, and the same greedy
 // request would then decode differently depending on what it is batched with.  One wave per row.
 template <typename Tag>
 __global__ void __launch_bounds__(64) topc_pick_kernel(const uint16_t *cand_logits, const int32_t *cand_idx,
@@ -749,7 +748,7 @@ __global__ void __launch_bounds__(64) topc_pick_kernel(const uint16_t *cand_logi
   if (lane == 0) tokens[r] = tok;
 }
 
-// f2 (SURVEY §8) for rows sampled from the WHOLE vocabulary (the default SamplingParams: top_k = -1, top_p = 1, min_p = 0)
+// f2 for rows sampled from the WHOLE vocabulary (the default SamplingParams: top_k = -1, top_p = 1, min_p = 0)
 // under tensor parallelism: an exact TWO-STAGE draw instead of the [B, V/tp] all-gather.  Every rank runs the ordinary
 // sampler on its own shard (token t_r drawn with the row's uniform u, row maximum m_r, mass S_r = sum exp((l - m_r)/T)),
 // the ranks exchange {m_r, S_r, t_r} per row — 16 bytes — through the slot scheme of the greedy path (exact 16-bit pieces
@@ -833,7 +832,7 @@ __global__ void mass_merge_kernel(const uint16_t *buf, const float *temperatures
 }
 
 
-// ---- nucleus (top-p) / min-p rows of vocabulary-sharded logits (SURVEY §8 f2) -----------------------------------
+// ---- nucleus (top-p) / min-p rows of vocabulary-sharded logits -----------------------------------
 // The edge of the nucleus is a property of the whole row: the smallest value v whose strictly-larger mass E(v) still
 // fits p * Z.  The ranks find it together by a two-level radix walk over the 16-bit order keys, counted DOWN from the
 // row's global maximum (offset = key(max) - key(x); level 0 bins the high byte of the offset, level 1 the low byte

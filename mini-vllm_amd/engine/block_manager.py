@@ -9,7 +9,7 @@ become the block tables and slot mappings the HIP kernels index with.  What fixe
   * a freed block keeps its digest/tokens until it is handed out again (so it can be revived).
 Method names, the deque-plus-tombstone pool and the order of its operations are the reference's by necessity (the ids
 they produce are compared bit for bit with reference traces, tests/test_host_logic.py); the error texts are this
-build's own, except the leading words of "No free blocks available", which DESIGN.md Q10 and the scheduler refer to.
+build's own, except the leading words of "No free blocks available", which the scheduler refers to.
 """
 from __future__ import annotations
 
@@ -77,7 +77,7 @@ class BlockManager:
             if q[0] in self._free_set:
                 return q[0]
             q.popleft()  # tombstone of a block that was taken since
-        raise RuntimeError("No free blocks available: the KV pool is exhausted")  # (first words = the reference's, DESIGN.md Q10)
+        raise RuntimeError("No free blocks available: the KV pool is exhausted")  # (first words = the reference's)
 
     def _take(self, block_id: int, reset: bool = True) -> Block:
         if not 0 <= block_id < self.num_blocks:
@@ -149,7 +149,7 @@ class BlockManager:
             sequence.block_table.append(block_id)
         if sequence.num_cached_tokens >= sequence.num_tokens:
             # every block hit (len % block_size == 0): the reference then prefills ZERO query tokens
-            # and samples from another sequence's row (SURVEY §9 Q3).  Recompute the last block
+            # and samples from another sequence's row.  Recompute the last block
             # instead, so that there is a last-token logit; the rewrite of the shared block is
             # byte-identical.
             sequence.num_cached_tokens -= self.block_size
@@ -177,7 +177,7 @@ class BlockManager:
     # -- decode-time growth (block_manager.py:369-450) ------------------------------------------
     def can_append(self, sequence: Sequence) -> bool:
         """Reference predicate, kept verbatim for trace parity: a block is "needed" when
-        len % block_size == 0 — one step BEFORE may_append actually takes it (DESIGN.md Q10)."""
+        len % block_size == 0 — one step BEFORE may_append actually takes it."""
         need = 1 if len(sequence) % self.block_size == 0 else 0
         return len(self._free_set) >= need
 

@@ -2,7 +2,7 @@
 one process per GPU, ``torch.distributed`` backend "nccl" (= RCCL over xGMI on ROCm) for the
 data plane (C1-C3) and a small gloo group on the host for the control plane (C4).
 
-Unlike the reference this runs BEFORE the model is built (SURVEY §9 Q1) and registers the
+Unlike the reference this runs BEFORE the model is built and registers the
 rank/size with ``parallel_state`` so that every layer shards itself."""
 from __future__ import annotations
 

@@ -3,13 +3,13 @@ model execution, sampling (mirror of minivllm/engine/inference_executor.py:35-94
 
 MI355X-first differences from the reference:
   * KV cache sized for 288 GB HBM3E with the LOCAL kv-head count (the reference uses the total
-    head count even under TP, SURVEY §9 Q1) — layout [2, L, num_blocks, block_size, Hkv/tp, D];
+    head count even under TP) — layout [2, L, num_blocks, block_size, Hkv/tp, D];
   * the decode step — model forward, LM head AND the sampler — is ONE captured hipGraph per
     batch-size bucket; every per-step quantity (ids, positions, slots, context lens, block
     tables, sampling params, RNG offset) lives in static device buffers that are refreshed by
     a handful of async copies; the only host sync of a step is reading back the B token ids;
   * the reference's graph path is dead code (row-0 broadcast bug, fp32 output buffer, host syncs
-    in the attention fallback: SURVEY §9 Q2); here graph replay is checked bit-identical
+    in the attention fallback); here graph replay is checked bit-identical
     against eager execution.
 """
 from __future__ import annotations

@@ -22,7 +22,7 @@ _DTYPES = {"float16": torch.float16, "bfloat16": torch.bfloat16, "float32": torc
 def resolve_dtype(config: Config) -> torch.dtype:
     if config.dtype != "auto":
         return _DTYPES[config.dtype]
-    # the reference leaves "auto" at fp32 whatever the checkpoint says (SURVEY §9 Q6); here it
+    # the reference leaves "auto" at fp32 whatever the checkpoint says; here it
     # means what it says: the checkpoint's own dtype
     hf = getattr(config.hf_config, "torch_dtype", None) or getattr(config.hf_config, "dtype", None)
     if isinstance(hf, str):

@@ -4,7 +4,7 @@ ever calls ``call("run", seqs, is_prefill) -> list[int]`` and ``call("exit")``.
 Execution is SPMD: every tensor-parallel rank holds the same scheduler state and calls ``run`` with
 the same batch, so — unlike the reference — no per-step pickle of ``Sequence`` objects crosses a
 process boundary; only ``generate`` requests do (see LLMEngine).  Worker errors are raised, not
-swallowed (SURVEY §9 Q7)."""
+swallowed."""
 from __future__ import annotations
 
 import logging

@@ -4,7 +4,7 @@ otherwise every running sequence decodes one token, preempting the newest when b
 out.  Preempted sequences lose their blocks and are re-prefilled from the front of the queue
 (recompute; the prefix cache often rescues them).
 
-Beyond the reference (SURVEY §8 f4, BASELINE config 4 "chunked prefill"): a prompt longer than
+Beyond the reference (BASELINE config 4 "chunked prefill"): a prompt longer than
 max_num_batched_tokens — which the reference can never schedule — is prefilled ALONE in chunks of at most
 max_num_batched_tokens tokens (whole blocks), one chunk per step, each attending the chunks before it through
 the paged KV cache (the prefix-cached form of the prefill kernel).  Only the last chunk's token is kept.  Every

@@ -32,7 +32,7 @@ class Sequence:
         self.num_tokens = len(self.token_ids)
         self.num_prompt_tokens = self.num_tokens
         self.num_cached_tokens = 0
-        # chunked prefill (beyond the reference, SURVEY §8 f4): a prefill step computes tokens
+        # chunked prefill (beyond the reference): a prefill step computes tokens
         # [num_cached_tokens, prefill_end); None = up to the end of the sequence (the reference's only mode)
         self.prefill_end: int | None = None
         self.block_table: list[int] = []

@@ -1,6 +1,6 @@
 """Qwen2 / Qwen3 decoder glue (mirror of minivllm/models/qwen_base.py, qwen2.py, qwen3.py).
 
-Op order per layer fixes the fusion boundaries (SURVEY §8 a14):
+Op order per layer fixes the fusion boundaries:
     qkv GEMM -> [q/k head RMSNorm] -> RoPE -> KV store   == ONE HIP launch (mv_rope_qk_store)
     -> attention (varlen prefill | paged decode)          == ONE HIP launch
     -> o_proj (+all-reduce) -> add+RMSNorm (fused HIP) -> gate_up GEMM -> SiluAndMul (HIP)

@@ -1,5 +1,5 @@
 """Architecture registry (mirror of minivllm/models/registry.py:30-52).  GPT-2 is not built:
-it is in none of the benchmark configurations (SURVEY §2 #24)."""
+it is in none of the benchmark configurations."""
 from typing import Any
 
 from .mofarax import MofaraxForCausalLM

@@ -726,7 +726,7 @@ def gate_up_silu_small_m(x, weight, shape: int = 0, packed=None, act: str = "sil
 # rows x vectors-per-norm-thread up to which the layer norm rides in the prologue of the small-M projection behind it.  The
 # kernel takes up to 8 (csrc/linear_small_m.hip: kNormRows, in passes of 4 / PT rows, round 4), but beyond one pass the
 # prologue costs more than the norm launch it saves — Qwen3-1.7B, ctx 1024: B = 5 1.52 -> 1.61 ms per step, B = 8 1.66 ->
-# 1.81 (gpurun_out/r4e_*) — so the default stays at one pass (4); MV_NORM_FOLD_MAX_ROWS=8 selects the longer fold
+# 1.81 — so the default stays at one pass (4); MV_NORM_FOLD_MAX_ROWS=8 selects the longer fold
 NORM_FUSED_MAX_ROWS = min(8, int(os.environ.get("MV_NORM_FOLD_MAX_ROWS", "4")))
 
 

@@ -1,7 +1,7 @@
 """Token sampler on the fused HIP kernel (replaces minivllm/sampling/sampler.py:12-110 and
 sampling/functional.py as wired by the engine: temperature -> top-k -> top-p -> min-p ->
 multinomial).  Penalties / typical / avoid-top-k are not reachable from ``SamplingParams`` in
-the reference and are not built (SURVEY §2 #26)."""
+the reference and are not built."""
 from __future__ import annotations
 
 import torch
@@ -21,7 +21,7 @@ class Sampler(nn.Module):
 
     def forward(self, logits, temperatures=None, top_ks=None, top_ps=None, min_ps=None, **unused):
         """logits [B,V] -> int64 [B].  temperature 0 = argmax (the reference's tensor-temperature
-        path turns 0 into softmax(l/1e-8) + multinomial, SURVEY §9 Q4)."""
+        path turns 0 into softmax(l/1e-8) + multinomial)."""
         if logits.dim() != 2:
             raise ValueError(f"logits must be 2D [batch_size, vocab_size], got {logits.shape}")
         b = logits.shape[0]

@@ -1,7 +1,7 @@
 """Tensor-parallel process state: one process per GPU, torch.distributed ("nccl" = RCCL over
 xGMI).  Set ONCE, before the model is built — the reference derives tp_size from
 ``dist.is_initialized()`` while constructing layers but only initialises the process group
-afterwards, so its TP>1 silently builds replicated models (SURVEY §9 Q1)."""
+afterwards, so its TP>1 silently builds replicated models."""
 from __future__ import annotations
 
 import torch
@@ -57,7 +57,7 @@ def tp_all_reduce(x: torch.Tensor) -> torch.Tensor:
 
 def tp_all_reduce_add_rmsnorm(x: torch.Tensor, residual: torch.Tensor, weight: torch.Tensor, eps: float):
     """``tp_all_reduce(x)`` followed by the fused residual-add + RMSNorm -> (normed, residual), residual
-    updated in place.  One launch on the peer-to-peer kernel when it takes the shape (SURVEY §8 f1),
+    updated in place.  One launch on the peer-to-peer kernel when it takes the shape,
     otherwise the two steps."""
     from . import hip_ops
 
@@ -96,7 +96,7 @@ def tp_all_gather_last_dim(x: torch.Tensor) -> torch.Tensor:
 
 
 def tp_merge_greedy(local_tokens: torch.Tensor, local_values: torch.Tensor, vocab_per_rank: int) -> torch.Tensor:
-    """Greedy decoding without the full-logit gather (SURVEY §8 f2): each rank brings the argmax of its
+    """Greedy decoding without the full-logit gather: each rank brings the argmax of its
     vocab shard (shard-local index, lowest on ties) and its value; the row's token is the global index
     of the largest value, the lowest global index on ties -- exactly ``argmax`` of the gathered row.
     One all-gather of B x 16 bytes per rank instead of B x V/tp logits."""
@@ -127,7 +127,7 @@ def tp_greedy_tokens(logits_local: torch.Tensor, local_tokens: torch.Tensor) -> 
 
 
 def tp_candidate_tokens(logits_local: torch.Tensor, sample_fn, temperatures: torch.Tensor | None = None) -> torch.Tensor:
-    """Sampled tokens without the full-logit gather (SURVEY §8 f2, sampled rows): valid for batches whose rows are
+    """Sampled tokens without the full-logit gather (sampled rows): valid for batches whose rows are
     greedy or have 1 <= top_k <= hip_ops.TOPC.  Every rank packs the 64 largest logits of its vocab shard per row
     (+ global indices) into its slot of a zeroed buffer, the all-reduce sums the slots (x + 0: an exact gather,
     on the peer-to-peer kernel when it is up: no backend collective), ``sample_fn(cand_logits [B, tp*64]) -> int64
@@ -149,7 +149,7 @@ def tp_candidate_tokens(logits_local: torch.Tensor, sample_fn, temperatures: tor
 def tp_mass_tokens(logits_local: torch.Tensor, sample_stats_fn, temperatures: torch.Tensor, seed: int, offset: int,
                    offset_dev=None) -> torch.Tensor:
     """Tokens of rows sampled from the WHOLE vocabulary (top_k off, top_p = 1, min_p = 0: the default SamplingParams)
-    or greedy, without the logit gather (SURVEY §8 f2): an exact two-stage draw.  ``sample_stats_fn(logits_local) ->
+    or greedy, without the logit gather: an exact two-stage draw.  ``sample_stats_fn(logits_local) ->
     (local tokens, fp32 [B, 2] {shard maximum, shard mass})`` is the ordinary sampler on this rank's shard; the ranks
     exchange 16 bytes per row through the slot scheme (peer-to-peer all-reduce when it is up: no backend collective)
     and pick the same rank with probability proportional to its mass from a second uniform of the same Philox counter
@@ -167,7 +167,7 @@ def tp_mass_tokens(logits_local: torch.Tensor, sample_stats_fn, temperatures: to
 def tp_nucleus_tokens(logits_local: torch.Tensor, sample_stats_fn, temperatures: torch.Tensor, top_ps: torch.Tensor,
                       min_ps: torch.Tensor, seed: int, offset: int, offset_dev=None) -> torch.Tensor:
     """Tokens of rows with a nucleus (top_p < 1) and / or a min-p filter and top_k off (plus greedy / unfiltered rows
-    in the same batch) without the logit gather (SURVEY §8 f2).  The ranks find the edge of the kept set together:
+    in the same batch) without the logit gather.  The ranks find the edge of the kept set together:
     the row maximum (MAX all-reduce of B floats), then a two-level radix walk over the 16-bit order keys below it with
     one all-reduced 256-bin histogram of fixed-point masses per level (mv_shard_key_hist / mv_nucleus_pick: integer
     sums, so every rank derives the same floor); every rank masks its shard below the floor and the batch finishes as

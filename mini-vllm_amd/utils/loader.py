@@ -3,7 +3,7 @@ local directory, HF names remapped onto the fused parameters (q_proj|k_proj|v_pr
 gate_proj|up_proj -> gate_up_proj) and sliced per tensor-parallel rank by each parameter's
 ``weight_loader``.  Local paths only: there is no network on the benchmark machines.
 
-Sharded, direct-to-device (SURVEY §8 f4; the reference reads every tensor whole onto the CPU and slices it
+Sharded, direct-to-device (the reference reads every tensor whole onto the CPU and slices it
 there): a safetensors tensor reaches the ``weight_loader`` as a ``LazyTensor`` — shape and dtype known, nothing
 read yet.  ``narrow`` / ``chunk`` (the only things the loaders do before ``copy_``) turn into a slice of the file,
 read straight onto the parameter's device: at TP = 8 a rank reads 1/8 of every sharded matrix (18 of 145 GB for

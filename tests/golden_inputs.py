@@ -60,7 +60,7 @@ def wide_decode_inputs(case):
 
 
 # prefill cases: packed varlen causal attention; the same outputs pin the prefix-cached form (the rows of the new
-# tokens of a FULL no-cache prefill are what a prefix-cached prefill must produce, SURVEY §9 Q3)
+# tokens of a FULL no-cache prefill are what a prefix-cached prefill must produce)
 WIDE_PREFILL = [
     dict(name="qwen3_16_8", H=16, Hkv=8, D=128, lens=[300, 77, 1024, 1], cached=[256, 64, 960, 0], seed=1201),
     dict(name="qwen2_28_4", H=28, Hkv=4, D=128, lens=[640, 129], cached=[576, 128], seed=1202),

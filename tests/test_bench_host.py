@@ -75,7 +75,7 @@ def test_projection_plan_ingest_figures_for_the_headline_shapes():
 
 
 def test_prefill_flops_formula():
-    # 4 H D (Sq Sk - Sq (Sq - 1) / 2); S = 4096, H = 28, D = 128 -> 1.20e11 per sequence and layer
+    # causal flash prefill: 4 H D (Sq Sk - Sq (Sq - 1) / 2); S = 4096, H = 28, D = 128 -> 1.20e11 per sequence and layer
     assert abs(bench.prefill_flops(28, 128, [4096]) / 1.20e11 - 1) < 0.01
     assert bench.prefill_flops(16, 128, [1024] * 16) == 16 * 4 * 16 * 128 * (1024 * 1024 - 1024 * 1023 // 2)
 

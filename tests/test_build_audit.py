@@ -3,7 +3,7 @@
 The default (PIPE) ``prefill_mfma_kernel`` retires its inline-assembly LDS reads with HAND-COUNTED ``s_waitcnt
 lgkmcnt(N)`` (csrc/prefill_mfma.hip).  ``lgkmcnt`` also counts scalar memory loads, so a count is only sound while the
 compiler places no ``s_load`` / ``s_buffer_load`` inside the span of the counted reads; and the kernel must neither
-spill nor use scratch.  A compiler or code change could silently break either (ADVICE r3): this test re-checks the
+spill nor use scratch.  A compiler or code change could silently break either: this test re-checks the
 shipped instantiations and the 64-rows-per-wave bench kernel (its accumulator file is asm-owned) on every run."""
 import os
 import re

@@ -100,7 +100,7 @@ def test_fp32_logits_match_reference(golden_dir, tmp_path, name):
 def test_bf16_logits_within_reference_noise(golden_dir, tmp_path, name):
     """north_star: 'matching the reference eager path logits within 1e-3 bf16'.  The reference's own
     bf16 run differs from its fp32 run by more than that on these models, so the
-    bound is max(1e-3 * scale, 1.5 x the reference's bf16-vs-fp32 error), per SURVEY §8c."""
+    bound is max(1e-3 * scale, 1.5 x the reference's bf16-vs-fp32 error)."""
     z = _load(golden_dir, name)
     _, _, ex = _build(tmp_path, z, torch.bfloat16)
     outs = _run(ex, z)
@@ -215,7 +215,7 @@ def test_other_legal_block_sizes_end_to_end(golden_dir, tmp_path, bs):
 
 def test_prefix_cached_prefill_matches_full_prefill(golden_dir, tmp_path):
     """A prompt whose first block is served by the prefix cache must give the logits of a clean
-    full prefill (the reference's fallback gets this wrong, SURVEY §9 Q3)."""
+    full prefill (the reference's fallback gets this wrong)."""
     from minivllm_amd.engine.block_manager import BlockManager
     from minivllm_amd.engine.sequence import Sequence
 
@@ -464,7 +464,7 @@ def test_config5_per_gpu_layer_shape_qwen2_72b_tp8(tmp_path):
         err = (got - want).abs().max().item()
         worst = max(worst, err / scale)
         worst_noise = max(worst_noise, noise / scale)
-        # the bar of every other e2e test (SURVEY §8c): max(1e-3 * scale, 1.5 x the bf16 noise of the eager op order)
+        # the bar of every other e2e test: max(1e-3 * scale, 1.5 x the bf16 noise of the eager op order)
         assert err <= max(1e-3 * scale, 1.5 * noise), f"step {step}: err {err:.4f} noise {noise:.4f} scale {scale:.3f}"
         assert torch.nn.functional.cosine_similarity(got.flatten(), want.flatten(), dim=0).item() > 0.9995
         for s, t in zip(seqs, want.argmax(-1).tolist()):

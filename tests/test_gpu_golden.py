@@ -162,7 +162,7 @@ def test_golden_prefill_wide_and_prefix_cached(H, GW, name, dtype):
     out = H.prefill_varlen(qd, kd, vd, cu.to(DEV), cu.to(DEV), max(lens), max(lens), D ** -0.5)
     torch.testing.assert_close(out.float().cpu()[rows], want[rows], **tol)
     # prefix-cached form: the first cached[i] tokens of sequence i live only in the paged cache; the rows of the
-    # remaining tokens must equal the SAME rows of the reference's full no-cache prefill (SURVEY §9 Q3)
+    # remaining tokens must equal the SAME rows of the reference's full no-cache prefill
     bs, Hkv = 64, case["Hkv"]
     nblk = [-(-n // bs) for n in lens]
     perm = torch.randperm(sum(nblk) + 1, generator=torch.Generator().manual_seed(9)).tolist()
@@ -188,7 +188,7 @@ def test_config2_qwen3_0p6b_full_depth_against_the_reference(golden_dir, tmp_pat
     """Qwen3-0.6B (28 layers, 16/8 heads, D = 128, vocab 151936), bf16, enforce_eager.  The
     fixture holds what the REFERENCE computed on the CPU in fp32 for the same seeded weights and prompts (logits at
     512 fixed vocabulary columns + the top-8 of every row) and the reference's own bf16-vs-fp32 error.  Bound, as
-    for the tiny models (SURVEY §8c): max(1e-3 * scale, 1.5 x the reference's bf16 noise); the error is printed."""
+    for the tiny models: max(1e-3 * scale, 1.5 x the reference's bf16 noise); the error is printed."""
     from minivllm_amd.config import Config
     from minivllm_amd.engine.block_manager import BlockManager
     from minivllm_amd.engine.inference_executor import InferenceExecutor

@@ -416,7 +416,7 @@ def test_prefill_mfma_strided_qkv_and_f16(H):
 @pytest.mark.parametrize("dtype", [torch.bfloat16, torch.float32])
 def test_prefill_paged_prefix(H, dtype):
     """Prefix-cache hit: queries are the uncached suffix, keys come from the paged cache
-    (flash-attn semantics; oracle = full no-cache prefill rows, SURVEY §9 Q3)."""
+    (flash-attn semantics; oracle = full no-cache prefill rows)."""
     Hq, Hkv, D, bs = 8, 4, 128, 64
     full = [64 + 5, 128 + 64, 40]       # total lengths
     cached = [64, 128, 0]               # cached prefix (multiples of bs)
@@ -710,7 +710,7 @@ def test_nucleus_floor_across_shards_is_the_full_row_keep_mask(H, dtype, world):
 
 @pytest.mark.parametrize("world", [2, 8])
 def test_nucleus_floor_with_ties_at_the_edge(H, world):
-    """ADVICE r3: rows made of a few distinct values, so that the nucleus edge falls ON a tie group, with p just below
+    """rows made of a few distinct values, so that the nucleus edge falls ON a tie group, with p just below
     and just above the group boundaries -- the case where the cross-rank floor (budget = trunc(p * Z) on 2^-40 fixed-point
     masses, `mv_nucleus_pick`) could part ways with `mv_sample` (fp32 masses) and with the reference's sort-based cut.
     Pinned here: (1) the emulated ranks keep EXACTLY `mv_sample`'s set, at every p; (2) both keep the edge's tie group
@@ -1014,7 +1014,7 @@ def test_linear_mid_m_every_tile(H, dtype, m, n, k, bias):
 
 
 def test_timing_ablation_switches_are_not_reachable_in_the_production_build(H):
-    """ADVICE r3: the bench-only switches of mv_linear_mid_m (cfg + 100 x flags: DMA ring only, no x / W DMA, clock
+    """the bench-only switches of mv_linear_mid_m (cfg + 100 x flags: DMA ring only, no x / W DMA, clock
     stamps INTO `bias`, no output stores) and of mv_prefill_varlen (no K/V refresh, no output stores) leave garbage or
     write out of bounds.  They are compiled only with `make ABLATE=1`; the shipped library answers MV_E_RANGE."""
     x = _randn(64, 256, dtype=torch.bfloat16, seed=1).to(DEV)

@@ -98,7 +98,7 @@ def _worker(rank, port, out_path):
             ok &= bool(torch.equal(out_n, eager[i][0]) and torch.equal(out_r, eager[i][1]))
         res["graph_replays_equal_eager"] = ok
         res["graph_all_gather_ok"] = bool(torch.equal(gathered, logits_local))
-    except Exception as e:  # recorded, not raised: whether RCCL captures is the finding (DESIGN.md §5)
+    except Exception as e:  # recorded, not raised: whether RCCL captures is the finding
         err = f"{type(e).__name__}: {e}"
     res["rccl_in_graph_capture"] = captured
     res["capture_error"] = err[:500]

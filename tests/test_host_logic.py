@@ -30,7 +30,7 @@ def fake_next_token(tokens, vocab):
 def test_xxh64_digests(traces):
     for case in traces["hashes"]:
         assert BlockManager.compute_hash(case["tokens"], case["prefix"]) == case["hash"]
-    # SURVEY §8 known answers
+    # known answers
     assert BlockManager.compute_hash([1, 2, 3]) == 13048208712247349756
     assert BlockManager.compute_hash([1, 2, 3], prefix=5) == 17518828517520909647
     assert BlockManager.compute_hash(list(range(64))) == 4138455281752509893
@@ -100,7 +100,7 @@ def test_replay_reference_trace(traces, idx):
 
 
 def test_survey_known_answer_trace():
-    """SURVEY §8: two prompts (130 and 3 tokens), fresh BlockManager(16, 64)."""
+    """two prompts (130 and 3 tokens), fresh BlockManager(16, 64)."""
     bm = BlockManager(16, 64)
     a, b = Sequence(list(range(1, 131))), Sequence(list(range(500, 503)))
     bm.allocate(a)
@@ -136,7 +136,7 @@ def test_prefix_cache_hit_shares_block():
 
 
 def test_fully_cached_prompt_keeps_a_query_block():
-    """Build semantics where the reference is broken (SURVEY §9 Q3): a prompt whose every block
+    """Build semantics where the reference is broken: a prompt whose every block
     hits the prefix cache recomputes its last block so that a last-token logit exists."""
     bm = BlockManager(8, 64)
     toks = list(range(1, 129))
@@ -151,7 +151,7 @@ def test_fully_cached_prompt_keeps_a_query_block():
 
 
 def test_block_pressure_preempts_instead_of_raising():
-    """DESIGN.md Q10: the reference raises 'No free blocks available' when a sequence needs its
+    """the reference raises 'No free blocks available' when a sequence needs its
     next block (len % bs == 1) and none is free; the build preempts the newest sequence instead."""
     cfg = SimpleNamespace(max_num_seqs=4, max_num_batched_tokens=512, eos=-1, num_kvcache_blocks=3,
                           kvcache_block_size=64)
@@ -432,7 +432,7 @@ def test_nucleus_batches_fall_back_to_the_gather_graphs_when_their_own_family_ca
     """Tensor parallel, a batch with top-p rows and top_k off ('nuc' mode).  Its graph family holds backend
     collectives and is captured lazily, only where the peer-to-peer all-reduce is up.  On an RCCL-only run (or after
     a failed capture) the family stays empty while the gathered-logits graphs exist: such a batch must replay THOSE,
-    not drop to an eager step (ADVICE r3).  The eager path and the replay ask the same helper, so they agree."""
+    not drop to an eager step.  The eager path and the replay ask the same helper, so they agree."""
     import torch
 
     from minivllm_amd.engine.inference_executor import InferenceExecutor

@@ -1,5 +1,5 @@
 """Tensor parallelism (SURVEY §8 a13 / e).  The reference never exercises TP>1 (its layers are built
-before the process group exists, SURVEY §9 Q1), so the oracle here is the build's own TP=1 result
+before the process group exists), so the oracle here is the build's own TP=1 result
 and, end to end, the reference's TP=1 logits.
   * CPU, gloo, world_size 2: sharded linears / embedding / LM head == unsharded math
   * GPU, 2 processes on the one card (gloo for the collectives): tiny Qwen3 with TP=2 reproduces the
@@ -208,7 +208,7 @@ def test_tp2_logits_match_reference_on_one_gpu(golden_dir, tmp_path):
 
 # ---------------------------------------------------------------------------------- sharded checkpoint loading (CPU)
 def _sharded_load_worker(rank, world, port, golden, ckpt_dir, out_path):
-    """SURVEY §8 f4: every rank reads from the safetensors file only the slices it owns (LazyTensor), and ends up
+    """every rank reads from the safetensors file only the slices it owns (LazyTensor), and ends up
     with exactly the shard the reference's loaders would cut from the whole tensor."""
     _init(rank, world, port)
     from transformers import AutoConfig
@@ -544,7 +544,7 @@ def test_llm_spawned_tp2_generates_like_tp1(golden_dir, tmp_path, monkeypatch):
         assert captured and spec_hits > 0
     assert not run(2, "float32", eager=False)[1]
     # sampled rows with a small top_k, 16-bit logits: no logit gather — every rank contributes its 64 best candidates
-    # per row (SURVEY §8 f2); the ranks draw the same tokens (the driver would otherwise diverge from its worker and
+    # per row; the ranks draw the same tokens (the driver would otherwise diverge from its worker and
     # the run would hang or mismatch), the mode really ran, eager and captured replay agree, and every generated
     # token has a non-zero probability under the same filters on TP = 1 logits is checked by the kernel test
     small_k = SamplingParams(temperature=0.8, top_p=0.95, top_k=40, max_tokens=12, ignore_eos=True)

@@ -1,5 +1,5 @@
 #!/usr/bin/env python3
-"""What mixed prefill/decode batches buy (Config.enable_mixed_batches, SURVEY §8 f4): a serving trace on one engine.
+"""What mixed prefill/decode batches buy (Config.enable_mixed_batches): a serving trace on one engine.
 
 `--running` sequences are decoding (context `--ctx`) while `--arrivals` prompts of `--prompt` tokens arrive, one every
 `--every` engine steps.  Reported per schedule (separate steps = the reference's: a prefill step stalls every decoder;

@@ -1,5 +1,5 @@
 #!/usr/bin/env python3
-"""Prefill tokens/s of the whole model step (SURVEY §8 d(ii), configs 3/4): batches of n prompts x len tokens
+"""Prefill tokens/s of the whole model step (configs 3/4): batches of n prompts x len tokens
 through ``InferenceExecutor.execute_batch(prefill=True)`` -- input build, H2D, every layer (hipBLASLt GEMMs,
 fused norm/rope/store kernels, the MFMA flash prefill), LM head on the last tokens and the sampler.
 Random-init weights at the true dimensions, fresh random prompts per repetition (no prefix-cache hits),

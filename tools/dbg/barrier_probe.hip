@@ -1,4 +1,4 @@
-// Grid-barrier price on MI355X for the persistent small-batch decode kernel (VERDICT r3 item 3): 256 workgroups of 512
+// Grid-barrier price on MI355X for the persistent small-batch decode kernel: 256 workgroups of 512
 // threads, one per CU, N barriers in a row; between two barriers every workgroup publishes a small record (16 B per
 // lane of wave 0, write-through stores) and after the barrier reads the record of ANOTHER workgroup and checks it
 // word for word.  Variants:
