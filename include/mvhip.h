@@ -297,8 +297,19 @@ int mv_silu_and_mul(const void *x, int64_t x_stride, void *out,
 int mv_gelu_and_mul(const void *x, int64_t x_stride, void *out, int64_t out_stride,
                     int rows, int cols, int dtype, void *stream);
 
+/* Activation of a gated projection, act(gate, up) (HOST struct, read during the call).  MV_ACT_CLAMPED: g = min(gate, limit),
+ * u = clamp(up, -limit, limit), g * sigmoid(alpha * g) * (u + 1). */
+enum { MV_ACT_SILU = 0, MV_ACT_GELU = 1, MV_ACT_CLAMPED = 2 };
+typedef struct MvGateAct {
+  int kind;
+  float limit, alpha;
+} MvGateAct;
+/* out[r, c] = act(x[r, c], x[r, cols + c]), fp32 inside */
+int mv_act_and_mul(const void *x, int64_t x_stride, void *out, int64_t out_stride, int rows, int cols,
+                   const MvGateAct *act, int dtype, void *stream);
+
 /* K13 — one edge of a residual stream kept in fp32.  Per row, with the stream x [rows][cols] (dense fp32, in place):
- *     b = x, or (embed_mode 1) nothing;   y' = y, or (y_norm_w) y / sqrt(mean(y^2) + eps) * y_norm_w
+ *     b = x, or (embed_mode 1) nothing;   y' = y, or (y_norm_w) y / sqrt(mean(y^2) + eps) * y_norm_w;   y' *= y_scale * y_mult
  *     x = b + y' + [embed_mode 1 or 2: embed_scale * embed[ids[row]]] + [vec]
  *     out = (norm_w) x / sqrt(mean(x^2) + eps) * (norm_offset + norm_w), else x, rounded to dtype   (out NULL: nothing)
  * y: rows of dtype at stride y_stride, or (y_splits > 0) fp32 partial sums [y_splits][rows][cols]; NULL = nothing.
@@ -312,6 +323,8 @@ typedef struct MvResidualArgs {
   int64_t y_stride, out_stride, vocab;
   float embed_scale, norm_offset, eps;
   int y_splits, embed_mode;
+  float y_mult;          /* 1 = none */
+  const void *y_scale;   /* [cols] of dtype; NULL = ones */
 } MvResidualArgs;
 int mv_residual_update(const MvResidualArgs *args, int rows, int cols, int cols_true, int dtype, void *stream);
 
@@ -364,6 +377,11 @@ int mv_gate_up_silu_small_m_packed(const void *x, int64_t x_stride, const void *
                                    void *out, int64_t out_stride, int m, int n_inter,
                                    int k, int dtype, int shape, void *stream);
 
+/* ... with the activation and its constants as an argument (packed != 0: w_gate_up is the fragment-ordered copy) */
+int mv_gated_act_small_m(const void *x, int64_t x_stride, const void *w_gate_up, int packed, void *out,
+                         int64_t out_stride, int m, int n_inter, int k, const MvGateAct *act, int dtype,
+                         int shape, void *stream);
+
 /* K6 + K10 — the RMSNorm in front of a projection folded into the projection's launch, for decode steps of <= 4
  * rows (K <= 2048; 2 rows to 4096, 1 row to 8192): every workgroup re-enacts the norm of those few rows in its
  * prologue (the arithmetic of mv_rmsnorm / mv_add_rmsnorm thread for thread), so the step loses two launches per
@@ -405,6 +423,9 @@ int mv_linear_mid_m(const void *x, int64_t x_stride, const void *w_packed, const
 int mv_gate_up_silu_mid_m(const void *x, int64_t x_stride, const void *w_gate_up_packed,
                           void *out, int64_t out_stride, int m, int n_inter, int k,
                           int dtype, int cfg, void *stream);
+int mv_gated_act_mid_m(const void *x, int64_t x_stride, const void *w_gate_up_packed, void *out,
+                       int64_t out_stride, int m, int n_inter, int k, const MvGateAct *act, int dtype,
+                       int cfg, void *stream);
 /* K11, K split over `splits` workgroup groups: out_partial [splits][m][n] fp32, unrounded, no bias; the
  * consumer kernel behind it sums the slices in split order (deterministic). */
 int mv_linear_mid_m_partial(const void *x, int64_t x_stride, const void *w_packed,
@@ -533,6 +554,116 @@ int mv_topc_unpack(const void *buf, int world, int rows, int rows_padded, void *
  * mv_greedy_merge name on ties (candidate order is shard-visiting order, not index order). */
 int mv_topc_pick(const void *cand_logits, const int32_t *cand_idx, const int64_t *pos,
                  const float *temperatures, int64_t *tokens, int rows, int width, int dtype, void *stream);
+
+/* ---- K14 — latent attention: keys and values of a token are one cached row [latent | rotated part], shared by all heads.
+ * A plane is [num_slots] rows of kv_cols + rot_cols elements (num_slots = blocks * block_size); columns beyond kv_rank and
+ * rot_dim hold zeros.  Rotation: dims 2i, 2i + 1 of the rotated part form a pair, cos / sin [max_pos, rot_dim / 2] fp32.
+ * Window: > 0: position i sees the keys i - window + 1 .. i; 0: every key up to i.  All sizes *_cols are multiples of 32. */
+
+/* `flags` of the two attention calls: MV_LATENT_SIMPLE = the vector-ALU kernel for 16-bit tensors too */
+enum { MV_LATENT_SIMPLE = 1 };
+
+/* One launch behind the merged down projection z: q_out = rms(z[q_off ..]) * q_norm_w; and (kv_rank > 0) the row
+ * [rms(z[kv_off ..]) * kv_norm_w | rotated z[rot_off ..]] into plane[slot_mapping[t]] (slots outside the plane: nothing)
+ * and / or rows_out[t].  Norm weights are zero-padded to q_cols / kv_cols. */
+typedef struct MvLatentPrepArgs {
+  const void *z;
+  int64_t z_stride;
+  const void *q_norm_w, *kv_norm_w;
+  void *q_out;
+  int64_t q_out_stride;
+  void *rows_out, *plane;
+  const int32_t *slot_mapping;
+  int64_t num_slots;
+  const int64_t *positions;
+  const float *cos, *sin;
+  int64_t max_pos;
+  int q_off, q_rank, q_cols, kv_off, kv_rank, kv_cols, rot_off, rot_dim, rot_cols;
+  float eps;
+} MvLatentPrepArgs;
+int mv_latent_prep(const MvLatentPrepArgs *args, int n_tok, int dtype, void *stream);
+
+/* Per-head product: out[t, h, 0..n) = w[h] (n x k) . x[t, h, 0..k); w dense [heads][n][k]; n % 16 == 0, k % 32 == 0.  With
+ * rot_dim > 0 additionally out[t, h, n .. n + rot_cols) = the rotation of x[t, h, k .. k + rot_dim), zeros behind. */
+typedef struct MvHeadLinearArgs {
+  const void *x, *w;
+  void *out;
+  int64_t x_tok, x_head, out_tok, out_head;
+  const int64_t *positions;
+  const float *cos, *sin;
+  int64_t max_pos;
+  int heads, n, k, rot_dim, rot_cols;
+} MvHeadLinearArgs;
+int mv_head_linear(const MvHeadLinearArgs *args, int n_tok, int dtype, void *stream);
+
+/* out[g] = the plane row of position start[s] + (g - cu[s]) of sequence s, for cu[s] <= g < cu[s + 1]; zeros where the table
+ * has no block. */
+int mv_latent_gather(const void *plane, int64_t num_blocks, int block_size, int cols, const int32_t *block_tables,
+                     int64_t table_stride, int table_width, const int32_t *cu, const int32_t *start, int n_seqs, int max_len,
+                     void *out, int dtype, void *stream);
+
+/* Decode: one query row per sequence against the cached rows themselves.  q [B][heads][kv_cols + rot_cols] (the query in the
+ * latent's coordinates | its rotated part), out [B][heads][kv_cols] = the softmax-weighted latents; dense rows.  Rows with
+ * context_lens <= 0 give zeros.  workspace: mv_latent_decode_workspace_bytes(). */
+size_t mv_latent_decode_workspace_bytes(int batch, int heads, int kv_cols, int rot_cols, int block_size, int max_blocks,
+                                        int window, int dtype);
+int mv_latent_decode(const void *q, const void *plane, const int32_t *block_tables, int64_t table_stride,
+                     const int32_t *context_lens, void *out, int batch, int heads, int kv_cols, int rot_cols,
+                     int block_size, int max_blocks, int64_t num_blocks, int window, float scale, void *workspace,
+                     size_t workspace_bytes, int dtype, int flags, void *stream);
+
+/* Prefill on expanded keys and values: queries of sequence s are rows cu_q[s] .. cu_q[s + 1], its keys rows cu_k[s] ..
+ * cu_k[s + 1] of k / v / rot, the last query aligned with the last key.  q [T] rows, head h at h * dq: [plain_cols | rotated
+ * part, not yet rotated]; k: head h at h * plain_cols; v: head h at h * dv; rot: rows of rot_cols, shared by the heads; out:
+ * head h at h * dv.  dq >= plain_cols + rot_cols, q is zero beyond its true columns. */
+typedef struct MvLatentPrefillArgs {
+  const void *q, *k, *v, *rot;
+  void *out;
+  int64_t q_stride, k_stride, v_stride, rot_stride, out_stride;
+  const int32_t *cu_q, *cu_k;
+  const int64_t *positions;
+  const float *cos, *sin;
+  int64_t max_pos;
+  int n_seqs, max_q, max_k, heads, plain_cols, rot_dim, rot_cols, dq, dv, window;
+  float scale;
+} MvLatentPrefillArgs;
+int mv_latent_prefill(const MvLatentPrefillArgs *args, int dtype, int flags, void *stream);
+
+/* ---- K15 — selective state space layer (heads of `p` columns, `groups` of state keys b and readers c of `n` elements).
+ * Recurrent state lives in slots: ssm_state fp32 [2][slots][heads][n][p], conv_state [2][slots][taps - 1][channels] of dtype.
+ * The state after an even / odd number of tokens is in half 0 / 1: a step reads the half of the tokens before it and writes
+ * that of the tokens behind it, so running the same single-token step again gives the same state.  A sequence whose first token has
+ * position 0 starts from zeros; slot < 0: starts from zeros, nothing is kept.  Channels: x [heads * p] | b [groups * n] |
+ * c [groups * n] at offsets 0, b_off, c_off; p % 16 == 0, n % 32 == 0 (padding holds zeros). */
+typedef struct MvSsmArgs {
+  const void *x;              /* [T] rows of channels at x_stride: projected (conv, step) or convolved (prefill) */
+  int64_t x_stride;
+  const void *dt;             /* [T] rows of heads, raw */
+  int64_t dt_stride;
+  const void *conv_w, *conv_b;      /* [taps][channels], [channels] */
+  const void *dt_bias, *a_log, *d;  /* [heads] */
+  void *conv_state;
+  float *ssm_state;
+  const int32_t *state_slots;       /* [n_seqs] */
+  const int32_t *cu_q, *cu_k;       /* prefill: token ranges; tokens before the step = key length - query length */
+  const int32_t *context_lens;      /* step: tokens including this one */
+  void *out;
+  int64_t out_stride;
+  int64_t slots;
+  int n_seqs, max_q, channels, taps, heads, groups, p, n, b_off, c_off;
+} MvSsmArgs;
+/* out[t] = silu(causal convolution of x + conv_b), [T][channels]; writes conv_state */
+int mv_causal_conv(const MvSsmArgs *args, int dtype, void *stream);
+/* out[t] = y, [T][heads * p], from convolved channels; writes ssm_state.  flags: MV_SSM_SCAN = token by token */
+enum { MV_SSM_SCAN = 1 };
+int mv_ssm_prefill(const MvSsmArgs *args, int dtype, int flags, void *stream);
+/* one token per sequence: convolution and recurrence in one launch, from projected channels; writes both states */
+int mv_ssm_step(const MvSsmArgs *args, int dtype, void *stream);
+/* out[t] = rms over each of `norm_groups` equal parts of (y * silu(z)) * w.  Rows are heads of p columns of which p_true
+ * count (parts are parts of the true columns). */
+int mv_gated_group_norm(const void *y, int64_t y_stride, const void *z, int64_t z_stride, const void *w, void *out,
+                        int64_t out_stride, int rows, int heads, int p, int p_true, int norm_groups, float eps, int dtype,
+                        void *stream);
 
 #ifdef __cplusplus
 }

@@ -138,11 +138,18 @@ __device__ __forceinline__ float gelu_tanh(float z) {
   return z / (1.0f + expf(-u2));
 }
 
-// act(gate) * up on the fp32 accumulators of a gated projection.  gelu: fp32 throughout.  silu: the rounding points of the
-// unfused pair (GEMM -> dtype, silu -> dtype, product in fp32; the caller rounds it)
+// clamped gate: g = min(gate, limit), u = clamp(up, -limit, limit): g sigmoid(alpha g) (u + 1)
+__device__ __forceinline__ float clamped_glu(float gate, float up, float limit, float alpha) {
+  const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+  return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
+}
+
+// act(gate) * up on the fp32 accumulators of a gated projection.  gelu, clamped: fp32 throughout.  silu: the rounding points
+// of the unfused pair (GEMM -> dtype, silu -> dtype, product in fp32; the caller rounds it)
 template <typename Tag>
-__device__ __forceinline__ float gated_act(float gate, float up, bool gelu) {
-  if (gelu) return __fmul_rn(gelu_tanh(gate), up);
+__device__ __forceinline__ float gated_act(float gate, float up, const MvGateAct &a) {
+  if (a.kind == MV_ACT_GELU) return __fmul_rn(gelu_tanh(gate), up);
+  if (a.kind == MV_ACT_CLAMPED) return clamped_glu(gate, up, a.limit, a.alpha);
   const float gt = elem<Tag>::ld(elem<Tag>::st(gate)), ut = elem<Tag>::ld(elem<Tag>::st(up));
   float sl = gt / (1.0f + expf(-gt));                        // rmsnorm.hip: silu_and_mul_kernel
   sl = elem<Tag>::ld(elem<Tag>::st(sl));
@@ -206,6 +213,11 @@ __device__ __forceinline__ void rot_apply(const float (&x)[VEC], const float (&c
 }
 
 // ---- host-side helpers ------------------------------------------------------
+static inline int mv_check_act(const MvGateAct *a) {
+  if (!a) return MV_E_NULLPTR;
+  if (a->kind < MV_ACT_SILU || a->kind > MV_ACT_CLAMPED) return MV_E_RANGE;
+  return a->kind == MV_ACT_CLAMPED && !(a->limit > 0.f) ? MV_E_RANGE : MV_OK;
+}
 static inline int mv_check_hip(hipError_t e) { return e == hipSuccess ? 0 : (int)e; }
 static inline bool mv_aligned16(const void *p) { return (((uintptr_t)p) & 15u) == 0; }
 

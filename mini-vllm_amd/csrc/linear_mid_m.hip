@@ -55,8 +55,8 @@ struct MidParams {
   int n_tiles, m_tiles;
   int kb_per_split;   // 64-element k-blocks per K split (blockIdx.y)
   int krot;           // rotate the K loop start per workgroup
-  int gelu;           // GATED: gelu (tanh form) instead of silu
   int ablate;         // bench only: bit 0 = no x DMA, bit 1 = no W DMA (the LDS slots keep whatever they hold)
+  MvGateAct act;      // GATED
 };
 
 template <int N>
@@ -330,7 +330,7 @@ __global__ void __launch_bounds__((WM * WN + NLX + NLW) * 64) linear_mid_m_kerne
         if (m < p.M && n < p.N) {
           float o[4];
 #pragma unroll
-          for (int e = 0; e < 4; ++e) o[e] = gated_act<Tag>(acc[a][b][e], acc[a + TN / 2][b][e], p.gelu != 0);
+          for (int e = 0; e < 4; ++e) o[e] = gated_act<Tag>(acc[a][b][e], acc[a + TN / 2][b][e], p.act);
           u32x2 pk;
           pk[0] = (uint32_t)elem<Tag>::st(o[0]) | ((uint32_t)elem<Tag>::st(o[1]) << 16);
           pk[1] = (uint32_t)elem<Tag>::st(o[2]) | ((uint32_t)elem<Tag>::st(o[3]) << 16);
@@ -533,7 +533,7 @@ extern "C" int mv_linear_mid_m(const void *x, int64_t x_stride, const void *w_pa
   if (flags) return MV_E_RANGE;
 #endif
   if (cfg == 0) cfg = auto_cfg(m, n, k, false);
-  MidParams p{x, w_packed, bias, out, x_stride, out_stride, m, n, k, 0, 0, 0, (flags & 2) ? 1 : 0, 0, flags >> 2};
+  MidParams p{x, w_packed, bias, out, x_stride, out_stride, m, n, k, 0, 0, 0, (flags & 2) ? 1 : 0, flags >> 2, {}};
   if ((flags & 16) && !bias) return MV_E_NULLPTR;
   if (flags & 1)
     return dtype == MV_BF16 ? launch_cfg<bf16_tag, EPI_INGEST>(p, cfg, 1, (hipStream_t)stream) : MV_E_DTYPE;
@@ -541,20 +541,27 @@ extern "C" int mv_linear_mid_m(const void *x, int64_t x_stride, const void *w_pa
                           : launch_cfg<f16_tag, EPI_PLAIN>(p, cfg, 1, (hipStream_t)stream);
 }
 
-extern "C" int mv_gate_up_silu_mid_m(const void *x, int64_t x_stride, const void *w_gate_up_packed, void *out,
-                                     int64_t out_stride, int m, int n_inter, int k, int dtype, int cfg,
-                                     void *stream) {
+extern "C" int mv_gated_act_mid_m(const void *x, int64_t x_stride, const void *w_gate_up_packed, void *out,
+                                  int64_t out_stride, int m, int n_inter, int k, const MvGateAct *act, int dtype, int cfg,
+                                  void *stream) {
   if (m == 0 || n_inter == 0) return MV_OK;
+  if (int e = mv_check_act(act)) return e;
   if (int e = check(x, x_stride, w_gate_up_packed, out, out_stride, m, n_inter, k, dtype)) return e;
   if (n_inter & 15) return MV_E_SHAPE;
-  const int gelu = (cfg & MV_GATE_GELU) ? 1 : 0;
-  cfg &= ~MV_GATE_GELU;
   if (cfg < 0 || cfg >= kNumCfgs) return MV_E_RANGE;
   if (cfg == 0) cfg = auto_cfg(m, n_inter, k, true);
   if (!kCfgs[cfg].gated_ok) return MV_E_RANGE;
-  MidParams p{x, w_gate_up_packed, nullptr, out, x_stride, out_stride, m, n_inter, k, 0, 0, 0, 0, gelu, 0};
+  MidParams p{x, w_gate_up_packed, nullptr, out, x_stride, out_stride, m, n_inter, k, 0, 0, 0, 0, 0, *act};
   return dtype == MV_BF16 ? launch_cfg<bf16_tag, EPI_GATED>(p, cfg, 1, (hipStream_t)stream)
                           : launch_cfg<f16_tag, EPI_GATED>(p, cfg, 1, (hipStream_t)stream);
+}
+
+extern "C" int mv_gate_up_silu_mid_m(const void *x, int64_t x_stride, const void *w_gate_up_packed, void *out,
+                                     int64_t out_stride, int m, int n_inter, int k, int dtype, int cfg,
+                                     void *stream) {
+  const MvGateAct act = {(cfg & MV_GATE_GELU) ? MV_ACT_GELU : MV_ACT_SILU, 0.f, 0.f};
+  return mv_gated_act_mid_m(x, x_stride, w_gate_up_packed, out, out_stride, m, n_inter, k, &act, dtype, cfg & ~MV_GATE_GELU,
+                            stream);
 }
 
 // fp32 partial sums of a K split: out_partial [splits][M][N] (row stride n), no bias, no rounding.
@@ -565,7 +572,7 @@ extern "C" int mv_linear_mid_m_partial(const void *x, int64_t x_stride, const vo
   if (!mv_aligned16(out_partial)) return MV_E_ALIGN;
   if (splits < 1 || splits > 16 || cfg < 0 || cfg >= kNumCfgs) return MV_E_RANGE;
   if (cfg == 0) cfg = auto_cfg(m, n * splits, k, false);
-  MidParams p{x, w_packed, nullptr, out_partial, x_stride, n, m, n, k, 0, 0, 0, 0, 0, 0};
+  MidParams p{x, w_packed, nullptr, out_partial, x_stride, n, m, n, k, 0, 0, 0, 0, 0, {}};
   return dtype == MV_BF16 ? launch_cfg<bf16_tag, EPI_PARTIAL>(p, cfg, splits, (hipStream_t)stream)
                           : launch_cfg<f16_tag, EPI_PARTIAL>(p, cfg, splits, (hipStream_t)stream);
 }

@@ -43,7 +43,7 @@ struct LinearParams {
   void *nres_out = nullptr;
   int64_t nres_stride = 0, nres_out_stride = 0;
   float eps = 0.f;
-  int gelu = 0;          // GATED: gelu (tanh form) instead of silu
+  MvGateAct act = {MV_ACT_SILU, 0.f, 0.f};   // GATED
   int norm_threads = 0;  // block size of the rmsnorm_kernel launch this prologue re-enacts
 };
 
@@ -348,7 +348,7 @@ linear_small_m_kernel(LinearParams p) {
     if constexpr (GATED) {
       const f32x4 up = tile_sum(t + RPW * MT);
 #pragma unroll
-      for (int i = 0; i < 4; ++i) o[i] = gated_act<Tag>(o[i], up[i], p.gelu != 0);
+      for (int i = 0; i < 4; ++i) o[i] = gated_act<Tag>(o[i], up[i], p.act);
     }
     if (m < p.M && n < p.N) {
       if (!GATED && p.bias) {
@@ -537,7 +537,7 @@ extern "C" int mv_gate_up_silu_small_m(const void *x, int64_t x_stride, const vo
   if (m == 0 || n_inter == 0) return MV_OK;
   if (int e = check(x, x_stride, w_gate_up, nullptr, out, out_stride, m, n_inter, k, dtype)) return e;
   LinearParams p{x, w_gate_up, nullptr, out, x_stride, out_stride, m, n_inter, k};
-  p.gelu = (shape & MV_GATE_GELU) ? 1 : 0;
+  p.act.kind = (shape & MV_GATE_GELU) ? MV_ACT_GELU : MV_ACT_SILU;
   return run<true>(p, dtype, shape, (hipStream_t)stream);
 }
 
@@ -560,8 +560,21 @@ extern "C" int mv_gate_up_silu_small_m_packed(const void *x, int64_t x_stride, c
   if (n_inter & 15) return MV_E_SHAPE;  // the up rows must start on a tile boundary of the packed copy
   if (int e = check(x, x_stride, w_gate_up_packed, nullptr, out, out_stride, m, n_inter, k, dtype)) return e;
   LinearParams p{x, w_gate_up_packed, nullptr, out, x_stride, out_stride, m, n_inter, k};
-  p.gelu = (shape & MV_GATE_GELU) ? 1 : 0;
+  p.act.kind = (shape & MV_GATE_GELU) ? MV_ACT_GELU : MV_ACT_SILU;
   return run<true, true>(p, dtype, shape, (hipStream_t)stream);
+}
+
+// ... with the activation and its constants as an argument; packed: w is the fragment-ordered copy
+extern "C" int mv_gated_act_small_m(const void *x, int64_t x_stride, const void *w_gate_up, int packed, void *out,
+                                    int64_t out_stride, int m, int n_inter, int k, const MvGateAct *act, int dtype, int shape,
+                                    void *stream) {
+  if (m == 0 || n_inter == 0) return MV_OK;
+  if (int e = mv_check_act(act)) return e;
+  if (packed && (n_inter & 15)) return MV_E_SHAPE;
+  if (int e = check(x, x_stride, w_gate_up, nullptr, out, out_stride, m, n_inter, k, dtype)) return e;
+  LinearParams p{x, w_gate_up, nullptr, out, x_stride, out_stride, m, n_inter, k};
+  p.act = *act;
+  return packed ? run<true, true>(p, dtype, shape, (hipStream_t)stream) : run<true>(p, dtype, shape, (hipStream_t)stream);
 }
 
 // The RMSNorm in front of a projection, folded into the projection's launch (<= 4 rows; see norm_prologue):

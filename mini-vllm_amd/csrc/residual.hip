@@ -1,6 +1,7 @@
 // K13 — steps of a 32-bit residual stream (models whose residual sum stays in fp32 whatever the activation dtype):
 //   mv_residual_update: one launch per edge of the stream — [start the row from a scaled embedding] + the output of the
-//     projections in front (plain, or RMS-normed by a weight of its own; or the fp32 partial sums of a K split)
+//     projections in front (plain, or RMS-normed by a weight of its own; or the fp32 partial sums of a K split; scaled by a
+//     vector and a number)
 //     [+ the scaled embedding] [+ a vector] -> the stream, and what the next projection reads: its RMSNorm or its cast;
 //   mv_gated_lookup: gelu(s) * a slice of a per-token table (the per-token layer input);
 //   mv_gated_lookup_linear: the same with the projection behind it, in one launch (decode-sized batches).
@@ -13,13 +14,14 @@ struct ResidualParams {
   float *x;                 // [rows][cols]
   const void *y;            // [rows] dtype rows (stride y_stride) or, y_splits > 0, fp32 [y_splits][rows][cols]
   const void *y_norm_w;     // RMS norm of y by a plain weight before it is added; NULL = y as it is
+  const void *y_scale;      // dtype [cols], multiplies y behind its norm; NULL = ones
   const void *embed;        // dtype [vocab][cols]
   const int64_t *ids;
   const void *vec;          // dtype [cols], added to every row
   const void *norm_w;       // out = rms(x) * (norm_offset + norm_w); NULL: out = x rounded to dtype
   void *out;
   int64_t y_stride, out_stride, vocab;
-  float embed_scale, norm_offset, eps;
+  float embed_scale, norm_offset, eps, y_mult;
   int y_splits, embed_mode; // embed_mode: 0 none, 1 the row starts from the embedding, 2 the embedding is added
   int rows, cols, cols_true;
 };
@@ -74,7 +76,7 @@ __global__ void __launch_bounds__(1024) residual_update_kernel(ResidualParams p)
   constexpr int VEC = elem<Tag>::VEC;
   __shared__ float red[2][16];
   const int row = blockIdx.x, nvec = p.cols / VEC;
-  float x[MAXV][VEC], y[MAXV][VEC], e[MAXV][VEC], vv[MAXV][VEC], wy[MAXV][VEC], wn[MAXV][VEC];
+  float x[MAXV][VEC], y[MAXV][VEC], e[MAXV][VEC], vv[MAXV][VEC], wy[MAXV][VEC], wn[MAXV][VEC], sy[MAXV][VEC];
   bool embed_ok = false;
   int64_t id = 0;
   if (p.embed_mode) {
@@ -86,7 +88,7 @@ __global__ void __launch_bounds__(1024) residual_update_kernel(ResidualParams p)
   for (int i = 0; i < MAXV; ++i) {
     const int c = (threadIdx.x + i * blockDim.x) * VEC;
 #pragma unroll
-    for (int j = 0; j < VEC; ++j) x[i][j] = y[i][j] = e[i][j] = vv[i][j] = wy[i][j] = wn[i][j] = 0.f;
+    for (int j = 0; j < VEC; ++j) x[i][j] = y[i][j] = e[i][j] = vv[i][j] = wy[i][j] = wn[i][j] = 0.f, sy[i][j] = 1.f;
     if (c < p.cols) {
       if (p.embed_mode != 1) load_f32<VEC>(p.x + (int64_t)row * p.cols + c, x[i]);
       if (p.y) {
@@ -103,6 +105,7 @@ __global__ void __launch_bounds__(1024) residual_update_kernel(ResidualParams p)
           load_row_vec<Tag>((const T *)p.y + (int64_t)row * p.y_stride + c, y[i]);
         }
         if (p.y_norm_w) load_row_vec<Tag>((const T *)p.y_norm_w + c, wy[i]);
+        if (p.y_scale) load_row_vec<Tag>((const T *)p.y_scale + c, sy[i]);
       }
       if (embed_ok) load_row_vec<Tag>((const T *)p.embed + id * p.cols + c, e[i]);
       if (p.vec) load_row_vec<Tag>((const T *)p.vec + c, vv[i]);
@@ -121,6 +124,12 @@ __global__ void __launch_bounds__(1024) residual_update_kernel(ResidualParams p)
     for (int i = 0; i < MAXV; ++i)
 #pragma unroll
       for (int j = 0; j < VEC; ++j) y[i][j] = y[i][j] * rs * wy[i][j];
+  }
+  if (p.y_scale || p.y_mult != 1.0f) {
+#pragma unroll
+    for (int i = 0; i < MAXV; ++i)
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) y[i][j] = y[i][j] * sy[i][j] * p.y_mult;
   }
   float ss = 0.f;
 #pragma unroll
@@ -291,10 +300,10 @@ extern "C" int mv_residual_update(const MvResidualArgs *a, int rows, int cols, i
   if (dtype != MV_BF16 && dtype != MV_F16 && dtype != MV_F32) return MV_E_DTYPE;
   if (a->embed_mode < 0 || a->embed_mode > 2) return MV_E_RANGE;
   if (a->embed_mode && (!a->embed || !a->ids || a->vocab <= 0)) return MV_E_NULLPTR;
-  if (a->y_norm_w && !a->y) return MV_E_NULLPTR;
+  if ((a->y_norm_w || a->y_scale) && !a->y) return MV_E_NULLPTR;
   const int vec = dtype == MV_F32 ? 4 : 8;
   if (cols % vec) return MV_E_SHAPE;
-  if (!mv_aligned16(a->x) || (a->y && !mv_aligned16(a->y)) || (a->y_norm_w && !mv_aligned16(a->y_norm_w)) ||
+  if (!mv_aligned16(a->x) || (a->y && !mv_aligned16(a->y)) || (a->y_norm_w && !mv_aligned16(a->y_norm_w)) || (a->y_scale && !mv_aligned16(a->y_scale)) ||
       (a->embed_mode && !mv_aligned16(a->embed)) || (a->vec && !mv_aligned16(a->vec)) ||
       (a->norm_w && !mv_aligned16(a->norm_w)) || (a->out && (!mv_aligned16(a->out) || a->out_stride % vec)) ||
       (a->y && a->y_splits == 0 && a->y_stride % vec))
@@ -302,6 +311,7 @@ extern "C" int mv_residual_update(const MvResidualArgs *a, int rows, int cols, i
   ResidualParams p;
   p.x = a->x, p.y = a->y, p.y_norm_w = a->y_norm_w, p.embed = a->embed, p.ids = a->ids, p.vec = a->vec;
   p.norm_w = a->norm_w, p.out = a->out, p.y_stride = a->y_stride, p.out_stride = a->out_stride, p.vocab = a->vocab;
+  p.y_scale = a->y_scale, p.y_mult = a->y_mult;
   p.embed_scale = a->embed_scale, p.norm_offset = a->norm_offset, p.eps = a->eps;
   p.y_splits = a->y_splits, p.embed_mode = a->embed_mode, p.rows = rows, p.cols = cols, p.cols_true = cols_true;
   const int nvec = cols / vec;

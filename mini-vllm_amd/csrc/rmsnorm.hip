@@ -202,14 +202,14 @@ extern "C" int mv_add_rmsnorm_partial(const float *partial, int splits, void *re
   return MV_OK;
 }
 
-// K9 — SiluAndMul (reference: minivllm/models/layers/activation.py:70-96) and, GELU, the tanh form of gelu in its place
-// (one rounding: gelu(x1) * x2 in fp32).
+// K9 — SiluAndMul (reference: minivllm/models/layers/activation.py:70-96) and, ACT, the tanh form of gelu or the clamped gate
+// in its place (fp32 inside, one rounding).
 // The reference rounds silu(x1) to the activation dtype before the multiply;
 // the same two rounding points are kept here.
-template <typename Tag, bool GELU>
+template <typename Tag, int ACT>
 __global__ void __launch_bounds__(256)
 silu_and_mul_kernel(const typename elem<Tag>::T *__restrict__ x, int64_t x_stride,
-                    typename elem<Tag>::T *__restrict__ out, int64_t out_stride, int rows, int cols) {
+                    typename elem<Tag>::T *__restrict__ out, int64_t out_stride, int rows, int cols, MvGateAct act) {
   constexpr int VEC = elem<Tag>::VEC;
   constexpr int U = 4;   // vectors per thread and trip: 2 U loads in flight before the first exp (prefill rows: 4.3 -> TB/s)
   const int nvec = cols / VEC;
@@ -239,8 +239,10 @@ silu_and_mul_kernel(const typename elem<Tag>::T *__restrict__ x, int64_t x_strid
           float y[VEC];
 #pragma unroll
           for (int j = 0; j < VEC; ++j) {
-            if constexpr (GELU) {
+            if constexpr (ACT == MV_ACT_GELU) {
               y[j] = __fmul_rn(gelu_tanh(a[u][j]), b[u][j]);
+            } else if constexpr (ACT == MV_ACT_CLAMPED) {
+              y[j] = clamped_glu(a[u][j], b[u][j], act.limit, act.alpha);
             } else {
               float s = a[u][j] / (1.0f + expf(-a[u][j]));
               s = elem<Tag>::ld(elem<Tag>::st(s));
@@ -254,9 +256,9 @@ silu_and_mul_kernel(const typename elem<Tag>::T *__restrict__ x, int64_t x_strid
   }
 }
 
-template <bool GELU>
+template <int ACT>
 static int act_and_mul(const void *x, int64_t x_stride, void *out, int64_t out_stride, int rows, int cols, int dtype,
-                       void *stream) {
+                       void *stream, MvGateAct act = {}) {
   if (rows == 0) return MV_OK;
   if (!x || !out) return MV_E_NULLPTR;
   if (rows < 0 || cols <= 0) return MV_E_SHAPE;
@@ -272,8 +274,8 @@ static int act_and_mul(const void *x, int64_t x_stride, void *out, int64_t out_s
     if (bx < 1) bx = 1;
     int by = rows < 65535 ? rows : 65535;
     while ((int64_t)bx * by > 16384 && by > 1) by = (by + 1) / 2;
-    hipLaunchKernelGGL((silu_and_mul_kernel<Tag, GELU>), dim3((unsigned)bx, (unsigned)by), dim3(256), 0,
-                       (hipStream_t)stream, (const T *)x, x_stride, (T *)out, out_stride, rows, cols);
+    hipLaunchKernelGGL((silu_and_mul_kernel<Tag, ACT>), dim3((unsigned)bx, (unsigned)by), dim3(256), 0,
+                       (hipStream_t)stream, (const T *)x, x_stride, (T *)out, out_stride, rows, cols, act);
   });
   MV_LAUNCH_CHECK();
   return MV_OK;
@@ -281,10 +283,19 @@ static int act_and_mul(const void *x, int64_t x_stride, void *out, int64_t out_s
 
 extern "C" int mv_silu_and_mul(const void *x, int64_t x_stride, void *out, int64_t out_stride,
                                int rows, int cols, int dtype, void *stream) {
-  return act_and_mul<false>(x, x_stride, out, out_stride, rows, cols, dtype, stream);
+  return act_and_mul<MV_ACT_SILU>(x, x_stride, out, out_stride, rows, cols, dtype, stream);
 }
 
 extern "C" int mv_gelu_and_mul(const void *x, int64_t x_stride, void *out, int64_t out_stride,
                                int rows, int cols, int dtype, void *stream) {
-  return act_and_mul<true>(x, x_stride, out, out_stride, rows, cols, dtype, stream);
+  return act_and_mul<MV_ACT_GELU>(x, x_stride, out, out_stride, rows, cols, dtype, stream);
+}
+
+extern "C" int mv_act_and_mul(const void *x, int64_t x_stride, void *out, int64_t out_stride, int rows, int cols,
+                              const MvGateAct *act, int dtype, void *stream) {
+  if (int e = mv_check_act(act)) return e;
+  if (act->kind == MV_ACT_CLAMPED)
+    return act_and_mul<MV_ACT_CLAMPED>(x, x_stride, out, out_stride, rows, cols, dtype, stream, *act);
+  return (act->kind == MV_ACT_GELU ? act_and_mul<MV_ACT_GELU> : act_and_mul<MV_ACT_SILU>)(x, x_stride, out, out_stride, rows,
+                                                                                        cols, dtype, stream, *act);
 }

@@ -19,6 +19,7 @@ from collections import deque
 import xxhash
 
 from .sequence import Sequence
+from .state_slots import StateSlots
 
 __all__ = ["Block", "BlockManager"]
 
@@ -45,7 +46,9 @@ class Block:
 
 
 class BlockManager:
-    def __init__(self, num_blocks: int, block_size: int) -> None:
+    def __init__(self, num_blocks: int, block_size: int, state_slots: int = 0) -> None:
+        """``state_slots`` > 0: the model has recurrent layers.  A sequence then also holds a state slot, and prompts share no
+        blocks: the state behind a shared prefix is not kept, so every token of a prompt has to be computed."""
         if num_blocks <= 0:
             raise ValueError(f"a block pool needs at least one block (num_blocks={num_blocks})")
         if block_size <= 0:
@@ -57,6 +60,7 @@ class BlockManager:
         self.free_block_ids: deque[int] = deque(range(num_blocks))
         self._free_set: set[int] = set(range(num_blocks))
         self.used_block_ids: set[int] = set()
+        self.states = StateSlots(state_slots) if state_slots else None
         self.stats = {"total_allocations": 0, "cache_hits": 0, "cache_misses": 0}
 
     # -- digests (block_manager.py:128-152) ---------------------------------------------------
@@ -115,6 +119,8 @@ class BlockManager:
 
     # -- prefill-time allocation (block_manager.py:252-344) -------------------------------------
     def can_allocate(self, sequence: Sequence) -> bool:
+        if self.states is not None and self.states.num_free == 0 and sequence.state_slot < 0:
+            return False
         return len(self._free_set) >= sequence.num_blocks
 
     def allocate(self, sequence: Sequence) -> None:
@@ -123,13 +129,15 @@ class BlockManager:
         if len(self._free_set) < sequence.num_blocks:
             raise ValueError(f"prompt needs {sequence.num_blocks} blocks, the pool has {len(self._free_set)} free "
                              f"(callers test can_allocate first)")
+        if self.states is not None:
+            self.states.take(sequence)
         chain = NO_HASH
         for i in range(sequence.num_blocks):
             tokens = sequence.block(i)
             full = len(tokens) == self.block_size
             chain = self.compute_hash(tokens, chain) if full else NO_HASH  # partial blocks break the chain
             hit_id = self.hash_to_block_id.get(chain, -1) if chain != NO_HASH else -1
-            hit = (chain != NO_HASH and 0 <= hit_id < self.num_blocks
+            hit = (self.states is None and chain != NO_HASH and 0 <= hit_id < self.num_blocks
                    and self.blocks[hit_id].token_ids == tokens)
             if hit:
                 self.stats["cache_hits"] += 1
@@ -160,6 +168,8 @@ class BlockManager:
         need = sequence.num_blocks - len(sequence.block_table)
         if need > len(self._free_set):
             raise RuntimeError(f"No free blocks available: {need} needed, {len(self._free_set)} free")
+        if self.states is not None:
+            self.states.take(sequence)
         for _ in range(need):
             block_id = self._get_any_free_block()
             self._take(block_id)
@@ -173,6 +183,8 @@ class BlockManager:
                 self._deallocate_block(block_id)
         sequence.num_cached_tokens = 0
         sequence.block_table.clear()
+        if self.states is not None:
+            self.states.release(sequence)
 
     # -- decode-time growth (block_manager.py:369-450) ------------------------------------------
     def can_append(self, sequence: Sequence) -> bool:

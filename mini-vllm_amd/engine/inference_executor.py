@@ -51,6 +51,16 @@ def kv_planes(model) -> list[tuple[int, int, int, int]]:
             if hasattr(m, "k_cache") and hasattr(m, "v_cache")]
 
 
+def latent_modules(model) -> list:
+    """Attention modules that own ONE plane of cached rows (``latent_cache``, ``row_cols`` elements a token), in cache order."""
+    return [m for m in model.modules() if hasattr(m, "latent_cache")]
+
+
+def state_modules(model) -> list:
+    """Modules with recurrent state: one slot per live sequence (``state_shapes``)."""
+    return [m for m in model.modules() if hasattr(m, "state_shapes")]
+
+
 def kv_block_bytes(num_layers: int, block_size: int, num_kv_heads_local: int, head_dim: int, itemsize: int) -> int:
     return 2 * num_layers * block_size * num_kv_heads_local * head_dim * itemsize
 
@@ -74,6 +84,10 @@ class InferenceExecutor:
             self.kv_shapes = []          # uniform: one [2, L, blocks, block_size, Hkv, D] tensor
             self.num_layers = len(planes) or self.num_layers
         self.attn_shapes = sorted({(h, hkv, d, c) for h, hkv, d, c in planes})
+        self.latents = latent_modules(model) if isinstance(model, torch.nn.Module) else []
+        self.state_modules = state_modules(model) if isinstance(model, torch.nn.Module) else []
+        self.span_windows = sorted({m.span_window for m in self.latents})
+        self._no_kv_planes = not planes and bool(self.latents or self.state_modules)
         try:
             self.dtype = next(model.parameters()).dtype
         except (StopIteration, AttributeError):
@@ -108,6 +122,8 @@ class InferenceExecutor:
         self._dev_slots = b_.pack_view(self._pack_dev, "slots")
         self._dev_ctx = b_.pack_view(self._pack_dev, "ctx")
         self._dev_rng = b_.pack_view(self._pack_dev, "rng")
+        self._dev_state = b_.pack_view(self._pack_dev, "state")
+        self._dev_state.fill_(-1)
         self._dev_tables = torch.full((ms, self.max_blocks_per_seq), -1, dtype=torch.int32, device=self.device)
         self._samp_rows = -1  # rows of the device sampling planes that are current (-1: stale)
         # speculative next-step replay (see _replay_graph): set by the engine when nothing is waiting
@@ -128,12 +144,23 @@ class InferenceExecutor:
 
     # ------------------------------------------------------------------ set-up
     def initialize(self, max_num_batched_tokens: int, max_num_seqs: int) -> None:
+        self._allocate_state()
         self._allocate_kv_cache()
         self._initialize_sampler()
         self._optimize_model()
         self._warmup_model(max_num_batched_tokens, max_num_seqs)
 
+    def _allocate_state(self) -> None:
+        """Recurrent state: max_num_seqs slots in every such module (before the KV pool, which takes what is left)."""
+        for m in self.state_modules:
+            for name, (shape, dtype) in m.state_shapes(self.dtype).items():
+                setattr(m, name, torch.empty((2, self.config.max_num_seqs, *shape), dtype=dtype, device=self.device))
+
     def _block_bytes(self) -> int:
+        rows = sum(m.row_cols for m in self.latents) * self.block_size * self.dtype.itemsize
+        return rows + (0 if self._no_kv_planes else self._kv_plane_bytes())
+
+    def _kv_plane_bytes(self) -> int:
         if self.kv_shapes:
             return sum(kv_block_bytes(1, self.block_size, hkv, d, self.dtype.itemsize) for hkv, d in self.kv_shapes)
         return kv_block_bytes(self.num_layers, self.block_size, self.num_kv_heads, self.head_dim, self.dtype.itemsize)
@@ -152,7 +179,7 @@ class InferenceExecutor:
             raise RuntimeError(f"Insufficient memory for KV cache allocation. Device: {self.device.type}, "
                                f"Available: {avail} bytes, Block size: {block_bytes} bytes")
         cap = cfg.max_num_seqs * self.max_blocks_per_seq
-        n = min(avail // block_bytes, cap)
+        n = min(avail // max(block_bytes, 1), cap)
         if get_tensor_parallel_world_size() > 1:
             # every rank runs the same scheduler: they must agree on the pool size
             import torch.distributed as dist
@@ -171,16 +198,19 @@ class InferenceExecutor:
             n = self._calculate_num_kv_blocks()
             self.config.num_kvcache_blocks = n  # the scheduler's BlockManager is sized from this
         shape = (2, self.num_layers, n, self.block_size, self.num_kv_heads, self.head_dim)
-        if self.kv_shapes:   # K plane, V plane of each module, one behind the other
-            shape = (n * self._block_bytes() // self.dtype.itemsize,)
+        if self._no_kv_planes:
+            shape = (0,)
+        elif self.kv_shapes:   # K plane, V plane of each module, one behind the other
+            shape = (n * self._kv_plane_bytes() // self.dtype.itemsize,)
         try:
             self.kv_cache = torch.empty(shape, device=self.device, dtype=self.dtype)
+            for m in self.latents:
+                m.latent_cache = torch.empty((n, self.block_size, m.row_cols), device=self.device, dtype=self.dtype)
         except torch.cuda.OutOfMemoryError as e:
             raise RuntimeError(f"OOM during KV cache allocation. Try reducing device_memory_utilization "
                                f"(current: {self.config.device_memory_utilization}) or max_num_seqs. Error: {e}") from e
         self._assign_kv_cache_to_layers()
-        logger.info("Allocated KV cache: %.2f GB (%d blocks x %d tokens)",
-                    self.kv_cache.numel() * self.kv_cache.element_size() / 2**30, n, self.block_size)
+        logger.info("Allocated KV cache: %.2f GB (%d blocks x %d tokens)", n * self._block_bytes() / 2**30, n, self.block_size)
 
     def _assign_kv_cache_to_layers(self) -> None:
         layer, at = 0, 0
@@ -194,7 +224,7 @@ class InferenceExecutor:
                     continue
                 module.k_cache, module.v_cache = self.kv_cache[0, layer], self.kv_cache[1, layer]
                 layer += 1
-        if layer == 0:
+        if layer == 0 and not self._no_kv_planes:
             logger.warning("No attention layers found with k_cache/v_cache attributes.")
 
     def _initialize_sampler(self) -> None:
@@ -340,18 +370,35 @@ class InferenceExecutor:
                     prefix_cached=any(s.num_cached_tokens > 0 for s in sequences),
                     decode_rows=inp.decode_rows, rest_cum_seqlens_q=self._to_dev(inp.rest_cum_seqlens_q),
                     rest_cum_seqlens_k=self._to_dev(inp.rest_cum_seqlens_k),
-                    rest_max_seqlen_q=inp.rest_max_seqlen_q, rest_max_seqlen_k=inp.rest_max_seqlen_k)
+                    rest_max_seqlen_q=inp.rest_max_seqlen_q, rest_max_seqlen_k=inp.rest_max_seqlen_k,
+                    state_slots=self._to_dev(inp.state_slots), key_spans=self._key_spans(sequences, inp.decode_rows))
         return self._to_dev(inp.input_ids), self._to_dev(inp.positions)
+
+    def _key_spans(self, sequences, decode_rows: int) -> dict | None:
+        """Context.key_spans of a step with cached tokens whose layers expand keys from cached rows."""
+        rest = sequences[decode_rows:]
+        if not self.latents or not rest or not any(s.num_cached_tokens > 0 for s in sequences):
+            return None
+        return {w: self._key_span(rest, w) for w in self.span_windows}
+
+    def _key_span(self, sequences, window: int):
+        first = [max(0, s.num_cached_tokens - window + 1) if window else 0 for s in sequences]
+        lens = [s.prefill_stop - f for s, f in zip(sequences, first)]
+        cu = [0]
+        for n in lens:
+            cu.append(cu[-1] + n)
+        both = torch.tensor(cu + first, dtype=torch.int32).to(self.device)
+        return both[:len(cu)], both[len(cu):], cu[-1], max(lens)
 
     def _ship_decode(self, inp: BatchInputs):
         b = inp.num_seqs
         if not inp.packed:  # oversize batch: one-off tensors (inference_executor.py:687-688)
             set_context(False, 0, 0, None, None, self._to_dev(inp.slot_mapping), self._to_dev(inp.context_lens),
-                        self._to_dev(inp.block_tables))
+                        self._to_dev(inp.block_tables), state_slots=self._to_dev(inp.state_slots))
             return self._to_dev(inp.input_ids), self._to_dev(inp.positions)
         self._pack_dev.copy_(self.builder.decode_pack, non_blocking=True)
         tables = self._ship_tables(inp)
-        set_context(False, 0, 0, None, None, self._dev_slots[:b], self._dev_ctx[:b], tables)
+        set_context(False, 0, 0, None, None, self._dev_slots[:b], self._dev_ctx[:b], tables, state_slots=self._dev_state[:b])
         return self._dev_ids[:b], self._dev_pos[:b]
 
     def _ship_tables(self, inp: BatchInputs):
@@ -543,7 +590,7 @@ class InferenceExecutor:
         gv = self.graph_vars = {
             "input_ids": self._dev_ids[:max_bs], "positions": self._dev_pos[:max_bs],
             "slot_mapping": self._dev_slots[:max_bs], "context_lens": self._dev_ctx[:max_bs],
-            "block_tables": self._dev_tables[:max_bs],
+            "block_tables": self._dev_tables[:max_bs], "state_slots": self._dev_state[:max_bs],
             "logits": torch.zeros((max_bs, vocab), dtype=self.dtype, device=dev),
             "logits_local": (torch.zeros((max_bs, vocab // self.tp_size), dtype=self.dtype, device=dev)
                              if self.tp_size > 1 else None),
@@ -555,9 +602,12 @@ class InferenceExecutor:
         heads = hf.num_attention_heads // get_tensor_parallel_world_size()
         # ... sized for every batch an EAGER step can carry too (max_num_seqs may exceed the largest graph bucket)
         shapes = self.attn_shapes or [(heads, self.num_kv_heads, self.head_dim, 0)]
-        hip_ops.workspace(max(hip_ops.paged_decode_workspace_bytes(bs, h, hkv, d, self.block_size, self.max_blocks_per_seq,
-                                                                   chunk=c)
-                              for bs in list(self.graph_bs) + [self.config.max_num_seqs] for h, hkv, d, c in shapes), dev)
+        batches = list(self.graph_bs) + [self.config.max_num_seqs]
+        latent = {(m.heads, m.kv_cols, m.rot_cols, m.window) for m in self.model.modules() if hasattr(m, "row_cols")}
+        hip_ops.workspace(max([hip_ops.paged_decode_workspace_bytes(bs, h, hkv, d, self.block_size, self.max_blocks_per_seq,
+                                                                    chunk=c) for bs in batches for h, hkv, d, c in shapes]
+                              + [hip_ops.latent_decode_workspace_bytes(bs, h, kv, r, self.block_size, self.max_blocks_per_seq, w,
+                                                                       self.dtype) for bs in batches for h, kv, r, w in latent]), dev)
         self._general_capture = "no" if not general_ok else "done"
         try:
             if self.tp_size > 1:   # the family without a backend collective inside (peer-to-peer kernels only)
@@ -615,6 +665,7 @@ class InferenceExecutor:
         gv = self.graph_vars
         gv["slot_mapping"].fill_(-1)
         gv["context_lens"].zero_()
+        gv["state_slots"].fill_(-1)
         gv["input_ids"].zero_()
         gv["positions"].zero_()
         torch.cuda.synchronize(self.device)
@@ -673,7 +724,7 @@ class InferenceExecutor:
         greedy = mode == "greedy"
         gv = self.graph_vars
         set_context(False, 0, 0, None, None, gv["slot_mapping"][:bs], gv["context_lens"][:bs],
-                    gv["block_tables"][:bs])
+                    gv["block_tables"][:bs], state_slots=gv["state_slots"][:bs])
         hidden = self.model(gv["input_ids"][:bs], gv["positions"][:bs])
         d = self._dev_samp_f32
         if greedy:  # TP > 1, every row at temperature 0: merge per-rank argmaxes, no logit gather

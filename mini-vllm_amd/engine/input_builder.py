@@ -10,6 +10,7 @@ Value and dtype contract (identical to the reference):
   input_ids, positions  int64 [T]          slot_mapping   int32 [T] or None
   cum_seqlens_q/k       int32 [n+1]        context_lens   int32 [B]
   block_tables          int32 [n, max blocks in batch], -1 padded, or None
+  state_slots           int32 [n]: Sequence.state_slot (not in the reference)
 """
 from __future__ import annotations
 
@@ -36,6 +37,7 @@ class BatchInputs:
     context_lens: torch.Tensor | None = None
     block_tables: torch.Tensor | None = None
     num_seqs: int = 0
+    state_slots: torch.Tensor | None = None
     # decode fast-path hints for the executor (values above are always complete and correct)
     packed: bool = False          # ids/positions/slots/context_lens are views of InputBuilder.decode_pack
     tables_dirty: bool = True     # block-table staging changed since the previous decode batch
@@ -59,31 +61,33 @@ class InputBuilder:
         # int64 plane: [input_ids | positions]; int32 plane: [slots | cu_q | cu_k / context_lens]
         self._i64 = self._alloc((2, cap_tok), torch.int64)
         self._slots = self._alloc((cap_tok,), torch.int32)
-        self._seq32 = self._alloc((5, max_num_seqs + 1), torch.int32)
+        self._seq32 = self._alloc((6, max_num_seqs + 1), torch.int32)
         self._tables = self._alloc((max_num_seqs, self.max_blocks_per_seq), torch.int32)
         self._np_i64 = self._i64.numpy()
         self._np_slots = self._slots.numpy()
         self._np_seq32 = self._seq32.numpy()
         self._np_tables = self._tables.numpy()
         # decode pack: ONE pinned buffer -> one H2D copy per step.
-        # layout (bytes): ids i64[ms] | positions i64[ms] | slots i32[ms] | context_lens i32[ms] | rng i64[2]
+        # layout (bytes): ids i64[ms] | positions i64[ms] | slots i32[ms] | context_lens i32[ms] | rng i64[2] | state slots i32[ms]
         ms = max_num_seqs
         self.pack_layout = {"ids": (0, ms * 8), "pos": (ms * 8, ms * 8), "slots": (ms * 16, ms * 4),
-                            "ctx": (ms * 20, ms * 4), "rng": (ms * 24, 16)}
-        self.pack_nbytes = ms * 24 + 16
+                            "ctx": (ms * 20, ms * 4), "rng": (ms * 24, 16), "state": (ms * 24 + 16, ms * 4)}
+        self.pack_nbytes = ms * 28 + 16
         self.decode_pack = torch.zeros(self.pack_nbytes, dtype=torch.uint8, pin_memory=self.pin)
         self._p_ids = self.pack_view(self.decode_pack, "ids")
         self._p_pos = self.pack_view(self.decode_pack, "pos")
         self._p_slots = self.pack_view(self.decode_pack, "slots")
         self._p_ctx = self.pack_view(self.decode_pack, "ctx")
         self.p_rng = self.pack_view(self.decode_pack, "rng")
+        self._p_state = self.pack_view(self.decode_pack, "state")
+        self._p_state.fill_(-1)
         self._last_batch: list | None = None   # decode batch whose block tables are in the staging buffer
         self._last_table_lens: list[int] = []
         self._last_width = -1
 
     def pack_view(self, buf: torch.Tensor, name: str) -> torch.Tensor:
         off, n = self.pack_layout[name]
-        return buf[off:off + n].view(torch.int32 if name in ("slots", "ctx") else torch.int64)
+        return buf[off:off + n].view(torch.int32 if name in ("slots", "ctx", "state") else torch.int64)
 
     def _alloc(self, shape, dtype) -> torch.Tensor:
         return torch.zeros(shape, dtype=dtype, pin_memory=self.pin)
@@ -132,7 +136,9 @@ class InputBuilder:
         tables = None
         if any(seq.block_table for seq in sequences):
             tables = self._tables_for(sequences, decode=False)
-        out = BatchInputs(True, out_ids, out_pos, max_q, max_k, cq, ck, slot_t, None, tables, n)
+        state = self._fit_seq32(5, n)
+        state.numpy()[:] = [seq.state_slot for seq in sequences]
+        out = BatchInputs(True, out_ids, out_pos, max_q, max_k, cq, ck, slot_t, None, tables, n, state_slots=state)
         # leading sequences that add exactly one token to a cached prefix are decode rows (mixed batches)
         nd = 0
         while nd < n and sequences[nd].block_table and sequences[nd].num_cached_tokens > 0 \
@@ -159,13 +165,15 @@ class InputBuilder:
         packed = b <= self.max_num_seqs
         if packed:
             ids, pos, slot_t, ctx = self._p_ids[:b], self._p_pos[:b], self._p_slots[:b], self._p_ctx[:b]
+            state = self._p_state[:b]
         else:
             ids, pos = self._fit_i64(0, b), self._fit_i64(1, b)
-            slot_t, ctx = self._fit_slots(b), self._fit_seq32(2, b)
+            slot_t, ctx, state = self._fit_slots(b), self._fit_seq32(2, b), self._fit_seq32(5, b)
         lens = np.fromiter((s.num_tokens for s in sequences), dtype=np.int64, count=b)
         ids.numpy()[:] = np.fromiter((s.last_token for s in sequences), dtype=np.int64, count=b)
         pos.numpy()[:] = lens - 1
         ctx.numpy()[:] = lens
+        state.numpy()[:] = np.fromiter((s.state_slot for s in sequences), dtype=np.int64, count=b)
         # slot of the token being written = last block * bs + (len-1) % bs  (== last_block_num_tokens - 1);
         # 0 without a table (warm-up)
         last_blk = np.fromiter((s.block_table[-1] if s.block_table else -1 for s in sequences),
@@ -174,13 +182,14 @@ class InputBuilder:
         if packed and pad_to is not None and pad_to > b:
             self._p_slots.numpy()[b:pad_to] = -1
             self._p_ctx.numpy()[b:pad_to] = 0
+            self._p_state.numpy()[b:pad_to] = -1
         last = self._last_batch
         same = (packed and last is not None and len(last) == b
                 and all(x is y for x, y in zip(sequences, last)))
         tables, dirty = self._tables_decode(sequences, same)
         self._last_batch = list(sequences) if packed else None
         return BatchInputs(False, ids, pos, 0, 0, None, None, slot_t, ctx, tables, b,
-                           packed=packed, tables_dirty=dirty, batch_changed=not same)
+                           state_slots=state, packed=packed, tables_dirty=dirty, batch_changed=not same)
 
     def _tables_decode(self, sequences: list[Sequence], same: bool):
         """Block tables of a decode batch; when the batch is the previous one, only rows whose table

@@ -31,7 +31,8 @@ class StepReplayer:
                              max_num_seqs=max_live, max_model_len=blocks * block_size,
                              max_num_batched_tokens=blocks * block_size, enforce_eager=True)
         self.runner = runner if runner is not None else ModelRunner(self.config, 0)
-        self.blocks = BlockManager(blocks, block_size)
+        self.blocks = BlockManager(blocks, block_size,
+                                   state_slots=max_live if getattr(self.config.hf_config, "recurrent_state", False) else 0)
         self.live: dict[str, Sequence] = {}
         self.vocab = self.config.hf_config.vocab_size
 

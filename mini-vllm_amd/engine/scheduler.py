@@ -34,7 +34,9 @@ class Scheduler:
         self.max_num_seqs = config.max_num_seqs
         self.max_num_batched_tokens = config.max_num_batched_tokens
         self.eos = config.eos
-        self.block_manager = BlockManager(config.num_kvcache_blocks, config.kvcache_block_size)
+        recurrent = getattr(getattr(config, "hf_config", None), "recurrent_state", False) is True
+        self.block_manager = BlockManager(config.num_kvcache_blocks, config.kvcache_block_size,
+                                          state_slots=config.max_num_seqs if recurrent else 0)
         # a sequence stops when it fills max_model_len -- or the whole KV pool (alone in it, it could only
         # preempt and re-prefill itself for ever)
         self.max_model_len = min(getattr(config, "max_model_len", None) or (1 << 62),

@@ -37,6 +37,7 @@ class Sequence:
         self.prefill_end: int | None = None
         self.block_table: list[int] = []
         self.block_size = block_size
+        self.state_slot = -1     # recurrent layers: where this sequence's state lives (engine/state_slots.py)
         self._adopt_sampling(sp)
 
     def _adopt_sampling(self, sp: SamplingParams) -> None:
@@ -117,11 +118,12 @@ class Sequence:
         payload = self.token_ids if self.num_completion_tokens == 0 else self.last_token
         return (self.num_tokens, self.num_prompt_tokens, self.num_cached_tokens, self.block_table,
                 self.block_size, payload, self.temperature, self.top_p, self.top_k, self.min_p,
-                self.max_tokens, self.ignore_eos, self.prefill_end)
+                self.max_tokens, self.ignore_eos, self.prefill_end, self.state_slot)
 
     def __setstate__(self, state) -> None:
         (self.num_tokens, self.num_prompt_tokens, self.num_cached_tokens, self.block_table,
-         self.block_size, payload, temperature, top_p, top_k, min_p, max_tokens, ignore_eos, prefill_end) = state
+         self.block_size, payload, temperature, top_p, top_k, min_p, max_tokens, ignore_eos, prefill_end,
+         self.state_slot) = state
         decoding = self.num_tokens - self.num_prompt_tokens > 0
         if isinstance(payload, int):
             if decoding:

@@ -19,11 +19,11 @@ import torch
 from torch import nn
 
 from .. import hip_ops
-from ..layers import Attention, ParallelLMHead, Segment, SegmentedLinear, get_rope
+from ..layers import Attention, ParallelLMHead, Segment, SegmentedLinear, get_rope, padded_parameter
 from ..layers.linear import MID_M_MAX, divide, gated_linear, pad_to
 from ..parallel_state import get_tensor_parallel_world_size
 from ..utils.context import get_context
-from ..utils.loader import load_weight, materialize
+from ..utils.loader import load_weight
 
 __all__ = ["MofaraxLayer", "MofaraxForCausalLM", "kernel_head_dim"]
 
@@ -39,20 +39,6 @@ def kernel_head_dim(dim: int) -> int:
     raise ValueError(f"head dims above 256 are not supported, got {dim}")
 
 
-def _padded(*shape: int) -> nn.Parameter:
-    """Zeros; a checkpoint tensor of the same rank fills the leading corner."""
-    p = nn.Parameter(torch.zeros(*shape))
-
-    def load(param, tensor, *args, **kwargs):
-        t = materialize(tensor)
-        if t.dim() != param.dim() or any(a > b for a, b in zip(t.shape, param.shape)):
-            raise ValueError(f"cannot place {tuple(t.shape)} in {tuple(param.shape)}")
-        param.data[tuple(slice(0, n) for n in t.shape)].copy_(t)
-
-    p.weight_loader = load
-    return p
-
-
 class SideInput(nn.Module):
     """gelu(W_gate x) * e[token], projected back to the stream's width (its RMS norm rides in the residual update)."""
 
@@ -61,7 +47,7 @@ class SideInput(nn.Module):
         self.dim, self.offset = dim, offset
         self.gate = SegmentedLinear(width, [Segment("gate", dim)], split="none")
         self.proj = SegmentedLinear(dim, [Segment("proj", width)], split="none")
-        self.norm = _padded(pad_to(width))
+        self.norm = padded_parameter(pad_to(width))
 
     def forward(self, x, ids, table):
         packed, n = self.proj.weight_packed, self.proj.weight.shape[0]
@@ -78,7 +64,7 @@ class MofaraxLayer(nn.Module):
         a, width = spec.attention, config.hidden_size
         self.heads, self.kv_heads, self.ff = divide(a.heads, tp), divide(a.kv_heads, tp), spec.ff
         self.head_dim = d = kernel_head_dim(a.dim)
-        self.norm1 = _padded(pad_to(width))
+        self.norm1 = padded_parameter(pad_to(width))
         rows = [Segment("o", a.heads, a.dim, d)]
         self.qk = SegmentedLinear(width, [Segment("q", a.heads, a.dim, d), Segment("k", a.kv_heads, a.dim, d)], split="out")
         if spec.ff:
@@ -137,15 +123,15 @@ class MofaraxForCausalLM(nn.Module):
         self.config = config
         w = pad_to(config.hidden_size)
         self.runs = config.layer_runs()
-        self.embed = _padded(config.vocab_size, w)
-        self.loop_step = _padded(config.loop[2], w) if config.loop else None
-        self.side_embed = _padded(config.vocab_size, config.side_dim * len(config.layers)) if config.side_dim else None
+        self.embed = padded_parameter(config.vocab_size, w)
+        self.loop_step = padded_parameter(config.loop[2], w) if config.loop else None
+        self.side_embed = padded_parameter(config.vocab_size, config.side_dim * len(config.layers)) if config.side_dim else None
         self.stack = []
         for i in range(len(config.layers)):
             layer = MofaraxLayer(config, i, 1 + max(t for j, t, _ in self.runs if j == i))
             self.add_module(f"l{i}", layer)
             self.stack.append(layer)
-        self.final_norm = _padded(w)
+        self.final_norm = padded_parameter(w)
         self.head = ParallelLMHead(config.vocab_size, config.hidden_size, storage_dim=w)
 
     # ---- the residual stream between two layer runs -------------------------------------------------------------------

@@ -2,14 +2,15 @@
 it is in none of the benchmark configurations."""
 from typing import Any
 
+from .kugulorn import KugulornForCausalLM
 from .mofarax import MofaraxForCausalLM
 from .opt import OPTForCausalLM
 from .qwen import Qwen2ForCausalLM, Qwen3ForCausalLM
 
 SUPPORTED_MODELS = {"Qwen2ForCausalLM": Qwen2ForCausalLM, "Qwen3ForCausalLM": Qwen3ForCausalLM,
-                    "OPTForCausalLM": OPTForCausalLM, "Mofarax": MofaraxForCausalLM}
+                    "OPTForCausalLM": OPTForCausalLM, "Mofarax": MofaraxForCausalLM, "Kugulorn": KugulornForCausalLM}
 TYPE_TO_ARCH = {"qwen2": "Qwen2ForCausalLM", "qwen3": "Qwen3ForCausalLM", "opt": "OPTForCausalLM",
-                "mofarax": "Mofarax"}
+                "mofarax": "Mofarax", "kugulorn": "Kugulorn"}
 
 
 def create_model(hf_config: Any) -> Any:

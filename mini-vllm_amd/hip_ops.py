@@ -75,6 +75,24 @@ _SIGNATURES = {
                                 c_int, c_int, c_int, c_void_p]),
     "mv_gated_lookup_linear": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int64, c_int, c_void_p, c_void_p, c_void_p,
                                        c_int64, c_int, c_int, c_int, c_int, c_int, c_void_p]),
+    "mv_act_and_mul": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int, c_int, c_void_p, c_int, c_void_p]),
+    "mv_latent_prep": (c_int, [c_void_p, c_int, c_int, c_void_p]),
+    "mv_head_linear": (c_int, [c_void_p, c_int, c_int, c_void_p]),
+    "mv_latent_gather": (c_int, [c_void_p, c_int64, c_int, c_int, c_void_p, c_int64, c_int, c_void_p, c_void_p, c_int, c_int,
+                                 c_void_p, c_int, c_void_p]),
+    "mv_latent_decode_workspace_bytes": (c_size_t, [c_int] * 8),
+    "mv_latent_decode": (c_int, [c_void_p, c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int,
+                                 c_int, c_int64, c_int, c_float, c_void_p, c_size_t, c_int, c_int, c_void_p]),
+    "mv_latent_prefill": (c_int, [c_void_p, c_int, c_int, c_void_p]),
+    "mv_causal_conv": (c_int, [c_void_p, c_int, c_void_p]),
+    "mv_ssm_prefill": (c_int, [c_void_p, c_int, c_int, c_void_p]),
+    "mv_ssm_step": (c_int, [c_void_p, c_int, c_void_p]),
+    "mv_gated_group_norm": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_int, c_int, c_int,
+                                    c_int, c_float, c_int, c_void_p]),
+    "mv_gated_act_small_m": (c_int, [c_void_p, c_int64, c_void_p, c_int, c_void_p, c_int64, c_int, c_int, c_int, c_void_p,
+                                     c_int, c_int, c_void_p]),
+    "mv_gated_act_mid_m": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_int, c_int, c_void_p, c_int, c_int,
+                                   c_void_p]),
     "mv_linear_small_m": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_int, c_int,
                                   c_int, c_int, c_int, c_void_p]),
     "mv_gate_up_silu_small_m": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_int, c_int,
@@ -145,7 +163,39 @@ class MvResidualArgs(ctypes.Structure):
     _fields_ = [("x", c_void_p), ("y", c_void_p), ("y_norm_w", c_void_p), ("embed", c_void_p), ("ids", c_void_p),
                 ("vec", c_void_p), ("norm_w", c_void_p), ("out", c_void_p), ("y_stride", c_int64), ("out_stride", c_int64),
                 ("vocab", c_int64), ("embed_scale", c_float), ("norm_offset", c_float), ("eps", c_float),
-                ("y_splits", c_int), ("embed_mode", c_int)]
+                ("y_splits", c_int), ("embed_mode", c_int), ("y_mult", c_float), ("y_scale", c_void_p)]
+
+
+class GateAct(ctypes.Structure):
+    """Activation of a gated projection with its constants (include/mvhip.h: MvGateAct)."""
+    _fields_ = [("kind", c_int), ("limit", c_float), ("alpha", c_float)]
+
+
+def clamped_glu(limit: float, alpha: float = 1.702) -> GateAct:
+    """g = min(gate, limit), u = clamp(up, -limit, limit): g * sigmoid(alpha * g) * (u + 1)."""
+    return GateAct(2, float(limit), float(alpha))
+
+
+def _struct(name: str, **fields):
+    return type(name, (ctypes.Structure,), {"_fields_": [(f, t) for k, t in fields.items() for f in k.split("__")]})
+
+
+# include/mvhip.h, field for field
+MvLatentPrepArgs = _struct(
+    "MvLatentPrepArgs", z=c_void_p, z_stride=c_int64, q_norm_w__kv_norm_w__q_out=c_void_p, q_out_stride=c_int64,
+    rows_out__plane__slot_mapping=c_void_p, num_slots=c_int64, positions__cos__sin=c_void_p, max_pos=c_int64,
+    q_off__q_rank__q_cols__kv_off__kv_rank__kv_cols__rot_off__rot_dim__rot_cols=c_int, eps=c_float)
+MvHeadLinearArgs = _struct(
+    "MvHeadLinearArgs", x__w__out=c_void_p, x_tok__x_head__out_tok__out_head=c_int64, positions__cos__sin=c_void_p,
+    max_pos=c_int64, heads__n__k__rot_dim__rot_cols=c_int)
+MvLatentPrefillArgs = _struct(
+    "MvLatentPrefillArgs", q__k__v__rot__out=c_void_p, q_stride__k_stride__v_stride__rot_stride__out_stride=c_int64,
+    cu_q__cu_k__positions__cos__sin=c_void_p, max_pos=c_int64,
+    n_seqs__max_q__max_k__heads__plain_cols__rot_dim__rot_cols__dq__dv__window=c_int, scale=c_float)
+MvSsmArgs = _struct(
+    "MvSsmArgs", x=c_void_p, x_stride=c_int64, dt=c_void_p, dt_stride=c_int64,
+    conv_w__conv_b__dt_bias__a_log__d__conv_state__ssm_state__state_slots__cu_q__cu_k__context_lens__out=c_void_p,
+    out_stride__slots=c_int64, n_seqs__max_q__channels__taps__heads__groups__p__n__b_off__c_off=c_int)
 
 
 def _attn_opts(interleaved_pairs=None, chunk: int = 0, out=None):
@@ -566,15 +616,29 @@ def gelu_and_mul(x, out=None):
     return out
 
 
+def act_and_mul(x, act, out=None):
+    """x [rows, 2 * cols] (row-strided view ok) -> act(x[:, :cols], x[:, cols:]); ``act``: "silu", "gelu_tanh" or a GateAct."""
+    if not isinstance(act, GateAct):
+        return (silu_and_mul if act == "silu" else gelu_and_mul)(x, out=out)
+    _need_cuda(x)
+    if x.dim() != 2 or x.stride(1) != 1 or x.shape[1] % 2:
+        raise ValueError(f"act_and_mul wants [rows, 2 * cols] rows, got {tuple(x.shape)}")
+    rows, cols = x.shape[0], x.shape[1] // 2
+    out = _gated_out(out, rows, cols, x)
+    _check(_lib.mv_act_and_mul(x.data_ptr(), x.stride(0), out.data_ptr(), out.stride(0), rows, cols, ctypes.byref(act), _dt(x),
+                               _stream()), "mv_act_and_mul")
+    return out
+
+
 # ---------------------------------------------------------------- K13
 def residual_update(x, y=None, y_norm_w=None, embed=None, ids=None, embed_scale: float = 1.0, start: bool = False,
                     vec=None, norm_w=None, norm_offset: float = 0.0, eps: float = 0.0, cols_true: int | None = None,
-                    out=None, want_out: bool = True, dtype=None):
+                    out=None, want_out: bool = True, dtype=None, y_scale=None, y_mult: float = 1.0):
     """One edge of the fp32 residual stream ``x`` [rows, cols] (updated in place; include/mvhip.h: mv_residual_update).
     ``y``: [rows, cols] of the activation dtype, or fp32 K-split partial sums [splits, rows, cols]; ``y_norm_w``: its RMS
-    norm.  ``embed`` / ``ids``: the scaled embedding is added (``start``: the row starts from it).  ``vec``: added to every
+    norm; ``y_scale`` (a vector) and ``y_mult`` multiply it.  ``embed`` / ``ids``: the scaled embedding is added (``start``: the row starts from it).  ``vec``: added to every
     row.  Returns rms(x) * (norm_offset + norm_w), or x cast to ``dtype`` when norm_w is None; None if not want_out."""
-    _need_cuda(x, y, y_norm_w, embed, ids, vec, norm_w)
+    _need_cuda(x, y, y_norm_w, embed, ids, vec, norm_w, y_scale)
     rows, cols = x.shape
     if x.dtype != torch.float32 or not x.is_contiguous():
         raise MvHipError("the residual stream must be a dense fp32 [rows, cols] tensor")
@@ -587,7 +651,7 @@ def residual_update(x, y=None, y_norm_w=None, embed=None, ids=None, embed_scale:
                 raise MvHipError("partial sums must be dense fp32 [splits, rows, cols]")
         elif tuple(y.shape) != (rows, cols) or y.dtype != dt or y.stride(1) != 1:
             raise MvHipError(f"y must be [{rows}, {cols}] of {dt}")
-    for name, w in (("y_norm_w", y_norm_w), ("vec", vec), ("norm_w", norm_w)):
+    for name, w in (("y_norm_w", y_norm_w), ("y_scale", y_scale), ("vec", vec), ("norm_w", norm_w)):
         if w is not None and (w.dtype != dt or w.numel() != cols or not w.is_contiguous()):
             raise MvHipError(f"{name} must be [{cols}] of {dt}")
     if embed is not None and (embed.dtype != dt or embed.shape[1] != cols or not embed.is_contiguous()
@@ -603,7 +667,7 @@ def residual_update(x, y=None, y_norm_w=None, embed=None, ids=None, embed_scale:
                        _ptr(vec), _ptr(norm_w), _ptr(out), y.stride(0) if y is not None and splits == 0 else 0,
                        out.stride(0) if out is not None else 0, embed.shape[0] if embed is not None else 0,
                        float(embed_scale), float(norm_offset), float(eps), splits,
-                       0 if embed is None else (1 if start else 2))
+                       0 if embed is None else (1 if start else 2), float(y_mult), _ptr(y_scale))
     _check(_lib.mv_residual_update(ctypes.byref(a), rows, cols, cols if cols_true is None else int(cols_true), _DTYPES[dt],
                                    _stream()), "mv_residual_update")
     return out
@@ -711,6 +775,12 @@ def gate_up_silu_small_m(x, weight, shape: int = 0, packed=None, act: str = "sil
         raise ValueError(f"weight {tuple(weight.shape)} is not a merged [2I, {k}] gate_up matrix")
     n = weight.shape[0] // 2
     given, out = out, _gated_out(out, x2.shape[0], n, x)
+    if isinstance(act, GateAct):
+        use = n % 16 == 0 and _packed_ok(packed, 2 * n, k, x.dtype)
+        _check(_lib.mv_gated_act_small_m(x2.data_ptr(), x2.stride(0), (packed if use else weight).data_ptr(), int(use),
+                                         out.data_ptr(), out.stride(0), x2.shape[0], n, k, ctypes.byref(act), _dt(x), int(shape),
+                                         _stream()), "mv_gated_act_small_m")
+        return out if given is not None else out.view(*x.shape[:-1], n)
     shape = int(shape) | GATE_ACTS[act]
     if n % 16 == 0 and _packed_ok(packed, 2 * n, k, x.dtype):
         _check(_lib.mv_gate_up_silu_small_m_packed(x2.data_ptr(), x2.stride(0), packed.data_ptr(), out.data_ptr(),
@@ -818,6 +888,11 @@ def gate_up_silu_mid_m(x, w_packed, n_inter: int, cfg: int = 0, act: str = "silu
     if w_packed.numel() != 2 * n_inter * k or n_inter % 16:
         raise ValueError(f"packed weight of {w_packed.numel()} elements is not a merged [2*{n_inter}, {k}] matrix")
     given, out = out, _gated_out(out, x2.shape[0], n_inter, x)
+    if isinstance(act, GateAct):
+        _check(_lib.mv_gated_act_mid_m(x2.data_ptr(), x2.stride(0), w_packed.data_ptr(), out.data_ptr(), out.stride(0),
+                                       x2.shape[0], n_inter, k, ctypes.byref(act), _dt(x), int(cfg), _stream()),
+               "mv_gated_act_mid_m")
+        return out if given is not None else out.view(*x.shape[:-1], n_inter)
     _check(_lib.mv_gate_up_silu_mid_m(x2.data_ptr(), x2.stride(0), w_packed.data_ptr(), out.data_ptr(),
                                       out.stride(0), x2.shape[0], n_inter, k, _dt(x), int(cfg) | GATE_ACTS[act], _stream()),
            "mv_gate_up_silu_mid_m")
@@ -1028,3 +1103,222 @@ def decode_advance(input_ids, tokens, positions, slot_mapping, context_lens, rng
     _check(_lib.mv_decode_advance(input_ids.data_ptr(), tokens.data_ptr(), positions.data_ptr(),
                                   slot_mapping.data_ptr(), context_lens.data_ptr(), _ptr(rng_offset),
                                   input_ids.shape[0], _stream()), "mv_decode_advance")
+
+
+# ---------------------------------------------------------------- K14
+MV_LATENT_SIMPLE = 1
+
+
+def _rows_ok(what: str, t, cols: int, dtype=None) -> None:
+    if t.dim() != 2 or t.stride(1) != 1 or t.shape[1] < cols or (dtype is not None and t.dtype != dtype):
+        raise MvHipError(f"{what}: rows of at least {cols} elements of {dtype} required, got {tuple(t.shape)} {t.dtype}")
+
+
+def _tables_ok(positions, cos, sin, n_tok: int, pairs: int) -> None:
+    if positions.dtype != torch.int64 or positions.numel() != n_tok or not positions.is_contiguous():
+        raise MvHipError(f"int64 positions of {n_tok} tokens required")
+    for t in (cos, sin):
+        if t.dtype != torch.float32 or t.dim() != 2 or t.shape[1] != pairs or not t.is_contiguous():
+            raise MvHipError(f"cos / sin must be dense fp32 [max_pos, {pairs}]")
+
+
+def latent_prep(z, q_norm_w, q_off: int, q_rank: int, eps: float, kv=None, positions=None, cos=None, sin=None, plane=None,
+                slot_mapping=None, want_rows: bool = False):
+    """Merged down projection ``z`` -> (normed query latent [T, q_cols], cached rows [T, kv_cols + rot_cols] or None).  ``kv``:
+    None (the layer has no latent of its own), or (norm weight, kv_off, kv_rank, rot_off, rot_dim, rot_cols); the rows also go to
+    ``plane`` [..., kv_cols + rot_cols] at ``slot_mapping``."""
+    _need_cuda(z, q_norm_w, plane, slot_mapping)
+    t, q_cols = z.shape[0], q_norm_w.numel()
+    _rows_ok("z", z, q_off + q_cols)
+    out = torch.empty((t, q_cols), dtype=z.dtype, device=z.device)
+    a = MvLatentPrepArgs(z=z.data_ptr(), z_stride=z.stride(0), q_norm_w=q_norm_w.data_ptr(), q_out=out.data_ptr(),
+                         q_out_stride=q_cols, q_off=q_off, q_rank=q_rank, q_cols=q_cols, eps=eps)
+    rows = None
+    if kv is not None:
+        w, kv_off, kv_rank, rot_off, rot_dim, rot_cols = kv
+        _rows_ok("z", z, max(kv_off + w.numel(), rot_off + rot_cols))
+        _tables_ok(positions, cos, sin, t, rot_dim // 2)
+        cols = w.numel() + rot_cols
+        if want_rows:
+            rows = torch.empty((t, cols), dtype=z.dtype, device=z.device)
+        a.kv_norm_w, a.kv_off, a.kv_rank, a.kv_cols = w.data_ptr(), kv_off, kv_rank, w.numel()
+        a.rot_off, a.rot_dim, a.rot_cols = rot_off, rot_dim, rot_cols
+        a.positions, a.cos, a.sin, a.max_pos = positions.data_ptr(), cos.data_ptr(), sin.data_ptr(), cos.shape[0]
+        a.rows_out = _ptr(rows)
+        if plane is not None and slot_mapping is not None and plane.numel():
+            if plane.dtype != z.dtype or plane.shape[-1] != cols or not plane.is_contiguous() or slot_mapping.numel() != t:
+                raise MvHipError(f"latent plane: dense rows of {cols} {z.dtype} and a slot per token required")
+            slots = _i32(slot_mapping)
+            a.plane, a.slot_mapping, a.num_slots = plane.data_ptr(), slots.data_ptr(), plane.numel() // cols
+    _check(_lib.mv_latent_prep(ctypes.byref(a), t, _dt(z), _stream()), "mv_latent_prep")
+    return out, rows
+
+
+def head_linear(x, w, out, rot=None):
+    """out[t, h, :n] = w[h] x[t, h, :k] for x [T, H, >= k], w [H, n, k], out [T, H, >= n]; ``rot`` (rot_dim, rot_cols, positions,
+    cos, sin): also out[t, h, n : n + rot_cols] = the rotated x[t, h, k : k + rot_dim]."""
+    _need_cuda(x, w, out)
+    t, h, n, k = x.shape[0], *w.shape
+    rot_cols = rot[1] if rot else 0
+    if (not w.is_contiguous() or w.dtype != x.dtype or out.dtype != x.dtype or x.shape[1] != h or tuple(out.shape[:2]) != (t, h)
+            or x.shape[2] < k + rot_cols or out.shape[2] < n + rot_cols or x.stride(2) != 1 or out.stride(2) != 1):
+        raise MvHipError(f"head_linear: {tuple(x.shape)} x {tuple(w.shape)} -> {tuple(out.shape)} does not fit")
+    a = MvHeadLinearArgs(x=x.data_ptr(), w=w.data_ptr(), out=out.data_ptr(), x_tok=x.stride(0), x_head=x.stride(1),
+                         out_tok=out.stride(0), out_head=out.stride(1), heads=h, n=n, k=k)
+    if rot:
+        rot_dim, _, positions, cos, sin = rot
+        _tables_ok(positions, cos, sin, t, rot_dim // 2)
+        a.positions, a.cos, a.sin, a.max_pos = positions.data_ptr(), cos.data_ptr(), sin.data_ptr(), cos.shape[0]
+        a.rot_dim, a.rot_cols = rot_dim, rot_cols
+    _check(_lib.mv_head_linear(ctypes.byref(a), t, _dt(x), _stream()), "mv_head_linear")
+    return out
+
+
+def latent_gather(plane, block_tables, cu, start, total: int, max_len: int):
+    """Rows of ``plane`` [blocks, block_size, cols]: positions start[s] .. of sequence s at cu[s] .. cu[s + 1] of [total, cols]."""
+    _need_cuda(plane, block_tables, cu, start)
+    cols = plane.shape[2]
+    out = torch.empty((total, cols), dtype=plane.dtype, device=plane.device)
+    bt = _i32(block_tables)
+    if bt.stride(1) != 1 or bt.shape[0] != start.numel() or cu.numel() != start.numel() + 1:
+        raise MvHipError("block tables [sequences, blocks], one start per sequence and cumulative lengths required")
+    _check(_lib.mv_latent_gather(plane.data_ptr(), plane.shape[0], plane.shape[1], cols, bt.data_ptr(), bt.stride(0), bt.shape[1],
+                                 cu.data_ptr(), start.data_ptr(), bt.shape[0], int(max_len), out.data_ptr(), _dt(plane),
+                                 _stream()), "mv_latent_gather")
+    return out
+
+
+def latent_decode_workspace_bytes(batch, heads, kv_cols, rot_cols, block_size, max_blocks, window, dtype) -> int:
+    return int(_lib.mv_latent_decode_workspace_bytes(int(batch), int(heads), int(kv_cols), int(rot_cols), int(block_size),
+                                                     int(max_blocks), int(window), _DTYPES[dtype]))
+
+
+def latent_decode(q, plane, block_tables, context_lens, kv_cols: int, scale: float, window: int = 0, flags: int = 0):
+    """q [B, H, kv_cols + rot_cols] (latent coordinates | rotated part) against the cached rows -> latents [B, H, kv_cols]."""
+    _need_cuda(q, plane, block_tables, context_lens)
+    b, h, cols = q.shape
+    if not q.is_contiguous() or plane.dtype != q.dtype or plane.shape[-1] != cols or not plane.is_contiguous():
+        raise MvHipError(f"latent_decode: dense q [B, H, {cols}] and a plane of such rows required")
+    bt, cl = _i32(block_tables), _i32(context_lens)
+    if bt.shape[1] and bt.stride(1) != 1 or bt.shape[0] != b or cl.numel() != b:
+        raise MvHipError("latent_decode: one block table and one length per row required")
+    out = torch.empty((b, h, kv_cols), dtype=q.dtype, device=q.device)
+    nb, bs, rot_cols = plane.shape[0], plane.shape[1], cols - kv_cols
+    ws = workspace(latent_decode_workspace_bytes(b, h, kv_cols, rot_cols, bs, bt.shape[1], window, q.dtype), q.device)
+    _check(_lib.mv_latent_decode(q.data_ptr(), plane.data_ptr(), bt.data_ptr(), bt.stride(0) if bt.shape[1] else 0, cl.data_ptr(),
+                                 out.data_ptr(), b, h, kv_cols, rot_cols, bs, bt.shape[1], nb, int(window), float(scale),
+                                 ws.data_ptr(), ws.numel(), _dt(q), int(flags), _stream()), "mv_latent_decode")
+    return out
+
+
+def latent_prefill(q, k, v, rot, cu_q, cu_k, max_q: int, max_k: int, positions, cos, sin, rot_dim: int, scale: float,
+                   window: int = 0, out=None, flags: int = 0):
+    """q [T, H, dq] ([plain | rotated part, not yet rotated]), k [G, H, plain], v [G, H, dv], rot [G, rot_cols] -> [T, H, dv]."""
+    _need_cuda(q, k, v, rot, cu_q, cu_k, positions)
+    t, h, dq = q.shape
+    dp, dv = k.shape[2], v.shape[2]
+    for x, d in ((q, dq), (k, dp), (v, dv)):
+        if x.shape[1] != h or x.stride(2) != 1 or x.stride(1) != d or x.dtype != q.dtype:
+            raise MvHipError("latent_prefill: heads must lie side by side in the rows of q, k and v")
+    _rows_ok("rot", rot, 1, q.dtype)
+    _tables_ok(positions, cos, sin, t, rot_dim // 2)
+    if out is None:
+        out = torch.empty((t, h, dv), dtype=q.dtype, device=q.device)
+    _out_rows(out, t, h, dv)
+    a = MvLatentPrefillArgs(q=q.data_ptr(), k=k.data_ptr(), v=v.data_ptr(), rot=rot.data_ptr(), out=out.data_ptr(),
+                            q_stride=q.stride(0), k_stride=k.stride(0), v_stride=v.stride(0), rot_stride=rot.stride(0),
+                            out_stride=out.stride(0), cu_q=cu_q.data_ptr(), cu_k=cu_k.data_ptr(), positions=positions.data_ptr(),
+                            cos=cos.data_ptr(), sin=sin.data_ptr(), max_pos=cos.shape[0], n_seqs=cu_q.numel() - 1,
+                            max_q=int(max_q), max_k=int(max_k), heads=h, plain_cols=dp, rot_dim=rot_dim, rot_cols=rot.shape[1],
+                            dq=dq, dv=dv, window=int(window), scale=float(scale))
+    _check(_lib.mv_latent_prefill(ctypes.byref(a), _dt(q), int(flags), _stream()), "mv_latent_prefill")
+    return out
+
+
+# ---------------------------------------------------------------- K15
+MV_SSM_SCAN = 1
+
+
+def _ssm_args(shape, x, state_slots, out, conv_w=None, conv_b=None, conv_state=None, ssm_state=None, dt=None, dt_bias=None,
+              a_log=None, d=None):
+    """``shape``: (heads, groups, p, n, b_off, c_off)."""
+    _need_cuda(x, state_slots, conv_state, ssm_state, dt)
+    heads, groups, p, n, b_off, c_off = shape
+    a = MvSsmArgs(x=x.data_ptr(), x_stride=x.stride(0), state_slots=state_slots.data_ptr(), out=out.data_ptr(),
+                  out_stride=out.stride(0), n_seqs=state_slots.numel(), channels=c_off + groups * n, taps=1, heads=heads,
+                  groups=groups, p=p, n=n, b_off=b_off, c_off=c_off)
+    _rows_ok("x", x, a.channels)
+    if state_slots.dtype != torch.int32 or not state_slots.is_contiguous():
+        raise MvHipError("int32 state slots required")
+    if conv_w is not None:
+        if conv_w.dtype != x.dtype or conv_b.dtype != x.dtype or conv_w.shape[1] != a.channels or conv_b.numel() != a.channels:
+            raise MvHipError(f"convolution weight [taps, {a.channels}] and bias of {x.dtype} required")
+        a.conv_w, a.conv_b, a.taps = conv_w.data_ptr(), conv_b.data_ptr(), conv_w.shape[0]
+    slots = 0
+    if conv_state is not None and conv_state.numel():
+        slots = conv_state.shape[1]
+        if conv_state.dtype != x.dtype or tuple(conv_state.shape) != (2, slots, a.taps - 1, a.channels) or not conv_state.is_contiguous():
+            raise MvHipError(f"convolution state must be dense [2, slots, {a.taps - 1}, {a.channels}] of {x.dtype}")
+        a.conv_state = conv_state.data_ptr()
+    if ssm_state is not None and ssm_state.numel():
+        slots = ssm_state.shape[1]
+        if ssm_state.dtype != torch.float32 or tuple(ssm_state.shape) != (2, slots, heads, n, p) or not ssm_state.is_contiguous():
+            raise MvHipError(f"recurrent state must be dense fp32 [2, slots, {heads}, {n}, {p}]")
+        a.ssm_state = ssm_state.data_ptr()
+    a.slots = slots
+    if dt is not None:
+        if dt.dtype != x.dtype or dt.shape[0] != x.shape[0] or dt.stride(1) != 1:
+            raise MvHipError("raw step sizes: rows of x's dtype, one per token")
+        for w in (dt_bias, a_log, d):
+            if w.dtype != x.dtype or w.numel() < heads:
+                raise MvHipError(f"per-head parameters of {x.dtype} required")
+        a.dt, a.dt_stride = dt.data_ptr(), dt.stride(0)
+        a.dt_bias, a.a_log, a.d = dt_bias.data_ptr(), a_log.data_ptr(), d.data_ptr()
+    return a
+
+
+def causal_conv(x, conv_w, conv_b, shape, conv_state, state_slots, cu_q, cu_k, max_q: int):
+    """silu(causal convolution) of the projected channels [T, channels] of a batch of sequences; keeps the last inputs."""
+    out = torch.empty((x.shape[0], conv_w.shape[1]), dtype=x.dtype, device=x.device)
+    a = _ssm_args(shape, x, state_slots, out, conv_w, conv_b, conv_state)
+    a.cu_q, a.cu_k, a.max_q = cu_q.data_ptr(), cu_k.data_ptr(), int(max_q)
+    _check(_lib.mv_causal_conv(ctypes.byref(a), _dt(x), _stream()), "mv_causal_conv")
+    return out
+
+
+def ssm_prefill(x, dt, dt_bias, a_log, d, shape, ssm_state, state_slots, cu_q, cu_k, max_q: int, out=None, flags: int = 0):
+    """The recurrence over convolved channels [T, channels] and raw step sizes [T, heads] -> y [T, heads * p]."""
+    if out is None:
+        out = torch.empty((x.shape[0], shape[0] * shape[2]), dtype=x.dtype, device=x.device)
+    a = _ssm_args(shape, x, state_slots, out, ssm_state=ssm_state, dt=dt, dt_bias=dt_bias, a_log=a_log, d=d)
+    a.cu_q, a.cu_k, a.max_q = cu_q.data_ptr(), cu_k.data_ptr(), int(max_q)
+    _check(_lib.mv_ssm_prefill(ctypes.byref(a), _dt(x), int(flags), _stream()), "mv_ssm_prefill")
+    return out
+
+
+def ssm_step(x, dt, conv_w, conv_b, dt_bias, a_log, d, shape, conv_state, ssm_state, state_slots, context_lens, out=None):
+    """One token per sequence: convolution and recurrence of the projected channels [B, channels] -> y [B, heads * p]."""
+    if out is None:
+        out = torch.empty((x.shape[0], shape[0] * shape[2]), dtype=x.dtype, device=x.device)
+    a = _ssm_args(shape, x, state_slots, out, conv_w, conv_b, conv_state, ssm_state, dt, dt_bias, a_log, d)
+    lens = _i32(context_lens)
+    if lens.numel() != x.shape[0] or state_slots.numel() != x.shape[0]:
+        raise MvHipError("one length and one state slot per row required")
+    a.context_lens = lens.data_ptr()
+    _check(_lib.mv_ssm_step(ctypes.byref(a), _dt(x), _stream()), "mv_ssm_step")
+    return out
+
+
+def gated_group_norm(y, z, w, heads: int, p: int, p_true: int, groups: int, eps: float):
+    """rms over each of ``groups`` equal parts of y * silu(z), times w: [T, heads * p] (p_true of each head's columns count)."""
+    _need_cuda(y, z, w)
+    cols = heads * p
+    _rows_ok("y", y, cols)
+    _rows_ok("z", z, cols, y.dtype)
+    if w.dtype != y.dtype or w.numel() != cols or y.shape[0] != z.shape[0]:
+        raise MvHipError(f"norm weight of {cols} {y.dtype} and as many rows of z required")
+    out = torch.empty((y.shape[0], cols), dtype=y.dtype, device=y.device)
+    _check(_lib.mv_gated_group_norm(y.data_ptr(), y.stride(0), z.data_ptr(), z.stride(0), w.data_ptr(), out.data_ptr(),
+                                    out.stride(0), y.shape[0], heads, p, p_true, groups, float(eps), _dt(y), _stream()),
+           "mv_gated_group_norm")
+    return out

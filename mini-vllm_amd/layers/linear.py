@@ -162,9 +162,10 @@ def linear(x, weight, bias=None, packed=None, kind: str = "col"):
     return F.linear(x, weight, bias)
 
 
-def gated_linear(x, lin, act: str = "silu", out=None):
-    """act(x W_gate^T) * (x W_up^T) for ``lin`` with the merged weight [gate rows ; up rows]: in the projection's epilogue for
-    decode-sized inputs, else the library GEMM and the activation kernel.  ``out``: where it goes (2-D, rows may be strided)."""
+def gated_linear(x, lin, act="silu", out=None):
+    """act(x W_gate^T, x W_up^T) ("silu" / "gelu_tanh": of the gate, times up; or a hip_ops.GateAct) for ``lin`` with the merged
+    weight [gate rows ; up rows]: in the projection's epilogue for decode-sized inputs, else the library GEMM and the activation
+    kernel.  ``out``: where it goes (2-D, rows may be strided)."""
     w = lin.weight
     if small_m(x, w):
         return hip_ops.gate_up_silu_small_m(x, w, packed=lin.weight_packed, act=act, out=out)
@@ -173,7 +174,7 @@ def gated_linear(x, lin, act: str = "silu", out=None):
         cfg, _ = mid_plan("gated", x.numel() // x.shape[-1], n_inter, w.shape[1])
         if cfg:
             return hip_ops.gate_up_silu_mid_m(x, lin.weight_packed, n_inter, cfg, act=act, out=out)
-    return (hip_ops.silu_and_mul if act == "silu" else hip_ops.gelu_and_mul)(lin(x), out=out)
+    return hip_ops.act_and_mul(lin(x), act, out=out)
 
 
 class LinearBase(nn.Module):
@@ -309,11 +310,13 @@ def pad_to(n: int, multiple: int = 64) -> int:
 @dataclass(frozen=True)
 class Segment:
     """One checkpoint matrix inside a merged weight: ``units`` (heads, features) of ``unit`` rows or columns each, stored
-    at ``stored`` >= unit apiece (zeros behind); a tensor-parallel rank owns a contiguous run of whole units."""
+    at ``stored`` >= unit apiece (zeros behind); a tensor-parallel rank owns a contiguous run of whole units.  ``parts``:
+    pieces (size, place) of a unit that do not lie one behind the other in the stored unit."""
     name: str
     units: int
     unit: int = 1
     stored: int | None = None
+    parts: tuple[tuple[int, int], ...] | None = None
 
     def local(self, tp: int) -> int:
         """Stored rows / columns of one rank: a multiple of 64, so that the next segment starts on a whole tile."""
@@ -345,8 +348,16 @@ class SegmentedLinear(LinearBase):
     def weight_loader(self, param, loaded_weight, loaded_shard_id: str | None = None, *args, **kwargs):
         if loaded_shard_id is None and len(self.segments) == 1:
             loaded_shard_id = next(iter(self.segments))
-        g = self.segments[loaded_shard_id]
         dim = 1 if self.split == "in" else 0
+        if isinstance(loaded_shard_id, tuple):      # one checkpoint tensor that holds several segments, one behind the other
+            at, sizes = 0, [self.segments[n].units * self.segments[n].unit for n in loaded_shard_id]
+            if loaded_weight.shape[dim] != sum(sizes):
+                raise ValueError(f"segments {loaded_shard_id}: expected {sum(sizes)}, got {loaded_weight.shape[dim]}")
+            for n, size in zip(loaded_shard_id, sizes):
+                self.weight_loader(param, loaded_weight.narrow(dim, at, size), n)
+                at += size
+            return
+        g = self.segments[loaded_shard_id]
         want = [self.other_size, self.other_size]
         want[dim] = g.units * g.unit
         if tuple(loaded_weight.shape) != tuple(want):
@@ -354,9 +365,12 @@ class SegmentedLinear(LinearBase):
         units, stored, off = divide(g.units, self.shards), g.stored or g.unit, self.offsets[g.name]
         rank = self.tp_rank if self.shards > 1 else 0
         piece = materialize(loaded_weight.narrow(dim, rank * units * g.unit, units * g.unit))
-        dst = param.data.narrow(dim, off, units * stored).unflatten(dim, (units, stored)).narrow(dim + 1, 0, g.unit)
+        dst = param.data.narrow(dim, off, units * stored).unflatten(dim, (units, stored))
         dst = dst.narrow(0 if dim == 1 else 2, 0, self.other_size)
-        dst.copy_(piece.unflatten(dim, (units, g.unit)))
+        piece, at = piece.unflatten(dim, (units, g.unit)), 0
+        for size, place in g.parts or ((g.unit, 0),):
+            dst.narrow(dim + 1, place, size).copy_(piece.narrow(dim + 1, at, size))
+            at += size
 
     def forward(self, x, partial_ok: bool = False):
         """``partial_ok`` (split="in", single rank): the caller takes a ``PartialSum``."""

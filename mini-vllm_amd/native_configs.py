@@ -7,7 +7,8 @@ import math
 from dataclasses import dataclass
 from pathlib import Path
 
-__all__ = ["AttentionSpec", "LayerSpec", "MofaraxConfig", "NATIVE_CONFIGS", "load_native_config"]
+__all__ = ["AttentionSpec", "LayerSpec", "MofaraxConfig", "LatentAttentionSpec", "Mamba2Spec", "ClampedMlpSpec", "MixerLayerSpec",
+           "KugulornConfig", "NATIVE_CONFIGS", "load_native_config"]
 
 
 def _need(d: dict, key: str, where: str):
@@ -147,7 +148,159 @@ class MofaraxConfig:
         return out
 
 
-NATIVE_CONFIGS = {"Mofarax": MofaraxConfig}
+@dataclass(frozen=True)
+class LatentAttentionSpec:
+    """Attention whose keys and values are one cached latent per token; see layers/latent_attention.py."""
+    heads: int
+    dim: int            # unrotated query / key dims of a head
+    rot_dim: int        # rotated ones, one key part for all heads
+    vdim: int
+    q_rank: int
+    kv_rank: int
+    rot_base: float
+    scale: float
+    window: int         # 0: every key up to the query
+    kv_from: int | None  # layer whose latents this one reads instead of its own
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str) -> "LatentAttentionSpec":
+        sizes = {k: _size(_need(m, k, where), f"{where}.{k}") for k in ("heads", "dim", "rot_dim", "vdim", "q_rank", "kv_rank")}
+        rot = _need(m, "rot", where)
+        dims = _size(rot.get("dims", sizes["rot_dim"]), f"{where}.rot.dims")
+        if sizes["rot_dim"] % 2 or dims != sizes["rot_dim"]:
+            raise ValueError(f"{where}: rot_dim must be even and all of it rotated, got {sizes['rot_dim']} and rot.dims {dims}")
+        base, scale = _real(_need(rot, "base", f"{where}.rot"), f"{where}.rot.base"), _real(_need(m, "scale", where), f"{where}.scale")
+        if scale <= 0 or base <= 0:
+            raise ValueError(f"{where}: scale and rot.base must be positive, got {scale} and {base}")
+        mask = m.get("mask") or {}
+        window = _size(mask["size"], f"{where}.mask.size") if mask.get("size") is not None else 0
+        source = m.get("kv_from")
+        if source is not None and (isinstance(source, bool) or not isinstance(source, int) or source < 0):
+            raise ValueError(f"{where}.kv_from must be a layer's index, got {source!r}")
+        return cls(**sizes, rot_base=base, scale=scale, window=window, kv_from=source)
+
+    def weight_shapes(self, width: int) -> dict[str, tuple[int, ...]]:
+        h, out = self.heads, {"dq": (self.q_rank, width), "dq.norm": (self.q_rank,)}
+        out["uq"], out["o"] = (h * (self.dim + self.rot_dim), self.q_rank), (width, h * self.vdim)
+        out["uk"], out["uv"] = (h * self.dim, self.kv_rank), (h * self.vdim, self.kv_rank)
+        if self.kv_from is None:
+            out["dkv"], out["dkv.norm"] = (self.kv_rank + self.rot_dim, width), (self.kv_rank,)
+        return out
+
+
+@dataclass(frozen=True)
+class Mamba2Spec:
+    """Selective state space mixer; see layers/mamba2.py."""
+    heads: int
+    vdim: int
+    state: int
+    groups: int
+    taps: int           # of the causal convolution
+    norm_groups: int
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str) -> "Mamba2Spec":
+        s = {k: _size(_need(m, k, where), f"{where}.{k}") for k in ("heads", "vdim", "state", "groups", "conv", "norm_groups")}
+        s["taps"] = s.pop("conv")
+        if s["heads"] % s["groups"]:
+            raise ValueError(f"{where}: {s['heads']} heads do not divide over {s['groups']} groups")
+        if s["heads"] * s["vdim"] % s["norm_groups"]:
+            raise ValueError(f"{where}: {s['heads'] * s['vdim']} columns do not divide into {s['norm_groups']} norm groups")
+        return cls(**s)
+
+    def weight_shapes(self, width: int) -> dict[str, tuple[int, ...]]:
+        inner, bc = self.heads * self.vdim, 2 * self.groups * self.state
+        out = {"in": (2 * inner + bc + self.heads, width), "conv": (inner + bc, self.taps), "conv.b": (inner + bc,)}
+        out["dt_bias"] = out["A_log"] = out["D"] = (self.heads,)
+        out["norm"], out["o"] = (inner,), (width, inner)
+        return out
+
+
+@dataclass(frozen=True)
+class ClampedMlpSpec:
+    ff: int
+    limit: float
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str) -> "ClampedMlpSpec":
+        if m.get("kind", "dense") != "dense":
+            raise ValueError(f"{where}: unsupported feed-forward {m.get('kind')!r}")
+        limit = _real(_need(m, "limit", where), f"{where}.limit")
+        if limit <= 0:
+            raise ValueError(f"{where}.limit must be positive, got {limit}")
+        return cls(_size(_need(m, "ff", where), f"{where}.ff"), limit)
+
+
+@dataclass(frozen=True)
+class MixerLayerSpec:
+    """A mixer of one of several kinds and an optional feed-forward."""
+    type: str
+    mixer: LatentAttentionSpec | Mamba2Spec
+    mlp: ClampedMlpSpec | None
+    KINDS = {"latent_attention": LatentAttentionSpec, "mamba2": Mamba2Spec}
+
+    @classmethod
+    def from_dict(cls, d: dict, where: str) -> "MixerLayerSpec":
+        kind = _need(d, "type", where)
+        if kind not in cls.KINDS:
+            raise ValueError(f"{where}: unsupported layer type {kind!r}; known: {sorted(cls.KINDS)}")
+        mlp = d.get("mlp")
+        return cls(kind, cls.KINDS[kind].from_dict(_need(d, "mixer", where), f"{where}.mixer"),
+                   None if mlp is None else ClampedMlpSpec.from_dict(mlp, f"{where}.mlp"))
+
+
+class KugulornConfig:
+    """Latent attention and state space layers, some sharing one layer's latents, over a 32-bit residual stream."""
+    model_type = "kugulorn"
+
+    def __init__(self, raw: dict) -> None:
+        self.architectures = ["Kugulorn"]
+        self.vocab_size = _size(_need(raw, "vocab", "config"), "vocab")
+        self.hidden_size = _size(_need(raw, "width", "config"), "width")
+        self.norm_eps = _real(_need(_need(raw, "norm", "config"), "eps", "norm"), "norm.eps")
+        self.residual_mult = _real(raw.get("residual_mult", 1.0), "residual_mult")
+        layers = _need(raw, "layers", "config")
+        if not isinstance(layers, list) or not layers:
+            raise ValueError("config: 'layers' must be a non-empty list")
+        self.layers = [MixerLayerSpec.from_dict(d, f"layers[{i}]") for i, d in enumerate(layers)]
+        for i, s in enumerate(self.layers):
+            j = getattr(s.mixer, "kv_from", None)
+            if j is None:
+                continue
+            src = self.layers[j] if j < i else None
+            if src is None or src.type != s.type or src.mixer.kv_from is not None:
+                raise ValueError(f"layers[{i}].mixer.kv_from: {j} is not an earlier layer with latents of its own")
+            a, b = src.mixer, s.mixer
+            if (a.kv_rank, a.rot_dim, a.rot_base) != (b.kv_rank, b.rot_dim, b.rot_base):
+                raise ValueError(f"layers[{i}].mixer: kv_rank, rot_dim and rot.base must equal those of layer {j}")
+        # what the engine asks of any configuration
+        self.num_hidden_layers = len(self.layers)
+        self.num_attention_heads = max(s.mixer.heads for s in self.layers)
+        self.num_key_value_heads = 1
+        self.head_dim = max((s.mixer.kv_rank + s.mixer.rot_dim for s in self.layers if s.type != "mamba2"), default=1)
+        self.intermediate_size = max((s.mlp.ff for s in self.layers if s.mlp), default=0)
+        self.recurrent_state = any(s.type == "mamba2" for s in self.layers)
+        self.max_position_embeddings: int | None = None    # none of its own; the engine's Config fills it in
+        self.torch_dtype = raw.get("dtype", "bfloat16")
+        self.eos_token_id = None
+        self.tie_word_embeddings = False
+
+    def weight_shapes(self) -> dict[str, tuple[int, ...]]:
+        """Name -> shape of every tensor of a checkpoint."""
+        v, d = self.vocab_size, self.hidden_size
+        out: dict[str, tuple[int, ...]] = {"embed": (v, d), "final.norm": (d,), "head": (v, d)}
+        for i, s in enumerate(self.layers):
+            p = f"l{i}."
+            out[p + "norm1"] = out[p + "norm1b"] = out[p + "ls1"] = (d,)
+            out.update({f"{p}mix.{k}": v for k, v in s.mixer.weight_shapes(d).items()})
+            if s.mlp:
+                out[p + "norm2"] = out[p + "norm2b"] = out[p + "ls2"] = (d,)
+                out[p + "mlp.gate"] = out[p + "mlp.up"] = (s.mlp.ff, d)
+                out[p + "mlp.down"] = (d, s.mlp.ff)
+        return out
+
+
+NATIVE_CONFIGS = {"Mofarax": MofaraxConfig, "Kugulorn": KugulornConfig}
 
 
 def load_native_config(model_dir: str):

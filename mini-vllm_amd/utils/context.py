@@ -33,6 +33,11 @@ class Context:
     rest_cum_seqlens_k: torch.Tensor | None = None
     rest_max_seqlen_q: int = 0
     rest_max_seqlen_k: int = 0
+    # build-only: where each sequence's recurrent state lives (int32 [n], -1 = nowhere)
+    state_slots: torch.Tensor | None = None
+    # build-only (layers that expand keys from cached rows, prefix_cached batches): window -> the spans of cached keys that the
+    # non-decode sequences read, (cumulative lengths, first positions, total, longest); window 0 = from the start
+    key_spans: dict | None = None
 
 
 _CURRENT: ContextVar[Context | None] = ContextVar("minivllm_amd_context", default=None)
@@ -46,10 +51,12 @@ def get_context() -> Context:
 def set_context(is_prefill: bool, max_seqlen_q: int = 0, max_seqlen_k: int = 0,
                 cum_seqlens_q=None, cum_seqlens_k=None, slot_mapping=None, context_lens=None,
                 block_tables=None, prefix_cached: bool = False, decode_rows: int = 0, rest_cum_seqlens_q=None,
-                rest_cum_seqlens_k=None, rest_max_seqlen_q: int = 0, rest_max_seqlen_k: int = 0) -> None:
+                rest_cum_seqlens_k=None, rest_max_seqlen_q: int = 0, rest_max_seqlen_k: int = 0, state_slots=None,
+                key_spans=None) -> None:
     _CURRENT.set(Context(is_prefill, max_seqlen_q, max_seqlen_k, cum_seqlens_q, cum_seqlens_k,
                          slot_mapping, context_lens, block_tables, prefix_cached, decode_rows,
-                         rest_cum_seqlens_q, rest_cum_seqlens_k, rest_max_seqlen_q, rest_max_seqlen_k))
+                         rest_cum_seqlens_q, rest_cum_seqlens_k, rest_max_seqlen_q, rest_max_seqlen_k,
+                         state_slots, key_spans))
 
 
 def reset_context() -> None:
