@@ -36,6 +36,13 @@ __device__ __forceinline__ void store_vec_row(typename elem<Tag>::T *p, const fl
   *reinterpret_cast<u32x4 *>(p) = raw;
 }
 
+// let kernel K use the CU's whole LDS (once per process)
+template <auto K>
+static inline int mv_allow_lds() {
+  static const hipError_t rc = hipFuncSetAttribute((const void *)K, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+  return mv_check_hip(rc);
+}
+
 // vector-ALU forms (every dtype and size)
 int mv_latent_decode_simple_launch(const void *q, const void *plane, const int32_t *tables, int64_t table_stride,
                                    const int32_t *lens, void *out, int batch, int heads, int kv_cols, int rot_cols,

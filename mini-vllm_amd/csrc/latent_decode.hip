@@ -1,0 +1,274 @@
+// K14 — latent attention, decode on the matrix cores (16-bit): every head's query row against the cached rows themselves
+// (scores over the whole row, values = its latent columns), so a row is read from HBM once for all heads.
+//
+// One workgroup = 4 waves = up to 16 HG heads of one sequence and one part of its visible keys; tiles of 32 keys (one page each),
+// double-buffered in LDS by LDS-DMA, two workgroups per CU.  LDS rows have an odd number of 16-byte chunks, so neither the row
+// reads nor the transposed reads meet in a bank.  Per tile:
+//   S^T[key][head] = rows . Q^T     wave w: keys 16 (w & 1) .., heads 16 (w >> 1) .. (HG = 1: two waves do the same work)
+//   softmax                         running maxima per head, exchanged through LDS; probabilities to LDS as 16-bit rows
+//   O^T[column][head] += V^T P^T    wave w: a quarter of the latent columns, all heads; V^T by transposed LDS reads
+// A context in several parts leaves fp32 sums and (maximum, sum) pairs in the workspace; a second launch merges them.
+#include "latent.h"
+
+namespace {
+
+typedef __attribute__((ext_vector_type(4))) short s16x4;
+typedef __attribute__((address_space(3))) s16x4 lds_s16x4;
+
+constexpr int TK = 32;   // keys per tile
+constexpr int kMaxRot = 64, kMaxSplits = 64;
+
+struct DecodeParams {
+  const void *q, *plane;
+  const int32_t *tables, *lens;
+  void *out;
+  float *part, *part_ml;   // [batch][heads][splits][kv_cols], [batch][heads][splits][2]
+  int64_t table_stride, num_blocks;
+  int heads, kv_cols, cols, block_size, max_blocks, window, splits;
+  float scale;
+};
+
+__host__ __device__ __forceinline__ int lds_chunks(int cols) { return cols / 8 + 1 - (cols / 8 & 1); }   // odd
+
+// CT: latent column tiles of 16 per wave (kv_cols <= 64 CT)
+template <typename Tag, int HG, int CT>
+__global__ void __launch_bounds__(256, 2) latent_decode_kernel(DecodeParams p) {
+  typedef typename elem<Tag>::T T;
+  constexpr int KSM = 2 * CT + kMaxRot / 32;   // 32-column steps of a row
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), r16 = lane & 15, g = lane >> 4;
+  const int split = blockIdx.x, h0 = blockIdx.y * 16 * HG, b = blockIdx.z;
+  const int CH = lds_chunks(p.cols), RB = CH * 16, ks = p.cols / 32, cts = p.kv_cols / 64;
+  const int dmas = (TK * CH + 63) / 64, BUF = dmas * 1024;
+  float *smax = (float *)(smem + 2 * BUF);                      // [2 key halves][16 HG heads]
+  char *prob = (char *)(smax + 2 * 16 * HG);                    // [16 HG heads][TK] 16-bit, rows of 80 bytes
+  constexpr int PR = 80;
+  const int len = min(p.lens[b], p.max_blocks * p.block_size), lo = p.window > 0 && len > p.window ? len - p.window : 0;
+  const int first = lo / TK, tiles = len > 0 ? (len + TK - 1) / TK - first : 0, per = (tiles + p.splits - 1) / p.splits;
+  const int t0 = first + split * per, t1 = min(first + tiles, t0 + per);
+
+  // Q^T fragments of this wave's heads
+  const int kg = wave & 1, hg = HG == 2 ? wave >> 1 : 0, qh = h0 + hg * 16 + r16;
+  u32x4 qf[KSM];
+  {
+    const T *qp = (const T *)p.q + ((int64_t)b * p.heads + min(qh, p.heads - 1)) * p.cols + g * 8;
+#pragma unroll
+    for (int s = 0; s < KSM; ++s)
+      if (s < ks) qf[s] = *(const u32x4 *)(qp + s * 32);
+  }
+  f32x4 acc[HG][CT] = {};
+  float m_run[HG], l_run[HG];
+#pragma unroll
+  for (int i = 0; i < HG; ++i) m_run[i] = -1e30f, l_run[i] = 0.f;
+  const float scale_log2 = p.scale * 1.4426950408889634f;
+
+  // page of a tile, or -1; kept one tile ahead so that the table entry is there when its rows are requested
+  auto page = [&](int t) {
+    const int blk = t < t1 ? p.tables[b * p.table_stride + t * TK / p.block_size] : -1;
+    return blk >= 0 && blk < p.num_blocks ? blk : -1;
+  };
+  const int q256 = 256 / CH, r256 = 256 % CH, row_first = (wave * 64 + lane) / CH, col_first = (wave * 64 + lane) % CH;
+  auto dma = [&](int t, int blk, int buf) {
+    if (blk < 0) return;
+    const T *src = (const T *)p.plane + ((int64_t)blk * p.block_size + t * TK % p.block_size) * p.cols;
+    const int last = min(TK, len - t * TK) - 1;   // rows past the end re-read the last key (probability 0, finite data)
+    int row = row_first, col = col_first;
+    for (int i = wave; i < dmas; i += 4) {
+      __builtin_amdgcn_global_load_lds(
+          (const __attribute__((address_space(1))) void *)(src + (int64_t)min(row, last) * p.cols + min(col, p.cols / 8 - 1) * 8),
+          (__attribute__((address_space(3))) void *)(smem + buf * BUF + i * 1024), 16, 0, 0);
+      row += q256, col += r256;
+      if (col >= CH) col -= CH, ++row;
+    }
+  };
+
+  int blk = page(t0), buf = 0;
+  dma(t0, blk, 0);
+  int blk_next = page(t0 + 1);
+  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+  __syncthreads();
+  for (int t = t0; t < t1; ++t, buf ^= 1) {
+    if (t + 1 < t1) dma(t + 1, blk_next, buf ^ 1);
+    const int blk_after = page(t + 2);
+    if (blk >= 0) {
+      const char *tile = smem + buf * BUF;
+      // ---- scores: 16 keys x 16 heads
+      f32x4 s = {0.f, 0.f, 0.f, 0.f};
+      const char *ka = tile + (kg * 16 + r16) * RB + g * 16;
+#pragma unroll
+      for (int i = 0; i < KSM; ++i)
+        if (i < ks) s = mfma16x16x32<Tag>(*(const u32x4 *)(ka + i * 64), qf[i], s);
+      float mx = -INFINITY;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int key = t * TK + kg * 16 + g * 4 + i;
+        s[i] = key < len && key >= lo ? s[i] * scale_log2 : -INFINITY;
+        mx = fmaxf(mx, s[i]);
+      }
+      mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+      mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+      if (g == 0) smax[kg * 16 * HG + hg * 16 + r16] = mx;
+      __syncthreads();
+      float alpha[HG];
+#pragma unroll
+      for (int i = 0; i < HG; ++i) {
+        const float m_new = fmaxf(m_run[i], fmaxf(smax[i * 16 + r16], smax[16 * HG + i * 16 + r16]));
+        alpha[i] = __builtin_amdgcn_exp2f(m_run[i] - m_new);
+        m_run[i] = m_new;
+        l_run[i] *= alpha[i];
+      }
+      float e[4], sum = 0.f;
+      const float m_own = HG == 2 && hg ? m_run[HG - 1] : m_run[0];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) e[i] = __builtin_amdgcn_exp2f(s[i] - m_own), sum += e[i];
+      if (HG == 2 && hg) l_run[HG - 1] += sum;
+      else l_run[0] += sum;
+      if (HG == 2 || wave < 2)
+        *(u32x2 *)(prob + (hg * 16 + r16) * PR + (kg * 16 + g * 4) * 2) =
+            u32x2{(uint32_t)elem<Tag>::st(e[0]) | ((uint32_t)elem<Tag>::st(e[1]) << 16),
+                  (uint32_t)elem<Tag>::st(e[2]) | ((uint32_t)elem<Tag>::st(e[3]) << 16)};
+      __syncthreads();
+      // ---- values
+      u32x4 pf[HG];
+#pragma unroll
+      for (int i = 0; i < HG; ++i) pf[i] = *(const u32x4 *)(prob + (i * 16 + r16) * PR + g * 16);
+      const char *va = tile + (g * 8 + (r16 >> 2)) * RB + (r16 & 3) * 8 + wave * 32;
+#pragma unroll
+      for (int c = 0; c < CT; ++c)
+        if (c < cts) {
+          const u32x2 a0 = __builtin_bit_cast(u32x2, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4 *)(va + c * 128)));
+          const u32x2 a1 = __builtin_bit_cast(u32x2, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4 *)(va + 4 * RB + c * 128)));
+          const u32x4 a = {a0.x, a0.y, a1.x, a1.y};
+#pragma unroll
+          for (int i = 0; i < HG; ++i) acc[i][c] = mfma16x16x32<Tag>(a, pf[i], acc[i][c] * alpha[i]);
+        }
+    }
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    __syncthreads();
+    blk = blk_next, blk_next = blk_after;
+  }
+  // ---- sums of a head: over the waves that scored it (its two key halves) and their four lane groups
+  float *sl = smax;   // [2][16 HG]
+  {
+    float l = HG == 2 && hg ? l_run[HG - 1] : l_run[0];
+    l += __shfl_xor(l, 16, 64);
+    l += __shfl_xor(l, 32, 64);
+    if (g == 0 && (HG == 2 || wave < 2)) sl[kg * 16 * HG + hg * 16 + r16] = l;
+  }
+  __syncthreads();
+#pragma unroll
+  for (int i = 0; i < HG; ++i) {
+    const int head = h0 + i * 16 + r16;
+    if (head >= p.heads) continue;
+    const float l = sl[i * 16 + r16] + sl[16 * HG + i * 16 + r16];
+    const int64_t row = (int64_t)b * p.heads + head;
+    if (p.splits == 1) {
+      const float inv = l > 0.f ? 1.0f / l : 0.f;
+      T *o = (T *)p.out + row * p.kv_cols + wave * 16 + g * 4;
+#pragma unroll
+      for (int c = 0; c < CT; ++c)
+        if (c < cts)
+          *(u32x2 *)(o + c * 64) = u32x2{(uint32_t)elem<Tag>::st(acc[i][c][0] * inv) | ((uint32_t)elem<Tag>::st(acc[i][c][1] * inv) << 16),
+                                         (uint32_t)elem<Tag>::st(acc[i][c][2] * inv) | ((uint32_t)elem<Tag>::st(acc[i][c][3] * inv) << 16)};
+    } else {
+      float *o = p.part + (row * p.splits + split) * p.kv_cols + wave * 16 + g * 4;
+#pragma unroll
+      for (int c = 0; c < CT; ++c)
+        if (c < cts) *(f32x4 *)(o + c * 64) = acc[i][c];
+      if (wave == 0 && g == 0) {
+        float *ml = p.part_ml + (row * p.splits + split) * 2;
+        ml[0] = m_run[i], ml[1] = l;
+      }
+    }
+  }
+}
+
+template <typename Tag>
+__global__ void __launch_bounds__(256) latent_merge_kernel(const float *part, const float *part_ml, void *out, int rows, int splits,
+                                                           int kv_cols) {
+  typedef typename elem<Tag>::T T;
+  const int per = kv_cols / 4, idx = blockIdx.x * 256 + threadIdx.x, row = idx / per, c = idx % per * 4;
+  if (row >= rows) return;
+  const float *ml = part_ml + (int64_t)row * splits * 2;
+  float m = -1e30f, l = 0.f;
+  for (int s = 0; s < splits; ++s) m = fmaxf(m, ml[2 * s]);
+  f32x4 o = {0.f, 0.f, 0.f, 0.f};
+  for (int s = 0; s < splits; ++s) {
+    if (!(ml[2 * s + 1] > 0.f)) continue;
+    const float w = __builtin_amdgcn_exp2f(ml[2 * s] - m);
+    l = fmaf(ml[2 * s + 1], w, l);
+    o += *(const f32x4 *)(part + ((int64_t)row * splits + s) * kv_cols + c) * w;
+  }
+  const float inv = l > 0.f ? 1.0f / l : 0.f;
+  *(u32x2 *)((T *)out + (int64_t)row * kv_cols + c) =
+      u32x2{(uint32_t)elem<Tag>::st(o[0] * inv) | ((uint32_t)elem<Tag>::st(o[1] * inv) << 16),
+            (uint32_t)elem<Tag>::st(o[2] * inv) | ((uint32_t)elem<Tag>::st(o[3] * inv) << 16)};
+}
+
+int head_groups(int heads) { return heads > 16 ? 2 : 1; }
+
+// parts of a context: enough workgroups for two per CU, at least two tiles each
+int split_count(int batch, int heads, int block_size, int max_blocks, int window) {
+  const int hg = head_groups(heads), wgs = batch * ((heads + 16 * hg - 1) / (16 * hg));
+  int64_t keys = (int64_t)max_blocks * block_size;
+  if (window > 0 && keys > window) keys = window;
+  const int64_t tiles = (keys + 2 * TK - 2) / TK;
+  int64_t s = (512 + wgs - 1) / wgs;
+  if (s > tiles / 2) s = tiles / 2;
+  if (s > kMaxSplits) s = kMaxSplits;
+  return s < 1 ? 1 : (int)s;
+}
+
+template <typename Tag, int HG>
+int launch(const DecodeParams &p, const dim3 &grid, size_t lds, hipStream_t stream) {
+#define MV_LD(CT_)                                                                                          \
+  if (p.kv_cols <= 64 * CT_) {                                                                              \
+    if (int e = mv_allow_lds<&latent_decode_kernel<Tag, HG, CT_>>()) return e;                              \
+    hipLaunchKernelGGL((latent_decode_kernel<Tag, HG, CT_>), grid, dim3(256), lds, stream, p);               \
+    MV_LAUNCH_CHECK();                                                                                      \
+    return MV_OK;                                                                                           \
+  }
+  MV_LD(2)
+  MV_LD(4)
+  MV_LD(8)
+#undef MV_LD
+  return MV_E_SHAPE;
+}
+
+}  // namespace
+
+size_t mv_latent_decode_mfma_workspace(int batch, int heads, int kv_cols, int rot_cols, int block_size, int max_blocks, int window) {
+  const int s = split_count(batch, heads, block_size, max_blocks, window);
+  return s == 1 ? 256 : ((size_t)batch * heads * s * (kv_cols + 2) * 4 + 255) / 256 * 256;
+}
+
+int mv_latent_decode_mfma_launch(const void *q, const void *plane, const int32_t *tables, int64_t table_stride,
+                                 const int32_t *lens, void *out, int batch, int heads, int kv_cols, int rot_cols, int block_size,
+                                 int max_blocks, int64_t num_blocks, int window, float scale, void *workspace,
+                                 size_t workspace_bytes, int dtype, hipStream_t stream) {
+  if ((kv_cols & 63) || kv_cols > 512 || rot_cols > kMaxRot || block_size % TK || batch > 65535) return MV_E_SHAPE;
+  const int splits = split_count(batch, heads, block_size, max_blocks, window), hg = head_groups(heads);
+  if (splits > 1 && (!workspace || workspace_bytes < mv_latent_decode_mfma_workspace(batch, heads, kv_cols, rot_cols, block_size,
+                                                                                     max_blocks, window)))
+    return MV_E_WORKSPACE;
+  DecodeParams p;
+  p.q = q, p.plane = plane, p.tables = tables, p.lens = lens, p.out = out;
+  p.part = (float *)workspace, p.part_ml = p.part + (int64_t)batch * heads * splits * kv_cols;
+  p.table_stride = table_stride, p.num_blocks = num_blocks, p.heads = heads, p.kv_cols = kv_cols, p.cols = kv_cols + rot_cols;
+  p.block_size = block_size, p.max_blocks = max_blocks, p.window = window, p.splits = splits, p.scale = scale;
+  const int CH = lds_chunks(p.cols);
+  const size_t lds = 2 * (size_t)((TK * CH + 63) / 64) * 1024 + 2 * 16 * hg * 4 + 16 * hg * 80;
+  const dim3 grid(splits, (heads + 16 * hg - 1) / (16 * hg), batch);
+  int rc;
+  if (dtype == MV_BF16) rc = hg == 2 ? launch<bf16_tag, 2>(p, grid, lds, stream) : launch<bf16_tag, 1>(p, grid, lds, stream);
+  else rc = hg == 2 ? launch<f16_tag, 2>(p, grid, lds, stream) : launch<f16_tag, 1>(p, grid, lds, stream);
+  if (rc != MV_OK || splits == 1) return rc;
+  const int rows = batch * heads;
+  const dim3 mgrid((rows * (kv_cols / 4) + 255) / 256);
+  if (dtype == MV_BF16)
+    hipLaunchKernelGGL((latent_merge_kernel<bf16_tag>), mgrid, dim3(256), 0, stream, p.part, p.part_ml, out, rows, splits, kv_cols);
+  else
+    hipLaunchKernelGGL((latent_merge_kernel<f16_tag>), mgrid, dim3(256), 0, stream, p.part, p.part_ml, out, rows, splits, kv_cols);
+  MV_LAUNCH_CHECK();
+  return MV_OK;
+}

@@ -192,11 +192,3 @@ extern "C" int mv_latent_prefill(const MvLatentPrefillArgs *a, int dtype, int fl
   }
   return mv_latent_prefill_simple_launch(*a, dtype, (hipStream_t)stream);
 }
-
-// matrix-core forms: not here yet
-size_t mv_latent_decode_mfma_workspace(int, int, int, int, int, int, int) { return 256; }
-int mv_latent_decode_mfma_launch(const void *, const void *, const int32_t *, int64_t, const int32_t *, void *, int, int, int, int,
-                                 int, int, int64_t, int, float, void *, size_t, int, hipStream_t) {
-  return MV_E_SHAPE;
-}
-int mv_latent_prefill_mfma_launch(const MvLatentPrefillArgs &, int, hipStream_t) { return MV_E_SHAPE; }
