@@ -352,6 +352,3 @@ extern "C" int mv_gated_group_norm(const void *y, int64_t y_stride, const void *
   MV_LAUNCH_CHECK();
   return MV_OK;
 }
-
-// in chunks on the matrix cores: not here yet
-int mv_ssm_chunk_launch(const MvSsmArgs &, int, hipStream_t) { return MV_E_SHAPE; }
