@@ -94,8 +94,33 @@ def _mofarax(like: str, side_dim: int = 128, layers: int = 20, loop=(8, 12, 3), 
                 head_dim=dim, intermediate_size=c["intermediate_size"])
 
 
-DESIGNS = {"mofarax": {"mofarax-0.6b": "qwen3-0.6b", "mofarax-1.7b": "qwen3-1.7b", "mofarax-7b": "qwen2-7b"}}
+def _kugulorn(like: str, q_rank: int, ssm_heads: int, groups: int, pairs: int, window: int = 2048, kv_rank: int = 512, rot: int = 64,
+              state: int = 128) -> dict:
+    """A Kugulorn configuration of ``pairs`` x [state space layer, latent attention layer with a feed-forward] with ``like``'s
+    width, heads and feed-forward; as many pairs as make the layers' weights ``like``'s.  Every second attention layer reads the
+    latents of the one before."""
+    c = MODELS[like]
+    heads, width, vocab = c["num_attention_heads"], c["hidden_size"], c["vocab_size"]
+    ssm = {"type": "mamba2", "mlp": None, "mixer": {"heads": ssm_heads, "vdim": 64, "state": state, "groups": groups, "conv": 4,
+                                                   "norm_groups": groups}}
+    layers = []
+    for i in range(pairs):
+        mixer = {"heads": heads, "dim": 128, "rot_dim": rot, "vdim": 128, "q_rank": q_rank, "kv_rank": kv_rank,
+                 "mask": {"size": window}, "rot": {"base": c["rope_theta"], "dims": rot}, "scale": (128 + rot) ** -0.5}
+        if i % 2:
+            mixer["kv_from"] = len(layers) - 1
+        layers += [ssm, {"type": "latent_attention", "mixer": mixer,
+                         "mlp": {"kind": "dense", "ff": c["intermediate_size"], "limit": 7.0}}]
+    return dict(architecture="Kugulorn", vocab=vocab, width=width, norm={"eps": 1e-6}, residual_mult=0.5, layers=layers, like=like,
+                window=window, vocab_size=vocab, hidden_size=width, num_attention_heads=heads, num_key_value_heads=1,
+                head_dim=kv_rank + rot, intermediate_size=c["intermediate_size"])
+
+
+DESIGNS = {"mofarax": {"mofarax-0.6b": "qwen3-0.6b", "mofarax-1.7b": "qwen3-1.7b", "mofarax-7b": "qwen2-7b"},
+           "kugulorn": {"kugulorn-0.6b": "qwen3-0.6b", "kugulorn-1.7b": "qwen3-1.7b", "kugulorn-7b": "qwen2-7b"}}
 MODELS.update({name: _mofarax(like) for name, like in DESIGNS["mofarax"].items()})
+MODELS.update({"kugulorn-0.6b": _kugulorn("qwen3-0.6b", 512, 32, 1, 19), "kugulorn-1.7b": _kugulorn("qwen3-1.7b", 768, 64, 1, 19),
+               "kugulorn-7b": _kugulorn("qwen2-7b", 1536, 112, 2, 21)})
 DESIGN_DECODE = ((256, 1024), (16, 1024), (1, 1024))      # (batch, context) of a design's decode records
 DESIGN_PREFILL = ((16, 1024), (4, 4096))
 HBM_PEAK_GBS = 8000.0  # MI355X_MICROARCH.md: HBM3E 8.0 TB/s spec (6.29 TB/s measured copy ceiling)
@@ -507,7 +532,7 @@ def step_roofline(engine, model, batch, ctx_mid, ms_per_step):
     ex = engine.model_runner.inference_executor
     seen, wbytes = set(), 0
     # weights of looped layers are read once a pass
-    passes = {id(m): len(layer.attn) for layer in getattr(ex.model, "stack", []) for m in layer.modules()}
+    passes = {id(m): len(layer.attn) for layer in getattr(ex.model, "stack", []) if hasattr(layer, "attn") for m in layer.modules()}
     for mod in ex.model.modules():
         w = getattr(mod, "weight", None)
         if w is None or w.dim() != 2 or w.data_ptr() in seen:
@@ -515,8 +540,14 @@ def step_roofline(engine, model, batch, ctx_mid, ms_per_step):
         if hasattr(mod, "input_size") or type(mod).__name__ == "ParallelLMHead":
             seen.add(w.data_ptr())
             wbytes += w.numel() * w.element_size() * passes.get(id(mod), 1)
-    L, nb, bs, hkv, d = ex.kv_cache.shape[1:]
-    kv = L * batch * ctx_mid * 2 * hkv * d * ex.dtype.itemsize
+    if ex.latents or ex.state_modules:    # cached rows seen by each attention layer; state read and written once
+        kv = sum(batch * min(ctx_mid, m.window or ctx_mid) * m.row_cols * ex.dtype.itemsize for m in ex.model.modules()
+                 if hasattr(m, "row_cols"))
+        kv += sum(2 * batch * t.numel() // (2 * t.shape[1]) * t.element_size() for m in ex.state_modules
+                  for t in (m.conv_state, m.ssm_state))
+    else:
+        L, nb, bs, hkv, d = ex.kv_cache.shape[1:]
+        kv = L * batch * ctx_mid * 2 * hkv * d * ex.dtype.itemsize
     gbs = (wbytes + kv) / (ms_per_step * 1e-3) / 1e9
     return {"bound": "hbm", "weight_bytes_per_gpu": wbytes, "kv_bytes_per_step_per_gpu": int(kv),
             "bytes_per_step_per_gpu": int(wbytes + kv), "achieved": round(gbs, 1), "peak": HBM_PEAK_GBS, "unit": "GB/s",
@@ -575,6 +606,8 @@ def prefill_records(engine, model, gpus=1, cases=PREFILL_CASES, reps=5):
     busy, busy_src = _mfma_busy_quote()
     g = torch.Generator().manual_seed(1)
     out = []
+    latent = bool(ex.latents)
+    entry = "latent_prefill" if latent else "prefill_varlen"
     for n, ln in cases:
         times, probe = [], _EventProbe()
         for rep in range(reps + 2):
@@ -582,9 +615,10 @@ def prefill_records(engine, model, gpus=1, cases=PREFILL_CASES, reps=5):
             for s in seqs:
                 bm.allocate(s)
             probing = rep == reps + 1
-            real = hip_ops.prefill_varlen
+            real, real_ssm = getattr(hip_ops, entry), hip_ops.ssm_prefill
             if probing:
-                attn_mod.hip_ops.prefill_varlen = probe.wrap("prefill", real)
+                setattr(attn_mod.hip_ops, entry, probe.wrap("prefill", real))
+                attn_mod.hip_ops.ssm_prefill = probe.wrap("ssm", real_ssm)
             try:
                 torch.cuda.synchronize()
                 t0 = time.perf_counter()
@@ -592,7 +626,8 @@ def prefill_records(engine, model, gpus=1, cases=PREFILL_CASES, reps=5):
                 torch.cuda.synchronize()
                 dt = time.perf_counter() - t0
             finally:
-                attn_mod.hip_ops.prefill_varlen = real
+                setattr(attn_mod.hip_ops, entry, real)
+                attn_mod.hip_ops.ssm_prefill = real_ssm
             for s in seqs:
                 bm.deallocate(s)
             if rep and not probing:
@@ -602,19 +637,31 @@ def prefill_records(engine, model, gpus=1, cases=PREFILL_CASES, reps=5):
         m = statistics.median(t_us)
         kept = [t for t in t_us if t <= 3 * m]
         us = sum(kept) / len(kept)
-        flops = prefill_flops(heads, head_dim, [ln] * n, cfgm.get("chunk", 0))
+        if latent:     # expanded form: scores over dim + rot columns, values of vdim columns, keys inside the window
+            m0 = next(m for m in ex.model.modules() if hasattr(m, "row_cols"))
+            seen = n * sum(min(i + 1, m0.window or ln) for i in range(ln))
+            flops = seen * m0.heads * 2 * (m0.dq + m0.dv)
+        else:
+            flops = prefill_flops(heads, head_dim, [ln] * n, cfgm.get("chunk", 0))
         tf = flops / us / 1e6
         out.append({"metric": "prefill tokens/s", "model": model, "tp": gpus, "prompts": n, "prompt_len": ln,
                     "batches_timed": reps, "warmup_batches": 1, "ms_per_batch": round(med * 1e3, 3),
                     "value": round(n * ln / med, 1), "unit": "tokens/s",
                     "timing": "wall clock around execute_batch(prefill=True) bracketed by torch.cuda.synchronize(), median",
-                    "roofline": {"bound": "mfma", "kernel": "prefill_mfma_kernel", "achieved": round(tf, 1),
+                    "roofline": {"bound": "mfma", "kernel": "latent_prefill_kernel" if latent else "prefill_mfma_kernel", "achieved": round(tf, 1),
                                  "peak": MFMA_PEAK_TFLOPS, "unit": "TFLOP/s", "frac": round(tf / MFMA_PEAK_TFLOPS, 4),
                                  "traffic": None, "flops_per_launch": flops, "us_per_launch": round(us, 2),
                                  "launches_timed": len(kept), "heads_per_rank": heads,
                                  "share_of_step": round(us * len(t_us) / (med * 1e6), 4),
                                  "mfma_busy": busy, "mfma_busy_source": busy_src,
-                                 "timing": "HIP event pairs around every mv_prefill_varlen launch of one extra (untimed) batch, on the launching stream"}})
+                                 "timing": f"HIP event pairs around every mv_{entry} launch of one extra (untimed) batch, on the launching stream"}})
+        if ex.state_modules:
+            m0, t_ssm = ex.state_modules[0], sorted(probe.times_us("ssm"))
+            us = t_ssm[len(t_ssm) // 2]
+            byt = n * ln * (2 * m0.heads * m0.p + 2 * m0.groups * m0.n + m0.heads) * ex.dtype.itemsize
+            out[-1]["ssm_roofline"] = {"bound": "hbm", "kernel": "ssm_chunk_kernel", "bytes_per_launch": byt, "us_per_launch": round(us, 2),
+                                       "achieved": round(byt / us / 1e3, 1), "peak": HBM_PEAK_GBS, "unit": "GB/s",
+                                       "frac": round(byt / us / 1e3 / HBM_PEAK_GBS, 4)}
     return out
 
 
@@ -923,8 +970,8 @@ def init_process_group(args):
     return dist
 
 
-def attention_graph_roofline(engine, model) -> dict:
-    """The decode attention launches of one step (every layer run, on the running batch's tables, lengths and K/V planes, query
+def attention_graph_roofline(engine, model) -> tuple:
+    """-> (attention, state space step or None).  The decode attention launches of one step (every layer run, on the running batch's tables, lengths and K/V planes, query
     rows random) captured into a graph and replayed.  A design's small batches are launch-bound when run eagerly: event pairs
     around its launches would time the host."""
     from minivllm_amd import hip_ops
@@ -936,8 +983,10 @@ def attention_graph_roofline(engine, model) -> dict:
     torch.cuda.synchronize()
     ex._ship_decode(ex.builder.decode(seqs))
     ctx = get_context()
-    tables, lens = ctx.block_tables, ctx.context_lens
+    tables, lens, slots = ctx.block_tables, ctx.context_lens, ctx.state_slots
     reset_context()
+    if ex.latents:
+        return _latent_graph_roofline(ex, tables, lens), _state_graph_roofline(ex, lens, slots)
     mods = [m for m in ex.model.modules() if hasattr(m, "k_cache") and hasattr(m, "v_cache")]
     m0 = mods[0]
     q = torch.randn((len(seqs), m0.num_heads, m0.head_dim), device=ex.device).to(ex.dtype)
@@ -950,7 +999,47 @@ def attention_graph_roofline(engine, model) -> dict:
     algo = (sum(seen) * 2 * m0.num_kv_heads * m0.head_dim + 2 * q.numel()) * ex.dtype.itemsize
     return {"bound": "hbm", "achieved": round(algo / us / 1e3, 1), "peak": HBM_PEAK_GBS, "unit": "GB/s",
             "frac": round(algo / us / 1e3 / HBM_PEAK_GBS, 4), "bytes_per_launch": algo, "us_per_launch": round(us, 2),
-            "timing": f"{len(mods)} launches (split-KV combine included) captured into a hipGraph, median of 5 replays / launches"}
+            "timing": f"{len(mods)} launches (split-KV combine included) captured into a hipGraph, median of 5 replays / launches"}, None
+
+
+def _graph_roofline(byt: int, us: float, launches: int) -> dict:
+    return {"bound": "hbm", "achieved": round(byt / us / 1e3, 1), "peak": HBM_PEAK_GBS, "unit": "GB/s",
+            "frac": round(byt / us / 1e3 / HBM_PEAK_GBS, 4), "bytes_per_launch": byt, "us_per_launch": round(us, 2),
+            "timing": f"{launches} launches (merges included) captured into a hipGraph, median of 5 replays / launches"}
+
+
+def _latent_graph_roofline(ex, tables, lens) -> dict:
+    """mv_latent_decode of every attention layer on the running batch, query rows random."""
+    from minivllm_amd import hip_ops
+
+    mods = [m for m in ex.model.modules() if hasattr(m, "row_cols")]
+    m0, b = mods[0], lens.numel()
+    q = torch.randn((b, m0.heads, m0.row_cols), device=ex.device).to(ex.dtype)
+
+    def run():
+        for m in mods:
+            hip_ops.latent_decode(q, m.owner.latent_cache, tables, lens, m.kv_cols, m.scale, m.window)
+    us = _graph_time_us(run, len(mods))
+    seen = sum(min(n, m0.window or n) for n in lens.tolist())
+    return _graph_roofline((seen * m0.row_cols + q.numel() + b * m0.heads * m0.kv_cols) * ex.dtype.itemsize, us, len(mods))
+
+
+def _state_graph_roofline(ex, lens, slots) -> dict:
+    """mv_ssm_step of every state space layer on the running batch (a step that is run again gives the same state)."""
+    from minivllm_amd import hip_ops
+
+    mods, b = ex.state_modules, lens.numel()
+    m0 = mods[0]
+    z = torch.randn((b, m0.in_proj.weight.shape[0]), device=ex.device).to(ex.dtype)
+
+    def run():
+        for m in mods:
+            hip_ops.ssm_step(z[:, m.x_off:m.x_off + m.channels], z[:, m.dt_off:m.dt_off + m.heads], m.conv, m.conv_b, m.dt_bias, m.A_log,
+                             m.D, m.shape, m.conv_state, m.ssm_state, slots, lens)
+    us = _graph_time_us(run, len(mods))
+    byt = 2 * b * (m0.ssm_state[0, 0].numel() * 4 + m0.conv_state[0, 0].numel() * ex.dtype.itemsize)
+    byt += b * (m0.channels + m0.heads + m0.heads * m0.p) * ex.dtype.itemsize
+    return _graph_roofline(byt, us, len(mods))
 
 
 def design_records(args, workdir) -> dict:
@@ -970,7 +1059,9 @@ def design_records(args, workdir) -> dict:
             for i, (batch, ctx) in enumerate(DESIGN_DECODE):
                 a.batch, a.ctx = batch, ctx
                 rec, _ = decode_record(engine, a, model, None, seed=i, probes=False)
-                rec["roofline"] = attention_graph_roofline(engine, model)
+                rec["roofline"], state = attention_graph_roofline(engine, model)
+                if state is not None:
+                    rec["state_roofline"] = state
                 rec["step_roofline"] = step_roofline(engine, model, batch, ctx + a.warmup + a.steps // 2, rec["ms_per_step"])
                 recs.append(rec)
                 release_all(engine)
@@ -995,6 +1086,7 @@ def design_line(args, records: dict) -> dict:
             pairs.append({"model": name, "peer": like, "workload": what, "tokens_per_s": [mine["value"], peer["value"]],
                           "ratio": round(mine["value"] / peer["value"], 4),
                           "attention_frac_of_peak": [mine["roofline"]["frac"], peer["roofline"]["frac"]],
+                          "state_frac_of_peak": (mine.get("state_roofline") or mine.get("ssm_roofline") or {}).get("frac"),
                           "step_frac_of_hbm_peak": [(r.get("step_roofline") or {}).get("frac") for r in (mine, peer)]})
     last = list(DESIGNS[args.design])[-1]
     head = records[last][0]

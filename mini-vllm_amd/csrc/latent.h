@@ -13,6 +13,17 @@ __device__ __forceinline__ f32x4 mfma16x16x32(const u32x4 &a, const u32x4 &b, co
     return __builtin_amdgcn_mfma_f32_16x16x32_f16(__builtin_bit_cast(mv_f16x8, a), __builtin_bit_cast(mv_f16x8, b), c, 0, 0, 0);
 }
 
+// two fp32 -> two 16-bit values in one register (one conversion instruction)
+template <typename Tag>
+__device__ __forceinline__ uint32_t pack_pair(float lo, float hi) {
+  if constexpr (__is_same(Tag, bf16_tag))
+    return __builtin_bit_cast(uint32_t, __builtin_convertvector(f32x2{lo, hi}, bf16x2_t));
+  else
+    return __builtin_bit_cast(uint32_t, __builtin_convertvector(f32x2{lo, hi}, f16x2_t));
+}
+template <typename Tag>
+__device__ __forceinline__ u32x2 pack_quad(const f32x4 &v) { return u32x2{pack_pair<Tag>(v[0], v[1]), pack_pair<Tag>(v[2], v[3])}; }
+
 // one 16-byte vector of a row
 template <typename Tag>
 __device__ __forceinline__ void load_vec_row(const typename elem<Tag>::T *p, float (&f)[elem<Tag>::VEC]) {

@@ -83,15 +83,14 @@ __global__ void __launch_bounds__(256) latent_prep_kernel(MvLatentPrepArgs p) {
   }
 }
 
-// rotated part of 64 tokens of one head: out[t, h, n ..] = rotation of x[t, h, k ..]
+// rotated part of tokens t0 .. end - 1 of one head: out[t, h, n ..] = rotation of x[t, h, k ..]
 template <typename Tag>
-__device__ __forceinline__ void head_rotation(const MvHeadLinearArgs &p, int head, int t0, int n_tok) {
+__device__ __forceinline__ void head_rotation(const MvHeadLinearArgs &p, int head, int t0, int end) {
   typedef typename elem<Tag>::T T;
   constexpr int VEC = elem<Tag>::VEC;
   const int per = p.rot_cols / VEC;
-  for (int i = threadIdx.x; i < 64 * per; i += 256) {
+  for (int i = threadIdx.x; i < (end - t0) * per; i += 256) {
     const int t = t0 + i / per, c = i % per * VEC;
-    if (t >= n_tok) continue;
     float f[VEC];
     load_vec_row<Tag>((const T *)p.x + t * p.x_tok + head * p.x_head + p.k + c, f);
     const int64_t pos = p.positions[t];
@@ -100,45 +99,58 @@ __device__ __forceinline__ void head_rotation(const MvHeadLinearArgs &p, int hea
   }
 }
 
-// 64 tokens x 64 outputs of one head per workgroup: wave w computes outputs 16 w .. 16 w + 15.  Both operands come straight
-// from memory in fragment order (a lane's 8 consecutive k), W rows as A, token rows as B.
-template <typename Tag>
+// 16 TT tokens x 64 outputs of one head per workgroup: wave w computes outputs 16 w .. 16 w + 15.  Both operands come straight
+// from memory in fragment order (a lane's 8 consecutive k), W rows as A, token rows as B; the loads of the next 128 k are in
+// flight while the current ones are multiplied.
+template <typename Tag, int TT>
 __global__ void __launch_bounds__(256) head_linear_mfma_kernel(MvHeadLinearArgs p, int n_tiles, int n_tok) {
   typedef typename elem<Tag>::T T;
-  const int head = blockIdx.y, t0 = blockIdx.z * 64;
-  if ((int)blockIdx.x == n_tiles) return head_rotation<Tag>(p, head, t0, n_tok);
+  const int head = blockIdx.y, t0 = blockIdx.z * (16 * TT);
+  if ((int)blockIdx.x == n_tiles) return head_rotation<Tag>(p, head, t0, min(n_tok, t0 + 16 * TT));
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r16 = lane & 15, g = lane >> 4;
   const int n0 = (int)blockIdx.x * 64 + wave * 16;
   if (n0 >= p.n) return;
   const T *w = (const T *)p.w + ((int64_t)head * p.n + n0 + r16) * p.k + g * 8;
-  const T *x[4];
+  const T *x[TT];
 #pragma unroll
-  for (int b = 0; b < 4; ++b) {
-    const int t = t0 + b * 16 + r16;
-    x[b] = (const T *)p.x + (int64_t)(t < n_tok ? t : n_tok - 1) * p.x_tok + head * p.x_head + g * 8;
+  for (int b = 0; b < TT; ++b)
+    x[b] = (const T *)p.x + (int64_t)min(t0 + b * 16 + r16, n_tok - 1) * p.x_tok + head * p.x_head + g * 8;
+  u32x4 wa[2][4], xa[2][TT][4];
+  auto load = [&](int set, int k0) {   // (steps behind the end: weights of zero, x of the last step)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int k = min(k0 + 32 * i, p.k - 32);
+      wa[set][i] = *(const u32x4 *)(w + k);
+      if (k0 + 32 * i >= p.k) wa[set][i] = u32x4{0u, 0u, 0u, 0u};
+#pragma unroll
+      for (int b = 0; b < TT; ++b) xa[set][b][i] = *(const u32x4 *)(x[b] + k);
+    }
+  };
+  f32x4 acc[TT] = {};
+  auto multiply = [&](int set) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int b = 0; b < TT; ++b) acc[b] = mfma16x16x32<Tag>(wa[set][i], xa[set][b][i], acc[b]);
+  };
+  load(0, 0);
+  for (int k = 0; k < p.k; k += 256) {
+    if (k + 128 < p.k) load(1, k + 128);
+    multiply(0);
+    if (k + 256 < p.k) load(0, k + 256);
+    if (k + 128 < p.k) multiply(1);
   }
-  const int tiles = min(4, (n_tok - t0 + 15) / 16);
-  f32x4 acc[4] = {};
-  for (int k = 0; k < p.k; k += 32) {
-    const u32x4 a = *(const u32x4 *)(w + k);
 #pragma unroll
-    for (int b = 0; b < 4; ++b)
-      if (b < tiles) acc[b] = mfma16x16x32<Tag>(a, *(const u32x4 *)(x[b] + k), acc[b]);
-  }
-#pragma unroll
-  for (int b = 0; b < 4; ++b) {
+  for (int b = 0; b < TT; ++b) {
     const int t = t0 + b * 16 + r16;
-    if (t >= n_tok) continue;
-    T *o = (T *)p.out + (int64_t)t * p.out_tok + head * p.out_head + n0 + g * 4;
-    *(u32x2 *)o = u32x2{(uint32_t)elem<Tag>::st(acc[b][0]) | ((uint32_t)elem<Tag>::st(acc[b][1]) << 16),
-                        (uint32_t)elem<Tag>::st(acc[b][2]) | ((uint32_t)elem<Tag>::st(acc[b][3]) << 16)};
+    if (t < n_tok) *(u32x2 *)((T *)p.out + (int64_t)t * p.out_tok + head * p.out_head + n0 + g * 4) = pack_quad<Tag>(acc[b]);
   }
 }
 
 // one output per thread, fp32
 __global__ void __launch_bounds__(256) head_linear_f32_kernel(MvHeadLinearArgs p, int n_tiles, int n_tok) {
   const int head = blockIdx.y, t0 = blockIdx.z * 64;
-  if ((int)blockIdx.x == n_tiles) return head_rotation<f32_tag>(p, head, t0, n_tok);
+  if ((int)blockIdx.x == n_tiles) return head_rotation<f32_tag>(p, head, t0, min(n_tok, t0 + 64));
   for (int i = threadIdx.x; i < 64 * 64; i += 256) {
     const int t = t0 + i / 64, n = (int)blockIdx.x * 64 + i % 64;
     if (t >= n_tok || n >= p.n) continue;
@@ -208,14 +220,25 @@ extern "C" int mv_head_linear(const MvHeadLinearArgs *a, int n_tok, int dtype, v
   if (!mv_aligned16(a->x) || !mv_aligned16(a->w) || !mv_aligned16(a->out) || a->x_tok % vec || a->x_head % vec ||
       a->out_tok % vec || a->out_head % vec)
     return MV_E_ALIGN;
-  const int n_tiles = (a->n + 63) / 64, z = (n_tok + 63) / 64;
+  const int n_tiles = (a->n + 63) / 64, x = n_tiles + (a->rot_dim ? 1 : 0);
+  // token tiles per workgroup: a tile of weights is read once per workgroup, but the chip should be full
+  int tt = 4;
+  while (dtype != MV_F32 && tt > 1 && (n_tok <= 8 * tt || (int64_t)x * a->heads * ((n_tok + 16 * tt - 1) / (16 * tt)) < 512)) tt /= 2;
+  const int z = (n_tok + 16 * tt - 1) / (16 * tt);
   if (z > 65535) return MV_E_SHAPE;
-  const dim3 grid(n_tiles + (a->rot_dim ? 1 : 0), a->heads, z), block(256);
+  const dim3 grid(x, a->heads, z), block(256);
   hipStream_t st = (hipStream_t)stream;
-  if (dtype == MV_BF16) hipLaunchKernelGGL((head_linear_mfma_kernel<bf16_tag>), grid, block, 0, st, *a, n_tiles, n_tok);
-  else if (dtype == MV_F16) hipLaunchKernelGGL((head_linear_mfma_kernel<f16_tag>), grid, block, 0, st, *a, n_tiles, n_tok);
+#define MV_HL(TAG)                                                                                                       \
+  do {                                                                                                                   \
+    if (tt == 4) hipLaunchKernelGGL((head_linear_mfma_kernel<TAG, 4>), grid, block, 0, st, *a, n_tiles, n_tok);          \
+    else if (tt == 2) hipLaunchKernelGGL((head_linear_mfma_kernel<TAG, 2>), grid, block, 0, st, *a, n_tiles, n_tok);     \
+    else hipLaunchKernelGGL((head_linear_mfma_kernel<TAG, 1>), grid, block, 0, st, *a, n_tiles, n_tok);                  \
+  } while (0)
+  if (dtype == MV_BF16) MV_HL(bf16_tag);
+  else if (dtype == MV_F16) MV_HL(f16_tag);
   else if (dtype == MV_F32) hipLaunchKernelGGL(head_linear_f32_kernel, grid, block, 0, st, *a, n_tiles, n_tok);
   else return MV_E_DTYPE;
+#undef MV_HL
   MV_LAUNCH_CHECK();
   return MV_OK;
 }

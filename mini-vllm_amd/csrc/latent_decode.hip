@@ -28,18 +28,17 @@ struct DecodeParams {
   float scale;
 };
 
-__host__ __device__ __forceinline__ int lds_chunks(int cols) { return cols / 8 + 1 - (cols / 8 & 1); }   // odd
+__host__ __device__ constexpr int lds_chunks(int cols) { return cols / 8 + 1 - (cols / 8 & 1); }   // odd
 
-// CT: latent column tiles of 16 per wave (kv_cols <= 64 CT)
-template <typename Tag, int HG, int CT>
+// CT: latent column tiles of 16 per wave (kv_cols = 64 CT); RT: rotated columns / 32
+template <typename Tag, int HG, int CT, int RT>
 __global__ void __launch_bounds__(256, 2) latent_decode_kernel(DecodeParams p) {
   typedef typename elem<Tag>::T T;
-  constexpr int KSM = 2 * CT + kMaxRot / 32;   // 32-column steps of a row
+  constexpr int KS = 2 * CT + RT, COLS = KS * 32, CH = lds_chunks(COLS), RB = CH * 16;   // 32-column steps of a row; its LDS form
+  constexpr int DMAS = (TK * CH + 63) / 64, BUF = DMAS * 1024;
   extern __shared__ __attribute__((aligned(16))) char smem[];
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), r16 = lane & 15, g = lane >> 4;
   const int split = blockIdx.x, h0 = blockIdx.y * 16 * HG, b = blockIdx.z;
-  const int CH = lds_chunks(p.cols), RB = CH * 16, ks = p.cols / 32, cts = p.kv_cols / 64;
-  const int dmas = (TK * CH + 63) / 64, BUF = dmas * 1024;
   float *smax = (float *)(smem + 2 * BUF);                      // [2 key halves][16 HG heads]
   char *prob = (char *)(smax + 2 * 16 * HG);                    // [16 HG heads][TK] 16-bit, rows of 80 bytes
   constexpr int PR = 80;
@@ -49,12 +48,11 @@ __global__ void __launch_bounds__(256, 2) latent_decode_kernel(DecodeParams p) {
 
   // Q^T fragments of this wave's heads
   const int kg = wave & 1, hg = HG == 2 ? wave >> 1 : 0, qh = h0 + hg * 16 + r16;
-  u32x4 qf[KSM];
+  u32x4 qf[KS];
   {
-    const T *qp = (const T *)p.q + ((int64_t)b * p.heads + min(qh, p.heads - 1)) * p.cols + g * 8;
+    const T *qp = (const T *)p.q + ((int64_t)b * p.heads + min(qh, p.heads - 1)) * COLS + g * 8;
 #pragma unroll
-    for (int s = 0; s < KSM; ++s)
-      if (s < ks) qf[s] = *(const u32x4 *)(qp + s * 32);
+    for (int s = 0; s < KS; ++s) qf[s] = *(const u32x4 *)(qp + s * 32);
   }
   f32x4 acc[HG][CT] = {};
   float m_run[HG], l_run[HG];
@@ -67,17 +65,19 @@ __global__ void __launch_bounds__(256, 2) latent_decode_kernel(DecodeParams p) {
     const int blk = t < t1 ? p.tables[b * p.table_stride + t * TK / p.block_size] : -1;
     return blk >= 0 && blk < p.num_blocks ? blk : -1;
   };
-  const int q256 = 256 / CH, r256 = 256 % CH, row_first = (wave * 64 + lane) / CH, col_first = (wave * 64 + lane) % CH;
+  const int row_first = (wave * 64 + lane) / CH, col_first = (wave * 64 + lane) % CH;
   auto dma = [&](int t, int blk, int buf) {
     if (blk < 0) return;
-    const T *src = (const T *)p.plane + ((int64_t)blk * p.block_size + t * TK % p.block_size) * p.cols;
+    const T *src = (const T *)p.plane + ((int64_t)blk * p.block_size + t * TK % p.block_size) * COLS;
     const int last = min(TK, len - t * TK) - 1;   // rows past the end re-read the last key (probability 0, finite data)
     int row = row_first, col = col_first;
-    for (int i = wave; i < dmas; i += 4) {
-      __builtin_amdgcn_global_load_lds(
-          (const __attribute__((address_space(1))) void *)(src + (int64_t)min(row, last) * p.cols + min(col, p.cols / 8 - 1) * 8),
-          (__attribute__((address_space(3))) void *)(smem + buf * BUF + i * 1024), 16, 0, 0);
-      row += q256, col += r256;
+#pragma unroll
+    for (int i = 0; i < (DMAS + 3) / 4; ++i) {
+      if (4 * i + wave < DMAS)
+        __builtin_amdgcn_global_load_lds(
+            (const __attribute__((address_space(1))) void *)(src + (min(row, last) * COLS + min(col, COLS / 8 - 1) * 8)),
+            (__attribute__((address_space(3))) void *)(smem + buf * BUF + (4 * i + wave) * 1024), 16, 0, 0);
+      row += 256 / CH, col += 256 % CH;
       if (col >= CH) col -= CH, ++row;
     }
   };
@@ -93,11 +93,14 @@ __global__ void __launch_bounds__(256, 2) latent_decode_kernel(DecodeParams p) {
     if (blk >= 0) {
       const char *tile = smem + buf * BUF;
       // ---- scores: 16 keys x 16 heads
-      f32x4 s = {0.f, 0.f, 0.f, 0.f};
+      f32x4 s = {0.f, 0.f, 0.f, 0.f}, s2 = {0.f, 0.f, 0.f, 0.f};   // (two chains: half the dependent latency)
       const char *ka = tile + (kg * 16 + r16) * RB + g * 16;
 #pragma unroll
-      for (int i = 0; i < KSM; ++i)
-        if (i < ks) s = mfma16x16x32<Tag>(*(const u32x4 *)(ka + i * 64), qf[i], s);
+      for (int i = 0; i < KS; i += 2) {
+        s = mfma16x16x32<Tag>(*(const u32x4 *)(ka + i * 64), qf[i], s);
+        if (i + 1 < KS) s2 = mfma16x16x32<Tag>(*(const u32x4 *)(ka + i * 64 + 64), qf[i + 1], s2);
+      }
+      s += s2;
       float mx = -INFINITY;
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
@@ -125,8 +128,7 @@ __global__ void __launch_bounds__(256, 2) latent_decode_kernel(DecodeParams p) {
       else l_run[0] += sum;
       if (HG == 2 || wave < 2)
         *(u32x2 *)(prob + (hg * 16 + r16) * PR + (kg * 16 + g * 4) * 2) =
-            u32x2{(uint32_t)elem<Tag>::st(e[0]) | ((uint32_t)elem<Tag>::st(e[1]) << 16),
-                  (uint32_t)elem<Tag>::st(e[2]) | ((uint32_t)elem<Tag>::st(e[3]) << 16)};
+            u32x2{pack_pair<Tag>(e[0], e[1]), pack_pair<Tag>(e[2], e[3])};
       __syncthreads();
       // ---- values
       u32x4 pf[HG];
@@ -134,8 +136,7 @@ __global__ void __launch_bounds__(256, 2) latent_decode_kernel(DecodeParams p) {
       for (int i = 0; i < HG; ++i) pf[i] = *(const u32x4 *)(prob + (i * 16 + r16) * PR + g * 16);
       const char *va = tile + (g * 8 + (r16 >> 2)) * RB + (r16 & 3) * 8 + wave * 32;
 #pragma unroll
-      for (int c = 0; c < CT; ++c)
-        if (c < cts) {
+      for (int c = 0; c < CT; ++c) {
           const u32x2 a0 = __builtin_bit_cast(u32x2, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4 *)(va + c * 128)));
           const u32x2 a1 = __builtin_bit_cast(u32x2, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4 *)(va + 4 * RB + c * 128)));
           const u32x4 a = {a0.x, a0.y, a1.x, a1.y};
@@ -166,15 +167,11 @@ __global__ void __launch_bounds__(256, 2) latent_decode_kernel(DecodeParams p) {
       const float inv = l > 0.f ? 1.0f / l : 0.f;
       T *o = (T *)p.out + row * p.kv_cols + wave * 16 + g * 4;
 #pragma unroll
-      for (int c = 0; c < CT; ++c)
-        if (c < cts)
-          *(u32x2 *)(o + c * 64) = u32x2{(uint32_t)elem<Tag>::st(acc[i][c][0] * inv) | ((uint32_t)elem<Tag>::st(acc[i][c][1] * inv) << 16),
-                                         (uint32_t)elem<Tag>::st(acc[i][c][2] * inv) | ((uint32_t)elem<Tag>::st(acc[i][c][3] * inv) << 16)};
+      for (int c = 0; c < CT; ++c) *(u32x2 *)(o + c * 64) = pack_quad<Tag>(acc[i][c] * inv);
     } else {
       float *o = p.part + (row * p.splits + split) * p.kv_cols + wave * 16 + g * 4;
 #pragma unroll
-      for (int c = 0; c < CT; ++c)
-        if (c < cts) *(f32x4 *)(o + c * 64) = acc[i][c];
+      for (int c = 0; c < CT; ++c) *(f32x4 *)(o + c * 64) = acc[i][c];
       if (wave == 0 && g == 0) {
         float *ml = p.part_ml + (row * p.splits + split) * 2;
         ml[0] = m_run[i], ml[1] = l;
@@ -183,26 +180,40 @@ __global__ void __launch_bounds__(256, 2) latent_decode_kernel(DecodeParams p) {
   }
 }
 
+// one (sequence, head) per workgroup: 4 columns per thread, the parts dealt to blockDim.x / (kv_cols / 4) groups of threads
 template <typename Tag>
-__global__ void __launch_bounds__(256) latent_merge_kernel(const float *part, const float *part_ml, void *out, int rows, int splits,
-                                                           int kv_cols) {
+__global__ void __launch_bounds__(256) latent_merge_kernel(const float *part, const float *part_ml, void *out, int splits, int kv_cols) {
   typedef typename elem<Tag>::T T;
-  const int per = kv_cols / 4, idx = blockIdx.x * 256 + threadIdx.x, row = idx / per, c = idx % per * 4;
-  if (row >= rows) return;
-  const float *ml = part_ml + (int64_t)row * splits * 2;
-  float m = -1e30f, l = 0.f;
-  for (int s = 0; s < splits; ++s) m = fmaxf(m, ml[2 * s]);
-  f32x4 o = {0.f, 0.f, 0.f, 0.f};
-  for (int s = 0; s < splits; ++s) {
-    if (!(ml[2 * s + 1] > 0.f)) continue;
-    const float w = __builtin_amdgcn_exp2f(ml[2 * s] - m);
-    l = fmaf(ml[2 * s + 1], w, l);
-    o += *(const f32x4 *)(part + ((int64_t)row * splits + s) * kv_cols + c) * w;
+  __shared__ float w[kMaxSplits];
+  __shared__ f32x4 sums[256];
+  const int64_t row = blockIdx.x;
+  const int tid = threadIdx.x, per = kv_cols / 4, groups = 256 / per, c = tid % per, first = tid / per;
+  float total;
+  {
+    const float *ml = part_ml + row * splits * 2;
+    const int lane = tid & 63;      // (kMaxSplits = one wave)
+    const float m = lane < splits ? ml[2 * lane] : -1e30f, l = lane < splits ? ml[2 * lane + 1] : 0.f;
+    const float top = wave_max(l > 0.f ? m : -1e30f);   // (all lanes take part)
+    const float e = l > 0.f ? __builtin_amdgcn_exp2f(m - top) : 0.f;
+    total = wave_sum(l * e);
+    if (tid < splits) w[tid] = e;
   }
-  const float inv = l > 0.f ? 1.0f / l : 0.f;
-  *(u32x2 *)((T *)out + (int64_t)row * kv_cols + c) =
-      u32x2{(uint32_t)elem<Tag>::st(o[0] * inv) | ((uint32_t)elem<Tag>::st(o[1] * inv) << 16),
-            (uint32_t)elem<Tag>::st(o[2] * inv) | ((uint32_t)elem<Tag>::st(o[3] * inv) << 16)};
+  __syncthreads();
+  f32x4 o = {0.f, 0.f, 0.f, 0.f};
+  if (first < groups) {
+    const float *p = part + row * splits * kv_cols + 4 * c;
+#pragma unroll 4
+    for (int s = first; s < splits; s += groups) {
+      const f32x4 v = *(const f32x4 *)(p + (int64_t)s * kv_cols);
+      o += w[s] > 0.f ? v * w[s] : f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+  }
+  sums[tid] = o;
+  __syncthreads();
+  if (tid < per) {
+    for (int i = 1; i < groups; ++i) o += sums[i * per + tid];
+    *(u32x2 *)((T *)out + row * kv_cols + 4 * c) = pack_quad<Tag>(o * (total > 0.f ? 1.0f / total : 0.f));
+  }
 }
 
 int head_groups(int heads) { return heads > 16 ? 2 : 1; }
@@ -221,16 +232,23 @@ int split_count(int batch, int heads, int block_size, int max_blocks, int window
 
 template <typename Tag, int HG>
 int launch(const DecodeParams &p, const dim3 &grid, size_t lds, hipStream_t stream) {
-#define MV_LD(CT_)                                                                                          \
-  if (p.kv_cols <= 64 * CT_) {                                                                              \
-    if (int e = mv_allow_lds<&latent_decode_kernel<Tag, HG, CT_>>()) return e;                              \
-    hipLaunchKernelGGL((latent_decode_kernel<Tag, HG, CT_>), grid, dim3(256), lds, stream, p);               \
+#define MV_LD(CT_, RT_)                                                                                     \
+  if (p.kv_cols == 64 * CT_ && p.cols - p.kv_cols == 32 * RT_) {                                            \
+    if (int e = mv_allow_lds<&latent_decode_kernel<Tag, HG, CT_, RT_>>()) return e;                         \
+    hipLaunchKernelGGL((latent_decode_kernel<Tag, HG, CT_, RT_>), grid, dim3(256), lds, stream, p);          \
     MV_LAUNCH_CHECK();                                                                                      \
     return MV_OK;                                                                                           \
   }
-  MV_LD(2)
-  MV_LD(4)
-  MV_LD(8)
+#define MV_LDR(CT_) MV_LD(CT_, 1) MV_LD(CT_, 2)
+  MV_LDR(1)
+  MV_LDR(2)
+  MV_LDR(3)
+  MV_LDR(4)
+  MV_LDR(5)
+  MV_LDR(6)
+  MV_LDR(7)
+  MV_LDR(8)
+#undef MV_LDR
 #undef MV_LD
   return MV_E_SHAPE;
 }
@@ -264,11 +282,10 @@ int mv_latent_decode_mfma_launch(const void *q, const void *plane, const int32_t
   else rc = hg == 2 ? launch<f16_tag, 2>(p, grid, lds, stream) : launch<f16_tag, 1>(p, grid, lds, stream);
   if (rc != MV_OK || splits == 1) return rc;
   const int rows = batch * heads;
-  const dim3 mgrid((rows * (kv_cols / 4) + 255) / 256);
   if (dtype == MV_BF16)
-    hipLaunchKernelGGL((latent_merge_kernel<bf16_tag>), mgrid, dim3(256), 0, stream, p.part, p.part_ml, out, rows, splits, kv_cols);
+    hipLaunchKernelGGL((latent_merge_kernel<bf16_tag>), dim3(rows), dim3(256), 0, stream, p.part, p.part_ml, out, splits, kv_cols);
   else
-    hipLaunchKernelGGL((latent_merge_kernel<f16_tag>), mgrid, dim3(256), 0, stream, p.part, p.part_ml, out, rows, splits, kv_cols);
+    hipLaunchKernelGGL((latent_merge_kernel<f16_tag>), dim3(rows), dim3(256), 0, stream, p.part, p.part_ml, out, splits, kv_cols);
   MV_LAUNCH_CHECK();
   return MV_OK;
 }

@@ -27,14 +27,6 @@ __device__ __forceinline__ f32x16 mfma32(const u32x4 &a, const u32x4 &b, const f
   else
     return __builtin_amdgcn_mfma_f32_32x32x16_f16(__builtin_bit_cast(mv_f16x8, a), __builtin_bit_cast(mv_f16x8, b), c, 0, 0, 0);
 }
-template <typename Tag>
-__device__ __forceinline__ uint32_t pack2(float lo, float hi) {
-  if constexpr (__is_same(Tag, bf16_tag))
-    return __builtin_bit_cast(uint32_t, __builtin_convertvector(f32x2{lo, hi}, bf16x2_t));
-  else
-    return __builtin_bit_cast(uint32_t, __builtin_convertvector(f32x2{lo, hi}, f16x2_t));
-}
-
 // chunk swizzles (XOR): rows of a multiple of 256 bytes all start in the same bank, other multiples of 128 in two
 template <int CH> __device__ __forceinline__ int k_swz(int row) { return CH % 16 == 0 ? (row & 15) : ((row >> 1) & 7); }
 template <int CH> __device__ __forceinline__ int v_swz(int row) {
@@ -207,7 +199,7 @@ __global__ void __launch_bounds__(NW * 64, 2) latent_prefill_kernel(MvLatentPref
         for (int s2 = 0; s2 < 2; ++s2) {
           u32x4 pf;
 #pragma unroll
-          for (int j = 0; j < 4; ++j) pf[j] = pack2<Tag>(sacc[kt][8 * s2 + 2 * j], sacc[kt][8 * s2 + 2 * j + 1]);
+          for (int j = 0; j < 4; ++j) pf[j] = pack_pair<Tag>(sacc[kt][8 * s2 + 2 * j], sacc[kt][8 * s2 + 2 * j + 1]);
           const char *vb = smem + BO + KB + (kt * 32 + 16 * s2) * (DV * 2);
 #pragma unroll
           for (int dt = 0; dt < NDT; ++dt) {
@@ -237,7 +229,7 @@ __global__ void __launch_bounds__(NW * 64, 2) latent_prefill_kernel(MvLatentPref
 #pragma unroll
     for (int c = 0; c < 4; ++c)
       *reinterpret_cast<u32x2 *>(stage + r * (DV * 2) + (((4 * dt + c) ^ (r & MASK)) << 4) + 8 * h) =
-          u32x2{pack2<Tag>(oacc[dt][4 * c] * inv, oacc[dt][4 * c + 1] * inv), pack2<Tag>(oacc[dt][4 * c + 2] * inv, oacc[dt][4 * c + 3] * inv)};
+          u32x2{pack_pair<Tag>(oacc[dt][4 * c] * inv, oacc[dt][4 * c + 1] * inv), pack_pair<Tag>(oacc[dt][4 * c + 2] * inv, oacc[dt][4 * c + 3] * inv)};
   const int row0 = qb * BM + wave * 32;
 #pragma unroll
   for (int it = 0; it < CV / 2; ++it) {

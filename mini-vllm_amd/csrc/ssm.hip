@@ -11,7 +11,7 @@ template <typename Tag>
 __device__ __forceinline__ float param(const void *p, int i) { return elem<Tag>::ld(((const typename elem<Tag>::T *)p)[i]); }
 
 // ---- convolution: 8 (fp32: 4) channels per thread, kConvRows tokens per workgroup, a sliding window of inputs in registers
-constexpr int kConvRows = 32, kMaxTaps = 8;
+constexpr int kConvRows = 32, kConvAhead = 8, kMaxTaps = 8;
 
 template <typename Tag, int TAPS>
 __global__ void __launch_bounds__(64) causal_conv_kernel(MvSsmArgs p) {
@@ -57,22 +57,33 @@ __global__ void __launch_bounds__(64) causal_conv_kernel(MvSsmArgs p) {
       if (j < back) store_vec_row<Tag>(ns + (int64_t)j * p.channels, last[j]);
   }
   const int t1 = min(len, t0 + kConvRows);
-  for (int t = t0; t < t1; ++t) {
-    float o[VEC];
+  for (int tb = t0; tb < t1; tb += kConvAhead) {
+    u32x4 raw[kConvAhead];
 #pragma unroll
-    for (int i = 0; i < TAPS - 1; ++i)
+    for (int u = 0; u < kConvAhead; ++u) raw[u] = *(const u32x4 *)(x + (int64_t)min(tb + u, len - 1) * p.x_stride);
 #pragma unroll
-      for (int j = 0; j < VEC; ++j) win[i][j] = win[i + 1][j];
-    load_vec_row<Tag>(x + (int64_t)t * p.x_stride, win[TAPS - 1]);
+    for (int u = 0; u < kConvAhead; ++u) {
+      float o[VEC];
 #pragma unroll
-    for (int j = 0; j < VEC; ++j) o[j] = bias[j];
+      for (int i = 0; i < TAPS - 1; ++i)
 #pragma unroll
-    for (int i = 0; i < TAPS; ++i)
+        for (int j = 0; j < VEC; ++j) win[i][j] = win[i + 1][j];
+      if constexpr (VEC == 8) {
+        unpack8<Tag>(raw[u], win[TAPS - 1]);
+      } else {
 #pragma unroll
-      for (int j = 0; j < VEC; ++j) o[j] = fmaf(win[i][j], w[i][j], o[j]);
+        for (int j = 0; j < VEC; ++j) win[TAPS - 1][j] = u2f(raw[u][j]);
+      }
 #pragma unroll
-    for (int j = 0; j < VEC; ++j) o[j] = silu_f32(o[j]);
-    store_vec_row<Tag>((T *)p.out + (int64_t)(q0 + t) * p.out_stride + c, o);
+      for (int j = 0; j < VEC; ++j) o[j] = bias[j];
+#pragma unroll
+      for (int i = 0; i < TAPS; ++i)
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) o[j] = fmaf(win[i][j], w[i][j], o[j]);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) o[j] = silu_of<Tag>(o[j]);
+      if (tb + u < t1) store_vec_row<Tag>((T *)p.out + (int64_t)(q0 + tb + u) * p.out_stride + c, o);
+    }
   }
 }
 
@@ -137,8 +148,11 @@ __global__ void __launch_bounds__(256) ssm_scan_kernel(MvSsmArgs p) {
   }
 }
 
-// ---- one token: workgroup = (head, sequence).  The convolution of the head's columns and of its group's b and c first (a few
-// hundred channels), then the state [n][p] in 16-byte pieces, each read, updated, multiplied into y and written once.
+// ---- one token: workgroup = (head, sequence).  The state [n][p] is requested first (up to kStepAhead 16-byte pieces per
+// thread); under that, the convolution of the head's columns and of its group's b and c (a few hundred channels); then each piece
+// of state is updated, multiplied into y and written once.
+constexpr int kStepAhead = 8;
+
 template <typename Tag>
 __global__ void __launch_bounds__(256) ssm_step_kernel(MvSsmArgs p) {
   typedef typename elem<Tag>::T T;
@@ -151,6 +165,18 @@ __global__ void __launch_bounds__(256) ssm_step_kernel(MvSsmArgs p) {
     return;
   }
   const bool keep = slot >= 0 && slot < p.slots, have = keep && before > 0;
+  const int64_t size = (int64_t)p.heads * p.n * p.p, at = (int64_t)(keep ? slot : 0) * size + (int64_t)head * p.n * p.p;
+  const f32x4 *os = (const f32x4 *)(p.ssm_state + (before & 1) * p.slots * size + at);
+  f32x4 *ns = (f32x4 *)(p.ssm_state + ((before + 1) & 1) * p.slots * size + at);
+  const int p4 = p.p / 4, rows = 256 / p4;   // threads across a state row; state rows per trip
+  const int c4 = tid % p4, r0 = tid / p4;
+  const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+  f32x4 v[kStepAhead];
+#pragma unroll
+  for (int i = 0; i < kStepAhead; ++i) {
+    const int r = r0 + i * rows;
+    v[i] = have && r0 < rows && r < p.n ? __builtin_nontemporal_load(os + r * p4 + c4) : zero;
+  }
   const int64_t chalf = p.slots * back * p.channels, cbase = (int64_t)(keep ? slot : 0) * back * p.channels;
   const T *x = (const T *)p.x + (int64_t)s * p.x_stride, *w = (const T *)p.conv_w;
   const T *oc = (const T *)p.conv_state + (before & 1) * chalf + cbase;
@@ -159,39 +185,44 @@ __global__ void __launch_bounds__(256) ssm_step_kernel(MvSsmArgs p) {
   for (int i = tid; i < p.p + 2 * p.n; i += 256) {
     const int ch = i < p.p ? head * p.p + i : (i < p.p + p.n ? p.b_off + g * p.n + i - p.p : p.c_off + g * p.n + i - p.p - p.n);
     const bool owner = keep && (i < p.p || head == g * per);   // b and c of a group: kept once
-    float o = param<Tag>(p.conv_b, ch), cur = elem<Tag>::ld(x[ch]);
-    for (int j = 0; j < back; ++j) {
-      const T raw = have ? oc[(int64_t)j * p.channels + ch] : elem<Tag>::st(0.f);
-      o = fmaf(elem<Tag>::ld(raw), elem<Tag>::ld(w[(int64_t)j * p.channels + ch]), o);
-      if (owner && j > 0) nc[(int64_t)(j - 1) * p.channels + ch] = raw;
+    const T cur = x[ch];
+    T raw[kMaxTaps - 1];
+    float wt[kMaxTaps - 1];
+#pragma unroll
+    for (int j = 0; j < kMaxTaps - 1; ++j) {
+      raw[j] = j < back && have ? oc[(int64_t)j * p.channels + ch] : elem<Tag>::st(0.f);
+      wt[j] = j < back ? elem<Tag>::ld(w[(int64_t)j * p.channels + ch]) : 0.f;
     }
-    if (owner && back > 0) nc[(int64_t)(back - 1) * p.channels + ch] = x[ch];
-    o = fmaf(cur, elem<Tag>::ld(w[(int64_t)back * p.channels + ch]), o);
-    lds[i] = elem<Tag>::ld(elem<Tag>::st(silu_f32(o)));   // (the rounding of the prefill's convolved rows)
+    float o = param<Tag>(p.conv_b, ch);
+    const float wc = elem<Tag>::ld(w[(int64_t)back * p.channels + ch]);
+#pragma unroll
+    for (int j = 0; j < kMaxTaps - 1; ++j) {
+      o = fmaf(elem<Tag>::ld(raw[j]), wt[j], o);
+      if (owner && j > 0 && j < back) nc[(int64_t)(j - 1) * p.channels + ch] = raw[j];
+    }
+    if (owner && back > 0) nc[(int64_t)(back - 1) * p.channels + ch] = cur;
+    o = fmaf(elem<Tag>::ld(cur), wc, o);
+    lds[i] = elem<Tag>::ld(elem<Tag>::st(silu_of<Tag>(o)));   // (the rounding of the prefill's convolved rows)
   }
   const float step = softplus_f32(elem<Tag>::ld(((const T *)p.dt)[(int64_t)s * p.dt_stride + head]) + param<Tag>(p.dt_bias, head));
   const float a = expf(-expf(param<Tag>(p.a_log, head)) * step), d = param<Tag>(p.d, head);
   __syncthreads();
-  const int64_t size = (int64_t)p.heads * p.n * p.p, at = (int64_t)(keep ? slot : 0) * size + (int64_t)head * p.n * p.p;
-  const f32x4 *os = (const f32x4 *)(p.ssm_state + (before & 1) * p.slots * size + at);
-  f32x4 *ns = (f32x4 *)(p.ssm_state + ((before + 1) & 1) * p.slots * size + at);
-  const int p4 = p.p / 4, rows = 256 / p4;   // threads across a state row; state rows per trip
-  const int c4 = tid % p4, r0 = tid / p4;
-  f32x4 y = {0.f, 0.f, 0.f, 0.f};
+  f32x4 y = zero;
   if (r0 < rows) {
     const f32x4 u = *(const f32x4 *)(xs + 4 * c4) * step;
-#pragma unroll 4
-    for (int r = r0; r < p.n; r += rows) {
-      f32x4 v = {0.f, 0.f, 0.f, 0.f};
-      if (have) v = os[r * p4 + c4];
+    auto advance = [&](f32x4 st, int r) {
       const float b = bs[r], c = cs[r];
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
-        v[j] = fmaf(a, v[j], b * u[j]);
-        y[j] = fmaf(v[j], c, y[j]);
+        st[j] = fmaf(a, st[j], b * u[j]);
+        y[j] = fmaf(st[j], c, y[j]);
       }
-      if (keep) ns[r * p4 + c4] = v;
-    }
+      if (keep) __builtin_nontemporal_store(st, ns + r * p4 + c4);
+    };
+#pragma unroll
+    for (int i = 0; i < kStepAhead; ++i)
+      if (r0 + i * rows < p.n) advance(v[i], r0 + i * rows);
+    for (int r = r0 + kStepAhead * rows; r < p.n; r += rows) advance(have ? os[r * p4 + c4] : zero, r);
     *(f32x4 *)(ys + r0 * p.p + 4 * c4) = y;
   }
   __syncthreads();
@@ -216,45 +247,66 @@ __global__ void __launch_bounds__(256) gated_group_norm_kernel(const typename el
   y += row * y_stride, z += row * z_stride, out += row * out_stride;
   auto place = [&](int i) { return p == p_true ? i : i / p_true * p + i % p_true; };   // true column -> stored column
   const bool vec = size % VEC == 0 && p_true % VEC == 0;
+  constexpr int KEEP = 4;   // vectors of the gated row that a thread keeps between the sum and the product
+  float v[KEEP][VEC];
   float ss = 0.f;
-  if (vec) {
-    for (int i = tid * VEC; i < size; i += 256 * VEC) {
-      float a[VEC], b[VEC];
-      const int c = place(g * size + i);
-      load_vec_row<Tag>(y + c, a);
-      load_vec_row<Tag>(z + c, b);
+  auto gated = [&](int c, float (&f)[VEC]) {
+    float b[VEC];
+    load_vec_row<Tag>(y + c, f);
+    load_vec_row<Tag>(z + c, b);
 #pragma unroll
-      for (int j = 0; j < VEC; ++j) {
-        const float v = a[j] * silu_f32(b[j]);
-        ss = fmaf(v, v, ss);
+    for (int j = 0; j < VEC; ++j) f[j] = f[j] * silu_of<Tag>(b[j]);
+  };
+  if (vec) {
+#pragma unroll
+    for (int k = 0; k < KEEP; ++k) {
+      const int i = (tid + 256 * k) * VEC;
+      if (i < size) {
+        gated(place(g * size + i), v[k]);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) ss = fmaf(v[k][j], v[k][j], ss);
       }
+    }
+    for (int i = (tid + 256 * KEEP) * VEC; i < size; i += 256 * VEC) {
+      float f[VEC];
+      gated(place(g * size + i), f);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) ss = fmaf(f[j], f[j], ss);
     }
   } else {
     for (int i = tid; i < size; i += 256) {
       const int c = place(g * size + i);
-      const float v = elem<Tag>::ld(y[c]) * silu_f32(elem<Tag>::ld(z[c]));
-      ss = fmaf(v, v, ss);
+      const float f = elem<Tag>::ld(y[c]) * silu_of<Tag>(elem<Tag>::ld(z[c]));
+      ss = fmaf(f, f, ss);
     }
   }
   ss = wave_sum(ss);
   if ((tid & 63) == 0) red[tid >> 6] = ss;
   __syncthreads();
   const float rs = 1.0f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / (float)size + eps);
-  if (vec) {
-    for (int i = tid * VEC; i < size; i += 256 * VEC) {
-      float a[VEC], b[VEC], f[VEC];
-      const int c = place(g * size + i);
-      load_vec_row<Tag>(y + c, a);
-      load_vec_row<Tag>(z + c, b);
-      load_vec_row<Tag>(w + c, f);
+  auto finish = [&](int c, const float (&f)[VEC]) {
+    float o[VEC];
+    load_vec_row<Tag>(w + c, o);
 #pragma unroll
-      for (int j = 0; j < VEC; ++j) f[j] = a[j] * silu_f32(b[j]) * rs * f[j];
-      store_vec_row<Tag>(out + c, f);
+    for (int j = 0; j < VEC; ++j) o[j] = f[j] * rs * o[j];
+    store_vec_row<Tag>(out + c, o);
+  };
+  if (vec) {
+#pragma unroll
+    for (int k = 0; k < KEEP; ++k) {
+      const int i = (tid + 256 * k) * VEC;
+      if (i < size) finish(place(g * size + i), v[k]);
+    }
+    for (int i = (tid + 256 * KEEP) * VEC; i < size; i += 256 * VEC) {
+      float f[VEC];
+      const int c = place(g * size + i);
+      gated(c, f);
+      finish(c, f);
     }
   } else {
     for (int i = tid; i < size; i += 256) {
       const int c = place(g * size + i);
-      out[c] = elem<Tag>::st(elem<Tag>::ld(y[c]) * silu_f32(elem<Tag>::ld(z[c])) * rs * elem<Tag>::ld(w[c]));
+      out[c] = elem<Tag>::st(elem<Tag>::ld(y[c]) * silu_of<Tag>(elem<Tag>::ld(z[c])) * rs * elem<Tag>::ld(w[c]));
     }
   }
   if (p != p_true) {   // padding columns: this part's share of the heads
@@ -305,7 +357,7 @@ extern "C" int mv_ssm_prefill(const MvSsmArgs *a, int dtype, int flags, void *st
   if (a->max_q < 0 || a->dt_stride < a->heads || a->out_stride < a->heads * a->p) return MV_E_SHAPE;
   if (a->ssm_state && !mv_aligned16(a->ssm_state)) return MV_E_ALIGN;
   if (dtype != MV_F32 && !(flags & MV_SSM_SCAN)) {
-    const int rc = mv_ssm_chunk_launch(*a, dtype, (hipStream_t)stream);
+    const int rc = mv_ssm_chunk_launch(*a, dtype, flags, (hipStream_t)stream);
     if (rc != MV_E_SHAPE) return rc;
   }
   const size_t lds = (size_t)(2 * kScanRows * a->n + kScanRows * 16 + 2 * kScanRows) * 4;

@@ -22,19 +22,22 @@ typedef __attribute__((address_space(3))) s16x4 lds_s16x4;
 
 constexpr int L = 64;   // tokens per chunk
 
-template <typename Tag>
-__device__ __forceinline__ uint32_t pair_hi(float a, float b, float &ra, float &rb) {   // high parts; ra, rb: the remainders
-  const auto ha = elem<Tag>::st(a), hb = elem<Tag>::st(b);
-  ra = a - elem<Tag>::ld(ha), rb = b - elem<Tag>::ld(hb);
-  return (uint32_t)ha | ((uint32_t)hb << 16);
-}
+// v = hi + lo in 16-bit parts
 template <typename Tag>
 __device__ __forceinline__ void split4(const f32x4 &v, u32x2 &hi, u32x2 &lo) {
-  float r[4];
-  hi.x = pair_hi<Tag>(v[0], v[1], r[0], r[1]);
-  hi.y = pair_hi<Tag>(v[2], v[3], r[2], r[3]);
-  lo.x = (uint32_t)elem<Tag>::st(r[0]) | ((uint32_t)elem<Tag>::st(r[1]) << 16);
-  lo.y = (uint32_t)elem<Tag>::st(r[2]) | ((uint32_t)elem<Tag>::st(r[3]) << 16);
+  hi = pack_quad<Tag>(v);
+  f32x4 r;
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    if constexpr (__is_same(Tag, bf16_tag)) {
+      r[2 * i] = v[2 * i] - u2f(hi[i] << 16);
+      r[2 * i + 1] = v[2 * i + 1] - u2f(hi[i] & 0xffff0000u);
+    } else {
+      r[2 * i] = v[2 * i] - f16_bits_to_f32((uint16_t)(hi[i] & 0xffffu));
+      r[2 * i + 1] = v[2 * i + 1] - f16_bits_to_f32((uint16_t)(hi[i] >> 16));
+    }
+  }
+  lo = pack_quad<Tag>(r);
 }
 __device__ __forceinline__ u32x4 join(const u32x2 &a, const u32x2 &b) { return u32x4{a.x, a.y, b.x, b.y}; }
 __device__ __forceinline__ u32x2 read_tr(const char *p) {
@@ -72,25 +75,34 @@ __global__ void __launch_bounds__(PT * 64, PT == 4 ? 2 : 1) ssm_chunk_kernel(MvS
     for (int e = 0; e < 4; ++e)
       st[i][e] = keep && before > 0 ? p.ssm_state[(before & 1) * p.slots * size + at + (int64_t)(i * 16 + g * 4 + e) * p.p] : 0.f;
 
-  // piece i of a chunk that starts at token t0: where it comes from, where it goes
-  auto source = [&](int i, int t0) -> const T * {
+  // piece i of a chunk: its row, where it comes from (of row 0), where it goes
+  auto piece = [&](int i, int &row, int &col) {
     const bool isx = i >= 2 * CB;
-    const int j = isx ? i - 2 * CB : (i >= CB ? i - CB : i);
-    const int row = isx ? j / (2 * PT) : j / (N / 8), c = isx ? j % (2 * PT) : j % (N / 8);
-    return x + (int64_t)min(t0 + row, len - 1) * p.x_stride + (isx ? xcol : (i >= CB ? ccol : bcol)) + c * 8;
+    const int j = isx ? i - 2 * CB : (i >= CB ? i - CB : i), c = isx ? j % (2 * PT) : j % (N / 8);
+    row = isx ? j / (2 * PT) : j / (N / 8);
+    col = (isx ? xcol : (i >= CB ? ccol : bcol)) + c * 8;
+    return (isx ? xs + row * RX : (i >= CB ? cs : bs) + row * RB) + c * 16;
   };
-  auto place = [&](int i) -> char * {
-    const bool isx = i >= 2 * CB;
-    const int j = isx ? i - 2 * CB : (i >= CB ? i - CB : i);
-    return isx ? xs + j / (2 * PT) * RX + j % (2 * PT) * 16 : (i >= CB ? cs : bs) + j / (N / 8) * RB + j % (N / 8) * 16;
-  };
+  char *dst[AHEAD];
+  const T *src[AHEAD];
+  int rows[AHEAD];
+#pragma unroll
+  for (int k = 0; k < AHEAD; ++k) {
+    int col;
+    dst[k] = piece(min(k * THREADS + tid, PIECES - 1), rows[k], col);
+    src[k] = x + (int64_t)rows[k] * p.x_stride + col;
+  }
   u32x4 ahead[AHEAD];
   float dt_ahead = 0.f;
   auto request = [&](int t0) {
+    if (t0 + L <= len) {
+      const int64_t off = (int64_t)t0 * p.x_stride;
 #pragma unroll
-    for (int k = 0; k < AHEAD; ++k) {
-      const int i = k * THREADS + tid;
-      if (PIECES % THREADS == 0 || i < PIECES) ahead[k] = *(const u32x4 *)source(i, t0);
+      for (int k = 0; k < AHEAD; ++k) ahead[k] = *(const u32x4 *)(src[k] + off);
+    } else {   // the last, short chunk: rows behind the end repeat the last token (weight 0)
+#pragma unroll
+      for (int k = 0; k < AHEAD; ++k)
+        ahead[k] = *(const u32x4 *)(src[k] + (int64_t)(min(t0 + rows[k], len - 1) - rows[k]) * p.x_stride);
     }
     if (wave == 0) dt_ahead = elem<Tag>::ld(dt[(int64_t)min(t0 + lane, len - 1) * p.dt_stride]);
   };
@@ -99,12 +111,13 @@ __global__ void __launch_bounds__(PT * 64, PT == 4 ? 2 : 1) ssm_chunk_kernel(MvS
   for (int t0 = 0; t0 < len; t0 += L) {
     const int nt = min(L, len - t0);
 #pragma unroll
-    for (int k = 0; k < AHEAD; ++k) {
-      const int i = k * THREADS + tid;
-      if (PIECES % THREADS == 0 || i < PIECES) *(u32x4 *)place(i) = ahead[k];
-    }
+    for (int k = 0; k < AHEAD; ++k) *(u32x4 *)dst[k] = ahead[k];   // (threads without a piece repeat the last one)
     if constexpr (PER > AHEAD) {
-      for (int i = AHEAD * THREADS + tid; i < PIECES; i += THREADS) *(u32x4 *)place(i) = *(const u32x4 *)source(i, t0);
+      for (int i = AHEAD * THREADS + tid; i < PIECES; i += THREADS) {
+        int row, col;
+        char *to = piece(i, row, col);
+        *(u32x4 *)to = *(const u32x4 *)(x + (int64_t)min(t0 + row, len - 1) * p.x_stride + col);
+      }
     }
     if (wave == 0) {   // step sizes and decays; tokens behind the end: dt = 0, no decay
       const float step = lane < nt ? softplus_f32(dt_ahead + bias) : 0.f;
@@ -211,8 +224,7 @@ __global__ void __launch_bounds__(PT * 64, PT == 4 ? 2 : 1) ssm_chunk_kernel(MvS
       }
       if (t < nt)
         *(u32x2 *)((T *)p.out + (int64_t)(q0 + t0 + t) * p.out_stride + xcol + wave * 16 + g * 4) =
-            u32x2{(uint32_t)elem<Tag>::st(o[0]) | ((uint32_t)elem<Tag>::st(o[1]) << 16),
-                  (uint32_t)elem<Tag>::st(o[2]) | ((uint32_t)elem<Tag>::st(o[3]) << 16)};
+            u32x2{pack_pair<Tag>(o[0], o[1]), pack_pair<Tag>(o[2], o[3])};
     }
     __syncthreads();
   }
@@ -226,11 +238,11 @@ __global__ void __launch_bounds__(PT * 64, PT == 4 ? 2 : 1) ssm_chunk_kernel(MvS
 }
 
 template <typename Tag, int NK>
-int launch(const MvSsmArgs &a, hipStream_t stream) {
+int launch(const MvSsmArgs &a, int flags, hipStream_t stream) {
   // column tiles per workgroup: as many as share the b / c rows and the scores, as long as the chip is full
   const int tiles = a.p / 16;
   int pt = tiles % 4 == 0 ? 4 : tiles % 3 == 0 ? 3 : tiles % 2 == 0 ? 2 : 1;
-  while (pt % 2 == 0 && (int64_t)a.n_seqs * a.heads * (tiles / pt) < 256) pt /= 2;
+  while (pt % 2 == 0 && (int64_t)a.n_seqs * a.heads * (tiles / pt) < ((flags >> 8) ? (flags >> 8) : 256)) pt /= 2;
   const dim3 grid(tiles / pt, a.heads, a.n_seqs);
 #define MV_SC(PT_) hipLaunchKernelGGL((ssm_chunk_kernel<Tag, NK, PT_>), grid, dim3(PT_ * 64), 0, stream, a)
   if (pt == 4) MV_SC(4);
@@ -244,9 +256,9 @@ int launch(const MvSsmArgs &a, hipStream_t stream) {
 
 }  // namespace
 
-int mv_ssm_chunk_launch(const MvSsmArgs &a, int dtype, hipStream_t stream) {
+int mv_ssm_chunk_launch(const MvSsmArgs &a, int dtype, int flags, hipStream_t stream) {
 #define MV_SN(N_) \
-  if (a.n == N_) return dtype == MV_BF16 ? launch<bf16_tag, N_ / 32>(a, stream) : launch<f16_tag, N_ / 32>(a, stream)
+  if (a.n == N_) return dtype == MV_BF16 ? launch<bf16_tag, N_ / 32>(a, flags, stream) : launch<f16_tag, N_ / 32>(a, flags, stream)
   MV_SN(32);
   MV_SN(64);
   MV_SN(96);
