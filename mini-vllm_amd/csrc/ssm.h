@@ -12,4 +12,4 @@ __device__ __forceinline__ float silu_of(float z) {
 __device__ __forceinline__ float softplus_f32(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
 
 // chunked form (16-bit); MV_E_SHAPE when it does not apply
-int mv_ssm_chunk_launch(const MvSsmArgs &a, int dtype, int flags, hipStream_t stream);
+int mv_ssm_chunk_launch(const MvSsmArgs &a, int dtype, hipStream_t stream);

@@ -357,7 +357,7 @@ extern "C" int mv_ssm_prefill(const MvSsmArgs *a, int dtype, int flags, void *st
   if (a->max_q < 0 || a->dt_stride < a->heads || a->out_stride < a->heads * a->p) return MV_E_SHAPE;
   if (a->ssm_state && !mv_aligned16(a->ssm_state)) return MV_E_ALIGN;
   if (dtype != MV_F32 && !(flags & MV_SSM_SCAN)) {
-    const int rc = mv_ssm_chunk_launch(*a, dtype, flags, (hipStream_t)stream);
+    const int rc = mv_ssm_chunk_launch(*a, dtype, (hipStream_t)stream);
     if (rc != MV_E_SHAPE) return rc;
   }
   const size_t lds = (size_t)(2 * kScanRows * a->n + kScanRows * 16 + 2 * kScanRows) * 4;

@@ -8,11 +8,12 @@
 // 16 bits of mantissa.
 //
 // One workgroup = PT waves = PT tiles of 16 columns of one head of one sequence, chunks one behind the other; wave w keeps S of
-// its columns in accumulators for the whole sequence (v_mfma_f32_16x16x32, S[n][p]: a lane holds 4 consecutive n of one column).
-// An accumulator pair of two tiles is an operand of the next product as it is, with the k index permuted (k = 8 g + e means row
-// 16 (e >> 2) + 4 g + (e & 3)); the other operand is read from LDS in that order.  So S stays in registers, and the weighted
-// scores go through LDS once (each wave computes some of the 4 token tiles, all waves read all).  The next chunk's rows are
-// requested before the current chunk's products.
+// its columns in accumulators for the whole sequence (v_mfma_f32_16x16x32, S[n][p]: a lane holds rows of one column).
+// Accumulators are operands of the next product as they are: the transposed reads of b deal the rows of S so that tiles 2 s and
+// 2 s + 1 together hold n = 32 s + 8 g .. + 7 in lane group g, the k order of an operand; the weighted scores' two key tiles are
+// one operand with k permuted (k = 8 g + e means key 16 (e >> 2) + 4 g + (e & 3)), and x is read in that order.  So S stays in
+// registers, and the scores go through LDS once (each wave computes some of the 4 token tiles, all waves read all).  The next
+// chunk's rows are requested before the current chunk's products.
 #include "ssm.h"
 
 namespace {
@@ -54,7 +55,7 @@ __global__ void __launch_bounds__(PT * 64, PT == 4 ? 2 : 1) ssm_chunk_kernel(MvS
   constexpr int PER = (PIECES + THREADS - 1) / THREADS, AHEAD = PER <= 20 ? PER : 20;
   __shared__ __attribute__((aligned(16))) char bs[L * RB], cs[L * RB], xs[L * RX];
   __shared__ u32x4 wf[2][4][2][64];            // weighted scores, high / remainder: [token tile][32 keys][lane]
-  __shared__ float rs[L], dts[L], ws[L];       // r_i (log2), dt_i, exp(r_last - r_i) dt_i
+  __shared__ float steps[2][3][L];             // of this and the next chunk: r_i (log2), dt_i, exp(r_last - r_i) dt_i
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), r16 = lane & 15, g = lane >> 4;
   const int slice = blockIdx.x, head = blockIdx.y, seq = blockIdx.z;
   const int q0 = p.cu_q[seq], len = p.cu_q[seq + 1] - q0;
@@ -68,12 +69,13 @@ __global__ void __launch_bounds__(PT * 64, PT == 4 ? 2 : 1) ssm_chunk_kernel(MvS
   const float na2 = -expf(elem<Tag>::ld(((const T *)p.a_log)[head])) * 1.4426950408889634f;
   const float bias = elem<Tag>::ld(((const T *)p.dt_bias)[head]), d = elem<Tag>::ld(((const T *)p.d)[head]);
 
+  auto state_row = [&](int i, int e) { return (i >> 1) * 32 + g * 8 + (i & 1) * 4 + e; };
   f32x4 st[2 * NK];
 #pragma unroll
   for (int i = 0; i < 2 * NK; ++i)
 #pragma unroll
     for (int e = 0; e < 4; ++e)
-      st[i][e] = keep && before > 0 ? p.ssm_state[(before & 1) * p.slots * size + at + (int64_t)(i * 16 + g * 4 + e) * p.p] : 0.f;
+      st[i][e] = keep && before > 0 ? p.ssm_state[(before & 1) * p.slots * size + at + (int64_t)state_row(i, e) * p.p] : 0.f;
 
   // piece i of a chunk: its row, where it comes from (of row 0), where it goes
   auto piece = [&](int i, int &row, int &col) {
@@ -95,6 +97,7 @@ __global__ void __launch_bounds__(PT * 64, PT == 4 ? 2 : 1) ssm_chunk_kernel(MvS
   u32x4 ahead[AHEAD];
   float dt_ahead = 0.f;
   auto request = [&](int t0) {
+    if (wave == 0) dt_ahead = elem<Tag>::ld(dt[(int64_t)min(t0 + lane, len - 1) * p.dt_stride]);
     if (t0 + L <= len) {
       const int64_t off = (int64_t)t0 * p.x_stride;
 #pragma unroll
@@ -104,12 +107,25 @@ __global__ void __launch_bounds__(PT * 64, PT == 4 ? 2 : 1) ssm_chunk_kernel(MvS
       for (int k = 0; k < AHEAD; ++k)
         ahead[k] = *(const u32x4 *)(src[k] + (int64_t)(min(t0 + rows[k], len - 1) - rows[k]) * p.x_stride);
     }
-    if (wave == 0) dt_ahead = elem<Tag>::ld(dt[(int64_t)min(t0 + lane, len - 1) * p.dt_stride]);
+  };
+  // step sizes and decays of the requested chunk (wave 0); tokens behind the end: dt = 0, no decay
+  auto scan = [&](int nt, float (*to)[L]) {
+    const float step = lane < nt ? softplus_f32(dt_ahead + bias) : 0.f;
+    float r = na2 * step;
+#pragma unroll
+    for (int o = 1; o < 64; o *= 2) {
+      const float v = __shfl_up(r, o, 64);
+      if (lane >= o) r += v;
+    }
+    to[0][lane] = r, to[1][lane] = step;
+    to[2][lane] = __builtin_amdgcn_exp2f(__shfl(r, 63, 64) - r) * step;
   };
   request(0);
+  if (wave == 0) scan(min(L, len), steps[0]);
 
   for (int t0 = 0; t0 < len; t0 += L) {
-    const int nt = min(L, len - t0);
+    const int nt = min(L, len - t0), cur = (t0 / L) & 1;
+    const float *rs = steps[cur][0], *dts = steps[cur][1], *ws = steps[cur][2];
 #pragma unroll
     for (int k = 0; k < AHEAD; ++k) *(u32x4 *)dst[k] = ahead[k];   // (threads without a piece repeat the last one)
     if constexpr (PER > AHEAD) {
@@ -118,17 +134,6 @@ __global__ void __launch_bounds__(PT * 64, PT == 4 ? 2 : 1) ssm_chunk_kernel(MvS
         char *to = piece(i, row, col);
         *(u32x4 *)to = *(const u32x4 *)(x + (int64_t)min(t0 + row, len - 1) * p.x_stride + col);
       }
-    }
-    if (wave == 0) {   // step sizes and decays; tokens behind the end: dt = 0, no decay
-      const float step = lane < nt ? softplus_f32(dt_ahead + bias) : 0.f;
-      float r = na2 * step;
-#pragma unroll
-      for (int o = 1; o < 64; o *= 2) {
-        const float v = __shfl_up(r, o, 64);
-        if (lane >= o) r += v;
-      }
-      rs[lane] = r, dts[lane] = step;
-      ws[lane] = __builtin_amdgcn_exp2f(__shfl(r, 63, 64) - r) * step;
     }
     __syncthreads();
     if (t0 + L < len) request(t0 + L);
@@ -141,13 +146,14 @@ __global__ void __launch_bounds__(PT * 64, PT == 4 ? 2 : 1) ssm_chunk_kernel(MvS
       split4<Tag>(st[2 * s], h0, l0);
       split4<Tag>(st[2 * s + 1], h1, l1);
       const u32x4 hi = join(h0, h1), lo = join(l0, l1);
+      u32x4 c[4];
 #pragma unroll
-      for (int it = 0; it < 4; ++it) {
-        const char *ca = cs + (it * 16 + r16) * RB + s * 64 + g * 8;
-        const u32x4 c = join(*(const u32x2 *)ca, *(const u32x2 *)(ca + 32));
-        y[it] = mfma16x16x32<Tag>(hi, c, y[it]);
-        y[it] = mfma16x16x32<Tag>(lo, c, y[it]);
-      }
+      for (int it = 0; it < 4; ++it) c[it] = *(const u32x4 *)(cs + (it * 16 + r16) * RB + s * 64 + g * 16);
+      // (products of one accumulator never back to back: the second would wait for the first's whole latency)
+#pragma unroll
+      for (int it = 0; it < 4; ++it) y[it] = mfma16x16x32<Tag>(hi, c[it], y[it]);
+#pragma unroll
+      for (int it = 0; it < 4; ++it) y[it] = mfma16x16x32<Tag>(lo, c[it], y[it]);
     }
     float ri[4];
 #pragma unroll
@@ -161,13 +167,17 @@ __global__ void __launch_bounds__(PT * 64, PT == 4 ? 2 : 1) ssm_chunk_kernel(MvS
 #pragma unroll
       for (int s = 0; s < NK; ++s) cf[s] = *(const u32x4 *)(cs + (it * 16 + r16) * RB + s * 64 + g * 16);
       const float r_tok = rs[it * 16 + r16];
+      f32x4 sc[4] = {};
+#pragma unroll
+      for (int s = 0; s < NK; ++s)
+#pragma unroll
+        for (int jt = 0; jt < 4; ++jt)
+          if (jt <= it) sc[jt] = mfma16x16x32<Tag>(*(const u32x4 *)(bs + (jt * 16 + r16) * RB + s * 64 + g * 16), cf[s], sc[jt]);
 #pragma unroll
       for (int jt = 0; jt < 4; ++jt) {
         u32x2 hi = {0u, 0u}, lo = {0u, 0u};
         if (jt <= it) {
-          f32x4 a = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-          for (int s = 0; s < NK; ++s) a = mfma16x16x32<Tag>(*(const u32x4 *)(bs + (jt * 16 + r16) * RB + s * 64 + g * 16), cf[s], a);
+          f32x4 a = sc[jt];
           const f32x4 rk = *(const f32x4 *)(rs + jt * 16 + g * 4), dk = *(const f32x4 *)(dts + jt * 16 + g * 4);
 #pragma unroll
           for (int e = 0; e < 4; ++e) {
@@ -180,6 +190,7 @@ __global__ void __launch_bounds__(PT * 64, PT == 4 ? 2 : 1) ssm_chunk_kernel(MvS
         *((u32x2 *)&wf[1][it][jt >> 1][lane] + (jt & 1)) = lo;
       }
     }
+    if (wave == 0 && t0 + L < len) scan(min(L, len - t0 - L), steps[cur ^ 1]);   // (wave 0 scored the fewest keys)
     __syncthreads();
     // ---- sum over the chunk's keys; then the state moves on
     const float tail = __builtin_amdgcn_exp2f(rs[L - 1]);
@@ -191,11 +202,9 @@ __global__ void __launch_bounds__(PT * 64, PT == 4 ? 2 : 1) ssm_chunk_kernel(MvS
       const u32x2 x0 = read_tr(xa), x1 = read_tr(xa + 16 * RX);
       const u32x4 xf = join(x0, x1);
 #pragma unroll
-      for (int it = 2 * s; it < 4; ++it) {
-        y[it] = mfma16x16x32<Tag>(xf, wf[0][it][s][lane], y[it]);
-        y[it] = mfma16x16x32<Tag>(xf, wf[1][it][s][lane], y[it]);
-      }
-      // (tokens 16 .. 31 of the chunk also need keys 0 .. 31, which is s = 0 above; s = 1 starts at token 32)
+      for (int part = 0; part < 2; ++part)
+#pragma unroll
+        for (int it = 2 * s; it < 4; ++it) y[it] = mfma16x16x32<Tag>(xf, wf[part][it][s][lane], y[it]);   // keys 32 s ..
       float f[8];
       unpack8<Tag>(xf, f);
       const f32x4 w0 = *(const f32x4 *)(ws + 32 * s + 4 * g), w1 = *(const f32x4 *)(ws + 32 * s + 16 + 4 * g);
@@ -203,12 +212,20 @@ __global__ void __launch_bounds__(PT * 64, PT == 4 ? 2 : 1) ssm_chunk_kernel(MvS
       split4<Tag>(f32x4{f[0], f[1], f[2], f[3]} * w0, h0, l0);
       split4<Tag>(f32x4{f[4], f[5], f[6], f[7]} * w1, h1, l1);
       const u32x4 hi = join(h0, h1), lo = join(l0, l1);
-      const char *ba = bs + (32 * s + 4 * g + (r16 >> 2)) * RB + (r16 & 3) * 8;
+      const char *ba = bs + (32 * s + 4 * g + (r16 >> 2)) * RB + (r16 & 3) * 16;
+      constexpr int IB = NK % 2 == 0 ? 4 : 2;   // state tiles at a time
 #pragma unroll
-      for (int i = 0; i < 2 * NK; ++i) {
-        const u32x4 b = join(read_tr(ba + i * 32), read_tr(ba + 16 * RB + i * 32));
-        st[i] = mfma16x16x32<Tag>(b, hi, st[i]);
-        st[i] = mfma16x16x32<Tag>(b, lo, st[i]);
+      for (int i = 0; i < 2 * NK; i += IB) {
+        u32x4 b[IB];
+#pragma unroll
+        for (int j = 0; j < IB; ++j) {
+          const int o = ((i + j) >> 1) * 64 + ((i + j) & 1) * 8;
+          b[j] = join(read_tr(ba + o), read_tr(ba + 16 * RB + o));
+        }
+#pragma unroll
+        for (int j = 0; j < IB; ++j) st[i + j] = mfma16x16x32<Tag>(b[j], hi, st[i + j]);
+#pragma unroll
+        for (int j = 0; j < IB; ++j) st[i + j] = mfma16x16x32<Tag>(b[j], lo, st[i + j]);
       }
     }
     // ---- out: lane (token r16, columns 4 g ..)
@@ -233,16 +250,15 @@ __global__ void __launch_bounds__(PT * 64, PT == 4 ? 2 : 1) ssm_chunk_kernel(MvS
 #pragma unroll
     for (int i = 0; i < 2 * NK; ++i)
 #pragma unroll
-      for (int e = 0; e < 4; ++e) ns[(int64_t)(i * 16 + g * 4 + e) * p.p] = st[i][e];
+      for (int e = 0; e < 4; ++e) ns[(int64_t)state_row(i, e) * p.p] = st[i][e];
   }
 }
 
 template <typename Tag, int NK>
-int launch(const MvSsmArgs &a, int flags, hipStream_t stream) {
-  // column tiles per workgroup: as many as share the b / c rows and the scores, as long as the chip is full
-  const int tiles = a.p / 16;
-  int pt = tiles % 4 == 0 ? 4 : tiles % 3 == 0 ? 3 : tiles % 2 == 0 ? 2 : 1;
-  while (pt % 2 == 0 && (int64_t)a.n_seqs * a.heads * (tiles / pt) < ((flags >> 8) ? (flags >> 8) : 256)) pt /= 2;
+int launch(const MvSsmArgs &a, hipStream_t stream) {
+  // column tiles per workgroup: as many as divide the head's.  They share the b / c rows and the scores; fewer per workgroup
+  // measured slower even where they fill an otherwise idle chip (a lone wave loads and scores everything by itself)
+  const int tiles = a.p / 16, pt = tiles % 4 == 0 ? 4 : tiles % 3 == 0 ? 3 : tiles % 2 == 0 ? 2 : 1;
   const dim3 grid(tiles / pt, a.heads, a.n_seqs);
 #define MV_SC(PT_) hipLaunchKernelGGL((ssm_chunk_kernel<Tag, NK, PT_>), grid, dim3(PT_ * 64), 0, stream, a)
   if (pt == 4) MV_SC(4);
@@ -256,9 +272,9 @@ int launch(const MvSsmArgs &a, int flags, hipStream_t stream) {
 
 }  // namespace
 
-int mv_ssm_chunk_launch(const MvSsmArgs &a, int dtype, int flags, hipStream_t stream) {
+int mv_ssm_chunk_launch(const MvSsmArgs &a, int dtype, hipStream_t stream) {
 #define MV_SN(N_) \
-  if (a.n == N_) return dtype == MV_BF16 ? launch<bf16_tag, N_ / 32>(a, flags, stream) : launch<f16_tag, N_ / 32>(a, flags, stream)
+  if (a.n == N_) return dtype == MV_BF16 ? launch<bf16_tag, N_ / 32>(a, stream) : launch<f16_tag, N_ / 32>(a, stream)
   MV_SN(32);
   MV_SN(64);
   MV_SN(96);
