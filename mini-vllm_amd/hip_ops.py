@@ -1309,15 +1309,17 @@ def ssm_step(x, dt, conv_w, conv_b, dt_bias, a_log, d, shape, conv_state, ssm_st
     return out
 
 
-def gated_group_norm(y, z, w, heads: int, p: int, p_true: int, groups: int, eps: float):
-    """rms over each of ``groups`` equal parts of y * silu(z), times w: [T, heads * p] (p_true of each head's columns count)."""
+def gated_group_norm(y, z, w, heads: int, p: int, p_true: int, groups: int, eps: float, out_cols: int | None = None):
+    """rms over each of ``groups`` equal parts of y * silu(z), times w: [T, heads * p] (p_true of each head's columns count);
+    ``out_cols``: rows of that many columns, zeros behind."""
     _need_cuda(y, z, w)
     cols = heads * p
     _rows_ok("y", y, cols)
     _rows_ok("z", z, cols, y.dtype)
     if w.dtype != y.dtype or w.numel() != cols or y.shape[0] != z.shape[0]:
         raise MvHipError(f"norm weight of {cols} {y.dtype} and as many rows of z required")
-    out = torch.empty((y.shape[0], cols), dtype=y.dtype, device=y.device)
+    wide = out_cols is not None and out_cols > cols
+    out = (torch.zeros if wide else torch.empty)((y.shape[0], out_cols if wide else cols), dtype=y.dtype, device=y.device)
     _check(_lib.mv_gated_group_norm(y.data_ptr(), y.stride(0), z.data_ptr(), z.stride(0), w.data_ptr(), out.data_ptr(),
                                     out.stride(0), y.shape[0], heads, p, p_true, groups, float(eps), _dt(y), _stream()),
            "mv_gated_group_norm")

@@ -98,5 +98,6 @@ class Mamba2(nn.Module):
             xc = hip_ops.causal_conv(x[nd:], self.conv, self.conv_b, self.shape, self.conv_state, slots[nd:], cu_q, cu_k, max_q)
             hip_ops.ssm_prefill(xc, dt[nd:], self.dt_bias, self.A_log, self.D, self.shape, self.ssm_state, slots[nd:], cu_q, cu_k,
                                 max_q, out=y[nd:])
-        g = hip_ops.gated_group_norm(y, z, self.norm, self.heads, self.p, self.vdim, self.norm_groups, self.eps)
+        g = hip_ops.gated_group_norm(y, z, self.norm, self.heads, self.p, self.vdim, self.norm_groups, self.eps,
+                                     self.o.weight.shape[1])
         return self.o(g, partial_ok=True)

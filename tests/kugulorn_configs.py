@@ -35,7 +35,7 @@ CONFIGS = {
     "ones": config(64, 64, [mamba(1, 16, 32, 1, 1, 1), latent(1, 32, 2, 16, 16, 32, 1, ff=64, limit=50.0),
                             latent(1, 8, 8, 8, 8, 16, 2, ff=64), mamba(2, 8, 8, 2, 8, 2)], mult=1.0),
     # recurrent layers only: no cache plane at all
-    "states": config(96, 97, [mamba(4, 48, 64, 4, 3, 4, ff=64), mamba(6, 80, 160, 2, 5, 3)], mult=0.5),
+    "states": config(96, 104, [mamba(4, 48, 64, 4, 3, 4, ff=64), mamba(6, 80, 160, 2, 5, 3)], mult=0.5),
 }
 
 

@@ -138,14 +138,25 @@ def test_design_configurations_have_the_layer_sizes_of_their_peers():
     and the framework reads the configuration."""
     from minivllm_amd.native_configs import NATIVE_CONFIGS
 
-    for design, pairs in bench.DESIGNS.items():
-        for name, like in pairs.items():
-            c, p = NATIVE_CONFIGS[bench.MODELS[name]["architecture"]](bench.MODELS[name]), bench.MODELS[like]
-            assert c.num_hidden_layers == p["num_hidden_layers"] and c.vocab_size == p["vocab_size"]
-            for run, _, _ in c.layer_runs():
-                a = c.layers[run].attention
-                assert (a.heads, a.kv_heads) == (p["num_attention_heads"], p["num_key_value_heads"])
-                assert a.dim == (p.get("head_dim") or p["hidden_size"] // p["num_attention_heads"]) and c.layers[run].ff == p["intermediate_size"]
+    for name, like in bench.DESIGNS["mofarax"].items():
+        c, p = NATIVE_CONFIGS[bench.MODELS[name]["architecture"]](bench.MODELS[name]), bench.MODELS[like]
+        assert c.num_hidden_layers == p["num_hidden_layers"] and c.vocab_size == p["vocab_size"]
+        for run, _, _ in c.layer_runs():
+            a = c.layers[run].attention
+            assert (a.heads, a.kv_heads) == (p["num_attention_heads"], p["num_key_value_heads"])
+            assert a.dim == (p.get("head_dim") or p["hidden_size"] // p["num_attention_heads"]) and c.layers[run].ff == p["intermediate_size"]
+    # layers of unlike kinds: the peer's width, heads and feed-forward, and as many weights in all layers together (within 5 %)
+    for name, like in bench.DESIGNS["kugulorn"].items():
+        c, p = NATIVE_CONFIGS["Kugulorn"](bench.MODELS[name]), bench.MODELS[like]
+        assert (c.vocab_size, c.hidden_size) == (p["vocab_size"], p["hidden_size"])
+        for s in c.layers:
+            if s.type == "latent_attention":
+                assert s.mixer.heads == p["num_attention_heads"] and s.mlp.ff == p["intermediate_size"]
+        count = lambda shapes: sum(a[0] * a[1] for k, a in shapes.items() if len(a) == 2 and k not in ("embed", "head"))
+        d, dim = p["hidden_size"], p.get("head_dim") or p["hidden_size"] // p["num_attention_heads"]
+        h, kv = p["num_attention_heads"], p["num_key_value_heads"]
+        layer = d * dim * (2 * h + 2 * kv) + 3 * d * p["intermediate_size"]
+        assert abs(count(c.weight_shapes()) / (layer * p["num_hidden_layers"]) - 1) < 0.05, name
     args = bench.parse(["--design", "mofarax"])
     assert args.design == "mofarax" and bench.parse([]).design is None and bench.parse([]).model == "qwen3-1.7b"
     # a chunk mask cuts the work of a prompt into the chunks' triangles
