@@ -50,7 +50,9 @@ template <typename Tag, int NK, int PT>
 __global__ void __launch_bounds__(PT * 64, PT == 4 ? 2 : 1) ssm_chunk_kernel(MvSsmArgs p) {
   typedef typename elem<Tag>::T T;
   constexpr int N = NK * 32, THREADS = PT * 64;
-  constexpr int RB = (N / 8 + 1) * 16, RX = (2 * PT + 1) * 16;   // LDS rows of an odd number of 16-byte pieces
+  // LDS rows: x an odd number of 16-byte pieces; b and c 2 (mod 4), so that the row reads stay apart over 8 rows and the
+  // transposed reads, whose pieces lie 16 bytes apart, meet at most in pairs
+  constexpr int RB = (N / 8 + 2) * 16, RX = (2 * PT + 1) * 16;
   constexpr int CB = L * N / 8, CX = L * 2 * PT, PIECES = 2 * CB + CX;   // 16-byte pieces of b, c and x
   constexpr int PER = (PIECES + THREADS - 1) / THREADS, AHEAD = PER <= 20 ? PER : 20;
   __shared__ __attribute__((aligned(16))) char bs[L * RB], cs[L * RB], xs[L * RX];
