@@ -2,6 +2,9 @@
 #pragma once
 #include "common.h"
 
+#include <type_traits>
+#include <utility>
+
 typedef __attribute__((ext_vector_type(8))) __bf16 mv_bf16x8;
 typedef __attribute__((ext_vector_type(8))) _Float16 mv_f16x8;
 
@@ -45,6 +48,52 @@ __device__ __forceinline__ void store_vec_row(typename elem<Tag>::T *p, const fl
     for (int i = 0; i < 4; ++i) raw[i] = f2u(f[i]);
   }
   *reinterpret_cast<u32x4 *>(p) = raw;
+}
+
+// ---- hand-counted LDS reads.  The compiler puts a wait for every outstanding LDS-DMA in front of an LDS read it can see, since
+// the transfer might write what is read; with tiles in flight to OTHER buffers that wait is the whole memory latency.  These
+// reads are opaque to it and are retired by counted waits that name the fragment as an operand, so that no use moves above its
+// wait.  LDS operations complete in order, so a count of one's own newer reads is safe beside LDS operations of the compiler's;
+// scalar loads share the counter out of order and must not be outstanding.
+__device__ __forceinline__ uint32_t lds_address(const void *p) {
+  return (uint32_t)(uintptr_t)(__attribute__((address_space(3))) const char *)p;
+}
+template <int OFF>
+__device__ __forceinline__ void lds_read128(u32x4 &d, uint32_t a) {
+  asm volatile("ds_read_b128 %0, %1 offset:%2" : "=v"(d) : "v"(a), "i"(OFF) : "memory");
+}
+template <int OFF>
+__device__ __forceinline__ void lds_read32(float &d, uint32_t a) {
+  asm volatile("ds_read_b32 %0, %1 offset:%2" : "=v"(d) : "v"(a), "i"(OFF) : "memory");
+}
+template <int OFF>
+__device__ __forceinline__ void lds_read64_tr(u32x2 &d, uint32_t a) {
+  asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(d) : "v"(a), "i"(OFF) : "memory");
+}
+template <int N, typename V>
+__device__ __forceinline__ void lds_wait(V &a) {
+  asm volatile("s_waitcnt lgkmcnt(%1)" : "+v"(a) : "n"(N));
+}
+template <int N, typename V>
+__device__ __forceinline__ void lds_wait(V &a, V &b) {
+  asm volatile("s_waitcnt lgkmcnt(%2)" : "+v"(a), "+v"(b) : "n"(N));
+}
+// the registers count as written here: loads into them are waited for now, not (with everything newer) at their first use
+template <int N>
+__device__ __forceinline__ void settle(u32x4 (&v)[N]) {
+#pragma unroll
+  for (int i = 0; i < N; ++i) asm volatile("" : "+v"(v[i]));
+}
+// workgroup barrier that leaves transfers to LDS in flight (__syncthreads waits for all of them)
+__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+// compile-time loop: f(integral_constant<int, 0>) ... f(integral_constant<int, N - 1>)
+template <typename F, int... I>
+__device__ __forceinline__ void static_for_impl(F &&f, std::integer_sequence<int, I...>) {
+  (f(std::integral_constant<int, I>{}), ...);
+}
+template <int N, typename F>
+__device__ __forceinline__ void static_for(F &&f) {
+  static_for_impl(f, std::make_integer_sequence<int, N>{});
 }
 
 // let kernel K use the CU's whole LDS (once per process)
