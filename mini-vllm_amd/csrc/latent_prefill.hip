@@ -14,9 +14,10 @@
 
 namespace {
 
-typedef __attribute__((ext_vector_type(4))) short s16x4;
 typedef __attribute__((ext_vector_type(16))) float f32x16;
+typedef __attribute__((ext_vector_type(4))) short s16x4;
 typedef __attribute__((address_space(3))) s16x4 lds_s16x4;
+typedef __attribute__((address_space(3))) const u32x4 lds_u32x4;
 
 constexpr int BN = 64;   // keys per tile
 
@@ -59,25 +60,34 @@ __global__ void __launch_bounds__(NW * 64, 2) latent_prefill_kernel(MvLatentPref
     const int64_t pos = p.positions[row];
     const bool pos_ok = pos >= 0 && pos < p.max_pos;
     const float *ct = p.cos + (pos_ok ? pos * pairs : 0), *st = p.sin + (pos_ok ? pos * pairs : 0);
+    float cs[NS][4], sn[NS][4];   // (every load of the row ahead of its arithmetic; only the rotated steps' are made)
 #pragma unroll
     for (int s = 0; s < NS; ++s) {
-      u32x4 v = *reinterpret_cast<const u32x4 *>(qp + 16 * s);
-      const int c = 16 * s + 8 * h - p.plain_cols;   // (plain_cols is a multiple of 32: uniform over the step)
+      qf[s] = *reinterpret_cast<const u32x4 *>(qp + 16 * s);
+      if (16 * s >= p.plain_cols)   // (plain_cols is a multiple of 32: uniform over the step)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const int i = min(((16 * s + 8 * h - p.plain_cols) >> 1) + j, pairs - 1);
+          cs[s][j] = ct[i], sn[s][j] = st[i];
+        }
+    }
+#pragma unroll
+    for (int s = 0; s < NS; ++s) {
       if (16 * s >= p.plain_cols) {
         float f[8];
-        unpack8<Tag>(v, f);
+        unpack8<Tag>(qf[s], f);
 #pragma unroll
-        for (int j = 0; j < 8; j += 2) {
-          const int i = (c + j) >> 1, ic = i < pairs ? i : pairs - 1;
-          const float cs = pos_ok ? ct[ic] : 1.0f, sn = pos_ok ? st[ic] : 0.0f;
-          const float a = f[j], b = f[j + 1];
-          f[j] = i < pairs ? __fsub_rn(__fmul_rn(a, cs), __fmul_rn(b, sn)) : 0.f;
-          f[j + 1] = i < pairs ? __fadd_rn(__fmul_rn(b, cs), __fmul_rn(a, sn)) : 0.f;
+        for (int j = 0; j < 4; ++j) {
+          const int i = ((16 * s + 8 * h - p.plain_cols) >> 1) + j;
+          const float c = pos_ok ? cs[s][j] : 1.0f, n = pos_ok ? sn[s][j] : 0.0f, a = f[2 * j], b = f[2 * j + 1];
+          f[2 * j] = i < pairs ? __fsub_rn(__fmul_rn(a, c), __fmul_rn(b, n)) : 0.f;
+          f[2 * j + 1] = i < pairs ? __fadd_rn(__fmul_rn(b, c), __fmul_rn(a, n)) : 0.f;
         }
-        v = pack8<Tag>(f);
+        qf[s] = pack8<Tag>(f);
       }
-      qf[s] = q_ok ? v : u32x4{0u, 0u, 0u, 0u};
+      if (!q_ok) qf[s] = u32x4{0u, 0u, 0u, 0u};
     }
+    settle(qf);
   }
 
   f32x16 oacc[NDT];
@@ -130,31 +140,61 @@ __global__ void __launch_bounds__(NW * 64, 2) latent_prefill_kernel(MvLatentPref
           (__attribute__((address_space(3))) void *)(dv + (NW * i + wave) * 1024), 16, 0, 0);
   };
 
-  // ---- LDS read offsets
-  int koff[NS];
+  // ---- LDS read addresses (hand-counted reads, latent.h); the buffer is an instruction immediate where it fits in 16 bits
+  constexpr bool IMM = BUF + (DQ * 2) * 32 < 65536 && BUF + 48 * (DV * 2) < 65536;
+  // PIPE: hand-counted reads ahead of their use.  Not where the registers run out: a fragment that is still on its way must not be
+  // moved to scratch
+  constexpr bool PIPE = DQ <= 192 && DV <= 128;
+  const uint32_t lds0 = lds_address(smem);
+  uint32_t koff[NS];
 #pragma unroll
-  for (int s = 0; s < NS; ++s) koff[s] = r * (DQ * 2) + (((2 * s + h) ^ k_swz<CQ>(r)) << 4);
+  for (int s = 0; s < NS; ++s) koff[s] = lds0 + r * (DQ * 2) + (((2 * s + h) ^ k_swz<CQ>(r)) << 4);
   const int g = (lane >> 4) & 1, q4 = (lane & 15) >> 2, pp = lane & 3;
-  int vlo[NDT], vhi[NDT];
+  uint32_t vlo[NDT], vhi[NDT];
 #pragma unroll
   for (int dt = 0; dt < NDT; ++dt) {
     const int ch = 4 * dt + 2 * g + (pp >> 1);
-    vlo[dt] = (4 * h + q4) * (DV * 2) + ((ch ^ v_swz<CV>(4 * h + q4)) << 4) + 8 * (pp & 1);
-    vhi[dt] = (4 * h + q4 + 8) * (DV * 2) + ((ch ^ v_swz<CV>(4 * h + q4 + 8)) << 4) + 8 * (pp & 1);
+    vlo[dt] = lds0 + KB + (4 * h + q4) * (DV * 2) + ((ch ^ v_swz<CV>(4 * h + q4)) << 4) + 8 * (pp & 1);
+    vhi[dt] = lds0 + KB + (4 * h + q4 + 8) * (DV * 2) + ((ch ^ v_swz<CV>(4 * h + q4 + 8)) << 4) + 8 * (pp & 1);
   }
 
   auto tile = [&](const int t, auto Bc) __attribute__((always_inline)) {
-    constexpr int BO = decltype(Bc)::value * BUF;
+    constexpr int BO = IMM ? decltype(Bc)::value * BUF : 0;
+    constexpr uint32_t add = IMM ? 0 : decltype(Bc)::value * BUF;
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");   // (nothing else may be counted below)
     if (t + 1 < n_tiles) dma(t + 1, 1 - decltype(Bc)::value);
     const int kv0 = kv_base + t * BN;
     if (kv0 <= wave_max && kv0 + BN > lo_min) {
       f32x16 sacc[2];
       const f32x16 zero = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-      const char *ka = smem + BO, *kb = ka + 32 * (DQ * 2);   // (the swizzle repeats every 16 rows)
+      u32x4 kf[2][2];            // K fragments, one step ahead
+      u32x2 va[NDT], vb[NDT];    // V^T fragments of 16 keys; the first ones go out before the softmax
+      if constexpr (PIPE) {
+        lds_read128<BO>(kf[0][0], koff[0] + add);
+        lds_read128<BO + 32 * (DQ * 2)>(kf[0][1], koff[0] + add);
+        static_for<NS>([&](auto S) {
+          constexpr int s = decltype(S)::value;
+          if constexpr (s + 1 < NS) {
+            lds_read128<BO>(kf[(s + 1) & 1][0], koff[s + 1] + add);
+            lds_read128<BO + 32 * (DQ * 2)>(kf[(s + 1) & 1][1], koff[s + 1] + add);
+            lds_wait<2>(kf[s & 1][0], kf[s & 1][1]);
+          } else {
+            static_for<NDT>([&](auto D) {
+              lds_read64_tr<BO>(va[decltype(D)::value], vlo[decltype(D)::value] + add);
+              lds_read64_tr<BO>(vb[decltype(D)::value], vhi[decltype(D)::value] + add);
+            });
+            lds_wait<(2 * NDT < 15 ? 2 * NDT : 15)>(kf[s & 1][0], kf[s & 1][1]);
+          }
+          sacc[0] = mfma32<Tag>(kf[s & 1][0], qf[s], s ? sacc[0] : zero);
+          sacc[1] = mfma32<Tag>(kf[s & 1][1], qf[s], s ? sacc[1] : zero);
+        });
+      } else {
 #pragma unroll
-      for (int s = 0; s < NS; ++s) {
-        sacc[0] = mfma32<Tag>(*reinterpret_cast<const u32x4 *>(ka + koff[s]), qf[s], s ? sacc[0] : zero);
-        sacc[1] = mfma32<Tag>(*reinterpret_cast<const u32x4 *>(kb + koff[s]), qf[s], s ? sacc[1] : zero);
+        for (int s = 0; s < NS; ++s) {
+          const u32x4 k_lo = *(lds_u32x4 *)(uintptr_t)(koff[s] + BO + add), k_hi = *(lds_u32x4 *)(uintptr_t)(koff[s] + BO + add + 32 * (DQ * 2));
+          sacc[0] = mfma32<Tag>(k_lo, qf[s], s ? sacc[0] : zero);
+          sacc[1] = mfma32<Tag>(k_hi, qf[s], s ? sacc[1] : zero);
+        }
       }
       if (kv0 + BN - 1 > wave_min || kv0 + BN > sk || kv0 < lo_max) {
         const int hi = min(qidx + shift, sk - 1), lo = qidx + shift - win + 1;
@@ -171,7 +211,11 @@ __global__ void __launch_bounds__(NW * 64, 2) latent_prefill_kernel(MvLatentPref
       for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
         for (int i = 0; i < 16; ++i) mx = fmaxf(mx, sacc[kt][i]);
-      mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+      {   // the other half of the row lies 32 lanes away (a vector instruction: an LDS one would wait for the reads in flight)
+        float other = mx;
+        asm volatile("s_nop 1\n\tv_permlane32_swap_b32 %0, %1" : "+v"(mx), "+v"(other));
+        mx = fmaxf(mx, other);
+      }
       const float m_new = fmaxf(m_run, mx * scale_log2);
       if (!__all(m_new - m_run <= 6.0f)) {   // rescale only when a maximum grew by more than 2^6
         const float alpha = __builtin_amdgcn_exp2f(m_run - m_new);
@@ -193,21 +237,30 @@ __global__ void __launch_bounds__(NW * 64, 2) latent_prefill_kernel(MvLatentPref
           rs[i & 3] += e;
         }
       l_run += (rs[0] + rs[1]) + (rs[2] + rs[3]);
+      u32x4 pf[4];
 #pragma unroll
-      for (int kt = 0; kt < 2; ++kt)
+      for (int i = 0; i < 4; ++i)
 #pragma unroll
-        for (int s2 = 0; s2 < 2; ++s2) {
-          u32x4 pf;
-#pragma unroll
-          for (int j = 0; j < 4; ++j) pf[j] = pack_pair<Tag>(sacc[kt][8 * s2 + 2 * j], sacc[kt][8 * s2 + 2 * j + 1]);
-          const char *vb = smem + BO + KB + (kt * 32 + 16 * s2) * (DV * 2);
-#pragma unroll
-          for (int dt = 0; dt < NDT; ++dt) {
-            const u32x2 lo = __builtin_bit_cast(u32x2, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4 *)(vb + vlo[dt])));
-            const u32x2 hi = __builtin_bit_cast(u32x2, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4 *)(vb + vhi[dt])));
-            oacc[dt] = mfma32<Tag>(u32x4{lo.x, lo.y, hi.x, hi.y}, pf, oacc[dt]);
+        for (int j = 0; j < 4; ++j)
+          pf[i][j] = pack_pair<Tag>(sacc[i >> 1][8 * (i & 1) + 2 * j], sacc[i >> 1][8 * (i & 1) + 2 * j + 1]);
+      // 16 keys at a time; a fragment register is requested again right behind the product that used it
+      static_for<4>([&](auto G) {
+        constexpr int gr = decltype(G)::value;
+        static_for<NDT>([&](auto D) {
+          constexpr int dt = decltype(D)::value;
+          if constexpr (!PIPE) {
+            constexpr uint32_t o = BO + add + gr * 16 * (DV * 2);
+            va[dt] = __builtin_bit_cast(u32x2, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4 *)(uintptr_t)(vlo[dt] + o)));
+            vb[dt] = __builtin_bit_cast(u32x2, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4 *)(uintptr_t)(vhi[dt] + o)));
+          } else if constexpr (gr < 3) lds_wait<2 * NDT - 2>(va[dt], vb[dt]);
+          else lds_wait<2 * (NDT - 1 - dt)>(va[dt], vb[dt]);
+          oacc[dt] = mfma32<Tag>(u32x4{va[dt].x, va[dt].y, vb[dt].x, vb[dt].y}, pf[gr], oacc[dt]);
+          if constexpr (PIPE && gr < 3) {
+            lds_read64_tr<BO + (gr + 1) * 16 * (DV * 2)>(va[dt], vlo[dt] + add);
+            lds_read64_tr<BO + (gr + 1) * 16 * (DV * 2)>(vb[dt], vhi[dt] + add);
           }
-        }
+        });
+      });
     }
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");   // this wave's share of the next tile has landed
     __syncthreads();
