@@ -50,10 +50,18 @@ enum {
  *       1 / n: dim 2i pairs with dim 2i + 1 for i < n, dims from 2n on pass unchanged, cos, sin are [max_pos, n].
  *   chunk: > 0: a query at position i sees only the keys of its own chunk of `chunk` positions (counted from the start of
  *       the sequence), i / chunk * chunk .. i.  0: every key up to i.
- *   out_stride: elements between the token rows of `out` (0: dense [.., H, D] rows). */
+ *   norm_dim: columns of a head that its norm is a mean over (0: all of them; the others hold zeros).
+ *   out_stride: elements between the token rows of `out` (0: dense [.., H, D] rows).
+ *   window / keep_first: window > 0: a query at position i sees key j <= i if i - j < window or j < keep_first (not with chunk).
+ *   softcap: > 0: scores s become softcap * tanh(s / softcap).
+ *   out_scale: multiplies the output (0: 1).
+ *   sink: [n_heads] of dtype: the softmax denominator of head h has one more term, exp(sink[h]) (not scaled, not capped). */
 typedef struct MvAttnOpts {
-  int rot_pairs, interleaved, chunk, reserved;
+  int rot_pairs, interleaved, chunk, norm_dim;
   int64_t out_stride;
+  int window, keep_first;
+  float softcap, out_scale;
+  const void *sink;
 } MvAttnOpts;
 
 int mv_version(void);
@@ -141,8 +149,8 @@ size_t mv_paged_decode_workspace_bytes(int batch, int n_heads, int n_kv_heads,
                                        int head_dim, int block_size,
                                        int max_blocks, int flags);
 size_t mv_paged_decode_workspace_bytes_ex(int batch, int n_heads, int n_kv_heads,
-                                          int head_dim, int block_size,
-                                          int max_blocks, int flags, int chunk);
+                                          int head_dim, int block_size, int max_blocks, int flags,
+                                          const MvAttnOpts *opts);
 int mv_paged_decode(const void *q, int64_t q_stride_tok, const void *k_cache,
                     const void *v_cache, const int32_t *block_tables,
                     int64_t table_stride, const int32_t *context_lens,
@@ -298,8 +306,8 @@ int mv_gelu_and_mul(const void *x, int64_t x_stride, void *out, int64_t out_stri
                     int rows, int cols, int dtype, void *stream);
 
 /* Activation of a gated projection, act(gate, up) (HOST struct, read during the call).  MV_ACT_CLAMPED: g = min(gate, limit),
- * u = clamp(up, -limit, limit), g * sigmoid(alpha * g) * (u + 1). */
-enum { MV_ACT_SILU = 0, MV_ACT_GELU = 1, MV_ACT_CLAMPED = 2 };
+ * u = clamp(up, -limit, limit), g * sigmoid(alpha * g) * (u + 1).  MV_ACT_RELU: max(gate, 0) * up. */
+enum { MV_ACT_SILU = 0, MV_ACT_GELU = 1, MV_ACT_CLAMPED = 2, MV_ACT_RELU = 3 };
 typedef struct MvGateAct {
   int kind;
   float limit, alpha;
@@ -313,7 +321,14 @@ int mv_act_and_mul(const void *x, int64_t x_stride, void *out, int64_t out_strid
  *     x = b + y' + [embed_mode 1 or 2: embed_scale * embed[ids[row]]] + [vec]
  *     out = (norm_w) x / sqrt(mean(x^2) + eps) * (norm_offset + norm_w), else x, rounded to dtype   (out NULL: nothing)
  * y: rows of dtype at stride y_stride, or (y_splits > 0) fp32 partial sums [y_splits][rows][cols]; NULL = nothing.
- * All weights / tables are of dtype.  Means are over cols_true <= cols columns; the others hold zeros. */
+ * All weights / tables are of dtype.  Means are over cols_true <= cols columns; the others hold zeros.
+ * layer_norm: both norms are layer norms instead, (z - mean) / sqrt(mean((z - mean)^2) + eps) * w + b (biases NULL = 0).
+ * pairs: a second table, [buckets + 1][cols], whose row (previous token * mul_prev + token * mul_cur) mod buckets is added where the
+ *     embedding is (a sequence's first token: row `buckets`).  The token before a step's first is kept in prev_tokens [2][slots],
+ *     half = number of tokens before it & 1, at state_slots[sequence] (< 0: as if it were 0); the step writes its last one to the
+ *     other tokens' half.  Sequences: rows cu_q[s] .. cu_q[s + 1]; cu_q NULL: one row each.  Rows at position < 0: padding.
+ * moe_rows: y' += sum over k < moe_top of moe_w[row][k] * moe_out[moe_rows[row][k]] ([..][cols] of dtype, dense), where a row
+ *     index < 0 stands for the stream itself, as it is before the update. */
 typedef struct MvResidualArgs {
   float *x;
   const void *y, *y_norm_w, *embed;
@@ -325,6 +340,15 @@ typedef struct MvResidualArgs {
   int y_splits, embed_mode;
   float y_mult;          /* 1 = none */
   const void *y_scale;   /* [cols] of dtype; NULL = ones */
+  const void *y_norm_b, *norm_b, *pairs;
+  const int64_t *positions;
+  const int32_t *state_slots, *cu_q;
+  int32_t *prev_tokens;
+  const void *moe_out;
+  const int32_t *moe_rows;
+  const float *moe_w;
+  int64_t buckets, mul_prev, mul_cur, slots;
+  int layer_norm, n_seqs, moe_top, reserved;
 } MvResidualArgs;
 int mv_residual_update(const MvResidualArgs *args, int rows, int cols, int cols_true, int dtype, void *stream);
 
@@ -652,7 +676,7 @@ typedef struct MvSsmArgs {
   int64_t slots;
   int n_seqs, max_q, channels, taps, heads, groups, p, n, b_off, c_off;
 } MvSsmArgs;
-/* out[t] = silu(causal convolution of x + conv_b), [T][channels]; writes conv_state */
+/* out[t] = silu(causal convolution of x + conv_b), [T][channels]; writes conv_state.  conv_b NULL: no bias */
 int mv_causal_conv(const MvSsmArgs *args, int dtype, void *stream);
 /* out[t] = y, [T][heads * p], from convolved channels; writes ssm_state.  flags: MV_SSM_SCAN = token by token */
 enum { MV_SSM_SCAN = 1 };
@@ -664,6 +688,63 @@ int mv_ssm_step(const MvSsmArgs *args, int dtype, void *stream);
 int mv_gated_group_norm(const void *y, int64_t y_stride, const void *z, int64_t z_stride, const void *w, void *out,
                         int64_t out_stride, int rows, int heads, int p, int p_true, int norm_groups, float eps, int dtype,
                         void *stream);
+
+/* ---- K16 — gated delta rule (heads with a state S of `n` key channels x `p` columns; `groups` of keys and queries).  Per token
+ *     S <- g S;   u = beta (v - S^T k);   S <- S + k u^T;   o = S^T q
+ * with unit k and q (q also times q_scale), beta = sigmoid(raw beta), g = exp(-exp(a_log) softplus(a + dt_bias)), one per head or
+ * (channel_decay) per head and key channel.  State slots as in K15: state fp32 [2][slots][heads][n][p].  Channels of x: v [heads * p] |
+ * k [groups * n] | q [groups * n] at offsets 0, k_off, q_off; p % 16 == 0, n % 32 == 0 (padding holds zeros). */
+enum { MV_GATE_SILU = 0, MV_GATE_SIGMOID = 1 };
+typedef struct MvDeltaArgs {
+  const void *x;                    /* [T] rows of channels at x_stride: projected (step) or convolved (prefill) */
+  const void *beta, *a;             /* raw: [T] rows of heads; of heads, or (channel_decay) heads * n */
+  const void *gate;                 /* step: raw, [T] rows of heads * p */
+  const void *conv_w;               /* step: [taps][channels], no bias */
+  const void *dt_bias, *a_log;      /* [heads] or [heads * n]; [heads] */
+  const void *norm_w;               /* step: [p] */
+  void *conv_state;
+  float *state;
+  const int32_t *state_slots;       /* [n_seqs] */
+  const int32_t *cu_q, *cu_k;       /* prefill: token ranges; tokens before the step = key length - query length */
+  const int32_t *context_lens;      /* step: tokens including this one */
+  void *out, *workspace;            /* workspace: prefill, mv_delta_prefill_workspace_bytes() bytes (NULL: token by token) */
+  int64_t x_stride, beta_stride, a_stride, gate_stride, out_stride, slots, ws_bytes;
+  int n_seqs, max_q, total_q, channels, taps, heads, groups, p, p_true, n, k_off, q_off, channel_decay, gate_kind;
+  float eps, unit_eps, q_scale, out_scale;
+} MvDeltaArgs;
+/* out[t] = o, [T][heads * p], from convolved channels; writes state.  flags: MV_DELTA_SCAN = token by token */
+enum { MV_DELTA_SCAN = 1 };
+size_t mv_delta_prefill_workspace_bytes(int n_seqs, int total_q, int heads, int p, int n, int dtype);
+int mv_delta_prefill(const MvDeltaArgs *args, int dtype, int flags, void *stream);
+/* one token per sequence, from projected channels: convolution, recurrence and mv_head_norm_gate in one launch; writes both states */
+int mv_delta_step(const MvDeltaArgs *args, int dtype, void *stream);
+/* out[t] = per head: rms(y) over its p_true columns * w (shared by the heads) * silu or sigmoid (gate_kind) of gate * out_scale */
+int mv_head_norm_gate(const void *y, int64_t y_stride, const void *gate, int64_t gate_stride, const void *w, void *out,
+                      int64_t out_stride, int rows, int heads, int p, int p_true, float eps, int gate_kind, float out_scale,
+                      int dtype, void *stream);
+
+/* ---- K17 — mixture of experts.  A pair = (token t, choice c) at index t * top + c.
+ * Router: s = softmax(W x) over `outputs` (logits in fp32), choice scores s + correction; only outputs of the `keep` groups (of `groups`
+ * equal runs) with the largest choice score can be chosen; the `top` with the largest choice scores get weights s / (sum of the chosen
+ * s + 1e-20) * scale.  w [outputs][k] dense.  -> ids, weights [rows][top] */
+int mv_moe_route(const void *x, int64_t x_stride, const void *w, const void *correction, int32_t *ids, float *weights, int rows, int k,
+                 int outputs, int top, int groups, int keep, float scale, int dtype, void *stream);
+/* Sorts the pairs by expert: rows[pair] = its place (-1: id >= experts, no product), tokens[place] = its token; tiles
+ * [max_tiles][3] = expert (-1: none), first place, places (at most tile_m).  max_tiles >= pairs / tile_m + experts */
+int mv_moe_group(const int32_t *ids, int pairs, int top, int experts, int tile_m, int max_tiles, int32_t *rows, int32_t *tokens,
+                 int32_t *tiles, void *stream);
+/* out[place] = W[expert] x[tokens[place]] (tokens NULL: x[place]), W [experts][n][k]; act: W [experts][2][n][k], out = act(gate, up).
+ * 16-bit: W packed per expert (mv_pack_weight of all rows), tile_m 16, 32, 64 or 128; fp32: W as it is, tile_m 16.  n % 16 == 0,
+ * k % 64 == 0. */
+typedef struct MvMoeLinearArgs {
+  const void *x, *w;
+  void *out;
+  const int32_t *tokens, *tiles;
+  const MvGateAct *act;
+  int64_t x_stride, out_stride;
+  int max_tiles, tile_m, n, k;
+} MvMoeLinearArgs;
+int mv_moe_linear(const MvMoeLinearArgs *args, int dtype, void *stream);
 
 #ifdef __cplusplus
 }

@@ -144,12 +144,13 @@ __device__ __forceinline__ float clamped_glu(float gate, float up, float limit, 
   return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
 }
 
-// act(gate) * up on the fp32 accumulators of a gated projection.  gelu, clamped: fp32 throughout.  silu: the rounding points
+// act(gate) * up on the fp32 accumulators of a gated projection.  gelu, clamped, relu: fp32 throughout.  silu: the rounding points
 // of the unfused pair (GEMM -> dtype, silu -> dtype, product in fp32; the caller rounds it)
 template <typename Tag>
 __device__ __forceinline__ float gated_act(float gate, float up, const MvGateAct &a) {
   if (a.kind == MV_ACT_GELU) return __fmul_rn(gelu_tanh(gate), up);
   if (a.kind == MV_ACT_CLAMPED) return clamped_glu(gate, up, a.limit, a.alpha);
+  if (a.kind == MV_ACT_RELU) return __fmul_rn(fmaxf(gate, 0.f), up);
   const float gt = elem<Tag>::ld(elem<Tag>::st(gate)), ut = elem<Tag>::ld(elem<Tag>::st(up));
   float sl = gt / (1.0f + expf(-gt));                        // rmsnorm.hip: silu_and_mul_kernel
   sl = elem<Tag>::ld(elem<Tag>::st(sl));
@@ -215,15 +216,53 @@ __device__ __forceinline__ void rot_apply(const float (&x)[VEC], const float (&c
 // ---- host-side helpers ------------------------------------------------------
 static inline int mv_check_act(const MvGateAct *a) {
   if (!a) return MV_E_NULLPTR;
-  if (a->kind < MV_ACT_SILU || a->kind > MV_ACT_CLAMPED) return MV_E_RANGE;
+  if (a->kind < MV_ACT_SILU || a->kind > MV_ACT_RELU) return MV_E_RANGE;
   return a->kind == MV_ACT_CLAMPED && !(a->limit > 0.f) ? MV_E_RANGE : MV_OK;
 }
 static inline int mv_check_hip(hipError_t e) { return e == hipSuccess ? 0 : (int)e; }
 static inline bool mv_aligned16(const void *p) { return (((uintptr_t)p) & 15u) == 0; }
 
+// ---- what a query sees and how its scores become weights (MvAttnOpts) --------------------------------------------------
+struct AttnMask {
+  int window = 0, keep_first = 0;   // window > 0: key j of position i if i - j < window or j < keep_first
+  float softcap = 0.f, out_scale = 1.f;
+  const void *sink = nullptr;       // [heads] of dtype: one more term of the denominator
+};
+static inline AttnMask mv_attn_mask(const MvAttnOpts *o) {
+  AttnMask m;
+  if (o) {
+    m.window = o->window, m.keep_first = o->window > 0 ? o->keep_first : 0, m.softcap = o->softcap, m.sink = o->sink;
+    if (o->out_scale != 0.f) m.out_scale = o->out_scale;
+  }
+  return m;
+}
+static inline int mv_check_mask(const MvAttnOpts *o) {
+  if (!o) return MV_OK;
+  if (o->chunk < 0 || o->window < 0 || o->keep_first < 0 || (o->chunk > 0 && o->window > 0)) return MV_E_SHAPE;
+  return o->softcap < 0.f ? MV_E_RANGE : MV_OK;
+}
+// most keys that one query reads, in whole units; 0 = no bound
+static inline int64_t mv_attn_span(const MvAttnOpts *o, int unit) {
+  if (!o) return 0;
+  if (o->chunk > 0) return (int64_t)o->chunk + unit;   // (a chunk's edge inside a unit)
+  if (o->window > 0) return (int64_t)o->window + unit + ((int64_t)o->keep_first + unit - 1) / unit * unit;
+  return 0;
+}
+// cap * tanh(s / cap) in log2 units: `raw` an unscaled score, to_cap = scale / cap, cap_log2 = cap * log2(e)
+template <typename Tag>
+__device__ __forceinline__ float capped_log2(float raw, float to_cap, float cap_log2) {
+  const float z = raw * to_cap;
+  if constexpr (__is_same(Tag, f32_tag)) return cap_log2 * tanhf(z);
+  // 1 - 2 / (exp(2 z) + 1): hardware exponential and reciprocal, about 1e-7 of the cap
+  const float e = __builtin_amdgcn_exp2f(z * 2.8853900817779268f);
+  return cap_log2 * (1.f - 2.f * __builtin_amdgcn_rcpf(e + 1.f));
+}
+
 // rotary / window options of the attention entry points (NULL = none)
+static inline bool mv_needs_tables(const MvAttnOpts *o) { return !(o && o->interleaved && o->rot_pairs == 0); }
 static inline int mv_check_rot(const MvAttnOpts *o, int head_dim) {
   if (!o) return MV_OK;
+  if (o->norm_dim < 0 || o->norm_dim > head_dim) return MV_E_SHAPE;
   if (o->interleaved) return (o->rot_pairs < 0 || o->rot_pairs > head_dim / 2) ? MV_E_SHAPE : MV_OK;
   return (o->rot_pairs != 0 && o->rot_pairs != head_dim / 2) ? MV_E_SHAPE : MV_OK;   // halves: whole rows only
 }

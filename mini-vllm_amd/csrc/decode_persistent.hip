@@ -647,7 +647,7 @@ extern "C" int mv_decode_layers_persistent(const MvPersistLayer *layers_dev, int
   dp.q_stride = nqkv, dp.k_stride = nqkv, dp.v_stride = nqkv, dp.table_stride = a->table_stride, dp.num_blocks = a->num_blocks;
   dp.n_heads = H, dp.n_kv_heads = Hkv, dp.g_total = H / Hkv, dp.block_size = a->block_size;
   dp.bs_shift = (a->block_size & (a->block_size - 1)) == 0 ? __builtin_ctz((unsigned)a->block_size) : -1;
-  dp.max_blocks = a->max_blocks, dp.nsplit = ns, dp.scale_log2 = a->scale * 1.4426950408889634f;
+  dp.norm_dim = D, dp.max_blocks = a->max_blocks, dp.nsplit = ns, dp.scale_log2 = a->scale * 1.4426950408889634f;
   dp.positions = a->positions, dp.cos = a->cos, dp.sin = a->sin, dp.max_pos = a->max_pos, dp.eps = a->eps;
   dp.slot_mapping = a->slot_mapping;
   p.att_gx = wide ? Hkv / 4 : Hkv, p.att_gy = ns;

@@ -37,13 +37,26 @@ struct DecodeParams {
   int pairs = 0, interleaved = 0;   // rotary layout (common.h: rot_factors)
   // chunk > 0: a query at position i reads only the keys of its own chunk of positions, [i / chunk * chunk, i]
   int chunk = 0;
+  AttnMask mask;
+  int norm_dim = 0;         // columns that the head norms are means over
   int64_t out_stride = 0;   // elements between token rows of out; 0 = n_heads * D
 };
 
 // first key the query of a sequence with `ctx` tokens (its own included) may read
 __device__ __forceinline__ int decode_first_key(const DecodeParams &p, int ctx) {
+  if (p.mask.window > 0) return max(0, ctx - p.mask.window);
   return p.chunk > 0 && ctx > 0 ? (ctx - 1) / p.chunk * p.chunk : 0;
 }
+// the units of keys it reads: [0, head) hold the first keys that a window keeps, then [first, end)
+struct DecodeUnits {
+  int head, first, count;
+  __device__ __forceinline__ DecodeUnits(const DecodeParams &p, int ctx, int first_key, int unit) {
+    first = first_key / unit;
+    head = min((p.mask.keep_first + unit - 1) / unit, first);
+    count = max(0, head + (ctx + unit - 1) / unit - first);
+  }
+  __device__ __forceinline__ int at(int i) const { return i < head ? i : first + i - head; }
+};
 
 
 // ---- accesses to bytes that ANOTHER workgroup of the same launch wrote or will read (persistent decode kernel) -------
@@ -107,7 +120,7 @@ __device__ __forceinline__ void st2(uint16_t *p, uint16_t v) {
 // one head row (D elements on LPT lanes, VEC per lane): optional RMSNorm over the row (result rounded to dtype) and
 // the rotation by (cs, sn) — rope_qk_store_kernel's arithmetic and rounding points, statement for statement
 template <typename Tag, int D>
-__device__ __forceinline__ u32x4 norm_rope_row(const u32x4 &raw, const typename elem<Tag>::T *nw, float eps, int sub,
+__device__ __forceinline__ u32x4 norm_rope_row(const u32x4 &raw, const typename elem<Tag>::T *nw, float eps, int norm_dim, int sub,
                                                const float (&cs)[elem<Tag>::VEC], const float (&sn)[elem<Tag>::VEC],
                                                bool interleaved = false) {
   constexpr int VEC = elem<Tag>::VEC, LPT = D / VEC;
@@ -119,7 +132,7 @@ __device__ __forceinline__ u32x4 norm_rope_row(const u32x4 &raw, const typename 
 #pragma unroll
     for (int j = 0; j < VEC; ++j) ss = fmaf(x[j], x[j], ss);
     for (int off = 1; off < LPT; off <<= 1) ss += __shfl_xor(ss, off, 64);
-    const float rs = 1.0f / sqrtf(ss / (float)D + eps);
+    const float rs = 1.0f / sqrtf(ss / (float)norm_dim + eps);
     float w[VEC];
     const u32x4 wraw = *(const MV_AS1 u32x4 *)(nw + sub * VEC);
     unpack8<Tag>(wraw, w);

@@ -44,7 +44,7 @@ int pick_g(int g_total) {
 }
 
 bool make_plan(int batch, int n_heads, int n_kv_heads, int head_dim, int block_size,
-               int max_blocks, int dtype, int flags, int chunk, DecodePlan *pl) {
+               int max_blocks, int dtype, int flags, const MvAttnOpts *opts, DecodePlan *pl) {
   if (n_kv_heads <= 0 || n_heads % n_kv_heads) return false;
   if (head_dim != 64 && head_dim != 128 && head_dim != 256) return false;
   const int g_total = n_heads / n_kv_heads;
@@ -74,7 +74,8 @@ bool make_plan(int batch, int n_heads, int n_kv_heads, int head_dim, int block_s
     if (pl->wide) kv_groups = n_kv_heads / tpl;
   }
   int64_t max_ctx = (int64_t)max_blocks * block_size;
-  if (chunk > 0 && max_ctx > (int64_t)chunk + pl->unit) max_ctx = (int64_t)chunk + pl->unit;   // (a chunk's edge inside a unit)
+  const int64_t span = mv_attn_span(opts, pl->unit);
+  if (span > 0 && max_ctx > span) max_ctx = span;
   const int max_units = (int)((max_ctx + pl->unit - 1) / pl->unit);
   const int64_t wg = (int64_t)batch * kv_groups * pl->n_chunks;
   // the matrix-core kernel keeps 4 workgroups per CU resident (LDS): one wave of 1024 is enough
@@ -101,18 +102,18 @@ size_t align256(size_t x) { return (x + 255) & ~(size_t)255; }
 int mv_paged_decode_plan(int batch, int n_heads, int n_kv_heads, int head_dim, int block_size, int max_blocks, int dtype,
                          int flags, int *g_chunk, int *n_chunks, int *nsplit, int *wide, int *mfma, int *uniform) {
   DecodePlan pl;
-  if (!make_plan(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, dtype, flags, 0, &pl)) return MV_E_SHAPE;
+  if (!make_plan(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, dtype, flags, nullptr, &pl)) return MV_E_SHAPE;
   *g_chunk = pl.g_chunk, *n_chunks = pl.n_chunks, *nsplit = pl.nsplit, *wide = pl.wide, *mfma = pl.mfma, *uniform = pl.uniform;
   return MV_OK;
 }
 
 extern "C" size_t mv_paged_decode_workspace_bytes_ex(int batch, int n_heads, int n_kv_heads, int head_dim, int block_size,
-                                                     int max_blocks, int flags, int chunk) {
+                                                     int max_blocks, int flags, const MvAttnOpts *opts) {
   // sized for the widest element type so one buffer serves every dtype
   DecodePlan a, b;
   if (batch <= 0 ||
-      !make_plan(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, MV_BF16, flags, chunk, &a) ||
-      !make_plan(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, MV_F32, flags, chunk, &b))
+      !make_plan(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, MV_BF16, flags, opts, &a) ||
+      !make_plan(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, MV_F32, flags, opts, &b))
     return 256;
   const int ns = a.nsplit > b.nsplit ? a.nsplit : b.nsplit;
   if (ns <= 1) return 256;
@@ -122,7 +123,7 @@ extern "C" size_t mv_paged_decode_workspace_bytes_ex(int batch, int n_heads, int
 
 extern "C" size_t mv_paged_decode_workspace_bytes(int batch, int n_heads, int n_kv_heads,
                                                   int head_dim, int block_size, int max_blocks, int flags) {
-  return mv_paged_decode_workspace_bytes_ex(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, flags, 0);
+  return mv_paged_decode_workspace_bytes_ex(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, flags, nullptr);
 }
 
 namespace {
@@ -182,7 +183,7 @@ extern "C" int mv_rope_paged_decode_ex(const void *q, int64_t q_stride_tok, cons
                                     int max_blocks, int64_t num_blocks, float scale, void *workspace, size_t ws_bytes,
                                     int dtype, int flags, const MvAttnOpts *opts, void *stream) {
   if (batch == 0) return MV_OK;
-  if (!k || !v || !positions || !cos || !sin || !slot_mapping) return MV_E_NULLPTR;
+  if (!k || !v || !positions || !slot_mapping || (mv_needs_tables(opts) && (!cos || !sin))) return MV_E_NULLPTR;
   if (dtype != MV_BF16 && dtype != MV_F16) return dtype == MV_F32 ? MV_E_SHAPE : MV_E_DTYPE;
   if (max_blocks == 0 || num_blocks == 0 || n_kv_heads <= 0 || n_heads % n_kv_heads) return MV_E_SHAPE;
   if (!mv_aligned16(k) || !mv_aligned16(v) || (k_stride_tok & 7) || (v_stride_tok & 7) ||
@@ -190,7 +191,7 @@ extern "C" int mv_rope_paged_decode_ex(const void *q, int64_t q_stride_tok, cons
     return MV_E_ALIGN;
   if (int e = mv_check_rot(opts, head_dim)) return e;
   DecodePlan pl;
-  if (!make_plan(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, dtype, flags, opts ? opts->chunk : 0, &pl))
+  if (!make_plan(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, dtype, flags, opts, &pl))
     return MV_E_SHAPE;
   // vector kernel: up to 4 query heads per kv head; matrix-core kernel: one chunk of <= 16 heads
   if (pl.n_chunks != 1) return MV_E_SHAPE;
@@ -242,8 +243,9 @@ int paged_decode_impl(const void *q, int64_t q_stride_tok, const void *k_cache,
   DecodePlan pl;
   const int chunk = opts ? opts->chunk : 0;
   const int64_t out_stride = opts && opts->out_stride ? opts->out_stride : (int64_t)n_heads * head_dim;
-  if (chunk < 0 || out_stride < (int64_t)n_heads * head_dim) return MV_E_SHAPE;
-  if (!make_plan(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, dtype, flags, chunk, &pl))
+  if (int e = mv_check_mask(opts)) return e;
+  if (out_stride < (int64_t)n_heads * head_dim) return MV_E_SHAPE;
+  if (!make_plan(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, dtype, flags, opts, &pl))
     return MV_E_SHAPE;
   if (!mv_aligned16(q) || !mv_aligned16(k_cache) || !mv_aligned16(v_cache) || !mv_aligned16(out) ||
       (q_stride_tok * esz) % 16 || (out_stride * esz) % 16)
@@ -267,6 +269,8 @@ int paged_decode_impl(const void *q, int64_t q_stride_tok, const void *k_cache,
   p.max_blocks = max_blocks;
   p.nsplit = pl.nsplit;
   p.chunk = chunk;
+  p.mask = mv_attn_mask(opts);
+  p.norm_dim = opts && opts->norm_dim ? opts->norm_dim : head_dim;
   p.out_stride = out_stride;
   p.scale_log2 = scale * 1.4426950408889634f;
   p.ws_acc = nullptr;

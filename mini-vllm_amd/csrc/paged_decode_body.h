@@ -99,10 +99,9 @@ __device__ __forceinline__ void paged_decode_body(const DecodeParams &p, const i
   if (ctx > cap) ctx = (int)cap;
   if (ctx < 0) ctx = 0;
   const int first = decode_first_key(p, ctx);
-  const int units = (ctx + UNIT - 1) / UNIT, u_first = first / UNIT;
-  const int ups = (units - u_first + p.nsplit - 1) / p.nsplit;
-  const int u_begin = u_first + split * ups;
-  const int u_end = min(units, u_begin + ups);
+  const DecodeUnits units(p, ctx, first, UNIT);
+  const int ups = (units.count + p.nsplit - 1) / p.nsplit;
+  const int u_begin = split * ups, u_end = min(units.count, u_begin + ups);   // (places among the units read)
 
   // q fragments: this lane's 16-byte piece of each of the G heads
   u32x4 qraw[G];
@@ -121,16 +120,16 @@ __device__ __forceinline__ void paged_decode_body(const DecodeParams &p, const i
     const bool il = p.interleaved != 0;
     rot_factors<D, VEC>(p.cos, p.sin, pos, pos_ok, sub, p.pairs, il, cs, sn);
 #pragma unroll
-    for (int g = 0; g < G; ++g) qraw[g] = norm_rope_row<Tag, D>(qraw[g], (const T *)p.q_norm_w, p.eps, sub, cs, sn, il);
+    for (int g = 0; g < G; ++g) qraw[g] = norm_rope_row<Tag, D>(qraw[g], (const T *)p.q_norm_w, p.eps, p.norm_dim, sub, cs, sn, il);
     // the workgroup that will read the sequence's last token writes its K / V rows first (one wave; WIDE: its four
     // lane groups are the four kv heads, else lane group 0 has the workgroup's kv head)
     int64_t slot = p.slot_mapping ? (int64_t)p.slot_mapping[b] : -1;
     if (slot >= p.num_blocks * p.block_size) slot = -1;
-    const int u_last = ctx > 0 ? (ctx - 1) / UNIT : -1;
+    const int u_last = units.count - 1;
     if (write && slot >= 0 && u_last >= u_begin && u_last < u_end && wave == 0 && (WIDE || grp == 0)) {
       const u32x4 kraw = ld16<COH>((const T *)p.k_new + (int64_t)b * p.k_stride + (int64_t)hkv * D + sub * VEC);
       const u32x4 vraw = ld16<COH>((const T *)p.v_new + (int64_t)b * p.v_stride + (int64_t)hkv * D + sub * VEC);
-      const u32x4 krot = norm_rope_row<Tag, D>(kraw, (const T *)p.k_norm_w, p.eps, sub, cs, sn, il);
+      const u32x4 krot = norm_rope_row<Tag, D>(kraw, (const T *)p.k_norm_w, p.eps, p.norm_dim, sub, cs, sn, il);
       *(MV_AS1 u32x4 *)((T *)p.k_cache + (slot * p.n_kv_heads + hkv) * D + sub * VEC) = krot;
       *(MV_AS1 u32x4 *)((T *)p.v_cache + (slot * p.n_kv_heads + hkv) * D + sub * VEC) = vraw;
       asm volatile("s_waitcnt vmcnt(0)" ::: "memory");   // the rows are in L2 before any wave of the workgroup asks
@@ -143,6 +142,10 @@ __device__ __forceinline__ void paged_decode_body(const DecodeParams &p, const i
   for (int g = 0; g < G; ++g) {
     m[g] = NEG_BIG;
     l[g] = 0.f;
+    if (p.mask.sink && split == 0 && wave == 0 && (WIDE || grp == 0) && ctx > 0) {
+      m[g] = elem<Tag>::ld(((const T *)p.mask.sink)[h0 + (g < g_live ? g : 0)]) * 1.4426950408889634f;
+      l[g] = 1.f;
+    }
 #pragma unroll
     for (int j = 0; j < VEC; ++j) acc[g][j] = 0.f;
   }
@@ -169,7 +172,7 @@ __device__ __forceinline__ void paged_decode_body(const DecodeParams &p, const i
       const int off = WIDE ? i : i * TPL + grp;  // token of this lane within the tile
       const int tok = tile_base + off;
       int64_t row;
-      bool ok = tok < ctx && tok >= first;
+      bool ok = tok < ctx && (tok >= first || tok < p.mask.keep_first);
       if constexpr (UNIFORM) {
         ok = ok && uni_row >= 0;
         row = (uni_row >= 0 ? uni_row : 0) + (ok ? off : 0);
@@ -189,6 +192,7 @@ __device__ __forceinline__ void paged_decode_body(const DecodeParams &p, const i
     }
   };
 
+  const float softcap = p.mask.softcap, to_cap = softcap > 0.f ? p.scale_log2 * 0.6931471805599453f / softcap : 0.f;
   auto consume_tile = [&](const u32x4 (&kraw)[NLOAD], const u32x4 (&vraw)[NLOAD], const bool (&valid)[NLOAD]) {
     // scores (log2 domain) + online softmax, per query head
     float pr[G][NLOAD];
@@ -197,7 +201,8 @@ __device__ __forceinline__ void paged_decode_body(const DecodeParams &p, const i
       float mx = m[g];
 #pragma unroll
       for (int i = 0; i < NLOAD; ++i) {
-        float s = token_sum<LPT>(dot16B<Tag>(qraw[g], kraw[i])) * p.scale_log2;
+        float s = token_sum<LPT>(dot16B<Tag>(qraw[g], kraw[i]));
+        s = softcap > 0.f ? capped_log2<Tag>(s, to_cap, softcap * 1.4426950408889634f) : s * p.scale_log2;
         s = valid[i] ? s : -INFINITY;
         pr[g][i] = s;
         mx = fmaxf(mx, s);
@@ -228,14 +233,14 @@ __device__ __forceinline__ void paged_decode_body(const DecodeParams &p, const i
     }
   };
 
-  // a tile at or past the context is skipped whole (wave-uniform)
-  auto live = [&](int u) { return u < u_end && (u * NW + wave) * TILE < ctx; };
+  // a tile at or past the context is skipped whole (wave-uniform; the units ascend)
+  auto live = [&](int u) { return u < u_end && (units.at(u) * NW + wave) * TILE < ctx; };
   // (round 2: a second register set with the next tile's loads in flight during the arithmetic — 256 VGPRs,
   //  2 waves per SIMD — measured no faster than this loop, 166 vs 165 us: the HBM side is the limit)
   for (int u = u_begin; live(u); ++u) {
     u32x4 kraw[NLOAD], vraw[NLOAD];
     bool valid[NLOAD];
-    load_tile(u, kraw, vraw, valid);
+    load_tile(units.at(u), kraw, vraw, valid);
     consume_tile(kraw, vraw, valid);
   }
 
@@ -294,7 +299,7 @@ __device__ __forceinline__ void paged_decode_body(const DecodeParams &p, const i
     const int h = (hkv0 + hg) * p.g_total + chunk * G + g;
     const int64_t os = p.out_stride ? p.out_stride : (int64_t)p.n_heads * D;
     if (p.nsplit == 1) {
-      const float o = L > 0.f ? A / L : 0.f;
+      const float o = L > 0.f ? A / L * p.mask.out_scale : 0.f;
       if constexpr (sizeof(T) == 2) st2<COH>((uint16_t *)p.out + (int64_t)b * os + h * D + d, elem<Tag>::st(o));
       else ((T *)p.out)[(int64_t)b * os + h * D + d] = elem<Tag>::st(o);
     } else {
@@ -330,7 +335,7 @@ struct ReduceLds {
 template <typename Tag, int D, bool COH = false>
 __device__ __forceinline__ void paged_decode_reduce_body(const float *ws_acc, const float *ws_ml, typename elem<Tag>::T *out,
                                                          const int nsplit, const int64_t bh, const int tid, const bool write,
-                                                         float *lds) {
+                                                         float *lds, const float out_scale = 1.f) {
   constexpr int D4 = D / 4, NQ = 128 / D4;    // column pieces; split groups (4 at D = 128, 8 at D = 64)
   constexpr int kMax = 64, PER = kMax / NQ;   // kMaxSplits; rows per thread at most
   typedef MV_AS3 f32x4 lds_f4;
@@ -385,11 +390,11 @@ __device__ __forceinline__ void paged_decode_reduce_body(const float *ws_acc, co
     if constexpr (COH && sizeof(typename elem<Tag>::T) == 2) {
       uint32_t r[4];
 #pragma unroll
-      for (int e = 0; e < 4; ++e) r[e] = elem<Tag>::st(L > 0.f ? A[e] / L : 0.f);
+      for (int e = 0; e < 4; ++e) r[e] = elem<Tag>::st(L > 0.f ? A[e] / L * out_scale : 0.f);
       st8<true>(o, u32x2{r[0] | (r[1] << 16), r[2] | (r[3] << 16)});
     } else {
 #pragma unroll
-      for (int e = 0; e < 4; ++e) o[e] = elem<Tag>::st(L > 0.f ? A[e] / L : 0.f);
+      for (int e = 0; e < 4; ++e) o[e] = elem<Tag>::st(L > 0.f ? A[e] / L * out_scale : 0.f);
     }
   }
 }
@@ -398,11 +403,11 @@ template <typename Tag, int D>
 __global__ void __launch_bounds__(128) paged_decode_reduce_kernel(const float *__restrict__ ws_acc,
                                                                   const float *__restrict__ ws_ml,
                                                                   typename elem<Tag>::T *__restrict__ out,
-                                                                  int nsplit, int n_heads, int64_t out_stride) {
+                                                                  int nsplit, int n_heads, int64_t out_stride, float out_scale) {
   __shared__ __attribute__((aligned(16))) float lds[ReduceLds<D>::FLOATS];
   // (the body writes row bh of a dense [B * H, D] array: shift the base so that this row lands in its strided place)
   const int64_t b = blockIdx.x / n_heads;
   paged_decode_reduce_body<Tag, D>(ws_acc, ws_ml, out + b * (out_stride - (int64_t)n_heads * D), nsplit, blockIdx.x, threadIdx.x,
-                                   true, lds);
+                                   true, lds, out_scale);
 }
 

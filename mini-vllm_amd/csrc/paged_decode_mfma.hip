@@ -86,10 +86,9 @@ __global__ void __launch_bounds__(256, KLDS ? 2 : 4) paged_decode_mfma_kernel(De
   if (ctx > cap) ctx = (int)cap;
   if (ctx < 0) ctx = 0;
   const int first = decode_first_key(p, ctx);
-  const int units = (ctx + UNIT - 1) / UNIT, u_first = first / UNIT;
-  const int ups = (units - u_first + p.nsplit - 1) / p.nsplit;
-  const int u_begin = u_first + split * ups;
-  const int u_end = min(units, u_begin + ups);
+  const DecodeUnits units(p, ctx, first, UNIT);
+  const int ups = (units.count + p.nsplit - 1) / p.nsplit;
+  const int u_begin = split * ups, u_end = min(units.count, u_begin + ups);   // (places among the units read)
 
   // Q^T fragments (B operand): lane (q = i16, quad) holds Q[q][32s + 8 quad .. +8)
   u32x4 qf[4];
@@ -123,7 +122,7 @@ __global__ void __launch_bounds__(256, KLDS ? 2 : 4) paged_decode_mfma_kernel(De
       const float tot[4] = {a0 + a2, a1 + a3, a2 + a0, a3 + a1};                                       // sub ^ 8
 #pragma unroll
       for (int s = 0; s < 4; ++s) {
-        const float rs = 1.0f / sqrtf(tot[s] / (float)D + p.eps);
+        const float rs = 1.0f / sqrtf(tot[s] / (float)p.norm_dim + p.eps);
         float w[8];
         unpack8<Tag>(*reinterpret_cast<const u32x4 *>((const T *)p.q_norm_w + 32 * s + 8 * quad), w);
 #pragma unroll
@@ -166,14 +165,14 @@ __global__ void __launch_bounds__(256, KLDS ? 2 : 4) paged_decode_mfma_kernel(De
     // the new token's K / V rows: written by the workgroup (chunk 0) that will read them, before anybody does
     int64_t slot = p.slot_mapping ? (int64_t)p.slot_mapping[b] : -1;
     if (slot >= p.num_blocks * p.block_size) slot = -1;
-    const int u_last = ctx > 0 ? (ctx - 1) / UNIT : -1;
+    const int u_last = units.count - 1;
     if (slot >= 0 && chunk == 0 && u_last >= u_begin && u_last < u_end && wave == 0 && lane < 16) {
       const int sub = lane;
       float cs[8], sn[8];
       rot_factors<D, 8>(p.cos, p.sin, pos, pos_ok, sub, p.pairs, p.interleaved != 0, cs, sn);
       const u32x4 kraw = *reinterpret_cast<const u32x4 *>((const T *)p.k_new + (int64_t)b * p.k_stride + (int64_t)hkv * D + sub * 8);
       const u32x4 vraw = *reinterpret_cast<const u32x4 *>((const T *)p.v_new + (int64_t)b * p.v_stride + (int64_t)hkv * D + sub * 8);
-      const u32x4 krot = norm_rope_row<Tag, D>(kraw, (const T *)p.k_norm_w, p.eps, sub, cs, sn, p.interleaved != 0);
+      const u32x4 krot = norm_rope_row<Tag, D>(kraw, (const T *)p.k_norm_w, p.eps, p.norm_dim, sub, cs, sn, p.interleaved != 0);
       *reinterpret_cast<u32x4 *>((T *)p.k_cache + (slot * p.n_kv_heads + hkv) * D + sub * 8) = krot;
       *reinterpret_cast<u32x4 *>((T *)p.v_cache + (slot * p.n_kv_heads + hkv) * D + sub * 8) = vraw;
       asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
@@ -184,6 +183,11 @@ __global__ void __launch_bounds__(256, KLDS ? 2 : 4) paged_decode_mfma_kernel(De
 #pragma unroll
   for (int dt = 0; dt < 8; ++dt) oacc[dt] = f32x4{0.f, 0.f, 0.f, 0.f};
   float m_run = -1e30f, l_run = 0.f;
+  if (p.mask.sink && split == 0 && wave == 0 && ctx > 0) {
+    m_run = elem<Tag>::ld(((const T *)p.mask.sink)[h0 + min(i16, g_live - 1)]) * 1.4426950408889634f;
+    l_run = quad == 0 ? 1.f : 0.f;
+  }
+  const float softcap = p.mask.softcap, to_cap = softcap > 0.f ? p.scale_log2 * 0.6931471805599453f / softcap : 0.f;
 
   const int32_t *table = p.block_tables + (int64_t)b * p.table_stride;
   const int64_t row_elems = (int64_t)p.n_kv_heads * D;
@@ -192,7 +196,7 @@ __global__ void __launch_bounds__(256, KLDS ? 2 : 4) paged_decode_mfma_kernel(De
   const int q4 = i16 >> 2, pp = i16 & 3;
 
   for (int u = u_begin; u < u_end; ++u) {
-    const int tile_base = (u * NW + wave) * TILE;
+    const int tile_base = (units.at(u) * NW + wave) * TILE;
     if (tile_base >= ctx) break;  // wave-uniform
     const int bi = p.bs_shift >= 0 ? (tile_base >> p.bs_shift) : (tile_base / p.block_size);
     const int blk = bi < p.max_blocks ? __builtin_amdgcn_readfirstlane(table[bi]) : -1;
@@ -268,8 +272,8 @@ __global__ void __launch_bounds__(256, KLDS ? 2 : 4) paged_decode_mfma_kernel(De
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int key = tile_base + 16 * kt + 4 * quad + r;
-        float s = sacc[kt][r] * p.scale_log2;
-        s = (blk_ok && key < ctx && key >= first) ? s : -INFINITY;
+        float s = softcap > 0.f ? capped_log2<Tag>(sacc[kt][r], to_cap, softcap * 1.4426950408889634f) : sacc[kt][r] * p.scale_log2;
+        s = (blk_ok && key < ctx && (key >= first || key < p.mask.keep_first)) ? s : -INFINITY;
         sacc[kt][r] = s;
         mx = fmaxf(mx, s);
       }
@@ -345,7 +349,7 @@ __global__ void __launch_bounds__(256, KLDS ? 2 : 4) paged_decode_mfma_kernel(De
     const int h = h0 + g;
     if (p.nsplit == 1) {
       const int64_t os = p.out_stride ? p.out_stride : (int64_t)p.n_heads * D;
-      ((T *)p.out)[(int64_t)b * os + h * D + d] = elem<Tag>::st(L > 0.f ? A / L : 0.f);
+      ((T *)p.out)[(int64_t)b * os + h * D + d] = elem<Tag>::st(L > 0.f ? A / L * p.mask.out_scale : 0.f);
     } else {
       const int64_t slot = ((int64_t)b * p.n_heads + h) * p.nsplit + split;
       p.ws_acc[slot * D + d] = A;

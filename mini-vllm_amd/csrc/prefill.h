@@ -12,6 +12,7 @@ struct PrefillParams {
   int n_heads, n_kv_heads, head_dim, block_size, table_width;
   float scale;
   int chunk;            // > 0: position i reads only the keys of its chunk of positions, [i / chunk * chunk, i]
+  AttnMask mask;
   int64_t out_stride;   // elements between token rows of out
 };
 

@@ -22,7 +22,8 @@ extern "C" int mv_prefill_varlen_ex(const void *q, int64_t q_stride_tok, const v
     return MV_E_SHAPE;
   if (head_dim != 64 && head_dim != 128 && head_dim != 256) return MV_E_SHAPE;
   const int64_t out_stride = opts && opts->out_stride ? opts->out_stride : (int64_t)n_heads * head_dim;
-  if (out_stride < (int64_t)n_heads * head_dim || (opts && opts->chunk < 0)) return MV_E_SHAPE;
+  if (out_stride < (int64_t)n_heads * head_dim) return MV_E_SHAPE;
+  if (int e = mv_check_mask(opts)) return e;
   if (dtype != MV_BF16 && dtype != MV_F16 && dtype != MV_F32) return MV_E_DTYPE;
   const int esz = dtype == MV_F32 ? 4 : 2;
   if (!mv_aligned16(q) || !mv_aligned16(out) || (q_stride_tok * esz) % 16 || (out_stride * esz) % 16 ||
@@ -41,6 +42,7 @@ extern "C" int mv_prefill_varlen_ex(const void *q, int64_t q_stride_tok, const v
   p.table_width = paged ? (int)((max_seqlen_k + block_size - 1) / block_size) : 0;
   p.scale = scale;
   p.chunk = opts ? opts->chunk : 0;
+  p.mask = mv_attn_mask(opts);
   p.out_stride = out_stride;
   hipStream_t st = (hipStream_t)stream;
   // MV_PREFILL_SIMPLE routes 16-bit tensors through the vector-ALU kernel (debug aid)

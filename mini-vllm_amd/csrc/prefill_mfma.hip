@@ -1,4 +1,4 @@
-// K2 (MFMA path) — packed varlen causal flash attention for gfx950, bf16/f16, D = 64 / 128, whole or chunked context
+// K2 (MFMA path) — packed varlen causal flash attention for gfx950, bf16/f16, D = 64 / 128, whole, chunked or windowed context
 // (reference call site: flash_attn_varlen_func, minivllm/models/layers/attention.py:422-433;
 //  semantics of the fallback :467-504,554-597 with bottom-right aligned causal mask).
 //
@@ -116,9 +116,12 @@ __device__ __forceinline__ void half_swap(float x, float &lo, float &hi) {
 // instructions — ~100 issue cycles apiece — are shared by twice the rows)
 // DH = head dim (64 or 128; the names below shadow the file's D = 128 constants).  CHUNK: position i reads only the keys of its
 // chunk of p.chunk positions: a workgroup starts at the tile of its first row's chunk, a wave skips the tiles in front of its
-// own first row's chunk, and the tiles that hold a chunk's edge take the masked path.
-template <typename Tag, int NW, bool PIPE, int DH, bool CHUNK>
+// own first row's chunk, and the tiles that hold a chunk's edge take the masked path.  WINDOW (MASK = 2): the same with the first key
+// of a row's window, the tiles of the first keys that the window keeps in front of the list; also capped scores, a sink in the
+// denominator and a factor of the output (common.h: AttnMask).
+template <typename Tag, int NW, bool PIPE, int DH, int MASK>
 __global__ void __launch_bounds__(NW * 64, 2) prefill_mfma_kernel(PrefillParams p, float rescale_thr) {
+  constexpr bool CHUNK = MASK == 1, WINDOW = MASK == 2;
   constexpr int NBUF = 2;   // K|V tile buffers in LDS
   constexpr int D = DH, NS = D / 16, NDT = D / 32, ROW_BYTES = D * 2, TILE_BYTES = BN * ROW_BYTES;
   constexpr int CH = D / 8, RPI = 64 / CH;   // 16-byte chunks of a row; rows that one 1-KiB DMA instruction fills
@@ -169,14 +172,24 @@ __global__ void __launch_bounds__(NW * 64, 2) prefill_mfma_kernel(PrefillParams 
 #pragma unroll
     for (int i = 0; i < 16; ++i) oacc[dt][i] = 0.f;
   float m_run = -1e30f, l_run = 0.f;
-  const float scale_log2 = p.scale * 1.4426950408889634f;
+  if (WINDOW && p.mask.sink) {   // (a row's two half-waves: the sink counts once)
+    m_run = elem<Tag>::ld(((const T *)p.mask.sink)[head]) * 1.4426950408889634f;
+    l_run = h == 0 ? 1.f : 0.f;
+  }
+  const bool capped = WINDOW && p.mask.softcap > 0.f;
+  const float cap_log2 = p.mask.softcap * 1.4426950408889634f, to_cap = capped ? p.scale / p.mask.softcap : 0.f;
+  const float scale_log2 = capped ? 1.f : p.scale * 1.4426950408889634f;
 
   // keys needed by this query block: everything up to its last row's diagonal
   const int q_last = min(sq, (qb + 1) * BM) - 1;
   const int kv_len = min(sk, q_last + shift + 1);
   // CHUNK: tiles count from the one that holds the first visible key of the workgroup's first row
-  const int kv_base = CHUNK ? (shift + qb * BM) / p.chunk * p.chunk / BN * BN : 0;
-  const int n_tiles = (kv_len - kv_base + BN - 1) / BN;
+  const int window = WINDOW && p.mask.window > 0 ? p.mask.window : 1 << 30, keep = WINDOW ? p.mask.keep_first : 0;
+  const int kv_base = CHUNK ? (shift + qb * BM) / p.chunk * p.chunk / BN * BN
+                            : WINDOW ? max(0, shift + qb * BM - window + 1) / BN * BN : 0;
+  const int head_tiles = WINDOW ? min((keep + BN - 1) / BN, kv_base / BN) : 0;   // of the kept first keys
+  const int n_tiles = head_tiles + (kv_len - kv_base + BN - 1) / BN;
+  auto tile_key = [&](int t) { return WINDOW && t < head_tiles ? t * BN : kv_base + (t - head_tiles) * BN; };
   const int wave_qpos_min = shift + qb * BM + wave * 32;  // smallest key limit among this wave's rows
   // ... and the largest: tiles that start beyond it are masked out for EVERY row of this wave (the workgroup walks the
   // tiles its LAST wave needs): such a wave skips the tile's arithmetic (p = 0 for all its scores: maximum, sum and
@@ -184,8 +197,8 @@ __global__ void __launch_bounds__(NW * 64, 2) prefill_mfma_kernel(PrefillParams 
   // each: 5 % of the MFMAs at 4096 tokens, 22 % at 1024, more for short prompts.
   const int wave_qpos_max = wave_qpos_min + 31;
   // CHUNK: first visible key of the wave's first and last row
-  const int wave_lo_min = CHUNK ? wave_qpos_min / p.chunk * p.chunk : 0;
-  const int wave_lo_max = CHUNK ? wave_qpos_max / p.chunk * p.chunk : 0;
+  const int wave_lo_min = CHUNK ? wave_qpos_min / p.chunk * p.chunk : WINDOW ? max(0, wave_qpos_min - window + 1) : 0;
+  const int wave_lo_max = CHUNK ? wave_qpos_max / p.chunk * p.chunk : WINDOW ? max(0, wave_qpos_max - window + 1) : 0;
 
   const bool paged = p.block_tables != nullptr;
   const T *ksrc = paged ? (const T *)p.k_cache : (const T *)p.k;
@@ -217,7 +230,7 @@ __global__ void __launch_bounds__(NW * 64, 2) prefill_mfma_kernel(PrefillParams 
   };
   auto dma = [&](int t, int buf) {
     {
-      const int kv0f = kv_base + t * BN;
+      const int kv0f = tile_key(t);
       if (kv0f + BN <= sk) {   // a full tile: one scalar base + the per-lane constants
         int64_t base_row = k0 + kv0f;
         tile_ok_next = true;
@@ -240,7 +253,7 @@ __global__ void __launch_bounds__(NW * 64, 2) prefill_mfma_kernel(PrefillParams 
         return;
       }
     }
-    const int kv0 = kv_base + t * BN;
+    const int kv0 = tile_key(t);
     int64_t base_row = k0 + kv0;
     tile_ok_next = true;
     if (paged) {
@@ -351,18 +364,24 @@ __global__ void __launch_bounds__(NW * 64, 2) prefill_mfma_kernel(PrefillParams 
     }
   };
   auto softmax_phase = [&](const int t, const bool tile_ok) __attribute__((always_inline)) {
-    const int kv0 = kv_base + t * BN;
+    const int kv0 = tile_key(t);
+    if (WINDOW && capped) {
+#pragma unroll
+      for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+        for (int i = 0; i < 16; ++i) sacc[kt][i] = capped_log2<Tag>(sacc[kt][i], to_cap, cap_log2);
+    }
     // ---- mask (only tiles that touch the diagonal / the ragged end: wave-uniform branch)
-    if ((kv0 + BN - 1 > wave_qpos_min) || (kv0 + BN > sk) || !tile_ok || (CHUNK && kv0 < wave_lo_max)) {
+    if ((kv0 + BN - 1 > wave_qpos_min) || (kv0 + BN > sk) || !tile_ok || ((CHUNK || WINDOW) && kv0 < wave_lo_max)) {
       const int klim = tile_ok ? min(qidx + shift, sk - 1) : -1;  // last key this query row may see
       // CHUNK: ... and the first.  A chunk is >= 32 positions here, so the wave's 32 rows meet at most one chunk edge
-      const int lane_lo = CHUNK ? (qidx + shift >= wave_lo_max ? wave_lo_max : wave_lo_min) : 0;
+      const int lane_lo = CHUNK ? (qidx + shift >= wave_lo_max ? wave_lo_max : wave_lo_min) : WINDOW ? qidx + shift - window + 1 : 0;
 #pragma unroll
       for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
           const int key = kv0 + kt * 32 + (i & 3) + 8 * (i >> 2) + 4 * h;
-          sacc[kt][i] = key <= klim && (!CHUNK || key >= lane_lo) ? sacc[kt][i] : -INFINITY;
+          sacc[kt][i] = key <= klim && (!(CHUNK || WINDOW) || key >= lane_lo || (WINDOW && key < keep)) ? sacc[kt][i] : -INFINITY;
         }
     }
     // ---- online softmax in the log2 domain: p = exp2(s*c - m), one FMA + one exp per score
@@ -492,7 +511,8 @@ __global__ void __launch_bounds__(NW * 64, 2) prefill_mfma_kernel(PrefillParams 
   auto tile = [&](const int t, auto BUF) __attribute__((always_inline)) {
     constexpr int BO = decltype(BUF)::value * 2 * TILE_BYTES;   // byte offset of this tile's K|V buffer
     tile_top(t);
-    if (kv_base + t * BN <= wave_qpos_max && (!CHUNK || kv_base + t * BN + BN > wave_lo_min)) {
+    const int kv0 = tile_key(t);
+    if (kv0 <= wave_qpos_max && (!(CHUNK || WINDOW) || kv0 + BN > wave_lo_min || (WINDOW && kv0 < keep))) {
       qk_phase(std::integral_constant<int, BO>{}, 0u);
       softmax_phase(t, tile_ok);
       pv_phase(std::integral_constant<int, BO>{}, 0u);
@@ -512,7 +532,7 @@ __global__ void __launch_bounds__(NW * 64, 2) prefill_mfma_kernel(PrefillParams 
   //      the (no longer needed) K|V buffers — 16-byte chunks XOR-swizzled by row so that both the 8-byte writes and the
   //      16-byte reads spread over the banks — and leaves as whole rows: one instruction = four contiguous 256-B rows.
   const float l_tot = l_run + __shfl_xor(l_run, 32, 64);
-  const float inv = l_tot > 0.f ? 1.0f / l_tot : 0.f;
+  const float inv = l_tot > 0.f ? (WINDOW ? p.mask.out_scale : 1.0f) / l_tot : 0.f;
   // (every wave passed the barrier that ends the last tile: nobody reads the K|V buffers any more; a wave then only
   //  touches its own 8 KiB, so no further barrier)
   char *stage = smem + wave * (32 * ROW_BYTES);
@@ -992,7 +1012,8 @@ __global__ void __launch_bounds__(256, 1) prefill_mfma64_kernel(PrefillParams p,
 
 int mv_prefill_mfma_launch(const PrefillParams &p, int dtype, int variant, hipStream_t stream) {
   if ((p.head_dim != 64 && p.head_dim != 128) || (dtype != MV_BF16 && dtype != MV_F16)) return MV_E_SHAPE;
-  if (p.chunk > 0 && p.chunk < 32) return MV_E_SHAPE;   // (a handful of keys per query: the vector kernel's job)
+  const bool general = p.mask.window > 0 || p.mask.softcap > 0.f || p.mask.sink || p.mask.out_scale != 1.f;
+  if (p.chunk > 0 && (p.chunk < 32 || general)) return MV_E_SHAPE;   // (a handful of keys per query: the vector kernel's job)
   if (p.block_tables && (p.block_size % BN) != 0) return MV_E_SHAPE;  // a 64-key tile must sit in one block
   // 8 waves (256 query rows) per workgroup share a K/V tile where the sequences are long enough that the larger
   // blocks still fill the chip evenly; short prompts keep 4 waves x 2 workgroups per CU (measured per shape,
@@ -1010,7 +1031,7 @@ int mv_prefill_mfma_launch(const PrefillParams &p, int dtype, int variant, hipSt
   const float thr_pick = 6.0f + 2.0f * (float)((variant >> 6) & 3);   // bench switch: rescale threshold 6 / 8 / 10 / 12
   variant &= 7;
   // the comparison variants (3, 4, 5) exist for whole-context attention at head dim 128
-  if ((p.head_dim != D || p.chunk > 0) && variant > 2) return MV_E_RANGE;
+  if ((p.head_dim != D || p.chunk > 0 || general) && variant > 2) return MV_E_RANGE;
   if (variant == 5) {   // bench switch: 64 query rows per wave, one wave per SIMD (profiles/r03_prefill_kernel.md)
     const int qblocks = (p.max_seqlen_q + 255) / 256;
     if (qblocks == 0 || p.n_seqs == 0) return MV_OK;
@@ -1037,20 +1058,22 @@ int mv_prefill_mfma_launch(const PrefillParams &p, int dtype, int variant, hipSt
   if (q_blocks == 0 || p.n_seqs == 0) return MV_OK;
   dim3 grid(p.n_heads, p.n_seqs, q_blocks), block(nw * 64);
   const size_t lds = (size_t)4 * BN * p.head_dim * 2;   // 2 x (K tile + V tile): 64 KiB at D = 128 -> two workgroups per CU
-#define MV_PF_LAUNCH(NWAVES, PIPED, DH, CHUNK)                                                                           \
+#define MV_PF_LAUNCH(NWAVES, PIPED, DH, MASK)                                                                            \
   do {                                                                                                                  \
-    if (dtype == MV_BF16) hipLaunchKernelGGL((prefill_mfma_kernel<bf16_tag, NWAVES, PIPED, DH, CHUNK>), grid, block, lds, stream, p, thr); \
-    else hipLaunchKernelGGL((prefill_mfma_kernel<f16_tag, NWAVES, PIPED, DH, CHUNK>), grid, block, lds, stream, p, thr);   \
+    if (dtype == MV_BF16) hipLaunchKernelGGL((prefill_mfma_kernel<bf16_tag, NWAVES, PIPED, DH, MASK>), grid, block, lds, stream, p, thr); \
+    else hipLaunchKernelGGL((prefill_mfma_kernel<f16_tag, NWAVES, PIPED, DH, MASK>), grid, block, lds, stream, p, thr);   \
   } while (0)
 #define MV_PF_DIMS(NWAVES)                                                   \
   do {                                                                       \
-    if (p.head_dim == 64 && p.chunk > 0) MV_PF_LAUNCH(NWAVES, true, 64, true);   \
-    else if (p.head_dim == 64) MV_PF_LAUNCH(NWAVES, true, 64, false);          \
-    else if (p.chunk > 0) MV_PF_LAUNCH(NWAVES, true, 128, true);               \
-    else MV_PF_LAUNCH(NWAVES, true, 128, false);                               \
+    if (p.head_dim == 64 && general) MV_PF_LAUNCH(NWAVES, true, 64, 2);      \
+    else if (p.head_dim == 64 && p.chunk > 0) MV_PF_LAUNCH(NWAVES, true, 64, 1); \
+    else if (p.head_dim == 64) MV_PF_LAUNCH(NWAVES, true, 64, 0);            \
+    else if (general) MV_PF_LAUNCH(NWAVES, true, 128, 2);                    \
+    else if (p.chunk > 0) MV_PF_LAUNCH(NWAVES, true, 128, 1);                \
+    else MV_PF_LAUNCH(NWAVES, true, 128, 0);                                 \
   } while (0)
-  if (!pipe && nw == 8) MV_PF_LAUNCH(8, false, 128, false);
-  else if (!pipe) MV_PF_LAUNCH(4, false, 128, false);
+  if (!pipe && nw == 8) MV_PF_LAUNCH(8, false, 128, 0);
+  else if (!pipe) MV_PF_LAUNCH(4, false, 128, 0);
   else if (nw == 8) MV_PF_DIMS(8);
   else MV_PF_DIMS(4);
 #undef MV_PF_DIMS

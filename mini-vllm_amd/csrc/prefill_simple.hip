@@ -53,18 +53,23 @@ __global__ void __launch_bounds__(256) prefill_simple_kernel(PrefillParams p) {
   const int k0 = p.cu_k[seq], sk = p.cu_k[seq + 1] - k0;
   const int pos = (tok - q0) + (sk - sq);       // bottom-right aligned causal
   const int nkeys = min(sk, pos + 1);
-  const int first = p.chunk > 0 ? pos / p.chunk * p.chunk : 0;
+  const int keep = p.mask.keep_first;
+  const int first = p.chunk > 0 ? pos / p.chunk * p.chunk : p.mask.window > 0 ? max(0, pos - p.mask.window + 1) : 0;
+  // keys [0, head) and [first, nkeys), TPL at a time
+  const int head_keys = min(keep, first), skip = (head_keys + TPL - 1) / TPL * TPL;
 
   const T *qp = (const T *)p.q + (int64_t)tok * p.q_stride + (int64_t)h * D + sub * VEC;
   const u32x4 qraw = *reinterpret_cast<const u32x4 *>(qp);
   float m = -1e30f, l = 0.f, acc[VEC];
+  if (p.mask.sink && grp == 0) m = elem<Tag>::ld(((const T *)p.mask.sink)[h]) * 1.4426950408889634f, l = 1.f;
 #pragma unroll
   for (int j = 0; j < VEC; ++j) acc[j] = 0.f;
   const float scale_log2 = p.scale * 1.4426950408889634f;
+  const float cap = p.mask.softcap, to_cap = cap > 0.f ? p.scale / cap : 0.f, cap_log2 = cap * 1.4426950408889634f;
 
-  for (int base = first; base < nkeys; base += TPL) {
-    const int key = base + grp;
-    bool ok = key < nkeys;
+  for (int at = 0; at < skip + nkeys - first; at += TPL) {
+    const int key = (at < skip ? at : first + at - skip) + grp;
+    bool ok = at < skip ? key < head_keys : key < nkeys;
     const T *kp = nullptr, *vp = nullptr;
     if (p.block_tables) {
       int blk = -1;
@@ -83,7 +88,8 @@ __global__ void __launch_bounds__(256) prefill_simple_kernel(PrefillParams p) {
     const u32x4 vraw = ok ? *reinterpret_cast<const u32x4 *>(vp) : zero;
     float s = dot16<Tag>(qraw, kraw);
     for (int off = 1; off < LPT; off <<= 1) s += __shfl_xor(s, off, 64);
-    s = ok ? s * scale_log2 : -INFINITY;
+    s = cap > 0.f ? capped_log2<Tag>(s, to_cap, cap_log2) : s * scale_log2;
+    s = ok ? s : -INFINITY;
     const float mx = fmaxf(m, s);
     const float alpha = __builtin_amdgcn_exp2f(m - mx);
     const float e = __builtin_amdgcn_exp2f(s - mx);
@@ -109,7 +115,7 @@ __global__ void __launch_bounds__(256) prefill_simple_kernel(PrefillParams p) {
   for (int j = 0; j < VEC; ++j) {
     float a = acc[j] * f;
     for (int off = LPT; off < 64; off <<= 1) a += __shfl_xor(a, off, 64);
-    o[j] = ll > 0.f ? a / ll : 0.f;
+    o[j] = ll > 0.f ? a / ll * p.mask.out_scale : 0.f;
   }
   if (grp == 0) {
     T *op = (T *)p.out + (int64_t)tok * p.out_stride + h * D + sub * VEC;

@@ -21,6 +21,16 @@ struct ResidualParams {
   const void *norm_w;       // out = rms(x) * (norm_offset + norm_w); NULL: out = x rounded to dtype
   void *out;
   int64_t y_stride, out_stride, vocab;
+  // see MvResidualArgs
+  const void *y_norm_b, *norm_b, *pairs;
+  const int64_t *positions;
+  const int32_t *state_slots, *cu_q;
+  int32_t *prev_tokens;
+  const void *moe_out;
+  const int32_t *moe_rows;
+  const float *moe_w;
+  int64_t buckets, mul_prev, mul_cur, slots;
+  int n_seqs, moe_top;
   float embed_scale, norm_offset, eps, y_mult;
   int y_splits, embed_mode; // embed_mode: 0 none, 1 the row starts from the embedding, 2 the embedding is added
   int rows, cols, cols_true;
@@ -69,12 +79,68 @@ __device__ __forceinline__ float group_sum(float x, float *red) {
   return t;
 }
 
+// Row of the pair table for this row's token (uniform in the workgroup); < 0: none.  The workgroup of a sequence's first row, the
+// only one that reads the token kept from the step before, also keeps the step's last one.
+__device__ __forceinline__ int64_t pair_row(const ResidualParams &p, int row, int64_t id) {
+  int lo = row, first = row, last = row;
+  if (p.cu_q) {
+    lo = 0;
+    for (int hi = p.n_seqs; hi - lo > 1;) {
+      const int mid = (lo + hi) >> 1;
+      if (p.cu_q[mid] <= row) lo = mid;
+      else hi = mid;
+    }
+    first = p.cu_q[lo], last = p.cu_q[lo + 1] - 1;
+  }
+  const int64_t pos = p.positions[row];
+  if (pos < 0) return -1;
+  const int slot = p.state_slots[lo];
+  const bool keep = slot >= 0 && slot < p.slots;
+  int64_t prev = 0;
+  if (row > first) {
+    prev = p.ids[row - 1];
+  } else {
+    __shared__ int32_t kept;
+    if (threadIdx.x == 0) {
+      kept = pos > 0 && keep ? p.prev_tokens[(pos & 1) * p.slots + slot] : 0;
+      if (keep) p.prev_tokens[((pos + last - first + 1) & 1) * p.slots + slot] = (int32_t)p.ids[last];
+    }
+    __syncthreads();
+    prev = kept;
+  }
+  return pos == 0 ? p.buckets : (prev * p.mul_prev + id * p.mul_cur) % p.buckets;
+}
+
+// Per row z (held VEC at a time): the factors of its norm, (z - mean) * rs.  LN: mean over the true columns, else 0
+template <bool LN, int MAXV, int VEC>
+__device__ __forceinline__ float norm_factors(float (&z)[MAXV][VEC], int cols_true, float eps, float *red0, float *red1) {
+  float ss = 0.f;
+  if constexpr (LN) {
+    float sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < MAXV; ++i)
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) sum += z[i][j];
+    const float mean = group_sum(sum, red0) / (float)cols_true;
+#pragma unroll
+    for (int i = 0; i < MAXV; ++i)
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) z[i][j] = (threadIdx.x + i * blockDim.x) * VEC + j < cols_true ? z[i][j] - mean : 0.f;
+  }
+#pragma unroll
+  for (int i = 0; i < MAXV; ++i)
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) ss = fmaf(z[i][j], z[i][j], ss);
+  ss = group_sum(ss, red1);
+  return 1.0f / sqrtf(ss / (float)cols_true + eps);
+}
+
 // MAXV = vectors per thread
-template <typename Tag, int MAXV>
+template <typename Tag, int MAXV, bool LN>
 __global__ void __launch_bounds__(1024) residual_update_kernel(ResidualParams p) {
   typedef typename elem<Tag>::T T;
   constexpr int VEC = elem<Tag>::VEC;
-  __shared__ float red[2][16];
+  __shared__ float red[4][16];
   const int row = blockIdx.x, nvec = p.cols / VEC;
   float x[MAXV][VEC], y[MAXV][VEC], e[MAXV][VEC], vv[MAXV][VEC], wy[MAXV][VEC], wn[MAXV][VEC], sy[MAXV][VEC];
   bool embed_ok = false;
@@ -83,6 +149,7 @@ __global__ void __launch_bounds__(1024) residual_update_kernel(ResidualParams p)
     id = p.ids[row];
     embed_ok = id >= 0 && id < p.vocab;
   }
+  const int64_t pair = embed_ok && p.pairs ? pair_row(p, row, id) : -1;
   // every load of the row before the first reduction
 #pragma unroll
   for (int i = 0; i < MAXV; ++i) {
@@ -104,26 +171,40 @@ __global__ void __launch_bounds__(1024) residual_update_kernel(ResidualParams p)
         } else {
           load_row_vec<Tag>((const T *)p.y + (int64_t)row * p.y_stride + c, y[i]);
         }
-        if (p.y_norm_w) load_row_vec<Tag>((const T *)p.y_norm_w + c, wy[i]);
-        if (p.y_scale) load_row_vec<Tag>((const T *)p.y_scale + c, sy[i]);
       }
+      if (p.y_norm_w) load_row_vec<Tag>((const T *)p.y_norm_w + c, wy[i]);
+      if (p.y_scale) load_row_vec<Tag>((const T *)p.y_scale + c, sy[i]);
       if (embed_ok) load_row_vec<Tag>((const T *)p.embed + id * p.cols + c, e[i]);
+      if (pair >= 0) {
+        float t[VEC];
+        load_row_vec<Tag>((const T *)p.pairs + pair * p.cols + c, t);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) e[i][j] += t[j];
+      }
+      for (int k = 0; k < p.moe_top; ++k) {
+        const int from = p.moe_rows[(int64_t)row * p.moe_top + k];
+        const float mw = p.moe_w[(int64_t)row * p.moe_top + k];
+        float t[VEC];
+        if (from >= 0) load_row_vec<Tag>((const T *)p.moe_out + (int64_t)from * p.cols + c, t);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) y[i][j] = fmaf(mw, from >= 0 ? t[j] : x[i][j], y[i][j]);
+      }
       if (p.vec) load_row_vec<Tag>((const T *)p.vec + c, vv[i]);
       if (p.norm_w) load_row_vec<Tag>((const T *)p.norm_w + c, wn[i]);
     }
   }
   if (p.y_norm_w) {
-    float ss = 0.f;
+    const float rs = norm_factors<LN>(y, p.cols_true, p.eps, red[0], red[1]);
 #pragma unroll
-    for (int i = 0; i < MAXV; ++i)
+    for (int i = 0; i < MAXV; ++i) {
+      const int c = (threadIdx.x + i * blockDim.x) * VEC;
+      float b[VEC];
 #pragma unroll
-      for (int j = 0; j < VEC; ++j) ss = fmaf(y[i][j], y[i][j], ss);
-    ss = group_sum(ss, red[0]);
-    const float rs = 1.0f / sqrtf(ss / (float)p.cols_true + p.eps);
+      for (int j = 0; j < VEC; ++j) b[j] = 0.f;
+      if (LN && p.y_norm_b && c < p.cols) load_row_vec<Tag>((const T *)p.y_norm_b + c, b);
 #pragma unroll
-    for (int i = 0; i < MAXV; ++i)
-#pragma unroll
-      for (int j = 0; j < VEC; ++j) y[i][j] = y[i][j] * rs * wy[i][j];
+      for (int j = 0; j < VEC; ++j) y[i][j] = LN ? y[i][j] * rs * wy[i][j] + b[j] : y[i][j] * rs * wy[i][j];
+    }
   }
   if (p.y_scale || p.y_mult != 1.0f) {
 #pragma unroll
@@ -131,15 +212,11 @@ __global__ void __launch_bounds__(1024) residual_update_kernel(ResidualParams p)
 #pragma unroll
       for (int j = 0; j < VEC; ++j) y[i][j] = y[i][j] * sy[i][j] * p.y_mult;
   }
-  float ss = 0.f;
 #pragma unroll
   for (int i = 0; i < MAXV; ++i) {
     const int c = (threadIdx.x + i * blockDim.x) * VEC;
 #pragma unroll
-    for (int j = 0; j < VEC; ++j) {
-      x[i][j] = x[i][j] + y[i][j] + e[i][j] * p.embed_scale + vv[i][j];
-      ss = fmaf(x[i][j], x[i][j], ss);
-    }
+    for (int j = 0; j < VEC; ++j) x[i][j] = x[i][j] + y[i][j] + e[i][j] * p.embed_scale + vv[i][j];
     if (c < p.cols) {
       float *xr = p.x + (int64_t)row * p.cols + c;
 #pragma unroll
@@ -149,17 +226,20 @@ __global__ void __launch_bounds__(1024) residual_update_kernel(ResidualParams p)
   }
   if (!p.out) return;
   float rs = 1.0f;
-  if (p.norm_w) {
-    ss = group_sum(ss, red[1]);
-    rs = 1.0f / sqrtf(ss / (float)p.cols_true + p.eps);
-  }
+  if (p.norm_w) rs = norm_factors<LN>(x, p.cols_true, p.eps, red[2], red[3]);
 #pragma unroll
   for (int i = 0; i < MAXV; ++i) {
     const int c = (threadIdx.x + i * blockDim.x) * VEC;
     if (c < p.cols) {
-      float o[VEC];
+      float o[VEC], b[VEC];
 #pragma unroll
-      for (int j = 0; j < VEC; ++j) o[j] = p.norm_w ? x[i][j] * rs * (p.norm_offset + wn[i][j]) : x[i][j];
+      for (int j = 0; j < VEC; ++j) b[j] = 0.f;
+      if (LN && p.norm_b) load_row_vec<Tag>((const T *)p.norm_b + c, b);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) {
+        o[j] = p.norm_w ? x[i][j] * rs * (p.norm_offset + wn[i][j]) : x[i][j];
+        if constexpr (LN) o[j] += b[j];
+      }
       store_row_vec<Tag>((T *)p.out + (int64_t)row * p.out_stride + c, o);
     }
   }
@@ -300,12 +380,20 @@ extern "C" int mv_residual_update(const MvResidualArgs *a, int rows, int cols, i
   if (dtype != MV_BF16 && dtype != MV_F16 && dtype != MV_F32) return MV_E_DTYPE;
   if (a->embed_mode < 0 || a->embed_mode > 2) return MV_E_RANGE;
   if (a->embed_mode && (!a->embed || !a->ids || a->vocab <= 0)) return MV_E_NULLPTR;
-  if ((a->y_norm_w || a->y_scale) && !a->y) return MV_E_NULLPTR;
+  if ((a->y_norm_w || a->y_scale) && !a->y && a->moe_top == 0) return MV_E_NULLPTR;
+  if (a->moe_top < 0 || (!a->layer_norm && (a->y_norm_b || a->norm_b))) return MV_E_SHAPE;
+  if (a->moe_top && (!a->moe_out || !a->moe_rows || !a->moe_w || a->embed_mode == 1)) return MV_E_NULLPTR;
+  if (a->pairs) {
+    if (!a->embed_mode || !a->positions || !a->state_slots || (a->slots > 0 && !a->prev_tokens)) return MV_E_NULLPTR;
+    if (a->buckets <= 0 || a->mul_prev < 0 || a->mul_cur < 0 || a->slots < 0 || (a->cu_q && a->n_seqs <= 0)) return MV_E_SHAPE;
+  }
   const int vec = dtype == MV_F32 ? 4 : 8;
   if (cols % vec) return MV_E_SHAPE;
   if (!mv_aligned16(a->x) || (a->y && !mv_aligned16(a->y)) || (a->y_norm_w && !mv_aligned16(a->y_norm_w)) || (a->y_scale && !mv_aligned16(a->y_scale)) ||
       (a->embed_mode && !mv_aligned16(a->embed)) || (a->vec && !mv_aligned16(a->vec)) ||
-      (a->norm_w && !mv_aligned16(a->norm_w)) || (a->out && (!mv_aligned16(a->out) || a->out_stride % vec)) ||
+      (a->norm_w && !mv_aligned16(a->norm_w)) || (a->y_norm_b && !mv_aligned16(a->y_norm_b)) ||
+      (a->norm_b && !mv_aligned16(a->norm_b)) || (a->pairs && !mv_aligned16(a->pairs)) ||
+      (a->moe_top && !mv_aligned16(a->moe_out)) || (a->out && (!mv_aligned16(a->out) || a->out_stride % vec)) ||
       (a->y && a->y_splits == 0 && a->y_stride % vec))
     return MV_E_ALIGN;
   ResidualParams p;
@@ -313,14 +401,21 @@ extern "C" int mv_residual_update(const MvResidualArgs *a, int rows, int cols, i
   p.norm_w = a->norm_w, p.out = a->out, p.y_stride = a->y_stride, p.out_stride = a->out_stride, p.vocab = a->vocab;
   p.y_scale = a->y_scale, p.y_mult = a->y_mult;
   p.embed_scale = a->embed_scale, p.norm_offset = a->norm_offset, p.eps = a->eps;
+  p.y_norm_b = a->y_norm_b, p.norm_b = a->norm_b, p.pairs = a->pairs, p.positions = a->positions;
+  p.state_slots = a->state_slots, p.cu_q = a->cu_q, p.prev_tokens = a->prev_tokens;
+  p.moe_out = a->moe_out, p.moe_rows = a->moe_rows, p.moe_w = a->moe_w, p.moe_top = a->moe_top;
+  p.buckets = a->buckets, p.mul_prev = a->mul_prev, p.mul_cur = a->mul_cur, p.slots = a->slots, p.n_seqs = a->n_seqs;
   p.y_splits = a->y_splits, p.embed_mode = a->embed_mode, p.rows = rows, p.cols = cols, p.cols_true = cols_true;
   const int nvec = cols / vec;
   int threads = (nvec + 63) / 64 * 64;
   if (threads > 1024) threads = 1024;
   const int per = (nvec + threads - 1) / threads;
   hipStream_t st = (hipStream_t)stream;
-#define MV_RES(MV) \
-  MV_DISPATCH_DTYPE(dtype, hipLaunchKernelGGL((residual_update_kernel<Tag, MV>), dim3(rows), dim3(threads), 0, st, p))
+#define MV_RES(MV)                                                                                                              \
+  MV_DISPATCH_DTYPE(dtype, {                                                                                                    \
+    if (a->layer_norm) hipLaunchKernelGGL((residual_update_kernel<Tag, MV, true>), dim3(rows), dim3(threads), 0, st, p);       \
+    else hipLaunchKernelGGL((residual_update_kernel<Tag, MV, false>), dim3(rows), dim3(threads), 0, st, p);                    \
+  })
   if (per <= 1) MV_RES(1)
   else if (per <= 2) MV_RES(2)
   else return MV_E_SHAPE;   // > 16384 (16-bit) / 8192 (fp32) columns

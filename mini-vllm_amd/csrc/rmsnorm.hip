@@ -202,8 +202,8 @@ extern "C" int mv_add_rmsnorm_partial(const float *partial, int splits, void *re
   return MV_OK;
 }
 
-// K9 — SiluAndMul (reference: minivllm/models/layers/activation.py:70-96) and, ACT, the tanh form of gelu or the clamped gate
-// in its place (fp32 inside, one rounding).
+// K9 — SiluAndMul (reference: minivllm/models/layers/activation.py:70-96) and, ACT, the tanh form of gelu, the clamped gate or
+// relu in its place (fp32 inside, one rounding).
 // The reference rounds silu(x1) to the activation dtype before the multiply;
 // the same two rounding points are kept here.
 template <typename Tag, int ACT>
@@ -243,6 +243,8 @@ silu_and_mul_kernel(const typename elem<Tag>::T *__restrict__ x, int64_t x_strid
               y[j] = __fmul_rn(gelu_tanh(a[u][j]), b[u][j]);
             } else if constexpr (ACT == MV_ACT_CLAMPED) {
               y[j] = clamped_glu(a[u][j], b[u][j], act.limit, act.alpha);
+            } else if constexpr (ACT == MV_ACT_RELU) {
+              y[j] = __fmul_rn(fmaxf(a[u][j], 0.f), b[u][j]);
             } else {
               float s = a[u][j] / (1.0f + expf(-a[u][j]));
               s = elem<Tag>::ld(elem<Tag>::st(s));
@@ -296,6 +298,8 @@ extern "C" int mv_act_and_mul(const void *x, int64_t x_stride, void *out, int64_
   if (int e = mv_check_act(act)) return e;
   if (act->kind == MV_ACT_CLAMPED)
     return act_and_mul<MV_ACT_CLAMPED>(x, x_stride, out, out_stride, rows, cols, dtype, stream, *act);
+  if (act->kind == MV_ACT_RELU)
+    return act_and_mul<MV_ACT_RELU>(x, x_stride, out, out_stride, rows, cols, dtype, stream, *act);
   return (act->kind == MV_ACT_GELU ? act_and_mul<MV_ACT_GELU> : act_and_mul<MV_ACT_SILU>)(x, x_stride, out, out_stride, rows,
                                                                                         cols, dtype, stream, *act);
 }

@@ -19,6 +19,7 @@ struct RopeParams {
   int64_t max_pos;
   const void *q_norm_w, *k_norm_w;
   float eps;
+  int norm_dim;   // columns that the head norms are means over
   void *q_out, *k_out, *k_cache, *v_cache;
   const int32_t *slot_mapping;
   int64_t num_slots;
@@ -79,7 +80,7 @@ __global__ void __launch_bounds__(256) rope_qk_store_kernel(RopeParams p) {
 #pragma unroll
       for (int j = 0; j < VEC; ++j) ss = fmaf(x[j], x[j], ss);
       ss = lpt_sum<LPT>(ss);
-      const float rs = 1.0f / sqrtf(ss / (float)D + p.eps);
+      const float rs = 1.0f / sqrtf(ss / (float)p.norm_dim + p.eps);
       float w[VEC];
       const u32x4 wraw = *reinterpret_cast<const u32x4 *>(nw + sub * VEC);
       if constexpr (VEC == 8) unpack8<Tag>(wraw, w);
@@ -124,11 +125,11 @@ extern "C" int mv_rope_qk_store_ex(const void *q, const void *k, const void *v, 
                                 int n_heads, int n_kv_heads, int head_dim, int dtype,
                                 const MvAttnOpts *opts, void *stream) {
   if (n_tok == 0) return MV_OK;
-  if (!q || !k || !positions || !cos || !sin || !q_out) return MV_E_NULLPTR;
+  if (!q || !k || !positions || (mv_needs_tables(opts) && (!cos || !sin)) || !q_out) return MV_E_NULLPTR;
   if ((q_norm_w == nullptr) != (k_norm_w == nullptr)) return MV_E_NULLPTR;
   const bool has_cache = k_cache != nullptr || v_cache != nullptr || slot_mapping != nullptr;
   if (has_cache && (!k_cache || !v_cache || !slot_mapping || !v)) return MV_E_NULLPTR;
-  if (n_tok < 0 || n_heads <= 0 || n_kv_heads <= 0 || max_pos <= 0) return MV_E_SHAPE;
+  if (n_tok < 0 || n_heads <= 0 || n_kv_heads <= 0 || (mv_needs_tables(opts) && max_pos <= 0)) return MV_E_SHAPE;
   if (head_dim != 64 && head_dim != 128 && head_dim != 256) return MV_E_SHAPE;
   if (int e = mv_check_rot(opts, head_dim)) return e;
   if (dtype != MV_BF16 && dtype != MV_F16 && dtype != MV_F32) return MV_E_DTYPE;
@@ -150,6 +151,7 @@ extern "C" int mv_rope_qk_store_ex(const void *q, const void *k, const void *v, 
   p.slot_mapping = has_cache ? slot_mapping : nullptr;
   p.num_slots = num_slots;
   p.n_heads = n_heads; p.n_kv_heads = n_kv_heads;
+  p.norm_dim = opts && opts->norm_dim ? opts->norm_dim : head_dim;
   p.interleaved = opts && opts->interleaved;
   p.pairs = p.interleaved ? opts->rot_pairs : head_dim / 2;
   hipStream_t st = (hipStream_t)stream;

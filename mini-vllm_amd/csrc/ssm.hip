@@ -47,7 +47,9 @@ __global__ void __launch_bounds__(64) causal_conv_kernel(MvSsmArgs p) {
       if (i < TAPS - 1) input(t0 + i - (TAPS - 1), win[i + 1]);   // shifted down below
     }
   }
-  load_vec_row<Tag>((const T *)p.conv_b + c, bias);
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) bias[j] = 0.f;
+  if (p.conv_b) load_vec_row<Tag>((const T *)p.conv_b + c, bias);
   if (t0 == 0 && keep && back > 0) {   // the only workgroup that reads the old state writes the new one, behind its reads
     float last[kMaxTaps - 1][VEC];
     for (int j = 0; j < kMaxTaps - 1; ++j)
@@ -335,9 +337,9 @@ static int check_ssm(const MvSsmArgs *a, int dtype) {
 extern "C" int mv_causal_conv(const MvSsmArgs *a, int dtype, void *stream) {
   if (a && (a->n_seqs == 0 || a->max_q == 0)) return MV_OK;
   if (int e = check_ssm(a, dtype)) return e;
-  if (!a->conv_w || !a->conv_b || !a->cu_q || !a->cu_k || (a->slots > 0 && a->taps > 1 && !a->conv_state)) return MV_E_NULLPTR;
+  if (!a->conv_w || !a->cu_q || !a->cu_k || (a->slots > 0 && a->taps > 1 && !a->conv_state)) return MV_E_NULLPTR;
   if (a->max_q < 0 || a->out_stride < a->channels) return MV_E_SHAPE;
-  if (!mv_aligned16(a->conv_w) || !mv_aligned16(a->conv_b) || (a->conv_state && !mv_aligned16(a->conv_state))) return MV_E_ALIGN;
+  if (!mv_aligned16(a->conv_w) || (a->conv_b && !mv_aligned16(a->conv_b)) || (a->conv_state && !mv_aligned16(a->conv_state))) return MV_E_ALIGN;
   const int vec = dtype == MV_F32 ? 4 : 8, y = (a->max_q + kConvRows - 1) / kConvRows;
   if (y > 65535) return MV_E_SHAPE;
   const dim3 grid((a->channels / vec + 63) / 64, y, a->n_seqs);

@@ -4,13 +4,15 @@ from typing import Any
 
 from .kugulorn import KugulornForCausalLM
 from .mofarax import MofaraxForCausalLM
+from .pununex import PununexForCausalLM
 from .opt import OPTForCausalLM
 from .qwen import Qwen2ForCausalLM, Qwen3ForCausalLM
 
 SUPPORTED_MODELS = {"Qwen2ForCausalLM": Qwen2ForCausalLM, "Qwen3ForCausalLM": Qwen3ForCausalLM,
-                    "OPTForCausalLM": OPTForCausalLM, "Mofarax": MofaraxForCausalLM, "Kugulorn": KugulornForCausalLM}
+                    "OPTForCausalLM": OPTForCausalLM, "Mofarax": MofaraxForCausalLM, "Kugulorn": KugulornForCausalLM,
+                    "Pununex": PununexForCausalLM}
 TYPE_TO_ARCH = {"qwen2": "Qwen2ForCausalLM", "qwen3": "Qwen3ForCausalLM", "opt": "OPTForCausalLM",
-                "mofarax": "Mofarax", "kugulorn": "Kugulorn"}
+                "mofarax": "Mofarax", "kugulorn": "Kugulorn", "pununex": "Pununex"}
 
 
 def create_model(hf_config: Any) -> Any:

@@ -10,6 +10,7 @@ from __future__ import annotations
 import ctypes
 import os
 from ctypes import c_char_p, c_float, c_int, c_int64, c_size_t, c_uint64, c_void_p
+from typing import NamedTuple
 
 import torch
 
@@ -40,7 +41,7 @@ _SIGNATURES = {
                                  c_void_p, c_void_p, c_void_p, c_void_p, c_int64, c_int, c_int, c_int,
                                  c_int, c_int, c_void_p, c_void_p]),
     "mv_paged_decode_workspace_bytes": (c_size_t, [c_int, c_int, c_int, c_int, c_int, c_int, c_int]),
-    "mv_paged_decode_workspace_bytes_ex": (c_size_t, [c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int]),
+    "mv_paged_decode_workspace_bytes_ex": (c_size_t, [c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p]),
     "mv_paged_decode": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_void_p,
                                 c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int64, c_float,
                                 c_void_p, c_size_t, c_int, c_int, c_void_p]),
@@ -89,6 +90,15 @@ _SIGNATURES = {
     "mv_ssm_step": (c_int, [c_void_p, c_int, c_void_p]),
     "mv_gated_group_norm": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_int, c_int, c_int,
                                     c_int, c_float, c_int, c_void_p]),
+    "mv_delta_prefill_workspace_bytes": (c_size_t, [c_int] * 6),
+    "mv_delta_prefill": (c_int, [c_void_p, c_int, c_int, c_void_p]),
+    "mv_delta_step": (c_int, [c_void_p, c_int, c_void_p]),
+    "mv_head_norm_gate": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_int, c_int, c_int,
+                                  c_float, c_int, c_float, c_int, c_void_p]),
+    "mv_moe_route": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
+                             c_float, c_int, c_void_p]),
+    "mv_moe_group": (c_int, [c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p]),
+    "mv_moe_linear": (c_int, [c_void_p, c_int, c_void_p]),
     "mv_gated_act_small_m": (c_int, [c_void_p, c_int64, c_void_p, c_int, c_void_p, c_int64, c_int, c_int, c_int, c_void_p,
                                      c_int, c_int, c_void_p]),
     "mv_gated_act_mid_m": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_int, c_int, c_void_p, c_int, c_int,
@@ -156,19 +166,40 @@ class MvHipError(RuntimeError):
 
 class MvAttnOpts(ctypes.Structure):
     """Options of the ``_ex`` attention entry points (include/mvhip.h)."""
-    _fields_ = [("rot_pairs", c_int), ("interleaved", c_int), ("chunk", c_int), ("reserved", c_int), ("out_stride", c_int64)]
+    _fields_ = [("rot_pairs", c_int), ("interleaved", c_int), ("chunk", c_int), ("norm_dim", c_int), ("out_stride", c_int64),
+                ("window", c_int), ("keep_first", c_int), ("softcap", c_float), ("out_scale", c_float), ("sink", c_void_p)]
+
+
+class AttnMask(NamedTuple):
+    """What a query sees and how its scores become weights (include/mvhip.h: MvAttnOpts): a window of positions with the first
+    ``keep_first`` tokens kept, capped scores, a factor of the output, one more term per head in the softmax denominator."""
+    window: int = 0
+    keep_first: int = 0
+    softcap: float = 0.0
+    out_scale: float = 1.0
+    sink: torch.Tensor | None = None
+
+
+NO_MASK = AttnMask()
 
 
 class MvResidualArgs(ctypes.Structure):
     _fields_ = [("x", c_void_p), ("y", c_void_p), ("y_norm_w", c_void_p), ("embed", c_void_p), ("ids", c_void_p),
                 ("vec", c_void_p), ("norm_w", c_void_p), ("out", c_void_p), ("y_stride", c_int64), ("out_stride", c_int64),
                 ("vocab", c_int64), ("embed_scale", c_float), ("norm_offset", c_float), ("eps", c_float),
-                ("y_splits", c_int), ("embed_mode", c_int), ("y_mult", c_float), ("y_scale", c_void_p)]
+                ("y_splits", c_int), ("embed_mode", c_int), ("y_mult", c_float), ("y_scale", c_void_p),
+                ("y_norm_b", c_void_p), ("norm_b", c_void_p), ("pairs", c_void_p), ("positions", c_void_p),
+                ("state_slots", c_void_p), ("cu_q", c_void_p), ("prev_tokens", c_void_p), ("moe_out", c_void_p),
+                ("moe_rows", c_void_p), ("moe_w", c_void_p), ("buckets", c_int64), ("mul_prev", c_int64), ("mul_cur", c_int64),
+                ("slots", c_int64), ("layer_norm", c_int), ("n_seqs", c_int), ("moe_top", c_int), ("reserved", c_int)]
 
 
 class GateAct(ctypes.Structure):
     """Activation of a gated projection with its constants (include/mvhip.h: MvGateAct)."""
     _fields_ = [("kind", c_int), ("limit", c_float), ("alpha", c_float)]
+
+
+RELU_GLU = GateAct(3, 0.0, 0.0)     # max(gate, 0) * up
 
 
 def clamped_glu(limit: float, alpha: float = 1.702) -> GateAct:
@@ -198,11 +229,26 @@ MvSsmArgs = _struct(
     out_stride__slots=c_int64, n_seqs__max_q__channels__taps__heads__groups__p__n__b_off__c_off=c_int)
 
 
-def _attn_opts(interleaved_pairs=None, chunk: int = 0, out=None):
+MvDeltaArgs = _struct(
+    "MvDeltaArgs", x__beta__a__gate__conv_w__dt_bias__a_log__norm_w__conv_state__state__state_slots__cu_q__cu_k__context_lens__out__workspace=c_void_p,
+    x_stride__beta_stride__a_stride__gate_stride__out_stride__slots__ws_bytes=c_int64,
+    n_seqs__max_q__total_q__channels__taps__heads__groups__p__p_true__n__k_off__q_off__channel_decay__gate_kind=c_int,
+    eps__unit_eps__q_scale__out_scale=c_float)
+MvMoeLinearArgs = _struct(
+    "MvMoeLinearArgs", x__w__out__tokens__tiles__act=c_void_p, x_stride__out_stride=c_int64, max_tiles__tile_m__n__k=c_int)
+
+
+def _attn_opts(interleaved_pairs=None, chunk: int = 0, out=None, mask: AttnMask | None = None, norm_dim: int = 0, like=None):
     """``interleaved_pairs``: None = rotary halves, n = interleaved layout with n rotated pairs; ``chunk``: chunk size of
-    the causal mask (0 = whole context); ``out``: output tensor [rows, H, D] whose rows may be strided."""
-    il = interleaved_pairs is not None
-    o = MvAttnOpts(int(interleaved_pairs) if il else 0, int(il), int(chunk), 0, out.stride(0) if out is not None else 0)
+    the causal mask (0 = whole context); ``out``: output tensor [rows, H, D] whose rows may be strided; ``norm_dim``: columns that
+    the head norms are means over (0 = all); ``like``: q, whose dtype and heads the mask's sink must have."""
+    il, m = interleaved_pairs is not None, mask or NO_MASK
+    _need_cuda(m.sink)
+    if m.sink is not None and like is not None and (m.sink.dtype != like.dtype or m.sink.numel() != like.shape[1]
+                                                    or not m.sink.is_contiguous()):
+        raise MvHipError(f"sink: a number of {like.dtype} per head required")
+    o = MvAttnOpts(int(interleaved_pairs) if il else 0, int(il), int(chunk), int(norm_dim), out.stride(0) if out is not None else 0,
+                   int(m.window), int(m.keep_first), float(m.softcap), float(m.out_scale), _ptr(m.sink))
     return ctypes.byref(o)
 
 
@@ -396,14 +442,17 @@ def add_rmsnorm_partial(partial, residual, weight, eps: float):
 
 # ---------------------------------------------------------------- K7
 def _rot_tables_ok(cos, sin, d: int, interleaved_pairs) -> bool:
-    """cos / sin are dense fp32 [max_pos, rotated pairs] tables."""
+    """cos / sin are dense fp32 [max_pos, rotated pairs] tables (none if nothing is rotated)."""
+    if interleaved_pairs == 0:
+        return True
     want = d // 2 if interleaved_pairs is None else int(interleaved_pairs)
     return (cos.shape == sin.shape and cos.dim() == 2 and cos.shape[1] == want and cos.is_contiguous() and sin.is_contiguous()
             and cos.dtype == torch.float32 and sin.dtype == torch.float32)
 
 
 def rope_qk_store(q, k, v, positions, cos, sin, q_norm_w=None, k_norm_w=None, eps: float = 1e-6,
-                  k_cache=None, v_cache=None, slot_mapping=None, want_k_out: bool = True, interleaved_pairs=None):
+                  k_cache=None, v_cache=None, slot_mapping=None, want_k_out: bool = True, interleaved_pairs=None,
+                  norm_dim: int = 0):
     """q [T,H,D], k/v [T,Hkv,D] (views of the qkv GEMM output are fine).
     ``interleaved_pairs``: n = the interleaved layout on the first 2n dims (cos / sin [max_pos, n]); None = halves.
     Returns (q_rot [T,H,D], k_rot [T,Hkv,D] or None)."""
@@ -431,23 +480,24 @@ def rope_qk_store(q, k, v, positions, cos, sin, q_norm_w=None, k_norm_w=None, ep
         raise MvHipError(f"cos / sin: dense fp32 [max_pos, rotated pairs] tables required, got {tuple(cos.shape)}")
     _check(_lib.mv_rope_qk_store_ex(
         q.data_ptr(), k.data_ptr(), _ptr(v), q.stride(0), k.stride(0), v.stride(0) if v is not None else 0,
-        pos.data_ptr(), cos.data_ptr(), sin.data_ptr(), cos.shape[0], _ptr(qn), _ptr(kn), float(eps),
+        pos.data_ptr(), _ptr(cos), _ptr(sin), 0 if cos is None else cos.shape[0], _ptr(qn), _ptr(kn), float(eps),
         q_out.data_ptr(), _ptr(k_out),
         k_cache.data_ptr() if has_cache else None, v_cache.data_ptr() if has_cache else None,
         _i32(slot_mapping).data_ptr() if has_cache else None, num_slots, t, h, hkv, d, _dt(q),
-        _attn_opts(interleaved_pairs), _stream()), "mv_rope_qk_store")
+        _attn_opts(interleaved_pairs, norm_dim=norm_dim), _stream()), "mv_rope_qk_store")
     return q_out, k_out
 
 
 # ---------------------------------------------------------------- K3
 def paged_decode_workspace_bytes(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks,
-                                 flags: int | None = None, chunk: int = 0) -> int:
+                                 flags: int | None = None, chunk: int = 0, mask: AttnMask | None = None) -> int:
     return int(_lib.mv_paged_decode_workspace_bytes_ex(batch, n_heads, n_kv_heads, head_dim, block_size,
-                                                       max_blocks, DECODE_FLAGS if flags is None else flags, int(chunk)))
+                                                       max_blocks, DECODE_FLAGS if flags is None else flags,
+                                                       _attn_opts(None, chunk, mask=mask)))
 
 
 def paged_decode(q, k_cache, v_cache, block_tables, context_lens, scale: float, out=None, flags: int | None = None,
-                 chunk: int = 0):
+                 chunk: int = 0, mask: AttnMask | None = None):
     """q [B,H,D]; caches [nb,bs,Hkv,D]; block_tables int [B,nblk] (row-strided view ok);
     context_lens int [B].  ``chunk``: > 0 = only the keys of the last token's chunk of positions.  Returns [B,H,D] in
     q's dtype (``out``: a row-strided view is fine)."""
@@ -465,12 +515,12 @@ def paged_decode(q, k_cache, v_cache, block_tables, context_lens, scale: float, 
     cl = _i32(context_lens)
     max_blocks = bt.shape[1]
     flags = DECODE_FLAGS if flags is None else flags
-    ws_bytes = paged_decode_workspace_bytes(b, h, hkv, d, bs, max_blocks, flags, chunk)
+    ws_bytes = paged_decode_workspace_bytes(b, h, hkv, d, bs, max_blocks, flags, chunk, mask)
     ws = workspace(ws_bytes, q.device)
     _check(_lib.mv_paged_decode_ex(q.data_ptr(), q.stride(0), k_cache.data_ptr(), v_cache.data_ptr(),
                                 bt.data_ptr(), bt.stride(0) if max_blocks else 0, cl.data_ptr(),
                                 out.data_ptr(), b, h, hkv, d, bs, max_blocks, nb, float(scale),
-                                ws.data_ptr(), ws.numel(), _dt(q), flags, _attn_opts(None, chunk, out),
+                                ws.data_ptr(), ws.numel(), _dt(q), flags, _attn_opts(None, chunk, out, mask, like=q),
                                    _stream()), "mv_paged_decode")
     return out
 
@@ -478,7 +528,7 @@ def paged_decode(q, k_cache, v_cache, block_tables, context_lens, scale: float, 
 # ---------------------------------------------------------------- K2
 def rope_paged_decode(q, k, v, positions, cos, sin, q_norm_w, k_norm_w, eps: float, slot_mapping,
                       k_cache, v_cache, block_tables, context_lens, scale: float, flags: int | None = None,
-                      interleaved_pairs=None, chunk: int = 0, out=None):
+                      interleaved_pairs=None, chunk: int = 0, out=None, mask: AttnMask | None = None, norm_dim: int = 0):
     """Decode step of one layer in ONE launch: q [B,H,D], k/v [B,Hkv,D] RAW rows of the qkv projection (views are
     fine) -> per-head RMSNorm (weights or None) + RoPE on q and k, the new K/V rows stored at ``slot_mapping``, paged
     attention over ``block_tables`` / ``context_lens`` (which count the new token).  Returns [B,H,D], or None when
@@ -496,7 +546,7 @@ def rope_paged_decode(q, k, v, positions, cos, sin, q_norm_w, k_norm_w, eps: flo
     if bt.dim() != 2 or bt.stride(1) != 1 or bt.shape[1] == 0:
         return None
     flags = DECODE_FLAGS if flags is None else flags
-    ws_bytes = paged_decode_workspace_bytes(b, h, hkv, d, bs, bt.shape[1], flags, chunk)
+    ws_bytes = paged_decode_workspace_bytes(b, h, hkv, d, bs, bt.shape[1], flags, chunk, mask)
     ws = workspace(ws_bytes, q.device)
     if out is None:
         out = torch.empty((b, h, d), dtype=q.dtype, device=q.device)
@@ -508,10 +558,10 @@ def rope_paged_decode(q, k, v, positions, cos, sin, q_norm_w, k_norm_w, eps: flo
     kn = k_norm_w if k_norm_w is None or k_norm_w.dtype == q.dtype else k_norm_w.to(q.dtype)
     rc = _lib.mv_rope_paged_decode_ex(
         q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0), pos.data_ptr(),
-        cos.data_ptr(), sin.data_ptr(), cos.shape[0], _ptr(qn), _ptr(kn), float(eps), _i32(slot_mapping).data_ptr(),
+        _ptr(cos), _ptr(sin), 0 if cos is None else cos.shape[0], _ptr(qn), _ptr(kn), float(eps), _i32(slot_mapping).data_ptr(),
         k_cache.data_ptr(), v_cache.data_ptr(), bt.data_ptr(), bt.stride(0), cl.data_ptr(), out.data_ptr(), b, h, hkv,
         d, bs, bt.shape[1], nb, float(scale), ws.data_ptr(), ws.numel(), _dt(q), flags,
-        _attn_opts(interleaved_pairs, chunk, out), _stream())
+        _attn_opts(interleaved_pairs, chunk, out, mask, norm_dim, q), _stream())
     if rc == MV_E_SHAPE:
         return None
     _check(rc, "mv_rope_paged_decode")
@@ -520,7 +570,7 @@ def rope_paged_decode(q, k, v, positions, cos, sin, q_norm_w, k_norm_w, eps: flo
 
 def prefill_varlen(q, k, v, cu_seqlens_q, cu_seqlens_k, max_seqlen_q, max_seqlen_k, scale: float,
                    k_cache=None, v_cache=None, block_tables=None, out=None, flags: int | None = None,
-                   chunk: int = 0):
+                   chunk: int = 0, mask: AttnMask | None = None):
     """Packed causal prefill.  Contiguous K/V (k,v [Tk,Hkv,D]) unless ``block_tables`` is
     given, in which case keys come from the paged caches (prefix-cache hit).  ``chunk``: > 0 = a query sees only the
     keys of its own chunk of positions."""
@@ -550,7 +600,7 @@ def prefill_varlen(q, k, v, cu_seqlens_q, cu_seqlens_k, max_seqlen_q, max_seqlen
                                   _i32(cu_seqlens_q).data_ptr(), _i32(cu_seqlens_k).data_ptr(), n_seqs,
                                   int(max_seqlen_q), int(max_seqlen_k), h, hkv, d, bs, float(scale),
                                   _dt(q), PREFILL_FLAGS if flags is None else flags,
-                                     _attn_opts(None, chunk, out), _stream()), "mv_prefill_varlen")
+                                     _attn_opts(None, chunk, out, mask, like=q), _stream()), "mv_prefill_varlen")
     return out
 
 
@@ -633,12 +683,15 @@ def act_and_mul(x, act, out=None):
 # ---------------------------------------------------------------- K13
 def residual_update(x, y=None, y_norm_w=None, embed=None, ids=None, embed_scale: float = 1.0, start: bool = False,
                     vec=None, norm_w=None, norm_offset: float = 0.0, eps: float = 0.0, cols_true: int | None = None,
-                    out=None, want_out: bool = True, dtype=None, y_scale=None, y_mult: float = 1.0):
+                    out=None, want_out: bool = True, dtype=None, y_scale=None, y_mult: float = 1.0, y_norm_b=None, norm_b=None,
+                    layer_norm: bool = False, pairs=None, experts=None):
     """One edge of the fp32 residual stream ``x`` [rows, cols] (updated in place; include/mvhip.h: mv_residual_update).
     ``y``: [rows, cols] of the activation dtype, or fp32 K-split partial sums [splits, rows, cols]; ``y_norm_w``: its RMS
     norm; ``y_scale`` (a vector) and ``y_mult`` multiply it.  ``embed`` / ``ids``: the scaled embedding is added (``start``: the row starts from it).  ``vec``: added to every
-    row.  Returns rms(x) * (norm_offset + norm_w), or x cast to ``dtype`` when norm_w is None; None if not want_out."""
-    _need_cuda(x, y, y_norm_w, embed, ids, vec, norm_w, y_scale)
+    row.  ``layer_norm``: both norms are layer norms, with biases ``y_norm_b`` / ``norm_b``.  ``pairs`` (a ``PairTable``): a row
+    per (previous token, token) is added where the embedding is.  ``experts`` (rows [pairs, cols], place per pair, weight per pair):
+    y also gets the weighted rows of a token's choices, place < 0 standing for x itself.  Returns rms(x) * (norm_offset + norm_w), or x cast to ``dtype`` when norm_w is None; None if not want_out."""
+    _need_cuda(x, y, y_norm_w, embed, ids, vec, norm_w, y_scale, y_norm_b, norm_b)
     rows, cols = x.shape
     if x.dtype != torch.float32 or not x.is_contiguous():
         raise MvHipError("the residual stream must be a dense fp32 [rows, cols] tensor")
@@ -651,7 +704,8 @@ def residual_update(x, y=None, y_norm_w=None, embed=None, ids=None, embed_scale:
                 raise MvHipError("partial sums must be dense fp32 [splits, rows, cols]")
         elif tuple(y.shape) != (rows, cols) or y.dtype != dt or y.stride(1) != 1:
             raise MvHipError(f"y must be [{rows}, {cols}] of {dt}")
-    for name, w in (("y_norm_w", y_norm_w), ("y_scale", y_scale), ("vec", vec), ("norm_w", norm_w)):
+    for name, w in (("y_norm_w", y_norm_w), ("y_scale", y_scale), ("vec", vec), ("norm_w", norm_w), ("y_norm_b", y_norm_b),
+                    ("norm_b", norm_b)):
         if w is not None and (w.dtype != dt or w.numel() != cols or not w.is_contiguous()):
             raise MvHipError(f"{name} must be [{cols}] of {dt}")
     if embed is not None and (embed.dtype != dt or embed.shape[1] != cols or not embed.is_contiguous()
@@ -667,10 +721,47 @@ def residual_update(x, y=None, y_norm_w=None, embed=None, ids=None, embed_scale:
                        _ptr(vec), _ptr(norm_w), _ptr(out), y.stride(0) if y is not None and splits == 0 else 0,
                        out.stride(0) if out is not None else 0, embed.shape[0] if embed is not None else 0,
                        float(embed_scale), float(norm_offset), float(eps), splits,
-                       0 if embed is None else (1 if start else 2), float(y_mult), _ptr(y_scale))
+                       0 if embed is None else (1 if start else 2), float(y_mult), _ptr(y_scale), _ptr(y_norm_b), _ptr(norm_b))
+    a.layer_norm = int(layer_norm)
+    if pairs is not None:
+        _pair_args(a, pairs, rows, cols, dt)
+    if experts is not None:
+        rows_out, place, weight = experts
+        if (rows_out.dtype != dt or rows_out.shape[1] != cols or not rows_out.is_contiguous() or place.dtype != torch.int32
+                or weight.dtype != torch.float32 or place.numel() != weight.numel() or place.numel() % rows
+                or not place.is_contiguous() or not weight.is_contiguous()):
+            raise MvHipError(f"expert outputs: dense rows of {cols} {dt}, an int32 place and an fp32 weight per choice required")
+        a.moe_out, a.moe_rows, a.moe_w, a.moe_top = rows_out.data_ptr(), place.data_ptr(), weight.data_ptr(), place.numel() // rows
     _check(_lib.mv_residual_update(ctypes.byref(a), rows, cols, cols if cols_true is None else int(cols_true), _DTYPES[dt],
                                    _stream()), "mv_residual_update")
     return out
+
+
+class PairTable(NamedTuple):
+    """A table row per (previous token, token): (previous * mul_prev + token * mul_cur) mod (rows - 1), the last row for a
+    sequence's first token.  ``prev_tokens`` int32 [2, slots] keeps the token before a step's first at ``state_slots``."""
+    table: torch.Tensor
+    mul_prev: int
+    mul_cur: int
+    positions: torch.Tensor
+    prev_tokens: torch.Tensor
+    state_slots: torch.Tensor
+    cu_q: torch.Tensor | None = None     # None: one row per sequence
+
+
+def _pair_args(a, t: PairTable, rows: int, cols: int, dt) -> None:
+    n = rows if t.cu_q is None else t.cu_q.numel() - 1
+    slots = t.prev_tokens.shape[1] if t.prev_tokens.numel() else 0
+    _need_cuda(*t[:1], *t[3:])
+    if (t.table.dtype != dt or t.table.dim() != 2 or t.table.shape[1] != cols or t.table.shape[0] < 2 or not t.table.is_contiguous()
+            or t.positions.dtype != torch.int64 or t.positions.numel() != rows or not t.positions.is_contiguous()
+            or t.state_slots.dtype != torch.int32 or t.state_slots.numel() != n or not t.state_slots.is_contiguous()
+            or (slots and (t.prev_tokens.dtype != torch.int32 or t.prev_tokens.shape[0] != 2 or not t.prev_tokens.is_contiguous()))
+            or (t.cu_q is not None and t.cu_q.dtype != torch.int32)):
+        raise MvHipError(f"pair table [buckets + 1, {cols}] of {dt}, int64 positions, int32 state slots and kept tokens required")
+    a.pairs, a.buckets, a.mul_prev, a.mul_cur = t.table.data_ptr(), t.table.shape[0] - 1, int(t.mul_prev), int(t.mul_cur)
+    a.positions, a.state_slots, a.slots, a.n_seqs = t.positions.data_ptr(), t.state_slots.data_ptr(), slots, n
+    a.prev_tokens, a.cu_q = t.prev_tokens.data_ptr() if slots else None, _ptr(t.cu_q)
 
 
 def gated_lookup(s, table, offset: int, dim: int, ids, out=None):
@@ -1251,9 +1342,10 @@ def _ssm_args(shape, x, state_slots, out, conv_w=None, conv_b=None, conv_state=N
     if state_slots.dtype != torch.int32 or not state_slots.is_contiguous():
         raise MvHipError("int32 state slots required")
     if conv_w is not None:
-        if conv_w.dtype != x.dtype or conv_b.dtype != x.dtype or conv_w.shape[1] != a.channels or conv_b.numel() != a.channels:
-            raise MvHipError(f"convolution weight [taps, {a.channels}] and bias of {x.dtype} required")
-        a.conv_w, a.conv_b, a.taps = conv_w.data_ptr(), conv_b.data_ptr(), conv_w.shape[0]
+        if conv_w.dtype != x.dtype or conv_w.shape[1] != a.channels or (
+                conv_b is not None and (conv_b.dtype != x.dtype or conv_b.numel() != a.channels)):
+            raise MvHipError(f"convolution weight [taps, {a.channels}] (and bias) of {x.dtype} required")
+        a.conv_w, a.conv_b, a.taps = conv_w.data_ptr(), _ptr(conv_b), conv_w.shape[0]
     slots = 0
     if conv_state is not None and conv_state.numel():
         slots = conv_state.shape[1]
@@ -1323,4 +1415,159 @@ def gated_group_norm(y, z, w, heads: int, p: int, p_true: int, groups: int, eps:
     _check(_lib.mv_gated_group_norm(y.data_ptr(), y.stride(0), z.data_ptr(), z.stride(0), w.data_ptr(), out.data_ptr(),
                                     out.stride(0), y.shape[0], heads, p, p_true, groups, float(eps), _dt(y), _stream()),
            "mv_gated_group_norm")
+    return out
+
+
+# ---------------------------------------------------------------- K16
+MV_DELTA_SCAN = 1
+GATES = {"silu": 0, "sigmoid": 1}
+
+
+class DeltaShape(NamedTuple):
+    """Stored sizes of a gated delta rule: channels [v heads * p | k groups * n | q groups * n] at 0, k_off, q_off."""
+    heads: int
+    groups: int
+    p: int          # columns of a head (p_true of them count)
+    n: int          # key channels
+    k_off: int
+    q_off: int
+    p_true: int
+    q_scale: float
+    channel_decay: bool
+    eps: float = 1e-6
+    unit_eps: float = 1e-6
+
+    @property
+    def channels(self) -> int:
+        return self.q_off + self.groups * self.n
+
+    @property
+    def conv(self) -> tuple:
+        """The same channels as ``causal_conv`` takes them."""
+        return self.heads, self.groups, self.p, self.n, self.k_off, self.q_off
+
+
+def _delta_args(s: DeltaShape, x, beta, a, dt_bias, a_log, state, state_slots, out):
+    _need_cuda(x, beta, a, dt_bias, a_log, state, state_slots, out)
+    _rows_ok("x", x, s.channels)
+    _rows_ok("beta", beta, s.heads, x.dtype)
+    width = s.heads * (s.n if s.channel_decay else 1)
+    _rows_ok("decay", a, width, x.dtype)
+    _rows_ok("out", out, s.heads * s.p, x.dtype)
+    if dt_bias.dtype != x.dtype or dt_bias.numel() < width or a_log.dtype != x.dtype or a_log.numel() < s.heads:
+        raise MvHipError(f"decay parameters of {x.dtype}, {width} and {s.heads}, required")
+    if state_slots.dtype != torch.int32 or not state_slots.is_contiguous():
+        raise MvHipError("int32 state slots required")
+    g = MvDeltaArgs(x=x.data_ptr(), beta=beta.data_ptr(), a=a.data_ptr(), dt_bias=dt_bias.data_ptr(), a_log=a_log.data_ptr(),
+                    state_slots=state_slots.data_ptr(), out=out.data_ptr(), x_stride=x.stride(0), beta_stride=beta.stride(0),
+                    a_stride=a.stride(0), out_stride=out.stride(0), n_seqs=state_slots.numel(), total_q=x.shape[0],
+                    channels=s.channels, taps=1, heads=s.heads, groups=s.groups, p=s.p, p_true=s.p_true, n=s.n, k_off=s.k_off,
+                    q_off=s.q_off, channel_decay=int(s.channel_decay), eps=s.eps, unit_eps=s.unit_eps, q_scale=s.q_scale,
+                    out_scale=1.0)
+    if state is not None and state.numel():
+        if state.dtype != torch.float32 or tuple(state.shape[2:]) != (s.heads, s.n, s.p) or state.shape[0] != 2 or not state.is_contiguous():
+            raise MvHipError(f"recurrent state must be dense fp32 [2, slots, {s.heads}, {s.n}, {s.p}]")
+        g.state, g.slots = state.data_ptr(), state.shape[1]
+    return g
+
+
+def delta_prefill(s: DeltaShape, x, beta, a, dt_bias, a_log, state, state_slots, cu_q, cu_k, max_q: int, out=None, flags: int = 0):
+    """The gated delta rule over convolved channels [T, channels], raw beta [T, heads] and raw decays -> o [T, heads * p]."""
+    if out is None:
+        out = torch.empty((x.shape[0], s.heads * s.p), dtype=x.dtype, device=x.device)
+    g = _delta_args(s, x, beta, a, dt_bias, a_log, state, state_slots, out)
+    g.cu_q, g.cu_k, g.max_q = cu_q.data_ptr(), cu_k.data_ptr(), int(max_q)
+    n = 0 if flags & MV_DELTA_SCAN else int(_lib.mv_delta_prefill_workspace_bytes(g.n_seqs, g.total_q, s.heads, s.p, s.n, _dt(x)))
+    ws = torch.empty((n,), dtype=torch.uint8, device=x.device) if n else None
+    g.workspace, g.ws_bytes = _ptr(ws), n
+    _check(_lib.mv_delta_prefill(ctypes.byref(g), _dt(x), int(flags), _stream()), "mv_delta_prefill")
+    return out
+
+
+def delta_step(s: DeltaShape, x, beta, a, dt_bias, a_log, conv_w, conv_state, state, state_slots, context_lens, gate, norm_w,
+               gate_kind: str = "silu", out_scale: float = 1.0, out=None):
+    """One token per sequence, from projected channels [B, channels]: convolution, gated delta rule, ``head_norm_gate``."""
+    if out is None:
+        out = torch.empty((x.shape[0], s.heads * s.p), dtype=x.dtype, device=x.device)
+    g = _delta_args(s, x, beta, a, dt_bias, a_log, state, state_slots, out)
+    lens = _i32(context_lens)
+    _need_cuda(conv_w, gate, norm_w, lens)
+    _rows_ok("gate", gate, s.heads * s.p, x.dtype)
+    if lens.numel() != x.shape[0] or state_slots.numel() != x.shape[0]:
+        raise MvHipError("one length and one state slot per row required")
+    if conv_w.dtype != x.dtype or conv_w.shape[1] != s.channels or norm_w.dtype != x.dtype or norm_w.numel() < s.p:
+        raise MvHipError(f"convolution weight [taps, {s.channels}] and norm weight [{s.p}] of {x.dtype} required")
+    g.taps = conv_w.shape[0]
+    if g.slots and g.taps > 1:
+        if conv_state.dtype != x.dtype or tuple(conv_state.shape) != (2, g.slots, g.taps - 1, s.channels) or not conv_state.is_contiguous():
+            raise MvHipError(f"convolution state must be dense [2, {g.slots}, {g.taps - 1}, {s.channels}] of {x.dtype}")
+        g.conv_state = conv_state.data_ptr()
+    g.conv_w, g.norm_w, g.gate, g.gate_stride = conv_w.data_ptr(), norm_w.data_ptr(), gate.data_ptr(), gate.stride(0)
+    g.context_lens, g.gate_kind, g.out_scale = lens.data_ptr(), GATES[gate_kind], float(out_scale)
+    _check(_lib.mv_delta_step(ctypes.byref(g), _dt(x), _stream()), "mv_delta_step")
+    return out
+
+
+def head_norm_gate(y, gate, w, heads: int, p: int, p_true: int, eps: float, gate_kind: str = "silu", out_scale: float = 1.0, out=None):
+    """Per head of [T, heads * p]: rms(y) * w (shared by the heads) * act(gate) * out_scale."""
+    _need_cuda(y, gate, w)
+    _rows_ok("y", y, heads * p)
+    _rows_ok("gate", gate, heads * p, y.dtype)
+    if out is None:
+        out = torch.empty((y.shape[0], heads * p), dtype=y.dtype, device=y.device)
+    _rows_ok("out", out, heads * p, y.dtype)
+    if w.dtype != y.dtype or w.numel() < p or gate.shape[0] != y.shape[0] or out.shape[0] != y.shape[0]:
+        raise MvHipError(f"norm weight of {p} {y.dtype} and as many rows of the gate and the output required")
+    _check(_lib.mv_head_norm_gate(y.data_ptr(), y.stride(0), gate.data_ptr(), gate.stride(0), w.data_ptr(), out.data_ptr(), out.stride(0),
+                                  y.shape[0], heads, p, p_true, float(eps), GATES[gate_kind], float(out_scale), _dt(y), _stream()),
+           "mv_head_norm_gate")
+    return out
+
+
+# ---------------------------------------------------------------- K17
+def moe_route(x, w, correction, top: int, groups: int = 1, keep: int = 1, scale: float = 1.0):
+    """x [T, K], w [outputs, K] -> (ids int32 [T, top], weights fp32 [T, top])."""
+    _need_cuda(x, w, correction)
+    _rows_ok("x", x, w.shape[1])
+    if w.dtype != x.dtype or not w.is_contiguous() or correction.dtype != x.dtype or correction.numel() != w.shape[0]:
+        raise MvHipError(f"router weight [outputs, K] and correction [outputs] of {x.dtype} required")
+    ids = torch.empty((x.shape[0], top), dtype=torch.int32, device=x.device)
+    weights = torch.empty((x.shape[0], top), dtype=torch.float32, device=x.device)
+    _check(_lib.mv_moe_route(x.data_ptr(), x.stride(0), w.data_ptr(), correction.data_ptr(), ids.data_ptr(), weights.data_ptr(),
+                             x.shape[0], w.shape[1], w.shape[0], top, groups, keep, float(scale), _dt(x), _stream()), "mv_moe_route")
+    return ids, weights
+
+
+class ExpertGroups(NamedTuple):
+    place: torch.Tensor      # int32 [pairs]; -1: no product
+    tokens: torch.Tensor     # int32 [pairs], by place
+    tiles: torch.Tensor      # int32 [tiles, 3]
+    tile_m: int
+
+
+def moe_group(ids, experts: int, tile_m: int) -> ExpertGroups:
+    """(token, choice) pairs of ids [T, top] sorted by expert."""
+    _need_cuda(ids)
+    pairs, n = ids.numel(), ids.numel() // tile_m + experts
+    if ids.dtype != torch.int32 or not ids.is_contiguous():
+        raise MvHipError("dense int32 choices [T, top] required")
+    place, tokens, tiles = (torch.empty(s, dtype=torch.int32, device=ids.device) for s in ((pairs,), (pairs,), (n, 3)))
+    _check(_lib.mv_moe_group(ids.data_ptr(), pairs, ids.shape[1], experts, tile_m, n, place.data_ptr(), tokens.data_ptr(),
+                             tiles.data_ptr(), _stream()), "mv_moe_group")
+    return ExpertGroups(place, tokens, tiles, tile_m)
+
+
+def moe_linear(x, w, n: int, groups: ExpertGroups, act: GateAct | None = None, gather: bool = False, experts: int = 0):
+    """Rows by place: out[i] = W[expert of i] x[i] (``gather``: x[token of i]), W the experts' weights [experts, n, K] -- fp32: as
+    they are, 16-bit: packed per expert; ``act``: [experts, 2, n, K], out = act(gate, up)."""
+    _need_cuda(x, w)
+    pairs, k = groups.tokens.numel(), x.shape[1]
+    _rows_ok("x", x, 1, w.dtype)
+    if not w.is_contiguous() or w.numel() != experts * n * k * (2 if act is not None else 1) or (not gather and x.shape[0] < pairs):
+        raise MvHipError(f"expert weights of {experts} x {n} outputs and {k} inputs, and a row of x per place, required")
+    out = torch.empty((pairs, n), dtype=x.dtype, device=x.device)
+    a = MvMoeLinearArgs(x=x.data_ptr(), w=w.data_ptr(), out=out.data_ptr(), tokens=groups.tokens.data_ptr() if gather else None,
+                        tiles=groups.tiles.data_ptr(), act=ctypes.addressof(act) if act is not None else None, x_stride=x.stride(0),
+                        out_stride=out.stride(0), max_tiles=groups.tiles.shape[0], tile_m=groups.tile_m, n=n, k=k)
+    _check(_lib.mv_moe_linear(ctypes.byref(a), _dt(x), _stream()), "mv_moe_linear")
     return out

@@ -21,7 +21,7 @@ __all__ = ["Attention"]
 
 class Attention(nn.Module):
     def __init__(self, num_heads: int, head_dim: int, scale: float, num_kv_heads: int,
-                 use_buffered_page_attention: bool = False, chunk: int = 0) -> None:
+                 use_buffered_page_attention: bool = False, chunk: int = 0, mask: hip_ops.AttnMask | None = None) -> None:
         super().__init__()
         self.num_heads = num_heads
         self.head_dim = head_dim
@@ -29,6 +29,9 @@ class Attention(nn.Module):
         self.num_kv_heads = num_kv_heads
         # > 0: a query sees only the keys of its own chunk of ``chunk`` positions (counted from the sequence's start)
         self.chunk = int(chunk)
+        # a window that keeps the first tokens, capped scores, a factor of the output (hip_ops.AttnMask); with a sink, the number
+        # per head is a parameter of the layer that owns this module (``with_sink``)
+        self.mask = mask
         self.k_cache: torch.Tensor = torch.tensor([])
         self.v_cache: torch.Tensor = torch.tensor([])
         self._cache_initialized = False
@@ -36,6 +39,9 @@ class Attention(nn.Module):
     def extra_repr(self) -> str:
         return (f"num_heads={self.num_heads}, head_dim={self.head_dim}, num_kv_heads={self.num_kv_heads}, "
                 f"scale={self.scale}, chunk={self.chunk}, backend=mvhip")
+
+    def with_sink(self, sink) -> None:
+        self.mask = (self.mask or hip_ops.NO_MASK)._replace(sink=sink)
 
     def store_kv_cache(self, key, value, slot_mapping) -> None:
         hip_ops.store_kvcache(key, value, self.k_cache, self.v_cache, slot_mapping)
@@ -66,23 +72,23 @@ class Attention(nn.Module):
                 if out is None:
                     out = torch.empty((q.shape[0], self.num_heads, q.shape[2]), dtype=q.dtype, device=q.device)
                 hip_ops.paged_decode(q[:nd], self.k_cache, self.v_cache, ctx.block_tables[:nd], ctx.context_lens,
-                                     self.scale, out=out[:nd], chunk=self.chunk)
+                                     self.scale, out=out[:nd], chunk=self.chunk, mask=self.mask)
                 if q.shape[0] > nd:
                     hip_ops.prefill_varlen(q[nd:], None, None, ctx.rest_cum_seqlens_q, ctx.rest_cum_seqlens_k,
                                            ctx.rest_max_seqlen_q, ctx.rest_max_seqlen_k, self.scale,
                                            k_cache=self.k_cache, v_cache=self.v_cache,
-                                           block_tables=ctx.block_tables[nd:], out=out[nd:], chunk=self.chunk)
+                                           block_tables=ctx.block_tables[nd:], out=out[nd:], chunk=self.chunk, mask=self.mask)
                 return out
             if ctx.prefix_cached and has_cache and ctx.block_tables is not None:
                 # prefix-cache hit: the queries are the uncached suffix, the keys live in the cache
                 return hip_ops.prefill_varlen(q, None, None, ctx.cum_seqlens_q, ctx.cum_seqlens_k,
                                               ctx.max_seqlen_q, ctx.max_seqlen_k, self.scale,
                                               k_cache=self.k_cache, v_cache=self.v_cache,
-                                              block_tables=ctx.block_tables, out=out, chunk=self.chunk)
+                                              block_tables=ctx.block_tables, out=out, chunk=self.chunk, mask=self.mask)
             return hip_ops.prefill_varlen(q, k, v, ctx.cum_seqlens_q, ctx.cum_seqlens_k,
-                                          ctx.max_seqlen_q, ctx.max_seqlen_k, self.scale, out=out, chunk=self.chunk)
+                                          ctx.max_seqlen_q, ctx.max_seqlen_k, self.scale, out=out, chunk=self.chunk, mask=self.mask)
         if ctx.context_lens is None or ctx.block_tables is None:
             raise RuntimeError("Context lengths or block tables not set for decode phase. "
                                "This is a bug in the inference pipeline.")
         return hip_ops.paged_decode(q, self.k_cache, self.v_cache, ctx.block_tables, ctx.context_lens,
-                                    self.scale, out=out, chunk=self.chunk)
+                                    self.scale, out=out, chunk=self.chunk, mask=self.mask)

@@ -28,7 +28,7 @@ from ..parallel_state import (divide, get_tensor_parallel_rank, get_tensor_paral
 from ..utils.loader import materialize
 
 __all__ = ["LinearBase", "ReplicatedLinear", "ColumnParallelLinear", "MergedColumnParallelLinear",
-           "QKVParallelLinear", "RowParallelLinear", "SegmentedLinear", "Segment", "gated_linear", "pad_to", "divide", "linear", "small_m", "PartialSum", "mid_plan",
+           "QKVParallelLinear", "RowParallelLinear", "SegmentedLinear", "Segment", "BlockLinear", "gated_linear", "pad_to", "divide", "linear", "small_m", "PartialSum", "mid_plan",
            "tuned_plan", "mid_m"]
 
 # rows up to which the weight-streaming kernel beats the library GEMM (tools/bench_linear.py); 0 disables
@@ -377,3 +377,27 @@ class SegmentedLinear(LinearBase):
         kind = "row" if partial_ok and self.split == "in" and self.shards == 1 else "col"
         y = linear(x, self.weight, None, self.weight_packed, kind)
         return tp_all_reduce(y) if self.split == "in" and self.shards > 1 else y
+
+
+class BlockLinear(LinearBase):
+    """Several projections with inputs AND outputs of their own as one product: blocks on the diagonal of one weight, zeros elsewhere.
+    Block i reads its ``pad_to(inputs)`` columns behind those of the blocks before it; its outputs are the segment's.  One rank."""
+
+    def __init__(self, blocks: list[tuple[int, Segment]]) -> None:
+        self.blocks, self.offsets, n, k = {}, {}, 0, 0
+        for inputs, g in blocks:
+            self.blocks[g.name], self.offsets[g.name] = (inputs, k, g), n
+            n, k = n + g.local(1), k + pad_to(inputs)
+        super().__init__(k, n)
+        self.weight.data.zero_()
+
+    def weight_loader(self, param, loaded_weight, loaded_shard_id: str | None = None, *args, **kwargs):
+        inputs, k, g = self.blocks[loaded_shard_id]
+        if tuple(loaded_weight.shape) != (g.units * g.unit, inputs):
+            raise ValueError(f"block {g.name!r}: expected {(g.units * g.unit, inputs)}, got {tuple(loaded_weight.shape)}")
+        stored, at = g.stored or g.unit, self.offsets[g.name]
+        dst = param.data[at:at + g.units * stored, k:k + inputs].unflatten(0, (g.units, stored))
+        dst[:, :g.unit].copy_(materialize(loaded_weight).unflatten(0, (g.units, g.unit)))
+
+    def forward(self, x):
+        return linear(x, self.weight, None, self.weight_packed)

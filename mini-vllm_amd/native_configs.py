@@ -4,11 +4,13 @@ from __future__ import annotations
 
 import json
 import math
-from dataclasses import dataclass
+import struct
+from dataclasses import dataclass, replace
 from pathlib import Path
 
 __all__ = ["AttentionSpec", "LayerSpec", "MofaraxConfig", "LatentAttentionSpec", "Mamba2Spec", "ClampedMlpSpec", "MixerLayerSpec",
-           "KugulornConfig", "NATIVE_CONFIGS", "load_native_config"]
+           "KugulornConfig", "DeltaRuleSpec", "SinkAttentionSpec", "ParallelMixerSpec", "ReluMlpSpec", "MoeSpec", "DeltaLayerSpec",
+           "PununexConfig", "NATIVE_CONFIGS", "checkpoint_shapes", "load_native_config"]
 
 
 def _need(d: dict, key: str, where: str):
@@ -20,6 +22,12 @@ def _need(d: dict, key: str, where: str):
 def _size(v, what: str) -> int:
     if isinstance(v, bool) or not isinstance(v, int) or v <= 0:
         raise ValueError(f"{what} must be a positive integer, got {v!r}")
+    return v
+
+
+def _count(v, what: str) -> int:
+    if isinstance(v, bool) or not isinstance(v, int) or v < 0:
+        raise ValueError(f"{what} must be a non-negative integer, got {v!r}")
     return v
 
 
@@ -300,7 +308,226 @@ class KugulornConfig:
         return out
 
 
-NATIVE_CONFIGS = {"Mofarax": MofaraxConfig, "Kugulorn": KugulornConfig}
+@dataclass(frozen=True)
+class SinkAttentionSpec:
+    """Grouped-head attention without positions: normed queries and keys, a window that keeps the first tokens, capped scores, a
+    sink per head in the softmax denominator."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    softcap: float      # 0: none
+    window: int         # 0: every key up to the query
+    keep_first: int
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str) -> "SinkAttentionSpec":
+        s = {k: _size(_need(m, k, where), f"{where}.{k}") for k in ("heads", "kv_heads", "dim", "vdim")}
+        if s["heads"] % s["kv_heads"]:
+            raise ValueError(f"{where}: {s['heads']} query heads do not divide over {s['kv_heads']} key/value heads")
+        scale, cap = _real(_need(m, "scale", where), f"{where}.scale"), m.get("softcap")
+        cap = 0.0 if cap is None else _real(cap, f"{where}.softcap")
+        if scale <= 0 or cap < 0:
+            raise ValueError(f"{where}: scale must be positive and softcap not negative, got {scale} and {cap}")
+        mask = m.get("mask") or {}
+        window = _size(mask["size"], f"{where}.mask.size") if mask.get("size") is not None else 0
+        return cls(**s, scale=scale, softcap=cap, window=window,
+                   keep_first=_count(mask.get("keep_first") or 0, f"{where}.mask.keep_first"))
+
+    def weight_shapes(self, width: int) -> dict[str, tuple[int, ...]]:
+        return {"q": (self.heads * self.dim, width), "k": (self.kv_heads * self.dim, width), "v": (self.kv_heads * self.vdim, width),
+                "q.norm": (self.dim,), "k.norm": (self.dim,), "sink": (self.heads,), "o": (width, self.heads * self.vdim)}
+
+
+@dataclass(frozen=True)
+class DeltaRuleSpec:
+    """Gated delta rule; see layers/delta_rule.py.  ``channel_decay``: a decay per key channel and a sigmoid gate, each through a
+    projection of low rank; else a decay per head and a silu gate."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    taps: int           # of the causal convolutions
+    channel_decay: bool = False
+    decay_rank: int = 0  # of the low-rank projections; a checkpoint's tensors give them (0: not known yet)
+    gate_rank: int = 0
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str, channel_decay: bool = False) -> "DeltaRuleSpec":
+        s = {k: _size(_need(m, k, where), f"{where}.{k}") for k in ("heads", "kv_heads", "dim", "vdim", "conv")}
+        s["taps"] = s.pop("conv")
+        if s["heads"] % s["kv_heads"]:
+            raise ValueError(f"{where}: {s['heads']} heads do not divide over {s['kv_heads']} key heads")
+        rank = _count(m.get("rank") or 0, f"{where}.rank")
+        return cls(**s, channel_decay=channel_decay, decay_rank=rank, gate_rank=rank)
+
+    def weight_shapes(self, width: int) -> dict[str, tuple[int, ...]]:
+        h, k, v = self.heads, self.kv_heads * self.dim, self.heads * self.vdim
+        out = {"q": (k, width), "k": (k, width), "v": (v, width), "q.conv": (k, self.taps), "k.conv": (k, self.taps),
+               "v.conv": (v, self.taps), "b": (h, width), "A_log": (h,), "norm": (self.vdim,), "o": (width, v)}
+        if self.channel_decay:
+            if not self.decay_rank or not self.gate_rank:
+                raise ValueError("the ranks of the decay's and the gate's projections are not known: they come from the "
+                                 "checkpoint's tensors a1 and g1 (or 'rank' in the configuration)")
+            out.update(a1=(self.decay_rank, width), a2=(h * self.dim, self.decay_rank), dt_bias=(h * self.dim,),
+                       g1=(self.gate_rank, width), g2=(v, self.gate_rank))
+        else:
+            out.update(a=(h, width), dt_bias=(h,), g=(v, width))
+        return out
+
+
+@dataclass(frozen=True)
+class ParallelMixerSpec:
+    """Attention and a gated delta rule side by side on the same input, summed with a scale each."""
+    left: SinkAttentionSpec
+    right: DeltaRuleSpec
+    left_scale: float
+    right_scale: float
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str) -> "ParallelMixerSpec":
+        return cls(SinkAttentionSpec.from_dict(_need(m, "left", where), f"{where}.left"),
+                   DeltaRuleSpec.from_dict(_need(m, "right", where), f"{where}.right", channel_decay=True),
+                   _real(m.get("left_scale", 1.0), f"{where}.left_scale"), _real(m.get("right_scale", 1.0), f"{where}.right_scale"))
+
+    def weight_shapes(self, width: int) -> dict[str, tuple[int, ...]]:
+        return {f"{side}.{k}": s for side in ("left", "right") for k, s in getattr(self, side).weight_shapes(width).items()}
+
+
+@dataclass(frozen=True)
+class ReluMlpSpec:
+    ff: int
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str) -> "ReluMlpSpec":
+        return cls(_size(_need(m, "ff", where), f"{where}.ff"))
+
+    def weight_shapes(self, width: int) -> dict[str, tuple[int, ...]]:
+        return {"gate": (self.ff, width), "up": (self.ff, width), "down": (width, self.ff)}
+
+
+@dataclass(frozen=True)
+class MoeSpec:
+    """Experts behind a router with groups, a correction of the choice and identity experts; see layers/moe.py."""
+    experts: int
+    identity: int       # router outputs behind the experts whose output is the input itself
+    top: int
+    groups: int
+    keep: int           # groups that a token chooses from
+    scale: float
+    ff: int
+    shared_ff: int      # 0: no shared expert
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str) -> "MoeSpec":
+        r, at = _need(m, "router", where), f"{where}.router"
+        experts, top = _size(_need(r, "experts", at), f"{at}.experts"), _size(_need(r, "top", at), f"{at}.top")
+        identity, groups = _count(r.get("identity") or 0, f"{at}.identity"), r.get("groups") or {}
+        count, keep = _size(groups.get("count", 1), f"{at}.groups.count"), _size(groups.get("keep", 1), f"{at}.groups.keep")
+        outputs = experts + identity
+        if outputs % count or keep > count or top > outputs // count * keep:
+            raise ValueError(f"{at}: {outputs} outputs in {count} groups, of which {keep} count, cannot give {top} choices")
+        shared, ff = m.get("shared"), _need(_need(m, "expert", where), "ff", f"{where}.expert")
+        return cls(experts, identity, top, count, keep, _real(r.get("scale", 1.0), f"{at}.scale"), _size(ff, f"{where}.expert.ff"),
+                   _size(_need(shared, "ff", f"{where}.shared"), f"{where}.shared.ff") if shared else 0)
+
+    def weight_shapes(self, width: int) -> dict[str, tuple[int, ...]]:
+        n = self.experts + self.identity
+        out: dict[str, tuple[int, ...]] = {"router": (n, width), "correction": (n,)}
+        for name, ff in [(f"e{i}", self.ff) for i in range(self.experts)] + ([("shared", self.shared_ff)] if self.shared_ff else []):
+            out[name + ".gate"] = out[name + ".up"] = (ff, width)
+            out[name + ".down"] = (width, ff)
+        return out
+
+
+@dataclass(frozen=True)
+class DeltaLayerSpec:
+    """A mixer of one of several kinds and an optional feed-forward of one of several kinds."""
+    type: str
+    mixer: DeltaRuleSpec | ParallelMixerSpec
+    mlp: ReluMlpSpec | MoeSpec | None
+    MIXERS = {"delta": DeltaRuleSpec, "parallel": ParallelMixerSpec}
+    MLPS = {"dense": ReluMlpSpec, "moe": MoeSpec}
+
+    @classmethod
+    def from_dict(cls, d: dict, where: str) -> "DeltaLayerSpec":
+        kind, mlp = _need(d, "type", where), d.get("mlp")
+        if kind not in cls.MIXERS:
+            raise ValueError(f"{where}: unsupported layer type {kind!r}; known: {sorted(cls.MIXERS)}")
+        if mlp is not None and _need(mlp, "kind", f"{where}.mlp") not in cls.MLPS:
+            raise ValueError(f"{where}.mlp: unsupported feed-forward {mlp['kind']!r}; known: {sorted(cls.MLPS)}")
+        return cls(kind, cls.MIXERS[kind].from_dict(_need(d, "mixer", where), f"{where}.mixer"),
+                   None if mlp is None else cls.MLPS[mlp["kind"]].from_dict(mlp, f"{where}.mlp"))
+
+
+class PununexConfig:
+    """Gated delta rule layers, some beside windowed attention, dense or expert feed-forwards, and a table of token pairs."""
+    model_type = "pununex"
+    recurrent_state = True     # the token before, and the delta rules' states
+
+    def __init__(self, raw: dict) -> None:
+        self.architectures = ["Pununex"]
+        self.vocab_size = _size(_need(raw, "vocab", "config"), "vocab")
+        self.hidden_size = _size(_need(raw, "width", "config"), "width")
+        self.norm_eps = _real(_need(_need(raw, "norm", "config"), "eps", "norm"), "norm.eps")
+        pairs = (raw.get("embedding") or {}).get("bigram")
+        self.pair_buckets, self.pair_muls = 0, (0, 0)
+        if pairs:
+            at = "embedding.bigram"
+            self.pair_buckets = _size(_need(pairs, "buckets", at), f"{at}.buckets")
+            self.pair_muls = tuple(_count(_need(pairs, k, at), f"{at}.{k}") for k in ("mul_prev", "mul_cur"))
+        layers = _need(raw, "layers", "config")
+        if not isinstance(layers, list) or not layers:
+            raise ValueError("config: 'layers' must be a non-empty list")
+        self.layers = [DeltaLayerSpec.from_dict(d, f"layers[{i}]") for i, d in enumerate(layers)]
+        # what the engine asks of any configuration
+        attention = [s.mixer.left for s in self.layers if s.type == "parallel"]
+        self.num_hidden_layers = len(self.layers)
+        self.num_attention_heads = max([a.heads for a in attention], default=1)
+        self.num_key_value_heads = max([a.kv_heads for a in attention], default=1)
+        self.head_dim = max([max(a.dim, a.vdim) for a in attention], default=1)
+        self.intermediate_size = max((s.mlp.ff for s in self.layers if s.mlp), default=0)
+        self.max_position_embeddings: int | None = None    # none of its own; the engine's Config fills it in
+        self.torch_dtype = raw.get("dtype", "bfloat16")
+        self.eos_token_id = None
+        self.tie_word_embeddings = False
+
+    def take_shapes(self, shapes: dict[str, tuple[int, ...]]) -> None:
+        """Sizes that only a checkpoint's tensors give: the ranks of the low-rank projections."""
+        for i, s in enumerate(self.layers):
+            a1, g1 = (shapes.get(f"l{i}.mix.right.{k}") for k in ("a1", "g1"))
+            if s.type == "parallel" and a1 and g1:
+                self.layers[i] = replace(s, mixer=replace(s.mixer, right=replace(s.mixer.right, decay_rank=a1[0], gate_rank=g1[0])))
+
+    def weight_shapes(self) -> dict[str, tuple[int, ...]]:
+        """Name -> shape of every tensor of a checkpoint."""
+        v, d = self.vocab_size, self.hidden_size
+        out: dict[str, tuple[int, ...]] = {"embed": (v, d), "final.norm": (d,), "final.norm.b": (d,), "head": (v, d)}
+        if self.pair_buckets:
+            out["bigram"] = (self.pair_buckets + 1, d)
+        for i, s in enumerate(self.layers):
+            p = f"l{i}."
+            out.update({f"{p}mix.{k}": v for k, v in s.mixer.weight_shapes(d).items()})
+            out[p + "norm1"] = out[p + "norm1.b"] = out[p + "ls1"] = (d,)
+            if s.mlp:
+                out[p + "norm2"] = out[p + "norm2.b"] = out[p + "ls2"] = (d,)
+                out.update({f"{p}mlp.{k}": v for k, v in s.mlp.weight_shapes(d).items()})
+        return out
+
+
+NATIVE_CONFIGS = {"Mofarax": MofaraxConfig, "Kugulorn": KugulornConfig, "Pununex": PununexConfig}
+
+
+def checkpoint_shapes(model_dir) -> dict[str, tuple[int, ...]]:
+    """Tensor name -> shape of a directory's safetensors files, from their headers (an 8-byte length, then JSON)."""
+    out: dict[str, tuple[int, ...]] = {}
+    for path in sorted(Path(model_dir).glob("*.safetensors")):
+        with open(path, "rb") as f:
+            (n,) = struct.unpack("<Q", f.read(8))
+            header = json.loads(f.read(n))
+        out.update({k: tuple(v["shape"]) for k, v in header.items() if k != "__metadata__"})
+    return out
 
 
 def load_native_config(model_dir: str):
@@ -314,4 +541,7 @@ def load_native_config(model_dir: str):
         return None
     if name not in NATIVE_CONFIGS:
         raise ValueError(f"unsupported architecture {name!r} in {path}; known: {sorted(NATIVE_CONFIGS)}")
-    return NATIVE_CONFIGS[name](raw)
+    config = NATIVE_CONFIGS[name](raw)
+    if hasattr(config, "take_shapes"):
+        config.take_shapes(checkpoint_shapes(model_dir))
+    return config

@@ -39,7 +39,7 @@ def _facts(body):
 
 def test_pipe_prefill_kernels_keep_scalar_loads_out_of_the_counted_lds_reads(asm):
     pipe = {n: b for n, b in asm.items() if re.search(r"prefill_mfma_kernelI\w+?Li[48]ELb1E", n)}
-    assert len(pipe) == 16, sorted(asm)                      # bf16 / f16 x 4 / 8 waves x head dim 64 / 128 x whole / chunked
+    assert len(pipe) == 24, sorted(asm)                      # bf16 / f16 x 4 / 8 waves x head dim 64 / 128 x whole / chunked / windowed
     for name, body in pipe.items():
         lines = body.split("\n")
         # the counted waits are the hand-written ones: inside ;;#ASMSTART ... ;;#ASMEND blocks
