@@ -116,11 +116,34 @@ def _kugulorn(like: str, q_rank: int, ssm_heads: int, groups: int, pairs: int, w
                 head_dim=kv_rank + rot, intermediate_size=c["intermediate_size"])
 
 
+def _pununex(like: str, peer: str, pairs: int, window: int = 2048, experts: int = 32, rank: int = 128) -> dict:
+    """A Pununex configuration of ``pairs`` x [gated delta rule with a dense feed-forward, attention beside a gated delta rule with
+    experts], with ``like``'s width, heads and feed-forward: a token's experts (4, and a shared one) have its size together.  As many
+    pairs as make the weights that a token uses ``like``'s; ``peer``: the model it is compared with."""
+    c = MODELS[like]
+    heads, kv, width, ff = (c[k] for k in ("num_attention_heads", "num_key_value_heads", "hidden_size", "intermediate_size"))
+    delta = {"heads": heads, "kv_heads": heads // 2, "dim": 128, "vdim": 128, "conv": 4}
+    left = {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 30.0,
+            "mask": {"size": window, "keep_first": 4}}
+    right = {"heads": heads // 2, "kv_heads": heads // 2, "dim": 128, "vdim": 128, "conv": 4, "rank": rank}
+    moe = {"kind": "moe", "router": {"experts": experts, "identity": 2, "top": 4, "scale": 2.0,
+                                     "groups": {"count": 2, "keep": 1}}, "expert": {"ff": ff // 8}, "shared": {"ff": ff // 2}}
+    layers = [{"type": "delta", "mixer": delta, "mlp": {"kind": "dense", "ff": ff}},
+              {"type": "parallel", "mixer": {"left": left, "right": right, "left_scale": 0.7, "right_scale": 0.7}, "mlp": moe}] * pairs
+    return dict(architecture="Pununex", vocab=c["vocab_size"], width=width, norm={"eps": 1e-6}, layers=layers, like=peer, window=window,
+                embedding={"bigram": {"buckets": 65521, "mul_prev": 31, "mul_cur": 17}}, vocab_size=c["vocab_size"], hidden_size=width,
+                num_attention_heads=heads, num_key_value_heads=kv, head_dim=128, intermediate_size=ff)
+
+
 DESIGNS = {"mofarax": {"mofarax-0.6b": "qwen3-0.6b", "mofarax-1.7b": "qwen3-1.7b", "mofarax-7b": "qwen2-7b"},
-           "kugulorn": {"kugulorn-0.6b": "qwen3-0.6b", "kugulorn-1.7b": "qwen3-1.7b", "kugulorn-7b": "qwen2-7b"}}
+           "kugulorn": {"kugulorn-0.6b": "qwen3-0.6b", "kugulorn-1.7b": "qwen3-1.7b", "kugulorn-7b": "qwen2-7b"},
+           # (beside the design that also mixes attention with a recurrence)
+           "pununex": {"pununex-0.6b": "kugulorn-0.6b", "pununex-1.7b": "kugulorn-1.7b", "pununex-7b": "kugulorn-7b"}}
 MODELS.update({name: _mofarax(like) for name, like in DESIGNS["mofarax"].items()})
 MODELS.update({"kugulorn-0.6b": _kugulorn("qwen3-0.6b", 512, 32, 1, 19), "kugulorn-1.7b": _kugulorn("qwen3-1.7b", 768, 64, 1, 19),
                "kugulorn-7b": _kugulorn("qwen2-7b", 1536, 112, 2, 21)})
+MODELS.update({f"pununex-{s}": _pununex(like, f"kugulorn-{s}", n) for s, like, n in
+               (("0.6b", "qwen3-0.6b", 12), ("1.7b", "qwen3-1.7b", 13), ("7b", "qwen2-7b", 13))})
 DESIGN_DECODE = ((256, 1024), (16, 1024), (1, 1024))      # (batch, context) of a design's decode records
 DESIGN_PREFILL = ((16, 1024), (4, 4096))
 HBM_PEAK_GBS = 8000.0  # MI355X_MICROARCH.md: HBM3E 8.0 TB/s spec (6.29 TB/s measured copy ceiling)
@@ -540,11 +563,15 @@ def step_roofline(engine, model, batch, ctx_mid, ms_per_step):
         if hasattr(mod, "input_size") or type(mod).__name__ == "ParallelLMHead":
             seen.add(w.data_ptr())
             wbytes += w.numel() * w.element_size() * passes.get(id(mod), 1)
+    for mod in expert_modules(ex):        # (each choice a different expert, as far as there are enough of them)
+        wbytes += int(sum(p.numel() * p.element_size() for p in (mod.gate_up, mod.down)) * min(1.0, batch * mod.top / mod.experts))
     if ex.latents or ex.state_modules:    # cached rows seen by each attention layer; state read and written once
         kv = sum(batch * min(ctx_mid, m.window or ctx_mid) * m.row_cols * ex.dtype.itemsize for m in ex.model.modules()
                  if hasattr(m, "row_cols"))
-        kv += sum(2 * batch * t.numel() // (2 * t.shape[1]) * t.element_size() for m in ex.state_modules
-                  for t in (m.conv_state, m.ssm_state))
+        kv += sum(batch * min(ctx_mid, m.mask.window or ctx_mid) * 2 * m.num_kv_heads * m.head_dim * ex.dtype.itemsize
+                  for m in ex.model.modules() if hasattr(m, "k_cache"))
+        kv += sum(2 * batch * t.numel() // (2 * t.shape[1]) * t.element_size() for m in recurrent_modules(ex)
+                  for t in (m.conv_state, m.ssm_state if hasattr(m, "ssm_state") else m.state))
     else:
         L, nb, bs, hkv, d = ex.kv_cache.shape[1:]
         kv = L * batch * ctx_mid * 2 * hkv * d * ex.dtype.itemsize
@@ -552,6 +579,14 @@ def step_roofline(engine, model, batch, ctx_mid, ms_per_step):
     return {"bound": "hbm", "weight_bytes_per_gpu": wbytes, "kv_bytes_per_step_per_gpu": int(kv),
             "bytes_per_step_per_gpu": int(wbytes + kv), "achieved": round(gbs, 1), "peak": HBM_PEAK_GBS, "unit": "GB/s",
             "frac": round(gbs / HBM_PEAK_GBS, 4), "mean_context": ctx_mid}
+
+
+def recurrent_modules(ex) -> list:
+    return [m for m in ex.state_modules if hasattr(m, "conv_state")]
+
+
+def expert_modules(ex) -> list:
+    return [m for m in ex.model.modules() if type(m).__name__ == "ExpertMLP"]
 
 
 def release_all(engine):
@@ -570,9 +605,11 @@ def release_all(engine):
     torch.cuda.synchronize()
 
 
-def prefill_flops(heads: int, head_dim: int, lens, chunk: int = 0) -> int:
+def prefill_flops(heads: int, head_dim: int, lens, chunk: int = 0, window: int = 0) -> int:
     """Causal flash prefill without a cached prefix, one layer (K2): sum over sequences of
-    4 H D (Sq Sk - Sq (Sq - 1) / 2) with Sq = Sk = len; a chunk mask cuts a sequence into pieces of ``chunk`` tokens."""
+    4 H D (Sq Sk - Sq (Sq - 1) / 2) with Sq = Sk = len; a chunk mask cuts a sequence into pieces of ``chunk`` tokens; a window counts its pairs."""
+    if window:
+        return 4 * heads * head_dim * sum(min(i + 1, window) for n in lens for i in range(n))
     if chunk:
         lens = [m for n in lens for m in [chunk] * (n // chunk) + [n % chunk]]
     return sum(4 * heads * head_dim * (n * n - n * (n - 1) // 2) for n in lens)
@@ -615,10 +652,11 @@ def prefill_records(engine, model, gpus=1, cases=PREFILL_CASES, reps=5):
             for s in seqs:
                 bm.allocate(s)
             probing = rep == reps + 1
-            real, real_ssm = getattr(hip_ops, entry), hip_ops.ssm_prefill
+            entries = {entry: "prefill", "ssm_prefill": "ssm", "delta_prefill": "delta", "moe_linear": "experts"}
+            reals = {e: getattr(hip_ops, e) for e in entries}
             if probing:
-                setattr(attn_mod.hip_ops, entry, probe.wrap("prefill", real))
-                attn_mod.hip_ops.ssm_prefill = probe.wrap("ssm", real_ssm)
+                for e, key in entries.items():
+                    setattr(attn_mod.hip_ops, e, probe.wrap(key, reals[e]))
             try:
                 torch.cuda.synchronize()
                 t0 = time.perf_counter()
@@ -626,8 +664,8 @@ def prefill_records(engine, model, gpus=1, cases=PREFILL_CASES, reps=5):
                 torch.cuda.synchronize()
                 dt = time.perf_counter() - t0
             finally:
-                setattr(attn_mod.hip_ops, entry, real)
-                attn_mod.hip_ops.ssm_prefill = real_ssm
+                for e, real in reals.items():
+                    setattr(attn_mod.hip_ops, e, real)
             for s in seqs:
                 bm.deallocate(s)
             if rep and not probing:
@@ -642,7 +680,7 @@ def prefill_records(engine, model, gpus=1, cases=PREFILL_CASES, reps=5):
             seen = n * sum(min(i + 1, m0.window or ln) for i in range(ln))
             flops = seen * m0.heads * 2 * (m0.dq + m0.dv)
         else:
-            flops = prefill_flops(heads, head_dim, [ln] * n, cfgm.get("chunk", 0))
+            flops = prefill_flops(heads, head_dim, [ln] * n, cfgm.get("chunk", 0), cfgm.get("window", 0))
         tf = flops / us / 1e6
         out.append({"metric": "prefill tokens/s", "model": model, "tp": gpus, "prompts": n, "prompt_len": ln,
                     "batches_timed": reps, "warmup_batches": 1, "ms_per_batch": round(med * 1e3, 3),
@@ -655,13 +693,40 @@ def prefill_records(engine, model, gpus=1, cases=PREFILL_CASES, reps=5):
                                  "share_of_step": round(us * len(t_us) / (med * 1e6), 4),
                                  "mfma_busy": busy, "mfma_busy_source": busy_src,
                                  "timing": f"HIP event pairs around every mv_{entry} launch of one extra (untimed) batch, on the launching stream"}})
-        if ex.state_modules:
+        if recurrent_modules(ex) and hasattr(recurrent_modules(ex)[0], "state"):
+            out[-1].update(_delta_and_expert_prefill(ex, n * ln, probe))
+        elif ex.state_modules:
             m0, t_ssm = ex.state_modules[0], sorted(probe.times_us("ssm"))
             us = t_ssm[len(t_ssm) // 2]
             byt = n * ln * (2 * m0.heads * m0.p + 2 * m0.groups * m0.n + m0.heads) * ex.dtype.itemsize
             out[-1]["ssm_roofline"] = {"bound": "hbm", "kernel": "ssm_chunk_kernel", "bytes_per_launch": byt, "us_per_launch": round(us, 2),
                                        "achieved": round(byt / us / 1e3, 1), "peak": HBM_PEAK_GBS, "unit": "GB/s",
                                        "frac": round(byt / us / 1e3 / HBM_PEAK_GBS, 4)}
+    return out
+
+
+def _delta_and_expert_prefill(ex, tokens: int, probe) -> dict:
+    """Rooflines of mv_delta_prefill (bytes of its inputs and outputs, the layers of each kind apart) and of the two expert products."""
+    out, mods = {}, recurrent_modules(ex)
+    t = probe.times_us("delta")
+    for key, kind in (("ssm_roofline", False), ("channel_decay_roofline", True)):
+        mine = [(m, us) for m, us in zip(mods, t) if m.shape.channel_decay == kind]
+        if mine:
+            s, us = mine[0][0].shape, statistics.median(u for _, u in mine)
+            byt = tokens * (2 * s.heads * s.p + 2 * s.groups * s.n + s.heads * (1 + (s.n if kind else 1))) * ex.dtype.itemsize
+            out[key] = {"bound": "hbm", "kernel": "delta_prepare_kernel + delta_walk_kernel", "bytes_per_launch": byt,
+                        "us_per_launch": round(us, 2), "achieved": round(byt / us / 1e3, 1), "peak": HBM_PEAK_GBS, "unit": "GB/s",
+                        "frac": round(byt / us / 1e3 / HBM_PEAK_GBS, 4)}
+    experts, t = expert_modules(ex), probe.times_us("experts")
+    if experts:
+        m0 = experts[0]
+        pairs = tokens * m0.top * m0.experts / m0.router.shape[0]      # (identity experts have no product)
+        for key, us, n in (("gate_up", t[0::2], 2), ("down", t[1::2], 1)):
+            us, flops = statistics.median(us), 2 * pairs * n * m0.f * m0.w
+            out[f"expert_{key}_roofline"] = {"bound": "mfma", "kernel": "moe_tile_kernel", "flops_per_launch": int(flops),
+                                             "us_per_launch": round(us, 2), "achieved": round(flops / us / 1e6, 1),
+                                             "peak": MFMA_PEAK_TFLOPS, "unit": "TFLOP/s",
+                                             "frac": round(flops / us / 1e6 / MFMA_PEAK_TFLOPS, 4)}
     return out
 
 
@@ -993,13 +1058,16 @@ def attention_graph_roofline(engine, model) -> tuple:
 
     def run():
         for m in mods:
-            hip_ops.paged_decode(q, m.k_cache, m.v_cache, tables, lens, m.scale, chunk=m.chunk)
+            hip_ops.paged_decode(q, m.k_cache, m.v_cache, tables, lens, m.scale, chunk=m.chunk, mask=m.mask)
     us = _graph_time_us(run, len(mods))
     seen = [n - (n - 1) // m0.chunk * m0.chunk if m0.chunk else n for n in lens.tolist()]
+    if m0.mask and m0.mask.window:
+        seen = [min(n, m0.mask.window + m0.mask.keep_first) for n in seen]
     algo = (sum(seen) * 2 * m0.num_kv_heads * m0.head_dim + 2 * q.numel()) * ex.dtype.itemsize
     return {"bound": "hbm", "achieved": round(algo / us / 1e3, 1), "peak": HBM_PEAK_GBS, "unit": "GB/s",
             "frac": round(algo / us / 1e3 / HBM_PEAK_GBS, 4), "bytes_per_launch": algo, "us_per_launch": round(us, 2),
-            "timing": f"{len(mods)} launches (split-KV combine included) captured into a hipGraph, median of 5 replays / launches"}, None
+            "timing": f"{len(mods)} launches (split-KV combine included) captured into a hipGraph, median of 5 replays / launches"}, (
+                _delta_graph_roofline(ex, lens, slots) if recurrent_modules(ex) else None)
 
 
 def _graph_roofline(byt: int, us: float, launches: int) -> dict:
@@ -1042,6 +1110,56 @@ def _state_graph_roofline(ex, lens, slots) -> dict:
     return _graph_roofline(byt, us, len(mods))
 
 
+def _delta_graph_roofline(ex, lens, slots) -> dict:
+    """mv_delta_step of the layers with a decay per head on the running batch (a step that is run again gives the same state)."""
+    from minivllm_amd import hip_ops
+
+    mods, b = [m for m in recurrent_modules(ex) if not m.shape.channel_decay], lens.numel()
+    m0, s = mods[0], mods[0].shape
+    z = torch.randn((b, m0.columns), device=ex.device).to(ex.dtype)
+    at, cols = m0.at, s.heads * s.p
+
+    def run():
+        for m in mods:
+            hip_ops.delta_step(s, z[:, :s.channels], z[:, at["b"]:at["b"] + s.heads], z[:, at["a"]:at["a"] + s.heads], m.dt_bias, m.A_log,
+                               m.conv, m.conv_state, m.state, slots, lens, z[:, at["g"]:at["g"] + cols], m.norm, m.gate)
+    us = _graph_time_us(run, len(mods))
+    byt = 2 * b * (m0.state[0, 0].numel() * 4 + m0.conv_state[0, 0].numel() * ex.dtype.itemsize)
+    return _graph_roofline(byt + b * (s.channels + 2 * s.heads + 2 * cols) * ex.dtype.itemsize, us, len(mods))
+
+
+def expert_graph_rooflines(engine, batch: int) -> dict | None:
+    """Routing and the two expert products of every layer with experts, on random rows: weight bytes of the experts that were chosen."""
+    from minivllm_amd import hip_ops
+
+    ex = engine.model_runner.inference_executor
+    mods = expert_modules(ex)
+    if not mods:
+        return None
+    out, m0 = {}, mods[0]
+    h = torch.randn((batch, m0.w), device=ex.device).to(ex.dtype)
+    ids = [hip_ops.moe_route(h, m.router, m.correction, m.top, m.groups, m.keep, m.scale)[0] for m in mods]
+    used = statistics.mean(len({e for e in i.flatten().tolist() if e < m0.experts}) for i in ids)
+    groups = [hip_ops.moe_group(i, m.experts, m.tile_rows(batch)) for i, m in zip(ids, mods)]
+    zs = [torch.randn((batch * m.top, m.f), device=ex.device).to(ex.dtype) for m in mods]
+
+    def gate_up():
+        for m, g in zip(mods, groups):
+            hip_ops.moe_linear(h, m.gate_up, m.f, g, m.act, gather=True, experts=m.experts)
+
+    def down():
+        for m, g, z in zip(mods, groups, zs):
+            hip_ops.moe_linear(z, m.down, m.w, g, experts=m.experts)
+
+    def route():
+        for m in mods:
+            hip_ops.moe_group(hip_ops.moe_route(h, m.router, m.correction, m.top, m.groups, m.keep, m.scale)[0], m.experts, m.tile_rows(batch))
+    for name, run, n in (("gate_up", gate_up, 2), ("down", down, 1)):
+        out[name] = _graph_roofline(int(used * n * m0.f * m0.w * ex.dtype.itemsize), _graph_time_us(run, len(mods)), len(mods))
+    out["route_and_group_us"] = round(_graph_time_us(route, len(mods)), 2)
+    return out
+
+
 def design_records(args, workdir) -> dict:
     """``--design``: for every size of the design and for its peer, decode at several batches and prefill, on one engine each."""
     import gc
@@ -1062,6 +1180,9 @@ def design_records(args, workdir) -> dict:
                 rec["roofline"], state = attention_graph_roofline(engine, model)
                 if state is not None:
                     rec["state_roofline"] = state
+                experts = expert_graph_rooflines(engine, batch)
+                if experts is not None:
+                    rec["expert_rooflines"] = experts
                 rec["step_roofline"] = step_roofline(engine, model, batch, ctx + a.warmup + a.steps // 2, rec["ms_per_step"])
                 recs.append(rec)
                 release_all(engine)

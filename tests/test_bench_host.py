@@ -157,6 +157,22 @@ def test_design_configurations_have_the_layer_sizes_of_their_peers():
         h, kv = p["num_attention_heads"], p["num_key_value_heads"]
         layer = d * dim * (2 * h + 2 * kv) + 3 * d * p["intermediate_size"]
         assert abs(count(c.weight_shapes()) / (layer * p["num_hidden_layers"]) - 1) < 0.05, name
+    # layers of unlike kinds and experts: the weights that a token uses are those of the model the sizes are taken from (within 10 %)
+    for name, peer in bench.DESIGNS["pununex"].items():
+        c, p = NATIVE_CONFIGS["Pununex"](bench.MODELS[name]), bench.MODELS[bench.MODELS[peer]["like"]]
+        assert (c.vocab_size, c.hidden_size, c.num_attention_heads) == (p["vocab_size"], p["hidden_size"], p["num_attention_heads"])
+        used = 0
+        for s in c.layers:
+            if hasattr(s.mlp, "experts"):
+                assert s.mlp.top * s.mlp.ff + s.mlp.shared_ff == p["intermediate_size"]
+            else:
+                assert s.mlp.ff == p["intermediate_size"]
+            used += 3 * c.hidden_size * p["intermediate_size"]
+            used += sum(a[0] * a[1] for k, a in s.mixer.weight_shapes(c.hidden_size).items() if len(a) == 2)
+        d, dim = p["hidden_size"], p.get("head_dim") or p["hidden_size"] // p["num_attention_heads"]
+        layer = d * dim * 2 * (p["num_attention_heads"] + p["num_key_value_heads"]) + 3 * d * p["intermediate_size"]
+        assert abs(used / (layer * p["num_hidden_layers"]) - 1) < 0.1, name
+    assert bench.prefill_flops(2, 64, [100], 0, 30) == 4 * 2 * 64 * (sum(range(1, 31)) + 70 * 30)
     args = bench.parse(["--design", "mofarax"])
     assert args.design == "mofarax" and bench.parse([]).design is None and bench.parse([]).model == "qwen3-1.7b"
     # a chunk mask cuts the work of a prompt into the chunks' triangles
