@@ -734,7 +734,7 @@ int mv_moe_route(const void *x, int64_t x_stride, const void *w, const void *cor
 int mv_moe_group(const int32_t *ids, int pairs, int top, int experts, int tile_m, int max_tiles, int32_t *rows, int32_t *tokens,
                  int32_t *tiles, void *stream);
 /* out[place] = W[expert] x[tokens[place]] (tokens NULL: x[place]), W [experts][n][k]; act: W [experts][2][n][k], out = act(gate, up).
- * 16-bit: W packed per expert (mv_pack_weight of all rows), tile_m 16, 32, 64 or 128; fp32: W as it is, tile_m 16.  n % 16 == 0,
+ * 16-bit: W packed per expert (mv_pack_weight of all rows), tile_m 16, 32, 64, 128 or 256; fp32: W as it is, tile_m 16.  n % 16 == 0,
  * k % 64 == 0. */
 typedef struct MvMoeLinearArgs {
   const void *x, *w;

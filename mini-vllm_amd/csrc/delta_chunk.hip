@@ -5,9 +5,9 @@
 //     u_i = beta_i (v_i - (e^{r_i} k_i) S - sum_{j < i} A_ij u_j),    A_ij = sum_c k_ic k_jc e^{r_ic - r_jc}
 //     o_i = (e^{r_i} q_i) S + sum_{j <= i} B_ij u_j,                  B_ij = sum_c q_ic k_jc e^{r_ic - r_jc}
 //     S  <- e^{r_last} S + sum_j (e^{r_last - r_j} k_j)^T u_j
-// The u of a chunk solve a unit lower triangular system, so U = U0 - W S with (U0, W) its solutions for the right-hand sides
-// beta v and beta e^r k.  Two launches:
-//   prepare: everything that does not need S, one workgroup per (chunk, head): A, B, the solutions, the scaled operands;
+// The u of a chunk solve a unit lower triangular system: with T = (1 + A)^-1 diag(beta), U = U0 - W S, U0 = T v, W = T e^r k.
+// Two launches:
+//   prepare: everything that does not need S, one workgroup per (chunk, head): A, B, T, U0, W, the scaled operands;
 //   walk:    chunks one behind the other, one workgroup per (sequence, head, columns): four products with S and U.
 // What is fp32 by nature enters a product as the sum of two bf16 numbers (three MFMAs: high x high, high x rest, rest x high), about
 // 16 bits of mantissa.  The operands lie in the workspace as MFMA fragments (64 lanes x 16 bytes), which the walk fetches by LDS-DMA.
@@ -68,12 +68,12 @@ __global__ void __launch_bounds__(256, 2) delta_prepare_kernel(DeltaPrep q) {
   constexpr int N = NK * 32, RS = N + 4, KS = N + 8;   // LDS row strides: fp32, 16-bit
   const MvDeltaArgs &p = q.a;
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  float *rs = (float *)smem;                              // [L][RS] running log2 decays; later the solutions W
-  T *ks = (T *)(smem + L * RS * 4), *qs = ks + L * KS;    // [L][KS]; later (from qs on) the system's matrix
+  float *rs = (float *)smem;                              // [L][RS] running log2 decays
+  T *ks = (T *)(smem + L * RS * 4), *qs = ks + L * KS;    // [L][KS]; later (from qs on) -A, then T
   constexpr int TS = L + 4;
   float *ts = (float *)qs;                                // [L][TS]
   constexpr int QB = L * KS * 2 > L * TS * 4 ? L * KS * 2 : L * TS * 4;
-  float *fk = (float *)((char *)qs + QB), *fq = fk + L, *bt = fq + L;
+  float *fk = (float *)((char *)qs + QB), *fq = fk + L, *bt = fq + L, *part_sums = bt + L;   // [4][64]
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), r16 = lane & 15, g = lane >> 4;
   const int head = blockIdx.y;
   // chunk slot -> sequence (its slots start at cu_q / L + its number) and chunk
@@ -133,13 +133,26 @@ __global__ void __launch_bounds__(256, 2) delta_prepare_kernel(DeltaPrep q) {
       for (int c = tid & 3; c < N; c += 4) rs[t * RS + c] = v;
     }
     __syncthreads();
-    for (int c = tid; c < N; c += 256) {
-      float sum = 0.f;
+    // a thread a quarter of a channel's tokens (the threads of a wave: adjacent channels); then the quarters ahead are added
+    for (int c0 = 0; c0 < N; c0 += 64) {
+      const int c = c0 + lane;
+      float v[16], sum = 0.f;
+      if (c < N) {
 #pragma unroll
-      for (int t = 0; t < L; ++t) {
-        sum += rs[t * RS + c];
-        rs[t * RS + c] = sum;
+        for (int t = 0; t < 16; ++t) v[t] = rs[(16 * wave + t) * RS + c];
+#pragma unroll
+        for (int t = 0; t < 16; ++t) sum += v[t], v[t] = sum;
+        part_sums[wave * 64 + lane] = sum;
       }
+      __syncthreads();
+      if (c < N) {
+        float ahead = 0.f;
+#pragma unroll
+        for (int w = 0; w < 3; ++w) ahead += w < wave ? part_sums[w * 64 + lane] : 0.f;
+#pragma unroll
+        for (int t = 0; t < 16; ++t) rs[(16 * wave + t) * RS + c] = ahead + v[t];
+      }
+      if (c0 + 64 < N) __syncthreads();
     }
   }
   __syncthreads();
@@ -196,10 +209,10 @@ __global__ void __launch_bounds__(256, 2) delta_prepare_kernel(DeltaPrep q) {
     }
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
-      A[e] = j0 + e < i ? A[e] * (bt[i] * fk[i] * fk[j0 + e]) : 0.f;
+      A[e] = j0 + e < i ? -A[e] * (bt[i] * fk[i] * fk[j0 + e]) : 0.f;
       B[e] = j0 + e <= i ? B[e] * (fq[i] * fk[j0 + e]) : 0.f;
     }
-    blk[m] = A;
+    blk[m] = A;   // (the negative)
     // B as an operand whose k order is that of an accumulator pair: key 16 (e >> 2) + 4 g + (e & 3) of a step of 32
     const u32x2 hi = pack_quad<B16>(B);
     f32x4 rest;
@@ -227,20 +240,6 @@ __global__ void __launch_bounds__(256, 2) delta_prepare_kernel(DeltaPrep q) {
     u32x4 *dst = (u32x4 *)(ws + (8 * NK + f * 2) * 1024) + lane;
     dst[0] = hi, dst[64] = lo;
   }
-  for (int f = wave; f < 4 * NK; f += 4) {
-    const int i = f >> 1, s = f & 1, c = (i >> 1) * 32 + (r16 >> 2) * 8 + (i & 1) * 4 + (r16 & 3);
-    const float last = rs[(L - 1) * RS + c];
-    float v[8];
-    u32x4 hi, lo;
-#pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      const int t = 32 * s + 16 * (e >> 2) + 4 * g + (e & 3);
-      v[e] = elem<Tag>::ld(ks[t * KS + c]) * fk[t] * __builtin_amdgcn_exp2f(last - rs[t * RS + c]);
-    }
-    split8(v, hi, lo);
-    u32x4 *dst = (u32x4 *)(ws + (lay.k + f * 2) * 1024) + lane;
-    dst[0] = hi, dst[64] = lo;
-  }
   for (int c = tid; c < N; c += 256) ((float *)(ws + lay.tail * 1024))[c] = __builtin_amdgcn_exp2f(rs[(L - 1) * RS + c]);
   __syncthreads();   // q is done with
 #pragma unroll
@@ -252,54 +251,139 @@ __global__ void __launch_bounds__(256, 2) delta_prepare_kernel(DeltaPrep q) {
   }
   __syncthreads();
 
-  // ---- the triangular system: a thread a column of [beta e^r k | beta v]
-  for (int col0 = 0; col0 < N + p.p; col0 += 256) {
-    const int col = col0 + tid;
-    float sol[L];
-    if (col < N) {
+  // ---- T = (1 + A)^-1 diag(beta).  Its entries are at most 1, since no factor 1 - beta k k^T of the recurrence lengthens a vector.
+  // A wave inverts a diagonal block, a column in each of 16 lanes ..
+  {
+    float *d = ts + 16 * wave * TS + 16 * wave, x[16];
 #pragma unroll
-      for (int i = 0; i < L; ++i) sol[i] = bt[i] * fk[i] * __builtin_amdgcn_exp2f(rs[i * RS + col]) * elem<Tag>::ld(ks[i * KS + col]);
-    } else {
-      const T *v = x + head * p.p + min(col - N, p.p - 1);
-#pragma unroll
-      for (int i = 0; i < L; ++i) sol[i] = elem<Tag>::ld(v[(int64_t)min(i, nt - 1) * p.x_stride]);
-#pragma unroll
-      for (int i = 0; i < L; ++i) sol[i] *= bt[i];   // (0 behind the end)
-    }
-#pragma unroll
-    for (int i = 1; i < L; ++i) {
-      float a = sol[i], b = 0.f;
+    for (int i = 0; i < 16; ++i) {
+      float a = i == r16 ? 1.f : 0.f, b = 0.f;
 #pragma unroll
       for (int j = 0; j < i; j += 4) {   // (zeros from column i on)
-        const f32x4 t = *(const f32x4 *)(ts + i * TS + j);
-        a = fmaf(-t[0], sol[j], a);
-        b = fmaf(-t[1], sol[j + 1], b);
-        a = fmaf(-t[2], sol[j + 2], a);
-        b = fmaf(-t[3], sol[j + 3], b);
+        const f32x4 t = *(const f32x4 *)(d + i * TS + j);
+        a = fmaf(t[0], x[j], a);
+        if (j + 1 < i) b = fmaf(t[1], x[j + 1], b);
+        if (j + 2 < i) a = fmaf(t[2], x[j + 2], a);
+        if (j + 3 < i) b = fmaf(t[3], x[j + 3], b);
       }
-      sol[i] = a + b;
+      x[i] = a + b;
     }
-    if (col >= N && col < N + p.p) {   // U0 in the layout of an accumulator: column lane & 15, tokens 4 (lane >> 4) ..
-      const int c = col - N;
-      f32x4 *dst = (f32x4 *)(ws + (lay.u0 + (c >> 4) * 4) * 1024) + (c & 15);
+    if (lane < 16) {
 #pragma unroll
-      for (int i = 0; i < L; i += 4) dst[(i >> 4) * 64 + ((i >> 2) & 3) * 16] = f32x4{sol[i], sol[i + 1], sol[i + 2], sol[i + 3]};
+      for (int i = 0; i < 16; ++i) d[i * TS + r16] = x[i];
     }
-    if (col0 == 0) {   // -W, by rows (N <= 256)
-      __syncthreads();
-      if (col < N) {
+  }
+  __syncthreads();
+  // .. and then a wave a column of blocks, from the diagonal down: T_IJ = T_II sum_{J <= K < I} (-A_IK) T_KJ.  Accumulators are the
+  // right operand of the next product, whose keys are 4 g + step.
+  {
+    auto product = [&](int I, int K, const f32x4 &right, f32x4 acc) {
+      const f32x4 left = *(const f32x4 *)(ts + (16 * I + r16) * TS + 16 * K + 4 * g);
 #pragma unroll
-        for (int i = 0; i < L; ++i) rs[i * RS + col] = -sol[i];
+      for (int e = 0; e < 4; ++e) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(left[e], right[e], acc, 0, 0, 0);
+      return acc;
+    };
+    f32x4 t[4];
+#pragma unroll
+    for (int I = 0; I < 4; ++I) {
+      t[I] = f32x4{0.f, 0.f, 0.f, 0.f};
+      if (I < wave) continue;
+      if (I == wave) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) t[I][e] = ts[(16 * I + 4 * g + e) * TS + 16 * wave + r16];
+        continue;
       }
-      __syncthreads();
-      for (int f = wave; f < 4 * NK; f += 4) {
-        const int it = f / NK, s = f - it * NK;
-        const float *w = rs + (16 * it + r16) * RS + 32 * s + 8 * g;
+      f32x4 sum = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int K = 0; K < I; ++K)
+        if (K >= wave) sum = product(I, K, t[K], sum);
+      t[I] = product(I, I, sum, t[I]);
+    }
+    const float beta = bt[16 * wave + r16];
+    __syncthreads();   // every wave has read A
+#pragma unroll
+    for (int I = 0; I < 4; ++I)
+      if (I >= wave) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) ts[(16 * I + 4 * g + e) * TS + 16 * wave + r16] = t[I][e] * beta;
+      }
+  }
+  __syncthreads();
+  // T by rows as operands, either side: (token tile, step of 32 tokens) 0 0, 1 0, 2 0, 2 1, 3 0, 3 1; tokens 16 (e >> 2) + 4 g + (e & 3)
+  u32x4 th[6], tl[6];
+#pragma unroll
+  for (int m = 0; m < 6; ++m) {
+    const int it = m < 2 ? m : 2 + (m - 2) / 2, s = m < 2 ? 0 : m & 1;
+    const float *row = ts + (16 * it + r16) * TS + 32 * s + 4 * g;
+    f32x4 a = *(const f32x4 *)row, b = {0.f, 0.f, 0.f, 0.f};
+    if (2 * s + 1 <= it) b = *(const f32x4 *)(row + 16);
+    split44(a, b, th[m], tl[m]);
+  }
+  auto of = [](int it, int s) constexpr { return it < 2 ? it : 2 * it - 2 + s; };
+
+  // ---- by 32 channels: K = e^(r_last - r) k by state rows, in the order of the walk's accumulators, and -W = -T e^r k by tokens;
+  // by 16 columns of v: U0 = T v
+  for (int item = wave; item < NK + p.p / 16; item += 4) {
+    if (item < NK) {
+      f32x4 acc[2][4];
+#pragma unroll
+      for (int d = 0; d < 2; ++d) {
+        const int i = 2 * item + d, c = item * 32 + (r16 >> 2) * 8 + d * 4 + (r16 & 3);
+        const float last = rs[(L - 1) * RS + c];
+#pragma unroll
+        for (int it = 0; it < 4; ++it) acc[d][it] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int s = 0; s < 2; ++s) {
+          float v[8], w[8];
+          u32x4 hi, lo;
+#pragma unroll
+          for (int e = 0; e < 8; ++e) {
+            const int t = 32 * s + 16 * (e >> 2) + 4 * g + (e & 3);
+            const float k = elem<Tag>::ld(ks[t * KS + c]) * fk[t], r = rs[t * RS + c];
+            v[e] = k * __builtin_amdgcn_exp2f(last - r);
+            w[e] = k * __builtin_amdgcn_exp2f(r);
+          }
+          split8(v, hi, lo);
+          u32x4 *dst = (u32x4 *)(ws + (lay.k + (i * 2 + s) * 2) * 1024) + lane;
+          dst[0] = hi, dst[64] = lo;
+          split8(w, hi, lo);
+#pragma unroll
+          for (int it = 2 * s; it < 4; ++it) acc[d][it] = mfma3(hi, lo, th[of(it, s)], tl[of(it, s)], acc[d][it]);
+        }
+      }
+#pragma unroll
+      for (int it = 0; it < 4; ++it) {
         u32x4 hi, lo;
-        split44(*(const f32x4 *)w, *(const f32x4 *)(w + 4), hi, lo);
-        u32x4 *dst = (u32x4 *)(ws + f * 2 * 1024) + lane;
+        split44(-acc[0][it], -acc[1][it], hi, lo);
+        u32x4 *dst = (u32x4 *)(ws + (it * NK + item) * 2 * 1024) + lane;
         dst[0] = hi, dst[64] = lo;
       }
+    } else {
+      const int ct = item - NK;
+      const T *v = x + head * p.p + ct * 16 + r16;
+      T raw[16];
+#pragma unroll
+      for (int e = 0; e < 16; ++e) raw[e] = v[(int64_t)min(16 * (e >> 2) + 4 * g + (e & 3), nt - 1) * p.x_stride];
+      f32x4 acc[4];
+#pragma unroll
+      for (int it = 0; it < 4; ++it) acc[it] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int s = 0; s < 2; ++s) {
+        float f[8];
+        u32x4 hi, lo;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) f[e] = elem<Tag>::ld(raw[8 * s + e]);
+        split8(f, hi, lo);
+#pragma unroll
+        for (int it = 2 * s; it < 4; ++it) {
+          acc[it] = mfma16x16x32<B16>(th[of(it, s)], hi, acc[it]);
+          acc[it] = mfma16x16x32<B16>(tl[of(it, s)], hi, acc[it]);
+          if constexpr (!__is_same(Tag, B16)) acc[it] = mfma16x16x32<B16>(th[of(it, s)], lo, acc[it]);
+        }
+      }
+      // in the layout of an accumulator: column lane & 15, tokens 4 (lane >> 4) ..
+#pragma unroll
+      for (int it = 0; it < 4; ++it) *((f32x4 *)(ws + (lay.u0 + ct * 4 + it) * 1024) + lane) = acc[it];
     }
   }
 }
@@ -508,7 +592,7 @@ int launch(const DeltaPrep &q, hipStream_t stream) {
   constexpr int QB = L * KS * 2 > L * (L + 4) * 4 ? L * KS * 2 : L * (L + 4) * 4;
   if (int rc = mv_allow_lds<delta_prepare_kernel<Tag, NK>>()) return rc;
   hipLaunchKernelGGL((delta_prepare_kernel<Tag, NK>), dim3((unsigned)chunk_slots(a.n_seqs, a.total_q), a.heads), dim3(256),
-                     L * RS * 4 + L * KS * 2 + QB + 3 * L * 4, stream, q);
+                     L * RS * 4 + L * KS * 2 + QB + 7 * L * 4, stream, q);
   MV_LAUNCH_CHECK();
   // two column tiles a wave share every operand read, where that still leaves a workgroup per CU
   const int tiles = a.p / 16, wide = (tiles + 7) / 8;

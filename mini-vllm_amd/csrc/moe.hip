@@ -249,8 +249,13 @@ __global__ void __launch_bounds__(256) moe_small_kernel(MoeLinear p) {
   }
 }
 
+// A fragment of 16 rows x 32 inputs that LDS-DMA brings: four adjacent lanes fetch one row's 64 bytes (16 rows in adjacent lanes would be
+// 16 cache lines), in an order that spreads the rows' like pieces over the banks.
+__device__ __forceinline__ int row_chunk(int lane) { return (lane & 3) ^ ((lane >> 4) & 3); }              // the piece that a lane fetches
+__device__ __forceinline__ int row_place(int row, int chunk) { return row * 4 + (chunk ^ ((row >> 2) & 3)); }  // where a piece lies
+
 // many rows: BM x BN per workgroup of 2 x 2 waves, 64 inputs at a time.  Rows and weights reach LDS by DMA as fragments (16 rows x
-// 32 inputs, 1 KiB, in the order of the lanes), so every LDS read is linear; the next 64 inputs land while these are multiplied.
+// 32 inputs, 1 KiB; weights in the order of the lanes); the next 64 inputs land while these are multiplied.
 template <typename Tag, int BM, int BN, bool GATED>
 __global__ void __launch_bounds__(256, 2) moe_tile_kernel(MoeLinear p) {
   typedef typename elem<Tag>::T T;
@@ -269,8 +274,8 @@ __global__ void __launch_bounds__(256, 2) moe_tile_kernel(MoeLinear p) {
   for (int i = 0; i < PER; ++i) {
     const int piece = i * 4 + wave, half = piece & 1, t = piece >> 1;
     if (t < MT) {
-      const int place = m0 + min(t * 16 + r16, live - 1);
-      src[i] = (const T *)p.x + (int64_t)(p.tokens ? p.tokens[place] : place) * p.x_stride + half * 32 + g * 8;
+      const int place = m0 + min(t * 16 + (lane >> 2), live - 1);
+      src[i] = (const T *)p.x + (int64_t)(p.tokens ? p.tokens[place] : place) * p.x_stride + half * 32 + row_chunk(lane) * 8;
       step[i] = 64;
     } else {
       const int j = t - MT, wt = min(nt0 + (GATED ? j >> 1 : j), ntiles - 1) + (GATED && (j & 1) ? ntiles : 0);
@@ -287,14 +292,14 @@ __global__ void __launch_bounds__(256, 2) moe_tile_kernel(MoeLinear p) {
     }
   };
   f32x4 acc[WN][WM] = {};
-  const uint32_t base = lds_address(smem) + lane * 16;
+  const uint32_t base = lds_address(smem) + lane * 16, rows = lds_address(smem) + row_place(r16, g) * 16;
   const int trips = p.k / 64;
   fetch(0);
   asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");
   lds_barrier();
   for (int t = 0; t < trips; ++t) {
     if (t + 1 < trips) fetch((t + 1) & 1);
-    const uint32_t at = base + (t & 1) * STAGE, xa = at + wm * WM * 2048, wa = at + (MT + wn * WN) * 2048;
+    const uint32_t at = (t & 1) * STAGE, xa = rows + at + wm * WM * 2048, wa = base + at + (MT + wn * WN) * 2048;
     u32x4 a[2][WN], b[2][WM];
     static_for<2>([&](auto H) {
       constexpr int h = decltype(H)::value;
@@ -312,6 +317,95 @@ __global__ void __launch_bounds__(256, 2) moe_tile_kernel(MoeLinear p) {
     });
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     lds_barrier();
+  }
+#pragma unroll
+  for (int i = 0; i < WM; ++i) {
+    const int row = (wm * WM + i) * 16 + r16;
+    if (row >= live) continue;
+    T *out = (T *)p.out + (int64_t)(m0 + row) * p.out_stride + g * 4;
+#pragma unroll
+    for (int j = 0; j < (GATED ? WN / 2 : WN); ++j) {
+      const int nt = nt0 + (GATED ? wn * (WN / 2) + j : wn * WN + j);
+      if (nt >= ntiles) continue;
+      f32x4 o;
+      if constexpr (GATED) {
+#pragma unroll
+        for (int q = 0; q < 4; ++q) o[q] = gated_act<Tag>(acc[2 * j][i][q], acc[2 * j + 1][i][q], p.act);
+      } else {
+        o = acc[j][i];
+      }
+      *(u32x2 *)(out + nt * 16) = pack_quad<Tag>(o);
+    }
+  }
+}
+
+// very many rows: 256 x 256 per workgroup of 2 x 4 waves, so that a row operand read from LDS serves four products and a weight operand
+// eight.  Two stages of 64 inputs; a stage is handed back half way through its products, when all of it is in registers.
+template <typename Tag, bool GATED>
+__global__ void __launch_bounds__(512, 1) moe_wide_kernel(MoeLinear p, int nx, int max_tiles) {
+  typedef typename elem<Tag>::T T;
+  constexpr int TILES = 16, WM = 8, WN = 4, PER = 4, STAGE = 4 * TILES * 1024;
+  extern __shared__ __attribute__((aligned(16))) char smem[];   // 2 stages of [rows: TILES][2] | [weights: TILES][2] fragments
+  // Workgroups are dealt to the XCDs in turn: four row tiles and all their outputs stay on one of them, the row tiles first.
+  const int xcd = blockIdx.x & 7, turn = blockIdx.x >> 3, group = turn / (4 * nx) * 8 + xcd, in = turn % (4 * nx);
+  const int ty = group * 4 + (in & 3), tx = in >> 2;
+  if (ty >= max_tiles) return;
+  const int32_t *tile = p.tiles + 3 * ty;
+  const int e = tile[0], m0 = tile[1], live = tile[2];
+  if (e < 0) return;
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), r16 = lane & 15, g = lane >> 4;
+  const int wm = wave & 1, wn = wave >> 1, ntiles = p.n / 16, steps = p.k / 32, nt0 = tx * (GATED ? TILES / 2 : TILES);
+  // this wave's fragments: one half of the 64 inputs of every fourth tile, of the rows and of the weights
+  const int half = wave & 1, first = wave >> 1;
+  const T *xs[PER], *ws[PER];
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int j = 4 * i + first, place = m0 + min(j * 16 + (lane >> 2), live - 1);
+    xs[i] = (const T *)p.x + (int64_t)(p.tokens ? p.tokens[place] : place) * p.x_stride + half * 32 + row_chunk(lane) * 8;
+    const int wt = min(nt0 + (GATED ? j >> 1 : j), ntiles - 1) + (GATED && (j & 1) ? ntiles : 0);
+    ws[i] = (const T *)p.w + e * p.w_expert + ((int64_t)wt * steps + half) * 512;
+  }
+  const int lane8 = lane * 8;
+  auto fetch = [&](int t) {
+    char *to = smem + (t & 1) * STAGE + (first * 2 + half) * 1024;
+    const int64_t kx = (int64_t)t * 64, kw = (int64_t)t * 1024;
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void *)(xs[i] + kx),
+                                       (__attribute__((address_space(3))) void *)(to + i * 8192), 16, 0, 0);
+      __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void *)(ws[i] + kw + lane8),
+                                       (__attribute__((address_space(3))) void *)(to + (TILES * 2048) + i * 8192), 16, 0, 0);
+    }
+  };
+  f32x4 acc[WN][WM] = {};
+  const uint32_t base = lds_address(smem) + lane * 16, rows = lds_address(smem) + row_place(r16, g) * 16;
+  const int trips = p.k / 64;
+  fetch(0);
+  asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");
+  lds_barrier();
+  if (trips > 1) fetch(1);
+  for (int t = 0; t < trips; ++t) {
+    const uint32_t at = (t & 1) * STAGE, xa = rows + at + wm * WM * 2048, wa = base + at + (TILES + wn * WN) * 2048;
+    u32x4 a[2][WN], b[2][WM];
+    static_for<2>([&](auto H) {
+      constexpr int h = decltype(H)::value;
+      static_for<WN>([&](auto I) { lds_read128<decltype(I)::value * 2048 + h * 1024>(a[h][decltype(I)::value], wa); });
+      static_for<WM>([&](auto I) { lds_read128<decltype(I)::value * 2048 + h * 1024>(b[h][decltype(I)::value], xa); });
+    });
+    static_for<2>([&](auto H) {
+      constexpr int h = decltype(H)::value;
+      static_for<WN>([&](auto I) { lds_wait<h == 0 ? WM + WN : 0>(a[h][decltype(I)::value]); });
+      static_for<WM>([&](auto I) { lds_wait<h == 0 ? WM + WN : 0>(b[h][decltype(I)::value]); });
+      if (h == 1 && t + 1 < trips) {   // every wave has read this stage; the next has landed
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        lds_barrier();
+        if (t + 2 < trips) fetch(t + 2);
+      }
+#pragma unroll
+      for (int i = 0; i < WM; ++i)
+#pragma unroll
+        for (int j = 0; j < WN; ++j) acc[j][i] = mfma16x16x32<Tag>(a[h][j], b[h][i], acc[j][i]);
+    });
   }
 #pragma unroll
   for (int i = 0; i < WM; ++i) {
@@ -381,6 +475,10 @@ int launch_linear(const MoeLinear &p, int tile_m, int max_tiles, hipStream_t st)
     const dim3 grid((nt * 16 * (GATED ? 2 : 1) + BN - 1) / BN, max_tiles);
     if (tile_m == 64) hipLaunchKernelGGL((moe_tile_kernel<Tag, 64, BN, GATED>), grid, dim3(256), (64 + BN) * 256, st, p);
     else hipLaunchKernelGGL((moe_tile_kernel<Tag, 128, BN, GATED>), grid, dim3(256), (128 + BN) * 256, st, p);
+  } else if (tile_m == 256) {
+    const int nx = (nt * (GATED ? 2 : 1) + 15) / 16, groups = (max_tiles + 3) / 4;
+    if (int rc = mv_allow_lds<moe_wide_kernel<Tag, GATED>>()) return rc;
+    hipLaunchKernelGGL((moe_wide_kernel<Tag, GATED>), dim3((unsigned)((groups + 7) / 8 * 8) * 4u * nx), dim3(512), 128 * 1024, st, p, nx, max_tiles);
   } else {
     return MV_E_SHAPE;
   }

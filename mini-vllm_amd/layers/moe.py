@@ -18,7 +18,7 @@ from .linear import Segment, SegmentedLinear, gated_linear, pad_to
 __all__ = ["ExpertMLP"]
 
 # pairs per expert up to which a launch works on tiles of that many rows
-TILES = ((8, 16), (40, 32), (96, 64))
+TILES = ((8, 16), (40, 32), (96, 64), (768, 128))
 
 
 class ExpertMLP(nn.Module):
@@ -61,7 +61,7 @@ class ExpertMLP(nn.Module):
         if self.router.dtype == torch.float32:
             return 16
         per = tokens * self.top / self.experts
-        return next((rows for most, rows in TILES if per <= most), 128)
+        return next((rows for most, rows in TILES if per <= most), 256)
 
     def forward(self, h):
         """-> (shared expert's output or None, the routed experts' part for ``hip_ops.residual_update``)."""

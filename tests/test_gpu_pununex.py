@@ -459,7 +459,7 @@ def test_grouping_of_choices(H, T, top, experts, outputs, tile_m):
     assert sorted(seen) == list(range(len(order)))
 
 
-@pytest.mark.parametrize("dtype, tile_m", [(torch.float32, 16)] + [(torch.bfloat16, m) for m in (16, 32, 64, 128)] + [(torch.float16, 128)])
+@pytest.mark.parametrize("dtype, tile_m", [(torch.float32, 16)] + [(torch.bfloat16, m) for m in (16, 32, 64, 128, 256)] + [(torch.float16, 128), (torch.float16, 256)])
 @pytest.mark.parametrize("T, width, ff, experts, top", [(3, 64, 64, 4, 2), (90, 256, 192, 5, 2), (300, 192, 320, 3, 1)])
 def test_products_over_the_experts(H, dtype, tile_m, T, width, ff, experts, top):
     x = _rand(T, width, dtype=dtype, seed=1)
