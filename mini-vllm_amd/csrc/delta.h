@@ -9,3 +9,4 @@ __device__ __forceinline__ float decay_log(float rate, float a, float bias) { re
 // chunked form (16-bit); MV_E_SHAPE when it does not apply
 size_t mv_delta_chunk_workspace(int n_seqs, int total_q, int heads, int p, int n);
 int mv_delta_chunk_launch(const MvDeltaArgs &a, int dtype, hipStream_t stream);
+int mv_delta_scalar_launch(const MvDeltaArgs &a, hipStream_t stream);   // (from the above: bf16, one decay per head)

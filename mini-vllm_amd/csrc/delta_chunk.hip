@@ -12,54 +12,22 @@
 // What is fp32 by nature enters a product as the sum of two bf16 numbers (three MFMAs: high x high, high x rest, rest x high), about
 // 16 bits of mantissa.  The operands lie in the workspace as MFMA fragments (64 lanes x 16 bytes), which the walk fetches by LDS-DMA.
 //
+// One decay per head needs less (delta_scalar.hip, bf16).
+//
 // Exponentials never overflow: A and B are computed by blocks of 16 x 16 tokens with the sums taken relative to r at the end of the
 // block in front of the rows' (both factors at most 1), or in the middle of a diagonal block; where a block decays by more than
 // 2^kRange a diagonal block is summed pair by pair instead.
-#include "delta.h"
+#include "delta_chunk.h"
 
 namespace {
 
-constexpr int L = 64;              // tokens per chunk
 constexpr float kRange = 60.f;     // log2
-
-typedef bf16_tag B16;
-typedef __attribute__((ext_vector_type(4))) short s16x4;
 
 // sizes of a (chunk, head) in the workspace, in fragments of 1 KiB: [W | Q: 4 token tiles][NK][high, rest] | U0: 4 per 16 columns |
 // K: [2 NK state tiles][2][high, rest] | B: [4 token tiles][2][high, rest] | decay of the whole chunk
 struct Layout {
   int u0, k, b, tail, total;
   __host__ __device__ constexpr Layout(int nk, int p) : u0(16 * nk), k(16 * nk + p / 4), b(24 * nk + p / 4), tail(24 * nk + p / 4 + 16), total(24 * nk + p / 4 + 17) {}
-};
-
-__device__ __forceinline__ void split8(const float (&f)[8], u32x4 &hi, u32x4 &lo) {
-  float rest[8];
-#pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    hi[i] = pack_pair<B16>(f[2 * i], f[2 * i + 1]);
-    rest[2 * i] = f[2 * i] - u2f(hi[i] << 16);
-    rest[2 * i + 1] = f[2 * i + 1] - u2f(hi[i] & 0xffff0000u);
-  }
-#pragma unroll
-  for (int i = 0; i < 4; ++i) lo[i] = pack_pair<B16>(rest[2 * i], rest[2 * i + 1]);
-}
-__device__ __forceinline__ void split44(const f32x4 &a, const f32x4 &b, u32x4 &hi, u32x4 &lo) {
-  const float f[8] = {a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
-  split8(f, hi, lo);
-}
-__device__ __forceinline__ f32x4 mfma3(const u32x4 &ah, const u32x4 &al, const u32x4 &bh, const u32x4 &bl, f32x4 c) {
-  c = mfma16x16x32<B16>(ah, bh, c);
-  c = mfma16x16x32<B16>(ah, bl, c);
-  return mfma16x16x32<B16>(al, bh, c);
-}
-// softplus in hardware exponential and logarithm: an absolute error of about 1e-7
-__device__ __forceinline__ float softplus_fast(float z) {
-  return fmaxf(z, 0.f) + 0.6931471805599453f * __builtin_amdgcn_logf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * fabsf(z)));
-}
-
-struct DeltaPrep {
-  MvDeltaArgs a;
-  char *ws;
 };
 
 template <typename Tag, int NK>
@@ -70,19 +38,12 @@ __global__ void __launch_bounds__(256, 2) delta_prepare_kernel(DeltaPrep q) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
   float *rs = (float *)smem;                              // [L][RS] running log2 decays
   T *ks = (T *)(smem + L * RS * 4), *qs = ks + L * KS;    // [L][KS]; later (from qs on) -A, then T
-  constexpr int TS = L + 4;
   float *ts = (float *)qs;                                // [L][TS]
   constexpr int QB = L * KS * 2 > L * TS * 4 ? L * KS * 2 : L * TS * 4;
   float *fk = (float *)((char *)qs + QB), *fq = fk + L, *bt = fq + L, *part_sums = bt + L;   // [4][64]
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), r16 = lane & 15, g = lane >> 4;
   const int head = blockIdx.y;
-  // chunk slot -> sequence (its slots start at cu_q / L + its number) and chunk
-  int seq = 0;
-  for (int hi = p.n_seqs; hi - seq > 1;) {
-    const int mid = (seq + hi) >> 1;
-    if (p.cu_q[mid] / L + mid <= (int)blockIdx.x) seq = mid;
-    else hi = mid;
-  }
+  const int seq = chunk_sequence(p, blockIdx.x);
   const int q0 = p.cu_q[seq], len = p.cu_q[seq + 1] - q0, t0 = ((int)blockIdx.x - q0 / L - seq) * L;
   if (t0 >= len) return;
   const int nt = min(L, len - t0), grp = head / (p.heads / p.groups);
@@ -163,12 +124,16 @@ __global__ void __launch_bounds__(256, 2) delta_prepare_kernel(DeltaPrep q) {
   for (int m = 0; m < 3; ++m) {
     const int idx = wave + 4 * m;
     if (idx >= 10) continue;
-    const int I = idx < 4 ? 3 : idx < 7 ? 2 : idx < 9 ? 1 : 0, J = idx < 4 ? 3 - idx : idx < 7 ? 6 - idx : idx < 9 ? 8 - idx : 0;
+    int I, J;
+    block_place(idx, I, J);
     const int ref = I == J ? 16 * I + 7 : 16 * I - 1;
     const float *ri = rs + (16 * I + r16) * RS + 8 * g, *rj = rs + (16 * J + r16) * RS + 8 * g, *rr = rs + ref * RS + 8 * g;
     const T *ki = ks + (16 * I + r16) * KS + 8 * g, *kj = ks + (16 * J + r16) * KS + 8 * g, *qi = qs + (16 * I + r16) * KS + 8 * g;
     f32x4 A = {0.f, 0.f, 0.f, 0.f}, B = A;
-    bool fits = true;
+    bool fits = true;   // (the sums fall, so the ends of a diagonal block decide)
+    if (I == J)
+      for (int c = lane; c < N; c += 64)
+        fits = fits && rs[16 * I * RS + c] - rs[ref * RS + c] <= kRange && rs[ref * RS + c] - rs[(16 * I + 15) * RS + c] <= kRange;
 #pragma unroll
     for (int s = 0; s < NK; ++s) {
       float fi[8], fj[8], fp[8];
@@ -180,11 +145,9 @@ __global__ void __launch_bounds__(256, 2) delta_prepare_kernel(DeltaPrep q) {
         const f32x4 a = *(const f32x4 *)(ri + 32 * s + 4 * h), b = *(const f32x4 *)(rj + 32 * s + 4 * h), c = *(const f32x4 *)(rr + 32 * s + 4 * h);
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
-          const float l = a[e] - c[e], r = c[e] - b[e];
-          fits = fits && fabsf(l) <= kRange && fabsf(r) <= kRange;
-          const float el = __builtin_amdgcn_exp2f(l);
+          const float el = __builtin_amdgcn_exp2f(a[e] - c[e]);
           fi[4 * h + e] *= el, fp[4 * h + e] *= el;
-          fj[4 * h + e] *= __builtin_amdgcn_exp2f(r);
+          fj[4 * h + e] *= __builtin_amdgcn_exp2f(c[e] - b[e]);
         }
       }
       u32x4 ih, il, jh, jl, ph, pl;
@@ -214,16 +177,11 @@ __global__ void __launch_bounds__(256, 2) delta_prepare_kernel(DeltaPrep q) {
     }
     blk[m] = A;   // (the negative)
     // B as an operand whose k order is that of an accumulator pair: key 16 (e >> 2) + 4 g + (e & 3) of a step of 32
-    const u32x2 hi = pack_quad<B16>(B);
-    f32x4 rest;
-#pragma unroll
-    for (int e = 0; e < 2; ++e) {
-      rest[2 * e] = B[2 * e] - u2f(hi[e] << 16);
-      rest[2 * e + 1] = B[2 * e + 1] - u2f(hi[e] & 0xffff0000u);
-    }
+    u32x2 hi, lo;
+    split4(B, hi, lo);
     u32x2 *dst = (u32x2 *)(ws + (lay.b + (I * 2 + (J >> 1)) * 2) * 1024 + lane * 16) + (J & 1);
     dst[0] = hi;
-    dst[128] = pack_quad<B16>(rest);
+    dst[128] = lo;
     if (I == J && (I & 1) == 0) dst[1] = dst[129] = u32x2{0u, 0u};   // the columns behind, in the same step of 32
   }
 
@@ -246,80 +204,16 @@ __global__ void __launch_bounds__(256, 2) delta_prepare_kernel(DeltaPrep q) {
   for (int m = 0; m < 3; ++m) {
     const int idx = wave + 4 * m;
     if (idx >= 10) continue;
-    const int I = idx < 4 ? 3 : idx < 7 ? 2 : idx < 9 ? 1 : 0, J = idx < 4 ? 3 - idx : idx < 7 ? 6 - idx : idx < 9 ? 8 - idx : 0;
+    int I, J;
+    block_place(idx, I, J);
     *(f32x4 *)(ts + (16 * I + r16) * TS + 16 * J + 4 * g) = blk[m];
   }
   __syncthreads();
 
-  // ---- T = (1 + A)^-1 diag(beta).  Its entries are at most 1, since no factor 1 - beta k k^T of the recurrence lengthens a vector.
-  // A wave inverts a diagonal block, a column in each of 16 lanes ..
-  {
-    float *d = ts + 16 * wave * TS + 16 * wave, x[16];
+  solve_chunk(ts, bt, wave, lane);
+  u32x4 th[kTriangle], tl[kTriangle];
 #pragma unroll
-    for (int i = 0; i < 16; ++i) {
-      float a = i == r16 ? 1.f : 0.f, b = 0.f;
-#pragma unroll
-      for (int j = 0; j < i; j += 4) {   // (zeros from column i on)
-        const f32x4 t = *(const f32x4 *)(d + i * TS + j);
-        a = fmaf(t[0], x[j], a);
-        if (j + 1 < i) b = fmaf(t[1], x[j + 1], b);
-        if (j + 2 < i) a = fmaf(t[2], x[j + 2], a);
-        if (j + 3 < i) b = fmaf(t[3], x[j + 3], b);
-      }
-      x[i] = a + b;
-    }
-    if (lane < 16) {
-#pragma unroll
-      for (int i = 0; i < 16; ++i) d[i * TS + r16] = x[i];
-    }
-  }
-  __syncthreads();
-  // .. and then a wave a column of blocks, from the diagonal down: T_IJ = T_II sum_{J <= K < I} (-A_IK) T_KJ.  Accumulators are the
-  // right operand of the next product, whose keys are 4 g + step.
-  {
-    auto product = [&](int I, int K, const f32x4 &right, f32x4 acc) {
-      const f32x4 left = *(const f32x4 *)(ts + (16 * I + r16) * TS + 16 * K + 4 * g);
-#pragma unroll
-      for (int e = 0; e < 4; ++e) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(left[e], right[e], acc, 0, 0, 0);
-      return acc;
-    };
-    f32x4 t[4];
-#pragma unroll
-    for (int I = 0; I < 4; ++I) {
-      t[I] = f32x4{0.f, 0.f, 0.f, 0.f};
-      if (I < wave) continue;
-      if (I == wave) {
-#pragma unroll
-        for (int e = 0; e < 4; ++e) t[I][e] = ts[(16 * I + 4 * g + e) * TS + 16 * wave + r16];
-        continue;
-      }
-      f32x4 sum = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int K = 0; K < I; ++K)
-        if (K >= wave) sum = product(I, K, t[K], sum);
-      t[I] = product(I, I, sum, t[I]);
-    }
-    const float beta = bt[16 * wave + r16];
-    __syncthreads();   // every wave has read A
-#pragma unroll
-    for (int I = 0; I < 4; ++I)
-      if (I >= wave) {
-#pragma unroll
-        for (int e = 0; e < 4; ++e) ts[(16 * I + 4 * g + e) * TS + 16 * wave + r16] = t[I][e] * beta;
-      }
-  }
-  __syncthreads();
-  // T by rows as operands, either side: (token tile, step of 32 tokens) 0 0, 1 0, 2 0, 2 1, 3 0, 3 1; tokens 16 (e >> 2) + 4 g + (e & 3)
-  u32x4 th[6], tl[6];
-#pragma unroll
-  for (int m = 0; m < 6; ++m) {
-    const int it = m < 2 ? m : 2 + (m - 2) / 2, s = m < 2 ? 0 : m & 1;
-    const float *row = ts + (16 * it + r16) * TS + 32 * s + 4 * g;
-    f32x4 a = *(const f32x4 *)row, b = {0.f, 0.f, 0.f, 0.f};
-    if (2 * s + 1 <= it) b = *(const f32x4 *)(row + 16);
-    split44(a, b, th[m], tl[m]);
-  }
-  auto of = [](int it, int s) constexpr { return it < 2 ? it : 2 * it - 2 + s; };
+  for (int m = 0; m < kTriangle; ++m) solution_operand(ts, m, lane, th[m], tl[m]);
 
   // ---- by 32 channels: K = e^(r_last - r) k by state rows, in the order of the walk's accumulators, and -W = -T e^r k by tokens;
   // by 16 columns of v: U0 = T v
@@ -348,7 +242,7 @@ __global__ void __launch_bounds__(256, 2) delta_prepare_kernel(DeltaPrep q) {
           dst[0] = hi, dst[64] = lo;
           split8(w, hi, lo);
 #pragma unroll
-          for (int it = 2 * s; it < 4; ++it) acc[d][it] = mfma3(hi, lo, th[of(it, s)], tl[of(it, s)], acc[d][it]);
+          for (int it = 2 * s; it < 4; ++it) acc[d][it] = mfma3(hi, lo, th[triangle(it, s)], tl[triangle(it, s)], acc[d][it]);
         }
       }
 #pragma unroll
@@ -376,9 +270,9 @@ __global__ void __launch_bounds__(256, 2) delta_prepare_kernel(DeltaPrep q) {
         split8(f, hi, lo);
 #pragma unroll
         for (int it = 2 * s; it < 4; ++it) {
-          acc[it] = mfma16x16x32<B16>(th[of(it, s)], hi, acc[it]);
-          acc[it] = mfma16x16x32<B16>(tl[of(it, s)], hi, acc[it]);
-          if constexpr (!__is_same(Tag, B16)) acc[it] = mfma16x16x32<B16>(th[of(it, s)], lo, acc[it]);
+          acc[it] = mfma16x16x32<B16>(th[triangle(it, s)], hi, acc[it]);
+          acc[it] = mfma16x16x32<B16>(tl[triangle(it, s)], hi, acc[it]);
+          if constexpr (!__is_same(Tag, B16)) acc[it] = mfma16x16x32<B16>(th[triangle(it, s)], lo, acc[it]);
         }
       }
       // in the layout of an accumulator: column lane & 15, tokens 4 (lane >> 4) ..
@@ -583,8 +477,6 @@ __global__ void __launch_bounds__(256, 1) delta_walk_kernel(DeltaPrep q) {
   }
 }
 
-int64_t chunk_slots(int n_seqs, int total_q) { return (int64_t)total_q / L + n_seqs; }
-
 template <typename Tag, int NK>
 int launch(const DeltaPrep &q, hipStream_t stream) {
   const MvDeltaArgs &a = q.a;
@@ -622,6 +514,7 @@ int mv_delta_chunk_launch(const MvDeltaArgs &a, int dtype, hipStream_t stream) {
   if (!mv_aligned16(a.x) || (a.x_stride & 7) || (a.k_off & 7) || (a.q_off & 7) || a.total_q > 64 * 1000000) return MV_E_ALIGN;
   if (a.channel_decay && (!mv_aligned16(a.a) || (a.a_stride & 7) || !mv_aligned16(a.dt_bias))) return MV_E_ALIGN;
   const DeltaPrep q{a, (char *)a.workspace};
+  if (!a.channel_decay && dtype == MV_BF16) return mv_delta_scalar_launch(a, stream);
 #define MV_DN(NK_) \
   if (a.n == 32 * NK_) return dtype == MV_BF16 ? launch<bf16_tag, NK_>(q, stream) : launch<f16_tag, NK_>(q, stream)
   MV_DN(1);

@@ -253,7 +253,7 @@ def test_tiles_follow_the_pairs_per_expert():
     assert e.tile_rows(1) == 16                                          # (fp32: the only form)
     e = e.to(torch.bfloat16)
     rows = [e.tile_rows(t) for t in (1, 16, 256, 16384)]
-    assert rows == sorted(rows) and rows[0] == 16 and rows[-1] == 128
+    assert rows == sorted(rows) and rows[0] == 16 and rows[-1] == 256
 
 
 def test_header_shapes_of_a_checkpoint(tmp_path):
