@@ -72,12 +72,12 @@ constexpr int TS = L + 4;   // row stride of A and T in LDS
 constexpr int kTriangle = 6;
 __host__ __device__ constexpr int triangle(int it, int s) { return it < 2 ? it : 2 * it - 2 + s; }
 
-// T = (1 + A)^-1 diag(beta), in place of -A in LDS (4 waves; -A is there, behind a barrier; so is T afterwards).  T's entries are at most 1, since no
-// factor 1 - beta k k^T of the recurrence lengthens a vector.
+// T = (1 + A)^-1 diag(beta), in place of -A in LDS (-A is there, behind a barrier; so is T afterwards), by the first four waves.  T's entries are
+// at most 1, since no factor 1 - beta k k^T of the recurrence lengthens a vector.
 __device__ __forceinline__ void solve_chunk(float *ts, const float *bt, int wave, int lane) {
   const int r16 = lane & 15, g = lane >> 4;
   // A wave inverts a diagonal block, a column in each of 16 lanes ..
-  {
+  if (wave < 4) {
     float *d = ts + 16 * wave * TS + 16 * wave, x[16];
 #pragma unroll
     for (int i = 0; i < 16; ++i) {
@@ -100,14 +100,14 @@ __device__ __forceinline__ void solve_chunk(float *ts, const float *bt, int wave
   __syncthreads();
   // .. and then a wave a column of blocks, from the diagonal down: T_IJ = T_II sum_{J <= K < I} (-A_IK) T_KJ.  Accumulators are the
   // right operand of the next product, whose keys are 4 g + step.
-  {
+  f32x4 t[4];
+  if (wave < 4) {
     auto product = [&](int I, int K, const f32x4 &right, f32x4 acc) {
       const f32x4 left = *(const f32x4 *)(ts + (16 * I + r16) * TS + 16 * K + 4 * g);
 #pragma unroll
       for (int e = 0; e < 4; ++e) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(left[e], right[e], acc, 0, 0, 0);
       return acc;
     };
-    f32x4 t[4];
 #pragma unroll
     for (int I = 0; I < 4; ++I) {
       t[I] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -123,8 +123,10 @@ __device__ __forceinline__ void solve_chunk(float *ts, const float *bt, int wave
         if (K >= wave) sum = product(I, K, t[K], sum);
       t[I] = product(I, I, sum, t[I]);
     }
+  }
+  __syncthreads();   // every wave has read A
+  if (wave < 4) {
     const float beta = bt[16 * wave + r16];
-    __syncthreads();   // every wave has read A
 #pragma unroll
     for (int I = 0; I < 4; ++I)
       if (I >= wave) {
@@ -134,6 +136,7 @@ __device__ __forceinline__ void solve_chunk(float *ts, const float *bt, int wave
   }
   __syncthreads();
 }
+
 // rows of T as an operand of either side: row r16 of a token tile, tokens 16 (e >> 2) + 4 g + (e & 3) of a step of 32
 __device__ __forceinline__ void solution_operand(const float *ts, int m, int lane, u32x4 &hi, u32x4 &lo) {
   const int it = m < 2 ? m : 2 + (m - 2) / 2, s = m < 2 ? 0 : m & 1;

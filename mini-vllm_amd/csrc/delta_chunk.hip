@@ -22,6 +22,7 @@
 namespace {
 
 constexpr float kRange = 60.f;     // log2
+constexpr int kPrepareWaves = 8;
 
 // sizes of a (chunk, head) in the workspace, in fragments of 1 KiB: [W | Q: 4 token tiles][NK][high, rest] | U0: 4 per 16 columns |
 // K: [2 NK state tiles][2][high, rest] | B: [4 token tiles][2][high, rest] | decay of the whole chunk
@@ -31,16 +32,16 @@ struct Layout {
 };
 
 template <typename Tag, int NK>
-__global__ void __launch_bounds__(256, 2) delta_prepare_kernel(DeltaPrep q) {
+__global__ void __launch_bounds__(kPrepareWaves * 64, 4) delta_prepare_kernel(DeltaPrep q) {
   typedef typename elem<Tag>::T T;
-  constexpr int N = NK * 32, RS = N + 4, KS = N + 8;   // LDS row strides: fp32, 16-bit
+  constexpr int N = NK * 32, W = kPrepareWaves, RS = N + 4, KS = N + 8;   // LDS row strides: fp32, 16-bit
   const MvDeltaArgs &p = q.a;
   extern __shared__ __attribute__((aligned(16))) char smem[];
   float *rs = (float *)smem;                              // [L][RS] running log2 decays
   T *ks = (T *)(smem + L * RS * 4), *qs = ks + L * KS;    // [L][KS]; later (from qs on) -A, then T
   float *ts = (float *)qs;                                // [L][TS]
   constexpr int QB = L * KS * 2 > L * TS * 4 ? L * KS * 2 : L * TS * 4;
-  float *fk = (float *)((char *)qs + QB), *fq = fk + L, *bt = fq + L, *part_sums = bt + L;   // [4][64]
+  float *fk = (float *)((char *)qs + QB), *fq = fk + L, *bt = fq + L, *part_sums = bt + L;   // [W][64]
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), r16 = lane & 15, g = lane >> 4;
   const int head = blockIdx.y;
   const int seq = chunk_sequence(p, blockIdx.x);
@@ -51,12 +52,12 @@ __global__ void __launch_bounds__(256, 2) delta_prepare_kernel(DeltaPrep q) {
   char *ws = q.ws + ((int64_t)blockIdx.x * p.heads + head) * lay.total * 1024;
   const T *x = (const T *)p.x + (int64_t)(q0 + t0) * p.x_stride;
 
-  // ---- k, q (tokens behind the end: zeros) and their lengths: four threads a token
+  // ---- k, q (tokens behind the end: zeros) and their lengths: eight threads a token
   {
-    const int t = tid >> 2, part = tid & 3;
+    const int t = tid >> 3, part = tid & 7;
     const T *row = x + (int64_t)min(t, nt - 1) * p.x_stride;
     float sk = 0.f, sq = 0.f;
-    for (int c = part * 8; c < N; c += 32) {
+    for (int c = part * 8; c < N; c += 64) {
       u32x4 a = *(const u32x4 *)(row + p.k_off + grp * N + c), b = *(const u32x4 *)(row + p.q_off + grp * N + c);
       if (t >= nt) a = b = u32x4{0u, 0u, 0u, 0u};
       float fa[8], fb[8];
@@ -67,8 +68,8 @@ __global__ void __launch_bounds__(256, 2) delta_prepare_kernel(DeltaPrep q) {
       *(u32x4 *)(ks + t * KS + c) = a;
       *(u32x4 *)(qs + t * KS + c) = b;
     }
-    sk += __shfl_xor(sk, 1, 64), sq += __shfl_xor(sq, 1, 64);
-    sk += __shfl_xor(sk, 2, 64), sq += __shfl_xor(sq, 2, 64);
+#pragma unroll
+    for (int o = 1; o <= 4; o <<= 1) sk += __shfl_xor(sk, o, 64), sq += __shfl_xor(sq, o, 64);
     if (part == 0) {
       fk[t] = 1.f / sqrtf(sk + p.unit_eps), fq[t] = p.q_scale / sqrtf(sq + p.unit_eps);
       bt[t] = t < nt ? sigmoid_f32(elem<Tag>::ld(((const T *)p.beta)[(int64_t)(q0 + t0 + t) * p.beta_stride + head])) : 0.f;
@@ -79,39 +80,42 @@ __global__ void __launch_bounds__(256, 2) delta_prepare_kernel(DeltaPrep q) {
     const float rate = -expf(elem<Tag>::ld(((const T *)p.a_log)[head])) * 1.4426950408889634f;
     const T *a = (const T *)p.a + (int64_t)(q0 + t0) * p.a_stride, *bias = (const T *)p.dt_bias;
     if (p.channel_decay) {
-      for (int i = tid; i < L * N / 8; i += 256) {
+      for (int i = tid; i < L * N / 8; i += W * 64) {
         const int t = i / (N / 8), c = (i - t * (N / 8)) * 8;
         float f[8], b[8];
         unpack8<Tag>(*(const u32x4 *)(a + (int64_t)min(t, nt - 1) * p.a_stride + head * N + c), f);
         unpack8<Tag>(*(const u32x4 *)(bias + head * N + c), b);
 #pragma unroll
-        for (int j = 0; j < 8; ++j) rs[t * RS + c + j] = t < nt ? rate * softplus_fast(f[j] + b[j]) : 0.f;
+        for (int j = 0; j < 8; ++j) f[j] = t < nt ? rate * softplus_fast(f[j] + b[j]) : 0.f;
+        f32x4 *dst = (f32x4 *)(rs + t * RS + c);
+        dst[0] = f32x4{f[0], f[1], f[2], f[3]}, dst[1] = f32x4{f[4], f[5], f[6], f[7]};
       }
     } else {
       const float b = elem<Tag>::ld(bias[head]);
-      const int t = tid >> 2;
+      const int t = tid >> 3;
       const float v = t < nt ? rate * softplus_fast(elem<Tag>::ld(a[(int64_t)t * p.a_stride + head]) + b) : 0.f;
-      for (int c = tid & 3; c < N; c += 4) rs[t * RS + c] = v;
+      for (int c = tid & 7; c < N; c += 8) rs[t * RS + c] = v;
     }
     __syncthreads();
-    // a thread a quarter of a channel's tokens (the threads of a wave: adjacent channels); then the quarters ahead are added
+    // a thread TW of a channel's tokens (the threads of a wave: adjacent channels); then the sums ahead are added
+    constexpr int TW = L / W;
     for (int c0 = 0; c0 < N; c0 += 64) {
       const int c = c0 + lane;
-      float v[16], sum = 0.f;
+      float v[TW], sum = 0.f;
       if (c < N) {
 #pragma unroll
-        for (int t = 0; t < 16; ++t) v[t] = rs[(16 * wave + t) * RS + c];
+        for (int t = 0; t < TW; ++t) v[t] = rs[(TW * wave + t) * RS + c];
 #pragma unroll
-        for (int t = 0; t < 16; ++t) sum += v[t], v[t] = sum;
+        for (int t = 0; t < TW; ++t) sum += v[t], v[t] = sum;
         part_sums[wave * 64 + lane] = sum;
       }
       __syncthreads();
       if (c < N) {
         float ahead = 0.f;
 #pragma unroll
-        for (int w = 0; w < 3; ++w) ahead += w < wave ? part_sums[w * 64 + lane] : 0.f;
+        for (int w = 0; w < W - 1; ++w) ahead += w < wave ? part_sums[w * 64 + lane] : 0.f;
 #pragma unroll
-        for (int t = 0; t < 16; ++t) rs[(16 * wave + t) * RS + c] = ahead + v[t];
+        for (int t = 0; t < TW; ++t) rs[(TW * wave + t) * RS + c] = ahead + v[t];
       }
       if (c0 + 64 < N) __syncthreads();
     }
@@ -119,10 +123,11 @@ __global__ void __launch_bounds__(256, 2) delta_prepare_kernel(DeltaPrep q) {
   __syncthreads();
 
   // ---- A and B by blocks of 16 x 16 tokens (rows I, columns J <= I), ten of them over the waves; a lane gets row r16, columns 4 g ..
-  f32x4 blk[3];
+  constexpr int BW = (10 + W - 1) / W;
+  f32x4 blk[BW];
 #pragma unroll
-  for (int m = 0; m < 3; ++m) {
-    const int idx = wave + 4 * m;
+  for (int m = 0; m < BW; ++m) {
+    const int idx = wave + W * m;
     if (idx >= 10) continue;
     int I, J;
     block_place(idx, I, J);
@@ -186,7 +191,7 @@ __global__ void __launch_bounds__(256, 2) delta_prepare_kernel(DeltaPrep q) {
   }
 
   // ---- the operands that meet S and U: e^r q by rows; e^(r_last - r) k by state rows, in the order of the walk's accumulators
-  for (int f = wave; f < 4 * NK; f += 4) {
+  for (int f = wave; f < 4 * NK; f += W) {
     const int it = f / NK, s = f - it * NK, t = 16 * it + r16, c = 32 * s + 8 * g;
     float v[8];
     u32x4 hi, lo;
@@ -198,11 +203,11 @@ __global__ void __launch_bounds__(256, 2) delta_prepare_kernel(DeltaPrep q) {
     u32x4 *dst = (u32x4 *)(ws + (8 * NK + f * 2) * 1024) + lane;
     dst[0] = hi, dst[64] = lo;
   }
-  for (int c = tid; c < N; c += 256) ((float *)(ws + lay.tail * 1024))[c] = __builtin_amdgcn_exp2f(rs[(L - 1) * RS + c]);
+  for (int c = tid; c < N; c += W * 64) ((float *)(ws + lay.tail * 1024))[c] = __builtin_amdgcn_exp2f(rs[(L - 1) * RS + c]);
   __syncthreads();   // q is done with
 #pragma unroll
-  for (int m = 0; m < 3; ++m) {
-    const int idx = wave + 4 * m;
+  for (int m = 0; m < BW; ++m) {
+    const int idx = wave + W * m;
     if (idx >= 10) continue;
     int I, J;
     block_place(idx, I, J);
@@ -211,23 +216,23 @@ __global__ void __launch_bounds__(256, 2) delta_prepare_kernel(DeltaPrep q) {
   __syncthreads();
 
   solve_chunk(ts, bt, wave, lane);
-  u32x4 th[kTriangle], tl[kTriangle];
-#pragma unroll
-  for (int m = 0; m < kTriangle; ++m) solution_operand(ts, m, lane, th[m], tl[m]);
 
   // ---- by 32 channels: K = e^(r_last - r) k by state rows, in the order of the walk's accumulators, and -W = -T e^r k by tokens;
   // by 16 columns of v: U0 = T v
-  for (int item = wave; item < NK + p.p / 16; item += 4) {
+  for (int item = wave; item < NK + p.p / 16; item += W) {
     if (item < NK) {
       f32x4 acc[2][4];
 #pragma unroll
-      for (int d = 0; d < 2; ++d) {
-        const int i = 2 * item + d, c = item * 32 + (r16 >> 2) * 8 + d * 4 + (r16 & 3);
-        const float last = rs[(L - 1) * RS + c];
+      for (int it = 0; it < 4; ++it) acc[0][it] = acc[1][it] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int it = 0; it < 4; ++it) acc[d][it] = f32x4{0.f, 0.f, 0.f, 0.f};
+      for (int s = 0; s < 2; ++s) {
+        u32x4 th[4], tl[4];
 #pragma unroll
-        for (int s = 0; s < 2; ++s) {
+        for (int it = 2 * s; it < 4; ++it) solution_operand(ts, triangle(it, s), lane, th[it], tl[it]);
+#pragma unroll
+        for (int d = 0; d < 2; ++d) {
+          const int i = 2 * item + d, c = item * 32 + (r16 >> 2) * 8 + d * 4 + (r16 & 3);
+          const float last = rs[(L - 1) * RS + c];
           float v[8], w[8];
           u32x4 hi, lo;
 #pragma unroll
@@ -242,7 +247,7 @@ __global__ void __launch_bounds__(256, 2) delta_prepare_kernel(DeltaPrep q) {
           dst[0] = hi, dst[64] = lo;
           split8(w, hi, lo);
 #pragma unroll
-          for (int it = 2 * s; it < 4; ++it) acc[d][it] = mfma3(hi, lo, th[triangle(it, s)], tl[triangle(it, s)], acc[d][it]);
+          for (int it = 2 * s; it < 4; ++it) acc[d][it] = mfma3(hi, lo, th[it], tl[it], acc[d][it]);
         }
       }
 #pragma unroll
@@ -270,9 +275,11 @@ __global__ void __launch_bounds__(256, 2) delta_prepare_kernel(DeltaPrep q) {
         split8(f, hi, lo);
 #pragma unroll
         for (int it = 2 * s; it < 4; ++it) {
-          acc[it] = mfma16x16x32<B16>(th[triangle(it, s)], hi, acc[it]);
-          acc[it] = mfma16x16x32<B16>(tl[triangle(it, s)], hi, acc[it]);
-          if constexpr (!__is_same(Tag, B16)) acc[it] = mfma16x16x32<B16>(th[triangle(it, s)], lo, acc[it]);
+          u32x4 th, tl;
+          solution_operand(ts, triangle(it, s), lane, th, tl);
+          acc[it] = mfma16x16x32<B16>(th, hi, acc[it]);
+          acc[it] = mfma16x16x32<B16>(tl, hi, acc[it]);
+          if constexpr (!__is_same(Tag, B16)) acc[it] = mfma16x16x32<B16>(th, lo, acc[it]);
         }
       }
       // in the layout of an accumulator: column lane & 15, tokens 4 (lane >> 4) ..
@@ -483,8 +490,8 @@ int launch(const DeltaPrep &q, hipStream_t stream) {
   constexpr int RS = NK * 32 + 4, KS = NK * 32 + 8;
   constexpr int QB = L * KS * 2 > L * (L + 4) * 4 ? L * KS * 2 : L * (L + 4) * 4;
   if (int rc = mv_allow_lds<delta_prepare_kernel<Tag, NK>>()) return rc;
-  hipLaunchKernelGGL((delta_prepare_kernel<Tag, NK>), dim3((unsigned)chunk_slots(a.n_seqs, a.total_q), a.heads), dim3(256),
-                     L * RS * 4 + L * KS * 2 + QB + 7 * L * 4, stream, q);
+  hipLaunchKernelGGL((delta_prepare_kernel<Tag, NK>), dim3((unsigned)chunk_slots(a.n_seqs, a.total_q), a.heads),
+                     dim3(kPrepareWaves * 64), L * RS * 4 + L * KS * 2 + QB + (3 + kPrepareWaves) * L * 4, stream, q);
   MV_LAUNCH_CHECK();
   // two column tiles a wave share every operand read, where that still leaves a workgroup per CU
   const int tiles = a.p / 16, wide = (tiles + 7) / 8;
