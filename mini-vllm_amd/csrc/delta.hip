@@ -315,7 +315,8 @@ extern "C" int mv_delta_step(const MvDeltaArgs *a, int dtype, void *stream) {
   if (a->taps < 1 || a->taps > kMaxTaps || a->p_true <= 0 || a->p_true > a->p || a->gate_stride < (int64_t)a->heads * a->p) return MV_E_SHAPE;
   if (a->gate_kind != MV_GATE_SILU && a->gate_kind != MV_GATE_SIGMOID) return MV_E_RANGE;
   const int pieces = a->n * a->p / 4;
-  const int threads = pieces <= 256 * kStepAhead ? 256 : pieces <= 512 * kStepAhead ? 512 : 1024;
+  // (few workgroups: latency decides, and eight waves a head are quicker through its dependent phases)
+  const int threads = pieces > 512 * kStepAhead ? 1024 : pieces > 256 * kStepAhead || (int64_t)a->heads * a->n_seqs <= 512 ? 512 : 256;
   const size_t lds = (size_t)(3 * a->p + 3 * a->n + 2 * (threads / (a->p / 4)) * a->p) * 4;
   const dim3 grid(a->heads, a->n_seqs);
   MV_DISPATCH_DTYPE(dtype, {
