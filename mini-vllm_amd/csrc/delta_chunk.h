@@ -76,9 +76,11 @@ __host__ __device__ constexpr int triangle(int it, int s) { return it < 2 ? it :
 // at most 1, since no factor 1 - beta k k^T of the recurrence lengthens a vector.
 __device__ __forceinline__ void solve_chunk(float *ts, const float *bt, int wave, int lane) {
   const int r16 = lane & 15, g = lane >> 4;
-  // A wave inverts a diagonal block, a column in each of 16 lanes ..
-  if (wave < 4) {
-    float *d = ts + 16 * wave * TS + 16 * wave, x[16];
+  // A wave inverts a diagonal block, a column in each of 16 lanes, into one of the blocks above the diagonal, which nothing uses ..
+  auto inverse = [&](int I) { return ts + (I < 3 ? 16 * (I + 1) : 16 * TS + 32); };
+  if (wave < 4 && lane < 16) {
+    const float *d = ts + 16 * wave * TS + 16 * wave;
+    float *to = inverse(wave), x[16];
 #pragma unroll
     for (int i = 0; i < 16; ++i) {
       float a = i == r16 ? 1.f : 0.f, b = 0.f;
@@ -92,18 +94,16 @@ __device__ __forceinline__ void solve_chunk(float *ts, const float *bt, int wave
       }
       x[i] = a + b;
     }
-    if (lane < 16) {
 #pragma unroll
-      for (int i = 0; i < 16; ++i) d[i * TS + r16] = x[i];
-    }
+    for (int i = 0; i < 16; ++i) to[i * TS + r16] = x[i];
   }
   __syncthreads();
   // .. and then a wave a column of blocks, from the diagonal down: T_IJ = T_II sum_{J <= K < I} (-A_IK) T_KJ.  Accumulators are the
   // right operand of the next product, whose keys are 4 g + step.
   f32x4 t[4];
   if (wave < 4) {
-    auto product = [&](int I, int K, const f32x4 &right, f32x4 acc) {
-      const f32x4 left = *(const f32x4 *)(ts + (16 * I + r16) * TS + 16 * K + 4 * g);
+    auto product = [&](const float *block, const f32x4 &right, f32x4 acc) {
+      const f32x4 left = *(const f32x4 *)(block + r16 * TS + 4 * g);
 #pragma unroll
       for (int e = 0; e < 4; ++e) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(left[e], right[e], acc, 0, 0, 0);
       return acc;
@@ -114,14 +114,14 @@ __device__ __forceinline__ void solve_chunk(float *ts, const float *bt, int wave
       if (I < wave) continue;
       if (I == wave) {
 #pragma unroll
-        for (int e = 0; e < 4; ++e) t[I][e] = ts[(16 * I + 4 * g + e) * TS + 16 * wave + r16];
+        for (int e = 0; e < 4; ++e) t[I][e] = inverse(I)[(4 * g + e) * TS + r16];
         continue;
       }
       f32x4 sum = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int K = 0; K < I; ++K)
-        if (K >= wave) sum = product(I, K, t[K], sum);
-      t[I] = product(I, I, sum, t[I]);
+        if (K >= wave) sum = product(ts + 16 * I * TS + 16 * K, t[K], sum);
+      t[I] = product(inverse(I), sum, t[I]);
     }
   }
   __syncthreads();   // every wave has read A

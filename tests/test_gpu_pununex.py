@@ -374,6 +374,30 @@ def test_decays_of_every_speed_over_a_long_prompt(H, slow, fast, channel_decay):
     _close(s.prefill([(ins, 0, 900)], [1]), s.want(ins, False), torch.bfloat16, factor=1.5)
 
 
+@pytest.mark.parametrize("channel_decay", [False, True], ids=["head", "channel"])
+def test_many_heads_and_sequences(H, channel_decay):
+    """Enough workgroups that a wave takes two column tiles, one wave of them a single one."""
+    s = _Delta(H, 32, 16, 64, 112, 3, channel_decay, torch.bfloat16)
+    lens = (70, 5, 64, 65, 128, 1, 33, 90, 2)
+    ins = [s.inputs(n, i) for i, n in enumerate(lens)]
+    o = s.prefill([(v, 0, n) for v, n in zip(ins, lens)], [0, 3, 1, 4, 2, 5, -1, -1, -1])
+    at = 0
+    for i, (v, n) in enumerate(zip(ins, lens)):
+        if i in (0, 3, 4, 5, 7):
+            _close(o[at:at + n], s.want(v, False), torch.bfloat16, f"sequence {i}", factor=1.5)
+        at += n
+
+
+@pytest.mark.parametrize("channel_decay", [False, True], ids=["head", "channel"])
+def test_equal_keys_that_nothing_forgets(H, channel_decay):
+    """Every token writes at the same key at full strength and nothing decays: the triangular system at its worst."""
+    s = _Delta(H, 2, 1, 64, 32, 2, channel_decay, torch.bfloat16, slow=8.0, fast=1e-6)
+    x, beta, a, gate = s.inputs(200, 3)
+    x[:, s.shape.k_off:] = x[:1, s.shape.k_off:]
+    ins = (x, torch.full_like(beta, 9.0), torch.full_like(a, -30.0), gate)
+    _close(s.prefill([(ins, 0, 200)], [1]), s.want(ins, False), torch.bfloat16, factor=1.5)
+
+
 def test_a_repeated_step_changes_nothing_and_padding_rows_keep_nothing(H):
     s = _Delta(H, 4, 2, 48, 64, 4, True, torch.bfloat16)
     ins = s.inputs(20, 3)
