@@ -123,15 +123,15 @@ def _pununex(like: str, peer: str, pairs: int, window: int = 2048, experts: int 
     c = MODELS[like]
     heads, kv, width, ff = (c[k] for k in ("num_attention_heads", "num_key_value_heads", "hidden_size", "intermediate_size"))
     delta = {"heads": heads, "kv_heads": heads // 2, "dim": 128, "vdim": 128, "conv": 4}
-    left = {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 30.0,
-            "mask": {"size": window, "keep_first": 4}}
+    left = {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 50.0,
+            "mask": {"size": window, "keep_first": 8}}
     right = {"heads": heads // 2, "kv_heads": heads // 2, "dim": 128, "vdim": 128, "conv": 4, "rank": rank}
-    moe = {"kind": "moe", "router": {"experts": experts, "identity": 2, "top": 4, "scale": 2.0,
+    moe = {"kind": "moe", "router": {"experts": experts, "identity": 2, "top": 4, "scale": 2.5,
                                      "groups": {"count": 2, "keep": 1}}, "expert": {"ff": ff // 8}, "shared": {"ff": ff // 2}}
     layers = [{"type": "delta", "mixer": delta, "mlp": {"kind": "dense", "ff": ff}},
               {"type": "parallel", "mixer": {"left": left, "right": right, "left_scale": 0.7, "right_scale": 0.7}, "mlp": moe}] * pairs
     return dict(architecture="Pununex", vocab=c["vocab_size"], width=width, norm={"eps": 1e-6}, layers=layers, like=peer, window=window,
-                embedding={"bigram": {"buckets": 65521, "mul_prev": 31, "mul_cur": 17}}, vocab_size=c["vocab_size"], hidden_size=width,
+                embedding={"bigram": {"buckets": 65521, "mul_prev": 131, "mul_cur": 71}}, vocab_size=c["vocab_size"], hidden_size=width,
                 num_attention_heads=heads, num_key_value_heads=kv, head_dim=128, intermediate_size=ff)
 
 
@@ -714,7 +714,8 @@ def _delta_and_expert_prefill(ex, tokens: int, probe) -> dict:
         if mine:
             s, us = mine[0][0].shape, statistics.median(u for _, u in mine)
             byt = tokens * (2 * s.heads * s.p + 2 * s.groups * s.n + s.heads * (1 + (s.n if kind else 1))) * ex.dtype.itemsize
-            out[key] = {"bound": "hbm", "kernel": "delta_prepare_kernel + delta_walk_kernel", "bytes_per_launch": byt,
+            names = "delta_prepare_kernel + delta_walk_kernel" if kind else "delta_scalar_prepare_kernel + delta_scalar_walk_kernel"
+            out[key] = {"bound": "hbm", "kernel": names, "bytes_per_launch": byt,
                         "us_per_launch": round(us, 2), "achieved": round(byt / us / 1e3, 1), "peak": HBM_PEAK_GBS, "unit": "GB/s",
                         "frac": round(byt / us / 1e3 / HBM_PEAK_GBS, 4)}
     experts, t = expert_modules(ex), probe.times_us("experts")
