@@ -323,7 +323,7 @@ int mv_act_and_mul(const void *x, int64_t x_stride, void *out, int64_t out_strid
  * y: rows of dtype at stride y_stride, or (y_splits > 0) fp32 partial sums [y_splits][rows][cols]; NULL = nothing.
  * All weights / tables are of dtype.  Means are over cols_true <= cols columns; the others hold zeros.
  * layer_norm: both norms are layer norms instead, (z - mean) / sqrt(mean((z - mean)^2) + eps) * w + b (biases NULL = 0).
- * pairs: a second table, [buckets + 1][cols], whose row (previous token * mul_prev + token * mul_cur) mod buckets is added where the
+ * pairs: a second table, [buckets + 1][cols], whose row (mul_prev * id[t - 1] + mul_cur * id[t]) % buckets is added where the
  *     embedding is (a sequence's first token: row `buckets`).  The token before a step's first is kept in prev_tokens [2][slots],
  *     half = number of tokens before it & 1, at state_slots[sequence] (< 0: as if it were 0); the step writes its last one to the
  *     other tokens' half.  Sequences: rows cu_q[s] .. cu_q[s + 1]; cu_q NULL: one row each.  Rows at position < 0: padding.
@@ -690,7 +690,7 @@ int mv_gated_group_norm(const void *y, int64_t y_stride, const void *z, int64_t 
                         void *stream);
 
 /* ---- K16 — gated delta rule (heads with a state S of `n` key channels x `p` columns; `groups` of keys and queries).  Per token
- *     S <- g S;   u = beta (v - S^T k);   S <- S + k u^T;   o = S^T q
+ *     S' = g S_old,   u = beta (v - k S'),   S_new = S' + (k outer u),   o = q S_new   (vectors are rows)
  * with unit k and q (q also times q_scale), beta = sigmoid(raw beta), g = exp(-exp(a_log) softplus(a + dt_bias)), one per head or
  * (channel_decay) per head and key channel.  State slots as in K15: state fp32 [2][slots][heads][n][p].  Channels of x: v [heads * p] |
  * k [groups * n] | q [groups * n] at offsets 0, k_off, q_off; p % 16 == 0, n % 32 == 0 (padding holds zeros). */

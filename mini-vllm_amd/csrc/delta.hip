@@ -88,14 +88,14 @@ __global__ void __launch_bounds__(256) delta_scan_kernel(MvDeltaArgs p) {
 
 // ---- one token: workgroup = (head, sequence).  The state [n][p] is requested first (up to kStepAhead 16-byte pieces per thread)
 // and stays in registers; under that, the convolution of the head's v and of its group's k and q.  With S the decayed state,
-//     u = beta (v - S^T k),   o = S^T q + (k . q) u,   S <- S + k u^T
+//     u = beta (v - k S),   o = q S + (k . q) u,   S += k outer u            (vectors are rows)
 // so both reductions over the rows of S happen in one pass.  k and q enter as they are, their lengths as factors of the sums.
 constexpr int kStepAhead = 16;
 
 template <typename Tag, int THREADS>
 __global__ void __launch_bounds__(THREADS) delta_step_kernel(MvDeltaArgs p) {
   typedef typename elem<Tag>::T T;
-  extern __shared__ float lds[];   // v [p] | k [n] | q [n] | decay [n] | u [p] | o [p] | partial S^T k, S^T q [rows][p] each
+  extern __shared__ float lds[];   // v [p] | k [n] | q [n] | decay [n] | u [p] | o [p] | partial k S, q S [rows][p] each
   __shared__ float sums[3];        // |k|^2, |q|^2, k . q
   const int head = blockIdx.x, s = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int before = p.context_lens[s] - 1, slot = p.state_slots[s], back = p.taps - 1;

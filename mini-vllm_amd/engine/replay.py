@@ -69,8 +69,8 @@ class StepReplayer:
 
 
 def main(argv: list[str] | None = None) -> int:
-    ap = argparse.ArgumentParser(prog="trace_run", description="Feed given token ids through a model, step by step (one JSON "
-                                 "object a line on standard input), and write the logits asked for.")
+    ap = argparse.ArgumentParser(prog="trace_run", description="Replay steps of token ids (standard input, one JSON object "
+                                 "each) through a model and write the logits asked for.")
     ap.add_argument("--model", required=True, help="folder with config.json and model.safetensors")
     ap.add_argument("--dtype", choices=["bfloat16", "float32"], required=True)
     ap.add_argument("--out", required=True, help="folder for <step>.f32 (little-endian floats, [wanted, vocab])")

@@ -1,5 +1,5 @@
 """Gated delta rule on the gfx950 kernels of csrc/delta*.hip: per head a state S of key channels x columns,
-    S <- g S;   u = beta (v - S^T k);   S <- S + k u^T;   o = S^T q        (k and q unit vectors, fp32 throughout)
+    S' = g S_old,   u = beta (v - k S'),   S_new = S' + (k outer u),   o = q S_new     (rows; k and q of length 1; fp32 throughout)
 then o's RMS norm per head, a weight shared by the heads, and a gate.
 
     prompts: causal convolution + silu of [v | k | q], the recurrence in chunks, norm and gate

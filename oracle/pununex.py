@@ -74,7 +74,7 @@ def unit(x):
 
 def delta_scan(q, k, v, beta, decay, state=None):
     """q / k [T, H, D], v [T, H, V], beta [T, H], decay [T, H, D] (a factor per key channel) -> o [T, H, V], token by token:
-    S <- decay S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q."""
+    S' = decay S_old,  u = beta (v - k S'),  S_new = S' + (k outer u),  o = q S_new, vectors as rows."""
     s = torch.zeros(k.shape[1], k.shape[2], v.shape[2], dtype=v.dtype) if state is None else state.clone()
     o = torch.empty_like(v)
     for i in range(v.shape[0]):
