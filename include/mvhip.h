@@ -55,13 +55,17 @@ enum {
  *   window / keep_first: window > 0: a query at position i sees key j <= i if i - j < window or j < keep_first (not with chunk).
  *   softcap: > 0: scores s become softcap * tanh(s / softcap).
  *   out_scale: multiplies the output (0: 1).
- *   sink: [n_heads] of dtype: the softmax denominator of head h has one more term, exp(sink[h]) (not scaled, not capped). */
+ *   sink: [n_heads] of dtype: the softmax denominator of head h has one more term, exp(sink[h]) (not scaled, not capped).
+ *   gate / gate_stride: rows of [n_heads * head_dim] of dtype, one per query: the output is multiplied by sigmoid(gate) (NULL: nothing).
+ *   unit_norm: (rotating entry points) q and k are divided by their root mean square over norm_dim behind the rotation, no weight. */
 typedef struct MvAttnOpts {
   int rot_pairs, interleaved, chunk, norm_dim;
   int64_t out_stride;
   int window, keep_first;
   float softcap, out_scale;
-  const void *sink;
+  const void *sink, *gate;
+  int64_t gate_stride;
+  int unit_norm, reserved;
 } MvAttnOpts;
 
 int mv_version(void);
@@ -307,7 +311,7 @@ int mv_gelu_and_mul(const void *x, int64_t x_stride, void *out, int64_t out_stri
 
 /* Activation of a gated projection, act(gate, up) (HOST struct, read during the call).  MV_ACT_CLAMPED: g = min(gate, limit),
  * u = clamp(up, -limit, limit), g * sigmoid(alpha * g) * (u + 1).  MV_ACT_RELU: max(gate, 0) * up. */
-enum { MV_ACT_SILU = 0, MV_ACT_GELU = 1, MV_ACT_CLAMPED = 2, MV_ACT_RELU = 3 };
+enum { MV_ACT_SILU = 0, MV_ACT_GELU = 1, MV_ACT_CLAMPED = 2, MV_ACT_RELU = 3, MV_ACT_GELU_ERF = 4 /* plain projections only */ };
 typedef struct MvGateAct {
   int kind;
   float limit, alpha;
@@ -315,6 +319,12 @@ typedef struct MvGateAct {
 /* out[r, c] = act(x[r, c], x[r, cols + c]), fp32 inside */
 int mv_act_and_mul(const void *x, int64_t x_stride, void *out, int64_t out_stride, int rows, int cols,
                    const MvGateAct *act, int dtype, void *stream);
+
+/* out = 0.5 x (1 + erf(x / sqrt(2))), fp32 inside, one rounding; out may be x.  (Decode-sized projections take it into their
+ * epilogue: MV_LINEAR_GELU_ERF in the `shape` of mv_linear_small_m_packed / mv_linear_small_m and in the `cfg` of mv_linear_mid_m,
+ * behind the bias and before the rounding.) */
+enum { MV_LINEAR_GELU_ERF = 1 << 18 };
+int mv_gelu_erf(const void *x, int64_t x_stride, void *out, int64_t out_stride, int rows, int cols, int dtype, void *stream);
 
 /* K13 — one edge of a residual stream kept in fp32.  Per row, with the stream x [rows][cols] (dense fp32, in place):
  *     b = x, or (embed_mode 1) nothing;   y' = y, or (y_norm_w) y / sqrt(mean(y^2) + eps) * y_norm_w;   y' *= y_scale * y_mult
@@ -726,25 +736,77 @@ int mv_head_norm_gate(const void *y, int64_t y_stride, const void *gate, int64_t
 /* ---- K17 — mixture of experts.  A pair = (token t, choice c) at index t * top + c.
  * Router: s = softmax(W x) over `outputs` (logits in fp32), choice scores s + correction; only outputs of the `keep` groups (of `groups`
  * equal runs) with the largest choice score can be chosen; the `top` with the largest choice scores get weights s / (sum of the chosen
- * s + 1e-20) * scale.  w [outputs][k] dense.  -> ids, weights [rows][top] */
+ * s + 1e-20) * scale.  correction NULL: none.  w [outputs][k] dense.  -> ids, weights [rows][top]
+ * flags: MV_ROUTE_SIGMOID: s = sigmoid(W x) instead; MV_ROUTE_RAW: weights s * scale, not divided by their sum */
+enum { MV_ROUTE_SIGMOID = 1, MV_ROUTE_RAW = 2 };
 int mv_moe_route(const void *x, int64_t x_stride, const void *w, const void *correction, int32_t *ids, float *weights, int rows, int k,
-                 int outputs, int top, int groups, int keep, float scale, int dtype, void *stream);
+                 int outputs, int top, int groups, int keep, float scale, int flags, int dtype, void *stream);
 /* Sorts the pairs by expert: rows[pair] = its place (-1: id >= experts, no product), tokens[place] = its token; tiles
- * [max_tiles][3] = expert (-1: none), first place, places (at most tile_m).  max_tiles >= pairs / tile_m + experts */
+ * [max_tiles][3] = expert (-1: none), first place, places (at most tile_m).  max_tiles >= pairs / tile_m + experts.
+ * weights [pairs] (may be NULL): also weights_out[place] = weights[pair] */
 int mv_moe_group(const int32_t *ids, int pairs, int top, int experts, int tile_m, int max_tiles, int32_t *rows, int32_t *tokens,
-                 int32_t *tiles, void *stream);
+                 int32_t *tiles, const float *weights, float *weights_out, void *stream);
 /* out[place] = W[expert] x[tokens[place]] (tokens NULL: x[place]), W [experts][n][k]; act: W [experts][2][n][k], out = act(gate, up).
  * 16-bit: W packed per expert (mv_pack_weight of all rows), tile_m 16, 32, 64, 128 or 256; fp32: W as it is, tile_m 16.  n % 16 == 0,
- * k % 64 == 0. */
+ * k % 64 == 0.  in_scale [places] (may be NULL): the input x is multiplied by it (the sums are, in fp32, ahead of the activation). */
 typedef struct MvMoeLinearArgs {
   const void *x, *w;
   void *out;
   const int32_t *tokens, *tiles;
   const MvGateAct *act;
+  const float *in_scale;
   int64_t x_stride, out_stride;
   int max_tiles, tile_m, n, k;
 } MvMoeLinearArgs;
 int mv_moe_linear(const MvMoeLinearArgs *args, int dtype, void *stream);
+
+/* ---- K18 — one edge of several residual streams (hyper-connections), kept in fp32: x [rows][streams][cols].  Per row:
+ *     x'_j = sum_i mix[i][j] x_i + out_w[j] y      (embed given instead: x'_j = embed[ids[row]] for every j)
+ *     u = sum_j in_w[j] x'_j (in_w NULL: 1),   h = u / sqrt(mean(u^2) + eps) * norm_w
+ *     out = h, or (shift) h + (h_before - h) * shift with the h of the sequence's token before (zeros before the first)
+ * y: rows of dtype at y_stride, or (y_splits > 0) fp32 partial sums [y_splits][rows][cols]; plus the sum over k < moe_top of
+ * moe_w[row][k] * moe_out[moe_rows[row][k]] (moe_w NULL: 1; a row index < 0: nothing).  x_out (NULL: not kept) gets x'; it may be x
+ * unless shift is given with cu_q.  Means are over cols_true <= cols columns; the others hold zeros.
+ * The h of a step's last token is kept in prev fp32 [2][slots][cols], half = number of tokens so far & 1, at state_slots[sequence]
+ * (< 0: nothing is kept, the token before counts as zeros).  Sequences: rows cu_q[s] .. cu_q[s + 1]; cu_q NULL: one row each.  Rows at
+ * position < 0: padding.  streams <= 8; all weights are of dtype. */
+typedef struct MvStreamArgs {
+  const float *x;
+  float *x_out;
+  const void *y, *mix, *out_w, *embed;
+  const int64_t *ids;
+  const void *in_w, *norm_w, *shift;
+  void *out;
+  const void *moe_out;
+  const int32_t *moe_rows;
+  const float *moe_w;
+  float *prev;
+  const int64_t *positions;
+  const int32_t *state_slots, *cu_q;
+  int64_t y_stride, out_stride, vocab, slots;
+  int streams, y_splits, moe_top, n_seqs;
+  float eps;
+  int reserved;
+} MvStreamArgs;
+int mv_stream_update(const MvStreamArgs *args, int rows, int cols, int cols_true, int dtype, void *stream);
+
+/* ---- K19 — gated running mean over `n` channels, from raw projections z, u, g (rows of dtype at one stride):
+ *     S_t = (1 - sigmoid(z)) S_(t-1) + sigmoid(z) c(u),   c(u) = u + 1/2 for u >= 0, else sigmoid(u);   out = S_t silu(g)
+ * State slots as in K15: state fp32 [2][slots][n].  Prompts run in chunks (workspace: mv_gru_prefill_workspace_bytes()). */
+typedef struct MvGruArgs {
+  const void *z, *u, *g;
+  float *state;
+  const int32_t *state_slots;       /* [n_seqs] */
+  const int32_t *cu_q, *cu_k;       /* prefill: token ranges; tokens before the step = key length - query length */
+  const int32_t *context_lens;      /* step: tokens including this one */
+  void *out;
+  float *workspace;
+  int64_t stride, out_stride, slots, ws_bytes;
+  int n_seqs, max_q, total_q, n;
+} MvGruArgs;
+size_t mv_gru_prefill_workspace_bytes(int n_seqs, int total_q, int max_q, int n);
+int mv_gru_prefill(const MvGruArgs *args, int dtype, void *stream);
+int mv_gru_step(const MvGruArgs *args, int dtype, void *stream);
 
 #ifdef __cplusplus
 }

@@ -138,6 +138,25 @@ __device__ __forceinline__ float gelu_tanh(float z) {
   return z / (1.0f + expf(-u2));
 }
 
+// 0.5 z (1 + erf(z / sqrt(2))).  16-bit operands: erfc by Abramowitz & Stegun 7.1.26 (absolute error 1.5e-7), hardware exponential
+// and reciprocal; max(z, 0) - |z| / 2 erfc(|z| / sqrt(2)) holds on both sides
+template <typename Tag>
+__device__ __forceinline__ float gelu_erf(float z) {
+  if constexpr (__is_same(Tag, f32_tag)) {
+    return 0.5f * z * (1.0f + erff(z * 0.7071067811865476f));
+  } else {
+    const float a = fabsf(z), t = __builtin_amdgcn_rcpf(fmaf(0.3275911f * 0.7071067811865476f, a, 1.0f));
+    const float poly = t * fmaf(t, fmaf(t, fmaf(t, fmaf(t, 1.061405429f, -1.453152027f), 1.421413741f), -0.284496736f), 0.254829592f);
+    return fmaxf(z, 0.f) - 0.5f * a * poly * __builtin_amdgcn_exp2f(-0.7213475204444817f * a * a);   // exp(-z^2 / 2)
+  }
+}
+// 16-bit operands: hardware exponential and reciprocal (1 ulp of fp32 each)
+template <typename Tag>
+__device__ __forceinline__ float sigmoid_of(float z) {
+  if constexpr (__is_same(Tag, f32_tag)) return 1.0f / (1.0f + expf(-z));
+  else return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z));
+}
+
 // clamped gate: g = min(gate, limit), u = clamp(up, -limit, limit): g sigmoid(alpha g) (u + 1)
 __device__ __forceinline__ float clamped_glu(float gate, float up, float limit, float alpha) {
   const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
@@ -227,18 +246,28 @@ struct AttnMask {
   int window = 0, keep_first = 0;   // window > 0: key j of position i if i - j < window or j < keep_first
   float softcap = 0.f, out_scale = 1.f;
   const void *sink = nullptr;       // [heads] of dtype: one more term of the denominator
+  const void *gate = nullptr;       // a row of [heads * D] per query: the output is multiplied by its sigmoid
+  int64_t gate_stride = 0;
 };
+// what an output element is multiplied by
+template <typename Tag>
+__device__ __forceinline__ float attn_factor(const AttnMask &m, int64_t row, int col) {
+  if (!m.gate) return m.out_scale;
+  return m.out_scale * sigmoid_of<Tag>(elem<Tag>::ld(((const typename elem<Tag>::T *)m.gate)[row * m.gate_stride + col]));
+}
 static inline AttnMask mv_attn_mask(const MvAttnOpts *o) {
   AttnMask m;
   if (o) {
     m.window = o->window, m.keep_first = o->window > 0 ? o->keep_first : 0, m.softcap = o->softcap, m.sink = o->sink;
     if (o->out_scale != 0.f) m.out_scale = o->out_scale;
+    m.gate = o->gate, m.gate_stride = o->gate_stride;
   }
   return m;
 }
 static inline int mv_check_mask(const MvAttnOpts *o) {
   if (!o) return MV_OK;
   if (o->chunk < 0 || o->window < 0 || o->keep_first < 0 || (o->chunk > 0 && o->window > 0)) return MV_E_SHAPE;
+  if (o->gate && (!mv_aligned16(o->gate) || (o->gate_stride & 7))) return MV_E_ALIGN;
   return o->softcap < 0.f ? MV_E_RANGE : MV_OK;
 }
 // most keys that one query reads, in whole units; 0 = no bound

@@ -56,7 +56,7 @@ struct MidParams {
   int kb_per_split;   // 64-element k-blocks per K split (blockIdx.y)
   int krot;           // rotate the K loop start per workgroup
   int ablate;         // bench only: bit 0 = no x DMA, bit 1 = no W DMA (the LDS slots keep whatever they hold)
-  MvGateAct act;      // GATED
+  MvGateAct act;      // GATED; EPI_PLAIN: MV_ACT_GELU_ERF or nothing
 };
 
 template <int N>
@@ -355,6 +355,10 @@ __global__ void __launch_bounds__((WM * WN + NLX + NLW) * 64) linear_mid_m_kerne
 #pragma unroll
               for (int e = 0; e < 4; ++e) o[e] += elem<Tag>::ld(bp[e]);
             }
+            if (p.act.kind == MV_ACT_GELU_ERF) {
+#pragma unroll
+              for (int e = 0; e < 4; ++e) o[e] = gelu_erf<Tag>(o[e]);
+            }
             u32x2 pk;
             pk[0] = (uint32_t)elem<Tag>::st(o[0]) | ((uint32_t)elem<Tag>::st(o[1]) << 16);
             pk[1] = (uint32_t)elem<Tag>::st(o[2]) | ((uint32_t)elem<Tag>::st(o[3]) << 16);
@@ -524,6 +528,8 @@ extern "C" int mv_linear_mid_m(const void *x, int64_t x_stride, const void *w_pa
   if (m == 0 || n == 0) return MV_OK;
   if (int e = check(x, x_stride, w_packed, out, out_stride, m, n, k, dtype)) return e;
   if (bias && (((uintptr_t)bias) & 7u)) return MV_E_ALIGN;
+  const MvGateAct act = {(cfg & MV_LINEAR_GELU_ERF) ? MV_ACT_GELU_ERF : MV_ACT_SILU, 0.f, 0.f};
+  cfg &= ~MV_LINEAR_GELU_ERF;
   int flags = cfg / 100;          // bench only: +100 the DMA ring without the arithmetic (out untouched), +200 K rotation,
   cfg %= 100;                     // +400 no x DMA, +800 no W DMA (results are garbage: timing ablations)
   if (cfg < 0 || cfg >= kNumCfgs || flags > 63) return MV_E_RANGE;   // +1600: clock stamps into `bias`; +3200: no output stores (bench only)
@@ -533,7 +539,7 @@ extern "C" int mv_linear_mid_m(const void *x, int64_t x_stride, const void *w_pa
   if (flags) return MV_E_RANGE;
 #endif
   if (cfg == 0) cfg = auto_cfg(m, n, k, false);
-  MidParams p{x, w_packed, bias, out, x_stride, out_stride, m, n, k, 0, 0, 0, (flags & 2) ? 1 : 0, flags >> 2, {}};
+  MidParams p{x, w_packed, bias, out, x_stride, out_stride, m, n, k, 0, 0, 0, (flags & 2) ? 1 : 0, flags >> 2, act};
   if ((flags & 16) && !bias) return MV_E_NULLPTR;
   if (flags & 1)
     return dtype == MV_BF16 ? launch_cfg<bf16_tag, EPI_INGEST>(p, cfg, 1, (hipStream_t)stream) : MV_E_DTYPE;

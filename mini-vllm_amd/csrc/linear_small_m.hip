@@ -43,7 +43,7 @@ struct LinearParams {
   void *nres_out = nullptr;
   int64_t nres_stride = 0, nres_out_stride = 0;
   float eps = 0.f;
-  MvGateAct act = {MV_ACT_SILU, 0.f, 0.f};   // GATED
+  MvGateAct act = {MV_ACT_SILU, 0.f, 0.f};   // GATED; else MV_ACT_GELU_ERF or nothing
   int norm_threads = 0;  // block size of the rmsnorm_kernel launch this prologue re-enacts
 };
 
@@ -356,6 +356,10 @@ linear_small_m_kernel(LinearParams p) {
 #pragma unroll
         for (int i = 0; i < 4; ++i) o[i] += elem<Tag>::ld(bp[i]);
       }
+      if (!GATED && p.act.kind == MV_ACT_GELU_ERF) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) o[i] = gelu_erf<Tag>(o[i]);
+      }
       u32x2 pk;
       pk[0] = (uint32_t)elem<Tag>::st(o[0]) | ((uint32_t)elem<Tag>::st(o[1]) << 16);
       pk[1] = (uint32_t)elem<Tag>::st(o[2]) | ((uint32_t)elem<Tag>::st(o[3]) << 16);
@@ -406,6 +410,7 @@ static void norm_block(int cols, int *threads, int *per_thread) {
 template <bool GATED, bool PACKED = false, bool NORM = false>
 int run(LinearParams p, int dtype, int shape, hipStream_t st) {
   const bool groups = PACKED && !GATED && !NORM && (shape & MV_LINEAR_ROW_GROUPS) && p.M > 16;
+  if (!GATED && !NORM && (shape & MV_LINEAR_GELU_ERF)) p.act.kind = MV_ACT_GELU_ERF;
   const int m = groups ? 16 : p.M, n = p.N, mt = (m + 15) / 16, steps = p.K / 32;
   int rpw = GATED ? (m > 2 && n >= 16384 ? 2 : 1) : (m <= 2 ? 1 : (n >= 65536 ? 4 : (n >= 8192 ? 2 : 1)));
   // (on the packed copy 4 row tiles per wave never measured fastest, nor 2 + 2 tiles for the gated form:

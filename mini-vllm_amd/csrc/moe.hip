@@ -13,7 +13,7 @@ struct RouteParams {
   int32_t *ids;
   float *weights;
   int64_t x_stride;
-  int rows, k, outputs, top, groups, keep;
+  int rows, k, outputs, top, groups, keep, flags;
   float scale;
 };
 constexpr int kRouteTokens = 16, kRouteWaves = 8, kRouteTiles = 4;   // kRouteTiles: tiles of 16 outputs at a time
@@ -83,15 +83,18 @@ __global__ void __launch_bounds__(kRouteWaves * 64) moe_route_kernel(RouteParams
   for (int t = wave; t < kRouteTokens; t += kRouteWaves) {
     if (m0 + t >= p.rows) break;   // (uniform in the wave; no barrier below)
     float *s = sc + t * R, *c = ch + t * R;
+    const bool sigmoid = p.flags & MV_ROUTE_SIGMOID;
     float mx = -INFINITY, sum = 0.f;
-    for (int i = lane; i < R; i += 64) mx = fmaxf(mx, s[i]);
-    mx = wave_max(mx);
-    for (int i = lane; i < R; i += 64) sum += expf(s[i] - mx);
-    sum = wave_sum(sum);
+    if (!sigmoid) {
+      for (int i = lane; i < R; i += 64) mx = fmaxf(mx, s[i]);
+      mx = wave_max(mx);
+      for (int i = lane; i < R; i += 64) sum += expf(s[i] - mx);
+      sum = wave_sum(sum);
+    }
     for (int i = lane; i < R; i += 64) {
-      const float v = expf(s[i] - mx) / sum;
+      const float v = sigmoid ? 1.0f / (1.0f + expf(-s[i])) : expf(s[i] - mx) / sum;
       s[i] = v;
-      c[i] = v + elem<Tag>::ld(((const T *)p.correction)[i]);
+      c[i] = p.correction ? v + elem<Tag>::ld(((const T *)p.correction)[i]) : v;
     }
     __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
     if (p.keep < p.groups) {   // lane = group (at most 64)
@@ -127,7 +130,7 @@ __global__ void __launch_bounds__(kRouteWaves * 64) moe_route_kernel(RouteParams
     }
     if (lane < p.top) {
       p.ids[(int64_t)(m0 + t) * p.top + lane] = mine;
-      p.weights[(int64_t)(m0 + t) * p.top + lane] = weight / (total + 1e-20f) * p.scale;
+      p.weights[(int64_t)(m0 + t) * p.top + lane] = (p.flags & MV_ROUTE_RAW ? weight : weight / (total + 1e-20f)) * p.scale;
     }
   }
 }
@@ -137,7 +140,8 @@ __global__ void __launch_bounds__(kRouteWaves * 64) moe_route_kernel(RouteParams
 constexpr int kGroupThreads = 1024, kGroupWaves = kGroupThreads / 64;
 
 __global__ void __launch_bounds__(kGroupThreads) moe_group_kernel(const int32_t *ids, int pairs, int top, int experts, int tile_m,
-                                                                  int max_tiles, int32_t *rows, int32_t *tokens, int32_t *tiles) {
+                                                                  int max_tiles, int32_t *rows, int32_t *tokens, int32_t *tiles,
+                                                                  const float *weights, float *weights_out) {
   __shared__ int less[kGroupWaves], equal[kGroupWaves];
   const int e = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int per = (pairs + kGroupWaves * 64 - 1) / (kGroupWaves * 64) * 64, lo = wave * per, hi = min(pairs, lo + per);
@@ -162,6 +166,7 @@ __global__ void __launch_bounds__(kGroupThreads) moe_group_kernel(const int32_t 
     if (v == e) {
       const int place = at + __popcll(mask & ((1ull << lane) - 1));
       rows[i] = place, tokens[place] = i / top;
+      if (weights) weights_out[place] = weights[i];
     }
     if (e == 0 && v >= experts) rows[i] = -1;
     at += __popcll(mask);
@@ -179,10 +184,13 @@ struct MoeLinear {
   const void *x, *w;
   void *out;
   const int32_t *tokens, *tiles;   // tokens NULL: row = place
+  const float *in_scale;           // by place; NULL: 1
   int64_t x_stride, out_stride, w_expert;   // w_expert: elements between two experts' weights
   int n, k;                        // outputs (gated: of the product with up), inputs
   MvGateAct act;
 };
+
+__device__ __forceinline__ float in_scale_of(const MoeLinear &p, int place) { return p.in_scale ? p.in_scale[place] : 1.0f; }
 
 // few rows per expert: TM tiles of 16 rows, TN of 16 outputs; the waves split the inputs, weight fragments come straight from
 // memory in the order they are stored (1 KiB per instruction)
@@ -237,13 +245,14 @@ __global__ void __launch_bounds__(256) moe_small_kernel(MoeLinear p) {
   for (int t = wave; t < TN * TM; t += 4) {
     const int j = t / TM, i = t - j * TM, row = i * 16 + r16, n0 = ((int)blockIdx.x * TN + j) * 16;
     if (row >= live || n0 >= p.n) continue;
+    const float sc = in_scale_of(p, m0 + row);
     f32x4 o;
     if constexpr (GATED) {
-      const f32x4 gate = total(2 * j * TM + i), up = total((2 * j + 1) * TM + i);
+      const f32x4 gate = total(2 * j * TM + i) * sc, up = total((2 * j + 1) * TM + i) * sc;
 #pragma unroll
       for (int q = 0; q < 4; ++q) o[q] = gated_act<Tag>(gate[q], up[q], p.act);
     } else {
-      o = total(t);
+      o = total(t) * sc;
     }
     *(u32x2 *)((T *)p.out + (int64_t)(m0 + row) * p.out_stride + n0 + g * 4) = pack_quad<Tag>(o);
   }
@@ -322,6 +331,7 @@ __global__ void __launch_bounds__(256, 2) moe_tile_kernel(MoeLinear p) {
   for (int i = 0; i < WM; ++i) {
     const int row = (wm * WM + i) * 16 + r16;
     if (row >= live) continue;
+    const float sc = in_scale_of(p, m0 + row);
     T *out = (T *)p.out + (int64_t)(m0 + row) * p.out_stride + g * 4;
 #pragma unroll
     for (int j = 0; j < (GATED ? WN / 2 : WN); ++j) {
@@ -330,9 +340,9 @@ __global__ void __launch_bounds__(256, 2) moe_tile_kernel(MoeLinear p) {
       f32x4 o;
       if constexpr (GATED) {
 #pragma unroll
-        for (int q = 0; q < 4; ++q) o[q] = gated_act<Tag>(acc[2 * j][i][q], acc[2 * j + 1][i][q], p.act);
+        for (int q = 0; q < 4; ++q) o[q] = gated_act<Tag>(acc[2 * j][i][q] * sc, acc[2 * j + 1][i][q] * sc, p.act);
       } else {
-        o = acc[j][i];
+        o = acc[j][i] * sc;
       }
       *(u32x2 *)(out + nt * 16) = pack_quad<Tag>(o);
     }
@@ -411,6 +421,7 @@ __global__ void __launch_bounds__(512, 1) moe_wide_kernel(MoeLinear p, int nx, i
   for (int i = 0; i < WM; ++i) {
     const int row = (wm * WM + i) * 16 + r16;
     if (row >= live) continue;
+    const float sc = in_scale_of(p, m0 + row);
     T *out = (T *)p.out + (int64_t)(m0 + row) * p.out_stride + g * 4;
 #pragma unroll
     for (int j = 0; j < (GATED ? WN / 2 : WN); ++j) {
@@ -419,9 +430,9 @@ __global__ void __launch_bounds__(512, 1) moe_wide_kernel(MoeLinear p, int nx, i
       f32x4 o;
       if constexpr (GATED) {
 #pragma unroll
-        for (int q = 0; q < 4; ++q) o[q] = gated_act<Tag>(acc[2 * j][i][q], acc[2 * j + 1][i][q], p.act);
+        for (int q = 0; q < 4; ++q) o[q] = gated_act<Tag>(acc[2 * j][i][q] * sc, acc[2 * j + 1][i][q] * sc, p.act);
       } else {
-        o = acc[j][i];
+        o = acc[j][i] * sc;
       }
       *(u32x2 *)(out + nt * 16) = pack_quad<Tag>(o);
     }
@@ -459,8 +470,10 @@ __global__ void __launch_bounds__(256) moe_f32_kernel(MoeLinear p) {
   }
 #pragma unroll
   for (int i = 0; i < 4; ++i)
-    if (r + 4 * i < live && n0 + c < p.n)
-      ((float *)p.out)[(int64_t)(m0 + r + 4 * i) * p.out_stride + n0 + c] = GATED ? gated_act<f32_tag>(acc[i], up[i], p.act) : acc[i];
+    if (r + 4 * i < live && n0 + c < p.n) {
+      const float sc = in_scale_of(p, m0 + r + 4 * i);
+      ((float *)p.out)[(int64_t)(m0 + r + 4 * i) * p.out_stride + n0 + c] = GATED ? gated_act<f32_tag>(acc[i] * sc, up[i] * sc, p.act) : acc[i] * sc;
+    }
 }
 
 template <typename Tag, bool GATED>
@@ -489,14 +502,15 @@ int launch_linear(const MoeLinear &p, int tile_m, int max_tiles, hipStream_t st)
 }  // namespace
 
 extern "C" int mv_moe_route(const void *x, int64_t x_stride, const void *w, const void *correction, int32_t *ids, float *weights,
-                            int rows, int k, int outputs, int top, int groups, int keep, float scale, int dtype, void *stream) {
+                            int rows, int k, int outputs, int top, int groups, int keep, float scale, int flags, int dtype, void *stream) {
   if (rows == 0) return MV_OK;
-  if (!x || !w || !correction || !ids || !weights) return MV_E_NULLPTR;
+  if (!x || !w || !ids || !weights) return MV_E_NULLPTR;
+  if (flags & ~(MV_ROUTE_SIGMOID | MV_ROUTE_RAW)) return MV_E_RANGE;
   if (rows < 0 || k <= 0 || (k & 31) || outputs <= 0 || outputs > 512 || top <= 0 || top > 64 || top > outputs || groups <= 0 ||
       groups > 64 || outputs % groups || keep <= 0 || keep > groups || (int64_t)outputs / groups * keep < top || x_stride < k)
     return MV_E_SHAPE;
   if (!mv_aligned16(x) || !mv_aligned16(w) || x_stride % (dtype == MV_F32 ? 4 : 8)) return MV_E_ALIGN;
-  const RouteParams p{x, w, correction, ids, weights, x_stride, rows, k, outputs, top, groups, keep, scale};
+  const RouteParams p{x, w, correction, ids, weights, x_stride, rows, k, outputs, top, groups, keep, flags, scale};
   const size_t lds = (size_t)2 * kRouteTokens * outputs * 4 + (dtype == MV_F32 ? 0 : kRouteWaves * kRouteTiles * 1024);
   const dim3 grid((rows + kRouteTokens - 1) / kRouteTokens);
   MV_DISPATCH_DTYPE(dtype, {
@@ -508,12 +522,12 @@ extern "C" int mv_moe_route(const void *x, int64_t x_stride, const void *w, cons
 }
 
 extern "C" int mv_moe_group(const int32_t *ids, int pairs, int top, int experts, int tile_m, int max_tiles, int32_t *rows,
-                            int32_t *tokens, int32_t *tiles, void *stream) {
+                            int32_t *tokens, int32_t *tiles, const float *weights, float *weights_out, void *stream) {
   if (pairs == 0) return MV_OK;
-  if (!ids || !rows || !tokens || !tiles) return MV_E_NULLPTR;
+  if (!ids || !rows || !tokens || !tiles || (weights && !weights_out)) return MV_E_NULLPTR;
   if (pairs < 0 || top <= 0 || experts <= 0 || experts > 65535 || tile_m <= 0 || max_tiles < pairs / tile_m + experts) return MV_E_SHAPE;
   hipLaunchKernelGGL(moe_group_kernel, dim3(experts), dim3(kGroupThreads), 0, (hipStream_t)stream, ids, pairs, top, experts, tile_m,
-                     max_tiles, rows, tokens, tiles);
+                     max_tiles, rows, tokens, tiles, weights, weights_out);
   MV_LAUNCH_CHECK();
   return MV_OK;
 }
@@ -526,7 +540,7 @@ extern "C" int mv_moe_linear(const MvMoeLinearArgs *a, int dtype, void *stream) 
     return MV_E_SHAPE;
   const int vec = dtype == MV_F32 ? 4 : 8;
   if (!mv_aligned16(a->x) || !mv_aligned16(a->w) || !mv_aligned16(a->out) || a->x_stride % vec || a->out_stride % vec) return MV_E_ALIGN;
-  MoeLinear p{a->x, a->w, a->out, a->tokens, a->tiles, a->x_stride, a->out_stride, (int64_t)a->n * a->k * (a->act ? 2 : 1), a->n, a->k, {}};
+  MoeLinear p{a->x, a->w, a->out, a->tokens, a->tiles, a->in_scale, a->x_stride, a->out_stride, (int64_t)a->n * a->k * (a->act ? 2 : 1), a->n, a->k, {}};
   if (a->act) {
     if (int e = mv_check_act(a->act)) return e;
     p.act = *a->act;

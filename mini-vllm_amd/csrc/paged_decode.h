@@ -39,6 +39,7 @@ struct DecodeParams {
   int chunk = 0;
   AttnMask mask;
   int norm_dim = 0;         // columns that the head norms are means over
+  int unit = 0;             // ROPE: q and k divided by their rms (no weight), one rounding behind the rotation
   int64_t out_stride = 0;   // elements between token rows of out; 0 = n_heads * D
 };
 
@@ -122,17 +123,20 @@ __device__ __forceinline__ void st2(uint16_t *p, uint16_t v) {
 template <typename Tag, int D>
 __device__ __forceinline__ u32x4 norm_rope_row(const u32x4 &raw, const typename elem<Tag>::T *nw, float eps, int norm_dim, int sub,
                                                const float (&cs)[elem<Tag>::VEC], const float (&sn)[elem<Tag>::VEC],
-                                               bool interleaved = false) {
+                                               bool interleaved = false, bool unit = false) {
   constexpr int VEC = elem<Tag>::VEC, LPT = D / VEC;
   static_assert(VEC == 8, "16-bit dtypes");
   float x[VEC];
   unpack8<Tag>(raw, x);
-  if (nw != nullptr) {
+  float rs = 1.0f;
+  if (nw != nullptr || unit) {
     float ss = 0.f;
 #pragma unroll
     for (int j = 0; j < VEC; ++j) ss = fmaf(x[j], x[j], ss);
     for (int off = 1; off < LPT; off <<= 1) ss += __shfl_xor(ss, off, 64);
-    const float rs = 1.0f / sqrtf(ss / (float)norm_dim + eps);
+    rs = 1.0f / sqrtf(ss / (float)norm_dim + eps);
+  }
+  if (nw != nullptr) {
     float w[VEC];
     const u32x4 wraw = *(const MV_AS1 u32x4 *)(nw + sub * VEC);
     unpack8<Tag>(wraw, w);
@@ -141,6 +145,10 @@ __device__ __forceinline__ u32x4 norm_rope_row(const u32x4 &raw, const typename 
   }
   float y[VEC];
   rot_apply<D, VEC>(x, cs, sn, sub, interleaved, y);
+  if (unit) {
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) y[j] = __fmul_rn(y[j], rs);
+  }
   return pack8<Tag>(y);
 }
 

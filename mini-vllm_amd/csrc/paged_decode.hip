@@ -190,6 +190,7 @@ extern "C" int mv_rope_paged_decode_ex(const void *q, int64_t q_stride_tok, cons
       (q_norm_w && !mv_aligned16(q_norm_w)) || (k_norm_w && !mv_aligned16(k_norm_w)))
     return MV_E_ALIGN;
   if (int e = mv_check_rot(opts, head_dim)) return e;
+  if ((q_norm_w || k_norm_w) && opts && opts->unit_norm) return MV_E_SHAPE;
   DecodePlan pl;
   if (!make_plan(batch, n_heads, n_kv_heads, head_dim, block_size, max_blocks, dtype, flags, opts, &pl))
     return MV_E_SHAPE;
@@ -271,6 +272,7 @@ int paged_decode_impl(const void *q, int64_t q_stride_tok, const void *k_cache,
   p.chunk = chunk;
   p.mask = mv_attn_mask(opts);
   p.norm_dim = opts && opts->norm_dim ? opts->norm_dim : head_dim;
+  p.unit = opts && opts->unit_norm;
   p.out_stride = out_stride;
   p.scale_log2 = scale * 1.4426950408889634f;
   p.ws_acc = nullptr;

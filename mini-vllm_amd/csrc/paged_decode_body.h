@@ -120,7 +120,7 @@ __device__ __forceinline__ void paged_decode_body(const DecodeParams &p, const i
     const bool il = p.interleaved != 0;
     rot_factors<D, VEC>(p.cos, p.sin, pos, pos_ok, sub, p.pairs, il, cs, sn);
 #pragma unroll
-    for (int g = 0; g < G; ++g) qraw[g] = norm_rope_row<Tag, D>(qraw[g], (const T *)p.q_norm_w, p.eps, p.norm_dim, sub, cs, sn, il);
+    for (int g = 0; g < G; ++g) qraw[g] = norm_rope_row<Tag, D>(qraw[g], (const T *)p.q_norm_w, p.eps, p.norm_dim, sub, cs, sn, il, p.unit);
     // the workgroup that will read the sequence's last token writes its K / V rows first (one wave; WIDE: its four
     // lane groups are the four kv heads, else lane group 0 has the workgroup's kv head)
     int64_t slot = p.slot_mapping ? (int64_t)p.slot_mapping[b] : -1;
@@ -129,7 +129,7 @@ __device__ __forceinline__ void paged_decode_body(const DecodeParams &p, const i
     if (write && slot >= 0 && u_last >= u_begin && u_last < u_end && wave == 0 && (WIDE || grp == 0)) {
       const u32x4 kraw = ld16<COH>((const T *)p.k_new + (int64_t)b * p.k_stride + (int64_t)hkv * D + sub * VEC);
       const u32x4 vraw = ld16<COH>((const T *)p.v_new + (int64_t)b * p.v_stride + (int64_t)hkv * D + sub * VEC);
-      const u32x4 krot = norm_rope_row<Tag, D>(kraw, (const T *)p.k_norm_w, p.eps, p.norm_dim, sub, cs, sn, il);
+      const u32x4 krot = norm_rope_row<Tag, D>(kraw, (const T *)p.k_norm_w, p.eps, p.norm_dim, sub, cs, sn, il, p.unit);
       *(MV_AS1 u32x4 *)((T *)p.k_cache + (slot * p.n_kv_heads + hkv) * D + sub * VEC) = krot;
       *(MV_AS1 u32x4 *)((T *)p.v_cache + (slot * p.n_kv_heads + hkv) * D + sub * VEC) = vraw;
       asm volatile("s_waitcnt vmcnt(0)" ::: "memory");   // the rows are in L2 before any wave of the workgroup asks
@@ -299,7 +299,7 @@ __device__ __forceinline__ void paged_decode_body(const DecodeParams &p, const i
     const int h = (hkv0 + hg) * p.g_total + chunk * G + g;
     const int64_t os = p.out_stride ? p.out_stride : (int64_t)p.n_heads * D;
     if (p.nsplit == 1) {
-      const float o = L > 0.f ? A / L * p.mask.out_scale : 0.f;
+      const float o = L > 0.f ? A / L * attn_factor<Tag>(p.mask, b, h * D + d) : 0.f;
       if constexpr (sizeof(T) == 2) st2<COH>((uint16_t *)p.out + (int64_t)b * os + h * D + d, elem<Tag>::st(o));
       else ((T *)p.out)[(int64_t)b * os + h * D + d] = elem<Tag>::st(o);
     } else {
@@ -331,11 +331,13 @@ struct ReduceLds {
   static constexpr int BYTES = FLOATS * 4;
 };
 
-// body for the 128-thread workgroup `bh` = (sequence, head); see paged_decode_body for `write`
+// body for the 128-thread workgroup `bh` = (sequence, head); see paged_decode_body for `write`; the head starts at column `gate_col` of
+// gate row `gate_row`
 template <typename Tag, int D, bool COH = false>
 __device__ __forceinline__ void paged_decode_reduce_body(const float *ws_acc, const float *ws_ml, typename elem<Tag>::T *out,
                                                          const int nsplit, const int64_t bh, const int tid, const bool write,
-                                                         float *lds, const float out_scale = 1.f) {
+                                                         float *lds, const AttnMask &mask = {}, const int64_t gate_row = 0,
+                                                         const int gate_col = 0) {
   constexpr int D4 = D / 4, NQ = 128 / D4;    // column pieces; split groups (4 at D = 128, 8 at D = 64)
   constexpr int kMax = 64, PER = kMax / NQ;   // kMaxSplits; rows per thread at most
   typedef MV_AS3 f32x4 lds_f4;
@@ -390,11 +392,11 @@ __device__ __forceinline__ void paged_decode_reduce_body(const float *ws_acc, co
     if constexpr (COH && sizeof(typename elem<Tag>::T) == 2) {
       uint32_t r[4];
 #pragma unroll
-      for (int e = 0; e < 4; ++e) r[e] = elem<Tag>::st(L > 0.f ? A[e] / L * out_scale : 0.f);
+      for (int e = 0; e < 4; ++e) r[e] = elem<Tag>::st(L > 0.f ? A[e] / L * attn_factor<Tag>(mask, gate_row, gate_col + 4 * c + e) : 0.f);
       st8<true>(o, u32x2{r[0] | (r[1] << 16), r[2] | (r[3] << 16)});
     } else {
 #pragma unroll
-      for (int e = 0; e < 4; ++e) o[e] = elem<Tag>::st(L > 0.f ? A[e] / L * out_scale : 0.f);
+      for (int e = 0; e < 4; ++e) o[e] = elem<Tag>::st(L > 0.f ? A[e] / L * attn_factor<Tag>(mask, gate_row, gate_col + 4 * c + e) : 0.f);
     }
   }
 }
@@ -403,11 +405,11 @@ template <typename Tag, int D>
 __global__ void __launch_bounds__(128) paged_decode_reduce_kernel(const float *__restrict__ ws_acc,
                                                                   const float *__restrict__ ws_ml,
                                                                   typename elem<Tag>::T *__restrict__ out,
-                                                                  int nsplit, int n_heads, int64_t out_stride, float out_scale) {
+                                                                  int nsplit, int n_heads, int64_t out_stride, AttnMask mask) {
   __shared__ __attribute__((aligned(16))) float lds[ReduceLds<D>::FLOATS];
   // (the body writes row bh of a dense [B * H, D] array: shift the base so that this row lands in its strided place)
   const int64_t b = blockIdx.x / n_heads;
   paged_decode_reduce_body<Tag, D>(ws_acc, ws_ml, out + b * (out_stride - (int64_t)n_heads * D), nsplit, blockIdx.x, threadIdx.x,
-                                   true, lds, out_scale);
+                                   true, lds, mask, b, (int)(blockIdx.x - b * n_heads) * D);
 }
 

@@ -58,7 +58,7 @@ int launch_d(const DecodeParams &p, const DecodePlan &pl, int batch, int dtype, 
     if (pl.nsplit > 1) {
       hipLaunchKernelGGL((paged_decode_reduce_kernel<Tag, D>), dim3(batch * p.n_heads), dim3(128), 0,
                          stream, p.ws_acc, p.ws_ml, (typename elem<Tag>::T *)p.out, pl.nsplit, p.n_heads, p.out_stride,
-                         p.mask.out_scale);
+                         p.mask);
       MV_LAUNCH_CHECK();
     }
     return MV_OK;
@@ -78,7 +78,7 @@ int launch_d(const DecodeParams &p, const DecodePlan &pl, int batch, int dtype, 
   if (pl.nsplit > 1) {
     hipLaunchKernelGGL((paged_decode_reduce_kernel<Tag, D>), dim3(batch * p.n_heads), dim3(128), 0,
                        stream, p.ws_acc, p.ws_ml, (typename elem<Tag>::T *)p.out, pl.nsplit, p.n_heads, p.out_stride,
-                         p.mask.out_scale);
+                         p.mask);
     MV_LAUNCH_CHECK();
   }
   return MV_OK;

@@ -104,7 +104,8 @@ __global__ void __launch_bounds__(256, KLDS ? 2 : 4) paged_decode_mfma_kernel(De
   if constexpr (ROPE) {
     const int64_t pos = p.positions[b];
     const bool pos_ok = pos >= 0 && pos < p.max_pos;
-    if (p.q_norm_w != nullptr) {
+    float unit[4] = {1.f, 1.f, 1.f, 1.f};   // by fragment (the sums differ in their order only)
+    if (p.q_norm_w != nullptr || p.unit) {
       // per-head RMSNorm of q, rope_qk_store_kernel's sum order: there a head row sits on 16 lanes "sub" (8 dims each,
       // fmaf chain over them) and the lane sums meet in a butterfly over sub ^ 1, 2, 4, 8.  Here sub = 4 s + quad:
       // sub ^ 1 / ^ 2 are the lanes quad ^ 1 / ^ 2 (16 / 32 lanes away), sub ^ 4 / ^ 8 are fragments s ^ 1 / s ^ 2
@@ -123,6 +124,10 @@ __global__ void __launch_bounds__(256, KLDS ? 2 : 4) paged_decode_mfma_kernel(De
 #pragma unroll
       for (int s = 0; s < 4; ++s) {
         const float rs = 1.0f / sqrtf(tot[s] / (float)p.norm_dim + p.eps);
+        if (p.unit) {
+          unit[s] = rs;
+          continue;
+        }
         float w[8];
         unpack8<Tag>(*reinterpret_cast<const u32x4 *>((const T *)p.q_norm_w + 32 * s + 8 * quad), w);
 #pragma unroll
@@ -140,6 +145,8 @@ __global__ void __launch_bounds__(256, KLDS ? 2 : 4) paged_decode_mfma_kernel(De
         unpack8<Tag>(qf[s], x);
         rot_factors<D, 8>(p.cos, p.sin, pos, pos_ok, 4 * s + quad, p.pairs, true, cs, sn);
         rot_apply<D, 8>(x, cs, sn, 4 * s + quad, true, y);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) y[j] = __fmul_rn(y[j], unit[s]);
         qf[s] = live ? pack8<Tag>(y) : u32x4{0u, 0u, 0u, 0u};
       }
     } else {
@@ -154,8 +161,8 @@ __global__ void __launch_bounds__(256, KLDS ? 2 : 4) paged_decode_mfma_kernel(De
       for (int j = 0; j < 8; ++j) {
         const int i = 32 * s + 8 * quad + j;
         const float c = pos_ok ? p.cos[pos * (D / 2) + i] : 1.0f, sn = pos_ok ? p.sin[pos * (D / 2) + i] : 0.0f;
-        ylo[j] = __fsub_rn(__fmul_rn(lo[j], c), __fmul_rn(hi[j], sn));
-        yhi[j] = __fadd_rn(__fmul_rn(hi[j], c), __fmul_rn(lo[j], sn));
+        ylo[j] = __fmul_rn(__fsub_rn(__fmul_rn(lo[j], c), __fmul_rn(hi[j], sn)), unit[s]);
+        yhi[j] = __fmul_rn(__fadd_rn(__fmul_rn(hi[j], c), __fmul_rn(lo[j], sn)), unit[s + 2]);
       }
       const bool live = i16 < g_live;   // (rows beyond the live heads stay zero)
       qf[s] = live ? pack8<Tag>(ylo) : u32x4{0u, 0u, 0u, 0u};
@@ -172,7 +179,7 @@ __global__ void __launch_bounds__(256, KLDS ? 2 : 4) paged_decode_mfma_kernel(De
       rot_factors<D, 8>(p.cos, p.sin, pos, pos_ok, sub, p.pairs, p.interleaved != 0, cs, sn);
       const u32x4 kraw = *reinterpret_cast<const u32x4 *>((const T *)p.k_new + (int64_t)b * p.k_stride + (int64_t)hkv * D + sub * 8);
       const u32x4 vraw = *reinterpret_cast<const u32x4 *>((const T *)p.v_new + (int64_t)b * p.v_stride + (int64_t)hkv * D + sub * 8);
-      const u32x4 krot = norm_rope_row<Tag, D>(kraw, (const T *)p.k_norm_w, p.eps, p.norm_dim, sub, cs, sn, p.interleaved != 0);
+      const u32x4 krot = norm_rope_row<Tag, D>(kraw, (const T *)p.k_norm_w, p.eps, p.norm_dim, sub, cs, sn, p.interleaved != 0, p.unit);
       *reinterpret_cast<u32x4 *>((T *)p.k_cache + (slot * p.n_kv_heads + hkv) * D + sub * 8) = krot;
       *reinterpret_cast<u32x4 *>((T *)p.v_cache + (slot * p.n_kv_heads + hkv) * D + sub * 8) = vraw;
       asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
@@ -349,7 +356,7 @@ __global__ void __launch_bounds__(256, KLDS ? 2 : 4) paged_decode_mfma_kernel(De
     const int h = h0 + g;
     if (p.nsplit == 1) {
       const int64_t os = p.out_stride ? p.out_stride : (int64_t)p.n_heads * D;
-      ((T *)p.out)[(int64_t)b * os + h * D + d] = elem<Tag>::st(L > 0.f ? A / L * p.mask.out_scale : 0.f);
+      ((T *)p.out)[(int64_t)b * os + h * D + d] = elem<Tag>::st(L > 0.f ? A / L * attn_factor<Tag>(p.mask, b, h * D + d) : 0.f);
     } else {
       const int64_t slot = ((int64_t)b * p.n_heads + h) * p.nsplit + split;
       p.ws_acc[slot * D + d] = A;

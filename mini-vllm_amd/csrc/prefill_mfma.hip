@@ -554,7 +554,16 @@ __global__ void __launch_bounds__(NW * 64, 2) prefill_mfma_kernel(PrefillParams 
       const u32x4 v = *reinterpret_cast<const u32x4 *>(stage + row * ROW_BYTES + ((cc ^ (row & (CH - 1))) << 4));
       if (row0 + row < sq && !(rescale_thr <= -2.f && lane != 0)) {   // (thr <= -2: bench ablation, timing only)
         T *op = (T *)p.out + (int64_t)(q0 + row0 + row) * p.out_stride + head * D;
-        *reinterpret_cast<u32x4 *>(op + 8 * cc) = v;
+        if (WINDOW && p.mask.gate) {
+          float o[8], g[8];
+          unpack8<Tag>(v, o);
+          unpack8<Tag>(*reinterpret_cast<const u32x4 *>((const T *)p.mask.gate + (q0 + row0 + row) * p.mask.gate_stride + head * D + 8 * cc), g);
+#pragma unroll
+          for (int j = 0; j < 8; ++j) o[j] *= sigmoid_of<Tag>(g[j]);
+          *reinterpret_cast<u32x4 *>(op + 8 * cc) = pack8<Tag>(o);
+        } else {
+          *reinterpret_cast<u32x4 *>(op + 8 * cc) = v;
+        }
       }
     }
   }
@@ -1012,7 +1021,7 @@ __global__ void __launch_bounds__(256, 1) prefill_mfma64_kernel(PrefillParams p,
 
 int mv_prefill_mfma_launch(const PrefillParams &p, int dtype, int variant, hipStream_t stream) {
   if ((p.head_dim != 64 && p.head_dim != 128) || (dtype != MV_BF16 && dtype != MV_F16)) return MV_E_SHAPE;
-  const bool general = p.mask.window > 0 || p.mask.softcap > 0.f || p.mask.sink || p.mask.out_scale != 1.f;
+  const bool general = p.mask.window > 0 || p.mask.softcap > 0.f || p.mask.sink || p.mask.gate || p.mask.out_scale != 1.f;
   if (p.chunk > 0 && (p.chunk < 32 || general)) return MV_E_SHAPE;   // (a handful of keys per query: the vector kernel's job)
   if (p.block_tables && (p.block_size % BN) != 0) return MV_E_SHAPE;  // a 64-key tile must sit in one block
   // 8 waves (256 query rows) per workgroup share a K/V tile where the sequences are long enough that the larger

@@ -115,7 +115,7 @@ __global__ void __launch_bounds__(256) prefill_simple_kernel(PrefillParams p) {
   for (int j = 0; j < VEC; ++j) {
     float a = acc[j] * f;
     for (int off = LPT; off < 64; off <<= 1) a += __shfl_xor(a, off, 64);
-    o[j] = ll > 0.f ? a / ll * p.mask.out_scale : 0.f;
+    o[j] = ll > 0.f ? a / ll * attn_factor<Tag>(p.mask, tok, h * D + sub * VEC + j) : 0.f;
   }
   if (grp == 0) {
     T *op = (T *)p.out + (int64_t)tok * p.out_stride + h * D + sub * VEC;

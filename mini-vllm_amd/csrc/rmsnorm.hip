@@ -283,6 +283,51 @@ static int act_and_mul(const void *x, int64_t x_stride, void *out, int64_t out_s
   return MV_OK;
 }
 
+template <typename Tag>
+__global__ void __launch_bounds__(256)
+gelu_erf_kernel(const typename elem<Tag>::T *x, int64_t x_stride, typename elem<Tag>::T *out, int64_t out_stride, int rows, int nvec) {
+  constexpr int VEC = elem<Tag>::VEC, U = 4;   // vectors of a row per thread and trip, all loads ahead of the arithmetic
+  for (int r = blockIdx.y; r < rows; r += gridDim.y) {
+    const typename elem<Tag>::T *xr = x + (int64_t)r * x_stride;
+    for (int c0 = blockIdx.x * 256 + threadIdx.x; c0 < nvec; c0 += gridDim.x * 256 * U) {
+      float a[U][VEC];
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const int c = c0 + u * gridDim.x * 256;
+        if (c < nvec) load_vec<Tag>(xr + c * VEC, a[u]);
+      }
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const int c = c0 + u * gridDim.x * 256;
+        if (c >= nvec) continue;
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) a[u][j] = gelu_erf<Tag>(a[u][j]);
+        store_vec<Tag>(out + (int64_t)r * out_stride + c * VEC, a[u]);
+      }
+    }
+  }
+}
+
+extern "C" int mv_gelu_erf(const void *x, int64_t x_stride, void *out, int64_t out_stride, int rows, int cols, int dtype, void *stream) {
+  if (rows == 0) return MV_OK;
+  if (!x || !out) return MV_E_NULLPTR;
+  if (rows < 0 || cols <= 0) return MV_E_SHAPE;
+  if (!mv_aligned16(x) || !mv_aligned16(out)) return MV_E_ALIGN;
+  MV_DISPATCH_DTYPE(dtype, {
+    typedef typename elem<Tag>::T T;
+    constexpr int VEC = elem<Tag>::VEC;
+    if (cols % VEC) return MV_E_SHAPE;
+    if ((x_stride % VEC) || (out_stride % VEC)) return MV_E_ALIGN;
+    const int nvec = cols / VEC, bx = (nvec + 1023) / 1024;
+    int by = rows < 65535 ? rows : 65535;
+    while ((int64_t)bx * by > 16384 && by > 1) by = (by + 1) / 2;
+    hipLaunchKernelGGL((gelu_erf_kernel<Tag>), dim3((unsigned)bx, (unsigned)by), dim3(256), 0, (hipStream_t)stream, (const T *)x, x_stride,
+                       (T *)out, out_stride, rows, nvec);
+  });
+  MV_LAUNCH_CHECK();
+  return MV_OK;
+}
+
 extern "C" int mv_silu_and_mul(const void *x, int64_t x_stride, void *out, int64_t out_stride,
                                int rows, int cols, int dtype, void *stream) {
   return act_and_mul<MV_ACT_SILU>(x, x_stride, out, out_stride, rows, cols, dtype, stream);

@@ -20,6 +20,7 @@ struct RopeParams {
   const void *q_norm_w, *k_norm_w;
   float eps;
   int norm_dim;   // columns that the head norms are means over
+  int unit;       // rows divided by their rms, no weight, one rounding behind the rotation
   void *q_out, *k_out, *k_cache, *v_cache;
   const int32_t *slot_mapping;
   int64_t num_slots;
@@ -75,12 +76,15 @@ __global__ void __launch_bounds__(256) rope_qk_store_kernel(RopeParams p) {
         for (int j = 0; j < 4; ++j) x[j] = u2f(raw[j]);
       }
     }
-    if (nw != nullptr) {  // per-head RMSNorm, result rounded to dtype like the reference
+    float rs = 1.0f;
+    if (nw != nullptr || p.unit) {   // (a rotation keeps the length)
       float ss = 0.f;
 #pragma unroll
       for (int j = 0; j < VEC; ++j) ss = fmaf(x[j], x[j], ss);
       ss = lpt_sum<LPT>(ss);
-      const float rs = 1.0f / sqrtf(ss / (float)p.norm_dim + p.eps);
+      rs = 1.0f / sqrtf(ss / (float)p.norm_dim + p.eps);
+    }
+    if (nw != nullptr) {  // per-head RMSNorm, result rounded to dtype like the reference
       float w[VEC];
       const u32x4 wraw = *reinterpret_cast<const u32x4 *>(nw + sub * VEC);
       if constexpr (VEC == 8) unpack8<Tag>(wraw, w);
@@ -94,6 +98,10 @@ __global__ void __launch_bounds__(256) rope_qk_store_kernel(RopeParams p) {
     }
     float y[VEC];
     rot_apply<D, VEC>(x, cs, sn, sub, p.interleaved != 0, y);
+    if (p.unit) {
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) y[j] = __fmul_rn(y[j], rs);
+    }
     u32x4 packed;
     if constexpr (VEC == 8) packed = pack8<Tag>(y);
     else {
@@ -127,6 +135,7 @@ extern "C" int mv_rope_qk_store_ex(const void *q, const void *k, const void *v, 
   if (n_tok == 0) return MV_OK;
   if (!q || !k || !positions || (mv_needs_tables(opts) && (!cos || !sin)) || !q_out) return MV_E_NULLPTR;
   if ((q_norm_w == nullptr) != (k_norm_w == nullptr)) return MV_E_NULLPTR;
+  if (q_norm_w && opts && opts->unit_norm) return MV_E_SHAPE;
   const bool has_cache = k_cache != nullptr || v_cache != nullptr || slot_mapping != nullptr;
   if (has_cache && (!k_cache || !v_cache || !slot_mapping || !v)) return MV_E_NULLPTR;
   if (n_tok < 0 || n_heads <= 0 || n_kv_heads <= 0 || (mv_needs_tables(opts) && max_pos <= 0)) return MV_E_SHAPE;
@@ -152,6 +161,7 @@ extern "C" int mv_rope_qk_store_ex(const void *q, const void *k, const void *v, 
   p.num_slots = num_slots;
   p.n_heads = n_heads; p.n_kv_heads = n_kv_heads;
   p.norm_dim = opts && opts->norm_dim ? opts->norm_dim : head_dim;
+  p.unit = opts && opts->unit_norm;
   p.interleaved = opts && opts->interleaved;
   p.pairs = p.interleaved ? opts->rot_pairs : head_dim / 2;
   hipStream_t st = (hipStream_t)stream;

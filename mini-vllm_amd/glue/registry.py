@@ -6,13 +6,14 @@ from .kugulorn import KugulornForCausalLM
 from .mofarax import MofaraxForCausalLM
 from .pununex import PununexForCausalLM
 from .opt import OPTForCausalLM
+from .semezen import SemezenForCausalLM
 from .qwen import Qwen2ForCausalLM, Qwen3ForCausalLM
 
 SUPPORTED_MODELS = {"Qwen2ForCausalLM": Qwen2ForCausalLM, "Qwen3ForCausalLM": Qwen3ForCausalLM,
                     "OPTForCausalLM": OPTForCausalLM, "Mofarax": MofaraxForCausalLM, "Kugulorn": KugulornForCausalLM,
-                    "Pununex": PununexForCausalLM}
+                    "Pununex": PununexForCausalLM, "Semezen": SemezenForCausalLM}
 TYPE_TO_ARCH = {"qwen2": "Qwen2ForCausalLM", "qwen3": "Qwen3ForCausalLM", "opt": "OPTForCausalLM",
-                "mofarax": "Mofarax", "kugulorn": "Kugulorn", "pununex": "Pununex"}
+                "mofarax": "Mofarax", "kugulorn": "Kugulorn", "pununex": "Pununex", "semezen": "Semezen"}
 
 
 def create_model(hf_config: Any) -> Any:

@@ -96,8 +96,13 @@ _SIGNATURES = {
     "mv_head_norm_gate": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_int, c_int, c_int,
                                   c_float, c_int, c_float, c_int, c_void_p]),
     "mv_moe_route": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
-                             c_float, c_int, c_void_p]),
-    "mv_moe_group": (c_int, [c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p]),
+                             c_float, c_int, c_int, c_void_p]),
+    "mv_moe_group": (c_int, [c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p]),
+    "mv_gelu_erf": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int, c_int, c_int, c_void_p]),
+    "mv_stream_update": (c_int, [c_void_p, c_int, c_int, c_int, c_int, c_void_p]),
+    "mv_gru_prefill_workspace_bytes": (c_size_t, [c_int] * 4),
+    "mv_gru_prefill": (c_int, [c_void_p, c_int, c_void_p]),
+    "mv_gru_step": (c_int, [c_void_p, c_int, c_void_p]),
     "mv_moe_linear": (c_int, [c_void_p, c_int, c_void_p]),
     "mv_gated_act_small_m": (c_int, [c_void_p, c_int64, c_void_p, c_int, c_void_p, c_int64, c_int, c_int, c_int, c_void_p,
                                      c_int, c_int, c_void_p]),
@@ -167,17 +172,20 @@ class MvHipError(RuntimeError):
 class MvAttnOpts(ctypes.Structure):
     """Options of the ``_ex`` attention entry points (include/mvhip.h)."""
     _fields_ = [("rot_pairs", c_int), ("interleaved", c_int), ("chunk", c_int), ("norm_dim", c_int), ("out_stride", c_int64),
-                ("window", c_int), ("keep_first", c_int), ("softcap", c_float), ("out_scale", c_float), ("sink", c_void_p)]
+                ("window", c_int), ("keep_first", c_int), ("softcap", c_float), ("out_scale", c_float), ("sink", c_void_p),
+                ("gate", c_void_p), ("gate_stride", c_int64), ("unit_norm", c_int), ("reserved", c_int)]
 
 
 class AttnMask(NamedTuple):
     """What a query sees and how its scores become weights (include/mvhip.h: MvAttnOpts): a window of positions with the first
-    ``keep_first`` tokens kept, capped scores, a factor of the output, one more term per head in the softmax denominator."""
+    ``keep_first`` tokens kept, capped scores, a factor of the output, one more term per head in the softmax denominator, a gate
+    (rows [N, heads * D], one per query: the output is multiplied by its sigmoid)."""
     window: int = 0
     keep_first: int = 0
     softcap: float = 0.0
     out_scale: float = 1.0
     sink: torch.Tensor | None = None
+    gate: torch.Tensor | None = None
 
 
 NO_MASK = AttnMask()
@@ -200,6 +208,7 @@ class GateAct(ctypes.Structure):
 
 
 RELU_GLU = GateAct(3, 0.0, 0.0)     # max(gate, 0) * up
+MV_LINEAR_GELU_ERF = 1 << 18        # plain projections: 0.5 y (1 + erf(y / sqrt(2))) in the epilogue
 
 
 def clamped_glu(limit: float, alpha: float = 1.702) -> GateAct:
@@ -235,20 +244,34 @@ MvDeltaArgs = _struct(
     n_seqs__max_q__total_q__channels__taps__heads__groups__p__p_true__n__k_off__q_off__channel_decay__gate_kind=c_int,
     eps__unit_eps__q_scale__out_scale=c_float)
 MvMoeLinearArgs = _struct(
-    "MvMoeLinearArgs", x__w__out__tokens__tiles__act=c_void_p, x_stride__out_stride=c_int64, max_tiles__tile_m__n__k=c_int)
+    "MvMoeLinearArgs", x__w__out__tokens__tiles__act__in_scale=c_void_p, x_stride__out_stride=c_int64, max_tiles__tile_m__n__k=c_int)
 
 
-def _attn_opts(interleaved_pairs=None, chunk: int = 0, out=None, mask: AttnMask | None = None, norm_dim: int = 0, like=None):
+MvStreamArgs = _struct(
+    "MvStreamArgs", x__x_out__y__mix__out_w__embed__ids__in_w__norm_w__shift__out__moe_out__moe_rows__moe_w__prev__positions__state_slots__cu_q=c_void_p,
+    y_stride__out_stride__vocab__slots=c_int64, streams__y_splits__moe_top__n_seqs=c_int, eps=c_float, reserved=c_int)
+MvGruArgs = _struct(
+    "MvGruArgs", z__u__g__state__state_slots__cu_q__cu_k__context_lens__out__workspace=c_void_p,
+    stride__out_stride__slots__ws_bytes=c_int64, n_seqs__max_q__total_q__n=c_int)
+
+
+def _attn_opts(interleaved_pairs=None, chunk: int = 0, out=None, mask: AttnMask | None = None, norm_dim: int = 0, like=None,
+               unit_norm: bool = False):
     """``interleaved_pairs``: None = rotary halves, n = interleaved layout with n rotated pairs; ``chunk``: chunk size of
     the causal mask (0 = whole context); ``out``: output tensor [rows, H, D] whose rows may be strided; ``norm_dim``: columns that
-    the head norms are means over (0 = all); ``like``: q, whose dtype and heads the mask's sink must have."""
+    the head norms are means over (0 = all); ``like``: q, whose dtype and heads the mask's sink must have, whose rows and columns its
+    gate must have; ``unit_norm``: q and k divided by their rms behind the rotation."""
     il, m = interleaved_pairs is not None, mask or NO_MASK
     _need_cuda(m.sink)
     if m.sink is not None and like is not None and (m.sink.dtype != like.dtype or m.sink.numel() != like.shape[1]
                                                     or not m.sink.is_contiguous()):
         raise MvHipError(f"sink: a number of {like.dtype} per head required")
+    if m.gate is not None and like is not None and (m.gate.dtype != like.dtype or m.gate.stride(1) != 1 or m.gate.shape[0] < like.shape[0]
+                                                    or m.gate.shape[1] < like.shape[1] * like.shape[2]):
+        raise MvHipError(f"gate: a row of {like.shape[1] * like.shape[2]} {like.dtype} per query required")
     o = MvAttnOpts(int(interleaved_pairs) if il else 0, int(il), int(chunk), int(norm_dim), out.stride(0) if out is not None else 0,
-                   int(m.window), int(m.keep_first), float(m.softcap), float(m.out_scale), _ptr(m.sink))
+                   int(m.window), int(m.keep_first), float(m.softcap), float(m.out_scale), _ptr(m.sink), _ptr(m.gate),
+                   m.gate.stride(0) if m.gate is not None else 0, int(unit_norm))
     return ctypes.byref(o)
 
 
@@ -452,9 +475,10 @@ def _rot_tables_ok(cos, sin, d: int, interleaved_pairs) -> bool:
 
 def rope_qk_store(q, k, v, positions, cos, sin, q_norm_w=None, k_norm_w=None, eps: float = 1e-6,
                   k_cache=None, v_cache=None, slot_mapping=None, want_k_out: bool = True, interleaved_pairs=None,
-                  norm_dim: int = 0):
+                  norm_dim: int = 0, unit_norm: bool = False):
     """q [T,H,D], k/v [T,Hkv,D] (views of the qkv GEMM output are fine).
-    ``interleaved_pairs``: n = the interleaved layout on the first 2n dims (cos / sin [max_pos, n]); None = halves.
+    ``interleaved_pairs``: n = the interleaved layout on the first 2n dims (cos / sin [max_pos, n]); None = halves.  ``unit_norm``:
+    q and k are divided by their rms behind the rotation (no weights).
     Returns (q_rot [T,H,D], k_rot [T,Hkv,D] or None)."""
     _need_cuda(q, k, positions, cos, sin)
     t, h, d = q.shape
@@ -484,7 +508,7 @@ def rope_qk_store(q, k, v, positions, cos, sin, q_norm_w=None, k_norm_w=None, ep
         q_out.data_ptr(), _ptr(k_out),
         k_cache.data_ptr() if has_cache else None, v_cache.data_ptr() if has_cache else None,
         _i32(slot_mapping).data_ptr() if has_cache else None, num_slots, t, h, hkv, d, _dt(q),
-        _attn_opts(interleaved_pairs, norm_dim=norm_dim), _stream()), "mv_rope_qk_store")
+        _attn_opts(interleaved_pairs, norm_dim=norm_dim, unit_norm=unit_norm), _stream()), "mv_rope_qk_store")
     return q_out, k_out
 
 
@@ -528,7 +552,8 @@ def paged_decode(q, k_cache, v_cache, block_tables, context_lens, scale: float, 
 # ---------------------------------------------------------------- K2
 def rope_paged_decode(q, k, v, positions, cos, sin, q_norm_w, k_norm_w, eps: float, slot_mapping,
                       k_cache, v_cache, block_tables, context_lens, scale: float, flags: int | None = None,
-                      interleaved_pairs=None, chunk: int = 0, out=None, mask: AttnMask | None = None, norm_dim: int = 0):
+                      interleaved_pairs=None, chunk: int = 0, out=None, mask: AttnMask | None = None, norm_dim: int = 0,
+                      unit_norm: bool = False):
     """Decode step of one layer in ONE launch: q [B,H,D], k/v [B,Hkv,D] RAW rows of the qkv projection (views are
     fine) -> per-head RMSNorm (weights or None) + RoPE on q and k, the new K/V rows stored at ``slot_mapping``, paged
     attention over ``block_tables`` / ``context_lens`` (which count the new token).  Returns [B,H,D], or None when
@@ -561,7 +586,7 @@ def rope_paged_decode(q, k, v, positions, cos, sin, q_norm_w, k_norm_w, eps: flo
         _ptr(cos), _ptr(sin), 0 if cos is None else cos.shape[0], _ptr(qn), _ptr(kn), float(eps), _i32(slot_mapping).data_ptr(),
         k_cache.data_ptr(), v_cache.data_ptr(), bt.data_ptr(), bt.stride(0), cl.data_ptr(), out.data_ptr(), b, h, hkv,
         d, bs, bt.shape[1], nb, float(scale), ws.data_ptr(), ws.numel(), _dt(q), flags,
-        _attn_opts(interleaved_pairs, chunk, out, mask, norm_dim, q), _stream())
+        _attn_opts(interleaved_pairs, chunk, out, mask, norm_dim, q, unit_norm), _stream())
     if rc == MV_E_SHAPE:
         return None
     _check(rc, "mv_rope_paged_decode")
@@ -677,6 +702,17 @@ def act_and_mul(x, act, out=None):
     out = _gated_out(out, rows, cols, x)
     _check(_lib.mv_act_and_mul(x.data_ptr(), x.stride(0), out.data_ptr(), out.stride(0), rows, cols, ctypes.byref(act), _dt(x),
                                _stream()), "mv_act_and_mul")
+    return out
+
+
+def gelu_erf(x, out=None):
+    """0.5 x (1 + erf(x / sqrt(2))) of rows [rows, cols] (row-strided view ok; ``out`` may be x)."""
+    _need_cuda(x, out)
+    if x.dim() != 2 or x.stride(1) != 1:
+        raise ValueError(f"gelu_erf wants [rows, cols] rows, got {tuple(x.shape)}")
+    out = _gated_out(out, x.shape[0], x.shape[1], x)
+    _check(_lib.mv_gelu_erf(x.data_ptr(), x.stride(0), out.data_ptr(), out.stride(0), x.shape[0], x.shape[1], _dt(x), _stream()),
+           "mv_gelu_erf")
     return out
 
 
@@ -822,7 +858,7 @@ def _packed_ok(packed, n_rows: int, k: int, dtype) -> bool:
             and packed.numel() == -(-n_rows // 16) * 16 * k)
 
 
-def linear_narrow(x, packed, n: int, bias=None):
+def linear_narrow(x, packed, n: int, bias=None, shape: int = 0):
     """x [..., K] (any number of rows), packed = pack_weight(W [n, K]), n small -> [..., n]: rows in groups of 16."""
     _need_cuda(x, packed)
     x2, k = _rows2d(x)
@@ -830,7 +866,7 @@ def linear_narrow(x, packed, n: int, bias=None):
         raise ValueError(f"packed weight / bias do not match [{n}, {k}] of {x.dtype}")
     out = torch.empty((x2.shape[0], n), dtype=x.dtype, device=x.device)
     _check(_lib.mv_linear_small_m_packed(x2.data_ptr(), x2.stride(0), packed.data_ptr(), _ptr(bias), out.data_ptr(),
-                                         out.stride(0), x2.shape[0], n, k, _dt(x), 1 << 17, _stream()),   # MV_LINEAR_ROW_GROUPS
+                                         out.stride(0), x2.shape[0], n, k, _dt(x), 1 << 17 | int(shape), _stream()),   # MV_LINEAR_ROW_GROUPS
            "mv_linear_small_m_packed")
     return out.view(*x.shape[:-1], n)
 
@@ -1525,16 +1561,22 @@ def head_norm_gate(y, gate, w, heads: int, p: int, p_true: int, eps: float, gate
 
 
 # ---------------------------------------------------------------- K17
-def moe_route(x, w, correction, top: int, groups: int = 1, keep: int = 1, scale: float = 1.0):
-    """x [T, K], w [outputs, K] -> (ids int32 [T, top], weights fp32 [T, top])."""
+MV_ROUTE_SIGMOID, MV_ROUTE_RAW = 1, 2
+
+
+def moe_route(x, w, correction, top: int, groups: int = 1, keep: int = 1, scale: float = 1.0, sigmoid: bool = False, raw: bool = False):
+    """x [T, K], w [outputs, K] -> (ids int32 [T, top], weights fp32 [T, top]).  ``sigmoid``: scores are sigmoids, not a softmax;
+    ``raw``: weights are the scores, not divided by their sum."""
     _need_cuda(x, w, correction)
     _rows_ok("x", x, w.shape[1])
-    if w.dtype != x.dtype or not w.is_contiguous() or correction.dtype != x.dtype or correction.numel() != w.shape[0]:
+    if w.dtype != x.dtype or not w.is_contiguous() or (correction is not None and (correction.dtype != x.dtype
+                                                                                   or correction.numel() != w.shape[0])):
         raise MvHipError(f"router weight [outputs, K] and correction [outputs] of {x.dtype} required")
     ids = torch.empty((x.shape[0], top), dtype=torch.int32, device=x.device)
     weights = torch.empty((x.shape[0], top), dtype=torch.float32, device=x.device)
-    _check(_lib.mv_moe_route(x.data_ptr(), x.stride(0), w.data_ptr(), correction.data_ptr(), ids.data_ptr(), weights.data_ptr(),
-                             x.shape[0], w.shape[1], w.shape[0], top, groups, keep, float(scale), _dt(x), _stream()), "mv_moe_route")
+    flags = (MV_ROUTE_SIGMOID if sigmoid else 0) | (MV_ROUTE_RAW if raw else 0)
+    _check(_lib.mv_moe_route(x.data_ptr(), x.stride(0), w.data_ptr(), _ptr(correction), ids.data_ptr(), weights.data_ptr(),
+                             x.shape[0], w.shape[1], w.shape[0], top, groups, keep, float(scale), flags, _dt(x), _stream()), "mv_moe_route")
     return ids, weights
 
 
@@ -1543,31 +1585,146 @@ class ExpertGroups(NamedTuple):
     tokens: torch.Tensor     # int32 [pairs], by place
     tiles: torch.Tensor      # int32 [tiles, 3]
     tile_m: int
+    weights: torch.Tensor | None = None   # fp32 [pairs], by place
 
 
-def moe_group(ids, experts: int, tile_m: int) -> ExpertGroups:
-    """(token, choice) pairs of ids [T, top] sorted by expert."""
-    _need_cuda(ids)
+def moe_group(ids, experts: int, tile_m: int, weights=None) -> ExpertGroups:
+    """(token, choice) pairs of ids [T, top] sorted by expert; ``weights`` (fp32 [T, top]): sorted along."""
+    _need_cuda(ids, weights)
     pairs, n = ids.numel(), ids.numel() // tile_m + experts
     if ids.dtype != torch.int32 or not ids.is_contiguous():
         raise MvHipError("dense int32 choices [T, top] required")
     place, tokens, tiles = (torch.empty(s, dtype=torch.int32, device=ids.device) for s in ((pairs,), (pairs,), (n, 3)))
+    by_place = None
+    if weights is not None:
+        if weights.dtype != torch.float32 or weights.numel() != pairs or not weights.is_contiguous():
+            raise MvHipError("a dense fp32 weight per choice required")
+        by_place = torch.empty_like(weights)
     _check(_lib.mv_moe_group(ids.data_ptr(), pairs, ids.shape[1], experts, tile_m, n, place.data_ptr(), tokens.data_ptr(),
-                             tiles.data_ptr(), _stream()), "mv_moe_group")
-    return ExpertGroups(place, tokens, tiles, tile_m)
+                             tiles.data_ptr(), _ptr(weights), _ptr(by_place), _stream()), "mv_moe_group")
+    return ExpertGroups(place, tokens, tiles, tile_m, by_place)
 
 
-def moe_linear(x, w, n: int, groups: ExpertGroups, act: GateAct | None = None, gather: bool = False, experts: int = 0):
+def moe_linear(x, w, n: int, groups: ExpertGroups, act: GateAct | None = None, gather: bool = False, experts: int = 0,
+               in_scale=None):
     """Rows by place: out[i] = W[expert of i] x[i] (``gather``: x[token of i]), W the experts' weights [experts, n, K] -- fp32: as
-    they are, 16-bit: packed per expert; ``act``: [experts, 2, n, K], out = act(gate, up)."""
-    _need_cuda(x, w)
+    they are, 16-bit: packed per expert; ``act``: [experts, 2, n, K], out = act(gate, up).  ``in_scale`` (fp32 by
+    place): the inputs are multiplied by it."""
+    _need_cuda(x, w, in_scale)
     pairs, k = groups.tokens.numel(), x.shape[1]
     _rows_ok("x", x, 1, w.dtype)
     if not w.is_contiguous() or w.numel() != experts * n * k * (2 if act is not None else 1) or (not gather and x.shape[0] < pairs):
         raise MvHipError(f"expert weights of {experts} x {n} outputs and {k} inputs, and a row of x per place, required")
     out = torch.empty((pairs, n), dtype=x.dtype, device=x.device)
-    a = MvMoeLinearArgs(x=x.data_ptr(), w=w.data_ptr(), out=out.data_ptr(), tokens=groups.tokens.data_ptr() if gather else None,
+    if in_scale is not None and (in_scale.dtype != torch.float32 or in_scale.numel() != pairs or not in_scale.is_contiguous()):
+        raise MvHipError("a dense fp32 factor per place required")
+    a = MvMoeLinearArgs(x=x.data_ptr(), w=w.data_ptr(), out=out.data_ptr(), in_scale=_ptr(in_scale), tokens=groups.tokens.data_ptr() if gather else None,
                         tiles=groups.tiles.data_ptr(), act=ctypes.addressof(act) if act is not None else None, x_stride=x.stride(0),
                         out_stride=out.stride(0), max_tiles=groups.tiles.shape[0], tile_m=groups.tile_m, n=n, k=k)
     _check(_lib.mv_moe_linear(ctypes.byref(a), _dt(x), _stream()), "mv_moe_linear")
+    return out
+
+
+# ---------------------------------------------------------------- K18
+class StreamShift(NamedTuple):
+    """Blend of a normed row with the one of the sequence's token before (include/mvhip.h: mv_stream_update)."""
+    share: torch.Tensor         # [cols]
+    prev: torch.Tensor          # fp32 [2, slots, cols]
+    positions: torch.Tensor
+    state_slots: torch.Tensor
+    cu_q: torch.Tensor | None = None     # None: one row per sequence
+
+
+def stream_update(streams: int, norm_w, eps: float, x=None, x_out=None, y=None, mix=None, out_w=None, in_w=None, embed=None, ids=None,
+                  experts=None, shift: StreamShift | None = None, cols_true: int | None = None, want_out: bool = True):
+    """One edge of fp32 residual streams [rows, streams, cols].  ``embed`` / ``ids``: they start from the embedding; else ``x`` is mixed
+    (``mix`` [from, to]) and gets ``out_w`` times y: [rows, cols], fp32 partial sums [splits, rows, cols], and / or ``experts`` (rows
+    [pairs, cols], place per pair, weight per pair or None).  The new streams go to ``x_out`` (None: nowhere).  -> the rms norm of
+    their sum weighted by ``in_w`` (None: 1), times ``norm_w``, blended by ``shift``."""
+    rows, cols, dt = (ids.numel() if embed is not None else x.shape[0]), norm_w.numel(), norm_w.dtype
+    _need_cuda(norm_w, x, x_out, y, mix, out_w, in_w, embed, ids)
+    for name, t in (("streams", x), ("new streams", x_out)):
+        if t is not None and (t.dtype != torch.float32 or tuple(t.shape) != (rows, streams, cols) or not t.is_contiguous()):
+            raise MvHipError(f"{name}: dense fp32 [{rows}, {streams}, {cols}] required")
+    for name, t, n in (("mix", mix, streams * streams), ("out_w", out_w, streams), ("in_w", in_w, streams),
+                       ("shift", shift.share if shift else None, cols)):
+        if t is not None and (t.dtype != dt or t.numel() != n or not t.is_contiguous()):
+            raise MvHipError(f"{name}: {n} elements of {dt} required")
+    a = MvStreamArgs(x=_ptr(x), x_out=_ptr(x_out), mix=_ptr(mix), out_w=_ptr(out_w), in_w=_ptr(in_w), norm_w=norm_w.data_ptr(),
+                     streams=streams, eps=float(eps))
+    if embed is not None:
+        if embed.dtype != dt or embed.shape[1] != cols or not embed.is_contiguous() or ids.dtype != torch.int64 or not ids.is_contiguous():
+            raise MvHipError(f"embedding table [vocab, {cols}] of {dt} and int64 ids required")
+        a.embed, a.ids, a.vocab = embed.data_ptr(), ids.data_ptr(), embed.shape[0]
+    if y is not None:
+        if y.dim() == 3:
+            if y.dtype != torch.float32 or tuple(y.shape[1:]) != (rows, cols) or not y.is_contiguous():
+                raise MvHipError("partial sums must be dense fp32 [splits, rows, cols]")
+            a.y_splits = y.shape[0]
+        elif tuple(y.shape) != (rows, cols) or y.dtype != dt or y.stride(1) != 1:
+            raise MvHipError(f"y must be [{rows}, {cols}] of {dt}")
+        a.y, a.y_stride = y.data_ptr(), y.stride(-2)
+    if experts is not None:
+        rows_out, place, weight = experts
+        if (rows_out.dtype != dt or rows_out.shape[1] != cols or not rows_out.is_contiguous() or place.dtype != torch.int32
+                or place.numel() % rows or not place.is_contiguous() or (weight is not None and (
+                    weight.dtype != torch.float32 or weight.numel() != place.numel() or not weight.is_contiguous()))):
+            raise MvHipError(f"expert outputs: dense rows of {cols} {dt}, an int32 place (and an fp32 weight) per choice required")
+        a.moe_out, a.moe_rows, a.moe_w, a.moe_top = rows_out.data_ptr(), place.data_ptr(), _ptr(weight), place.numel() // rows
+    if shift is not None:
+        _need_cuda(*shift)
+        n = rows if shift.cu_q is None else shift.cu_q.numel() - 1
+        slots = shift.prev.shape[1] if shift.prev.numel() else 0
+        if (shift.positions.dtype != torch.int64 or shift.positions.numel() != rows or not shift.positions.is_contiguous()
+                or shift.state_slots.dtype != torch.int32 or shift.state_slots.numel() != n or not shift.state_slots.is_contiguous()
+                or (slots and (shift.prev.dtype != torch.float32 or tuple(shift.prev.shape) != (2, slots, cols)
+                               or not shift.prev.is_contiguous()))
+                or (shift.cu_q is not None and (shift.cu_q.dtype != torch.int32 or not shift.cu_q.is_contiguous()))):
+            raise MvHipError(f"shift: int64 positions, int32 state slots and fp32 kept rows [2, slots, {cols}] required")
+        a.shift, a.prev, a.positions = shift.share.data_ptr(), shift.prev.data_ptr() if slots else None, shift.positions.data_ptr()
+        a.state_slots, a.cu_q, a.n_seqs, a.slots = shift.state_slots.data_ptr(), _ptr(shift.cu_q), n, slots
+    out = torch.empty((rows, cols), dtype=dt, device=norm_w.device) if want_out else None
+    a.out, a.out_stride = _ptr(out), cols
+    _check(_lib.mv_stream_update(ctypes.byref(a), rows, cols, cols if cols_true is None else int(cols_true), _DTYPES[dt], _stream()),
+           "mv_stream_update")
+    return out
+
+
+# ---------------------------------------------------------------- K19
+def _gru_args(z, u, g, state, state_slots, out):
+    _need_cuda(z, u, g, state, state_slots, out)
+    rows, n = z.shape
+    for t in (z, u, g, out):
+        if tuple(t.shape) != (rows, n) or t.dtype != z.dtype or t.stride(1) != 1 or (t is not out and t.stride(0) != z.stride(0)):
+            raise MvHipError(f"z, u and g: [{rows}, {n}] of {z.dtype} at one row stride, and such an output, required")
+    if state_slots.dtype != torch.int32 or not state_slots.is_contiguous():
+        raise MvHipError("int32 state slots required")
+    a = MvGruArgs(z=z.data_ptr(), u=u.data_ptr(), g=g.data_ptr(), state_slots=state_slots.data_ptr(), out=out.data_ptr(),
+                  stride=z.stride(0), out_stride=out.stride(0), n_seqs=state_slots.numel(), total_q=rows, n=n)
+    if state is not None and state.numel():
+        if state.dtype != torch.float32 or state.shape[0] != 2 or state.shape[2:] != (n,) or not state.is_contiguous():
+            raise MvHipError(f"recurrent state must be dense fp32 [2, slots, {n}]")
+        a.state, a.slots = state.data_ptr(), state.shape[1]
+    return a
+
+
+def gru_prefill(z, u, g, state, state_slots, cu_q, cu_k, max_q: int, out):
+    """The gated running mean over raw projections [T, n] of a batch of sequences; ``out`` [T, n] gets S silu(g)."""
+    a = _gru_args(z, u, g, state, state_slots, out)
+    a.cu_q, a.cu_k, a.max_q = cu_q.data_ptr(), cu_k.data_ptr(), int(max_q)
+    size = int(_lib.mv_gru_prefill_workspace_bytes(a.n_seqs, a.total_q, a.max_q, a.n))
+    ws = torch.empty((size,), dtype=torch.uint8, device=z.device) if size else None
+    a.workspace, a.ws_bytes = _ptr(ws), size
+    _check(_lib.mv_gru_prefill(ctypes.byref(a), _dt(z), _stream()), "mv_gru_prefill")
+    return out
+
+
+def gru_step(z, u, g, state, state_slots, context_lens, out):
+    """One token per sequence."""
+    a = _gru_args(z, u, g, state, state_slots, out)
+    lens = _i32(context_lens)
+    if lens.numel() != z.shape[0] or state_slots.numel() != z.shape[0]:
+        raise MvHipError("one length and one state slot per row required")
+    a.context_lens = lens.data_ptr()
+    _check(_lib.mv_gru_step(ctypes.byref(a), _dt(z), _stream()), "mv_gru_step")
     return out

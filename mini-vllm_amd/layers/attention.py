@@ -43,14 +43,19 @@ class Attention(nn.Module):
     def with_sink(self, sink) -> None:
         self.mask = (self.mask or hip_ops.NO_MASK)._replace(sink=sink)
 
+    def gated(self, gate):
+        """The mask of a call whose output is gated."""
+        return self.mask if gate is None else (self.mask or hip_ops.NO_MASK)._replace(gate=gate)
+
     def store_kv_cache(self, key, value, slot_mapping) -> None:
         hip_ops.store_kvcache(key, value, self.k_cache, self.v_cache, slot_mapping)
 
-    def forward(self, q, k, v, kv_stored: bool = False, out=None):
+    def forward(self, q, k, v, kv_stored: bool = False, out=None, gate=None):
         """``kv_stored=True`` when the caller already wrote k/v into the cache (the fused
         RoPE+store kernel); otherwise this call stores them first, like the reference.  ``out``: where the result goes
-        ([N, H, D], rows may be strided)."""
+        ([N, H, D], rows may be strided).  ``gate`` ([N, H * D], rows may be strided): the result is multiplied by its sigmoid."""
         ctx = get_context()
+        mask = self.gated(gate)
         has_cache = self.k_cache.numel() > 0 and self.v_cache.numel() > 0
         if has_cache:
             self._cache_initialized = True
@@ -72,23 +77,25 @@ class Attention(nn.Module):
                 if out is None:
                     out = torch.empty((q.shape[0], self.num_heads, q.shape[2]), dtype=q.dtype, device=q.device)
                 hip_ops.paged_decode(q[:nd], self.k_cache, self.v_cache, ctx.block_tables[:nd], ctx.context_lens,
-                                     self.scale, out=out[:nd], chunk=self.chunk, mask=self.mask)
+                                     self.scale, out=out[:nd], chunk=self.chunk, mask=mask)
                 if q.shape[0] > nd:
+                    if gate is not None:
+                        mask = self.gated(gate[nd:])
                     hip_ops.prefill_varlen(q[nd:], None, None, ctx.rest_cum_seqlens_q, ctx.rest_cum_seqlens_k,
                                            ctx.rest_max_seqlen_q, ctx.rest_max_seqlen_k, self.scale,
                                            k_cache=self.k_cache, v_cache=self.v_cache,
-                                           block_tables=ctx.block_tables[nd:], out=out[nd:], chunk=self.chunk, mask=self.mask)
+                                           block_tables=ctx.block_tables[nd:], out=out[nd:], chunk=self.chunk, mask=mask)
                 return out
             if ctx.prefix_cached and has_cache and ctx.block_tables is not None:
                 # prefix-cache hit: the queries are the uncached suffix, the keys live in the cache
                 return hip_ops.prefill_varlen(q, None, None, ctx.cum_seqlens_q, ctx.cum_seqlens_k,
                                               ctx.max_seqlen_q, ctx.max_seqlen_k, self.scale,
                                               k_cache=self.k_cache, v_cache=self.v_cache,
-                                              block_tables=ctx.block_tables, out=out, chunk=self.chunk, mask=self.mask)
+                                              block_tables=ctx.block_tables, out=out, chunk=self.chunk, mask=mask)
             return hip_ops.prefill_varlen(q, k, v, ctx.cum_seqlens_q, ctx.cum_seqlens_k,
-                                          ctx.max_seqlen_q, ctx.max_seqlen_k, self.scale, out=out, chunk=self.chunk, mask=self.mask)
+                                          ctx.max_seqlen_q, ctx.max_seqlen_k, self.scale, out=out, chunk=self.chunk, mask=mask)
         if ctx.context_lens is None or ctx.block_tables is None:
             raise RuntimeError("Context lengths or block tables not set for decode phase. "
                                "This is a bug in the inference pipeline.")
         return hip_ops.paged_decode(q, self.k_cache, self.v_cache, ctx.block_tables, ctx.context_lens,
-                                    self.scale, out=out, chunk=self.chunk, mask=self.mask)
+                                    self.scale, out=out, chunk=self.chunk, mask=mask)

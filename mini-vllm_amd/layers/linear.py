@@ -28,7 +28,7 @@ from ..parallel_state import (divide, get_tensor_parallel_rank, get_tensor_paral
 from ..utils.loader import materialize
 
 __all__ = ["LinearBase", "ReplicatedLinear", "ColumnParallelLinear", "MergedColumnParallelLinear",
-           "QKVParallelLinear", "RowParallelLinear", "SegmentedLinear", "Segment", "BlockLinear", "gated_linear", "pad_to", "divide", "linear", "small_m", "PartialSum", "mid_plan",
+           "QKVParallelLinear", "RowParallelLinear", "SegmentedLinear", "Segment", "BlockLinear", "gated_linear", "gelu_linear", "pad_to", "divide", "linear", "small_m", "PartialSum", "mid_plan",
            "tuned_plan", "mid_m"]
 
 # rows up to which the weight-streaming kernel beats the library GEMM (tools/bench_linear.py); 0 disables
@@ -160,6 +160,22 @@ def linear(x, weight, bias=None, packed=None, kind: str = "col"):
             if cfg:
                 return hip_ops.linear_mid_m(x, packed, n, bias, cfg)
     return F.linear(x, weight, bias)
+
+
+def gelu_linear(x, lin):
+    """gelu(lin(x)), the erf form: in the projection's epilogue for decode-sized inputs, else the library GEMM and the activation
+    kernel."""
+    w, flag = lin.weight, hip_ops.MV_LINEAR_GELU_ERF
+    if small_m(x, w):
+        return hip_ops.linear_small_m(x, w, lin.bias, shape=flag, packed=lin.weight_packed)
+    if mid_m(x, lin.weight_packed) and hip_ops.linear_mid_m_ok(x, w.shape[0]):
+        if w.shape[0] <= NARROW_N_MAX and w.shape[1] >= 256:
+            return hip_ops.linear_narrow(x, lin.weight_packed, w.shape[0], lin.bias, shape=flag)
+        cfg, _ = mid_plan("col", x.numel() // x.shape[-1], *w.shape)
+        if cfg:
+            return hip_ops.linear_mid_m(x, lin.weight_packed, w.shape[0], lin.bias, cfg | flag)
+    y = lin(x)
+    return hip_ops.gelu_erf(y, out=y)
 
 
 def gated_linear(x, lin, act="silu", out=None):
@@ -311,12 +327,14 @@ def pad_to(n: int, multiple: int = 64) -> int:
 class Segment:
     """One checkpoint matrix inside a merged weight: ``units`` (heads, features) of ``unit`` rows or columns each, stored
     at ``stored`` >= unit apiece (zeros behind); a tensor-parallel rank owns a contiguous run of whole units.  ``parts``:
-    pieces (size, place) of a unit that do not lie one behind the other in the stored unit."""
+    pieces (size, place) of a unit that do not lie one behind the other in the stored unit.  ``order``: place of each element of a
+    unit in the stored unit."""
     name: str
     units: int
     unit: int = 1
     stored: int | None = None
     parts: tuple[tuple[int, int], ...] | None = None
+    order: tuple[int, ...] | None = None
 
     def local(self, tp: int) -> int:
         """Stored rows / columns of one rank: a multiple of 64, so that the next segment starts on a whole tile."""
@@ -329,9 +347,10 @@ class SegmentedLinear(LinearBase):
     ``split="out"``: segments stack along the output features (they read the same input: q | k | gate | up ...);
     ``split="in"``: along the input features (their products are SUMMED: attention output | mlp down ...), reduced over
     the tensor-parallel ranks; ``split="none"``: one replicated matrix.  The other dimension is padded to a multiple of
-    64; ``offsets[name]`` is where a segment starts.  Padding rows / columns are zero and stay zero."""
+    64; ``offsets[name]`` is where a segment starts.  Padding rows / columns are zero and stay zero.  ``bias``
+    (not for split="in"): a bias per output, loaded by segment; segments whose checkpoint has none keep zeros."""
 
-    def __init__(self, other_size: int, segments: list[Segment], split: str = "out") -> None:
+    def __init__(self, other_size: int, segments: list[Segment], split: str = "out", bias: bool = False) -> None:
         if split not in ("out", "in", "none"):
             raise ValueError(f"unknown split {split!r}")
         tp = 1 if split == "none" else get_tensor_parallel_world_size()
@@ -341,9 +360,13 @@ class SegmentedLinear(LinearBase):
             self.offsets[g.name] = n
             n += g.local(tp)
         rows, cols = (pad_to(other_size), n) if split == "in" else (n, pad_to(other_size))
-        super().__init__(cols, rows, False, {"out": 0, "in": 1, "none": None}[split])
+        if bias and split == "in":
+            raise ValueError("the bias of summed projections belongs to none of the segments")
+        super().__init__(cols, rows, bias, {"out": 0, "in": 1, "none": None}[split])
         self.shards = tp
         self.weight.data.zero_()
+        if bias:
+            self.bias.data.zero_()
 
     def weight_loader(self, param, loaded_weight, loaded_shard_id: str | None = None, *args, **kwargs):
         if loaded_shard_id is None and len(self.segments) == 1:
@@ -358,16 +381,21 @@ class SegmentedLinear(LinearBase):
                 at += size
             return
         g = self.segments[loaded_shard_id]
+        vector = param.data.dim() == 1
         want = [self.other_size, self.other_size]
         want[dim] = g.units * g.unit
-        if tuple(loaded_weight.shape) != tuple(want):
+        if tuple(loaded_weight.shape) != tuple(want[:1] if vector else want):
             raise ValueError(f"segment {g.name!r}: expected {tuple(want)}, got {tuple(loaded_weight.shape)}")
         units, stored, off = divide(g.units, self.shards), g.stored or g.unit, self.offsets[g.name]
         rank = self.tp_rank if self.shards > 1 else 0
         piece = materialize(loaded_weight.narrow(dim, rank * units * g.unit, units * g.unit))
         dst = param.data.narrow(dim, off, units * stored).unflatten(dim, (units, stored))
-        dst = dst.narrow(0 if dim == 1 else 2, 0, self.other_size)
+        if not vector:
+            dst = dst.narrow(0 if dim == 1 else 2, 0, self.other_size)
         piece, at = piece.unflatten(dim, (units, g.unit)), 0
+        if g.order is not None:
+            dst.index_copy_(dim + 1, torch.tensor(g.order, device=dst.device), piece.to(dst.dtype))
+            return
         for size, place in g.parts or ((g.unit, 0),):
             dst.narrow(dim + 1, place, size).copy_(piece.narrow(dim + 1, at, size))
             at += size
@@ -375,7 +403,7 @@ class SegmentedLinear(LinearBase):
     def forward(self, x, partial_ok: bool = False):
         """``partial_ok`` (split="in", single rank): the caller takes a ``PartialSum``."""
         kind = "row" if partial_ok and self.split == "in" and self.shards == 1 else "col"
-        y = linear(x, self.weight, None, self.weight_packed, kind)
+        y = linear(x, self.weight, self.bias, self.weight_packed, kind)
         return tp_all_reduce(y) if self.split == "in" and self.shards > 1 else y
 
 

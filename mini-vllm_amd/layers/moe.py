@@ -1,9 +1,10 @@
 """Mixture of experts on the gfx950 kernels of csrc/moe.hip.
 
-    router: fp32 logits, softmax, choice by groups with a correction, weights          (one launch)
+    router: fp32 logits, scores, choice by groups with a correction, weights           (one launch)
     pairs (token, choice) sorted by expert                                             (one launch)
     per expert [gate | up] with the activation, then down                              (one launch each)
-The weighted sum over a token's choices (identity experts: the token's own input) is left to the residual update behind the layer.
+The weighted sum over a token's choices (identity experts: the token's own input) is left to the residual update behind the layer;
+where the weight multiplies the expert's input instead, it multiplies the sums of [gate | up], ahead of the activation.
 Expert weights are kept in ONE form: as the checkpoint has them in fp32, fragment-ordered in 16 bits (``finish_weights``)."""
 from __future__ import annotations
 
@@ -23,13 +24,21 @@ TILES = ((8, 16), (40, 32), (96, 64), (768, 128))
 
 class ExpertMLP(nn.Module):
     def __init__(self, width: int, experts: int, identity: int, top: int, groups: int, keep: int, scale: float, ff: int,
-                 shared_ff: int = 0, act: hip_ops.GateAct | None = None) -> None:
+                 shared_ff: int = 0, act: hip_ops.GateAct | None = None, sigmoid: bool = False, corrected: bool = True,
+                 raw_weights: bool = False, weigh_inputs: bool = False) -> None:
+        """``sigmoid``: scores are sigmoids of the logits, not a softmax; ``corrected``: a number per output joins the scores in the
+        choice; ``raw_weights``: the weights are the chosen scores, not divided by their sum; ``weigh_inputs``: they multiply the
+        experts' inputs, not their outputs."""
         super().__init__()
+        if weigh_inputs and identity:
+            raise ValueError("identity experts have no product that could weigh its input")
+        self.sigmoid, self.raw_weights, self.weigh_inputs = sigmoid, raw_weights, weigh_inputs
         self.experts, self.top, self.groups, self.keep, self.scale = experts, top, groups, keep, float(scale)
         self.act = act or hip_ops.GateAct(0, 0.0, 0.0)     # silu
         w, f = pad_to(width), pad_to(ff)
         self.w, self.f, self.width, self.ff = w, f, width, ff
-        self.router, self.correction = padded_parameter(experts + identity, w), padded_parameter(experts + identity)
+        self.router = padded_parameter(experts + identity, w)
+        self.correction = padded_parameter(experts + identity) if corrected else None
         self.gate_up, self.down = nn.Parameter(torch.zeros(experts, 2, f, w)), nn.Parameter(torch.zeros(experts, w, f))
         self.gate_up.weight_loader = self.down.weight_loader = self._load
         self.packed = False
@@ -65,11 +74,12 @@ class ExpertMLP(nn.Module):
 
     def forward(self, h):
         """-> (shared expert's output or None, the routed experts' part for ``hip_ops.residual_update``)."""
-        ids, weights = hip_ops.moe_route(h, self.router, self.correction, self.top, self.groups, self.keep, self.scale)
-        g = hip_ops.moe_group(ids, self.experts, self.tile_rows(h.shape[0]))
-        z = hip_ops.moe_linear(h, self.gate_up, self.f, g, self.act, gather=True, experts=self.experts)
+        ids, weights = hip_ops.moe_route(h, self.router, self.correction, self.top, self.groups, self.keep, self.scale, self.sigmoid,
+                                         self.raw_weights)
+        g = hip_ops.moe_group(ids, self.experts, self.tile_rows(h.shape[0]), weights if self.weigh_inputs else None)
+        z = hip_ops.moe_linear(h, self.gate_up, self.f, g, self.act, gather=True, experts=self.experts, in_scale=g.weights)
         y = hip_ops.moe_linear(z, self.down, self.w, g, experts=self.experts)
         shared = None
         if self.shared_gate_up is not None:
             shared = self.shared_down(gated_linear(h, self.shared_gate_up, "silu"), partial_ok=True)
-        return shared, (y, g.place, weights)
+        return shared, (y, g.place, None if self.weigh_inputs else weights)

@@ -4,9 +4,11 @@ must match torch's fp32 cos/sin of fp32 ``arange * inv_freq``); application runs
 kernel, normally fused with qk-norm and the KV-cache store (see glue/qwen.py).
 
 ``interleaved=True`` is the other layout: dims 2i and 2i + 1 form a pair, on the first ``rotary_dim`` dims of a head; its
-tables are the exact angles (fp64 on the host) rounded once to fp32."""
+tables are the exact angles (fp64 on the host) rounded once to fp32.  A design that pairs dim i with dim i + rotary_dim / 2 of
+fewer dims than a head has takes this layout too, with its heads stored in another order (``halves_as_pairs``)."""
 from __future__ import annotations
 
+import math
 from functools import lru_cache
 from typing import Any
 
@@ -15,7 +17,14 @@ from torch import nn
 
 from .. import hip_ops
 
-__all__ = ["RotaryEmbedding", "get_rope"]
+__all__ = ["RotaryEmbedding", "get_rope", "halves_as_pairs"]
+
+
+def halves_as_pairs(dim: int, rotary_dim: int) -> tuple[int, ...]:
+    """Place of each of a head's ``dim`` elements such that i and i + rotary_dim / 2 (i < rotary_dim / 2) lie side by side.  Scores
+    do not depend on the order, so queries, keys, values, gates and the columns of the output projection just share it."""
+    n = rotary_dim // 2
+    return tuple(2 * i if i < n else 2 * (i - n) + 1 if i < 2 * n else i for i in range(dim))
 
 
 def build_cos_sin(rotary_dim: int, max_position: int, base: float,
@@ -35,10 +44,22 @@ def build_cos_sin(rotary_dim: int, max_position: int, base: float,
     return freqs.cos(), freqs.sin()
 
 
-def build_cos_sin_interleaved(rotary_dim: int, max_position: int, base: float):
-    """fp32 cos / sin [max_position, rotary_dim / 2] of position * base^(-2i / rotary_dim)."""
+def stretch_by_wavelength(freq, scaling: dict[str, Any]):
+    """Frequencies whose wavelength is at most original / high stay, those from original / low on are divided by the factor, and
+    between the two both are blended, linearly in original / wavelength."""
+    factor, low, high, original = (float(scaling[k]) for k in ("factor", "low", "high", "original"))
+    turns = original * freq / (2.0 * math.pi)                       # original / wavelength
+    keep = ((turns - low) / (high - low if high != low else 1.0)).clamp(0.0, 1.0)
+    blend = (1.0 - keep) * freq / factor + keep * freq
+    return torch.where(turns > high, freq, torch.where(turns < low, freq / factor, blend))
+
+
+def build_cos_sin_interleaved(rotary_dim: int, max_position: int, base: float, scaling: dict[str, Any] | None = None):
+    """fp32 cos / sin [max_position, rotary_dim / 2] of position * base^(-2i / rotary_dim), stretched by ``scaling`` if given."""
     i = torch.arange(rotary_dim // 2, dtype=torch.float64, device="cpu")
     freq = float(base) ** (-2.0 * i / max(rotary_dim, 1))
+    if scaling is not None:
+        freq = stretch_by_wavelength(freq, scaling)
     angle = torch.arange(max_position, dtype=torch.float64, device="cpu")[:, None] * freq[None, :]
     return angle.cos().float(), angle.sin().float()
 
@@ -50,15 +71,15 @@ class RotaryEmbedding(nn.Module):
         if interleaved:
             if rotary_dim % 2 or not 0 <= rotary_dim <= head_size:
                 raise ValueError(f"interleaved rotary dims must be even and at most head_size, got {rotary_dim} of {head_size}")
-            if rope_scaling is not None:
-                raise ValueError("rope_scaling is not defined for the interleaved layout")
+            if rope_scaling is not None and rope_scaling.get("type") != "wavelength":
+                raise ValueError("the interleaved layout takes rope_scaling of type 'wavelength' only")
         elif rotary_dim != head_size:
             raise ValueError("rotary_dim must equal head_size")
         self.head_size = head_size
         self.max_position_embeddings = max_position_embeddings
         self.interleaved_pairs = rotary_dim // 2 if interleaved else None
         if interleaved:
-            cos, sin = build_cos_sin_interleaved(rotary_dim, max_position_embeddings, base)
+            cos, sin = build_cos_sin_interleaved(rotary_dim, max_position_embeddings, base, rope_scaling)
         else:
             cos, sin = build_cos_sin(rotary_dim, max_position_embeddings, base, rope_scaling)
         self.register_buffer("cos_cache", cos, persistent=False)  # [max_pos, D/2] fp32
@@ -90,11 +111,12 @@ class RotaryEmbedding(nn.Module):
 
 def get_rope(head_size: int, rotary_dim: int, max_position: int, base: float,
              rope_scaling: dict[str, Any] | None = None, interleaved: bool = False) -> RotaryEmbedding:
-    if rope_scaling is not None:  # dicts are unhashable: no cache, as in the reference
+    if rope_scaling is not None and not interleaved:  # dicts are unhashable: no cache, as in the reference
         return RotaryEmbedding(head_size, rotary_dim, max_position, base, rope_scaling, interleaved)
-    return _get_rope_cached(head_size, rotary_dim, max_position, base, interleaved)
+    return _get_rope_cached(head_size, rotary_dim, max_position, base, interleaved, tuple(sorted((rope_scaling or {}).items())))
 
 
 @lru_cache(16)
-def _get_rope_cached(head_size: int, rotary_dim: int, max_position: int, base: float, interleaved: bool) -> RotaryEmbedding:
-    return RotaryEmbedding(head_size, rotary_dim, max_position, base, None, interleaved)
+def _get_rope_cached(head_size: int, rotary_dim: int, max_position: int, base: float, interleaved: bool,
+                     scaling: tuple = ()) -> RotaryEmbedding:
+    return RotaryEmbedding(head_size, rotary_dim, max_position, base, dict(scaling) or None, interleaved)

@@ -10,7 +10,8 @@ from pathlib import Path
 
 __all__ = ["AttentionSpec", "LayerSpec", "MofaraxConfig", "LatentAttentionSpec", "Mamba2Spec", "ClampedMlpSpec", "MixerLayerSpec",
            "KugulornConfig", "DeltaRuleSpec", "SinkAttentionSpec", "ParallelMixerSpec", "ReluMlpSpec", "MoeSpec", "DeltaLayerSpec",
-           "PununexConfig", "NATIVE_CONFIGS", "checkpoint_shapes", "load_native_config"]
+           "PununexConfig", "WavelengthScaling", "KeyValueAttentionSpec", "MinGruSpec", "GeluMlpSpec", "SigmoidMoeSpec", "StreamLayerSpec",
+           "SemezenConfig", "NATIVE_CONFIGS", "checkpoint_shapes", "load_native_config"]
 
 
 def _need(d: dict, key: str, where: str):
@@ -516,7 +517,164 @@ class PununexConfig:
         return out
 
 
-NATIVE_CONFIGS = {"Mofarax": MofaraxConfig, "Kugulorn": KugulornConfig, "Pununex": PununexConfig}
+@dataclass(frozen=True)
+class WavelengthScaling:
+    """Rotary frequencies divided by a factor where their wavelength is long; see layers/rotary_embedding.py."""
+    factor: float
+    low: float
+    high: float
+    original: float
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str) -> "WavelengthScaling":
+        s = {k: _real(_need(m, k, where), f"{where}.{k}") for k in ("factor", "low", "high", "original")}
+        if min(s.values()) <= 0 or s["high"] < s["low"]:
+            raise ValueError(f"{where}: positive numbers required, high at least low, got {s}")
+        return cls(**s)
+
+
+@dataclass(frozen=True)
+class KeyValueAttentionSpec:
+    """Grouped-head attention in a window whose values are the projected keys, with a gate on its output; queries and keys have a
+    length of one (times the root of their size) behind the rotation."""
+    heads: int
+    kv_heads: int
+    dim: int
+    rot_base: float
+    rot_dims: int
+    scaling: WavelengthScaling | None
+    scale: float
+    window: int         # 0: every key up to the query
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str) -> "KeyValueAttentionSpec":
+        a = AttentionSpec.from_dict(m, where)      # (sizes, rotation and scale; its mask's size is a window here)
+        scaling = m["rot"].get("scaling")
+        return cls(a.heads, a.kv_heads, a.dim, a.rot_base, a.rot_dims,
+                   WavelengthScaling.from_dict(scaling, f"{where}.rot.scaling") if scaling else None, a.scale, a.chunk)
+
+    def weight_shapes(self, width: int) -> dict[str, tuple[int, ...]]:
+        q, k = self.heads * self.dim, self.kv_heads * self.dim
+        return {"q": (q, width), "q.b": (q,), "k": (k, width), "k.b": (k,), "g": (q, width), "o": (width, q)}
+
+
+@dataclass(frozen=True)
+class MinGruSpec:
+    """Gated running mean; see layers/mingru.py."""
+    width: int
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str) -> "MinGruSpec":
+        return cls(_size(_need(m, "width", where), f"{where}.width"))
+
+    def weight_shapes(self, width: int) -> dict[str, tuple[int, ...]]:
+        n = self.width
+        return {"z": (n, width), "z.b": (n,), "x": (n, width), "x.b": (n,), "g": (n, width), "o": (width, n)}
+
+
+@dataclass(frozen=True)
+class GeluMlpSpec:
+    ff: int
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str) -> "GeluMlpSpec":
+        return cls(_size(_need(m, "ff", where), f"{where}.ff"))
+
+    def weight_shapes(self, width: int) -> dict[str, tuple[int, ...]]:
+        return {"up": (self.ff, width), "down": (width, self.ff)}
+
+
+@dataclass(frozen=True)
+class SigmoidMoeSpec:
+    """Experts with a clamped gate behind sigmoid scores that multiply their inputs; see layers/moe.py."""
+    experts: int
+    top: int
+    ff: int
+    limit: float
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str) -> "SigmoidMoeSpec":
+        r, e = _need(m, "router", where), _need(m, "expert", where)
+        experts, top = _size(_need(r, "experts", f"{where}.router"), f"{where}.router.experts"), _size(_need(r, "top", f"{where}.router"), f"{where}.router.top")
+        if top > experts:
+            raise ValueError(f"{where}.router: {experts} experts cannot give {top} choices")
+        mlp = ClampedMlpSpec.from_dict(dict(e, kind="dense"), f"{where}.expert")
+        return cls(experts, top, mlp.ff, mlp.limit)
+
+    def weight_shapes(self, width: int) -> dict[str, tuple[int, ...]]:
+        out: dict[str, tuple[int, ...]] = {"router": (self.experts, width)}
+        for i in range(self.experts):
+            out[f"e{i}.gate"] = out[f"e{i}.up"] = (self.ff, width)
+            out[f"e{i}.down"] = (width, self.ff)
+        return out
+
+
+@dataclass(frozen=True)
+class StreamLayerSpec:
+    type: str
+    mixer: KeyValueAttentionSpec | MinGruSpec
+    mlp: GeluMlpSpec | SigmoidMoeSpec | None
+    MIXERS = {"attention": KeyValueAttentionSpec, "mingru": MinGruSpec}
+    MLPS = {"dense": GeluMlpSpec, "moe": SigmoidMoeSpec}
+
+    @classmethod
+    def from_dict(cls, d: dict, where: str) -> "StreamLayerSpec":
+        kind, mlp = _need(d, "type", where), d.get("mlp")
+        if kind not in cls.MIXERS:
+            raise ValueError(f"{where}: unsupported layer type {kind!r}; known: {sorted(cls.MIXERS)}")
+        if mlp is not None and _need(mlp, "kind", f"{where}.mlp") not in cls.MLPS:
+            raise ValueError(f"{where}.mlp: unsupported feed-forward {mlp['kind']!r}; known: {sorted(cls.MLPS)}")
+        return cls(kind, cls.MIXERS[kind].from_dict(_need(d, "mixer", where), f"{where}.mixer"),
+                   None if mlp is None else cls.MLPS[mlp["kind"]].from_dict(mlp, f"{where}.mlp"))
+
+
+class SemezenConfig:
+    """Windowed attention and gated running means over several residual streams, each mixer reading a blend of two tokens."""
+    model_type = "semezen"
+    recurrent_state = True     # the normed row of the token before, in every layer
+    MAX_STREAMS = 8            # of the kernel
+
+    def __init__(self, raw: dict) -> None:
+        self.architectures = ["Semezen"]
+        self.vocab_size = _size(_need(raw, "vocab", "config"), "vocab")
+        self.hidden_size = _size(_need(raw, "width", "config"), "width")
+        self.norm_eps = _real(_need(_need(raw, "norm", "config"), "eps", "norm"), "norm.eps")
+        self.streams = _size(_need(raw, "streams", "config"), "streams")
+        if self.streams > self.MAX_STREAMS:
+            raise ValueError(f"streams: at most {self.MAX_STREAMS} are supported, got {self.streams}")
+        layers = _need(raw, "layers", "config")
+        if not isinstance(layers, list) or not layers:
+            raise ValueError("config: 'layers' must be a non-empty list")
+        self.layers = [StreamLayerSpec.from_dict(d, f"layers[{i}]") for i, d in enumerate(layers)]
+        # what the engine asks of any configuration
+        attention = [s.mixer for s in self.layers if s.type == "attention"]
+        self.num_hidden_layers = len(self.layers)
+        self.num_attention_heads = max([a.heads for a in attention], default=1)
+        self.num_key_value_heads = max([a.kv_heads for a in attention], default=1)
+        self.head_dim = max([a.dim for a in attention], default=1)
+        self.intermediate_size = max((s.mlp.ff for s in self.layers if s.mlp), default=0)
+        self.max_position_embeddings: int | None = None    # none of its own; the engine's Config fills it in
+        self.torch_dtype = raw.get("dtype", "bfloat16")
+        self.eos_token_id = None
+        self.tie_word_embeddings = False
+
+    def weight_shapes(self) -> dict[str, tuple[int, ...]]:
+        """Name -> shape of every tensor of a checkpoint."""
+        v, d, n = self.vocab_size, self.hidden_size, self.streams
+        out: dict[str, tuple[int, ...]] = {"embed": (v, d), "final.norm": (d,), "head": (v, d)}
+        for i, s in enumerate(self.layers):
+            p = f"l{i}."
+            out[p + "shift"] = (d,)
+            out.update({f"{p}mix.{k}": v for k, v in s.mixer.weight_shapes(d).items()})
+            if s.mlp:
+                out.update({f"{p}mlp.{k}": v for k, v in s.mlp.weight_shapes(d).items()})
+            for q in ("1", "2") if s.mlp else ("1",):
+                out[f"{p}norm{q}"] = (d,)
+                out[f"{p}hc{q}.in"], out[f"{p}hc{q}.out"], out[f"{p}hc{q}.mix"] = (n,), (n,), (n, n)
+        return out
+
+
+NATIVE_CONFIGS = {"Mofarax": MofaraxConfig, "Kugulorn": KugulornConfig, "Pununex": PununexConfig, "Semezen": SemezenConfig}
 
 
 def checkpoint_shapes(model_dir) -> dict[str, tuple[int, ...]]:
