@@ -1599,7 +1599,7 @@ def moe_group(ids, experts: int, tile_m: int, weights=None) -> ExpertGroups:
     if weights is not None:
         if weights.dtype != torch.float32 or weights.numel() != pairs or not weights.is_contiguous():
             raise MvHipError("a dense fp32 weight per choice required")
-        by_place = torch.empty_like(weights)
+        by_place = torch.empty((pairs,), dtype=torch.float32, device=ids.device)
     _check(_lib.mv_moe_group(ids.data_ptr(), pairs, ids.shape[1], experts, tile_m, n, place.data_ptr(), tokens.data_ptr(),
                              tiles.data_ptr(), _ptr(weights), _ptr(by_place), _stream()), "mv_moe_group")
     return ExpertGroups(place, tokens, tiles, tile_m, by_place)
