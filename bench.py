@@ -135,15 +135,35 @@ def _pununex(like: str, peer: str, pairs: int, window: int = 2048, experts: int 
                 num_attention_heads=heads, num_key_value_heads=kv, head_dim=128, intermediate_size=ff)
 
 
+def _semezen(like: str, peer: str, pairs: int, window: int = 2048, experts: int = 32, streams: int = 4) -> dict:
+    """A Semezen configuration of ``pairs`` x [attention with a dense feed-forward, gated running mean with experts], with ``like``'s
+    width, heads and feed-forward weights (two matrices have the size of three, a token's 8 experts together too); as many pairs as
+    make the weights that a token uses ``like``'s.  ``peer``: the model it is compared with."""
+    c = MODELS[like]
+    heads, kv, width, ff = (c[k] for k in ("num_attention_heads", "num_key_value_heads", "hidden_size", "intermediate_size"))
+    mixer = {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "mask": {"size": window},
+             "rot": {"base": c["rope_theta"], "dims": 64, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+    moe = {"kind": "moe", "router": {"experts": experts, "top": 8}, "expert": {"ff": ff // 8, "limit": 7.0}}
+    layers = [{"type": "attention", "mixer": mixer, "mlp": {"kind": "dense", "ff": ff * 3 // 2}},
+              {"type": "mingru", "mixer": {"width": heads * 128}, "mlp": moe}] * pairs
+    return dict(architecture="Semezen", vocab=c["vocab_size"], width=width, streams=streams, norm={"eps": 1e-6}, layers=layers, like=peer,
+                window=window, vocab_size=c["vocab_size"], hidden_size=width, num_attention_heads=heads, num_key_value_heads=kv,
+                head_dim=128, intermediate_size=ff)
+
+
 DESIGNS = {"mofarax": {"mofarax-0.6b": "qwen3-0.6b", "mofarax-1.7b": "qwen3-1.7b", "mofarax-7b": "qwen2-7b"},
            "kugulorn": {"kugulorn-0.6b": "qwen3-0.6b", "kugulorn-1.7b": "qwen3-1.7b", "kugulorn-7b": "qwen2-7b"},
            # (beside the design that also mixes attention with a recurrence)
-           "pununex": {"pununex-0.6b": "kugulorn-0.6b", "pununex-1.7b": "kugulorn-1.7b", "pununex-7b": "kugulorn-7b"}}
+           "pununex": {"pununex-0.6b": "kugulorn-0.6b", "pununex-1.7b": "kugulorn-1.7b", "pununex-7b": "kugulorn-7b"},
+           # (beside the design with windowed attention, a recurrence and experts too)
+           "semezen": {"semezen-0.6b": "pununex-0.6b", "semezen-1.7b": "pununex-1.7b", "semezen-7b": "pununex-7b"}}
 MODELS.update({name: _mofarax(like) for name, like in DESIGNS["mofarax"].items()})
 MODELS.update({"kugulorn-0.6b": _kugulorn("qwen3-0.6b", 512, 32, 1, 19), "kugulorn-1.7b": _kugulorn("qwen3-1.7b", 768, 64, 1, 19),
                "kugulorn-7b": _kugulorn("qwen2-7b", 1536, 112, 2, 21)})
 MODELS.update({f"pununex-{s}": _pununex(like, f"kugulorn-{s}", n) for s, like, n in
                (("0.6b", "qwen3-0.6b", 12), ("1.7b", "qwen3-1.7b", 13), ("7b", "qwen2-7b", 13))})
+MODELS.update({f"semezen-{s}": _semezen(like, f"pununex-{s}", 13) for s, like in
+               (("0.6b", "qwen3-0.6b"), ("1.7b", "qwen3-1.7b"), ("7b", "qwen2-7b"))})
 DESIGN_DECODE = ((256, 1024), (16, 1024), (1, 1024))      # (batch, context) of a design's decode records
 DESIGN_PREFILL = ((16, 1024), (4, 4096))
 HBM_PEAK_GBS = 8000.0  # MI355X_MICROARCH.md: HBM3E 8.0 TB/s spec (6.29 TB/s measured copy ceiling)
@@ -572,6 +592,7 @@ def step_roofline(engine, model, batch, ctx_mid, ms_per_step):
                   for m in ex.model.modules() if hasattr(m, "k_cache"))
         kv += sum(2 * batch * t.numel() // (2 * t.shape[1]) * t.element_size() for m in recurrent_modules(ex)
                   for t in (m.conv_state, m.ssm_state if hasattr(m, "ssm_state") else m.state))
+        kv += sum(2 * batch * m.n * 4 for m in gru_modules(ex))
     else:
         L, nb, bs, hkv, d = ex.kv_cache.shape[1:]
         kv = L * batch * ctx_mid * 2 * hkv * d * ex.dtype.itemsize
@@ -583,6 +604,10 @@ def step_roofline(engine, model, batch, ctx_mid, ms_per_step):
 
 def recurrent_modules(ex) -> list:
     return [m for m in ex.state_modules if hasattr(m, "conv_state")]
+
+
+def gru_modules(ex) -> list:
+    return [m for m in ex.state_modules if type(m).__name__ == "MinGRU"]
 
 
 def expert_modules(ex) -> list:
@@ -652,7 +677,8 @@ def prefill_records(engine, model, gpus=1, cases=PREFILL_CASES, reps=5):
             for s in seqs:
                 bm.allocate(s)
             probing = rep == reps + 1
-            entries = {entry: "prefill", "ssm_prefill": "ssm", "delta_prefill": "delta", "moe_linear": "experts"}
+            entries = {entry: "prefill", "ssm_prefill": "ssm", "delta_prefill": "delta", "moe_linear": "experts", "gru_prefill": "gru",
+                       "stream_update": "edges", "residual_update": "edges", "gelu_erf": "act", "act_and_mul": "act"}
             reals = {e: getattr(hip_ops, e) for e in entries}
             if probing:
                 for e, key in entries.items():
@@ -693,7 +719,12 @@ def prefill_records(engine, model, gpus=1, cases=PREFILL_CASES, reps=5):
                                  "share_of_step": round(us * len(t_us) / (med * 1e6), 4),
                                  "mfma_busy": busy, "mfma_busy_source": busy_src,
                                  "timing": f"HIP event pairs around every mv_{entry} launch of one extra (untimed) batch, on the launching stream"}})
-        if recurrent_modules(ex) and hasattr(recurrent_modules(ex)[0], "state"):
+        out[-1].update(_edge_prefill(ex, n * ln, probe))
+        if gru_modules(ex):
+            m0, us = gru_modules(ex)[0], statistics.median(probe.times_us("gru"))
+            out[-1]["ssm_roofline"] = dict(_hbm(n * ln * m0.n * 4 * ex.dtype.itemsize, us), kernel="gru_chunk_kernel + gru_walk_kernel")
+            out[-1].update(_delta_and_expert_prefill(ex, n * ln, probe))
+        elif recurrent_modules(ex) and hasattr(recurrent_modules(ex)[0], "state"):
             out[-1].update(_delta_and_expert_prefill(ex, n * ln, probe))
         elif ex.state_modules:
             m0, t_ssm = ex.state_modules[0], sorted(probe.times_us("ssm"))
@@ -702,6 +733,32 @@ def prefill_records(engine, model, gpus=1, cases=PREFILL_CASES, reps=5):
             out[-1]["ssm_roofline"] = {"bound": "hbm", "kernel": "ssm_chunk_kernel", "bytes_per_launch": byt, "us_per_launch": round(us, 2),
                                        "achieved": round(byt / us / 1e3, 1), "peak": HBM_PEAK_GBS, "unit": "GB/s",
                                        "frac": round(byt / us / 1e3 / HBM_PEAK_GBS, 4)}
+    return out
+
+
+def _hbm(byt: int, us: float) -> dict:
+    return {"bound": "hbm", "bytes_per_launch": int(byt), "us_per_launch": round(us, 2), "achieved": round(byt / us / 1e3, 1),
+            "peak": HBM_PEAK_GBS, "unit": "GB/s", "frac": round(byt / us / 1e3 / HBM_PEAK_GBS, 4)}
+
+
+def _edge_prefill(ex, tokens: int, probe) -> dict:
+    """The launches between two sublayers (layers of a mixer and a feed-forward each): behind the mixers, and behind the dense
+    feed-forwards, as bytes of the stream(s) read and written, the sublayer's output and the next one's input; the activation kernel of
+    the dense feed-forwards."""
+    stack, out, item = getattr(ex.model, "stack", []), {}, ex.dtype.itemsize
+    t = probe.times_us("edges") if stack and all(getattr(la, "mlp", None) is not None for la in stack) else []
+    if len(t) == 1 + 2 * len(stack):
+        w, n = ex.model.embed.shape[1], getattr(ex.model.config, "streams", 1)
+        dense = [i for i, la in enumerate(stack) if not hasattr(la.mlp, "experts")][:-1]      # (not the last edge: it reads differently)
+        for key, us in (("edge_roofline", t[1::2]), ("shift_edge_roofline" if n > 1 else "ff_edge_roofline", [t[2 + 2 * i] for i in dense])):
+            if us:
+                out[key] = _hbm(tokens * w * (8 * n + 2 * item), statistics.median(us))
+        dense = next((la.mlp for la in stack if not hasattr(la.mlp, "experts")), None)
+        acts = probe.times_us("act")
+        if acts:
+            lin = getattr(dense, "up", None)
+            byt = 2 * lin.weight.shape[0] if lin is not None else 3 * (dense.gate_up.weight.shape[0] // 2)
+            out["act_roofline"] = _hbm(tokens * byt * item, statistics.median(acts))
     return out
 
 
@@ -1056,19 +1113,20 @@ def attention_graph_roofline(engine, model) -> tuple:
     mods = [m for m in ex.model.modules() if hasattr(m, "k_cache") and hasattr(m, "v_cache")]
     m0 = mods[0]
     q = torch.randn((len(seqs), m0.num_heads, m0.head_dim), device=ex.device).to(ex.dtype)
+    gate = torch.randn_like(q).flatten(1) if type(ex.model).__name__ == "SemezenForCausalLM" else None
 
     def run():
         for m in mods:
-            hip_ops.paged_decode(q, m.k_cache, m.v_cache, tables, lens, m.scale, chunk=m.chunk, mask=m.mask)
+            hip_ops.paged_decode(q, m.k_cache, m.v_cache, tables, lens, m.scale, chunk=m.chunk, mask=m.gated(gate))
     us = _graph_time_us(run, len(mods))
     seen = [n - (n - 1) // m0.chunk * m0.chunk if m0.chunk else n for n in lens.tolist()]
     if m0.mask and m0.mask.window:
         seen = [min(n, m0.mask.window + m0.mask.keep_first) for n in seen]
-    algo = (sum(seen) * 2 * m0.num_kv_heads * m0.head_dim + 2 * q.numel()) * ex.dtype.itemsize
+    algo = (sum(seen) * 2 * m0.num_kv_heads * m0.head_dim + (2 if gate is None else 3) * q.numel()) * ex.dtype.itemsize
     return {"bound": "hbm", "achieved": round(algo / us / 1e3, 1), "peak": HBM_PEAK_GBS, "unit": "GB/s",
             "frac": round(algo / us / 1e3 / HBM_PEAK_GBS, 4), "bytes_per_launch": algo, "us_per_launch": round(us, 2),
             "timing": f"{len(mods)} launches (split-KV combine included) captured into a hipGraph, median of 5 replays / launches"}, (
-                _delta_graph_roofline(ex, lens, slots) if recurrent_modules(ex) else None)
+                _gru_graph_roofline(ex, lens, slots) if gru_modules(ex) else _delta_graph_roofline(ex, lens, slots) if recurrent_modules(ex) else None)
 
 
 def _graph_roofline(byt: int, us: float, launches: int) -> dict:
@@ -1111,6 +1169,47 @@ def _state_graph_roofline(ex, lens, slots) -> dict:
     return _graph_roofline(byt, us, len(mods))
 
 
+def _gru_graph_roofline(ex, lens, slots) -> dict:
+    """mv_gru_step of every such layer on the running batch (a step that is run again gives the same state)."""
+    from minivllm_amd import hip_ops
+
+    mods, b = gru_modules(ex), lens.numel()
+    n = mods[0].n
+    z = torch.randn((b, 3 * n), device=ex.device).to(ex.dtype)
+    out = torch.empty((b, n), dtype=ex.dtype, device=ex.device)
+
+    def run():
+        for m in mods:
+            hip_ops.gru_step(z[:, :n], z[:, n:2 * n], z[:, 2 * n:], m.state, slots, lens, out)
+    return _graph_roofline(b * n * (8 + 4 * ex.dtype.itemsize), _graph_time_us(run, len(mods)), len(mods))
+
+
+def edge_graph_us(engine, batch: int) -> float | None:
+    """One launch between a feed-forward and the next mixer, on random rows inside a graph: streams with a token shift, or a normed
+    residual stream."""
+    from minivllm_amd import hip_ops
+
+    ex = engine.model_runner.inference_executor
+    stack, kind = getattr(ex.model, "stack", []), type(ex.model).__name__
+    if kind not in ("SemezenForCausalLM", "PununexForCausalLM"):
+        return None
+    w, c = ex.model.embed.shape[1], ex.model.config
+    y = torch.randn((batch, w), device=ex.device).to(ex.dtype)
+    n, pos = getattr(c, "streams", 1), torch.ones((batch,), dtype=torch.int64, device=ex.device)
+    x, new = (torch.randn((batch, n, w), device=ex.device) for _ in range(2))
+    slots = torch.arange(batch, dtype=torch.int32, device=ex.device)
+
+    def run():
+        for a, b in zip(stack, stack[1:]):
+            if kind == "SemezenForCausalLM":
+                hip_ops.stream_update(n, b.norm1, 1e-6, x=x, x_out=new, y=y, mix=a.hc2.mix, out_w=a.hc2.write, in_w=b.hc1.read,
+                                      shift=hip_ops.StreamShift(b.shift.share, b.shift.prev, pos, slots))
+            else:
+                hip_ops.residual_update(x[:, 0], y=y, y_norm_w=a.norm2, y_norm_b=a.norm2_b, y_scale=a.ls2, layer_norm=True, eps=1e-6,
+                                        dtype=ex.dtype)
+    return round(_graph_time_us(run, len(stack) - 1), 2)
+
+
 def _delta_graph_roofline(ex, lens, slots) -> dict:
     """mv_delta_step of the layers with a decay per head on the running batch (a step that is run again gives the same state)."""
     from minivllm_amd import hip_ops
@@ -1139,14 +1238,13 @@ def expert_graph_rooflines(engine, batch: int) -> dict | None:
         return None
     out, m0 = {}, mods[0]
     h = torch.randn((batch, m0.w), device=ex.device).to(ex.dtype)
-    ids = [hip_ops.moe_route(h, m.router, m.correction, m.top, m.groups, m.keep, m.scale)[0] for m in mods]
-    used = statistics.mean(len({e for e in i.flatten().tolist() if e < m0.experts}) for i in ids)
-    groups = [hip_ops.moe_group(i, m.experts, m.tile_rows(batch)) for i, m in zip(ids, mods)]
+    groups = [m.route(h)[1] for m in mods]
+    used = statistics.mean(len({e for e in g.tiles[:, 0].tolist() if e >= 0}) for g in groups)
     zs = [torch.randn((batch * m.top, m.f), device=ex.device).to(ex.dtype) for m in mods]
 
     def gate_up():
         for m, g in zip(mods, groups):
-            hip_ops.moe_linear(h, m.gate_up, m.f, g, m.act, gather=True, experts=m.experts)
+            hip_ops.moe_linear(h, m.gate_up, m.f, g, m.act, gather=True, experts=m.experts, in_scale=g.weights)
 
     def down():
         for m, g, z in zip(mods, groups, zs):
@@ -1154,7 +1252,7 @@ def expert_graph_rooflines(engine, batch: int) -> dict | None:
 
     def route():
         for m in mods:
-            hip_ops.moe_group(hip_ops.moe_route(h, m.router, m.correction, m.top, m.groups, m.keep, m.scale)[0], m.experts, m.tile_rows(batch))
+            m.route(h)
     for name, run, n in (("gate_up", gate_up, 2), ("down", down, 1)):
         out[name] = _graph_roofline(int(used * n * m0.f * m0.w * ex.dtype.itemsize), _graph_time_us(run, len(mods)), len(mods))
     out["route_and_group_us"] = round(_graph_time_us(route, len(mods)), 2)
@@ -1184,6 +1282,7 @@ def design_records(args, workdir) -> dict:
                 experts = expert_graph_rooflines(engine, batch)
                 if experts is not None:
                     rec["expert_rooflines"] = experts
+                rec["edge_us"] = edge_graph_us(engine, batch)
                 rec["step_roofline"] = step_roofline(engine, model, batch, ctx + a.warmup + a.steps // 2, rec["ms_per_step"])
                 recs.append(rec)
                 release_all(engine)

@@ -21,8 +21,9 @@ int chunk_len(int total_q, int max_q, int n) {
 // one token: the factor a = 1 - sigmoid(z) and what is added, sigmoid(z) c(u)
 template <typename Tag>
 __device__ __forceinline__ void operands(float z, float u, float &a, float &b) {
-  a = sigmoid_of<Tag>(-z);
-  b = sigmoid_of<Tag>(z) * (u >= 0.f ? u + 0.5f : sigmoid_of<Tag>(u));
+  const float s = sigmoid_of<Tag>(z);
+  a = 1.0f - s;
+  b = s * (u >= 0.f ? u + 0.5f : sigmoid_of<Tag>(u));
 }
 
 // fn(token, z, u) for the tokens t0 .. t1 of a thread's four channels

@@ -72,11 +72,15 @@ class ExpertMLP(nn.Module):
         per = tokens * self.top / self.experts
         return next((rows for most, rows in TILES if per <= most), 256)
 
-    def forward(self, h):
-        """-> (shared expert's output or None, the routed experts' part for ``hip_ops.residual_update``)."""
+    def route(self, h):
+        """-> (weights [T, top], the pairs sorted by expert)."""
         ids, weights = hip_ops.moe_route(h, self.router, self.correction, self.top, self.groups, self.keep, self.scale, self.sigmoid,
                                          self.raw_weights)
-        g = hip_ops.moe_group(ids, self.experts, self.tile_rows(h.shape[0]), weights if self.weigh_inputs else None)
+        return weights, hip_ops.moe_group(ids, self.experts, self.tile_rows(h.shape[0]), weights if self.weigh_inputs else None)
+
+    def forward(self, h):
+        """-> (shared expert's output or None, the routed experts' part for ``hip_ops.residual_update``)."""
+        weights, g = self.route(h)
         z = hip_ops.moe_linear(h, self.gate_up, self.f, g, self.act, gather=True, experts=self.experts, in_scale=g.weights)
         y = hip_ops.moe_linear(z, self.down, self.w, g, experts=self.experts)
         shared = None

@@ -172,6 +172,18 @@ def test_design_configurations_have_the_layer_sizes_of_their_peers():
         d, dim = p["hidden_size"], p.get("head_dim") or p["hidden_size"] // p["num_attention_heads"]
         layer = d * dim * 2 * (p["num_attention_heads"] + p["num_key_value_heads"]) + 3 * d * p["intermediate_size"]
         assert abs(used / (layer * p["num_hidden_layers"]) - 1) < 0.1, name
+    for name, peer in bench.DESIGNS["semezen"].items():
+        c, like = NATIVE_CONFIGS["Semezen"](bench.MODELS[name]), bench.MODELS[bench.MODELS[peer]["like"]]
+        p = bench.MODELS[like["like"]] if "like" in like else like
+        assert (c.vocab_size, c.hidden_size, c.num_attention_heads) == (p["vocab_size"], p["hidden_size"], p["num_attention_heads"])
+        used = 0
+        for s in c.layers:
+            ff = 3 * s.mlp.top * s.mlp.ff if hasattr(s.mlp, "experts") else 2 * s.mlp.ff
+            assert ff == 3 * p["intermediate_size"]
+            used += c.hidden_size * ff + sum(a[0] * a[1] for a in s.mixer.weight_shapes(c.hidden_size).values() if len(a) == 2)
+        d, dim = p["hidden_size"], p.get("head_dim") or p["hidden_size"] // p["num_attention_heads"]
+        layer = d * dim * 2 * (p["num_attention_heads"] + p["num_key_value_heads"]) + 3 * d * p["intermediate_size"]
+        assert abs(used / (layer * p["num_hidden_layers"]) - 1) < 0.1, name
     assert bench.prefill_flops(2, 64, [100], 0, 30) == 4 * 2 * 64 * (sum(range(1, 31)) + 70 * 30)
     args = bench.parse(["--design", "mofarax"])
     assert args.design == "mofarax" and bench.parse([]).design is None and bench.parse([]).model == "qwen3-1.7b"

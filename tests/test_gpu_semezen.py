@@ -49,7 +49,7 @@ def _i32(values):
 @pytest.mark.parametrize("dtype", DTYPES + [torch.float16])
 @pytest.mark.parametrize("streams", [1, 2, 3, 4, 5, 8])
 @pytest.mark.parametrize("cols, true, how", [(256, 200, "rows"), (64, 64, "splits"), (320, 320, "experts"), (4160, 4100, "rows"), (128, 100, "all"),
-                                             (8320, 8320, "splits")])
+                                             (8192, 8190, "splits")])
 def test_streams_are_mixed_written_and_read(H, dtype, streams, cols, true, how):
     rows, eps, top, n = 7, 1e-3, 2, streams
     pad = lambda t: torch.nn.functional.pad(t, (0, cols - true))
