@@ -137,7 +137,7 @@ __global__ void __launch_bounds__(kRouteWaves * 64) moe_route_kernel(RouteParams
 
 // ---- grouping.  Workgroup e = expert e: its pairs start behind those of the experts before it.  Each wave walks a part of the
 // pairs, in order, so places are the same in every run.
-constexpr int kGroupThreads = 1024, kGroupWaves = kGroupThreads / 64;
+constexpr int kGroupThreads = 1024, kGroupWaves = kGroupThreads / 64, kGroupAhead = 8;   // kGroupAhead: choices of a lane requested at a time
 
 __global__ void __launch_bounds__(kGroupThreads) moe_group_kernel(const int32_t *ids, int pairs, int top, int experts, int tile_m,
                                                                   int max_tiles, int32_t *rows, int32_t *tokens, int32_t *tiles,
@@ -146,9 +146,20 @@ __global__ void __launch_bounds__(kGroupThreads) moe_group_kernel(const int32_t 
   const int e = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int per = (pairs + kGroupWaves * 64 - 1) / (kGroupWaves * 64) * 64, lo = wave * per, hi = min(pairs, lo + per);
   int nl = 0, ne = 0;
-  for (int i = lo + lane; i < hi; i += 64) {
-    const int v = ids[i];
-    nl += v < e, ne += v == e;
+  // the choices i0 + 64 u + lane of this wave's part (-1 behind its end)
+  auto choices = [&](int i0, int (&v)[kGroupAhead]) {
+#pragma unroll
+    for (int u = 0; u < kGroupAhead; ++u) {
+      const int i = i0 + 64 * u + lane;
+      v[u] = ids[min(i, pairs - 1)];
+      if (i >= hi) v[u] = -1;
+    }
+  };
+  for (int i0 = lo; i0 < hi; i0 += 64 * kGroupAhead) {
+    int v[kGroupAhead];
+    choices(i0, v);
+#pragma unroll
+    for (int u = 0; u < kGroupAhead; ++u) nl += v[u] >= 0 && v[u] < e, ne += v[u] == e;
   }
 #pragma unroll
   for (int o = 32; o >= 1; o >>= 1) nl += __shfl_xor(nl, o, 64), ne += __shfl_xor(ne, o, 64);
@@ -160,16 +171,25 @@ __global__ void __launch_bounds__(kGroupThreads) moe_group_kernel(const int32_t 
     if (w < wave) ahead += equal[w];
   }
   int at = start + ahead;
-  for (int i0 = lo; i0 < hi; i0 += 64) {
-    const int i = i0 + lane, v = i < hi ? ids[i] : -1;
-    const unsigned long long mask = __ballot(v == e);
-    if (v == e) {
-      const int place = at + __popcll(mask & ((1ull << lane) - 1));
-      rows[i] = place, tokens[place] = i / top;
-      if (weights) weights_out[place] = weights[i];
+  for (int i0 = lo; i0 < hi; i0 += 64 * kGroupAhead) {
+    int v[kGroupAhead];
+    float w[kGroupAhead];
+    choices(i0, v);
+#pragma unroll
+    for (int u = 0; u < kGroupAhead; ++u)
+      if (weights && v[u] == e) w[u] = weights[i0 + 64 * u + lane];
+#pragma unroll
+    for (int u = 0; u < kGroupAhead; ++u) {
+      const int i = i0 + 64 * u + lane;
+      const unsigned long long mask = __ballot(v[u] == e);
+      if (v[u] == e) {
+        const int place = at + __popcll(mask & ((1ull << lane) - 1));
+        rows[i] = place, tokens[place] = i / top;
+        if (weights) weights_out[place] = w[u];
+      }
+      if (e == 0 && v[u] >= experts) rows[i] = -1;
+      at += __popcll(mask);
     }
-    if (e == 0 && v >= experts) rows[i] = -1;
-    at += __popcll(mask);
   }
   // tiles of this expert: entries start / tile_m + e on, up to the next expert's; the last expert also clears what is left
   const int t0 = start / tile_m + e, t1 = e + 1 < experts ? (start + count) / tile_m + e + 1 : max_tiles;
