@@ -769,7 +769,7 @@ int mv_moe_linear(const MvMoeLinearArgs *args, int dtype, void *stream);
  * unless shift is given with cu_q.  Means are over cols_true <= cols columns; the others hold zeros.
  * The h of a step's last token is kept in prev fp32 [2][slots][cols], half = number of tokens so far & 1, at state_slots[sequence]
  * (< 0: nothing is kept, the token before counts as zeros).  Sequences: rows cu_q[s] .. cu_q[s + 1]; cu_q NULL: one row each.  Rows at
- * position < 0: padding.  streams <= 8; all weights are of dtype. */
+ * position < 0: padding.  streams <= 8, cols <= 8192; all weights are of dtype. */
 typedef struct MvStreamArgs {
   const float *x;
   float *x_out;
